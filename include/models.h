@@ -24,6 +24,13 @@
 
 namespace xft {
 
+// One entry of Model::step
+struct StepEntry {
+    int seqID = -1; // -1: a new sequence; step() writes its id here
+    std::vector<int32_t> tokens; // the sequence's next tokens: a prompt, a portion of one, a decoded token
+    std::vector<int> want; // places among them whose logits are asked for
+};
+
 struct ModelImpl; // device model, weights and searcher state (private to the library)
 
 class Model {
@@ -99,6 +106,14 @@ public:
     // One step: the first call after input() runs the prompt, every later call one new token per
     // sequence.  Returns the batch's next token ids (models.cpp:834-846).
     std::vector<int32_t> generate();
+
+    // One batch of unequal parts: every entry brings the next tokens of a sequence, whatever their number.  Returns (logits,
+    // rows, vocab), one row a wanted place, in the order of the entries.  freeSeqs() gives a sequence's pages and slot back.
+    // Models from config.json (layer plans) only.  No counterpart in the reference.
+    std::tuple<float *, int, int> step(std::vector<StepEntry> &entries);
+
+    // Sizes the page pool (tokens over all live sequences) and the number of sequence slots step() works with.
+    void setCachePool(int tokens, int sequences);
 
     void createSearcher(SearcherConfig &config_);
 

@@ -148,6 +148,10 @@ int xfthip_gemm(xfthip_weight_t w, int M, const void *A, int lda, void *C, int l
  */
 int xfthip_gemm_gateup_silu(xfthip_weight_t w, int M, const void *A, int lda, void *out, int ldo, int out_dtype,
         xfthip_stream_t stream);
+/* out[M,I] = g * sigmoid(alpha * g) * (u + 1) with g = min(A*Wgate, limit), u = A*Wup held to [-limit, limit], for a weight
+ * created with XFTHIP_WF_GATEUP (no counterpart in the reference). */
+int xfthip_gemm_gateup_clamped(xfthip_weight_t w, int M, const void *A, int lda, void *out, int ldo, int out_dtype, float limit, float alpha,
+        xfthip_stream_t stream);
 
 /*
  * The two decode-step fusions of the M <= 32 kernel, for up to 4 activation rows (the model
@@ -539,6 +543,75 @@ int xfthip_moe_forward(xfthip_moe_t m, const float *x_in, int in_stride, float *
  * pass, decode steps (graph replay included) and the per-sequence entry points run it like any other layer.
  */
 int xfthip_model_set_moe(xfthip_model_t m, int idx, xfthip_moe_t moe);
+
+/* ---- layer plans: decoder stacks of several kinds of layers --------------------------- */
+/*
+ * A plan describes a stack whose layers differ: what mixes the tokens (latent attention or a gated delta-rule recurrence),
+ * its sizes, its constants, and the feed-forward behind it, if any.  Keys live in pages of a pool shared by all sequences,
+ * recurrent state in one slot a sequence.  The reference has no counterpart; a model built from a plan is a xfthip_model_t and
+ * runs behind the same calls as the others.
+ *
+ * Every sublayer has a norm in front and a norm behind it (RMS norms whose stored weights are distances from one), the latter
+ * multiplied by a learned scale per channel; layers [loop_start, loop_stop) run loop_times times, every run with its own cache
+ * or state, the embedding output joining the residual in front of every pass but the first.
+ */
+enum { XFTHIP_MIXER_LATENT = 1, XFTHIP_MIXER_DELTA = 2 };
+typedef struct {
+    int mixer;
+    int heads, kv_heads; /* kv_heads: query / key heads of the delta rule */
+    int dim, vdim; /* query / key (latent attention: their unrotated part) and value dimensions of a head */
+    /* latent attention */
+    int rot_dim, kv_rank, q_rank;
+    int rot_interleaved; /* 1: pairs (2i, 2i + 1), 0: pairs (i, i + rot_dim / 2) */
+    int window; /* tokens a position sees, itself included; 0 = all before it */
+    int has_sink; /* a learned logit a head in the softmax denominator */
+    float scale;
+    double rot_base;
+    /* delta rule */
+    int taps; /* of the short convolutions */
+    int decay_rank, gate_rank; /* inner widths of the two gates' projections */
+    /* feed-forward (inter 0: none): xfthip_gemm_gateup_clamped */
+    int inter;
+    float glu_limit, glu_alpha;
+} xfthip_plan_layer;
+typedef struct {
+    int layers;
+    int hidden, vocab;
+    int loop_start, loop_stop, loop_times; /* loop_times <= 1: no loop */
+    float eps, logit_scale;
+} xfthip_plan_config;
+typedef struct xfthip_plan *xfthip_plan_t;
+int xfthip_plan_create(const xfthip_plan_config *cfg, const xfthip_plan_layer *layers, xfthip_plan_t *out);
+int xfthip_plan_destroy(xfthip_plan_t p);
+/*
+ * Tensors by name, host memory, bf16 bit patterns, row-major [rows, cols] (linear weights [out, in]; vectors cols = 1): layer -1:
+ * embed, head, final.norm; a layer: norm1, norm1b, ls1, norm2, norm2b, ls2, mlp.gate / up / down, and in front of its
+ * mixer's names "mix.": latent attention dq, dq.norm, uq, dkv, dkv.norm, uk, uv, o, sink; delta rule q, k, v (each with
+ * .conv), b, A_log, a1, a2, dt_bias, g1, g2, norm, o.  xfthip_plan_finish checks that all are there, packs and uploads them.
+ */
+int xfthip_plan_set_tensor(xfthip_plan_t p, int layer, const char *name, const uint16_t *data_host, int rows, int cols);
+int xfthip_plan_finish(xfthip_plan_t p);
+size_t xfthip_plan_weight_bytes(xfthip_plan_t p);
+/*
+ * A device model over a finished plan, which must outlive it.  act_dtype: XFTHIP_BF16 (activations and cache in bf16, products
+ * on the bf16 matrix units) or XFTHIP_F32 (everything in 32 bits).  max_batch: sequence slots; pool_tokens: tokens the page
+ * pool holds over all sequences (0 = max_batch * max_seq).
+ */
+int xfthip_model_create_from_plan(xfthip_plan_t p, int act_dtype, int max_batch, int max_seq, int max_tokens, int pool_tokens,
+        xfthip_model_t *out);
+/*
+ * One step of a batch of unequal parts: entry i brings the next lens_host[i] tokens of slot rows_host[i] (a prompt, a portion of
+ * one or a single token; ids back to back in ids_host); a slot that holds no sequence starts one at position 0.  want_host: n_want
+ * indices into the step's tokens, ascending or not, whose logits go to logits_host (fp32 [n_want, vocab]).  Models from a plan only.
+ */
+int xfthip_model_step(xfthip_model_t m, int n, const int *rows_host, const int *lens_host, const int *ids_host, int n_want,
+        const int *want_host, float *logits_host, xfthip_stream_t stream);
+/* Residual stream after every layer run of the model's next steps, fp32 [runs, tokens, hidden] of the last step that ran
+ * (enable = 1 before the step; out_host NULL asks for the number of runs only). */
+int xfthip_model_trace_residual(xfthip_model_t m, int enable);
+int xfthip_model_read_residual(xfthip_model_t m, float *out_host, int *runs, int *tokens);
+/* pages of the pool that no sequence holds, and all of them */
+int xfthip_model_pool_pages(xfthip_model_t m, int *free_pages, int *total_pages);
 
 #ifdef __cplusplus
 }

@@ -18,6 +18,7 @@ if not os.path.exists(_LIB_PATH):
 _lib = C.CDLL(_LIB_PATH)
 _lib.xft_automodel_create.restype = C.c_void_p
 _lib.xft_automodel_create.argtypes = [C.c_char_p, C.c_char_p, C.c_char_p]
+_lib.xft_automodel_is_plan.argtypes = [C.c_char_p]
 _lib.xft_automodel_destroy.argtypes = [C.c_void_p]
 _lib.xft_automodel_destroy.restype = None
 _lib.xft_automodel_config.restype = None
@@ -34,6 +35,10 @@ _lib.xft_automodel_max_seq_len.argtypes = [C.c_void_p]
 _lib.xft_automodel_set_input.argtypes = [C.c_void_p, C.c_void_p, C.c_void_p, C.c_int, C.c_void_p, C.c_int, C.c_int, C.c_int, C.c_int,
                                          C.c_float, C.c_void_p]
 _lib.xft_automodel_free_seqs.argtypes = [C.c_void_p, C.c_void_p, C.c_int]
+_lib.xft_automodel_set_cache_pool.restype = None
+_lib.xft_automodel_set_cache_pool.argtypes = [C.c_void_p, C.c_int, C.c_int]
+_lib.xft_automodel_step.restype = None
+_lib.xft_automodel_step.argtypes = [C.c_void_p, C.c_int] + [C.c_void_p] * 6
 _lib.xft_automodel_set_prefix.restype = None
 _lib.xft_automodel_set_prefix.argtypes = [C.c_void_p, C.c_void_p, C.c_int]
 _lib.xft_sample_candidates.argtypes = [C.c_void_p, C.c_int, C.c_int, C.c_float, C.c_float, C.c_void_p, C.c_void_p]
@@ -52,6 +57,7 @@ _DTYPES = ["fp16", "bf16", "int8", "w8a8", "int4", "nf4", "bf16_fp16", "bf16_int
            "w8a8_int4", "w8a8_nf4"]
 _REFERENCE_DTYPES = _DTYPES + ["fp8_e4m3"]
 _KV_DTYPES = ["fp16", "int8"]
+_PLAN_DTYPES = ["bf16", "fp16", "fp32"]  # models described by config.json (layer plans)
 
 
 def _is_torch(x):
@@ -125,13 +131,14 @@ class BeamSearcher:
 
 class AutoModel:
     def __init__(self, path, dtype: str = "fp16", kv_cache_dtype: str = "fp16"):
-        if dtype not in _REFERENCE_DTYPES:
+        from_plan = bool(_lib.xft_automodel_is_plan(os.fsencode(path)))
+        if dtype not in _REFERENCE_DTYPES and not (from_plan and dtype in _PLAN_DTYPES):
             raise Exception(f"{self.__class__.__name__} don't support {dtype}.")
-        if dtype not in _DTYPES:
+        if dtype not in (_PLAN_DTYPES if from_plan else _DTYPES):
             raise Exception(f"{self.__class__.__name__} of this build don't support the type {dtype}.")
         if kv_cache_dtype not in _KV_DTYPES:
             raise Exception(f"{self.__class__.__name__} don't support KV cache data type: {kv_cache_dtype}.")
-        if not os.path.exists(os.path.join(path, "config.ini")):
+        if not from_plan and not os.path.exists(os.path.join(path, "config.ini")):
             raise FileNotFoundError(os.path.join(path, "config.ini"))
         self._h = _lib.xft_automodel_create(os.fsencode(path), dtype.encode(), kv_cache_dtype.encode())
         self._torch_out = False
@@ -196,6 +203,23 @@ class AutoModel:
     def forward_cb(self):
         """One step of the sequences chosen by set_input_cb: their next tokens, in that order."""
         return self.forward().ravel().tolist()
+
+    def set_cache_pool(self, tokens, sequences):
+        """Page pool (tokens over all live sequences) and sequence slots of step()."""
+        _lib.xft_automodel_set_cache_pool(self._h, int(tokens), int(sequences))
+
+    def step(self, entries):
+        """One batch of unequal parts.  entries: (sequence id or None for a new one, its next tokens, places among them whose
+        logits are wanted).  Returns (sequence ids in that order, fp32 logits [wanted, vocab])."""
+        seq = np.asarray([-1 if e[0] is None else int(e[0]) for e in entries], np.int32)
+        lens = np.asarray([len(e[1]) for e in entries], np.int32)
+        ids = np.asarray([t for e in entries for t in e[1]], np.int32)
+        wants = np.asarray([len(e[2]) for e in entries], np.int32)
+        want = np.asarray([w for e in entries for w in e[2]], np.int32)
+        out = np.zeros((len(want), self.vocab_size), np.float32)
+        _lib.xft_automodel_step(self._h, len(entries), seq.ctypes.data, lens.ctypes.data, ids.ctypes.data, wants.ctypes.data,
+                                want.ctypes.data, out.ctypes.data)
+        return seq.tolist(), out
 
     def prefix_sharing(self, input_ids=None, truncate_tail=0):
         """The reference's AutoModel.prefix_sharing (automodel.py:180-184): input_ids [1, n] is run once; inputs that

@@ -117,6 +117,14 @@ def build_test_drivers(force=True):
     return out
 
 
+def use_or_build_plan_libraries():
+    """For programs that may run in a checkout nothing was built in: leaves a built checkout alone."""
+    if os.path.exists(LIB_HIP) and os.path.exists(LIB_LAYERS):
+        return
+    build_hip(False)
+    build_host(False)
+
+
 def build_all(force=True):
     build_hip(force)
     build_host(force)

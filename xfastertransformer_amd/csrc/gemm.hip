@@ -133,6 +133,27 @@ int xfthip_gemm_gateup_silu(xfthip_weight_t w, int M, const void *A, int lda, vo
     return qgemm_mfma(pw, p, (hipStream_t)stream);
 }
 
+int xfthip_gemm_gateup_clamped(xfthip_weight_t w, int M, const void *A, int lda, void *out, int ldo, int out_dtype, float limit, float alpha,
+        xfthip_stream_t stream) {
+    if (int rc = check_common("xfthip_gemm_gateup_clamped", w, M, A, lda, out, ldo)) return rc;
+    const PackedWeight &pw = w->pw;
+    XFT_REQUIRE(pw.flags & XFTHIP_WF_GATEUP, "xfthip_gemm_gateup_clamped: weight was not created with XFTHIP_WF_GATEUP");
+    XFT_REQUIRE(ldo >= pw.N / 2, "xfthip_gemm_gateup_clamped: ldo=%d < I=%d", ldo, pw.N / 2);
+    XFT_REQUIRE(out_dtype == XFTHIP_F32 || out_dtype == XFTHIP_BF16, "xfthip_gemm_gateup_clamped: out_dtype must be f32 or bf16");
+    XFT_REQUIRE(pw.kind != XFTHIP_W_W8A8, "xfthip_gemm_gateup_clamped: not for W8A8 weights");
+    SkinnyParams p = {};
+    p.M = M;
+    p.A = (const uint16_t *)A;
+    p.lda = lda;
+    p.C = out;
+    p.ldc = ldo;
+    p.c_dtype = out_dtype;
+    p.gateup = 2;
+    p.glu_limit = limit, p.glu_alpha = alpha;
+    if (M <= 32) return qgemm_skinny(pw, p, (hipStream_t)stream);
+    return qgemm_mfma(pw, p, (hipStream_t)stream);
+}
+
 int xfthip_gemm_gateup_silu_rmsnorm(xfthip_weight_t w, int M, const float *x, int ldx, const float *norm_weight, float eps,
         void *out, int ldo, int out_dtype, xfthip_stream_t stream) {
     XFT_REQUIRE(w && x && norm_weight && out, "xfthip_gemm_gateup_silu_rmsnorm: null argument");

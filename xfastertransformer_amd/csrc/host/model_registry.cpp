@@ -1,0 +1,410 @@
+// Readers and registry of model_registry.h.
+#include "model_registry.h"
+
+#include <fcntl.h>
+#include <sys/mman.h>
+#include <sys/stat.h>
+#include <unistd.h>
+
+#include <cctype>
+#include <cstdio>
+#include <cstdlib>
+#include <cstring>
+#include <fstream>
+#include <sstream>
+
+#include "host_util.h"
+
+namespace xfthost {
+
+namespace {
+
+[[noreturn]] void broken(const std::string &what) {
+    printf("Could not load the model: %s\n", what.c_str());
+    exit(-1);
+}
+
+struct Parser {
+    const char *p, *end;
+    std::string error;
+    int depth = 0;
+
+    bool fail(const char *what) {
+        if (error.empty()) error = what;
+        return false;
+    }
+    void space() {
+        while (p < end && (*p == ' ' || *p == '\t' || *p == '\n' || *p == '\r')) ++p;
+    }
+    bool word(const char *w) {
+        const size_t n = strlen(w);
+        if ((size_t)(end - p) < n || strncmp(p, w, n) != 0) return fail("unknown word");
+        p += n;
+        return true;
+    }
+    static void utf8(std::string &s, unsigned c) {
+        if (c < 0x80) s += (char)c;
+        else if (c < 0x800) s += (char)(0xC0 | (c >> 6)), s += (char)(0x80 | (c & 63));
+        else if (c < 0x10000) s += (char)(0xE0 | (c >> 12)), s += (char)(0x80 | ((c >> 6) & 63)), s += (char)(0x80 | (c & 63));
+        else s += (char)(0xF0 | (c >> 18)), s += (char)(0x80 | ((c >> 12) & 63)), s += (char)(0x80 | ((c >> 6) & 63)), s += (char)(0x80 | (c & 63));
+    }
+    bool hex4(unsigned &c) {
+        c = 0;
+        for (int i = 0; i < 4; ++i) {
+            if (p >= end || !isxdigit((unsigned char)*p)) return fail("bad \\u escape");
+            const char d = *p++;
+            c = c * 16 + (unsigned)(d <= '9' ? d - '0' : (d | 32) - 'a' + 10);
+        }
+        return true;
+    }
+    bool str(std::string &out) {
+        ++p; // the quote
+        while (p < end && *p != '"') {
+            if (*p != '\\') {
+                out += *p++;
+                continue;
+            }
+            if (++p >= end) break;
+            const char e = *p++;
+            switch (e) {
+                case 'n': out += '\n'; break;
+                case 't': out += '\t'; break;
+                case 'r': out += '\r'; break;
+                case 'b': out += '\b'; break;
+                case 'f': out += '\f'; break;
+                case 'u': {
+                    unsigned c;
+                    if (!hex4(c)) return false;
+                    if (c >= 0xD800 && c < 0xDC00 && end - p >= 6 && p[0] == '\\' && p[1] == 'u') {
+                        unsigned lo;
+                        p += 2;
+                        if (!hex4(lo)) return false;
+                        c = 0x10000 + ((c - 0xD800) << 10) + (lo - 0xDC00);
+                    }
+                    utf8(out, c);
+                    break;
+                }
+                default: out += e;
+            }
+        }
+        if (p >= end) return fail("unterminated string");
+        ++p;
+        return true;
+    }
+    bool value(Json &v) {
+        space();
+        if (p >= end) return fail("unexpected end");
+        if (++depth > 64) return fail("nested too deeply");
+        bool ok = true;
+        switch (*p) {
+            case '{':
+                v.kind = Json::Object;
+                ++p, space();
+                if (p < end && *p == '}') {
+                    ++p;
+                    break;
+                }
+                for (;;) {
+                    space();
+                    if (p >= end || *p != '"') return fail("a key is missing");
+                    std::string key;
+                    if (!str(key)) return false;
+                    space();
+                    if (p >= end || *p != ':') return fail("a colon is missing");
+                    ++p;
+                    if (!value(v.fields[key])) return false;
+                    space();
+                    if (p < end && *p == ',') {
+                        ++p;
+                        continue;
+                    }
+                    if (p < end && *p == '}') {
+                        ++p;
+                        break;
+                    }
+                    return fail("an object does not end");
+                }
+                break;
+            case '[':
+                v.kind = Json::Array;
+                ++p, space();
+                if (p < end && *p == ']') {
+                    ++p;
+                    break;
+                }
+                for (;;) {
+                    v.items.emplace_back();
+                    if (!value(v.items.back())) return false;
+                    space();
+                    if (p < end && *p == ',') {
+                        ++p;
+                        continue;
+                    }
+                    if (p < end && *p == ']') {
+                        ++p;
+                        break;
+                    }
+                    return fail("an array does not end");
+                }
+                break;
+            case '"': v.kind = Json::String, ok = str(v.text); break;
+            case 't': v.kind = Json::Bool, v.flag = true, ok = word("true"); break;
+            case 'f': v.kind = Json::Bool, ok = word("false"); break;
+            case 'n': ok = word("null"); break;
+            default: {
+                const std::string rest(p, end - p < 64 ? end : p + 64);
+                char *stop = nullptr;
+                v.kind = Json::Number;
+                v.number = strtod(rest.c_str(), &stop);
+                if (stop == rest.c_str()) return fail("not a value");
+                p += stop - rest.c_str();
+            }
+        }
+        --depth;
+        return ok;
+    }
+};
+
+std::string read_file(const std::string &path, bool &ok) {
+    std::ifstream f(path, std::ios::binary);
+    ok = (bool)f;
+    std::stringstream s;
+    if (ok) s << f.rdbuf();
+    return s.str();
+}
+
+} // namespace
+
+bool Json::parse(const std::string &src, Json &out, std::string &error) {
+    Parser ps {src.data(), src.data() + src.size(), "", 0};
+    out = Json();
+    bool ok = ps.value(out);
+    ps.space();
+    if (ok && ps.p != ps.end) ok = ps.fail("text behind the value");
+    error = ps.error;
+    return ok;
+}
+
+bool Json::has(const std::string &key) const {
+    auto it = fields.find(key);
+    return it != fields.end() && it->second.kind != Null;
+}
+const Json &Json::at(const std::string &key) const {
+    auto it = fields.find(key);
+    if (it == fields.end()) broken("config.json lacks '" + key + "'");
+    return it->second;
+}
+long Json::integer(const std::string &key) const {
+    const double v = real(key);
+    if (v != (double)(long)v) broken("'" + key + "' of config.json is not a whole number");
+    return (long)v;
+}
+double Json::real(const std::string &key) const {
+    const Json &v = at(key);
+    if (v.kind != Number) broken("'" + key + "' of config.json is not a number");
+    return v.number;
+}
+const std::string &Json::string(const std::string &key) const {
+    const Json &v = at(key);
+    if (v.kind != String) broken("'" + key + "' of config.json is not a string");
+    return v.text;
+}
+
+long TensorRef::count() const {
+    long n = 1;
+    for (long d : shape) n *= d;
+    return n;
+}
+
+SafeTensors::~SafeTensors() {
+    if (base) munmap(base, length);
+}
+
+bool SafeTensors::open(const std::string &path, std::string &error) {
+    const int fd = ::open(path.c_str(), O_RDONLY);
+    struct stat st;
+    if (fd < 0 || fstat(fd, &st) != 0 || st.st_size < 8) {
+        if (fd >= 0) close(fd);
+        error = "cannot read " + path;
+        return false;
+    }
+    length = (size_t)st.st_size;
+    base = mmap(nullptr, length, PROT_READ, MAP_PRIVATE, fd, 0);
+    close(fd);
+    if (base == MAP_FAILED) {
+        base = nullptr;
+        error = "cannot map " + path;
+        return false;
+    }
+    const unsigned char *b = (const unsigned char *)base;
+    uint64_t header = 0;
+    for (int i = 7; i >= 0; --i) header = header << 8 | b[i];
+    if (header > length - 8) {
+        error = path + " is shorter than its header says";
+        return false;
+    }
+    Json j;
+    if (!Json::parse(std::string((const char *)b + 8, (size_t)header), j, error) || j.kind != Json::Object) {
+        error = "header of " + path + ": " + error;
+        return false;
+    }
+    const size_t room = length - 8 - (size_t)header;
+    for (auto &kv : j.fields) {
+        if (kv.first == "__metadata__") continue;
+        TensorRef t;
+        t.dtype = kv.second.string("dtype");
+        long n = 1;
+        for (const Json &d : kv.second.at("shape").items) t.shape.push_back((long)d.number), n *= (long)d.number;
+        const Json &off = kv.second.at("data_offsets");
+        const size_t width = t.dtype == "BF16" || t.dtype == "F16" || t.dtype == "I16" ? 2 : t.dtype == "F32" || t.dtype == "I32" ? 4 : t.dtype == "F64" || t.dtype == "I64" ? 8 : 1;
+        if (off.items.size() != 2 || off.items[0].number < 0 || off.items[1].number < off.items[0].number || off.items[1].number > (double)room
+                || n < 0 || (double)n * width != off.items[1].number - off.items[0].number) {
+            error = "tensor " + kv.first + " of " + path + " does not fit the file";
+            return false;
+        }
+        t.data = b + 8 + header + (size_t)off.items[0].number;
+        t.bytes = (size_t)(off.items[1].number - off.items[0].number);
+        tensors[kv.first] = t;
+    }
+    return true;
+}
+
+const TensorRef *SafeTensors::find(const std::string &name) const {
+    auto it = tensors.find(name);
+    return it == tensors.end() ? nullptr : &it->second;
+}
+
+namespace {
+
+long first_dim(const SafeTensors &w, const std::string &name) {
+    const TensorRef *t = w.find(name);
+    if (!t || t->shape.empty()) broken("model.safetensors lacks " + name);
+    return t->shape[0];
+}
+
+// ---- Pinepel: latent attention (windowed with interleaved rotation, or over everything with a sink and half rotation) and a
+// channel-wise gated delta rule, clamped gated feed-forwards, a norm on both sides of every sublayer, layers run in a loop ----
+PlanSpec pinepel(const Json &c, const SafeTensors &w) {
+    PlanSpec s;
+    s.cfg.hidden = (int)c.integer("width");
+    s.cfg.vocab = (int)c.integer("vocab");
+    s.cfg.eps = (float)c.at("norm").real("eps");
+    s.cfg.logit_scale = (float)c.real("logit_scale");
+    s.cfg.loop_times = 1;
+    if (c.has("loop")) {
+        const Json &l = c.at("loop");
+        s.cfg.loop_start = (int)l.integer("start"), s.cfg.loop_stop = (int)l.integer("stop"), s.cfg.loop_times = (int)l.integer("times");
+    }
+    const Json &layers = c.at("layers");
+    for (size_t i = 0; i < layers.items.size(); ++i) {
+        const Json &e = layers.items[i], &m = e.at("mixer");
+        const std::string &type = e.string("type"), mix = "l" + std::to_string(i) + ".mix.";
+        xfthip_plan_layer L {};
+        L.heads = (int)m.integer("heads"), L.dim = (int)m.integer("dim"), L.vdim = (int)m.integer("vdim");
+        if (type == "latent_attention" || type == "latent_attention_2") {
+            const bool windowed = type == "latent_attention";
+            L.mixer = XFTHIP_MIXER_LATENT;
+            L.kv_rank = (int)m.integer("kv_rank"), L.q_rank = (int)m.integer("q_rank"), L.rot_dim = (int)m.integer("rot_dim");
+            L.scale = (float)m.real("scale");
+            L.rot_base = m.at("rot").real("base");
+            if (m.at("rot").integer("dims") != L.rot_dim) broken("layer " + std::to_string(i) + ": rot.dims differs from rot_dim");
+            L.rot_interleaved = windowed ? 1 : 0;
+            L.window = windowed ? (int)m.at("mask").integer("size") : 0;
+            if (windowed && L.window < 1) broken("layer " + std::to_string(i) + ": an empty window");
+            L.has_sink = windowed ? 0 : 1;
+        } else if (type == "channel_delta") {
+            L.mixer = XFTHIP_MIXER_DELTA;
+            L.kv_heads = (int)m.integer("kv_heads"), L.taps = (int)m.integer("conv");
+            L.decay_rank = (int)first_dim(w, mix + "a1"), L.gate_rank = (int)first_dim(w, mix + "g1");
+        } else {
+            broken("layer type '" + type + "' of config.json is not known");
+        }
+        if (e.has("mlp")) {
+            const Json &f = e.at("mlp");
+            if (f.string("kind") != "dense") broken("feed-forward '" + f.string("kind") + "' of config.json is not known");
+            L.inter = (int)f.integer("ff");
+            L.glu_limit = (float)f.real("limit");
+            L.glu_alpha = 1.702f;
+        }
+        s.layers.push_back(L);
+    }
+    s.cfg.layers = (int)s.layers.size();
+    return s;
+}
+
+struct Architecture {
+    const char *name;
+    PlanSpec (*describe)(const Json &config, const SafeTensors &weights);
+};
+const Architecture kArchitectures[] = {{"Pinepel", pinepel}};
+
+const Architecture *find_architecture(const Json &c) {
+    if (c.kind != Json::Object || !c.has("architecture") || c.at("architecture").kind != Json::String) return nullptr;
+    for (const Architecture &a : kArchitectures)
+        if (c.at("architecture").text == a.name) return &a;
+    return nullptr;
+}
+
+} // namespace
+
+bool plan_architecture(const std::string &dir, std::string &name) {
+    bool ok = false;
+    const std::string src = read_file(dir + "/config.json", ok);
+    Json c;
+    std::string error;
+    if (!ok || !Json::parse(src, c, error)) return false;
+    const Architecture *a = find_architecture(c);
+    if (a) name = a->name;
+    return a != nullptr;
+}
+
+xfthip_plan_t load_plan(const std::string &dir, PlanSpec &spec) {
+    bool ok = false;
+    const std::string src = read_file(dir + "/config.json", ok);
+    Json c;
+    std::string error;
+    if (!ok) broken("cannot read " + dir + "/config.json");
+    if (!Json::parse(src, c, error)) broken("config.json: " + error);
+    const Architecture *a = find_architecture(c);
+    if (!a) broken("the architecture of config.json is not known");
+    SafeTensors w;
+    if (!w.open(dir + "/model.safetensors", error)) broken(error);
+    spec = a->describe(c, w);
+    xfthip_plan_t plan = nullptr;
+    CK(xfthip_plan_create(&spec.cfg, spec.layers.data(), &plan));
+    std::vector<uint16_t> widened;
+    for (auto &kv : w.all()) {
+        // 'l<i>.<name>' belongs to layer i, everything else to the model
+        int layer = -1;
+        std::string name = kv.first;
+        if (name.size() > 2 && name[0] == 'l' && isdigit((unsigned char)name[1])) {
+            char *end = nullptr;
+            const long i = strtol(name.c_str() + 1, &end, 10);
+            if (*end == '.' && i < spec.cfg.layers) layer = (int)i, name = std::string(end + 1);
+        }
+        const TensorRef &t = kv.second;
+        const long rows = t.shape.empty() ? 1 : t.shape[0], n = t.count();
+        if (rows <= 0 || n <= 0) continue;
+        const uint16_t *data = (const uint16_t *)t.data;
+        if (t.dtype == "F32") {
+            widened.resize((size_t)n);
+            for (long i = 0; i < n; ++i) {
+                float f;
+                memcpy(&f, t.data + 4 * i, 4);
+                widened[(size_t)i] = to_bf16(f);
+            }
+            data = widened.data();
+        } else if (t.dtype != "BF16") {
+            continue; // integer tables: none of the known plans has any
+        } else if ((uintptr_t)t.data & 1) {
+            widened.resize((size_t)n);
+            memcpy(widened.data(), t.data, (size_t)n * 2);
+            data = widened.data();
+        }
+        CK(xfthip_plan_set_tensor(plan, layer, name.c_str(), data, (int)rows, (int)(n / rows)));
+    }
+    CK(xfthip_plan_finish(plan));
+    return plan;
+}
+
+} // namespace xfthost

@@ -29,6 +29,7 @@
 #include "../../../include/models.h"
 #include "../../../include/xft_hip.h"
 #include "host_util.h"
+#include "model_registry.h"
 
 using namespace xfthost;
 
@@ -456,6 +457,25 @@ struct ModelImpl {
     xfthip_model_t model = nullptr;
     xfthip_model_config cfg {};
 
+    // models from config.json (model_registry.h): the layer plan instead of the uniform stack's weights above
+    xfthip_plan_t plan = nullptr;
+    PlanSpec planSpec;
+    int planAct = XFTHIP_BF16;
+    int poolTokens = 0; // tokens of the page pool over all sequences; 0: cache rows times their length
+
+    // device bytes of one sequence of `len` positions
+    double plan_row_bytes(int len) const {
+        double b = 0;
+        const int times = planSpec.cfg.loop_times > 1 ? planSpec.cfg.loop_times : 1;
+        for (int i = 0; i < planSpec.cfg.layers; ++i) {
+            const xfthip_plan_layer &y = planSpec.layers[i];
+            const int runs = i >= planSpec.cfg.loop_start && i < planSpec.cfg.loop_stop ? times : 1;
+            const double e = planAct == XFTHIP_F32 ? 4 : 2;
+            b += runs * (y.mixer == XFTHIP_MIXER_LATENT ? (double)len * (y.kv_rank + y.rot_dim) * e : (double)y.heads * y.dim * y.vdim * 4);
+        }
+        return b;
+    }
+
     // searcher state (GreedySearch / SampleSearch members of the reference)
     bool haveSearcher = false, sampling = false;
     int maxLen = 0, eosTokenId = -1, padTokenId = -1, topK = 50;
@@ -510,7 +530,7 @@ struct ModelImpl {
             size_t free_b = 0;
             if (xfthip_device_memory(&free_b, nullptr) == 0 && free_b > 0) {
                 const double per_value = cfg.kv_dtype == XFTHIP_INT8 ? 1.0 + 4.0 / cfg.head_size : 2.0;
-                const double row_b = (double)cfg.layers * 2.0 * cfg.kv_heads * ((maxLen + 1 + 31) / 32 * 32) * cfg.head_size * per_value;
+                const double row_b = plan ? plan_row_bytes(maxLen + 1) : (double)cfg.layers * 2.0 * cfg.kv_heads * ((maxLen + 1 + 31) / 32 * 32) * cfg.head_size * per_value;
                 const double fit_rows_d = 0.4 * (double)free_b / (row_b > 1.0 ? row_b : 1.0);
                 rows = fit_rows_d >= 64.0 ? 64 : (fit_rows_d <= 8.0 ? 8 : (int)fit_rows_d);
             }
@@ -550,6 +570,7 @@ struct ModelImpl {
                 if (w) xfthip_weight_destroy(w);
         }
         if (lmHead) xfthip_weight_destroy(lmHead);
+        if (plan) xfthip_plan_destroy(plan);
     }
 
     // the sparse MLPs work in the first one's buffers: the others go first
@@ -681,6 +702,14 @@ struct ModelImpl {
         model = nullptr;
         prefixOnDevice = false;
         drop_moe();
+        if (plan) {
+            cfg.max_batch = std::max(cfg.max_batch, B);
+            cfg.max_tokens = std::max(std::max(cfg.max_tokens, B * S), cfg.max_batch);
+            cfg.max_seq = std::max(cfg.max_seq, needLen);
+            const int pool = poolTokens > 0 ? std::max(poolTokens, B * needLen) : 0;
+            CK(xfthip_model_create_from_plan(plan, planAct, cfg.max_batch, cfg.max_seq, cfg.max_tokens, pool, &model));
+            return;
+        }
         cfg.layers = layers, cfg.hidden = hidden, cfg.intermediate = inter;
         cfg.q_heads = heads, cfg.kv_heads = kvHeads, cfg.head_size = headSize;
         cfg.vocab = vocab;
@@ -718,7 +747,8 @@ struct ModelImpl {
     // The prompt pass of a lockstep input.  With a prefix set, the first prefix.size() tokens of every sequence are
     // taken to be the prefix (as the reference takes them, common_decoder.h:337-350) and only the rest runs.
     void prompt_pass(const std::vector<int32_t> &ids, int B, int S, float *logits) {
-        if (prefix.empty()) {
+        if (prefix.empty() || plan) {
+            // (a plan's recurrent layers keep no state from the middle of a sequence: its prompts run whole)
             prefixOnDevice = false;
             CK(xfthip_model_prefill(model, ids.data(), B, S, logits, nullptr));
             return;
@@ -1542,7 +1572,135 @@ void Model::initMaxSeqLen() {
     maxSeqLen = impl->maxSeqLength > 0 ? impl->maxSeqLength : impl->maxPositions;
 }
 
+// ---- steps of unequal parts ------------------------------------------------------------------------
+void Model::setCachePool(int tokens, int sequences) {
+    ModelImpl &s = *impl;
+    if (!s.plan) unsupported("Model::setCachePool for a model without a page pool");
+    if (tokens <= 0 || sequences <= 0) {
+        printf("[ERROR] Model::setCachePool(%d, %d).\n", tokens, sequences);
+        exit(-1);
+    }
+    if (!s.pool.empty()) {
+        printf("[ERROR] %zu sequences are alive; free them before the pool changes.\n", s.pool.size());
+        exit(-1);
+    }
+    if (s.model) CK(xfthip_model_destroy(s.model));
+    s.model = nullptr;
+    s.poolTokens = tokens;
+    s.cfg.max_batch = sequences, s.cfg.max_seq = tokens;
+    s.cfg.max_tokens = std::max(std::min(tokens, 8192), sequences);
+    CK(xfthip_model_create_from_plan(s.plan, s.planAct, sequences, s.cfg.max_seq, s.cfg.max_tokens, tokens, &s.model));
+}
+
+std::tuple<float *, int, int> Model::step(std::vector<StepEntry> &entries) {
+    ModelImpl &s = *impl;
+    if (!s.plan) unsupported("Model::step for this model");
+    if (entries.empty()) {
+        printf("[ERROR] Model::step without entries.\n");
+        exit(-1);
+    }
+    s.cbMode = true;
+    s.working.clear();
+    if (!s.model) setCachePool(maxSeqLen, 8);
+    const int n = (int)entries.size();
+    std::vector<int> done(n, 0), rows(n);
+    std::vector<size_t> firstLogits(n);
+    size_t total = 0;
+    for (int i = 0; i < n; ++i) {
+        StepEntry &e = entries[i];
+        if (e.tokens.empty()) {
+            printf("[ERROR] Empty input for a sequence.\n");
+            exit(-1);
+        }
+        for (int w : e.want)
+            if (w < 0 || w >= (int)e.tokens.size()) {
+                printf("[ERROR] Logits of token %d of %zu asked for.\n", w, e.tokens.size());
+                exit(-1);
+            }
+        for (int32_t t : e.tokens)
+            if (t < 0 || t >= s.vocab) {
+                printf("[ERROR] Token %d is outside the vocabulary.\n", t);
+                exit(-1);
+            }
+        if (e.seqID < 0) {
+            ModelImpl::Seq q;
+            q.id = s.nextSeqId++;
+            q.forwardOnly = true;
+            q.row = s.free_row();
+            if (q.row < 0) {
+                printf("[ERROR] No free sequence slot.\n");
+                exit(-1);
+            }
+            s.pool[q.id] = q;
+            e.seqID = q.id;
+        }
+        auto it = s.pool.find(e.seqID);
+        if (it == s.pool.end()) {
+            printf("[ERROR] Sequence ID %d not found.\n", e.seqID);
+            exit(-1);
+        }
+        rows[i] = it->second.row;
+        it->second.prompt.insert(it->second.prompt.end(), e.tokens.begin(), e.tokens.end());
+        it->second.step++;
+        s.working.push_back(e.seqID);
+        firstLogits[i] = total;
+        total += e.want.size();
+    }
+    s.logitsHost.resize(total * (size_t)s.vocab);
+    // as few passes as the model's token capacity allows (one, unless the step is larger than that)
+    for (;;) {
+        std::vector<int> r, lens, ids, want, dest;
+        int room = s.cfg.max_tokens;
+        for (int i = 0; i < n && room > 0; ++i) {
+            const StepEntry &e = entries[i];
+            const int k = std::min(room, (int)e.tokens.size() - done[i]);
+            if (k <= 0) continue;
+            for (size_t j = 0; j < e.want.size(); ++j)
+                if (e.want[j] >= done[i] && e.want[j] < done[i] + k) {
+                    want.push_back((int)ids.size() + e.want[j] - done[i]);
+                    dest.push_back((int)(firstLogits[i] + j));
+                }
+            r.push_back(rows[i]), lens.push_back(k);
+            ids.insert(ids.end(), e.tokens.begin() + done[i], e.tokens.begin() + done[i] + k);
+            done[i] += k;
+            room -= k;
+        }
+        if (r.empty()) break;
+        std::vector<float> lg(want.size() * (size_t)s.vocab);
+        CK(xfthip_model_step(s.model, (int)r.size(), r.data(), lens.data(), ids.data(), (int)want.size(), want.data(), lg.data(), nullptr));
+        for (size_t j = 0; j < want.size(); ++j)
+            memcpy(s.logitsHost.data() + (size_t)dest[j] * s.vocab, lg.data() + j * s.vocab, (size_t)s.vocab * 4);
+    }
+    return std::make_tuple(s.logitsHost.data(), (int)total, s.vocab);
+}
+
 AutoModel::AutoModel(std::string modelPath, xft::DataType dataType, xft::DataType KVCacheDataType) : Model() {
+    std::string architecture;
+    if (!file_exists(modelPath + "/config.ini") && plan_architecture(modelPath, architecture)) {
+        const bool full = dataType == xft::DataType::fp32;
+        if ((!full && dataType != xft::DataType::bf16 && dataType != xft::DataType::fp16) || KVCacheDataType != xft::DataType::fp16) {
+            // (the cache holds the activations' own type; the weights are bf16)
+            printf("Unsupported data type or KV cache data type: %s-%s-%s\n", architecture.c_str(), type_name(dataType), type_name(KVCacheDataType));
+            exit(-1);
+        }
+        ensure_init();
+        impl = new ModelImpl();
+        ModelImpl &s = *impl;
+        s.path = modelPath;
+        s.modelType = architecture;
+        s.planAct = full ? XFTHIP_F32 : XFTHIP_BF16;
+        s.plan = load_plan(modelPath, s.planSpec);
+        s.weightBytes = xfthip_plan_weight_bytes(s.plan);
+        s.layers = s.planSpec.cfg.layers, s.hidden = s.planSpec.cfg.hidden, s.vocab = s.planSpec.cfg.vocab;
+        s.startId = 0, s.endId = -1; // such a directory names no end token: the caller does
+        // nothing in it bounds the positions either; XFT_MAX_POSITIONS does
+        s.maxPositions = 8192;
+        if (const char *e = getenv("XFT_MAX_POSITIONS"))
+            if (atoi(e) > 0) s.maxPositions = atoi(e);
+        setVocabSize(s.vocab);
+        maxSeqLen = s.maxPositions;
+        return;
+    }
     const std::string configPath = modelPath + "/config.ini";
     Ini ini(configPath);
     if (!ini.ok || ini.sections.empty()) {
@@ -1671,6 +1829,12 @@ static xft::DataType dtype_from_name(const char *name) {
     return xft::DataType::unknown;
 }
 
+// is the directory one of a model described by config.json (a layer plan)
+int xft_automodel_is_plan(const char *path) {
+    std::string name;
+    return !file_exists(std::string(path) + "/config.ini") && plan_architecture(path, name) ? 1 : 0;
+}
+
 void *xft_automodel_create(const char *path, const char *dtype, const char *kv_dtype) {
     return new xft::AutoModel(path, dtype_from_name(dtype), dtype_from_name(kv_dtype));
 }
@@ -1756,6 +1920,25 @@ void xft_automodel_set_prefix(void *h, const int *ids, int n) {
     }
     std::vector<int32_t> v(ids, ids + n);
     ((xft::AutoModel *)h)->setPrefix(v);
+}
+
+void xft_automodel_set_cache_pool(void *h, int tokens, int sequences) {
+    ((xft::AutoModel *)h)->setCachePool(tokens, sequences);
+}
+
+// Model::step: entry i brings lens[i] tokens (ids back to back) of sequence seq_ids[i] (-1: a new one, its id is written
+// there) and asks for the logits of wants[i] of them (places back to back in want); logits_out fp32 [sum of wants, vocab]
+void xft_automodel_step(void *h, int n, int *seq_ids, const int *lens, const int *ids, const int *wants, const int *want, float *logits_out) {
+    std::vector<xft::StepEntry> entries(n);
+    for (int i = 0; i < n; ++i) {
+        entries[i].seqID = seq_ids[i];
+        entries[i].tokens.assign(ids, ids + lens[i]);
+        entries[i].want.assign(want, want + wants[i]);
+        ids += lens[i], want += wants[i];
+    }
+    auto t = ((xft::AutoModel *)h)->step(entries);
+    for (int i = 0; i < n; ++i) seq_ids[i] = entries[i].seqID;
+    if (std::get<1>(t) > 0) memcpy(logits_out, std::get<0>(t), (size_t)std::get<1>(t) * std::get<2>(t) * 4);
 }
 
 int xft_automodel_free_seqs(void *h, const int *seq_ids, int n) {

@@ -18,23 +18,10 @@
 #include <utility>
 #include <vector>
 
-#include "attention_dev.h"
-#include "kvcache.h"
-#include "qgemm.h"
+#include "model_impl.h"
+#include "plan.h"
 
 namespace xfthip {
-
-struct LayerW {
-    xfthip_weight_t qkv = nullptr, o = nullptr, gateup = nullptr, down = nullptr;
-    // optional second set used by the prompt pass only (the reference's HybridModel: one weight type for the
-    // first token, another for the following ones, src/models/hybrid_model.h:25-84)
-    xfthip_weight_t first_qkv = nullptr, first_o = nullptr, first_gateup = nullptr, first_down = nullptr;
-    float *ln1 = nullptr, *ln2 = nullptr, *qkv_bias = nullptr, *o_bias = nullptr;
-    // set: the layer's two norms are LayerNorms with these shifts (NormType::LN of the layer API) instead of RMSNorms
-    float *ln1_beta = nullptr, *ln2_beta = nullptr;
-    // set: the layer's MLP is this sparse one (MixtralMLP; it carries its own norm weight and router), not gateup / down
-    xfthip_moe_t moe = nullptr;
-};
 
 __global__ void embed_kernel(const uint16_t *__restrict__ table, const int *__restrict__ ids, float *__restrict__ x,
         int hidden, int vocab) {
@@ -58,8 +45,9 @@ __global__ void gather_last_kernel(const float *__restrict__ x, float *__restric
 // here so that the step needs no launches of its own for them
 // active: optional per-row flags; a row whose flag is 0 keeps its id and its position (a sequence
 // that sits out this step of a continuously batched decode)
+// rows: optional, where row b's id and position live (b itself without)
 __global__ __launch_bounds__(1024) void argmax_kernel(const float *__restrict__ logits, int cols, int *__restrict__ ids,
-        int *advance_pos, int *advance_step, const int *__restrict__ active) {
+        int *advance_pos, int *advance_step, const int *__restrict__ active, const int *__restrict__ rows) {
     __shared__ float sv[1024];
     __shared__ int si[1024];
     const float *p = logits + (size_t)blockIdx.x * cols;
@@ -96,8 +84,9 @@ __global__ __launch_bounds__(1024) void argmax_kernel(const float *__restrict__ 
     }
     if (threadIdx.x == 0) {
         const bool on = active == nullptr || active[blockIdx.x] != 0;
-        if (on) ids[blockIdx.x] = si[0];
-        if (advance_pos && on) advance_pos[blockIdx.x] += 1;
+        const int at = rows ? rows[blockIdx.x] : blockIdx.x;
+        if (on) ids[at] = si[0];
+        if (advance_pos && on) advance_pos[at] += 1;
         if (advance_step && blockIdx.x == 0) advance_step[0] += 1;
     }
 }
@@ -155,57 +144,16 @@ __global__ void fill_int_kernel(int *p, int n, int v) {
     if (i < n) p[i] = v;
 }
 
+int argmax_rows(const float *logits, int n, int cols, int *ids, const int *rows, int *advance_pos, int *advance_step, hipStream_t st) {
+    hipLaunchKernelGGL(argmax_kernel, dim3(n), dim3(1024), 0, st, logits, cols, ids, advance_pos, advance_step, (const int *)nullptr, rows);
+    XFT_CHECK_HIP(hipGetLastError());
+    return 0;
+}
+
 
 } // namespace xfthip
 
 using namespace xfthip;
-
-struct xfthip_model {
-    xfthip_model_config cfg;
-    std::vector<LayerW> layers;
-    std::vector<xfthip_kvcache_t> caches;
-    // INT8 KV: the first-token pass attends over unquantised keys/values, as the reference's
-    // flash path does on its bf16 copies (src/layers/attention.h:1121-1188); they live here
-    xfthip_kvcache_t prefill_cache = nullptr;
-    AttnWorkspace attn_ws; // split-KV partials and tickets of this model's attention launches
-    // W8A8 layers: int8 activation rows + per-row (scale, zero, sum), and the [tokens, 2 * inter]
-    // bf16 result of the gate/up projection (which runs as a plain GEMM for this kind)
-    int8_t *w8a8_qa = nullptr;
-    size_t w8a8_qa_bytes = 0;
-    float *w8a8_stat = nullptr;
-    uint16_t *gu = nullptr;
-    float *cosT = nullptr, *sinT = nullptr;
-    // scratch
-    uint16_t *xn = nullptr, *qkv = nullptr, *att = nullptr, *h = nullptr;
-    float *x = nullptr, *xlast = nullptr, *logits = nullptr;
-    int *ids = nullptr, *pos = nullptr, *step = nullptr, *idlog = nullptr;
-    int idlog_cap = 0;
-    // head
-    uint16_t *embedding = nullptr;
-    float *final_norm = nullptr;
-    xfthip_weight_t lm_head = nullptr;
-    // decode state
-    int cur_B = 0, cur_pos = 0;
-    int prompt_rows = 0; // rows of `x` that hold the last layer's output of the most recent prompt pass (0 after a decode step)
-    int prefix_len = 0; // positions [0, prefix_len) of cache row 0 hold a shared prefix (xfthip_model_set_prefix)
-    // continuous batching: sequences live in cache rows of their own, each at its own position
-    int row0 = 0; // cache row of the first sequence of the forward call in flight
-    bool ragged = false; // rows may differ in position or sit out a step (set by the xfthip_model_seq_* calls)
-    int *active = nullptr; // device [max_batch]: rows taking part in the next decode call
-    int *prompt_ids = nullptr; // device [max_tokens]: prompt of a single-sequence prefill
-    std::vector<int> row_pos; // host copy of every row's position (-1 = free row)
-    unsigned char *kv_stage = nullptr; // staging buffer of xfthip_model_seq_reorder (grown on demand)
-    size_t kv_stage_bytes = 0;
-    int *reorder_rows = nullptr; // device [2 * max_batch]: source rows, destination rows
-    hipGraphExec_t graph = nullptr;
-    int graph_B = 0;
-    int graph_nsplit = 0; // attention split count the captured step was built with
-    bool graph_ragged = false; // the captured step's last node holds the `active` mask only in this mode
-    int len_hint = 0; // upper bound of the sequence length during the current decode call (0 = unknown)
-    hipStream_t graph_stream = nullptr;
-    bool use_graph = true;
-    bool fuse_decode = true; // RMSNorm prologue / RoPE + cache-append epilogue inside the decode GEMVs
-};
 
 // While one of these lives, the layers that hold first-token weights run with them.
 struct FirstTokenWeights {
@@ -430,13 +378,14 @@ static int head_forward(xfthip_model *m, const float *xrows, int B, bool advance
                  nullptr, 0, XFTHIP_F32, 1.0f, st)))
         return rc;
     hipLaunchKernelGGL(argmax_kernel, dim3(B), dim3(1024), 0, st, m->logits + (size_t)r0 * c.vocab, c.vocab, m->ids + r0,
-            advance ? m->pos + r0 : nullptr, advance ? m->step : nullptr, (advance && m->ragged) ? m->active + r0 : nullptr);
+            advance ? m->pos + r0 : nullptr, advance ? m->step : nullptr, (advance && m->ragged) ? m->active + r0 : nullptr, (const int *)nullptr);
     XFT_CHECK_HIP(hipGetLastError());
     return 0;
 }
 
 // the decode step that gets captured: everything reads its position from device memory
 static int decode_step(xfthip_model *m, int B, hipStream_t st) {
+    if (m->plan) return plan_decode_step(m, B, st);
     const xfthip_model_config &c = m->cfg;
     hipLaunchKernelGGL(decode_begin_kernel, dim3(B), dim3(256), 0, st, m->embedding, m->ids, m->x, c.hidden, c.vocab, m->idlog, m->step);
     for (int l = 0; l < c.layers; ++l)
@@ -449,7 +398,7 @@ extern "C" {
 int xfthip_argmax(const float *logits, int rows, int cols, int *ids_dev, xfthip_stream_t stream) {
     XFT_REQUIRE(logits && ids_dev && rows > 0 && cols > 0, "xfthip_argmax: bad argument");
     hipLaunchKernelGGL(argmax_kernel, dim3(rows), dim3(1024), 0, (hipStream_t)stream, logits, cols, ids_dev, (int *)nullptr, (int *)nullptr,
-            (const int *)nullptr);
+            (const int *)nullptr, (const int *)nullptr);
     XFT_CHECK_HIP(hipGetLastError());
     return 0;
 }
@@ -514,6 +463,10 @@ int xfthip_model_create(const xfthip_model_config *cfg, xfthip_model_t *out) {
 int xfthip_model_destroy(xfthip_model_t m) {
     if (!m) return 0;
     if (m->graph) (void)hipGraphExecDestroy(m->graph);
+    if (m->plan) {
+        plan_state_destroy(m->plan);
+        m->final_norm = nullptr; // the plan's
+    }
     for (auto c : m->caches) xfthip_kvcache_destroy(c);
     xfthip_kvcache_destroy(m->prefill_cache);
     attention_workspace_destroy(&m->attn_ws);
@@ -536,6 +489,7 @@ int xfthip_model_destroy(xfthip_model_t m) {
 int xfthip_model_set_attention(xfthip_model_t m, int idx, xfthip_weight_t qkv, xfthip_weight_t o, const float *ln1_host,
         const float *qkv_bias_host, const float *o_bias_host) {
     XFT_REQUIRE(m && qkv && o, "xfthip_model_set_attention: null argument");
+    XFT_REQUIRE(!m->plan, "xfthip_model_set_attention: the model follows a plan");
     XFT_REQUIRE(idx >= 0 && idx < m->cfg.layers, "xfthip_model_set_attention: layer %d out of range", idx);
     const xfthip_model_config &c = m->cfg;
     const int qcols = c.q_heads * c.head_size, qkv_cols = qcols + 2 * c.kv_heads * c.head_size;
@@ -561,6 +515,7 @@ int xfthip_model_set_attention(xfthip_model_t m, int idx, xfthip_weight_t qkv, x
 
 int xfthip_model_set_mlp(xfthip_model_t m, int idx, xfthip_weight_t gateup, xfthip_weight_t down, const float *ln2_host) {
     XFT_REQUIRE(m && gateup && down, "xfthip_model_set_mlp: null argument");
+    XFT_REQUIRE(!m->plan, "xfthip_model_set_mlp: the model follows a plan");
     XFT_REQUIRE(idx >= 0 && idx < m->cfg.layers, "xfthip_model_set_mlp: layer %d out of range", idx);
     const xfthip_model_config &c = m->cfg;
     // W8A8 gate/up weights stay in plain cat(gate, up) column order: the int8 GEMM has no fused SwiGLU
@@ -587,6 +542,7 @@ int xfthip_model_set_mlp(xfthip_model_t m, int idx, xfthip_weight_t gateup, xfth
 
 int xfthip_model_set_moe(xfthip_model_t m, int idx, xfthip_moe_t moe) {
     XFT_REQUIRE(m && moe, "xfthip_model_set_moe: null argument");
+    XFT_REQUIRE(!m->plan, "xfthip_model_set_moe: the model follows a plan");
     XFT_REQUIRE(idx >= 0 && idx < m->cfg.layers, "xfthip_model_set_moe: layer %d out of range", idx);
     const xfthip_model_config &c = m->cfg;
     int hidden = 0, inter = 0, experts = 0, max_tokens = 0;
@@ -614,7 +570,7 @@ int xfthip_model_set_layer(xfthip_model_t m, int idx, xfthip_weight_t qkv, xfthi
 }
 
 int xfthip_model_set_layer_norm_shifts(xfthip_model_t m, int idx, const float *ln1_beta_host, const float *ln2_beta_host) {
-    XFT_REQUIRE(m && idx >= 0 && idx < m->cfg.layers, "xfthip_model_set_layer_norm_shifts: bad model or layer");
+    XFT_REQUIRE(m && !m->plan && idx >= 0 && idx < m->cfg.layers, "xfthip_model_set_layer_norm_shifts: bad model or layer");
     LayerW &L = m->layers[idx];
     // a captured decode step holds the kernels of the other norm
     if (m->graph) {
@@ -629,7 +585,7 @@ int xfthip_model_set_layer_norm_shifts(xfthip_model_t m, int idx, const float *l
 
 int xfthip_model_set_first_token_weights(xfthip_model_t m, int idx, xfthip_weight_t qkv, xfthip_weight_t o, xfthip_weight_t gateup,
         xfthip_weight_t down) {
-    XFT_REQUIRE(m && idx >= 0 && idx < m->cfg.layers, "xfthip_model_set_first_token_weights: bad model or layer");
+    XFT_REQUIRE(m && !m->plan && idx >= 0 && idx < m->cfg.layers, "xfthip_model_set_first_token_weights: bad model or layer");
     LayerW &L = m->layers[idx];
     if (!qkv && !o && !gateup && !down) { // back to one weight set
         L.first_qkv = L.first_o = L.first_gateup = L.first_down = nullptr;
@@ -656,6 +612,7 @@ int xfthip_model_set_head(xfthip_model_t m, const uint16_t *embedding_fp16_host,
         xfthip_weight_t lm_head) {
     XFT_REQUIRE(m && embedding_fp16_host && final_norm_host && lm_head, "xfthip_model_set_head: null argument");
     const xfthip_model_config &c = m->cfg;
+    XFT_REQUIRE(!m->plan, "xfthip_model_set_head: the model follows a plan");
     XFT_REQUIRE(c.vocab > 0, "xfthip_model_set_head: model was created without a vocabulary");
     XFT_REQUIRE(lm_head->pw.K == c.hidden && lm_head->pw.N == c.vocab, "xfthip_model_set_head: lm_head is [%d,%d], expected [%d,%d]",
             lm_head->pw.K, lm_head->pw.N, c.hidden, c.vocab);
@@ -678,6 +635,7 @@ int xfthip_model_set_head(xfthip_model_t m, const uint16_t *embedding_fp16_host,
 static int check_forward(xfthip_model_t m, const char *fn, int idx, const void *x_in, const void *x_out, int in_stride,
         int out_stride, int B, int S, int past) {
     XFT_REQUIRE(m && x_in && x_out, "%s: null argument", fn);
+    XFT_REQUIRE(!m->plan, "%s: the model follows a plan", fn);
     XFT_REQUIRE(idx >= 0 && idx < m->cfg.layers, "%s: layer %d out of range", fn, idx);
     XFT_REQUIRE(B > 0 && B <= m->cfg.max_batch && S > 0 && B * S <= m->cfg.max_tokens, "%s: B=%d S=%d exceed max_batch=%d / max_tokens=%d",
             fn, B, S, m->cfg.max_batch, m->cfg.max_tokens);
@@ -709,6 +667,19 @@ int xfthip_model_mlp_forward(xfthip_model_t m, int idx, const float *x_in, int i
 // the prompt pass of B sequences of S tokens whose cache rows already hold `past` positions each
 static int prompt_pass(xfthip_model_t m, const char *who, const int *ids_host, int B, int S, int past, float *logits_host, hipStream_t st) {
     const xfthip_model_config &c = m->cfg;
+    if (m->plan) {
+        XFT_REQUIRE(B > 0 && B <= c.max_batch && S > 0 && B * S <= c.max_tokens && S <= c.max_seq, "%s: B=%d S=%d exceed the model limits", who, B, S);
+        m->row_pos.assign(c.max_batch, -1);
+        std::vector<int> rows(B);
+        for (int r = 0; r < c.max_batch; ++r) plan_release(m, r);
+        for (int b = 0; b < B; ++b) rows[b] = b;
+        m->ragged = false;
+        if (int rc = plan_prompt_pass(m, rows.data(), B, S, ids_host, logits_host, st)) return rc;
+        m->cur_B = B;
+        m->cur_pos = S;
+        m->prompt_rows = B * S;
+        return 0;
+    }
     XFT_REQUIRE(m->embedding && m->lm_head, "%s: embedding / lm_head not set", who);
     XFT_REQUIRE(B > 0 && B <= c.max_batch && S > 0 && B * S <= c.max_tokens && past + S <= c.max_seq, "%s: B=%d S=%d past=%d exceed the model limits",
             who, B, S, past);
@@ -742,6 +713,8 @@ int xfthip_model_prefill(xfthip_model_t m, const int *ids_host, int B, int S, fl
 
 int xfthip_model_set_prefix(xfthip_model_t m, const int *ids_host, int n, xfthip_stream_t stream) {
     XFT_REQUIRE(m && ids_host && n > 0, "xfthip_model_set_prefix: bad argument");
+    // (a recurrent state behind the prefix is gone as soon as its sequence goes on)
+    XFT_REQUIRE(!m->plan, "xfthip_model_set_prefix: the model follows a plan; run whole prompts");
     if (int rc = prompt_pass(m, "xfthip_model_set_prefix", ids_host, 1, n, 0, nullptr, (hipStream_t)stream)) return rc;
     m->prefix_len = n;
     return 0;
@@ -782,7 +755,15 @@ int xfthip_model_decode(xfthip_model_t m, int steps, int *ids_out_host, xfthip_s
     // (capture) time: it follows an upper bound of the length, rounded up so that the graph is
     // re-captured only every 128 tokens
     m->len_hint = ((m->cur_pos + steps + 127) / 128) * 128;
-    const int nsplit = attention_split_count(m->len_hint < c.max_seq ? m->len_hint : c.max_seq, B * c.kv_heads);
+    const int hint = m->len_hint < c.max_seq ? m->len_hint : c.max_seq;
+    if (m->plan) {
+        if (!m->ragged) {
+            m->plan->dec_list.resize(B);
+            for (int b = 0; b < B; ++b) m->plan->dec_list[b] = b;
+        }
+        if (int rc = plan_decode_begin(m, steps, st)) return rc;
+    }
+    const int nsplit = m->plan ? plan_decode_splits(m, B, hint) : attention_split_count(hint, B * c.kv_heads);
     if (!m->use_graph) {
         for (int i = 0; i < steps; ++i)
             if (int rc = decode_step(m, B, st)) return rc;
@@ -841,15 +822,63 @@ int xfthip_model_decode(xfthip_model_t m, int steps, int *ids_out_host, xfthip_s
     return 0;
 }
 
+int xfthip_model_step(xfthip_model_t m, int n, const int *rows_host, const int *lens_host, const int *ids_host, int n_want, const int *want_host,
+        float *logits_host, xfthip_stream_t stream) {
+    XFT_REQUIRE(m && n > 0 && rows_host && lens_host && ids_host && n_want >= 0 && (n_want == 0 || (want_host && logits_host)), "xfthip_model_step: bad argument");
+    XFT_REQUIRE(m->plan, "xfthip_model_step: only for models from a plan");
+    const xfthip_model_config &c = m->cfg;
+    hipStream_t st = (hipStream_t)stream;
+    if ((int)m->row_pos.size() != c.max_batch || !m->ragged) {
+        m->row_pos.assign(c.max_batch, -1);
+        for (int r = 0; r < c.max_batch; ++r) plan_release(m, r);
+    }
+    m->ragged = true;
+    long total = 0;
+    for (int i = 0; i < n; ++i) {
+        XFT_REQUIRE(lens_host[i] > 0, "xfthip_model_step: entry %d brings no tokens", i);
+        total += lens_host[i];
+    }
+    for (int i = 0; i < n_want; ++i) XFT_REQUIRE(want_host[i] >= 0 && want_host[i] < total, "xfthip_model_step: logits of token %d of %ld asked for", want_host[i], total);
+    if (int rc = plan_run(m, n, rows_host, lens_host, ids_host, st)) return rc;
+    m->prompt_rows = (int)total;
+    m->cur_B = 0;
+    for (int r = 0; r < c.max_batch; ++r)
+        if (m->row_pos[r] >= 0) m->cur_B = r + 1;
+    const int chunk = m->plan->logit_rows;
+    for (int i = 0; i < n_want; i += chunk) {
+        const int k = n_want - i < chunk ? n_want - i : chunk;
+        XFT_CHECK_HIP(hipMemcpyAsync(m->plan->want, want_host + i, (size_t)k * 4, hipMemcpyHostToDevice, st));
+        if (int rc = plan_head(m, m->plan->want, k, 0, st)) return rc;
+        XFT_CHECK_HIP(hipMemcpyAsync(logits_host + (size_t)i * c.vocab, m->logits, (size_t)k * c.vocab * 4, hipMemcpyDeviceToHost, st));
+        XFT_CHECK_HIP(hipStreamSynchronize(st));
+    }
+    XFT_CHECK_HIP(hipStreamSynchronize(st));
+    return 0;
+}
+
 // ---- continuous batching: sequences come and go, each in a cache row of its own ------------------
 int xfthip_model_seq_prefill(xfthip_model_t m, int row, const int *ids_host, int S, float *logits_host, xfthip_stream_t stream) {
     XFT_REQUIRE(m && ids_host, "xfthip_model_seq_prefill: null argument");
     const xfthip_model_config &c = m->cfg;
-    XFT_REQUIRE(m->embedding && m->lm_head, "xfthip_model_seq_prefill: embedding / lm_head not set");
+    XFT_REQUIRE(m->plan || (m->embedding && m->lm_head), "xfthip_model_seq_prefill: embedding / lm_head not set");
     XFT_REQUIRE(row >= 0 && row < c.max_batch, "xfthip_model_seq_prefill: row %d outside the %d cache rows", row, c.max_batch);
     XFT_REQUIRE(S > 0 && S <= c.max_tokens && S < c.max_seq, "xfthip_model_seq_prefill: %d tokens exceed max_tokens %d / max_seq %d", S,
             c.max_tokens, c.max_seq);
     hipStream_t st = (hipStream_t)stream;
+    if (m->plan) {
+        if ((int)m->row_pos.size() != c.max_batch || !m->ragged) {
+            m->row_pos.assign(c.max_batch, -1);
+            for (int r = 0; r < c.max_batch; ++r) plan_release(m, r);
+            m->cur_B = 0;
+        }
+        m->ragged = true;
+        plan_release(m, row);
+        m->row_pos[row] = -1;
+        if (int rc = plan_prompt_pass(m, &row, 1, S, ids_host, logits_host, st)) return rc;
+        if (row + 1 > m->cur_B) m->cur_B = row + 1;
+        m->prompt_rows = S;
+        return 0;
+    }
     if (row == 0) m->prefix_len = 0; // the row of a shared prefix is written from position 0
     if ((int)m->row_pos.size() != c.max_batch) m->row_pos.assign(c.max_batch, -1);
     if (!m->active) {
@@ -892,6 +921,7 @@ int xfthip_model_seq_release(xfthip_model_t m, int row) {
     XFT_REQUIRE(m && row >= 0 && row < m->cfg.max_batch, "xfthip_model_seq_release: bad row");
     if ((int)m->row_pos.size() != m->cfg.max_batch) m->row_pos.assign(m->cfg.max_batch, -1);
     m->row_pos[row] = -1;
+    if (m->plan) plan_release(m, row);
     // a free row keeps decoding along (at position 0, results dropped) until the rows above it are free too
     XFT_CHECK_HIP(hipDeviceSynchronize());
     int zero = 0;
@@ -907,7 +937,7 @@ int xfthip_model_seq_release(xfthip_model_t m, int row) {
 int xfthip_model_seq_decode(xfthip_model_t m, const int *rows_host, int n, int *ids_out_host, xfthip_stream_t stream) {
     XFT_REQUIRE(m && rows_host && n > 0, "xfthip_model_seq_decode: bad argument");
     const xfthip_model_config &c = m->cfg;
-    XFT_REQUIRE(m->ragged && m->active, "xfthip_model_seq_decode: no sequence was started with xfthip_model_seq_prefill");
+    XFT_REQUIRE(m->ragged && (m->active || m->plan), "xfthip_model_seq_decode: no sequence was started with xfthip_model_seq_prefill");
     std::vector<int> act(c.max_batch, 0);
     int top = 0, deepest = 0;
     for (int i = 0; i < n; ++i) {
@@ -923,6 +953,26 @@ int xfthip_model_seq_decode(xfthip_model_t m, const int *rows_host, int n, int *
             if (m->row_pos[r] > deepest) deepest = m->row_pos[r];
         }
     hipStream_t st = (hipStream_t)stream;
+    if (m->plan) {
+        // the listed slots only, side by side: a recurrent state must not move for a sequence that sits out
+        m->plan->dec_list.assign(rows_host, rows_host + n);
+        m->cur_B = n;
+        m->cur_pos = 0;
+        for (int i = 0; i < n; ++i) m->cur_pos = m->row_pos[rows_host[i]] > m->cur_pos ? m->row_pos[rows_host[i]] : m->cur_pos;
+        const int rc = xfthip_model_decode(m, 1, nullptr, stream);
+        m->cur_B = top;
+        if (rc) return rc;
+        for (int i = 0; i < n; ++i) {
+            m->row_pos[rows_host[i]] += 1;
+            m->plan->logit_of_row[rows_host[i]] = i;
+        }
+        if (ids_out_host) {
+            std::vector<int> all(c.max_batch);
+            XFT_CHECK_HIP(hipMemcpy(all.data(), m->ids, (size_t)c.max_batch * 4, hipMemcpyDeviceToHost));
+            for (int i = 0; i < n; ++i) ids_out_host[i] = all[rows_host[i]];
+        }
+        return 0;
+    }
     XFT_CHECK_HIP(hipMemcpyAsync(m->active, act.data(), (size_t)c.max_batch * 4, hipMemcpyHostToDevice, st));
     XFT_CHECK_HIP(hipStreamSynchronize(st));
     // one step over rows 0 .. top - 1; the split count of the attention follows the deepest row
@@ -1016,6 +1066,7 @@ int xfthip_model_seq_reorder(xfthip_model_t m, const int *dst_rows_host, const i
         XFT_CHECK_HIP(hipMemcpy(m->ids + d, &ids_new[i], 4, hipMemcpyHostToDevice));
         if (d + 1 > m->cur_B) m->cur_B = d + 1;
     }
+    if (m->plan) return identity ? 0 : plan_reorder(m, dst_rows_host, src_rows_host, n, st); // (state and pages as a whole)
     if (identity || pos1 == pos0) return 0;
     const int blk0 = pos0 / 32, nblk = (pos1 + 31) / 32 - blk0;
     const KvView &k0 = m->caches[0]->kv;
@@ -1056,6 +1107,7 @@ int xfthip_model_seq_set_next_id(xfthip_model_t m, int row, int id) {
 
 int xfthip_model_seq_logits(xfthip_model_t m, int row, float *logits_host) {
     XFT_REQUIRE(m && logits_host && row >= 0 && row < m->cfg.max_batch && m->logits, "xfthip_model_seq_logits: bad argument");
+    if (m->plan) row = m->plan->logit_of_row[row];
     XFT_CHECK_HIP(hipMemcpy(logits_host, m->logits + (size_t)row * m->cfg.vocab, (size_t)m->cfg.vocab * 4, hipMemcpyDeviceToHost));
     return 0;
 }
@@ -1106,6 +1158,19 @@ int xfthip_model_prompt_logits(xfthip_model_t m, int first_row, int rows, float 
             first_row + rows, m->prompt_rows);
     const xfthip_model_config &c = m->cfg;
     hipStream_t st = (hipStream_t)stream;
+    if (m->plan) {
+        const int chunk = m->plan->logit_rows;
+        for (int r = 0; r < rows; r += chunk) {
+            const int n = rows - r < chunk ? rows - r : chunk;
+            std::vector<int> list(n);
+            for (int i = 0; i < n; ++i) list[i] = first_row + r + i;
+            XFT_CHECK_HIP(hipMemcpyAsync(m->plan->want, list.data(), (size_t)n * 4, hipMemcpyHostToDevice, st));
+            if (int rc = plan_head(m, m->plan->want, n, 0, st)) return rc;
+            XFT_CHECK_HIP(hipMemcpyAsync(logits_host + (size_t)r * c.vocab, m->logits, (size_t)n * c.vocab * 4, hipMemcpyDeviceToHost, st));
+            XFT_CHECK_HIP(hipStreamSynchronize(st));
+        }
+        return 0;
+    }
     // final norm + lm_head over the prompt's residual rows, a chunk at a time through a buffer that lives for the
     // call (not a hot path: the reference's logitsAll = true serves scoring, not generation)
     const int chunk = rows < 256 ? rows : 256;

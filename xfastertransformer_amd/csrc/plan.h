@@ -1,0 +1,177 @@
+// Layer plans: decoder stacks whose layers differ in kind (latent attention, delta-rule recurrence), whose keys live
+// in a page pool shared by all sequences and whose recurrent layers keep a state per sequence slot.  Declarations
+// shared by the plan's driver (plan_model.hip) and its kernels (plan_layers.hip, latent_attention.hip, delta_rule.hip,
+// tile_gemm.hip).
+//
+// Every inner width is padded to whole 32-value groups (the state's key dimension to a power of two) by zero rows and
+// columns of the packed weights, so that the kernels see whole MFMA steps whatever sizes a model has.
+#pragma once
+#include <string>
+#include <vector>
+
+#include "common.h"
+#include "qgemm.h"
+
+namespace xfthip {
+
+constexpr int kPageTokens = 64; // tokens of a page of the latent cache
+
+// One step: B segments (one a sequence), T tokens, back to back.  All pointers are device memory.
+struct StepView {
+    int B, T;
+    int longest; // tokens of the longest segment
+    const int *tok_seg, *tok_pos; // [T] segment and position of a token
+    const int *seg_row, *seg_off, *seg_len, *seg_pos; // [B] slot, first token, tokens, position of the first token
+    const int *table; // [slots][table_stride] page numbers
+    int table_stride;
+};
+
+struct PlanLayer {
+    xfthip_plan_layer s;
+    // latent attention: padded widths of a head's unrotated / rotated / value part, of the key and the query latent
+    int D = 0, RD = 0, V = 0, R = 0, QR = 0;
+    // delta rule: padded key / value width of a head, padded rank of the two gates and columns of one gate
+    int KD = 0, VD = 0, rank = 0, gcols = 0;
+    int ff = 0; // padded
+    xfthip_weight_t in = nullptr, o = nullptr, gateup = nullptr, down = nullptr;
+    // latent: queries from their latent; W_uk turned round (query -> latent), W_uk and W_uv (latent -> key / value)
+    xfthip_weight_t uq = nullptr, absorb = nullptr, uk = nullptr, uv = nullptr;
+    float *q_norm = nullptr, *kv_norm = nullptr, *sink = nullptr;
+    float *cosT = nullptr, *sinT = nullptr; // [max positions][rot_dim / 2], shared by layers of the same rotation
+    // delta rule: both gates' second projections (decay | output gate), filters [channels][taps], exp(A_log), ...
+    xfthip_weight_t gates = nullptr;
+    float *conv = nullptr, *decay = nullptr, *dt_bias = nullptr, *out_norm = nullptr;
+    // norm weights: 1 + w in front of a sublayer, (1 + w) * layer scale behind it
+    float *pre1 = nullptr, *post1 = nullptr, *pre2 = nullptr, *post2 = nullptr;
+
+    int row_in() const { return s.mixer == XFTHIP_MIXER_LATENT ? QR + R + RD : (2 * s.kv_heads * KD + s.heads * VD) + beta_cols() + 2 * rank; }
+    int beta_cols() const { return (s.heads + 31) / 32 * 32; }
+    int channels() const { return 2 * s.kv_heads * KD + s.heads * VD; } // of the short convolution: q | k | v
+};
+
+struct LayerRun {
+    int layer;
+    bool add_embedding; // the embedding output joins the residual in front of this run
+};
+
+// ---- kernels -----------------------------------------------------------------------------------------------------
+// (act: XFTHIP_BF16 or XFTHIP_F32, the type of activations between kernels; the residual is fp32)
+
+// x[t] = table[ids[t]] (bf16 table, ids clamped to the vocabulary)
+int plan_embed(const uint16_t *table, const int *ids, float *x, int T, int hidden, int vocab, hipStream_t st);
+// x += rms(y) * post (y may be null), then x += table[ids] (table may be null), then xn = rms(x) * pre (pre may be null).
+// Means over `width` of the `hidden` columns.  rows: xn row i comes from x row rows[i] (only without y and table).
+int plan_norm(int act, float *x, const float *y, const float *post, const uint16_t *table, const int *ids, int vocab, const float *pre, void *xn,
+        const int *rows, int T, int hidden, int width, float eps, hipStream_t st);
+
+// C[t][n] = sum_k A[t][block(n) * a_block_stride + k] W[k][n], block(n) = n / block_cols: a plain product of 32-bit
+// activations (block_cols = 0), or heads side by side.  BF16 weights; act_in / c_dtype XFTHIP_BF16 or XFTHIP_F32; glu: 1
+// the weight holds gate / up pairs (XFTHIP_WF_GATEUP), combined as clamped_glu.
+int tile_gemm(xfthip_weight_t w, int act_in, int M, const void *A, int lda, int block_cols, int a_block_stride, void *C, int ldc, int c_dtype,
+        int glu, float glu_limit, float glu_alpha, hipStream_t st);
+
+struct LatentCacheView {
+    void *pool; // [pages][kPageTokens][R + RD] of the activation type: normalised latent | rotated shared key part
+    int R, RD;
+};
+// the query latent's norm -> cq; the key latent's norm and the shared key part's rotation -> cache
+int latent_prepare(int act, const PlanLayer &L, const StepView &v, const void *a, void *cq, const LatentCacheView &cache, float eps, hipStream_t st);
+// rotates the rotated parts of q [T][heads][D + RD] in place
+int latent_rotate_q(int act, const PlanLayer &L, const StepView &v, void *q, hipStream_t st);
+// absorbed form: qa [T][heads][R] queries in the latent space, q their rotated parts; out [T][heads][R] weighted latents.
+// part: workspace of attn_part_floats floats (split contexts).  hint: upper bound of the sequence lengths
+int latent_attention(int act, const PlanLayer &L, const StepView &v, const void *qa, const void *q, void *out, const LatentCacheView &cache,
+        int hint, float *part, size_t part_floats, hipStream_t st);
+int latent_split_count(const PlanLayer &L, int B, int longest, int hint);
+
+struct DeltaBuffers {
+    void *in; // [T][row_in] of the activation type: q | k | v | beta | decay rank | gate rank
+    float *gates; // [T][2 * gcols]: decay step (before softplus) | output gate (before the sigmoid)
+    float *q, *k, *qk; // [T][kv_heads][KD] twice, [T][kv_heads]
+    float *g, *v, *beta; // [T][heads][KD], [T][heads][VD], [T][heads]
+    float *o; // [T][heads][VD]
+    void *on; // [T][heads * VD] of the activation type
+    float *state; // [slots][heads][VD][KD]
+    void *conv_state; // [slots][taps - 1][channels] of the activation type
+};
+int delta_prepare(int act, const PlanLayer &L, const StepView &v, const DeltaBuffers &b, hipStream_t st);
+int delta_scan(const PlanLayer &L, const StepView &v, const DeltaBuffers &b, hipStream_t st);
+int delta_output(int act, const PlanLayer &L, const StepView &v, const DeltaBuffers &b, float eps, hipStream_t st);
+
+} // namespace xfthip
+
+struct xfthip_plan {
+    xfthip_plan_config cfg;
+    std::vector<xfthip::PlanLayer> layers;
+    std::vector<xfthip::LayerRun> runs;
+    int hidden = 0; // width padded to whole 32-value groups
+    uint16_t *embedding = nullptr; // [vocab][hidden] bf16
+    float *final_norm = nullptr; // (1 + w) * logit scale
+    xfthip_weight_t head = nullptr;
+    struct Tensor {
+        std::vector<uint16_t> data;
+        int rows = 0, cols = 0;
+    };
+    std::vector<std::pair<std::string, Tensor>> pending; // tensors given so far, until the plan is finished
+    bool finished = false;
+    size_t weight_bytes = 0;
+};
+
+namespace xfthip {
+
+// What a model from a plan adds to xfthip_model: the page pool and the state slots, scratch, the step's description.
+struct PlanState {
+    xfthip_plan *plan = nullptr;
+    std::vector<PlanLayer> layers; // the plan's, with this model's rotation tables
+    int act = XFTHIP_BF16, esz = 2;
+    int slots = 0;
+    // by layer run: page pool of a latent attention, state and convolution inputs of a delta rule
+    std::vector<LatentCacheView> cache;
+    std::vector<float *> state;
+    std::vector<void *> conv_state;
+    // pages: free ones, those of every slot in position order, and the device table [slots][table_stride]
+    int pages = 0, table_stride = 0;
+    std::vector<int> free_pages;
+    std::vector<std::vector<int>> held;
+    std::vector<int> table_host;
+    int *table = nullptr;
+    bool table_dirty = true;
+    // step description on the device, its host image (pinned) and the views into it
+    int *desc = nullptr, *desc_host = nullptr;
+    int *tok_seg = nullptr, *tok_pos = nullptr, *ids = nullptr, *seg = nullptr, *dec_rows = nullptr, *want = nullptr;
+    std::vector<int> dec_list; // slots of the decode call in flight
+    std::vector<int> logit_of_row; // which row of the logits a slot's last ones are in
+    int logit_rows = 0;
+    // scratch (activation type unless float)
+    void *xn = nullptr, *a = nullptr, *cq = nullptr, *q = nullptr, *qa = nullptr, *oc = nullptr, *ov = nullptr, *h = nullptr, *on = nullptr;
+    float *y = nullptr, *gates = nullptr, *dq = nullptr, *dk = nullptr, *dqk = nullptr, *dg = nullptr, *dv = nullptr, *dbeta = nullptr, *do_ = nullptr;
+    float *part = nullptr; // split contexts
+    size_t part_floats = 0;
+    std::vector<float *> tables; // rotation tables
+    std::vector<void *> owned; // every device buffer above
+    bool trace = false;
+    float *trace_buf = nullptr;
+    size_t trace_floats = 0;
+    int trace_tokens = 0;
+};
+
+// pages for the first `tokens` positions of a slot
+int plan_reserve(xfthip_model *m, int row, int tokens);
+void plan_release(xfthip_model *m, int row);
+// residual rows of a step: entry i = the next lens[i] tokens of slot rows[i] (m->row_pos says where they stand; it moves on)
+int plan_run(xfthip_model *m, int n, const int *rows, const int *lens, const int *ids, hipStream_t st);
+// final norm and head of the residual rows rows_dev[0 .. n) (null: rows 0 .. n - 1) into m->logits + at * vocab
+int plan_head(xfthip_model *m, const int *rows_dev, int n, int at, hipStream_t st);
+// upload of what a decode call of the slots in dec_list needs, for `steps` steps
+int plan_decode_begin(xfthip_model *m, int steps, hipStream_t st);
+// one decode step of the slots in dec_rows (recordable): positions and input ids from m->pos / m->ids
+int plan_decode_step(xfthip_model *m, int B, hipStream_t st);
+int plan_decode_splits(xfthip_model *m, int B, int hint);
+int plan_prompt_pass(xfthip_model *m, const int *rows, int B, int S, const int *ids, float *logits_host, hipStream_t st);
+int plan_reorder(xfthip_model *m, const int *dst, const int *src, int n, hipStream_t st);
+void plan_state_destroy(PlanState *p);
+
+// model.hip: first-maximum arg-max of n rows of logits; entry b goes to ids[rows ? rows[b] : b] (and bumps advance_pos there)
+int argmax_rows(const float *logits, int n, int cols, int *ids, const int *rows, int *advance_pos, int *advance_step, hipStream_t st);
+
+} // namespace xfthip

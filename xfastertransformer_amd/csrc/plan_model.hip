@@ -1,0 +1,775 @@
+// Driver of layer plans: the plan's weights (composed, padded and packed from the model's tensors), the page pool and the
+// state slots, and the order of kernels a step runs.  One step is a ragged batch: segments of any length, each the next
+// tokens of one sequence; a decode step is the same with one token a segment and everything position-dependent read from
+// device memory, so that it can be recorded.
+#include <math.h>
+#include <string.h>
+
+#include <algorithm>
+#include <map>
+
+#include "model_impl.h"
+#include "plan.h"
+
+namespace xfthip {
+
+namespace {
+
+int pad32(int n) { return (n + 31) / 32 * 32; }
+
+float bf16_value(uint16_t b) {
+    const uint32_t u = (uint32_t)b << 16;
+    float f;
+    memcpy(&f, &u, 4);
+    return f;
+}
+
+using Tensor = xfthip_plan::Tensor;
+
+struct Matrix { // [K][N] bf16, zero where nothing is placed
+    int K, N;
+    std::vector<uint16_t> w;
+    Matrix(int k, int n) : K(k), N(n), w((size_t)k * n, 0) {}
+    // rows [r0, r0 + rows) and columns [c0, c0 + cols) of an [out, in] tensor to columns n0 .. / rows k0 ..
+    void place(const Tensor &t, int r0, int rows, int c0, int cols, int k0, int n0) {
+        for (int cb = 0; cb < cols; cb += 32)
+            for (int rb = 0; rb < rows; rb += 32)
+                for (int c = cb; c < cols && c < cb + 32; ++c)
+                    for (int r = rb; r < rows && r < rb + 32; ++r) w[(size_t)(k0 + c) * N + n0 + r] = t.data[(size_t)(r0 + r) * t.cols + c0 + c];
+    }
+    // the same block turned round: tensor rows along K
+    void place_turned(const Tensor &t, int r0, int rows, int c0, int cols, int k0, int n0) {
+        for (int r = 0; r < rows; ++r) memcpy(&w[(size_t)(k0 + r) * N + n0], &t.data[(size_t)(r0 + r) * t.cols + c0], (size_t)cols * 2);
+    }
+};
+
+__global__ void plan_decode_begin_kernel(const uint16_t *table, const int *dec_rows, const int *pos, const int *ids, float *x, int hidden, int vocab,
+        int *tok_seg, int *tok_pos, int *tok_ids, int *seg, int seg_cap, int *log, const int *step, int max_seq) {
+    const int b = blockIdx.x, row = dec_rows[b];
+    int id = ids[row], at = pos[row];
+    at = at < 0 ? 0 : (at >= max_seq ? max_seq - 1 : at);
+    if (threadIdx.x == 0) {
+        log[(size_t)step[0] * gridDim.x + b] = id;
+        tok_seg[b] = b, tok_pos[b] = at, tok_ids[b] = id;
+        seg[b] = row, seg[seg_cap + b] = b, seg[2 * seg_cap + b] = 1, seg[3 * seg_cap + b] = at;
+    }
+    id = id < 0 ? 0 : (id >= vocab ? vocab - 1 : id);
+    const uint16_t *src = table + (size_t)id * hidden;
+    for (int c = threadIdx.x; c < hidden; c += blockDim.x) x[(size_t)b * hidden + c] = bf16_to_f32(src[c]);
+}
+
+__global__ void plan_set_pos_kernel(const int *seg, int seg_cap, int n, int *pos) {
+    const int b = blockIdx.x * blockDim.x + threadIdx.x;
+    if (b < n) pos[seg[b]] = seg[3 * seg_cap + b] + seg[2 * seg_cap + b];
+}
+
+__global__ void plan_fill_kernel(int *p, int n, int v) {
+    const int i = blockIdx.x * blockDim.x + threadIdx.x;
+    if (i < n) p[i] = v;
+}
+
+// rotation tables [positions][dims / 2]: angles in double, as far apart as positions can be
+int rotation_tables(double base, int dims, int positions, float **cosT, float **sinT) {
+    const int half = dims / 2;
+    std::vector<float> c((size_t)positions * half), s((size_t)positions * half);
+    for (int i = 0; i < half; ++i) {
+        const double f = pow(base, -2.0 * i / dims);
+        for (int p = 0; p < positions; ++p) c[(size_t)p * half + i] = (float)cos(p * f), s[(size_t)p * half + i] = (float)sin(p * f);
+    }
+    XFT_CHECK_HIP(hipMalloc((void **)cosT, c.size() * 4 + 16));
+    XFT_CHECK_HIP(hipMalloc((void **)sinT, s.size() * 4 + 16));
+    XFT_CHECK_HIP(hipMemcpy(*cosT, c.data(), c.size() * 4, hipMemcpyHostToDevice));
+    XFT_CHECK_HIP(hipMemcpy(*sinT, s.data(), s.size() * 4, hipMemcpyHostToDevice));
+    return 0;
+}
+
+int plan_gemm(xfthip_model *m, xfthip_weight_t w, int M, const void *A, int lda, void *C, int ldc, int c_dtype, hipStream_t st) {
+    if (m->plan->act == XFTHIP_F32) return tile_gemm(w, XFTHIP_F32, M, A, lda, 0, 0, C, ldc, c_dtype, 0, 0, 0, st);
+    return xfthip_gemm(w, M, A, lda, C, ldc, c_dtype, XFTHIP_EPI_NONE, nullptr, nullptr, 0, XFTHIP_F32, 1.0f, st);
+}
+
+int run_latent(xfthip_model *m, const PlanLayer &L, int run, const StepView &v, hipStream_t st) {
+    PlanState &p = *m->plan;
+    const int T = v.T, H = L.s.heads, act = p.act, hidden = m->cfg.hidden;
+    const int qcols = H * (L.D + L.RD);
+    int rc;
+    if ((rc = plan_gemm(m, L.in, T, p.xn, hidden, p.a, L.row_in(), act, st))) return rc;
+    if ((rc = latent_prepare(act, L, v, p.a, p.cq, p.cache[run], m->cfg.rms_eps, st))) return rc;
+    if ((rc = plan_gemm(m, L.uq, T, p.cq, L.QR, p.q, qcols, act, st))) return rc;
+    if ((rc = latent_rotate_q(act, L, v, p.q, st))) return rc;
+    if ((rc = tile_gemm(L.absorb, act, T, p.q, qcols, L.R, L.D + L.RD, p.qa, H * L.R, act, 0, 0, 0, st))) return rc;
+    if ((rc = latent_attention(act, L, v, p.qa, p.q, p.oc, p.cache[run], m->len_hint, p.part, p.part_floats, st))) return rc;
+    if ((rc = tile_gemm(L.uv, act, T, p.oc, H * L.R, L.V, L.R, p.ov, H * L.V, act, 0, 0, 0, st))) return rc;
+    return plan_gemm(m, L.o, T, p.ov, H * L.V, p.y, hidden, XFTHIP_F32, st);
+}
+
+int run_delta(xfthip_model *m, const PlanLayer &L, int run, const StepView &v, hipStream_t st) {
+    PlanState &p = *m->plan;
+    const int T = v.T, act = p.act, hidden = m->cfg.hidden, ld = L.row_in();
+    int rc;
+    const DeltaBuffers b = {p.a, p.gates, p.dq, p.dk, p.dqk, p.dg, p.dv, p.dbeta, p.do_, p.on, p.state[run], p.conv_state[run]};
+    if ((rc = plan_gemm(m, L.in, T, p.xn, hidden, p.a, ld, act, st))) return rc;
+    const int first = L.channels() + L.beta_cols();
+    if ((rc = tile_gemm(L.gates, act, T, (const char *)p.a + (size_t)first * p.esz, ld, L.gcols, L.rank, p.gates, 2 * L.gcols, XFTHIP_F32, 0, 0, 0, st)))
+        return rc;
+    if ((rc = delta_prepare(act, L, v, b, st))) return rc;
+    if ((rc = delta_scan(L, v, b, st))) return rc;
+    if ((rc = delta_output(act, L, v, b, m->cfg.rms_eps, st))) return rc;
+    return plan_gemm(m, L.o, T, p.on, L.s.heads * L.VD, p.y, hidden, XFTHIP_F32, st);
+}
+
+// all layer runs over the step's tokens, whose embeddings are in m->x
+int plan_layers(xfthip_model *m, const StepView &v, hipStream_t st) {
+    PlanState &p = *m->plan;
+    const xfthip_plan &plan = *p.plan;
+    const int T = v.T, hidden = m->cfg.hidden, width = plan.cfg.hidden, vocab = m->cfg.vocab;
+    const float eps = m->cfg.rms_eps;
+    const int nruns = (int)plan.runs.size();
+    int rc;
+    auto norm = [&](const float *y, const float *post, bool again, const float *pre) {
+        return plan_norm(p.act, m->x, y, post, again ? plan.embedding : nullptr, p.ids, vocab, pre, p.xn, nullptr, T, hidden, width, eps, st);
+    };
+    if ((rc = norm(nullptr, nullptr, plan.runs[0].add_embedding, p.layers[plan.runs[0].layer].pre1))) return rc;
+    for (int r = 0; r < nruns; ++r) {
+        const PlanLayer &L = p.layers[plan.runs[r].layer];
+        const bool last = r + 1 == nruns;
+        // (a traced run keeps the embedding of a further pass apart, so that the trace shows the layer's own result)
+        const bool again = !last && plan.runs[r + 1].add_embedding;
+        const float *next = last ? nullptr : p.layers[plan.runs[r + 1].layer].pre1;
+        rc = L.s.mixer == XFTHIP_MIXER_LATENT ? run_latent(m, L, r, v, st) : run_delta(m, L, r, v, st);
+        if (rc) return rc;
+        const bool ff = L.ff > 0;
+        if ((rc = norm(p.y, L.post1, !ff && again && !p.trace, ff ? L.pre2 : (p.trace ? nullptr : next)))) return rc;
+        if (ff) {
+            if (p.act == XFTHIP_F32)
+                rc = tile_gemm(L.gateup, XFTHIP_F32, T, p.xn, hidden, 0, 0, p.h, L.ff, XFTHIP_F32, 1, L.s.glu_limit, L.s.glu_alpha, st);
+            else
+                rc = xfthip_gemm_gateup_clamped(L.gateup, T, p.xn, hidden, p.h, L.ff, XFTHIP_BF16, L.s.glu_limit, L.s.glu_alpha, st);
+            if (rc) return rc;
+            if ((rc = plan_gemm(m, L.down, T, p.h, L.ff, p.y, hidden, XFTHIP_F32, st))) return rc;
+            if ((rc = norm(p.y, L.post2, again && !p.trace, p.trace ? nullptr : next))) return rc;
+        }
+        if (p.trace) {
+            XFT_CHECK_HIP(hipMemcpyAsync(p.trace_buf + (size_t)r * T * hidden, m->x, (size_t)T * hidden * 4, hipMemcpyDeviceToDevice, st));
+            if (!last && (rc = norm(nullptr, nullptr, again, next))) return rc;
+        }
+    }
+    return 0;
+}
+
+int upload_table(PlanState &p, hipStream_t st) {
+    if (!p.table_dirty) return 0;
+    XFT_CHECK_HIP(hipMemcpyAsync(p.table, p.table_host.data(), p.table_host.size() * 4, hipMemcpyHostToDevice, st));
+    XFT_CHECK_HIP(hipStreamSynchronize(st));
+    p.table_dirty = false;
+    return 0;
+}
+
+StepView view_of(const xfthip_model *m, int B, int T, int longest) {
+    const PlanState &p = *m->plan;
+    const int cap = p.slots;
+    return StepView {B, T, longest, p.tok_seg, p.tok_pos, p.seg, p.seg + cap, p.seg + 2 * cap, p.seg + 3 * cap, p.table, p.table_stride};
+}
+
+} // namespace
+
+int plan_reserve(xfthip_model *m, int row, int tokens) {
+    PlanState &p = *m->plan;
+    const int need = (tokens + kPageTokens - 1) / kPageTokens;
+    XFT_REQUIRE(need <= p.table_stride, "the sequence of slot %d is longer than the model's %d positions", row, m->cfg.max_seq);
+    while ((int)p.held[row].size() < need) {
+        XFT_REQUIRE(!p.free_pages.empty(), "the page pool (%d pages of %d tokens) is exhausted", p.pages, kPageTokens);
+        const int page = p.free_pages.back();
+        p.free_pages.pop_back();
+        p.table_host[(size_t)row * p.table_stride + p.held[row].size()] = page;
+        p.held[row].push_back(page);
+        p.table_dirty = true;
+    }
+    return 0;
+}
+
+void plan_release(xfthip_model *m, int row) {
+    PlanState &p = *m->plan;
+    for (size_t i = p.held[row].size(); i-- > 0;) p.free_pages.push_back(p.held[row][i]);
+    p.held[row].clear();
+}
+
+int plan_run(xfthip_model *m, int n, const int *rows, const int *lens, const int *ids, hipStream_t st) {
+    PlanState &p = *m->plan;
+    const xfthip_model_config &c = m->cfg;
+    XFT_REQUIRE(n > 0 && n <= p.slots, "a step of %d entries; the model has %d slots", n, p.slots);
+    std::vector<char> seen(p.slots, 0);
+    long T = 0;
+    int longest = 0, deepest = 0;
+    for (int i = 0; i < n; ++i) {
+        XFT_REQUIRE(rows[i] >= 0 && rows[i] < p.slots && !seen[rows[i]], "slot %d listed twice or outside the model's %d", rows[i], p.slots);
+        seen[rows[i]] = 1;
+        const int at = m->row_pos[rows[i]] < 0 ? 0 : m->row_pos[rows[i]];
+        XFT_REQUIRE(lens[i] > 0 && at + lens[i] <= c.max_seq, "slot %d: %d tokens at position %d exceed the model's %d positions", rows[i], lens[i], at, c.max_seq);
+        T += lens[i];
+        longest = std::max(longest, lens[i]);
+        deepest = std::max(deepest, at + lens[i]);
+    }
+    XFT_REQUIRE(T <= c.max_tokens, "a step of %ld tokens; the model takes %d", T, c.max_tokens);
+    for (int i = 0; i < n; ++i)
+        if (int rc = plan_reserve(m, rows[i], std::max(m->row_pos[rows[i]], 0) + lens[i])) return rc;
+    if (int rc = upload_table(p, st)) return rc;
+    // the description: tok_seg | tok_pos | ids | seg (4 arrays of `slots`), one copy each way
+    const int cap = p.slots, mt = c.max_tokens;
+    int *hs = p.desc_host, *hp = hs + mt, *hi = hp + mt, *hg = hi + mt;
+    int t = 0;
+    for (int i = 0; i < n; ++i) {
+        const int at = std::max(m->row_pos[rows[i]], 0);
+        hg[i] = rows[i], hg[cap + i] = t, hg[2 * cap + i] = lens[i], hg[3 * cap + i] = at;
+        for (int k = 0; k < lens[i]; ++k, ++t) hs[t] = i, hp[t] = at + k, hi[t] = ids[t];
+    }
+    XFT_CHECK_HIP(hipMemcpyAsync(p.tok_seg, hs, (size_t)T * 4, hipMemcpyHostToDevice, st));
+    XFT_CHECK_HIP(hipMemcpyAsync(p.tok_pos, hp, (size_t)T * 4, hipMemcpyHostToDevice, st));
+    XFT_CHECK_HIP(hipMemcpyAsync(p.ids, hi, (size_t)T * 4, hipMemcpyHostToDevice, st));
+    XFT_CHECK_HIP(hipMemcpyAsync(p.seg, hg, (size_t)4 * cap * 4, hipMemcpyHostToDevice, st));
+    if (int rc = plan_embed(p.plan->embedding, p.ids, m->x, (int)T, c.hidden, c.vocab, st)) return rc;
+    m->len_hint = deepest;
+    if (p.trace) {
+        const size_t need = p.plan->runs.size() * (size_t)T * c.hidden;
+        if (need > p.trace_floats) {
+            XFT_CHECK_HIP(hipStreamSynchronize(st));
+            if (p.trace_buf) (void)hipFree(p.trace_buf);
+            p.trace_buf = nullptr, p.trace_floats = 0;
+            XFT_CHECK_HIP(hipMalloc((void **)&p.trace_buf, need * 4));
+            p.trace_floats = need;
+        }
+        p.trace_tokens = (int)T;
+    }
+    if (int rc = plan_layers(m, view_of(m, n, (int)T, longest), st)) return rc;
+    hipLaunchKernelGGL(plan_set_pos_kernel, dim3((n + 63) / 64), dim3(64), 0, st, p.seg, cap, n, m->pos);
+    XFT_CHECK_HIP(hipGetLastError());
+    for (int i = 0; i < n; ++i) m->row_pos[rows[i]] = std::max(m->row_pos[rows[i]], 0) + lens[i];
+    return 0;
+}
+
+int plan_head(xfthip_model *m, const int *rows_dev, int n, int at, hipStream_t st) {
+    PlanState &p = *m->plan;
+    const xfthip_plan &plan = *p.plan;
+    const xfthip_model_config &c = m->cfg;
+    if (int rc = plan_norm(p.act, m->x, nullptr, nullptr, nullptr, nullptr, c.vocab, plan.final_norm, p.xn, rows_dev, n, c.hidden, plan.cfg.hidden, c.rms_eps, st))
+        return rc;
+    return plan_gemm(m, plan.head, n, p.xn, c.hidden, m->logits + (size_t)at * c.vocab, c.vocab, XFTHIP_F32, st);
+}
+
+int plan_prompt_pass(xfthip_model *m, const int *rows, int B, int S, const int *ids, float *logits_host, hipStream_t st) {
+    PlanState &p = *m->plan;
+    const xfthip_model_config &c = m->cfg;
+    std::vector<int> lens(B, S), last(B);
+    if (int rc = plan_run(m, B, rows, lens.data(), ids, st)) return rc;
+    for (int b = 0; b < B; ++b) last[b] = (b + 1) * S - 1;
+    XFT_CHECK_HIP(hipMemcpyAsync(p.want, last.data(), (size_t)B * 4, hipMemcpyHostToDevice, st));
+    // (the prompts of one call sit in neighbouring slots)
+    if (int rc = plan_head(m, p.want, B, rows[0], st)) return rc;
+    if (int rc = argmax_rows(m->logits + (size_t)rows[0] * c.vocab, B, c.vocab, m->ids, p.seg, nullptr, nullptr, st)) return rc;
+    hipLaunchKernelGGL(plan_fill_kernel, dim3(1), dim3(64), 0, st, m->step, 1, 0);
+    XFT_CHECK_HIP(hipGetLastError());
+    XFT_CHECK_HIP(hipStreamSynchronize(st));
+    if (logits_host) XFT_CHECK_HIP(hipMemcpy(logits_host, m->logits + (size_t)rows[0] * c.vocab, (size_t)B * c.vocab * 4, hipMemcpyDeviceToHost));
+    for (int b = 0; b < B; ++b) p.logit_of_row[rows[b]] = rows[0] + b;
+    return 0;
+}
+
+int plan_decode_begin(xfthip_model *m, int steps, hipStream_t st) {
+    PlanState &p = *m->plan;
+    for (int r : p.dec_list)
+        if (int rc = plan_reserve(m, r, m->row_pos[r] + steps)) return rc;
+    if (int rc = upload_table(p, st)) return rc;
+    XFT_CHECK_HIP(hipMemcpyAsync(p.dec_rows, p.dec_list.data(), p.dec_list.size() * 4, hipMemcpyHostToDevice, st));
+    XFT_CHECK_HIP(hipStreamSynchronize(st));
+    for (size_t b = 0; b < p.dec_list.size(); ++b) p.logit_of_row[p.dec_list[b]] = (int)b;
+    return 0;
+}
+
+int plan_decode_step(xfthip_model *m, int B, hipStream_t st) {
+    PlanState &p = *m->plan;
+    const xfthip_model_config &c = m->cfg;
+    hipLaunchKernelGGL(plan_decode_begin_kernel, dim3(B), dim3(256), 0, st, p.plan->embedding, p.dec_rows, m->pos, m->ids, m->x, c.hidden, c.vocab, p.tok_seg,
+            p.tok_pos, p.ids, p.seg, p.slots, m->idlog, m->step, c.max_seq);
+    XFT_CHECK_HIP(hipGetLastError());
+    const bool trace = p.trace;
+    p.trace = false;
+    int rc = plan_layers(m, view_of(m, B, B, 1), st);
+    p.trace = trace;
+    if (rc) return rc;
+    if ((rc = plan_head(m, nullptr, B, 0, st))) return rc;
+    return argmax_rows(m->logits, B, c.vocab, m->ids, p.dec_rows, m->pos, m->step, st);
+}
+
+int plan_decode_splits(xfthip_model *m, int B, int hint) {
+    int s = 0; // the split counts of the attentions, as far as a recorded step depends on them
+    for (auto &L : m->plan->layers)
+        if (L.s.mixer == XFTHIP_MIXER_LATENT) s = s * 31 + latent_split_count(L, B, 1, hint);
+    return s;
+}
+
+// Slot dst[i] becomes a copy of slot src[i]: pages, recurrent state, convolution inputs.  Everything is read before anything
+// is written (through a staging buffer, run by run).
+int plan_reorder(xfthip_model *m, const int *dst, const int *src, int n, hipStream_t st) {
+    PlanState &p = *m->plan;
+    XFT_CHECK_HIP(hipStreamSynchronize(st));
+    std::vector<std::vector<int>> from(n);
+    for (int i = 0; i < n; ++i) from[i] = p.held[src[i]];
+    for (int i = 0; i < n; ++i) {
+        const int have = (int)p.held[dst[i]].size(), want = (int)from[i].size();
+        for (int k = have; k > want; --k) {
+            p.free_pages.push_back(p.held[dst[i]].back());
+            p.held[dst[i]].pop_back();
+        }
+    }
+    // (a slot whose pages another one reads keeps them: it is a destination itself only if it is listed, with as many or more pages)
+    size_t bytes = 0;
+    for (size_t r = 0; r < p.plan->runs.size(); ++r) {
+        const PlanLayer &L = p.layers[p.plan->runs[r].layer];
+        size_t need = 0;
+        for (int i = 0; i < n; ++i)
+            need += L.s.mixer == XFTHIP_MIXER_LATENT ? from[i].size() * (size_t)kPageTokens * (L.R + L.RD) * p.esz
+                                                     : ((size_t)L.s.heads * L.VD * L.KD * 4 + (size_t)(L.s.taps - 1) * L.channels() * p.esz);
+        bytes = std::max(bytes, need);
+    }
+    char *stage = nullptr;
+    XFT_CHECK_HIP(hipMalloc((void **)&stage, bytes + 16));
+    int rc = 0;
+    for (int i = 0; i < n && rc == 0; ++i) rc = plan_reserve(m, dst[i], (int)from[i].size() * kPageTokens);
+    if (rc == 0) rc = upload_table(p, st);
+    hipError_t e = hipSuccess;
+    auto copy = [&](void *d, const void *s, size_t b) {
+        if (e == hipSuccess && b) e = hipMemcpyAsync(d, s, b, hipMemcpyDeviceToDevice, st);
+    };
+    for (size_t r = 0; r < p.plan->runs.size() && rc == 0; ++r) {
+        const PlanLayer &L = p.layers[p.plan->runs[r].layer];
+        for (int write = 0; write < 2; ++write) {
+            size_t at = 0;
+            for (int i = 0; i < n; ++i) {
+                if (L.s.mixer == XFTHIP_MIXER_LATENT) {
+                    const size_t page = (size_t)kPageTokens * (L.R + L.RD) * p.esz;
+                    for (size_t k = 0; k < from[i].size(); ++k, at += page) {
+                        char *pool = (char *)p.cache[r].pool;
+                        if (write) copy(pool + (size_t)p.held[dst[i]][k] * page, stage + at, page);
+                        else copy(stage + at, pool + (size_t)from[i][k] * page, page);
+                    }
+                } else {
+                    const size_t sb = (size_t)L.s.heads * L.VD * L.KD * 4, cb = (size_t)(L.s.taps - 1) * L.channels() * p.esz;
+                    char *state = (char *)p.state[r], *conv = (char *)p.conv_state[r];
+                    if (write) {
+                        copy(state + dst[i] * sb, stage + at, sb);
+                        copy(conv + dst[i] * cb, stage + at + sb, cb);
+                    } else {
+                        copy(stage + at, state + src[i] * sb, sb);
+                        copy(stage + at + sb, conv + src[i] * cb, cb);
+                    }
+                    at += sb + cb;
+                }
+            }
+        }
+    }
+    if (e == hipSuccess) e = hipStreamSynchronize(st);
+    (void)hipFree(stage);
+    if (rc) return rc;
+    XFT_CHECK_HIP(e);
+    return 0;
+}
+
+void plan_state_destroy(PlanState *p) {
+    for (void *b : p->owned) (void)hipFree(b);
+    if (p->trace_buf) (void)hipFree(p->trace_buf);
+    if (p->desc_host) (void)hipHostFree(p->desc_host);
+    delete p;
+}
+
+} // namespace xfthip
+
+using namespace xfthip;
+
+extern "C" {
+
+int xfthip_plan_create(const xfthip_plan_config *cfg, const xfthip_plan_layer *layers, xfthip_plan_t *out) {
+    XFT_REQUIRE(cfg && layers && out, "xfthip_plan_create: null argument");
+    const xfthip_plan_config &c = *cfg;
+    XFT_REQUIRE(c.layers > 0 && c.hidden > 0 && c.hidden <= 16384 && c.vocab > 0, "xfthip_plan_create: bad sizes");
+    const bool loop = c.loop_times > 1;
+    XFT_REQUIRE(!loop || (c.loop_start >= 0 && c.loop_start < c.loop_stop && c.loop_stop <= c.layers), "xfthip_plan_create: loop over layers %d .. %d of %d",
+            c.loop_start, c.loop_stop, c.layers);
+    xfthip_plan *p = new xfthip_plan();
+    p->cfg = c;
+    p->hidden = pad32(c.hidden);
+    for (int i = 0; i < c.layers; ++i) {
+        PlanLayer L;
+        L.s = layers[i];
+        const xfthip_plan_layer &s = L.s;
+        bool ok = s.heads > 0 && s.dim > 0 && s.vdim > 0 && s.inter >= 0;
+        if (s.mixer == XFTHIP_MIXER_LATENT) {
+            ok = ok && s.rot_dim > 0 && s.rot_dim % 2 == 0 && s.kv_rank > 0 && s.kv_rank <= 1024 && s.q_rank > 0 && s.window >= 0;
+            L.D = pad32(s.dim), L.RD = pad32(s.rot_dim), L.V = pad32(s.vdim), L.R = pad32(s.kv_rank), L.QR = pad32(s.q_rank);
+        } else if (s.mixer == XFTHIP_MIXER_DELTA) {
+            ok = ok && s.kv_heads > 0 && s.heads % s.kv_heads == 0 && s.dim <= 256 && s.taps >= 1 && s.decay_rank > 0 && s.gate_rank > 0;
+            L.KD = 32;
+            while (L.KD < s.dim) L.KD *= 2;
+            L.VD = pad32(s.vdim);
+            L.rank = pad32(std::max(s.decay_rank, s.gate_rank));
+            L.gcols = s.heads * std::max(L.KD, L.VD);
+        } else {
+            ok = false;
+        }
+        L.ff = pad32(s.inter);
+        if (!ok) {
+            delete p;
+            XFT_REQUIRE(false, "xfthip_plan_create: layer %d has sizes this library does not serve", i);
+        }
+        p->layers.push_back(L);
+    }
+    auto add = [&](int from, int to, bool again) {
+        for (int i = from; i < to; ++i) p->runs.push_back({i, again && i == from});
+    };
+    add(0, loop ? c.loop_start : c.layers, false);
+    if (loop) {
+        for (int t = 0; t < c.loop_times; ++t) add(c.loop_start, c.loop_stop, t > 0);
+        add(c.loop_stop, c.layers, false);
+    }
+    *out = p;
+    return 0;
+}
+
+int xfthip_plan_destroy(xfthip_plan_t p) {
+    if (!p) return 0;
+    for (PlanLayer &L : p->layers) {
+        for (xfthip_weight_t w : {L.in, L.o, L.gateup, L.down, L.uq, L.absorb, L.uk, L.uv, L.gates}) xfthip_weight_destroy(w);
+        for (float *f : {L.q_norm, L.kv_norm, L.sink, L.conv, L.decay, L.dt_bias, L.out_norm, L.pre1, L.post1, L.pre2, L.post2})
+            if (f) (void)hipFree(f);
+    }
+    xfthip_weight_destroy(p->head);
+    if (p->embedding) (void)hipFree(p->embedding);
+    if (p->final_norm) (void)hipFree(p->final_norm);
+    delete p;
+    return 0;
+}
+
+int xfthip_plan_set_tensor(xfthip_plan_t p, int layer, const char *name, const uint16_t *data_host, int rows, int cols) {
+    XFT_REQUIRE(p && name && data_host && rows > 0 && cols > 0, "xfthip_plan_set_tensor: bad argument");
+    XFT_REQUIRE(!p->finished, "xfthip_plan_set_tensor: the plan is finished");
+    XFT_REQUIRE(layer >= -1 && layer < p->cfg.layers, "xfthip_plan_set_tensor: layer %d out of range", layer);
+    Tensor t;
+    t.rows = rows, t.cols = cols;
+    t.data.assign(data_host, data_host + (size_t)rows * cols);
+    p->pending.emplace_back((layer < 0 ? std::string() : std::to_string(layer) + "/") + name, std::move(t));
+    return 0;
+}
+
+int xfthip_plan_finish(xfthip_plan_t p) {
+    XFT_REQUIRE(p && !p->finished, "xfthip_plan_finish: bad plan");
+    std::map<std::string, Tensor> all;
+    for (auto &kv : p->pending) all[kv.first] = std::move(kv.second);
+    p->pending.clear();
+    std::string prefix, missing;
+    static const Tensor empty;
+    auto get = [&](const char *name, int rows, int cols) -> const Tensor & {
+        auto it = all.find(prefix + name);
+        if (it == all.end() || it->second.rows != rows || it->second.cols != cols) {
+            if (missing.empty()) {
+                missing = prefix + name + ": ";
+                missing += it == all.end() ? std::string("missing")
+                                           : "[" + std::to_string(it->second.rows) + ", " + std::to_string(it->second.cols) + "] instead of ["
+                                + std::to_string(rows) + ", " + std::to_string(cols) + "]";
+            }
+            return empty;
+        }
+        return it->second;
+    };
+    int rc = 0;
+    auto upload = [&](const std::vector<float> &v, float **dst) {
+        if (rc) return;
+        if (hipMalloc((void **)dst, v.size() * 4 + 16) != hipSuccess || hipMemcpy(*dst, v.data(), v.size() * 4, hipMemcpyHostToDevice) != hipSuccess) {
+            set_error("xfthip_plan_finish: upload failed");
+            rc = 1;
+        }
+    };
+    auto pack = [&](const Matrix &w, int flags, xfthip_weight_t *dst) {
+        if (rc) return;
+        rc = xfthip_weight_create(XFTHIP_W_BF16, w.K, w.N, w.w.data(), nullptr, nullptr, flags, dst);
+        if (rc == 0) p->weight_bytes += xfthip_weight_bytes(*dst);
+    };
+    auto values = [&](const Tensor &t, int n) {
+        std::vector<float> v(n, 0.0f);
+        for (int i = 0; i < t.rows * t.cols && i < n; ++i) v[i] = bf16_value(t.data[i]);
+        return v;
+    };
+    const int W = p->cfg.hidden, Wp = p->hidden, V = p->cfg.vocab;
+    auto one_plus = [&](const Tensor &t, const Tensor *scale) {
+        std::vector<float> v(Wp, 0.0f);
+        for (int i = 0; i < t.rows; ++i) v[i] = (1.0f + bf16_value(t.data[i])) * (scale ? bf16_value(scale->data[i]) : 1.0f);
+        return v;
+    };
+#define NEED(var, name, r, c)                 \
+    const Tensor &var = get(name, r, c);      \
+    if (!missing.empty()) break
+    do {
+        NEED(embed, "embed", V, W);
+        NEED(head, "head", V, W);
+        NEED(fin, "final.norm", W, 1);
+        std::vector<uint16_t> table((size_t)V * Wp, 0);
+        for (int v = 0; v < V; ++v) memcpy(&table[(size_t)v * Wp], &embed.data[(size_t)v * W], (size_t)W * 2);
+        if (hipMalloc((void **)&p->embedding, table.size() * 2) != hipSuccess
+                || hipMemcpy(p->embedding, table.data(), table.size() * 2, hipMemcpyHostToDevice) != hipSuccess) {
+            set_error("xfthip_plan_finish: upload failed");
+            rc = 1;
+            break;
+        }
+        std::vector<float> fn = one_plus(fin, nullptr);
+        for (float &f : fn) f *= p->cfg.logit_scale; // the logits are linear in the normed row
+        upload(fn, &p->final_norm);
+        Matrix hm(Wp, V);
+        hm.place(head, 0, V, 0, W, 0, 0);
+        pack(hm, XFTHIP_WF_NONE, &p->head);
+    } while (false);
+    for (int i = 0; i < p->cfg.layers && missing.empty() && rc == 0; ++i) do {
+        PlanLayer &L = p->layers[i];
+        const xfthip_plan_layer &s = L.s;
+        const int H = s.heads;
+        prefix = std::to_string(i) + "/";
+        NEED(n1, "norm1", W, 1);
+        NEED(n1b, "norm1b", W, 1);
+        NEED(ls1, "ls1", W, 1);
+        upload(one_plus(n1, nullptr), &L.pre1);
+        upload(one_plus(n1b, &ls1), &L.post1);
+        if (s.inter > 0) {
+            NEED(n2, "norm2", W, 1);
+            NEED(n2b, "norm2b", W, 1);
+            NEED(ls2, "ls2", W, 1);
+            NEED(gate, "mlp.gate", s.inter, W);
+            NEED(up, "mlp.up", s.inter, W);
+            NEED(down, "mlp.down", W, s.inter);
+            upload(one_plus(n2, nullptr), &L.pre2);
+            upload(one_plus(n2b, &ls2), &L.post2);
+            Matrix gu(Wp, 2 * L.ff), dn(L.ff, Wp);
+            gu.place(gate, 0, s.inter, 0, W, 0, 0);
+            gu.place(up, 0, s.inter, 0, W, 0, L.ff);
+            dn.place(down, 0, W, 0, s.inter, 0, 0);
+            pack(gu, XFTHIP_WF_GATEUP, &L.gateup);
+            pack(dn, XFTHIP_WF_NONE, &L.down);
+        }
+        Matrix in(Wp, L.row_in());
+        if (s.mixer == XFTHIP_MIXER_LATENT) {
+            const int d = s.dim, r = s.rot_dim, dv = s.vdim, R = s.kv_rank;
+            NEED(dq, "mix.dq", s.q_rank, W);
+            NEED(dqn, "mix.dq.norm", s.q_rank, 1);
+            NEED(uq, "mix.uq", H * (d + r), s.q_rank);
+            NEED(dkv, "mix.dkv", R + r, W);
+            NEED(dkvn, "mix.dkv.norm", R, 1);
+            NEED(uk, "mix.uk", H * d, R);
+            NEED(uv, "mix.uv", H * dv, R);
+            NEED(o, "mix.o", W, H * dv);
+            in.place(dq, 0, s.q_rank, 0, W, 0, 0);
+            in.place(dkv, 0, R, 0, W, 0, L.QR);
+            in.place(dkv, R, r, 0, W, 0, L.QR + L.R);
+            Matrix mq(L.QR, H * (L.D + L.RD)), ma(L.D, H * L.R), mk(L.R, H * L.D), mv(L.R, H * L.V), mo(H * L.V, Wp);
+            for (int h = 0; h < H; ++h) {
+                mq.place(uq, h * (d + r), d, 0, s.q_rank, 0, h * (L.D + L.RD));
+                mq.place(uq, h * (d + r) + d, r, 0, s.q_rank, 0, h * (L.D + L.RD) + L.D);
+                ma.place_turned(uk, h * d, d, 0, R, 0, h * L.R);
+                mk.place(uk, h * d, d, 0, R, 0, h * L.D);
+                mv.place(uv, h * dv, dv, 0, R, 0, h * L.V);
+                mo.place(o, 0, W, h * dv, dv, h * L.V, 0);
+            }
+            pack(mq, XFTHIP_WF_NONE, &L.uq);
+            pack(ma, XFTHIP_WF_NONE, &L.absorb);
+            pack(mk, XFTHIP_WF_NONE, &L.uk);
+            pack(mv, XFTHIP_WF_NONE, &L.uv);
+            pack(mo, XFTHIP_WF_NONE, &L.o);
+            upload(values(dqn, L.QR), &L.q_norm);
+            upload(values(dkvn, L.R), &L.kv_norm);
+            if (s.has_sink) {
+                NEED(sink, "mix.sink", H, 1);
+                upload(values(sink, H), &L.sink);
+            }
+        } else {
+            const int KH = s.kv_heads, d = s.dim, dv = s.vdim, n = s.taps;
+            NEED(q, "mix.q", KH * d, W);
+            NEED(k, "mix.k", KH * d, W);
+            NEED(v, "mix.v", H * dv, W);
+            NEED(qc, "mix.q.conv", KH * d, n);
+            NEED(kc, "mix.k.conv", KH * d, n);
+            NEED(vc, "mix.v.conv", H * dv, n);
+            NEED(b, "mix.b", H, W);
+            NEED(al, "mix.A_log", H, 1);
+            NEED(nm, "mix.norm", dv, 1);
+            NEED(a1, "mix.a1", s.decay_rank, W);
+            NEED(a2, "mix.a2", H * d, s.decay_rank);
+            NEED(dt, "mix.dt_bias", H * d, 1);
+            NEED(g1, "mix.g1", s.gate_rank, W);
+            NEED(g2, "mix.g2", H * dv, s.gate_rank);
+            NEED(o, "mix.o", W, H * dv);
+            std::vector<float> conv((size_t)L.channels() * n, 0.0f), dtb((size_t)H * L.KD, 0.0f), dec(H);
+            const int k0 = KH * L.KD, v0 = 2 * KH * L.KD, b0 = L.channels(), a0 = b0 + L.beta_cols(), g0 = a0 + L.rank;
+            auto filters = [&](const Tensor &t, int from, int count, int to) {
+                for (int i2 = 0; i2 < count * n; ++i2) conv[(size_t)to * n + i2] = bf16_value(t.data[(size_t)from * n + i2]);
+            };
+            for (int h = 0; h < KH; ++h) {
+                in.place(q, h * d, d, 0, W, 0, h * L.KD);
+                in.place(k, h * d, d, 0, W, 0, k0 + h * L.KD);
+                filters(qc, h * d, d, h * L.KD);
+                filters(kc, h * d, d, k0 + h * L.KD);
+            }
+            Matrix gt(L.rank, 2 * L.gcols), mo(H * L.VD, Wp);
+            for (int h = 0; h < H; ++h) {
+                in.place(v, h * dv, dv, 0, W, 0, v0 + h * L.VD);
+                filters(vc, h * dv, dv, v0 + h * L.VD);
+                gt.place(a2, h * d, d, 0, s.decay_rank, 0, h * L.KD);
+                gt.place(g2, h * dv, dv, 0, s.gate_rank, 0, L.gcols + h * L.VD);
+                mo.place(o, 0, W, h * dv, dv, h * L.VD, 0);
+                for (int e = 0; e < d; ++e) dtb[(size_t)h * L.KD + e] = bf16_value(dt.data[(size_t)h * d + e]);
+                dec[h] = expf(bf16_value(al.data[h]));
+            }
+            in.place(b, 0, H, 0, W, 0, b0);
+            in.place(a1, 0, s.decay_rank, 0, W, 0, a0);
+            in.place(g1, 0, s.gate_rank, 0, W, 0, g0);
+            pack(gt, XFTHIP_WF_NONE, &L.gates);
+            pack(mo, XFTHIP_WF_NONE, &L.o);
+            upload(conv, &L.conv);
+            upload(dtb, &L.dt_bias);
+            upload(dec, &L.decay);
+            upload(values(nm, L.VD), &L.out_norm);
+        }
+        pack(in, XFTHIP_WF_NONE, &L.in);
+    } while (false);
+#undef NEED
+    XFT_REQUIRE(missing.empty(), "xfthip_plan_finish: tensor %s", missing.c_str());
+    p->finished = rc == 0;
+    return rc;
+}
+
+size_t xfthip_plan_weight_bytes(xfthip_plan_t p) { return p ? p->weight_bytes : 0; }
+
+int xfthip_model_create_from_plan(xfthip_plan_t plan, int act_dtype, int max_batch, int max_seq, int max_tokens, int pool_tokens, xfthip_model_t *out) {
+    XFT_REQUIRE(plan && plan->finished && out, "xfthip_model_create_from_plan: needs a finished plan");
+    XFT_REQUIRE(act_dtype == XFTHIP_BF16 || act_dtype == XFTHIP_F32, "xfthip_model_create_from_plan: activations are bf16 or fp32");
+    XFT_REQUIRE(max_batch > 0 && max_seq > 0 && max_tokens >= max_batch && pool_tokens >= 0, "xfthip_model_create_from_plan: bad limits");
+    xfthip_model *m = new xfthip_model();
+    memset(&m->cfg, 0, sizeof(m->cfg));
+    m->cfg.layers = plan->cfg.layers, m->cfg.hidden = plan->hidden, m->cfg.vocab = plan->cfg.vocab;
+    m->cfg.max_batch = max_batch, m->cfg.max_seq = max_seq, m->cfg.max_tokens = max_tokens, m->cfg.max_pos_embed = max_seq;
+    m->cfg.rms_eps = plan->cfg.eps;
+    m->final_norm = plan->final_norm;
+    m->lm_head = plan->head;
+    m->row_pos.assign(max_batch, -1);
+    PlanState *p = new PlanState();
+    m->plan = p;
+    p->plan = plan, p->layers = plan->layers, p->act = act_dtype, p->esz = act_dtype == XFTHIP_F32 ? 4 : 2, p->slots = max_batch;
+    p->table_stride = (max_seq + kPageTokens - 1) / kPageTokens;
+    p->pages = pool_tokens > 0 ? (pool_tokens + kPageTokens - 1) / kPageTokens : max_batch * p->table_stride;
+    for (int i = p->pages; i-- > 0;) p->free_pages.push_back(i);
+    p->held.resize(max_batch);
+    p->table_host.assign((size_t)max_batch * p->table_stride, 0);
+    p->logit_of_row.resize(max_batch);
+    for (int r = 0; r < max_batch; ++r) p->logit_of_row[r] = r;
+    p->logit_rows = std::max(max_batch, 64);
+    bool ok = true;
+    auto alloc = [&](void *dst, size_t bytes, bool clear = false) {
+        void *b = nullptr;
+        if (!ok) return;
+        if (hipMalloc(&b, bytes + 256) != hipSuccess || (clear && hipMemset(b, 0, bytes + 256) != hipSuccess)) {
+            ok = false;
+            return;
+        }
+        p->owned.push_back(b);
+        memcpy(dst, &b, sizeof(b));
+    };
+    const size_t T = max_tokens, e = p->esz, hidden = plan->hidden;
+    size_t a = 0, cq = 0, q = 0, qa = 0, ov = 0, h = 0, gates = 0, dk = 0, dqk = 0, dg = 0, dv = 0, heads = 0, on = 0;
+    for (const PlanLayer &L : p->layers) {
+        const size_t H = L.s.heads;
+        a = std::max(a, (size_t)L.row_in());
+        h = std::max(h, (size_t)L.ff);
+        if (L.s.mixer == XFTHIP_MIXER_LATENT) {
+            cq = std::max(cq, (size_t)L.QR), q = std::max(q, H * (L.D + L.RD)), qa = std::max(qa, H * L.R), ov = std::max(ov, H * L.V);
+        } else {
+            const size_t KH = L.s.kv_heads;
+            gates = std::max(gates, (size_t)2 * L.gcols), dk = std::max(dk, KH * L.KD), dqk = std::max(dqk, KH), dg = std::max(dg, H * L.KD);
+            dv = std::max(dv, H * L.VD), heads = std::max(heads, H), on = std::max(on, H * L.VD);
+        }
+    }
+    alloc(&p->xn, std::max(T, (size_t)p->logit_rows) * hidden * e);
+    alloc(&p->y, T * hidden * 4);
+    alloc(&p->a, T * a * e), alloc(&p->cq, T * cq * e), alloc(&p->q, T * q * e), alloc(&p->qa, T * qa * e), alloc(&p->oc, T * qa * e);
+    alloc(&p->ov, T * ov * e), alloc(&p->h, T * h * e), alloc(&p->on, T * on * e);
+    alloc(&p->gates, T * gates * 4), alloc(&p->dq, T * dk * 4), alloc(&p->dk, T * dk * 4), alloc(&p->dqk, T * dqk * 4), alloc(&p->dg, T * dg * 4);
+    alloc(&p->dv, T * dv * 4), alloc(&p->dbeta, T * heads * 4), alloc(&p->do_, T * dv * 4);
+    for (const LayerRun &r : plan->runs) {
+        const PlanLayer &L = p->layers[r.layer];
+        LatentCacheView cv = {nullptr, L.R, L.RD};
+        float *state = nullptr;
+        void *conv = nullptr;
+        if (L.s.mixer == XFTHIP_MIXER_LATENT) {
+            // cleared: keys that lie behind a sequence's end are multiplied by zero weights and must be numbers
+            alloc(&cv.pool, (size_t)p->pages * kPageTokens * (L.R + L.RD) * e, true);
+        } else {
+            alloc(&state, (size_t)max_batch * L.s.heads * L.VD * L.KD * 4, true);
+            alloc(&conv, (size_t)max_batch * (L.s.taps - 1) * L.channels() * e, true);
+        }
+        p->cache.push_back(cv), p->state.push_back(state), p->conv_state.push_back(conv);
+    }
+    alloc(&p->table, p->table_host.size() * 4, true);
+    alloc(&p->desc, (3 * T + 4 * (size_t)max_batch) * 4, true);
+    alloc(&p->dec_rows, (size_t)max_batch * 4, true);
+    alloc(&p->want, (size_t)p->logit_rows * 4, true);
+    std::map<std::pair<double, int>, std::pair<float *, float *>> rot;
+    for (PlanLayer &L : p->layers) {
+        if (L.s.mixer != XFTHIP_MIXER_LATENT || !ok) continue;
+        auto &t = rot[{L.s.rot_base, L.s.rot_dim}];
+        if (!t.first) {
+            ok = rotation_tables(L.s.rot_base, L.s.rot_dim, max_seq, &t.first, &t.second) == 0;
+            if (t.first) p->owned.push_back(t.first);
+            if (t.second) p->owned.push_back(t.second);
+        }
+        L.cosT = t.first, L.sinT = t.second;
+    }
+    ok = ok && hipHostMalloc((void **)&p->desc_host, (3 * T + 4 * (size_t)max_batch) * 4) == hipSuccess;
+    p->tok_seg = p->desc, p->tok_pos = p->desc + T, p->ids = p->desc + 2 * T, p->seg = p->desc + 3 * T;
+    const size_t nids = T > 64 ? T : 64;
+    m->idlog_cap = max_seq + 1;
+    ok = ok && hipMalloc((void **)&m->x, T * hidden * 4) == hipSuccess && hipMalloc((void **)&m->ids, nids * 4) == hipSuccess
+            && hipMemset(m->ids, 0, nids * 4) == hipSuccess && hipMalloc((void **)&m->pos, (size_t)max_batch * 4) == hipSuccess
+            && hipMemset(m->pos, 0, (size_t)max_batch * 4) == hipSuccess && hipMalloc((void **)&m->step, 64) == hipSuccess
+            && hipMemset(m->step, 0, 64) == hipSuccess
+            && hipMalloc((void **)&m->logits, (size_t)p->logit_rows * plan->cfg.vocab * 4) == hipSuccess
+            && hipMalloc((void **)&m->idlog, (size_t)m->idlog_cap * max_batch * 4) == hipSuccess;
+    if (!ok) {
+        set_error("xfthip_model_create_from_plan: out of device memory");
+        xfthip_model_destroy(m);
+        return 1;
+    }
+    *out = m;
+    return 0;
+}
+
+int xfthip_model_trace_residual(xfthip_model_t m, int enable) {
+    XFT_REQUIRE(m && m->plan, "xfthip_model_trace_residual: only for models from a plan");
+    m->plan->trace = enable != 0;
+    m->plan->trace_tokens = 0;
+    return 0;
+}
+
+int xfthip_model_read_residual(xfthip_model_t m, float *out_host, int *runs, int *tokens) {
+    XFT_REQUIRE(m && m->plan, "xfthip_model_read_residual: only for models from a plan");
+    const PlanState &p = *m->plan;
+    const int n = (int)p.plan->runs.size(), T = p.trace_tokens, W = p.plan->cfg.hidden, Wp = p.plan->hidden;
+    if (runs) *runs = n;
+    if (tokens) *tokens = T;
+    if (!out_host) return 0;
+    XFT_REQUIRE(T > 0, "xfthip_model_read_residual: nothing traced yet");
+    XFT_CHECK_HIP(hipDeviceSynchronize());
+    XFT_CHECK_HIP(hipMemcpy2D(out_host, (size_t)W * 4, p.trace_buf, (size_t)Wp * 4, (size_t)W * 4, (size_t)n * T, hipMemcpyDeviceToHost));
+    return 0;
+}
+
+int xfthip_model_pool_pages(xfthip_model_t m, int *free_pages, int *total_pages) {
+    XFT_REQUIRE(m && m->plan, "xfthip_model_pool_pages: only for models from a plan");
+    if (free_pages) *free_pages = (int)m->plan->free_pages.size();
+    if (total_pages) *total_pages = m->plan->pages;
+    return 0;
+}
+
+} // extern "C"

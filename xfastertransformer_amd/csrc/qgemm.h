@@ -25,7 +25,8 @@ struct SkinnyParams {
     const void *res;
     int ldres, res_dtype;
     float gamma;
-    int gateup; // 1: combine tile pairs as silu(gate)*up, N counts cat columns
+    int gateup; // 1: combine tile pairs as silu(gate)*up, N counts cat columns; 2: as clamped_glu (below)
+    float glu_limit, glu_alpha; // gateup == 2
     int nblocks; // column blocks of the launch (set by the launcher)
     // K split of the M > 32 kernel (few rows against few columns and a deep K): workgroup row blockIdx.y
     // multiplies k tiles [y * split_ktiles, (y + 1) * split_ktiles) and writes its scaled partial result as
@@ -62,6 +63,12 @@ struct SkinnyParams {
     int qH, kvH;
     KvView kv;
 };
+
+// The clamped gated unit: g = min(gate, limit), u = clamp(up, -limit, limit), g * sigmoid(alpha g) * (u + 1)
+__device__ inline float clamped_glu(float gate, float up, float limit, float alpha) {
+    const float g = fminf(gate, limit), u = fminf(fmaxf(up, -limit), limit);
+    return g / (1.0f + fast_exp(-alpha * g)) * (u + 1.0f);
+}
 
 int qgemm_skinny(const PackedWeight &pw, const SkinnyParams &p, hipStream_t stream); // M <= 32
 bool skinny_can_fuse_norm(const PackedWeight &pw, int M); // may SkinnyParams::norm_x be used

@@ -774,7 +774,7 @@ __global__ __launch_bounds__(256 * KG, (DIRECT && KG == 1) ? 2 : 1) void qgemm_m
                         x = s[t] * x;
                     }
                     const float other = __shfl_xor(x, 16, 64); // gate <-> up partner
-                    put_at(put_base, 16 * t, j, other * silu_big(x));
+                    put_at(put_base, 16 * t, j, p.gateup == 2 ? clamped_glu(x, other, p.glu_limit, p.glu_alpha) : other * silu_big(x));
                 }
             }
             flush(std::integral_constant<int, XFTHIP_EPI_NONE> {}, row_tile(m), n32_0 * 16, 16 * WN, p.N / 2);

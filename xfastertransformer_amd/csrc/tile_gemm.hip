@@ -1,0 +1,158 @@
+// Matrix products of layer plans that the weight-only GEMMs do not cover: 32-bit activations (true fp32 products on the
+// fp32 matrix units), and heads side by side (every block of output columns multiplies its own slice of the activation
+// row, the per-head products of latent attention and the two gates of the delta rule).  BF16 weights in the packed layout
+// of common.h.
+#include "plan.h"
+
+namespace xfthip {
+
+namespace {
+
+struct TileGemm {
+    const uint8_t *packed;
+    int KT, ktiles, NTILES, N, M;
+    const void *A;
+    int lda, tiles_per_block, a_block_stride;
+    void *C;
+    int ldc, c_dtype, glu;
+    float glu_limit, glu_alpha;
+};
+
+typedef uint32_t u32x4 __attribute__((ext_vector_type(4)));
+
+__device__ inline float precise_glu(float gate, float up, float limit, float alpha) {
+    const float g = fminf(gate, limit), u = fminf(fmaxf(up, -limit), limit);
+    return g / (1.0f + expf(-alpha * g)) * (u + 1.0f);
+}
+
+// A wave: two column tiles (16 weight columns each) x MT row tiles (16 activation rows each).  The weight tile is the MFMA
+// A operand, the activation rows the B operand: a lane ends up with four neighbouring columns of one row.  With fp32
+// activations step j of a 32-row weight tile multiplies rows 8 g + j of the four lane groups g.
+template <bool F32, int MT>
+__global__ __launch_bounds__(256) void tile_gemm_kernel(TileGemm p) {
+    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+    const int g = lane >> 4, ml = lane & 15;
+    const int nt0 = (blockIdx.x * 4 + wave) * 2;
+    if (nt0 >= p.NTILES) return;
+    const int m0 = blockIdx.y * 16 * MT;
+    const uint8_t *w[2];
+    int aofs[2];
+#pragma unroll
+    for (int t = 0; t < 2; ++t) {
+        const int nt = nt0 + t < p.NTILES ? nt0 + t : p.NTILES - 1;
+        w[t] = p.packed + (size_t)nt * p.KT * 1024 + lane * 16;
+        aofs[t] = p.tiles_per_block ? nt / p.tiles_per_block * p.a_block_stride : 0;
+    }
+    const bool same = aofs[0] == aofs[1];
+    size_t row[MT];
+#pragma unroll
+    for (int m = 0; m < MT; ++m) {
+        const int r = m0 + m * 16 + ml;
+        row[m] = (size_t)(r < p.M ? r : p.M - 1) * p.lda + 8 * g;
+    }
+    f32x4 acc[2][MT];
+#pragma unroll
+    for (int t = 0; t < 2; ++t)
+#pragma unroll
+        for (int m = 0; m < MT; ++m) acc[t][m] = f32x4 {0.f, 0.f, 0.f, 0.f};
+
+#pragma unroll 2
+    for (int kt = 0; kt < p.ktiles; ++kt) {
+        u32x4 wq[2];
+#pragma unroll
+        for (int t = 0; t < 2; ++t) wq[t] = *(const u32x4 *)(w[t] + (size_t)kt * 1024);
+        if constexpr (F32) {
+            const float *A = (const float *)p.A;
+#pragma unroll
+            for (int m = 0; m < MT; ++m) {
+                f32x4 a[2][2];
+                a[0][0] = *(const f32x4 *)(A + row[m] + aofs[0] + kt * 32), a[0][1] = *(const f32x4 *)(A + row[m] + aofs[0] + kt * 32 + 4);
+                if (same) {
+                    a[1][0] = a[0][0], a[1][1] = a[0][1];
+                } else {
+                    a[1][0] = *(const f32x4 *)(A + row[m] + aofs[1] + kt * 32), a[1][1] = *(const f32x4 *)(A + row[m] + aofs[1] + kt * 32 + 4);
+                }
+#pragma unroll
+                for (int t = 0; t < 2; ++t)
+#pragma unroll
+                    for (int j = 0; j < 8; ++j) {
+                        const uint32_t pair = wq[t][j >> 1];
+                        const float wv = u2f((j & 1) ? (pair & 0xFFFF0000u) : (pair << 16));
+                        acc[t][m] = __builtin_amdgcn_mfma_f32_16x16x4f32(wv, a[t][j >> 2][j & 3], acc[t][m], 0, 0, 0);
+                    }
+            }
+        } else {
+            const uint16_t *A = (const uint16_t *)p.A;
+#pragma unroll
+            for (int m = 0; m < MT; ++m) {
+                u32x4 a0 = *(const u32x4 *)(A + row[m] + aofs[0] + kt * 32), a1 = a0;
+                if (!same) a1 = *(const u32x4 *)(A + row[m] + aofs[1] + kt * 32);
+                acc[0][m] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, wq[0]), __builtin_bit_cast(bf16x8, a0), acc[0][m], 0, 0, 0);
+                acc[1][m] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, wq[1]), __builtin_bit_cast(bf16x8, a1), acc[1][m], 0, 0, 0);
+            }
+        }
+    }
+
+#pragma unroll
+    for (int m = 0; m < MT; ++m) {
+        const int r = m0 + m * 16 + ml;
+        if (r >= p.M) continue;
+        if (p.glu) { // tile pairs: 16 gate columns, the matching 16 up columns
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+                const int n = (nt0 >> 1) * 16 + 4 * g + i;
+                if (n < p.N / 2)
+                    store_from_f32(p.C, p.c_dtype, (size_t)r * p.ldc + n, precise_glu(acc[0][m][i], acc[1][m][i], p.glu_limit, p.glu_alpha));
+            }
+            continue;
+        }
+#pragma unroll
+        for (int t = 0; t < 2; ++t) {
+            const int n = (nt0 + t) * 16 + 4 * g;
+            const size_t at = (size_t)r * p.ldc + n;
+            if (n + 4 <= p.N && (p.ldc & 3) == 0) {
+                if (p.c_dtype == XFTHIP_F32)
+                    *(f32x4 *)((float *)p.C + at) = acc[t][m];
+                else
+                    *(uint2 *)((uint16_t *)p.C + at) = make_uint2(f32_to_bf16_ref(acc[t][m][0]) | ((uint32_t)f32_to_bf16_ref(acc[t][m][1]) << 16),
+                            f32_to_bf16_ref(acc[t][m][2]) | ((uint32_t)f32_to_bf16_ref(acc[t][m][3]) << 16));
+            } else {
+#pragma unroll
+                for (int i = 0; i < 4; ++i)
+                    if (n + i < p.N) store_from_f32(p.C, p.c_dtype, at + i, acc[t][m][i]);
+            }
+        }
+    }
+}
+
+} // namespace
+
+int tile_gemm(xfthip_weight_t w, int act_in, int M, const void *A, int lda, int block_cols, int a_block_stride, void *C, int ldc, int c_dtype,
+        int glu, float glu_limit, float glu_alpha, hipStream_t st) {
+    XFT_REQUIRE(w && A && C && M > 0, "tile_gemm: null argument");
+    const PackedWeight &pw = w->pw;
+    XFT_REQUIRE(pw.kind == XFTHIP_W_BF16 && pw.K % 32 == 0, "tile_gemm: BF16 weights with K a multiple of 32 (K=%d)", pw.K);
+    XFT_REQUIRE(block_cols % 16 == 0 && lda % 8 == 0 && a_block_stride % 8 == 0 && ((uintptr_t)A & 15) == 0, "tile_gemm: unaligned operands");
+    const int blocks = block_cols ? (pw.N + block_cols - 1) / block_cols : 1;
+    XFT_REQUIRE((long)(blocks - 1) * a_block_stride + pw.K <= lda, "tile_gemm: %d blocks of K=%d reach past the row (%d)", blocks, pw.K, lda);
+    XFT_REQUIRE(ldc >= (glu ? pw.N / 2 : pw.N) && (glu != 0) == ((pw.flags & XFTHIP_WF_GATEUP) != 0), "tile_gemm: ldc=%d N=%d glu=%d", ldc, pw.N, glu);
+    TileGemm p = {pw.packed, pw.KT, pw.K / 32, pw.NTILES, pw.N, M, A, lda, block_cols / 16, a_block_stride, C, ldc, c_dtype, glu, glu_limit, glu_alpha};
+    const unsigned gx = (unsigned)((pw.NTILES + 7) / 8);
+    const bool few = M <= 16 || (long)gx * ((M + 63) / 64) < 2L * device_cu_count();
+    const unsigned gy = (unsigned)((M + (few ? 16 : 64) - 1) / (few ? 16 : 64));
+    if (act_in == XFTHIP_F32) {
+        if (few)
+            hipLaunchKernelGGL((tile_gemm_kernel<true, 1>), dim3(gx, gy), dim3(256), 0, st, p);
+        else
+            hipLaunchKernelGGL((tile_gemm_kernel<true, 4>), dim3(gx, gy), dim3(256), 0, st, p);
+    } else {
+        if (few)
+            hipLaunchKernelGGL((tile_gemm_kernel<false, 1>), dim3(gx, gy), dim3(256), 0, st, p);
+        else
+            hipLaunchKernelGGL((tile_gemm_kernel<false, 4>), dim3(gx, gy), dim3(256), 0, st, p);
+    }
+    XFT_CHECK_HIP(hipGetLastError());
+    return 0;
+}
+
+} // namespace xfthip
