@@ -4,7 +4,7 @@
     python bench.py [--gpus 1] [--steps K] [--warmup W] [--batch B] [--weights int8|uint4] [--kv fp16|int8]
                     [--eager | --no-fusion]                       (variants of the decode step)
                     [--no-extras] [--no-cpu-baseline]
-                    [--prefill-gemm | --attention | --moe | --stream-floor]   (one of the extra measurements alone, one JSON line)
+                    [--prefill-gemm | --attention | --moe | --plan | --stream-floor]   (one of the extra measurements alone, one JSON line)
                     [--pmc-workload | --pmc-summary FETCH_CSV WRITE_CSV]   (hardware-counter traffic)
 
 Workload (configs[3] of the benchmark definition): a 32-layer Llama-2-7B-shape model with random weights
@@ -606,6 +606,122 @@ def moe_layer(xh, iters=5):
                      "counts stay on the device)")
 
 
+PLAN_SIZES = {
+    # width, ff, heads, query latent (the rest: 128 / 64 query dims, 128 value dims, key latent 512, 128-dim delta heads)
+    "2048": dict(width=2048, ff=5632, heads=16, q_rank=768),
+    "4096": dict(width=4096, ff=11008, heads=32, q_rank=1536),
+}
+
+
+def plan_shapes(sz):
+    """Layer descriptions and tensor shapes of a Pinepel stack at a real model's sizes: windowed latent attention, latent
+    attention with a sink, delta rule, twice over."""
+    W, F, H, Q = sz["width"], sz["ff"], sz["heads"], sz["q_rank"]
+    ff = dict(inter=F, glu_limit=7.0, glu_alpha=1.702)
+    latent = dict(mixer=1, heads=H, dim=128, vdim=128, rot_dim=64, kv_rank=512, q_rank=Q, scale=192 ** -0.5, rot_base=1e6, **ff)
+    kinds = [dict(latent, rot_interleaved=1, window=1024), dict(latent, has_sink=1),
+             dict(mixer=2, heads=H, kv_heads=H, dim=128, vdim=128, taps=4, decay_rank=128, gate_rank=128, **ff)]
+    norms = {n: (W,) for n in ("norm1", "norm1b", "ls1", "norm2", "norm2b", "ls2")}
+    mlp = {"mlp.gate": (F, W), "mlp.up": (F, W), "mlp.down": (W, F)}
+    lat = {"mix.dq": (Q, W), "mix.dq.norm": (Q,), "mix.uq": (H * 192, Q), "mix.dkv": (576, W), "mix.dkv.norm": (512,), "mix.uk": (H * 128, 512),
+           "mix.uv": (H * 128, 512), "mix.o": (W, H * 128)}
+    D = H * 128
+    delta = {"mix.b": (H, W), "mix.A_log": (H,), "mix.norm": (128,), "mix.a1": (128, W), "mix.a2": (D, 128), "mix.dt_bias": (D,),
+             "mix.g1": (128, W), "mix.g2": (D, 128), "mix.o": (W, D)}
+    for n in ("q", "k", "v"):
+        delta["mix." + n], delta["mix." + n + ".conv"] = (D, W), (D, 4)
+    shapes = [dict(norms, **mlp, **lat), dict(norms, **mlp, **lat, **{"mix.sink": (H,)}), dict(norms, **mlp, **delta)]
+    return kinds * 2, shapes * 2
+
+
+def build_plan(xh, sz, vocab=32000):
+    layers, shapes = plan_shapes(sz)
+    pool = xh.f32_to_bf16_bits(np.random.default_rng(5).standard_normal(1 << 22, dtype=np.float32) * 0.02)
+    plan = xh.Plan(sz["width"], vocab, layers)
+    cache = {}
+
+    def bits(shape):
+        if shape not in cache:
+            n = int(np.prod(shape))
+            cache[shape] = np.resize(pool, n).reshape(shape)
+        return cache[shape]
+
+    for n, s in (("embed", (vocab, sz["width"])), ("head", (vocab, sz["width"])), ("final.norm", (sz["width"],))):
+        plan.set(-1, n, bits(s))
+    for l, tensors in enumerate(shapes):
+        for n, s in tensors.items():
+            plan.set(l, n, bits(s))
+    plan.finish()
+    return plan
+
+
+def build_llama_bf16(xh, sz, layers, batch, max_seq, max_tokens, vocab=32000):
+    """The closest uniform stack: same width, feed-forward and layer count, multi-head attention, BF16 weights."""
+    W, F, H = sz["width"], sz["ff"], sz["width"] // 128
+    pool = xh.f32_to_bf16_bits(np.random.default_rng(5).standard_normal(1 << 22, dtype=np.float32) * 0.02)
+    model = xh.Model(layers, W, F, H, H, 128, vocab=vocab, max_batch=batch, max_seq=max_seq, max_tokens=max_tokens, max_pos_embed=max_seq)
+    ones = np.ones(W, np.float32)
+    ws = []
+    for l in range(layers):
+        w = [xh.Weight(xh.W_BF16, K, N, np.resize(pool, K * N), flags=xh.WF_GATEUP if i == 2 else xh.WF_NONE)
+             for i, (K, N) in enumerate(((W, 3 * W), (W, W), (W, 2 * F), (F, W)))]
+        model.set_layer(l, *w, ones, ones)
+        ws += w
+    lm = xh.Weight(xh.W_BF16, W, vocab, np.resize(pool, W * vocab))
+    emb = (np.random.default_rng(6).standard_normal((vocab, W), dtype=np.float32) * 0.02).astype(np.float16).view(np.uint16)
+    model.set_head(emb, ones, lm)
+    return model, ws + [lm]
+
+
+def plan_bench(xh, prompt=2048, batches=(1, 8, 32), steps=32, only=None, sizes=None, eager=False):
+    """Prefill (one prompt) and decode (behind prompts of that length) of Pinepel beside the uniform stack, six layers
+    each, in the same run.  Prompts of a decode batch are run one by one."""
+    out = []
+    for name in sizes or PLAN_SIZES:
+        sz = PLAN_SIZES[name]
+        for which in ("pinepel", "llama_bf16"):
+            if only and which != only:
+                continue
+            B, max_seq = max(batches), prompt + 4 * (steps + 8)
+            keep = []
+            if which == "pinepel":
+                plan = build_plan(xh, sz)
+                model, wbytes = xh.PlanModel(plan, xh.BF16, B, max_seq, prompt), plan.bytes()
+                keep = [plan]
+            else:
+                model, keep = build_llama_bf16(xh, sz, 6, B, max_seq, prompt)
+                wbytes = sum(w.bytes() for w in keep)
+            model.use_graph(not eager)
+            ids = np.random.default_rng(7).integers(0, 32000, (1, prompt)).astype(np.int32)
+            times = []
+            for _ in range(4):
+                t0 = time.time()
+                model.prefill(ids)
+                xh.synchronize()
+                times.append(time.time() - t0)
+            r = dict(model=which, width=sz["width"], layers=6, weight_bytes=wbytes, prompt=prompt, prefill_ms=round(min(times[1:]) * 1e3, 3),
+                     prefill_tok_s=round(prompt / min(times[1:]), 1), decode=[])
+            for b in batches:
+                for row in range(b):
+                    model.seq_prefill(row, ids[0])
+                rows = list(range(b))
+                for _ in range(4):
+                    model.seq_decode(rows)
+                t0 = time.time()
+                for _ in range(steps):
+                    model.seq_decode(rows)
+                dt = time.time() - t0
+                r["decode"].append(dict(batch=b, ms_per_step=round(dt * 1e3 / steps, 4), tok_s=round(b * steps / dt, 1)))
+                for row in rows:
+                    model.seq_release(row)
+            out.append(r)
+            print(json.dumps(r), file=sys.stderr, flush=True)
+            model.free()
+            for k in keep:
+                k.free()
+    return out
+
+
 def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -624,6 +740,9 @@ def main():
     ap.add_argument("--prefill-gemm", action="store_true", help="only the weight-only GEMM sweep: M = 256, 2048 against the MFMA peak, M = 1, 8, 32 against the HBM peak (one JSON line)")
     ap.add_argument("--attention", action="store_true", help="only the GQA attention sweep (one JSON line)")
     ap.add_argument("--moe", action="store_true", help="only the sparse-MLP layer (one JSON line)")
+    ap.add_argument("--plan", action="store_true", help="only the layer-plan stack (Pinepel) beside the uniform BF16 stack of equal size: prefill and decode (one JSON line; progress on stderr)")
+    ap.add_argument("--plan-only", choices=["pinepel", "llama_bf16"], help="with --plan: one of the two")
+    ap.add_argument("--plan-size", choices=sorted(PLAN_SIZES), help="with --plan: one width")
     ap.add_argument("--no-live-traffic", action="store_true", help="do not run the two rocprofv3 counter passes for roofline.traffic (the recorded figure under profiles/ is reported instead)")
     ap.add_argument("--stream-floor", action="store_true", help="only the read-only streaming floor at the decode GEMVs' byte counts (one JSON line)")
     args = ap.parse_args()
@@ -636,7 +755,7 @@ def main():
 
     # HBM counters of the dominant kernel, measured by two profiler passes over child runs of this file: only in the
     # full default run (the headline configuration), and first, while this process has not touched the GPU
-    single = args.prefill_gemm or args.attention or args.moe or args.stream_floor or args.pmc_workload or args.eager or args.no_extras
+    single = args.prefill_gemm or args.attention or args.moe or args.plan or args.stream_floor or args.pmc_workload or args.eager or args.no_extras
     live = None
     if not single and not args.no_live_traffic and args.weights == "int8" and args.batch == 1 and args.kv == "fp16":
         live = live_traffic()
@@ -652,6 +771,9 @@ def main():
         return
     if args.moe:
         print(json.dumps({"moe": moe_layer(xh)}))
+        return
+    if args.plan:
+        print(json.dumps({"plan": plan_bench(xh, only=args.plan_only, sizes=[args.plan_size] if args.plan_size else None, eager=args.eager)}))
         return
     if args.stream_floor:
         print(json.dumps({"stream_floor": stream_floor(xh), "hbm_peak_gbs": HBM_PEAK_GBS}))

@@ -71,7 +71,7 @@ def build_hip(force=True):
         reap(running.pop(0))
     if failed:
         raise RuntimeError("hipcc failed")
-    if force or built or not os.path.exists(LIB_HIP):
+    if force or built or _stale(LIB_HIP, objs):
         _run([HIPCC, "--offload-arch=gfx950", "-shared", "-fPIC", "-o", LIB_HIP] + objs)
     return LIB_HIP
 

@@ -530,6 +530,97 @@ class Model:
             pass
 
 
+class PlanLayer(C.Structure):
+    _fields_ = [("mixer", C.c_int), ("heads", C.c_int), ("kv_heads", C.c_int), ("dim", C.c_int), ("vdim", C.c_int), ("rot_dim", C.c_int),
+                ("kv_rank", C.c_int), ("q_rank", C.c_int), ("rot_interleaved", C.c_int), ("window", C.c_int), ("has_sink", C.c_int),
+                ("scale", C.c_float), ("rot_base", C.c_double), ("taps", C.c_int), ("decay_rank", C.c_int), ("gate_rank", C.c_int),
+                ("inter", C.c_int), ("glu_limit", C.c_float), ("glu_alpha", C.c_float)]
+
+
+class PlanConfig(C.Structure):
+    _fields_ = [("layers", C.c_int), ("hidden", C.c_int), ("vocab", C.c_int), ("loop_start", C.c_int), ("loop_stop", C.c_int),
+                ("loop_times", C.c_int), ("eps", C.c_float), ("logit_scale", C.c_float)]
+
+
+MIXER_LATENT, MIXER_DELTA = 1, 2
+lib.xfthip_plan_weight_bytes.restype = C.c_size_t
+lib.xfthip_plan_weight_bytes.argtypes = [C.c_void_p]
+
+
+class Plan:
+    """A stack of layers of several kinds (xfthip_plan_*).  layers: dicts of PlanLayer fields."""
+
+    def __init__(self, hidden, vocab, layers, loop=(0, 0, 1), eps=1e-6, logit_scale=1.0):
+        arr = (PlanLayer * len(layers))(*[PlanLayer(**f) for f in layers])
+        self.cfg = PlanConfig(len(layers), hidden, vocab, loop[0], loop[1], loop[2], eps, logit_scale)
+        self.layers = layers
+        h = C.c_void_p()
+        check(lib.xfthip_plan_create(C.byref(self.cfg), arr, C.byref(h)))
+        self.h = h
+
+    def set(self, layer, name, bits):
+        """bits: uint16 bf16 patterns, [rows, cols] or [n]"""
+        bits = np.ascontiguousarray(bits, np.uint16)
+        rows = bits.shape[0]
+        check(lib.xfthip_plan_set_tensor(self.h, layer, name.encode(), _hp(bits), rows, bits.size // rows))
+
+    def finish(self):
+        check(lib.xfthip_plan_finish(self.h))
+
+    def bytes(self):
+        return int(lib.xfthip_plan_weight_bytes(self.h))
+
+    def free(self):
+        if self.h is not None:
+            lib.xfthip_plan_destroy(self.h)
+            self.h = None
+
+    def __del__(self):
+        try:
+            self.free()
+        except Exception:
+            pass
+
+
+class PlanModel(Model):
+    """A device model over a finished Plan; act = BF16 or F32."""
+
+    def __init__(self, plan, act=BF16, max_batch=1, max_seq=256, max_tokens=None, pool_tokens=0):
+        c = plan.cfg
+        self.cfg = ModelConfig(c.layers, c.hidden, 0, 0, 0, 0, c.vocab, max_batch, max_seq, max_tokens or max_batch * max_seq, max_seq, 0, FP16,
+                               c.eps)
+        h = C.c_void_p()
+        check(lib.xfthip_model_create_from_plan(plan.h, act, max_batch, max_seq, self.cfg.max_tokens, pool_tokens, C.byref(h)))
+        self.h = h
+        self._keep = [plan]
+
+    def step(self, entries, stream=None):
+        """entries: (slot, tokens, places wanted) each; logits fp32 [wanted, vocab]"""
+        rows = np.asarray([e[0] for e in entries], np.int32)
+        lens = np.asarray([len(e[1]) for e in entries], np.int32)
+        ids = np.asarray([t for e in entries for t in e[1]], np.int32)
+        starts = np.concatenate([[0], np.cumsum(lens)[:-1]])
+        want = np.asarray([s + w for e, s in zip(entries, starts) for w in e[2]], np.int32)
+        out = np.empty((len(want), self.cfg.vocab), np.float32)
+        check(lib.xfthip_model_step(self.h, len(entries), _hp(rows), _hp(lens), _hp(ids), len(want), _hp(want), _hp(out), stream))
+        return out
+
+    def trace_residual(self, enable):
+        check(lib.xfthip_model_trace_residual(self.h, int(enable)))
+
+    def read_residual(self):
+        runs, tokens = C.c_int(), C.c_int()
+        check(lib.xfthip_model_read_residual(self.h, None, C.byref(runs), C.byref(tokens)))
+        out = np.empty((runs.value, tokens.value, self.cfg.hidden), np.float32)
+        check(lib.xfthip_model_read_residual(self.h, _hp(out), None, None))
+        return out
+
+    def pool_pages(self):
+        free, total = C.c_int(), C.c_int()
+        check(lib.xfthip_model_pool_pages(self.h, C.byref(free), C.byref(total)))
+        return free.value, total.value
+
+
 def paged_attention_decode(out_dev, q_dev, k_dev, v_dev, q_heads, kv_heads, head, q_stride, kv_stride, o_stride, scale, batch,
                            kcache_dev, vcache_dev, block_num, block_size, tables_dev, table_stride, ctx_dev, slots_dev, max_context,
                            stream=None):

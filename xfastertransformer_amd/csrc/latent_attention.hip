@@ -3,7 +3,8 @@
 //
 // Absorbed form: a query is carried into the latent space by its head's W_uk turned round, scores are products with the
 // cached rows themselves, and the weighted sum of latents is carried to the value space by W_uv behind the softmax.  All
-// heads of a token then read the same cache rows.
+// heads of a token then read the same cache rows.  Expanded form: keys and values of every head are made from the latents of
+// the whole context first, which pays when many tokens attend to them.
 #include "plan.h"
 
 namespace xfthip {
@@ -108,7 +109,7 @@ struct AttendParams {
     void *out;
     LatentCacheView cache;
     const float *sink; // or null
-    int H, D, window;
+    int H, D, window, max_len; // segments longer than max_len are somebody else's
     float scale;
 };
 
@@ -122,6 +123,7 @@ __global__ __launch_bounds__(256) void latent_attend_kernel(AttendParams p) {
     size_t *kr = (size_t *)(part + 8); // (8-byte aligned: R, RD are multiples of 32)
     const int t = blockIdx.x, h = blockIdx.y;
     const int seg = p.v.tok_seg[t], pos = p.v.tok_pos[t], slot = p.v.seg_row[seg];
+    if (p.v.seg_len[seg] > p.max_len) return;
     for (int c = threadIdx.x; c < R; c += 256) qs[c] = ldact<BF16>(p.qa, ((size_t)t * p.H + h) * R + c), o[c] = 0.0f;
     for (int c = threadIdx.x; c < RD; c += 256) qs[R + c] = ldact<BF16>(p.q, ((size_t)t * p.H + h) * (p.D + RD) + p.D + c);
     const int first = p.window > 0 && pos + 1 > p.window ? pos + 1 - p.window : 0;
@@ -160,6 +162,417 @@ __global__ __launch_bounds__(256) void latent_attend_kernel(AttendParams p) {
     for (int c = threadIdx.x; c < R; c += 256) stact<BF16>(p.out, ((size_t)t * p.H + h) * R + c, o[c] / l);
 }
 
+typedef uint32_t u32x4 __attribute__((ext_vector_type(4)));
+typedef __attribute__((ext_vector_type(4))) short s16x4;
+typedef __attribute__((ext_vector_type(8))) short s16x8;
+#define LDS_PTR(type, p) ((__attribute__((address_space(3))) type *)(p))
+
+constexpr float kUnseen = -1.0e30f; // score of a masked key, maximum of a column that has seen none
+constexpr float kLog2e = 1.4426950408889634f;
+
+__device__ inline bf16x8 pack_bf16x8(const float (&v)[8]) {
+    u32x4 u;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) u[i] = f32_to_bf16_ref(v[2 * i]) | ((uint32_t)f32_to_bf16_ref(v[2 * i + 1]) << 16);
+    return __builtin_bit_cast(bf16x8, u);
+}
+
+// Two transposing LDS reads: within 16 lanes, lane i names token row i / 4 and dims 4 (i % 4) of a block of 4 tokens x 16 dims
+// and receives the four tokens of dim i.  `second` lies where the lane's other four tokens start.
+__device__ inline bf16x8 transposed_pair(const unsigned char *first, const unsigned char *second) {
+    const s16x4 a = __builtin_amdgcn_ds_read_tr16_b64_v4i16(LDS_PTR(s16x4, first)), b = __builtin_amdgcn_ds_read_tr16_b64_v4i16(LDS_PTR(s16x4, second));
+    return __builtin_bit_cast(bf16x8, __builtin_shufflevector(a, b, 0, 1, 2, 3, 4, 5, 6, 7));
+}
+
+struct MfmaParams {
+    AttendParams a;
+    int RD, nsplit, max_len;
+    float *part; // [units][nsplit][32][R] outputs, behind them [units][nsplit][32][2] maxima and sums
+    size_t part_ml;
+};
+
+// BF16, absorbed form: 32 columns (neighbouring (token, head) pairs of one segment, which all read the same cache rows) a
+// workgroup, the context split over gridDim.z.  32 tokens at a time go through LDS: a wave scores 16 of them for 16 columns
+// (A = cached rows, B = the columns' queries in registers), the scores meet in LDS, every wave turns them into
+// probabilities and adds up its own quarter of the latent dimensions (A = the same rows read transposed).
+// DT: 16-dim tiles of a wave (R <= 64 DT); KSMAX: most 32-dim steps of a row.
+template <int DT, int KSMAX>
+__global__ __launch_bounds__(256, 2) void latent_mfma_kernel(MfmaParams p) {
+    extern __shared__ unsigned char lds[];
+    const StepView &v = p.a.v;
+    const int seg = blockIdx.y, n = v.seg_len[seg], H = p.a.H, R = p.a.cache.R, RD = p.RD;
+    const int c0 = blockIdx.x * 32, ncols = n * H;
+    if (n > p.max_len || c0 >= ncols) return;
+    const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), g = lane >> 4, i16 = lane & 15;
+    const int off = v.seg_off[seg], start = v.seg_pos[seg];
+    const int *table = v.table + (size_t)v.seg_row[seg] * v.table_stride;
+    const int last = c0 + 31 < ncols ? c0 + 31 : ncols - 1;
+    const int lo = start + c0 / H, hi = start + last / H; // positions of the first and the last column's token
+    const int first_vis = p.a.window > 0 && lo + 1 > p.a.window ? lo + 1 - p.a.window : 0;
+    const int b0 = first_vis >> 5, b1 = (hi >> 5) + 1;
+    const int per = (b1 - b0 + p.nsplit - 1) / p.nsplit;
+    const int bb = b0 + (int)blockIdx.z * per, be = bb + per < b1 ? bb + per : b1;
+    const int row_len = R + RD, ks_n = row_len / 32, row_chunks = row_len / 8, chunks = 32 * row_chunks;
+    const int pitch = row_len * 2 + 16;
+    float *sc = (float *)(lds + 2 * 32 * pitch); // [32 columns][36]
+
+    const int ct_s = wave >> 1, tt = wave & 1; // this wave's score tile
+    bf16x8 qf[KSMAX];
+    {
+        const int c = c0 + 16 * ct_s + i16;
+        const size_t at = (size_t)off * H + (c < ncols ? c : ncols - 1);
+        const uint16_t *qa = (const uint16_t *)p.a.qa + at * R + 8 * g;
+        const uint16_t *qr = (const uint16_t *)p.a.q + at * (p.a.D + RD) + p.a.D + 8 * g - R;
+#pragma unroll
+        for (int ks = 0; ks < KSMAX; ++ks)
+            if (ks < ks_n) qf[ks] = *(const bf16x8 *)((ks * 32 < R ? qa : qr) + ks * 32);
+    }
+    // this lane's column of either column tile: position, running maximum (log2 domain) and this lane's part of the sum
+    int cpos[2];
+    float m[2], l[2];
+    f32x4 o[DT][2];
+#pragma unroll
+    for (int ct = 0; ct < 2; ++ct) {
+        const int c = c0 + 16 * ct + i16;
+        cpos[ct] = c < ncols ? start + c / H : -1;
+        m[ct] = kUnseen, l[ct] = 0.0f;
+#pragma unroll
+        for (int d = 0; d < DT; ++d) o[d][ct] = f32x4 {0.f, 0.f, 0.f, 0.f};
+    }
+    const float scale2 = p.a.scale * kLog2e;
+
+    constexpr int PER = (KSMAX + 1) / 2;
+    u32x4 stage[PER];
+    auto fetch = [&](int blk, int page) {
+        const u32x4 *src = (const u32x4 *)((const uint16_t *)p.a.cache.pool + ((size_t)page * kPageTokens + (blk & 1) * 32) * row_len);
+#pragma unroll
+        for (int i = 0; i < PER; ++i) {
+            const int e = i * 256 + threadIdx.x;
+            if (e < chunks) stage[i] = src[e];
+        }
+    };
+    int lds_off[PER]; // chunk e of a block: 16 bytes of padding behind every row before it
+#pragma unroll
+    for (int i = 0; i < PER; ++i) {
+        const int e = i * 256 + threadIdx.x;
+        lds_off[i] = (e + e / row_chunks) * 16;
+    }
+    if (bb < be) fetch(bb, table[bb >> 1]);
+    int page = bb + 1 < be ? table[(bb + 1) >> 1] : 0;
+    int buf = 0;
+    for (int blk = bb; blk < be; ++blk, buf ^= 1) {
+        unsigned char *kv = lds + buf * 32 * pitch;
+#pragma unroll
+        for (int i = 0; i < PER; ++i)
+            if (i * 256 + (int)threadIdx.x < chunks) *(u32x4 *)(kv + lds_off[i]) = stage[i];
+        __syncthreads();
+        if (blk + 1 < be) fetch(blk + 1, page);
+        if (blk + 2 < be) page = table[(blk + 2) >> 1];
+        f32x4 s = {0.f, 0.f, 0.f, 0.f};
+        const unsigned char *krow = kv + (16 * tt + i16) * pitch + 16 * g;
+#pragma unroll
+        for (int ks = 0; ks < KSMAX; ++ks)
+            if (ks < ks_n) s = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*(const bf16x8 *)(krow + ks * 64), qf[ks], s, 0, 0, 0);
+        *(f32x4 *)(sc + (16 * ct_s + i16) * 36 + 16 * tt + 4 * g) = s;
+        __syncthreads();
+        bf16x8 pf[2];
+        float alpha[2];
+#pragma unroll
+        for (int ct = 0; ct < 2; ++ct) {
+            const float *row = sc + (16 * ct + i16) * 36 + 8 * g;
+            const f32x4 x0 = *(const f32x4 *)row, x1 = *(const f32x4 *)(row + 4);
+            float x[8], bm = kUnseen;
+#pragma unroll
+            for (int j = 0; j < 8; ++j) {
+                const int t = blk * 32 + 8 * g + j;
+                const bool seen = t <= cpos[ct] && (p.a.window <= 0 || t > cpos[ct] - p.a.window);
+                x[j] = seen ? (j < 4 ? x0[j & 3] : x1[j & 3]) * scale2 : kUnseen;
+                bm = fmaxf(bm, x[j]);
+            }
+            bm = fmaxf(bm, __shfl_xor(bm, 16, 64));
+            bm = fmaxf(bm, __shfl_xor(bm, 32, 64));
+            const float m_new = fmaxf(m[ct], bm);
+            alpha[ct] = __builtin_amdgcn_exp2f(m[ct] - m_new);
+            m[ct] = m_new;
+            float sum = 0.0f;
+#pragma unroll
+            for (int j = 0; j < 8; ++j) {
+                x[j] = x[j] > 0.5f * kUnseen ? __builtin_amdgcn_exp2f(x[j] - m_new) : 0.0f;
+                sum += x[j];
+            }
+            l[ct] = l[ct] * alpha[ct] + sum;
+            pf[ct] = pack_bf16x8(x);
+        }
+        if (__builtin_amdgcn_ballot_w64(alpha[0] != 1.0f || alpha[1] != 1.0f) != 0) {
+#pragma unroll
+            for (int d = 0; d < DT; ++d) o[d][0] *= alpha[0], o[d][1] *= alpha[1];
+        }
+        const unsigned char *vrow = kv + (8 * g + (i16 >> 2)) * pitch + 8 * (i16 & 3);
+#pragma unroll
+        for (int d = 0; d < DT; ++d) {
+            const int tile = wave * DT + d;
+            if (tile * 16 < R) {
+                const bf16x8 a = transposed_pair(vrow + tile * 32, vrow + tile * 32 + 4 * pitch);
+                o[d][0] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, pf[0], o[d][0], 0, 0, 0);
+                o[d][1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, pf[1], o[d][1], 0, 0, 0);
+            }
+        }
+    }
+#pragma unroll
+    for (int ct = 0; ct < 2; ++ct) {
+        l[ct] += __shfl_xor(l[ct], 16, 64);
+        l[ct] += __shfl_xor(l[ct], 32, 64);
+        const int c = c0 + 16 * ct + i16;
+        if (p.nsplit > 1) {
+            const size_t slot = (((size_t)seg * gridDim.x + blockIdx.x) * p.nsplit + blockIdx.z) * 32 + 16 * ct + i16;
+            if (wave == 0 && g == 0) *(float2 *)(p.part + p.part_ml + slot * 2) = make_float2(m[ct], l[ct]);
+            if (bb < be && c < ncols) {
+#pragma unroll
+                for (int d = 0; d < DT; ++d) {
+                    const int tile = wave * DT + d;
+                    if (tile * 16 < R) *(f32x4 *)(p.part + slot * R + tile * 16 + 4 * g) = o[d][ct];
+                }
+            }
+        } else if (c < ncols) {
+            float den = l[ct], mul = 1.0f;
+            if (p.a.sink) {
+                const float s2 = p.a.sink[c % H] * kLog2e, mt = fmaxf(m[ct], s2);
+                mul = __builtin_amdgcn_exp2f(m[ct] - mt);
+                den = den * mul + __builtin_amdgcn_exp2f(s2 - mt);
+            }
+            mul /= den;
+            uint16_t *dst = (uint16_t *)p.a.out + ((size_t)off * H + c) * R;
+#pragma unroll
+            for (int d = 0; d < DT; ++d) {
+                const int tile = wave * DT + d;
+                if (tile * 16 < R) {
+                    const f32x4 y = o[d][ct] * mul;
+                    *(uint2 *)(dst + tile * 16 + 4 * g) = make_uint2(f32_to_bf16_ref(y[0]) | ((uint32_t)f32_to_bf16_ref(y[1]) << 16),
+                            f32_to_bf16_ref(y[2]) | ((uint32_t)f32_to_bf16_ref(y[3]) << 16));
+                }
+            }
+        }
+    }
+}
+
+// sum of a column's splits; grid (column groups, segments, 32 columns)
+__global__ __launch_bounds__(128) void latent_merge_kernel(MfmaParams p) {
+    const StepView &v = p.a.v;
+    const int seg = blockIdx.y, n = v.seg_len[seg], H = p.a.H, R = p.a.cache.R;
+    const int c = blockIdx.x * 32 + blockIdx.z;
+    if (n > p.max_len || c >= n * H) return;
+    const size_t unit = ((size_t)seg * gridDim.x + blockIdx.x) * p.nsplit;
+    float mt = p.a.sink ? p.a.sink[c % H] * kLog2e : kUnseen;
+    const float s2 = mt;
+    for (int s = 0; s < p.nsplit; ++s) mt = fmaxf(mt, p.part[p.part_ml + ((unit + s) * 32 + blockIdx.z) * 2]);
+    float den = p.a.sink ? __builtin_amdgcn_exp2f(s2 - mt) : 0.0f;
+    for (int s = 0; s < p.nsplit; ++s) {
+        const float2 ml = *(const float2 *)(p.part + p.part_ml + ((unit + s) * 32 + blockIdx.z) * 2);
+        if (ml.x > 0.5f * kUnseen) den += ml.y * __builtin_amdgcn_exp2f(ml.x - mt);
+    }
+    const float inv = 1.0f / den;
+    uint16_t *dst = (uint16_t *)p.a.out + ((size_t)v.seg_off[seg] * H + c) * R;
+    for (int d = threadIdx.x * 4; d < R; d += 512) {
+        f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+        for (int s = 0; s < p.nsplit; ++s) {
+            const size_t slot = (unit + s) * 32 + blockIdx.z;
+            const float ms = p.part[p.part_ml + slot * 2];
+            if (ms > 0.5f * kUnseen) acc += *(const f32x4 *)(p.part + slot * R + d) * __builtin_amdgcn_exp2f(ms - mt);
+        }
+        acc *= inv;
+        *(uint2 *)(dst + d) = make_uint2(f32_to_bf16_ref(acc[0]) | ((uint32_t)f32_to_bf16_ref(acc[1]) << 16),
+                f32_to_bf16_ref(acc[2]) | ((uint32_t)f32_to_bf16_ref(acc[3]) << 16));
+    }
+}
+
+// cache rows of positions [base, base + rows) of a slot, side by side
+__global__ __launch_bounds__(256) void latent_gather_kernel(StepView v, int slot, int base, const uint16_t *pool, int row_len, uint16_t *out) {
+    const size_t src = cache_row(v, slot, base + blockIdx.x) * row_len;
+    for (int c = threadIdx.x * 8; c < row_len; c += 2048) *(u32x4 *)(out + (size_t)blockIdx.x * row_len + c) = *(const u32x4 *)(pool + src + c);
+}
+
+struct ExpandedParams {
+    const uint16_t *q, *k, *vv, *rows; // queries [T][H][D + RD]; keys [ctx][H D], values [ctx][H V]; cache rows [ctx][R + RD]
+    uint16_t *out; // [T][H V]
+    const float *sink;
+    int off, start, n, base, H, D, RD, V, R, window;
+    float scale;
+};
+
+// BF16, expanded form, for long segments: keys and values of every head made from the latents beforehand.  A workgroup takes
+// 128 query tokens of one head (32 a wave) and walks the visible context in blocks of 32 tokens, on 32 x 32 tiles:
+//   S^T = K Q^T (A = keys from LDS, B = the wave's queries in registers), O^T += V^T P^T (A = values from LDS read
+// transposed, B = probabilities straight from the score registers: half h of the wave holds tokens 8 q + 4 h + s of a block,
+// and the value operand takes its tokens in that order).
+// KSM: most 16-dim steps of a query; VTM: most 32-dim tiles of a value.  grid (heads, query blocks)
+template <int KSM, int VTM>
+__global__ __launch_bounds__(256, 2) void latent_expanded_kernel(ExpandedParams p) {
+    extern __shared__ unsigned char lds[];
+    const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), h = lane >> 5, cl = lane & 31;
+    const int head = blockIdx.x, q0 = ((int)gridDim.y - 1 - (int)blockIdx.y) * 128; // the blocks with the longest contexts first
+    const int Dq = p.D + p.RD, ks_n = Dq / 16, vt_n = p.V / 32;
+    const int kpitch = Dq * 2 + 16, vpitch = p.V * 2 + 16, bufb = 32 * (kpitch + vpitch);
+    const int qi = q0 + wave * 32 + cl;
+    const int pos = p.start + (qi < p.n ? qi : p.n - 1);
+    const int wlo = p.start + q0 + wave * 32, whi_q = q0 + wave * 32 + 31;
+    const int whi = p.start + (whi_q < p.n ? whi_q : p.n - 1); // last position of the wave's queries
+    const bool wave_on = q0 + wave * 32 < p.n;
+    bf16x8 qf[KSM];
+    {
+        const uint16_t *row = p.q + ((size_t)(p.off + (qi < p.n ? qi : p.n - 1)) * p.H + head) * Dq + 8 * h;
+#pragma unroll
+        for (int ks = 0; ks < KSM; ++ks)
+            if (ks < ks_n) qf[ks] = *(const bf16x8 *)(row + ks * 16);
+    }
+    f32x16 o[VTM];
+#pragma unroll
+    for (int d = 0; d < VTM; ++d)
+#pragma unroll
+        for (int r = 0; r < 16; ++r) o[d][r] = 0.0f;
+    float m = kUnseen, l = 0.0f;
+    const float scale2 = p.scale * kLog2e;
+    const int first = p.window > 0 && p.start + q0 + 1 > p.window ? p.start + q0 + 1 - p.window : 0;
+    const int last_q = q0 + 127 < p.n ? q0 + 127 : p.n - 1;
+    const int b0 = first >> 5, b1 = ((p.start + last_q) >> 5) + 1;
+    const int wfirst = p.window > 0 && wlo + 1 > p.window ? wlo + 1 - p.window : 0;
+
+    constexpr int PER = (16 * KSM + 32 * VTM + 63) / 64;
+    const int kd = p.D / 8, kr = p.RD / 8, kv8 = p.V / 8;
+    u32x4 stage[PER];
+    // chunk e of a block: 32 rows of unrotated keys, of rotated parts, of values
+    const uint16_t *src[PER];
+    size_t step[PER];
+    int dst[PER];
+#pragma unroll
+    for (int i = 0; i < PER; ++i) {
+        int e = i * 256 + threadIdx.x;
+        src[i] = nullptr, step[i] = 0, dst[i] = 0;
+        if (e < 32 * kd) {
+            const int r = e / kd, c = e % kd;
+            step[i] = (size_t)p.H * p.D, src[i] = p.k + r * step[i] + (size_t)head * p.D + c * 8, dst[i] = r * kpitch + c * 16;
+        } else if ((e -= 32 * kd) < 32 * kr) {
+            const int r = e / kr, c = e % kr;
+            step[i] = (size_t)(p.R + p.RD), src[i] = p.rows + r * step[i] + p.R + c * 8, dst[i] = r * kpitch + p.D * 2 + c * 16;
+        } else if ((e -= 32 * kr) < 32 * kv8) {
+            const int r = e / kv8, c = e % kv8;
+            step[i] = (size_t)p.H * p.V, src[i] = p.vv + r * step[i] + (size_t)head * p.V + c * 8, dst[i] = 32 * kpitch + r * vpitch + c * 16;
+        }
+    }
+    // (rows behind the segment's end lie inside the buffers, which hold whole blocks)
+    auto fetch = [&](int blk) {
+#pragma unroll
+        for (int i = 0; i < PER; ++i)
+            if (src[i]) stage[i] = *(const u32x4 *)(src[i] + (size_t)(blk * 32 - p.base) * step[i]);
+    };
+    fetch(b0);
+    int buf = 0;
+    for (int blk = b0; blk < b1; ++blk, buf ^= 1) {
+        unsigned char *kb = lds + buf * bufb, *vb = kb + 32 * kpitch;
+#pragma unroll
+        for (int i = 0; i < PER; ++i)
+            if (src[i]) *(u32x4 *)(kb + dst[i]) = stage[i];
+        __syncthreads();
+        if (blk + 1 < b1) fetch(blk + 1);
+        const int t0 = blk * 32;
+        if (!wave_on || t0 > whi || t0 + 31 < wfirst) continue; // (the same for the whole wave; the barriers above are all there are)
+        f32x16 s;
+#pragma unroll
+        for (int r = 0; r < 16; ++r) s[r] = 0.0f;
+        const unsigned char *krow = kb + cl * kpitch + 16 * h;
+#pragma unroll
+        for (int ks = 0; ks < KSM; ++ks)
+            if (ks < ks_n) s = __builtin_amdgcn_mfma_f32_32x32x16_bf16(*(const bf16x8 *)(krow + ks * 32), qf[ks], s, 0, 0, 0);
+        const bool masked = t0 + 31 > wlo || (p.window > 0 && t0 + p.window <= whi);
+        float bm = kUnseen;
+#pragma unroll
+        for (int r = 0; r < 16; ++r) s[r] *= scale2;
+        if (masked) {
+#pragma unroll
+            for (int r = 0; r < 16; ++r) {
+                const int t = t0 + 8 * (r >> 2) + 4 * h + (r & 3);
+                s[r] = t <= pos && (p.window <= 0 || t > pos - p.window) ? s[r] : kUnseen;
+            }
+        }
+#pragma unroll
+        for (int r = 0; r < 16; ++r) bm = fmaxf(bm, s[r]);
+        bm = fmaxf(bm, __shfl_xor(bm, 32, 64));
+        const float m_new = bm > m + 8.0f ? bm : m; // (the reference point moves only when it has to)
+        const float alpha = __builtin_amdgcn_exp2f(m - m_new);
+        m = m_new;
+        float sum = 0.0f;
+#pragma unroll
+        for (int r = 0; r < 16; ++r) s[r] = __builtin_amdgcn_exp2f(s[r] - m_new);
+        if (masked) {
+            // (a column that has seen no key yet has its reference point at the masked score)
+#pragma unroll
+            for (int r = 0; r < 16; ++r) {
+                const int t = t0 + 8 * (r >> 2) + 4 * h + (r & 3);
+                s[r] = t <= pos && (p.window <= 0 || t > pos - p.window) ? s[r] : 0.0f;
+            }
+        }
+#pragma unroll
+        for (int r = 0; r < 16; ++r) sum += s[r];
+        l = l * alpha + sum;
+        if (__builtin_amdgcn_ballot_w64(alpha != 1.0f) != 0) {
+#pragma unroll
+            for (int d = 0; d < VTM; ++d) o[d] *= alpha;
+        }
+#pragma unroll
+        for (int t = 0; t < 2; ++t) {
+            float pr[8];
+#pragma unroll
+            for (int j = 0; j < 8; ++j) pr[j] = s[8 * t + j];
+            const bf16x8 pf = pack_bf16x8(pr);
+            const unsigned char *vrow = vb + (16 * t + 4 * h + ((lane & 15) >> 2)) * vpitch + 32 * ((lane >> 4) & 1) + 8 * (lane & 3);
+#pragma unroll
+            for (int d = 0; d < VTM; ++d)
+                if (d < vt_n) o[d] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(transposed_pair(vrow + d * 64, vrow + d * 64 + 8 * vpitch), pf, o[d], 0, 0, 0);
+        }
+    }
+    l += __shfl_xor(l, 32, 64);
+    if (qi >= p.n) return;
+    float mul = 1.0f;
+    if (p.sink) {
+        const float s2 = p.sink[head] * kLog2e, mt = fmaxf(m, s2);
+        mul = __builtin_amdgcn_exp2f(m - mt);
+        l = l * mul + __builtin_amdgcn_exp2f(s2 - mt);
+    }
+    mul /= l;
+    uint16_t *out = p.out + (size_t)(p.off + qi) * p.H * p.V + (size_t)head * p.V;
+#pragma unroll
+    for (int d = 0; d < VTM; ++d)
+        if (d < vt_n) {
+#pragma unroll
+            for (int q = 0; q < 4; ++q)
+                *(uint2 *)(out + d * 32 + 8 * q + 4 * h) =
+                        make_uint2(f32_to_bf16_ref(o[d][4 * q] * mul) | ((uint32_t)f32_to_bf16_ref(o[d][4 * q + 1] * mul) << 16),
+                                f32_to_bf16_ref(o[d][4 * q + 2] * mul) | ((uint32_t)f32_to_bf16_ref(o[d][4 * q + 3] * mul) << 16));
+        }
+}
+
+template <int DT, int KSMAX>
+int launch_mfma(const MfmaParams &p, dim3 grid, size_t smem, hipStream_t st) {
+    static const hipError_t attr = hipFuncSetAttribute((const void *)latent_mfma_kernel<DT, KSMAX>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
+    XFT_CHECK_HIP(attr);
+    hipLaunchKernelGGL((latent_mfma_kernel<DT, KSMAX>), grid, dim3(256), smem, st, p);
+    XFT_CHECK_HIP(hipGetLastError());
+    return 0;
+}
+template <int KSM, int VTM>
+int launch_expanded(const ExpandedParams &p, dim3 grid, size_t smem, hipStream_t st) {
+    static const hipError_t attr = hipFuncSetAttribute((const void *)latent_expanded_kernel<KSM, VTM>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
+    XFT_CHECK_HIP(attr);
+    hipLaunchKernelGGL((latent_expanded_kernel<KSM, VTM>), grid, dim3(256), smem, st, p);
+    XFT_CHECK_HIP(hipGetLastError());
+    return 0;
+}
+
+// does the matrix-unit form of the absorbed attention take this layer
+bool mfma_takes(const PlanLayer &L) {
+    const int ks = (L.R + L.RD) / 32;
+    return (L.R <= 64 && ks <= 6) || (L.R <= 128 && ks <= 8) || (L.R <= 256 && ks <= 12) || (L.R <= 512 && ks <= 20);
+}
+
 } // namespace
 
 int latent_prepare(int act, const PlanLayer &L, const StepView &v, const void *a, void *cq, const LatentCacheView &cache, float eps, hipStream_t st) {
@@ -185,20 +598,75 @@ int latent_rotate_q(int act, const PlanLayer &L, const StepView &v, void *q, hip
     return 0;
 }
 
-int latent_split_count(const PlanLayer &, int, int, int) { return 1; }
+// Parts a context of `hint` tokens is split into: as many as give every compute unit a workgroup, blocks of 32 tokens permitting.
+int latent_split_count(const PlanLayer &L, int B, int longest, int hint) {
+    if (!mfma_takes(L)) return 1;
+    const long units = (long)B * ((longest * L.s.heads + 31) / 32);
+    const int ctx = L.s.window > 0 && L.s.window + longest < hint ? L.s.window + longest : hint;
+    const int blocks = (ctx + 31) / 32;
+    const long want = device_cu_count() / units;
+    return (int)(want < 1 ? 1 : (want < blocks ? want : (blocks < 1 ? 1 : blocks)));
+}
 
-int latent_attention(int act, const PlanLayer &L, const StepView &v, const void *qa, const void *q, void *out, const LatentCacheView &cache, int hint,
-        float *part, size_t part_floats, hipStream_t st) {
-    (void)hint, (void)part, (void)part_floats;
-    const AttendParams p = {v, qa, q, out, cache, L.sink, L.s.heads, L.D, L.s.window, L.s.scale};
+size_t latent_part_floats(const PlanLayer &L) { return mfma_takes(L) ? (size_t)device_cu_count() * 32 * (L.R + 2) : 0; }
+
+int latent_attention(int act, const PlanLayer &L, const StepView &v, int longest, const void *qa, const void *q, void *out, const LatentCacheView &cache,
+        int hint, float *part, size_t part_floats, hipStream_t st) {
+    const AttendParams a = {v, qa, q, out, cache, L.sink, L.s.heads, L.D, L.s.window, longest, L.s.scale};
+    if (act == XFTHIP_BF16 && mfma_takes(L)) {
+        MfmaParams p = {a, L.RD, latent_split_count(L, v.B, longest, hint), longest, part, 0};
+        const unsigned groups = (unsigned)((longest * L.s.heads + 31) / 32);
+        const size_t slots = (size_t)v.B * groups * p.nsplit * 32;
+        p.part_ml = slots * L.R;
+        XFT_REQUIRE(p.nsplit == 1 || slots * (L.R + 2) <= part_floats, "latent_attention: workspace too small for %zu partial columns", slots);
+        const dim3 grid(groups, v.B, p.nsplit);
+        const size_t smem = (size_t)2 * 32 * ((L.R + L.RD) * 2 + 16) + 32 * 36 * 4;
+        const int ks = (L.R + L.RD) / 32;
+        int rc;
+        if (L.R <= 64 && ks <= 6) rc = launch_mfma<1, 6>(p, grid, smem, st);
+        else if (L.R <= 128 && ks <= 8) rc = launch_mfma<2, 8>(p, grid, smem, st);
+        else if (L.R <= 256 && ks <= 12) rc = launch_mfma<4, 12>(p, grid, smem, st);
+        else if (ks <= 18) rc = launch_mfma<8, 18>(p, grid, smem, st);
+        else rc = launch_mfma<8, 20>(p, grid, smem, st);
+        if (rc || p.nsplit == 1) return rc;
+        hipLaunchKernelGGL(latent_merge_kernel, dim3(groups, v.B, 32), dim3(128), 0, st, p);
+        XFT_CHECK_HIP(hipGetLastError());
+        return 0;
+    }
     const size_t smem = (size_t)(2 * L.R + L.RD + 256 + 8) * 4 + 256 * 8;
     XFT_REQUIRE(smem <= 64 * 1024, "latent_attention: latent of %d values too wide", L.R);
     if (act == XFTHIP_BF16)
-        hipLaunchKernelGGL(latent_attend_kernel<true>, dim3(v.T, L.s.heads), dim3(256), smem, st, p);
+        hipLaunchKernelGGL(latent_attend_kernel<true>, dim3(v.T, L.s.heads), dim3(256), smem, st, a);
     else
-        hipLaunchKernelGGL(latent_attend_kernel<false>, dim3(v.T, L.s.heads), dim3(256), smem, st, p);
+        hipLaunchKernelGGL(latent_attend_kernel<false>, dim3(v.T, L.s.heads), dim3(256), smem, st, a);
     XFT_CHECK_HIP(hipGetLastError());
     return 0;
+}
+
+bool latent_expanded_takes(int act, const PlanLayer &L, int n, int ctx) {
+    if (act != XFTHIP_BF16 || n < 32) return false;
+    const int ks = (L.D + L.RD) / 16, vt = L.V / 32;
+    if (!((ks <= 4 && vt <= 2) || (ks <= 8 && vt <= 4) || (ks <= 12 && vt <= 4))) return false;
+    // what the narrower products save against making keys and values of the context that came before
+    return (double)n * ctx * (2.0 * L.R - L.D - L.V) >= (double)(ctx - n) * L.R * (L.D + L.V);
+}
+
+int latent_gather(const StepView &v, int slot, int base, int rows, const LatentCacheView &cache, void *out, hipStream_t st) {
+    hipLaunchKernelGGL(latent_gather_kernel, dim3(rows), dim3(256), 0, st, v, slot, base, (const uint16_t *)cache.pool, cache.R + cache.RD, (uint16_t *)out);
+    XFT_CHECK_HIP(hipGetLastError());
+    return 0;
+}
+
+int latent_expanded(const PlanLayer &L, int off, int start, int n, int base, const void *q, const void *k, const void *values, const void *rows, void *out,
+        hipStream_t st) {
+    const ExpandedParams p = {(const uint16_t *)q, (const uint16_t *)k, (const uint16_t *)values, (const uint16_t *)rows, (uint16_t *)out, L.sink, off, start, n,
+            base, L.s.heads, L.D, L.RD, L.V, L.R, L.s.window, L.s.scale};
+    const dim3 grid(L.s.heads, (n + 127) / 128);
+    const size_t smem = (size_t)2 * 32 * ((L.D + L.RD) * 2 + 16 + L.V * 2 + 16);
+    const int ks = (L.D + L.RD) / 16, vt = L.V / 32;
+    if (ks <= 4 && vt <= 2) return launch_expanded<4, 2>(p, grid, smem, st);
+    if (ks <= 8 && vt <= 4) return launch_expanded<8, 4>(p, grid, smem, st);
+    return launch_expanded<12, 4>(p, grid, smem, st);
 }
 
 } // namespace xfthip

@@ -844,14 +844,7 @@ int xfthip_model_step(xfthip_model_t m, int n, const int *rows_host, const int *
     m->cur_B = 0;
     for (int r = 0; r < c.max_batch; ++r)
         if (m->row_pos[r] >= 0) m->cur_B = r + 1;
-    const int chunk = m->plan->logit_rows;
-    for (int i = 0; i < n_want; i += chunk) {
-        const int k = n_want - i < chunk ? n_want - i : chunk;
-        XFT_CHECK_HIP(hipMemcpyAsync(m->plan->want, want_host + i, (size_t)k * 4, hipMemcpyHostToDevice, st));
-        if (int rc = plan_head(m, m->plan->want, k, 0, st)) return rc;
-        XFT_CHECK_HIP(hipMemcpyAsync(logits_host + (size_t)i * c.vocab, m->logits, (size_t)k * c.vocab * 4, hipMemcpyDeviceToHost, st));
-        XFT_CHECK_HIP(hipStreamSynchronize(st));
-    }
+    if (int rc = plan_logits(m, want_host, n_want, logits_host, st)) return rc;
     XFT_CHECK_HIP(hipStreamSynchronize(st));
     return 0;
 }
@@ -1159,17 +1152,9 @@ int xfthip_model_prompt_logits(xfthip_model_t m, int first_row, int rows, float 
     const xfthip_model_config &c = m->cfg;
     hipStream_t st = (hipStream_t)stream;
     if (m->plan) {
-        const int chunk = m->plan->logit_rows;
-        for (int r = 0; r < rows; r += chunk) {
-            const int n = rows - r < chunk ? rows - r : chunk;
-            std::vector<int> list(n);
-            for (int i = 0; i < n; ++i) list[i] = first_row + r + i;
-            XFT_CHECK_HIP(hipMemcpyAsync(m->plan->want, list.data(), (size_t)n * 4, hipMemcpyHostToDevice, st));
-            if (int rc = plan_head(m, m->plan->want, n, 0, st)) return rc;
-            XFT_CHECK_HIP(hipMemcpyAsync(logits_host + (size_t)r * c.vocab, m->logits, (size_t)n * c.vocab * 4, hipMemcpyDeviceToHost, st));
-            XFT_CHECK_HIP(hipStreamSynchronize(st));
-        }
-        return 0;
+        std::vector<int> list(rows);
+        for (int i = 0; i < rows; ++i) list[i] = first_row + i;
+        return plan_logits(m, list.data(), rows, logits_host, st);
     }
     // final norm + lm_head over the prompt's residual rows, a chunk at a time through a buffer that lives for the
     // call (not a hot path: the reference's logitsAll = true serves scoring, not generation)

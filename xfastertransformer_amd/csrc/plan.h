@@ -78,11 +78,21 @@ struct LatentCacheView {
 int latent_prepare(int act, const PlanLayer &L, const StepView &v, const void *a, void *cq, const LatentCacheView &cache, float eps, hipStream_t st);
 // rotates the rotated parts of q [T][heads][D + RD] in place
 int latent_rotate_q(int act, const PlanLayer &L, const StepView &v, void *q, hipStream_t st);
-// absorbed form: qa [T][heads][R] queries in the latent space, q their rotated parts; out [T][heads][R] weighted latents.
-// part: workspace of attn_part_floats floats (split contexts).  hint: upper bound of the sequence lengths
-int latent_attention(int act, const PlanLayer &L, const StepView &v, const void *qa, const void *q, void *out, const LatentCacheView &cache,
+// absorbed form: qa [T][heads][R] queries in the latent space, q their rotated parts; out [T][heads][R] weighted latents;
+// segments of up to `longest` tokens.  part: workspace of part_floats floats (split contexts).  hint: upper bound of the
+// sequence lengths
+int latent_attention(int act, const PlanLayer &L, const StepView &v, int longest, const void *qa, const void *q, void *out, const LatentCacheView &cache,
         int hint, float *part, size_t part_floats, hipStream_t st);
 int latent_split_count(const PlanLayer &L, int B, int longest, int hint);
+size_t latent_part_floats(const PlanLayer &L);
+// expanded form: should a segment of n tokens that ends at position ctx take it
+bool latent_expanded_takes(int act, const PlanLayer &L, int n, int ctx);
+// cache rows of positions base .. base + rows - 1 of a slot -> out [rows][R + RD]
+int latent_gather(const StepView &v, int slot, int base, int rows, const LatentCacheView &cache, void *out, hipStream_t st);
+// one segment: tokens off .. off + n - 1 of the step at positions start .., q [T][heads][D + RD]; keys [ctx][heads D], values
+// [ctx][heads V] and gathered cache rows of the positions from base (a multiple of 32) on, whole blocks of 32; out [T][heads V]
+int latent_expanded(const PlanLayer &L, int off, int start, int n, int base, const void *q, const void *k, const void *values, const void *rows, void *out,
+        hipStream_t st);
 
 struct DeltaBuffers {
     void *in; // [T][row_in] of the activation type: q | k | v | beta | decay rank | gate rank
@@ -138,13 +148,18 @@ struct PlanState {
     bool table_dirty = true;
     // step description on the device, its host image (pinned) and the views into it
     int *desc = nullptr, *desc_host = nullptr;
+    // pinned images of what else a step copies: the rows whose logits are wanted, a decode call's slots, the page table, logits
+    int *want_host = nullptr, *dec_host = nullptr, *table_pinned = nullptr;
+    float *logits_pinned = nullptr;
     int *tok_seg = nullptr, *tok_pos = nullptr, *ids = nullptr, *seg = nullptr, *dec_rows = nullptr, *want = nullptr;
+    std::vector<int> seg_off_host, seg_len_host, seg_pos_host, seg_row_host; // the step's segments
     std::vector<int> dec_list; // slots of the decode call in flight
     std::vector<int> logit_of_row; // which row of the logits a slot's last ones are in
     int logit_rows = 0;
     // scratch (activation type unless float)
     void *xn = nullptr, *a = nullptr, *cq = nullptr, *q = nullptr, *qa = nullptr, *oc = nullptr, *ov = nullptr, *h = nullptr, *on = nullptr;
     float *y = nullptr, *gates = nullptr, *dq = nullptr, *dk = nullptr, *dqk = nullptr, *dg = nullptr, *dv = nullptr, *dbeta = nullptr, *do_ = nullptr;
+    void *rows = nullptr, *kx = nullptr, *vx = nullptr; // gathered latents, keys and values of a long segment's context
     float *part = nullptr; // split contexts
     size_t part_floats = 0;
     std::vector<float *> tables; // rotation tables
@@ -162,6 +177,8 @@ void plan_release(xfthip_model *m, int row);
 int plan_run(xfthip_model *m, int n, const int *rows, const int *lens, const int *ids, hipStream_t st);
 // final norm and head of the residual rows rows_dev[0 .. n) (null: rows 0 .. n - 1) into m->logits + at * vocab
 int plan_head(xfthip_model *m, const int *rows_dev, int n, int at, hipStream_t st);
+// final norm and head of the residual rows list[0 .. n) (host), logits to host memory, as many rows at a time as fit
+int plan_logits(xfthip_model *m, const int *list, int n, float *logits_host, hipStream_t st);
 // upload of what a decode call of the slots in dec_list needs, for `steps` steps
 int plan_decode_begin(xfthip_model *m, int steps, hipStream_t st);
 // one decode step of the slots in dec_rows (recordable): positions and input ids from m->pos / m->ids

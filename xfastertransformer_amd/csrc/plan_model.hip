@@ -97,9 +97,44 @@ int run_latent(xfthip_model *m, const PlanLayer &L, int run, const StepView &v, 
     if ((rc = latent_prepare(act, L, v, p.a, p.cq, p.cache[run], m->cfg.rms_eps, st))) return rc;
     if ((rc = plan_gemm(m, L.uq, T, p.cq, L.QR, p.q, qcols, act, st))) return rc;
     if ((rc = latent_rotate_q(act, L, v, p.q, st))) return rc;
-    if ((rc = tile_gemm(L.absorb, act, T, p.q, qcols, L.R, L.D + L.RD, p.qa, H * L.R, act, 0, 0, 0, st))) return rc;
-    if ((rc = latent_attention(act, L, v, p.qa, p.q, p.oc, p.cache[run], m->len_hint, p.part, p.part_floats, st))) return rc;
-    if ((rc = tile_gemm(L.uv, act, T, p.oc, H * L.R, L.V, L.R, p.ov, H * L.V, act, 0, 0, 0, st))) return rc;
+    // long segments one by one in the expanded form; the others, as far as they are neighbours, together in the absorbed one
+    const size_t B = p.seg_len_host.size();
+    const char *q = (const char *)p.q;
+    int longest = 0, short_from = -1;
+    auto absorb = [&](int from, int to) {
+        return tile_gemm(L.absorb, act, to - from, q + (size_t)from * qcols * p.esz, qcols, L.R, L.D + L.RD, (char *)p.qa + (size_t)from * H * L.R * p.esz, H * L.R,
+                act, 0, 0, 0, st);
+    };
+    auto to_values = [&](int from, int to) {
+        return tile_gemm(L.uv, act, to - from, (char *)p.oc + (size_t)from * H * L.R * p.esz, H * L.R, L.V, L.R, (char *)p.ov + (size_t)from * H * L.V * p.esz,
+                H * L.V, act, 0, 0, 0, st);
+    };
+    std::vector<std::pair<int, int>> spans; // token ranges of the absorbed form
+    for (size_t i = 0; i < B; ++i) {
+        const int n = p.seg_len_host[i], off = p.seg_off_host[i], start = p.seg_pos_host[i];
+        const int from = L.s.window > 0 && start + 1 > L.s.window ? (start + 1 - L.s.window) & ~31 : 0, rows = start + n - from;
+        const bool expand = p.kx != nullptr && latent_expanded_takes(act, L, n, rows);
+        if (!expand) {
+            longest = std::max(longest, n);
+            if (short_from < 0) short_from = off;
+        }
+        if (short_from >= 0 && (expand || i + 1 == B)) {
+            spans.push_back({short_from, expand ? off : off + n});
+            short_from = -1;
+        }
+        if (!expand) continue;
+        if ((rc = latent_gather(v, p.seg_row_host[i], from, rows, p.cache[run], p.rows, st))) return rc;
+        if ((rc = xfthip_gemm(L.uk, rows, p.rows, L.R + L.RD, p.kx, H * L.D, XFTHIP_BF16, XFTHIP_EPI_NONE, nullptr, nullptr, 0, XFTHIP_F32, 1.0f, st))) return rc;
+        if ((rc = xfthip_gemm(L.uv, rows, p.rows, L.R + L.RD, p.vx, H * L.V, XFTHIP_BF16, XFTHIP_EPI_NONE, nullptr, nullptr, 0, XFTHIP_F32, 1.0f, st))) return rc;
+        if ((rc = latent_expanded(L, off, start, n, from, p.q, p.kx, p.vx, p.rows, p.ov, st))) return rc;
+    }
+    if (!spans.empty()) {
+        for (auto &s : spans)
+            if ((rc = absorb(s.first, s.second))) return rc;
+        if ((rc = latent_attention(act, L, v, longest, p.qa, p.q, p.oc, p.cache[run], m->len_hint, p.part, p.part_floats, st))) return rc;
+        for (auto &s : spans)
+            if ((rc = to_values(s.first, s.second))) return rc;
+    }
     return plan_gemm(m, L.o, T, p.ov, H * L.V, p.y, hidden, XFTHIP_F32, st);
 }
 
@@ -159,8 +194,8 @@ int plan_layers(xfthip_model *m, const StepView &v, hipStream_t st) {
 
 int upload_table(PlanState &p, hipStream_t st) {
     if (!p.table_dirty) return 0;
-    XFT_CHECK_HIP(hipMemcpyAsync(p.table, p.table_host.data(), p.table_host.size() * 4, hipMemcpyHostToDevice, st));
-    XFT_CHECK_HIP(hipStreamSynchronize(st));
+    memcpy(p.table_pinned, p.table_host.data(), p.table_host.size() * 4);
+    XFT_CHECK_HIP(hipMemcpyAsync(p.table, p.table_pinned, p.table_host.size() * 4, hipMemcpyHostToDevice, st));
     p.table_dirty = false;
     return 0;
 }
@@ -218,8 +253,10 @@ int plan_run(xfthip_model *m, int n, const int *rows, const int *lens, const int
     const int cap = p.slots, mt = c.max_tokens;
     int *hs = p.desc_host, *hp = hs + mt, *hi = hp + mt, *hg = hi + mt;
     int t = 0;
+    p.seg_off_host.resize(n), p.seg_len_host.assign(lens, lens + n), p.seg_pos_host.resize(n), p.seg_row_host.assign(rows, rows + n);
     for (int i = 0; i < n; ++i) {
         const int at = std::max(m->row_pos[rows[i]], 0);
+        p.seg_off_host[i] = t, p.seg_pos_host[i] = at;
         hg[i] = rows[i], hg[cap + i] = t, hg[2 * cap + i] = lens[i], hg[3 * cap + i] = at;
         for (int k = 0; k < lens[i]; ++k, ++t) hs[t] = i, hp[t] = at + k, hi[t] = ids[t];
     }
@@ -256,20 +293,37 @@ int plan_head(xfthip_model *m, const int *rows_dev, int n, int at, hipStream_t s
     return plan_gemm(m, plan.head, n, p.xn, c.hidden, m->logits + (size_t)at * c.vocab, c.vocab, XFTHIP_F32, st);
 }
 
+int plan_logits(xfthip_model *m, const int *list, int n, float *logits_host, hipStream_t st) {
+    PlanState &p = *m->plan;
+    const size_t vocab = m->cfg.vocab;
+    for (int i = 0; i < n; i += p.logit_rows) {
+        const int k = std::min(n - i, p.logit_rows);
+        memcpy(p.want_host, list + i, (size_t)k * 4);
+        XFT_CHECK_HIP(hipMemcpyAsync(p.want, p.want_host, (size_t)k * 4, hipMemcpyHostToDevice, st));
+        if (int rc = plan_head(m, p.want, k, 0, st)) return rc;
+        XFT_CHECK_HIP(hipMemcpyAsync(p.logits_pinned, m->logits, (size_t)k * vocab * 4, hipMemcpyDeviceToHost, st));
+        XFT_CHECK_HIP(hipStreamSynchronize(st));
+        memcpy(logits_host + (size_t)i * vocab, p.logits_pinned, (size_t)k * vocab * 4);
+    }
+    return 0;
+}
+
 int plan_prompt_pass(xfthip_model *m, const int *rows, int B, int S, const int *ids, float *logits_host, hipStream_t st) {
     PlanState &p = *m->plan;
     const xfthip_model_config &c = m->cfg;
-    std::vector<int> lens(B, S), last(B);
+    std::vector<int> lens(B, S);
     if (int rc = plan_run(m, B, rows, lens.data(), ids, st)) return rc;
-    for (int b = 0; b < B; ++b) last[b] = (b + 1) * S - 1;
-    XFT_CHECK_HIP(hipMemcpyAsync(p.want, last.data(), (size_t)B * 4, hipMemcpyHostToDevice, st));
+    for (int b = 0; b < B; ++b) p.want_host[b] = (b + 1) * S - 1;
+    XFT_CHECK_HIP(hipMemcpyAsync(p.want, p.want_host, (size_t)B * 4, hipMemcpyHostToDevice, st));
     // (the prompts of one call sit in neighbouring slots)
     if (int rc = plan_head(m, p.want, B, rows[0], st)) return rc;
     if (int rc = argmax_rows(m->logits + (size_t)rows[0] * c.vocab, B, c.vocab, m->ids, p.seg, nullptr, nullptr, st)) return rc;
     hipLaunchKernelGGL(plan_fill_kernel, dim3(1), dim3(64), 0, st, m->step, 1, 0);
     XFT_CHECK_HIP(hipGetLastError());
+    if (logits_host)
+        XFT_CHECK_HIP(hipMemcpyAsync(p.logits_pinned, m->logits + (size_t)rows[0] * c.vocab, (size_t)B * c.vocab * 4, hipMemcpyDeviceToHost, st));
     XFT_CHECK_HIP(hipStreamSynchronize(st));
-    if (logits_host) XFT_CHECK_HIP(hipMemcpy(logits_host, m->logits + (size_t)rows[0] * c.vocab, (size_t)B * c.vocab * 4, hipMemcpyDeviceToHost));
+    if (logits_host) memcpy(logits_host, p.logits_pinned, (size_t)B * c.vocab * 4);
     for (int b = 0; b < B; ++b) p.logit_of_row[rows[b]] = rows[0] + b;
     return 0;
 }
@@ -279,8 +333,8 @@ int plan_decode_begin(xfthip_model *m, int steps, hipStream_t st) {
     for (int r : p.dec_list)
         if (int rc = plan_reserve(m, r, m->row_pos[r] + steps)) return rc;
     if (int rc = upload_table(p, st)) return rc;
-    XFT_CHECK_HIP(hipMemcpyAsync(p.dec_rows, p.dec_list.data(), p.dec_list.size() * 4, hipMemcpyHostToDevice, st));
-    XFT_CHECK_HIP(hipStreamSynchronize(st));
+    memcpy(p.dec_host, p.dec_list.data(), p.dec_list.size() * 4);
+    XFT_CHECK_HIP(hipMemcpyAsync(p.dec_rows, p.dec_host, p.dec_list.size() * 4, hipMemcpyHostToDevice, st));
     for (size_t b = 0; b < p.dec_list.size(); ++b) p.logit_of_row[p.dec_list[b]] = (int)b;
     return 0;
 }
@@ -293,6 +347,9 @@ int plan_decode_step(xfthip_model *m, int B, hipStream_t st) {
     XFT_CHECK_HIP(hipGetLastError());
     const bool trace = p.trace;
     p.trace = false;
+    // (lengths and offsets only: where the segments stand is known on the device)
+    p.seg_off_host.resize(B), p.seg_len_host.assign(B, 1), p.seg_pos_host.assign(B, 0), p.seg_row_host.assign(B, 0);
+    for (int b = 0; b < B; ++b) p.seg_off_host[b] = b;
     int rc = plan_layers(m, view_of(m, B, B, 1), st);
     p.trace = trace;
     if (rc) return rc;
@@ -378,6 +435,7 @@ void plan_state_destroy(PlanState *p) {
     for (void *b : p->owned) (void)hipFree(b);
     if (p->trace_buf) (void)hipFree(p->trace_buf);
     if (p->desc_host) (void)hipHostFree(p->desc_host);
+    if (p->logits_pinned) (void)hipHostFree(p->logits_pinned);
     delete p;
 }
 
@@ -697,6 +755,17 @@ int xfthip_model_create_from_plan(xfthip_plan_t plan, int act_dtype, int max_bat
     alloc(&p->ov, T * ov * e), alloc(&p->h, T * h * e), alloc(&p->on, T * on * e);
     alloc(&p->gates, T * gates * 4), alloc(&p->dq, T * dk * 4), alloc(&p->dk, T * dk * 4), alloc(&p->dqk, T * dqk * 4), alloc(&p->dg, T * dg * 4);
     alloc(&p->dv, T * dv * 4), alloc(&p->dbeta, T * heads * 4), alloc(&p->do_, T * dv * 4);
+    // the expanded form's context (whole blocks of 32 tokens; cleared: rows behind the end meet zero weights)
+    if (act_dtype == XFTHIP_BF16 && max_tokens >= 32) {
+        const size_t ctx = pad32(max_seq) + 32;
+        size_t kx = 0, vx = 0, rl = 0;
+        for (const PlanLayer &L : p->layers)
+            if (L.s.mixer == XFTHIP_MIXER_LATENT && latent_expanded_takes(act_dtype, L, 1 << 20, 1 << 20))
+                kx = std::max(kx, (size_t)L.s.heads * L.D), vx = std::max(vx, (size_t)L.s.heads * L.V), rl = std::max(rl, (size_t)(L.R + L.RD));
+        if (kx) alloc(&p->rows, ctx * rl * e, true), alloc(&p->kx, ctx * kx * e, true), alloc(&p->vx, ctx * vx * e, true);
+    }
+    for (const PlanLayer &L : p->layers) p->part_floats = std::max(p->part_floats, L.s.mixer == XFTHIP_MIXER_LATENT ? latent_part_floats(L) : 0);
+    alloc(&p->part, p->part_floats * 4);
     for (const LayerRun &r : plan->runs) {
         const PlanLayer &L = p->layers[r.layer];
         LatentCacheView cv = {nullptr, L.R, L.RD};
@@ -726,7 +795,11 @@ int xfthip_model_create_from_plan(xfthip_plan_t plan, int act_dtype, int max_bat
         }
         L.cosT = t.first, L.sinT = t.second;
     }
-    ok = ok && hipHostMalloc((void **)&p->desc_host, (3 * T + 4 * (size_t)max_batch) * 4) == hipSuccess;
+    ok = ok && hipHostMalloc((void **)&p->desc_host, (3 * T + 5 * (size_t)max_batch + p->logit_rows + p->table_host.size()) * 4) == hipSuccess
+            && hipHostMalloc((void **)&p->logits_pinned, (size_t)p->logit_rows * plan->cfg.vocab * 4) == hipSuccess;
+    p->dec_host = p->desc_host + 3 * T + 4 * (size_t)max_batch;
+    p->want_host = p->dec_host + max_batch;
+    p->table_pinned = p->want_host + p->logit_rows;
     p->tok_seg = p->desc, p->tok_pos = p->desc + T, p->ids = p->desc + 2 * T, p->seg = p->desc + 3 * T;
     const size_t nids = T > 64 ? T : 64;
     m->idlog_cap = max_seq + 1;

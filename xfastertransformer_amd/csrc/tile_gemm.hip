@@ -56,7 +56,6 @@ __global__ __launch_bounds__(256) void tile_gemm_kernel(TileGemm p) {
 #pragma unroll
         for (int m = 0; m < MT; ++m) acc[t][m] = f32x4 {0.f, 0.f, 0.f, 0.f};
 
-#pragma unroll 2
     for (int kt = 0; kt < p.ktiles; ++kt) {
         u32x4 wq[2];
 #pragma unroll
