@@ -13,6 +13,41 @@ __device__ inline float wave_total(float v) {
     return v;
 }
 
+template <bool BF16>
+__device__ inline float ldb(const void *p, size_t i) {
+    if constexpr (BF16) return bf16_to_f32(((const uint16_t *)p)[i]);
+    else return ((const float *)p)[i];
+}
+
+// exp, x / (1 + exp(-x)), 1 / (1 + exp(-x)) and log(1 + exp(x)): the library functions with 32-bit activations; with bf16
+// ones the hardware's exp2 / log2 / reciprocal, each good to a few units in the last place (log(1 + y) through
+// y log(u) / (u - 1), u = 1 + y rounded, which keeps small y exact)
+template <bool FAST>
+__device__ inline float exp_of(float x) {
+    if constexpr (FAST) return fast_exp(x);
+    else return expf(x);
+}
+template <bool FAST>
+__device__ inline float sigmoid_of(float x) {
+    if constexpr (FAST) return __builtin_amdgcn_rcpf(1.0f + fast_exp(-x));
+    else return 1.0f / (1.0f + expf(-x));
+}
+template <bool FAST>
+__device__ inline float silu_of(float x) {
+    if constexpr (FAST) return x * __builtin_amdgcn_rcpf(1.0f + fast_exp(-x));
+    else return x / (1.0f + expf(-x));
+}
+template <bool FAST>
+__device__ inline float softplus_of(float x) {
+    if (x > 20.0f) return x;
+    if constexpr (FAST) {
+        const float y = fast_exp(x), u = 1.0f + y, d = u - 1.0f;
+        return d > 0.0f ? y * (__logf(u) * __builtin_amdgcn_rcpf(d)) : y;
+    } else {
+        return log1pf(expf(x));
+    }
+}
+
 struct PrepParams {
     StepView v;
     DeltaBuffers b;
@@ -84,6 +119,140 @@ __global__ __launch_bounds__(256) void delta_prepare_kernel(PrepParams p) {
         p.b.g[((size_t)t * p.H + head) * p.KD + c] = expf(-a * sp);
     }
     if (lane == 0) p.b.beta[(size_t)t * p.H + head] = 1.0f / (1.0f + expf(-load_as_f32(p.b.in, DT, (size_t)t * p.ld + p.beta_col + head)));
+}
+
+// The same for the usual shapes (TAPS taps, head widths of at most 256): a wave walks TT consecutive tokens of one segment and
+// head, two neighbouring channels a lane, the convolutions' last inputs in registers - every input is read once and every
+// result leaves as a pair.  grid (token tiles of a segment, ceil(heads / 4), segments)
+constexpr int kPrepTokens = 8;
+
+template <bool BF16>
+__device__ inline float2 load2(const void *p, size_t i) {
+    if constexpr (BF16) {
+        const uint32_t u = *(const uint32_t *)((const uint16_t *)p + i);
+        return make_float2(u2f(u << 16), u2f(u & 0xFFFF0000u));
+    } else {
+        return *(const float2 *)((const float *)p + i);
+    }
+}
+template <bool BF16>
+__device__ inline void store2(void *p, size_t i, float2 v) {
+    if constexpr (BF16) *(uint32_t *)((uint16_t *)p + i) = f32_bits_to_bf16_sel(f2u(v.x)) | (f32_bits_to_bf16_sel(f2u(v.y)) << 16);
+    else *(float2 *)((float *)p + i) = v;
+}
+
+template <bool BF16, int TAPS, int J> // J: turns of 128 channels that cover a head's width
+__global__ __launch_bounds__(256) void delta_prepare_tiled_kernel(PrepParams p) {
+    const int lane = threadIdx.x & 63, head = blockIdx.y * 4 + (threadIdx.x >> 6), seg = blockIdx.z;
+    const int n = p.v.seg_len[seg], i0 = blockIdx.x * kPrepTokens;
+    if (head >= p.H || i0 >= n) return;
+    const int off = p.v.seg_off[seg], row = p.v.seg_row[seg], start = p.v.seg_pos[seg];
+    const int cnt = n - i0 < kPrepTokens ? n - i0 : kPrepTokens;
+    const bool qk_head = head < p.KH;
+    const size_t hist = (size_t)row * (TAPS - 1) * p.channels;
+    const int vbase = 2 * p.KH * p.KD + head * p.VD;
+    // input of channel pair c at local index i (negative: what earlier steps left; before the sequence's start: zero)
+    auto input = [&](int c, int i) {
+        if (start + i < 0) return make_float2(0.0f, 0.0f);
+        return i >= 0 ? load2<BF16>(p.b.in, (size_t)(off + i) * p.ld + c) : load2<BF16>(p.b.conv_state, hist + (size_t)(TAPS - 1 + i) * p.channels + c);
+    };
+    struct Window {
+        float2 w[TAPS]; // filter of either channel, tap by tap
+        float2 x[TAPS > 1 ? TAPS - 1 : 1];
+    };
+    Window q[J], k[J], v[J];
+    auto open = [&](Window &win, int c) {
+#pragma unroll
+        for (int t = 0; t < TAPS; ++t) win.w[t] = make_float2(p.conv[(size_t)c * TAPS + t], p.conv[(size_t)(c + 1) * TAPS + t]);
+#pragma unroll
+        for (int t = 0; t < TAPS - 1; ++t) win.x[t] = input(c, i0 - (TAPS - 1) + t);
+    };
+    auto advance = [&](Window &win, float2 in) { // silu of the filtered inputs; the window moves on by one token
+        float2 a = make_float2(0.0f, 0.0f);
+#pragma unroll
+        for (int t = 0; t < TAPS - 1; ++t) a.x = fmaf(win.w[t].x, win.x[t].x, a.x), a.y = fmaf(win.w[t].y, win.x[t].y, a.y);
+        a.x = fmaf(win.w[TAPS - 1].x, in.x, a.x), a.y = fmaf(win.w[TAPS - 1].y, in.y, a.y);
+#pragma unroll
+        for (int t = 0; t + 1 < TAPS - 1; ++t) win.x[t] = win.x[t + 1];
+        if constexpr (TAPS > 1) win.x[TAPS - 2] = in;
+        return make_float2(silu_of<BF16>(a.x), silu_of<BF16>(a.y));
+    };
+    float2 dtb[J];
+#pragma unroll
+    for (int j = 0; j < J; ++j) {
+        const int c = j * 128 + lane * 2;
+        if (qk_head && c < p.KD) open(q[j], head * p.KD + c), open(k[j], (p.KH + head) * p.KD + c);
+        if (c < p.VD) open(v[j], vbase + c);
+        dtb[j] = c < p.KD ? *(const float2 *)(p.dt_bias + head * p.KD + c) : make_float2(0.0f, 0.0f);
+    }
+    const float decay = p.decay[head];
+    float2 nq[J], nk[J], nv[J], ng[J]; // the next token's values, requested a token ahead
+    float nb = 0.0f;
+    auto request = [&](int i) {
+        const int t = off + i;
+        const size_t in_row = (size_t)t * p.ld;
+#pragma unroll
+        for (int j = 0; j < J; ++j) {
+            const int c = j * 128 + lane * 2;
+            nq[j] = nk[j] = nv[j] = ng[j] = make_float2(0.0f, 0.0f);
+            if (qk_head && c < p.KD) nq[j] = load2<BF16>(p.b.in, in_row + head * p.KD + c), nk[j] = load2<BF16>(p.b.in, in_row + (p.KH + head) * p.KD + c);
+            if (c < p.VD) nv[j] = load2<BF16>(p.b.in, in_row + vbase + c);
+            if (c < p.KD) ng[j] = *(const float2 *)(p.b.gates + (size_t)t * 2 * p.gcols + head * p.KD + c);
+        }
+        nb = ldb<BF16>(p.b.in, in_row + p.beta_col + head);
+    };
+    request(i0);
+    for (int i = i0; i < i0 + cnt; ++i) {
+        const int t = off + i;
+        float2 xq[J], xk[J], xv[J], xg[J];
+#pragma unroll
+        for (int j = 0; j < J; ++j) xq[j] = nq[j], xk[j] = nk[j], xv[j] = nv[j], xg[j] = ng[j];
+        const float bl = nb;
+        if (i + 1 < i0 + cnt) request(i + 1);
+        float sq = 0.0f, sk = 0.0f, dot = 0.0f;
+#pragma unroll
+        for (int j = 0; j < J; ++j) {
+            const int c = j * 128 + lane * 2;
+            if (qk_head && c < p.KD) {
+                xq[j] = advance(q[j], xq[j]), xk[j] = advance(k[j], xk[j]);
+                sq = fmaf(xq[j].x, xq[j].x, fmaf(xq[j].y, xq[j].y, sq));
+                sk = fmaf(xk[j].x, xk[j].x, fmaf(xk[j].y, xk[j].y, sk));
+                dot = fmaf(xq[j].x, xk[j].x, fmaf(xq[j].y, xk[j].y, dot));
+            }
+            if (c < p.VD) *(float2 *)(p.b.v + ((size_t)t * p.H + head) * p.VD + c) = advance(v[j], xv[j]);
+            if (c < p.KD) {
+                *(float2 *)(p.b.g + ((size_t)t * p.H + head) * p.KD + c) = make_float2(exp_of<BF16>(-decay * softplus_of<BF16>(xg[j].x + dtb[j].x)),
+                        exp_of<BF16>(-decay * softplus_of<BF16>(xg[j].y + dtb[j].y)));
+            }
+        }
+        if (qk_head) { // (the same for the whole wave)
+            sq = 1.0f / sqrtf(wave_total(sq) + 1e-6f) * p.qscale, sk = 1.0f / sqrtf(wave_total(sk) + 1e-6f);
+            dot = wave_total(dot) * sq * sk;
+            const size_t at = ((size_t)t * p.KH + head) * p.KD;
+#pragma unroll
+            for (int j = 0; j < J; ++j) {
+                const int c = j * 128 + lane * 2;
+                if (c < p.KD) {
+                    *(float2 *)(p.b.q + at + c) = make_float2(xq[j].x * sq, xq[j].y * sq);
+                    *(float2 *)(p.b.k + at + c) = make_float2(xk[j].x * sk, xk[j].y * sk);
+                }
+            }
+            if (lane == 0) p.b.qk[(size_t)t * p.KH + head] = dot;
+        }
+        if (lane == 0) p.b.beta[(size_t)t * p.H + head] = sigmoid_of<BF16>(bl);
+    }
+    if (n == 1 && TAPS > 1) { // a single new token: nobody else reads these channels of the slot
+        auto keep = [&](const Window &win, int c) {
+#pragma unroll
+            for (int t = 0; t < TAPS - 1; ++t) store2<BF16>(p.b.conv_state, hist + (size_t)t * p.channels + c, win.x[t]);
+        };
+#pragma unroll
+        for (int j = 0; j < J; ++j) {
+            const int c = j * 128 + lane * 2;
+            if (qk_head && c < p.KD) keep(q[j], head * p.KD + c), keep(k[j], (p.KH + head) * p.KD + c);
+            if (c < p.VD) keep(v[j], vbase + c);
+        }
+    }
 }
 
 // the last taps - 1 inputs of a segment of several tokens; one thread a channel
@@ -189,25 +358,38 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(ScanParams p) {
     for (int c0 = 0; c0 < n; c0 += CT, buf ^= 1) {
         const int m = n - c0 < CT ? n - c0 : CT;
         if (c0 + CT < n) fetch(c0 + CT);
-        const float *lq = lds[buf] + 4 * li, *lk = lq + CT * KD, *lg = lk + CT * KD;
-        for (int i = 0; i < m; ++i) {
-            const f32x4 q0 = *(const f32x4 *)(lq + i * KD), q1 = *(const f32x4 *)(lq + i * KD + 4 * L);
-            const f32x4 k0 = *(const f32x4 *)(lk + i * KD), k1 = *(const f32x4 *)(lk + i * KD + 4 * L);
-            const f32x4 g0 = *(const f32x4 *)(lg + i * KD), g1 = *(const f32x4 *)(lg + i * KD + 4 * L);
-            const float vv = vlds[buf][i * COLS + lc], beta = sc[buf][i], qk = sc[buf][CT + i];
-            float a = 0.0f, b = 0.0f;
+        const float *lq = lds[buf] + 4 * li;
+        struct Operands {
+            f32x4 q0, q1, k0, k1, g0, g1;
+            float v, beta, qk;
+        };
+        auto read = [&](int i) {
+            const float *q = lq + i * KD, *k = q + CT * KD, *g = k + CT * KD;
+            return Operands {*(const f32x4 *)q, *(const f32x4 *)(q + 4 * L), *(const f32x4 *)k, *(const f32x4 *)(k + 4 * L), *(const f32x4 *)g,
+                    *(const f32x4 *)(g + 4 * L), vlds[buf][i * COLS + lc], sc[buf][i], sc[buf][CT + i]};
+        };
+        // the operands of the next token are on their way from LDS while this one's sums go round
+        auto token = [&](const Operands &x, int i) {
+            float a0 = 0.0f, a1 = 0.0f, b0 = 0.0f, b1 = 0.0f;
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
-                s0[r] *= g0[r], s1[r] *= g1[r];
-                a = fmaf(k0[r], s0[r], a), b = fmaf(q0[r], s0[r], b);
+                s0[r] *= x.g0[r], s1[r] *= x.g1[r];
+                a0 = fmaf(x.k0[r], s0[r], a0), b0 = fmaf(x.q0[r], s0[r], b0);
+                a1 = fmaf(x.k1[r], s1[r], a1), b1 = fmaf(x.q1[r], s1[r], b1);
             }
+            const float a = group_sum<L>(a0 + a1), b = group_sum<L>(b0 + b1);
+            const float u = x.beta * (x.v - a);
 #pragma unroll
-            for (int r = 0; r < 4; ++r) a = fmaf(k1[r], s1[r], a), b = fmaf(q1[r], s1[r], b);
-            a = group_sum<L>(a), b = group_sum<L>(b);
-            const float u = beta * (vv - a);
-#pragma unroll
-            for (int r = 0; r < 4; ++r) s0[r] = fmaf(k0[r], u, s0[r]), s1[r] = fmaf(k1[r], u, s1[r]);
-            if (li == 0) olds[i * COLS + lc] = fmaf(qk, u, b);
+            for (int r = 0; r < 4; ++r) s0[r] = fmaf(x.k0[r], u, s0[r]), s1[r] = fmaf(x.k1[r], u, s1[r]);
+            if (li == 0) olds[i * COLS + lc] = fmaf(x.qk, u, b);
+        };
+        Operands even = read(0), odd;
+        for (int i = 0; i < m; i += 2) {
+            odd = read(i + 1 < m ? i + 1 : i);
+            token(even, i);
+            if (i + 1 >= m) break;
+            even = read(i + 2 < m ? i + 2 : i + 1);
+            token(odd, i + 1);
         }
         if (c0 + CT < n) stash(buf ^ 1); // (the other buffer was last read before the barrier below, one chunk ago)
         __syncthreads();
@@ -218,6 +400,37 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(ScanParams p) {
         __syncthreads();
     }
     if (own) *(f32x4 *)(state + 4 * li) = s0, *(f32x4 *)(state + 4 * (L + li)) = s1;
+}
+
+// The same step for segments of one token: nothing to stage, the kernel is a read and a write of the state.
+template <int L>
+__global__ __launch_bounds__(256) void delta_step_kernel(ScanParams p) {
+    constexpr int KD = 8 * L, COLS = 256 / L;
+    const int seg = blockIdx.x, head = blockIdx.y, kvh = head / (p.H / p.KH), t = p.v.seg_off[seg];
+    const int li = threadIdx.x % L, col = blockIdx.z * COLS + threadIdx.x / L;
+    if (col >= p.VD) return; // (whole groups of L lanes)
+    float *state = p.b.state + (((size_t)p.v.seg_row[seg] * p.H + head) * p.VD + col) * KD;
+    f32x4 s0 = *(const f32x4 *)(state + 4 * li), s1 = *(const f32x4 *)(state + 4 * (L + li));
+    const float *q = p.b.q + ((size_t)t * p.KH + kvh) * KD + 4 * li, *k = p.b.k + ((size_t)t * p.KH + kvh) * KD + 4 * li;
+    const float *g = p.b.g + ((size_t)t * p.H + head) * KD + 4 * li;
+    const f32x4 q0 = *(const f32x4 *)q, q1 = *(const f32x4 *)(q + 4 * L), k0 = *(const f32x4 *)k, k1 = *(const f32x4 *)(k + 4 * L);
+    const f32x4 g0 = *(const f32x4 *)g, g1 = *(const f32x4 *)(g + 4 * L);
+    const float v = p.b.v[((size_t)t * p.H + head) * p.VD + col], beta = p.b.beta[(size_t)t * p.H + head], qk = p.b.qk[(size_t)t * p.KH + kvh];
+    if (p.v.seg_pos[seg] == 0) s0 = s1 = f32x4 {0.f, 0.f, 0.f, 0.f};
+    float a = 0.0f, b = 0.0f;
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+        s0[r] *= g0[r], s1[r] *= g1[r];
+        a = fmaf(k0[r], s0[r], a), b = fmaf(q0[r], s0[r], b);
+    }
+#pragma unroll
+    for (int r = 0; r < 4; ++r) a = fmaf(k1[r], s1[r], a), b = fmaf(q1[r], s1[r], b);
+    a = group_sum<L>(a), b = group_sum<L>(b);
+    const float u = beta * (v - a);
+#pragma unroll
+    for (int r = 0; r < 4; ++r) s0[r] = fmaf(k0[r], u, s0[r]), s1[r] = fmaf(k1[r], u, s1[r]);
+    *(f32x4 *)(state + 4 * li) = s0, *(f32x4 *)(state + 4 * (L + li)) = s1;
+    if (li == 0) p.b.o[((size_t)t * p.H + head) * p.VD + col] = fmaf(qk, u, b);
 }
 
 struct OutParams {
@@ -237,10 +450,15 @@ __global__ __launch_bounds__(256) void delta_output_kernel(OutParams p) {
     const float *o = p.o + idx * p.VD;
     const float *gate = p.gates + (size_t)t * 2 * p.gcols + p.gcols + head * p.VD;
     float sq = 0.0f;
-    for (int c = lane; c < p.VD; c += 64) sq = fmaf(o[c], o[c], sq);
+    for (int c = lane * 2; c < p.VD; c += 128) {
+        const float2 x = *(const float2 *)(o + c);
+        sq = fmaf(x.x, x.x, fmaf(x.y, x.y, sq));
+    }
     const float r = 1.0f / sqrtf(wave_total(sq) / (float)p.vdim + p.eps);
-    for (int c = lane; c < p.VD; c += 64)
-        store_from_f32(p.on, BF16 ? XFTHIP_BF16 : XFTHIP_F32, idx * p.VD + c, o[c] * r * p.norm[c] / (1.0f + expf(-gate[c])));
+    for (int c = lane * 2; c < p.VD; c += 128) {
+        const float2 x = *(const float2 *)(o + c), w = *(const float2 *)(p.norm + c), z = *(const float2 *)(gate + c);
+        store2<BF16>(p.on, idx * p.VD + c, make_float2(x.x * r * w.x * sigmoid_of<BF16>(z.x), x.y * r * w.y * sigmoid_of<BF16>(z.y)));
+    }
 }
 
 PrepParams prep_params(const PlanLayer &L, const StepView &v, const DeltaBuffers &b) {
@@ -259,11 +477,31 @@ int delta_prepare(int act, const PlanLayer &L, const StepView &v, const DeltaBuf
     const PrepParams p = prep_params(L, v, b);
     const dim3 grid(v.T, (p.H + 3) / 4), tail((p.channels + 255) / 256, v.B);
     const bool long_segments = v.longest > 1 && p.taps > 1;
+    const int width = p.KD > p.VD ? p.KD : p.VD;
+    const bool tiled = p.taps >= 2 && p.taps <= 4 && width <= 256;
+    if (tiled) {
+        const dim3 tiles((v.longest + kPrepTokens - 1) / kPrepTokens, (p.H + 3) / 4, v.B);
+        const int key = (act == XFTHIP_BF16 ? 0 : 10) + p.taps + (width > 128 ? 100 : 0);
+        switch (key) {
+            case 2: hipLaunchKernelGGL((delta_prepare_tiled_kernel<true, 2, 1>), tiles, dim3(256), 0, st, p); break;
+            case 3: hipLaunchKernelGGL((delta_prepare_tiled_kernel<true, 3, 1>), tiles, dim3(256), 0, st, p); break;
+            case 4: hipLaunchKernelGGL((delta_prepare_tiled_kernel<true, 4, 1>), tiles, dim3(256), 0, st, p); break;
+            case 12: hipLaunchKernelGGL((delta_prepare_tiled_kernel<false, 2, 1>), tiles, dim3(256), 0, st, p); break;
+            case 13: hipLaunchKernelGGL((delta_prepare_tiled_kernel<false, 3, 1>), tiles, dim3(256), 0, st, p); break;
+            case 14: hipLaunchKernelGGL((delta_prepare_tiled_kernel<false, 4, 1>), tiles, dim3(256), 0, st, p); break;
+            case 102: hipLaunchKernelGGL((delta_prepare_tiled_kernel<true, 2, 2>), tiles, dim3(256), 0, st, p); break;
+            case 103: hipLaunchKernelGGL((delta_prepare_tiled_kernel<true, 3, 2>), tiles, dim3(256), 0, st, p); break;
+            case 104: hipLaunchKernelGGL((delta_prepare_tiled_kernel<true, 4, 2>), tiles, dim3(256), 0, st, p); break;
+            case 112: hipLaunchKernelGGL((delta_prepare_tiled_kernel<false, 2, 2>), tiles, dim3(256), 0, st, p); break;
+            case 113: hipLaunchKernelGGL((delta_prepare_tiled_kernel<false, 3, 2>), tiles, dim3(256), 0, st, p); break;
+            default: hipLaunchKernelGGL((delta_prepare_tiled_kernel<false, 4, 2>), tiles, dim3(256), 0, st, p); break;
+        }
+    }
     if (act == XFTHIP_BF16) {
-        hipLaunchKernelGGL(delta_prepare_kernel<true>, grid, dim3(256), 0, st, p);
+        if (!tiled) hipLaunchKernelGGL(delta_prepare_kernel<true>, grid, dim3(256), 0, st, p);
         if (long_segments) hipLaunchKernelGGL(conv_tail_kernel<true>, tail, dim3(256), 0, st, p);
     } else {
-        hipLaunchKernelGGL(delta_prepare_kernel<false>, grid, dim3(256), 0, st, p);
+        if (!tiled) hipLaunchKernelGGL(delta_prepare_kernel<false>, grid, dim3(256), 0, st, p);
         if (long_segments) hipLaunchKernelGGL(conv_tail_kernel<false>, tail, dim3(256), 0, st, p);
     }
     XFT_CHECK_HIP(hipGetLastError());
@@ -275,6 +513,16 @@ int delta_scan(const PlanLayer &L, const StepView &v, const DeltaBuffers &b, hip
     p.v = v, p.b = b, p.H = L.s.heads, p.KH = L.s.kv_heads, p.VD = L.VD;
     const int lanes = L.KD / 8, cols = 256 / lanes;
     const dim3 grid(v.B, p.H, (L.VD + cols - 1) / cols);
+    if (v.longest == 1 && (lanes == 4 || lanes == 8 || lanes == 16 || lanes == 32)) {
+        switch (lanes) {
+            case 4: hipLaunchKernelGGL(delta_step_kernel<4>, grid, dim3(256), 0, st, p); break;
+            case 8: hipLaunchKernelGGL(delta_step_kernel<8>, grid, dim3(256), 0, st, p); break;
+            case 16: hipLaunchKernelGGL(delta_step_kernel<16>, grid, dim3(256), 0, st, p); break;
+            default: hipLaunchKernelGGL(delta_step_kernel<32>, grid, dim3(256), 0, st, p); break;
+        }
+        XFT_CHECK_HIP(hipGetLastError());
+        return 0;
+    }
     switch (lanes) {
         case 4: hipLaunchKernelGGL(delta_scan_kernel<4>, grid, dim3(256), 0, st, p); break;
         case 8: hipLaunchKernelGGL(delta_scan_kernel<8>, grid, dim3(256), 0, st, p); break;

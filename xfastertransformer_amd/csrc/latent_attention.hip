@@ -49,28 +49,49 @@ struct PrepareParams {
 };
 
 template <bool BF16>
+__device__ inline void load8(const void *p, size_t i, float (&v)[8]) {
+    if constexpr (BF16) {
+        const uint4 q = *(const uint4 *)((const uint16_t *)p + i);
+        const uint32_t w[4] = {q.x, q.y, q.z, q.w};
+#pragma unroll
+        for (int k = 0; k < 4; ++k) v[2 * k] = u2f(w[k] << 16), v[2 * k + 1] = u2f(w[k] & 0xFFFF0000u);
+    } else {
+        const f32x4 x = *(const f32x4 *)((const float *)p + i), y = *(const f32x4 *)((const float *)p + i + 4);
+#pragma unroll
+        for (int k = 0; k < 4; ++k) v[k] = x[k], v[4 + k] = y[k];
+    }
+}
+template <bool BF16>
+__device__ inline void store8(void *p, size_t i, const float (&v)[8]) {
+    if constexpr (BF16) {
+        uint32_t w[4];
+#pragma unroll
+        for (int k = 0; k < 4; ++k) w[k] = f32_bits_to_bf16_sel(f2u(v[2 * k])) | (f32_bits_to_bf16_sel(f2u(v[2 * k + 1])) << 16);
+        *(uint4 *)((uint16_t *)p + i) = make_uint4(w[0], w[1], w[2], w[3]);
+    } else {
+        *(f32x4 *)((float *)p + i) = f32x4 {v[0], v[1], v[2], v[3]};
+        *(f32x4 *)((float *)p + i + 4) = f32x4 {v[4], v[5], v[6], v[7]};
+    }
+}
+
+// One token a workgroup, 8 neighbouring values a thread and turn; the row and the norm weights are in registers (CH turns)
+// before the sums meet.
+template <bool BF16, int CH>
 __global__ __launch_bounds__(256) void latent_prepare_kernel(PrepareParams p) {
     __shared__ float part[2][4];
-    const int t = blockIdx.x, R = p.cache.R;
-    const size_t base = (size_t)t * (p.QR + R + p.RD);
-    float sq = 0.0f, sk = 0.0f;
-    for (int c = threadIdx.x; c < p.QR; c += 256) {
-        const float x = ldact<BF16>(p.a, base + c);
-        sq = fmaf(x, x, sq);
-    }
-    for (int c = threadIdx.x; c < R; c += 256) {
-        const float x = ldact<BF16>(p.a, base + p.QR + c);
-        sk = fmaf(x, x, sk);
-    }
-    sq = wave_total(sq), sk = wave_total(sk);
-    if ((threadIdx.x & 63) == 0) part[0][threadIdx.x >> 6] = sq, part[1][threadIdx.x >> 6] = sk;
-    __syncthreads();
-    sq = (part[0][0] + part[0][1]) + (part[0][2] + part[0][3]), sk = (part[1][0] + part[1][1]) + (part[1][2] + part[1][3]);
-    const float rq = 1.0f / sqrtf(sq / (float)p.q_rank + p.eps), rk = 1.0f / sqrtf(sk / (float)p.kv_rank + p.eps);
-    for (int c = threadIdx.x; c < p.QR; c += 256) stact<BF16>(p.cq, (size_t)t * p.QR + c, ldact<BF16>(p.a, base + c) * rq * p.q_norm[c]);
+    const int t = blockIdx.x, R = p.cache.R, len = p.QR + R + p.RD;
+    const size_t base = (size_t)t * len;
     const int seg = p.v.tok_seg[t], pos = p.v.tok_pos[t];
+    float x[CH][8], w[CH][8], sq = 0.0f, sk = 0.0f;
+#pragma unroll
+    for (int i = 0; i < CH; ++i) {
+        const int c = (i * 256 + (int)threadIdx.x) * 8;
+        if (c >= p.QR + R) continue;
+        load8<BF16>(p.a, base + c, x[i]);
+        load8<false>(c < p.QR ? p.q_norm : p.kv_norm - p.QR, c, w[i]);
+    }
     const size_t dst = cache_row(p.v, p.v.seg_row[seg], pos) * (R + p.RD);
-    for (int c = threadIdx.x; c < R; c += 256) stact<BF16>(p.cache.pool, dst + c, ldact<BF16>(p.a, base + p.QR + c) * rk * p.kv_norm[c]);
+    // the shared key part: one value a thread, its partner read beside it
     const int half = p.rot / 2;
     for (int c = threadIdx.x; c < p.RD; c += 256) {
         float y = 0.0f;
@@ -78,11 +99,35 @@ __global__ __launch_bounds__(256) void latent_prepare_kernel(PrepareParams p) {
             const int i = p.interleaved ? c >> 1 : (c < half ? c : c - half);
             const bool second = p.interleaved ? (c & 1) != 0 : c >= half;
             const float u = ldact<BF16>(p.a, base + p.QR + R + (p.interleaved ? 2 * i : i));
-            const float w = ldact<BF16>(p.a, base + p.QR + R + (p.interleaved ? 2 * i + 1 : i + half));
+            const float z = ldact<BF16>(p.a, base + p.QR + R + (p.interleaved ? 2 * i + 1 : i + half));
             const float cs = p.cosT[(size_t)pos * half + i], sn = p.sinT[(size_t)pos * half + i];
-            y = second ? fmaf(w, cs, u * sn) : fmaf(u, cs, -(w * sn));
+            y = second ? fmaf(z, cs, u * sn) : fmaf(u, cs, -(z * sn));
         }
         stact<BF16>(p.cache.pool, dst + R + c, y);
+    }
+#pragma unroll
+    for (int i = 0; i < CH; ++i) {
+        const int c = (i * 256 + (int)threadIdx.x) * 8;
+        if (c >= p.QR + R) continue;
+        float s = 0.0f;
+#pragma unroll
+        for (int k = 0; k < 8; ++k) s = fmaf(x[i][k], x[i][k], s);
+        (c < p.QR ? sq : sk) += s;
+    }
+    sq = wave_total(sq), sk = wave_total(sk);
+    if ((threadIdx.x & 63) == 0) part[0][threadIdx.x >> 6] = sq, part[1][threadIdx.x >> 6] = sk;
+    __syncthreads();
+    sq = (part[0][0] + part[0][1]) + (part[0][2] + part[0][3]), sk = (part[1][0] + part[1][1]) + (part[1][2] + part[1][3]);
+    const float rq = 1.0f / sqrtf(sq / (float)p.q_rank + p.eps), rk = 1.0f / sqrtf(sk / (float)p.kv_rank + p.eps);
+#pragma unroll
+    for (int i = 0; i < CH; ++i) {
+        const int c = (i * 256 + (int)threadIdx.x) * 8;
+        if (c >= p.QR + R) continue;
+        const float r = c < p.QR ? rq : rk;
+#pragma unroll
+        for (int k = 0; k < 8; ++k) x[i][k] = x[i][k] * r * w[i][k];
+        if (c < p.QR) store8<BF16>(p.cq, (size_t)t * p.QR + c, x[i]);
+        else store8<BF16>(p.cache.pool, dst + c - p.QR, x[i]);
     }
 }
 
@@ -170,10 +215,13 @@ typedef __attribute__((ext_vector_type(8))) short s16x8;
 constexpr float kUnseen = -1.0e30f; // score of a masked key, maximum of a column that has seen none
 constexpr float kLog2e = 1.4426950408889634f;
 
+typedef __attribute__((ext_vector_type(2))) __bf16 bf16x2;
+// two values -> packed bf16 pair, round to nearest even (v_cvt_pk_bf16_f32)
+__device__ inline uint32_t pack_pair(float lo, float hi) { return __builtin_bit_cast(uint32_t, bf16x2 {(__bf16)lo, (__bf16)hi}); }
 __device__ inline bf16x8 pack_bf16x8(const float (&v)[8]) {
     u32x4 u;
 #pragma unroll
-    for (int i = 0; i < 4; ++i) u[i] = f32_to_bf16_ref(v[2 * i]) | ((uint32_t)f32_to_bf16_ref(v[2 * i + 1]) << 16);
+    for (int i = 0; i < 4; ++i) u[i] = pack_pair(v[2 * i], v[2 * i + 1]);
     return __builtin_bit_cast(bf16x8, u);
 }
 
@@ -195,12 +243,13 @@ struct MfmaParams {
 // workgroup, the context split over gridDim.z.  32 tokens at a time go through LDS: a wave scores 16 of them for 16 columns
 // (A = cached rows, B = the columns' queries in registers), the scores meet in LDS, every wave turns them into
 // probabilities and adds up its own quarter of the latent dimensions (A = the same rows read transposed).
-// DT: 16-dim tiles of a wave (R <= 64 DT); KSMAX: most 32-dim steps of a row.
-template <int DT, int KSMAX>
+// DT: 16-dim tiles of a wave (R <= 64 DT); KSMAX: most 32-dim steps of a row; EXACT: R = 64 DT and a row is KSMAX steps, so
+// that the loops over them are straight-line code.
+template <int DT, int KSMAX, bool EXACT>
 __global__ __launch_bounds__(256, 2) void latent_mfma_kernel(MfmaParams p) {
     extern __shared__ unsigned char lds[];
     const StepView &v = p.a.v;
-    const int seg = blockIdx.y, n = v.seg_len[seg], H = p.a.H, R = p.a.cache.R, RD = p.RD;
+    const int seg = blockIdx.y, n = v.seg_len[seg], H = p.a.H, R = EXACT ? 64 * DT : p.a.cache.R, RD = p.RD;
     const int c0 = blockIdx.x * 32, ncols = n * H;
     if (n > p.max_len || c0 >= ncols) return;
     const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), g = lane >> 4, i16 = lane & 15;
@@ -212,7 +261,7 @@ __global__ __launch_bounds__(256, 2) void latent_mfma_kernel(MfmaParams p) {
     const int b0 = first_vis >> 5, b1 = (hi >> 5) + 1;
     const int per = (b1 - b0 + p.nsplit - 1) / p.nsplit;
     const int bb = b0 + (int)blockIdx.z * per, be = bb + per < b1 ? bb + per : b1;
-    const int row_len = R + RD, ks_n = row_len / 32, row_chunks = row_len / 8, chunks = 32 * row_chunks;
+    const int row_len = EXACT ? KSMAX * 32 : R + RD, ks_n = row_len / 32, row_chunks = row_len / 8, chunks = 32 * row_chunks;
     const int pitch = row_len * 2 + 16;
     float *sc = (float *)(lds + 2 * 32 * pitch); // [32 columns][36]
 
@@ -225,7 +274,7 @@ __global__ __launch_bounds__(256, 2) void latent_mfma_kernel(MfmaParams p) {
         const uint16_t *qr = (const uint16_t *)p.a.q + at * (p.a.D + RD) + p.a.D + 8 * g - R;
 #pragma unroll
         for (int ks = 0; ks < KSMAX; ++ks)
-            if (ks < ks_n) qf[ks] = *(const bf16x8 *)((ks * 32 < R ? qa : qr) + ks * 32);
+            if (EXACT || ks < ks_n) qf[ks] = *(const bf16x8 *)((ks * 32 < R ? qa : qr) + ks * 32);
     }
     // this lane's column of either column tile: position, running maximum (log2 domain) and this lane's part of the sum
     int cpos[2];
@@ -248,13 +297,14 @@ __global__ __launch_bounds__(256, 2) void latent_mfma_kernel(MfmaParams p) {
 #pragma unroll
         for (int i = 0; i < PER; ++i) {
             const int e = i * 256 + threadIdx.x;
-            if (e < chunks) stage[i] = src[e];
+            stage[i] = src[e < chunks ? e : chunks - 1]; // (past the block: its last chunk once more)
         }
     };
     int lds_off[PER]; // chunk e of a block: 16 bytes of padding behind every row before it
 #pragma unroll
     for (int i = 0; i < PER; ++i) {
-        const int e = i * 256 + threadIdx.x;
+        int e = i * 256 + threadIdx.x;
+        e = e < chunks ? e : chunks - 1;
         lds_off[i] = (e + e / row_chunks) * 16;
     }
     if (bb < be) fetch(bb, table[bb >> 1]);
@@ -263,17 +313,16 @@ __global__ __launch_bounds__(256, 2) void latent_mfma_kernel(MfmaParams p) {
     for (int blk = bb; blk < be; ++blk, buf ^= 1) {
         unsigned char *kv = lds + buf * 32 * pitch;
 #pragma unroll
-        for (int i = 0; i < PER; ++i)
-            if (i * 256 + (int)threadIdx.x < chunks) *(u32x4 *)(kv + lds_off[i]) = stage[i];
+        for (int i = 0; i < PER; ++i) *(u32x4 *)(kv + lds_off[i]) = stage[i];
         __syncthreads();
         if (blk + 1 < be) fetch(blk + 1, page);
         if (blk + 2 < be) page = table[(blk + 2) >> 1];
-        f32x4 s = {0.f, 0.f, 0.f, 0.f};
+        f32x4 s = {0.f, 0.f, 0.f, 0.f}, s1 = s; // (two chains of products)
         const unsigned char *krow = kv + (16 * tt + i16) * pitch + 16 * g;
 #pragma unroll
         for (int ks = 0; ks < KSMAX; ++ks)
-            if (ks < ks_n) s = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*(const bf16x8 *)(krow + ks * 64), qf[ks], s, 0, 0, 0);
-        *(f32x4 *)(sc + (16 * ct_s + i16) * 36 + 16 * tt + 4 * g) = s;
+            if (EXACT || ks < ks_n) (ks & 1 ? s1 : s) = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*(const bf16x8 *)(krow + ks * 64), qf[ks], ks & 1 ? s1 : s, 0, 0, 0);
+        *(f32x4 *)(sc + (16 * ct_s + i16) * 36 + 16 * tt + 4 * g) = s + s1;
         __syncthreads();
         bf16x8 pf[2];
         float alpha[2];
@@ -311,7 +360,7 @@ __global__ __launch_bounds__(256, 2) void latent_mfma_kernel(MfmaParams p) {
 #pragma unroll
         for (int d = 0; d < DT; ++d) {
             const int tile = wave * DT + d;
-            if (tile * 16 < R) {
+            if (EXACT || tile * 16 < R) {
                 const bf16x8 a = transposed_pair(vrow + tile * 32, vrow + tile * 32 + 4 * pitch);
                 o[d][0] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, pf[0], o[d][0], 0, 0, 0);
                 o[d][1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, pf[1], o[d][1], 0, 0, 0);
@@ -330,7 +379,7 @@ __global__ __launch_bounds__(256, 2) void latent_mfma_kernel(MfmaParams p) {
 #pragma unroll
                 for (int d = 0; d < DT; ++d) {
                     const int tile = wave * DT + d;
-                    if (tile * 16 < R) *(f32x4 *)(p.part + slot * R + tile * 16 + 4 * g) = o[d][ct];
+                    if (EXACT || tile * 16 < R) *(f32x4 *)(p.part + slot * R + tile * 16 + 4 * g) = o[d][ct];
                 }
             }
         } else if (c < ncols) {
@@ -345,43 +394,55 @@ __global__ __launch_bounds__(256, 2) void latent_mfma_kernel(MfmaParams p) {
 #pragma unroll
             for (int d = 0; d < DT; ++d) {
                 const int tile = wave * DT + d;
-                if (tile * 16 < R) {
+                if (EXACT || tile * 16 < R) {
                     const f32x4 y = o[d][ct] * mul;
-                    *(uint2 *)(dst + tile * 16 + 4 * g) = make_uint2(f32_to_bf16_ref(y[0]) | ((uint32_t)f32_to_bf16_ref(y[1]) << 16),
-                            f32_to_bf16_ref(y[2]) | ((uint32_t)f32_to_bf16_ref(y[3]) << 16));
+                    *(uint2 *)(dst + tile * 16 + 4 * g) = make_uint2(pack_pair(y[0], y[1]), pack_pair(y[2], y[3]));
                 }
             }
         }
     }
 }
 
-// sum of a column's splits; grid (column groups, segments, 32 columns)
+// sum of a column's splits; grid (column groups, segments, 32 columns).  The splits' weights are worked out once, side by
+// side, and the outputs are added four splits at a time.
+constexpr int kMaxSplits = 64;
 __global__ __launch_bounds__(128) void latent_merge_kernel(MfmaParams p) {
+    __shared__ float w[kMaxSplits];
+    __shared__ float inv_den;
     const StepView &v = p.a.v;
     const int seg = blockIdx.y, n = v.seg_len[seg], H = p.a.H, R = p.a.cache.R;
     const int c = blockIdx.x * 32 + blockIdx.z;
     if (n > p.max_len || c >= n * H) return;
     const size_t unit = ((size_t)seg * gridDim.x + blockIdx.x) * p.nsplit;
-    float mt = p.a.sink ? p.a.sink[c % H] * kLog2e : kUnseen;
-    const float s2 = mt;
-    for (int s = 0; s < p.nsplit; ++s) mt = fmaxf(mt, p.part[p.part_ml + ((unit + s) * 32 + blockIdx.z) * 2]);
-    float den = p.a.sink ? __builtin_amdgcn_exp2f(s2 - mt) : 0.0f;
-    for (int s = 0; s < p.nsplit; ++s) {
-        const float2 ml = *(const float2 *)(p.part + p.part_ml + ((unit + s) * 32 + blockIdx.z) * 2);
-        if (ml.x > 0.5f * kUnseen) den += ml.y * __builtin_amdgcn_exp2f(ml.x - mt);
+    if (threadIdx.x < 64) {
+        float2 ml = make_float2(kUnseen, 0.0f);
+        if ((int)threadIdx.x < p.nsplit) ml = *(const float2 *)(p.part + p.part_ml + ((unit + threadIdx.x) * 32 + blockIdx.z) * 2);
+        const float s2 = p.a.sink ? p.a.sink[c % H] * kLog2e : kUnseen;
+        const float mt = fmaxf(wave_largest(ml.x), s2);
+        const float e = ml.x > 0.5f * kUnseen ? __builtin_amdgcn_exp2f(ml.x - mt) : 0.0f;
+        const float den = wave_total(ml.y * e) + (p.a.sink ? __builtin_amdgcn_exp2f(s2 - mt) : 0.0f);
+        w[threadIdx.x] = e;
+        if (threadIdx.x == 0) inv_den = 1.0f / den;
     }
-    const float inv = 1.0f / den;
+    __syncthreads();
+    const float inv = inv_den;
     uint16_t *dst = (uint16_t *)p.a.out + ((size_t)v.seg_off[seg] * H + c) * R;
+    const float *src = p.part + (unit * 32 + blockIdx.z) * R;
     for (int d = threadIdx.x * 4; d < R; d += 512) {
-        f32x4 acc = {0.f, 0.f, 0.f, 0.f};
-        for (int s = 0; s < p.nsplit; ++s) {
-            const size_t slot = (unit + s) * 32 + blockIdx.z;
-            const float ms = p.part[p.part_ml + slot * 2];
-            if (ms > 0.5f * kUnseen) acc += *(const f32x4 *)(p.part + slot * R + d) * __builtin_amdgcn_exp2f(ms - mt);
+        f32x4 acc[4];
+#pragma unroll
+        for (int i = 0; i < 4; ++i) acc[i] = f32x4 {0.f, 0.f, 0.f, 0.f};
+        for (int s0 = 0; s0 < p.nsplit; s0 += 4) {
+            f32x4 x[4];
+#pragma unroll
+            for (int i = 0; i < 4; ++i) x[i] = *(const f32x4 *)(src + (size_t)(s0 + i < p.nsplit ? s0 + i : p.nsplit - 1) * 32 * R + d);
+            // (a part nobody wrote has weight 0 and may hold anything)
+#pragma unroll
+            for (int i = 0; i < 4; ++i)
+                if (s0 + i < p.nsplit && w[s0 + i] > 0.0f) acc[i] += x[i] * w[s0 + i];
         }
-        acc *= inv;
-        *(uint2 *)(dst + d) = make_uint2(f32_to_bf16_ref(acc[0]) | ((uint32_t)f32_to_bf16_ref(acc[1]) << 16),
-                f32_to_bf16_ref(acc[2]) | ((uint32_t)f32_to_bf16_ref(acc[3]) << 16));
+        const f32x4 y = ((acc[0] + acc[1]) + (acc[2] + acc[3])) * inv;
+        *(uint2 *)(dst + d) = make_uint2(pack_pair(y[0], y[1]), pack_pair(y[2], y[3]));
     }
 }
 
@@ -404,14 +465,14 @@ struct ExpandedParams {
 //   S^T = K Q^T (A = keys from LDS, B = the wave's queries in registers), O^T += V^T P^T (A = values from LDS read
 // transposed, B = probabilities straight from the score registers: half h of the wave holds tokens 8 q + 4 h + s of a block,
 // and the value operand takes its tokens in that order).
-// KSM: most 16-dim steps of a query; VTM: most 32-dim tiles of a value.  grid (heads, query blocks)
-template <int KSM, int VTM>
+// KSM: most 16-dim steps of a query; VTM: most 32-dim tiles of a value; EXACT: as many.  grid (heads, query blocks)
+template <int KSM, int VTM, bool EXACT>
 __global__ __launch_bounds__(256, 2) void latent_expanded_kernel(ExpandedParams p) {
     extern __shared__ unsigned char lds[];
     const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), h = lane >> 5, cl = lane & 31;
     const int head = blockIdx.x, q0 = ((int)gridDim.y - 1 - (int)blockIdx.y) * 128; // the blocks with the longest contexts first
-    const int Dq = p.D + p.RD, ks_n = Dq / 16, vt_n = p.V / 32;
-    const int kpitch = Dq * 2 + 16, vpitch = p.V * 2 + 16, bufb = 32 * (kpitch + vpitch);
+    const int Dq = EXACT ? KSM * 16 : p.D + p.RD, ks_n = Dq / 16, V = EXACT ? VTM * 32 : p.V, vt_n = V / 32;
+    const int kpitch = Dq * 2 + 16, vpitch = V * 2 + 16, bufb = 32 * (kpitch + vpitch);
     const int qi = q0 + wave * 32 + cl;
     const int pos = p.start + (qi < p.n ? qi : p.n - 1);
     const int wlo = p.start + q0 + wave * 32, whi_q = q0 + wave * 32 + 31;
@@ -422,7 +483,7 @@ __global__ __launch_bounds__(256, 2) void latent_expanded_kernel(ExpandedParams 
         const uint16_t *row = p.q + ((size_t)(p.off + (qi < p.n ? qi : p.n - 1)) * p.H + head) * Dq + 8 * h;
 #pragma unroll
         for (int ks = 0; ks < KSM; ++ks)
-            if (ks < ks_n) qf[ks] = *(const bf16x8 *)(row + ks * 16);
+            if (EXACT || ks < ks_n) qf[ks] = *(const bf16x8 *)(row + ks * 16);
     }
     f32x16 o[VTM];
 #pragma unroll
@@ -437,40 +498,39 @@ __global__ __launch_bounds__(256, 2) void latent_expanded_kernel(ExpandedParams 
     const int wfirst = p.window > 0 && wlo + 1 > p.window ? wlo + 1 - p.window : 0;
 
     constexpr int PER = (16 * KSM + 32 * VTM + 63) / 64;
-    const int kd = p.D / 8, kr = p.RD / 8, kv8 = p.V / 8;
+    const int kd = p.D / 8, kr = p.RD / 8, kv8 = V / 8;
     u32x4 stage[PER];
-    // chunk e of a block: 32 rows of unrotated keys, of rotated parts, of values
+    // chunk e of a block: 32 rows of unrotated keys, of rotated parts, of values (past them: the last one once more)
     const uint16_t *src[PER];
-    size_t step[PER];
+    uint32_t step[PER];
     int dst[PER];
 #pragma unroll
     for (int i = 0; i < PER; ++i) {
         int e = i * 256 + threadIdx.x;
-        src[i] = nullptr, step[i] = 0, dst[i] = 0;
         if (e < 32 * kd) {
             const int r = e / kd, c = e % kd;
-            step[i] = (size_t)p.H * p.D, src[i] = p.k + r * step[i] + (size_t)head * p.D + c * 8, dst[i] = r * kpitch + c * 16;
+            step[i] = (uint32_t)(p.H * p.D), src[i] = p.k + (size_t)r * step[i] + (size_t)head * p.D + c * 8, dst[i] = r * kpitch + c * 16;
         } else if ((e -= 32 * kd) < 32 * kr) {
             const int r = e / kr, c = e % kr;
-            step[i] = (size_t)(p.R + p.RD), src[i] = p.rows + r * step[i] + p.R + c * 8, dst[i] = r * kpitch + p.D * 2 + c * 16;
-        } else if ((e -= 32 * kr) < 32 * kv8) {
+            step[i] = (uint32_t)(p.R + p.RD), src[i] = p.rows + (size_t)r * step[i] + p.R + c * 8, dst[i] = r * kpitch + p.D * 2 + c * 16;
+        } else {
+            e -= 32 * kr;
+            e = e < 32 * kv8 ? e : 32 * kv8 - 1;
             const int r = e / kv8, c = e % kv8;
-            step[i] = (size_t)p.H * p.V, src[i] = p.vv + r * step[i] + (size_t)head * p.V + c * 8, dst[i] = 32 * kpitch + r * vpitch + c * 16;
+            step[i] = (uint32_t)(p.H * V), src[i] = p.vv + (size_t)r * step[i] + (size_t)head * V + c * 8, dst[i] = 32 * kpitch + r * vpitch + c * 16;
         }
     }
     // (rows behind the segment's end lie inside the buffers, which hold whole blocks)
     auto fetch = [&](int blk) {
 #pragma unroll
-        for (int i = 0; i < PER; ++i)
-            if (src[i]) stage[i] = *(const u32x4 *)(src[i] + (size_t)(blk * 32 - p.base) * step[i]);
+        for (int i = 0; i < PER; ++i) stage[i] = *(const u32x4 *)(src[i] + (size_t)(uint32_t)(blk * 32 - p.base) * step[i]);
     };
     fetch(b0);
     int buf = 0;
     for (int blk = b0; blk < b1; ++blk, buf ^= 1) {
         unsigned char *kb = lds + buf * bufb, *vb = kb + 32 * kpitch;
 #pragma unroll
-        for (int i = 0; i < PER; ++i)
-            if (src[i]) *(u32x4 *)(kb + dst[i]) = stage[i];
+        for (int i = 0; i < PER; ++i) *(u32x4 *)(kb + dst[i]) = stage[i];
         __syncthreads();
         if (blk + 1 < b1) fetch(blk + 1);
         const int t0 = blk * 32;
@@ -481,7 +541,7 @@ __global__ __launch_bounds__(256, 2) void latent_expanded_kernel(ExpandedParams 
         const unsigned char *krow = kb + cl * kpitch + 16 * h;
 #pragma unroll
         for (int ks = 0; ks < KSM; ++ks)
-            if (ks < ks_n) s = __builtin_amdgcn_mfma_f32_32x32x16_bf16(*(const bf16x8 *)(krow + ks * 32), qf[ks], s, 0, 0, 0);
+            if (EXACT || ks < ks_n) s = __builtin_amdgcn_mfma_f32_32x32x16_bf16(*(const bf16x8 *)(krow + ks * 32), qf[ks], s, 0, 0, 0);
         const bool masked = t0 + 31 > wlo || (p.window > 0 && t0 + p.window <= whi);
         float bm = kUnseen;
 #pragma unroll
@@ -526,7 +586,7 @@ __global__ __launch_bounds__(256, 2) void latent_expanded_kernel(ExpandedParams 
             const unsigned char *vrow = vb + (16 * t + 4 * h + ((lane & 15) >> 2)) * vpitch + 32 * ((lane >> 4) & 1) + 8 * (lane & 3);
 #pragma unroll
             for (int d = 0; d < VTM; ++d)
-                if (d < vt_n) o[d] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(transposed_pair(vrow + d * 64, vrow + d * 64 + 8 * vpitch), pf, o[d], 0, 0, 0);
+                if (EXACT || d < vt_n) o[d] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(transposed_pair(vrow + d * 64, vrow + d * 64 + 8 * vpitch), pf, o[d], 0, 0, 0);
         }
     }
     l += __shfl_xor(l, 32, 64);
@@ -541,28 +601,27 @@ __global__ __launch_bounds__(256, 2) void latent_expanded_kernel(ExpandedParams 
     uint16_t *out = p.out + (size_t)(p.off + qi) * p.H * p.V + (size_t)head * p.V;
 #pragma unroll
     for (int d = 0; d < VTM; ++d)
-        if (d < vt_n) {
+        if (EXACT || d < vt_n) {
 #pragma unroll
             for (int q = 0; q < 4; ++q)
                 *(uint2 *)(out + d * 32 + 8 * q + 4 * h) =
-                        make_uint2(f32_to_bf16_ref(o[d][4 * q] * mul) | ((uint32_t)f32_to_bf16_ref(o[d][4 * q + 1] * mul) << 16),
-                                f32_to_bf16_ref(o[d][4 * q + 2] * mul) | ((uint32_t)f32_to_bf16_ref(o[d][4 * q + 3] * mul) << 16));
+                        make_uint2(pack_pair(o[d][4 * q] * mul, o[d][4 * q + 1] * mul), pack_pair(o[d][4 * q + 2] * mul, o[d][4 * q + 3] * mul));
         }
 }
 
-template <int DT, int KSMAX>
+template <int DT, int KSMAX, bool EXACT>
 int launch_mfma(const MfmaParams &p, dim3 grid, size_t smem, hipStream_t st) {
-    static const hipError_t attr = hipFuncSetAttribute((const void *)latent_mfma_kernel<DT, KSMAX>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
+    static const hipError_t attr = hipFuncSetAttribute((const void *)latent_mfma_kernel<DT, KSMAX, EXACT>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
     XFT_CHECK_HIP(attr);
-    hipLaunchKernelGGL((latent_mfma_kernel<DT, KSMAX>), grid, dim3(256), smem, st, p);
+    hipLaunchKernelGGL((latent_mfma_kernel<DT, KSMAX, EXACT>), grid, dim3(256), smem, st, p);
     XFT_CHECK_HIP(hipGetLastError());
     return 0;
 }
-template <int KSM, int VTM>
+template <int KSM, int VTM, bool EXACT>
 int launch_expanded(const ExpandedParams &p, dim3 grid, size_t smem, hipStream_t st) {
-    static const hipError_t attr = hipFuncSetAttribute((const void *)latent_expanded_kernel<KSM, VTM>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
+    static const hipError_t attr = hipFuncSetAttribute((const void *)latent_expanded_kernel<KSM, VTM, EXACT>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
     XFT_CHECK_HIP(attr);
-    hipLaunchKernelGGL((latent_expanded_kernel<KSM, VTM>), grid, dim3(256), smem, st, p);
+    hipLaunchKernelGGL((latent_expanded_kernel<KSM, VTM, EXACT>), grid, dim3(256), smem, st, p);
     XFT_CHECK_HIP(hipGetLastError());
     return 0;
 }
@@ -578,10 +637,15 @@ bool mfma_takes(const PlanLayer &L) {
 int latent_prepare(int act, const PlanLayer &L, const StepView &v, const void *a, void *cq, const LatentCacheView &cache, float eps, hipStream_t st) {
     const PrepareParams p = {v, a, cq, cache, L.q_norm, L.kv_norm, L.cosT, L.sinT, L.QR, L.RD, L.s.q_rank, L.s.kv_rank, L.s.rot_dim,
             L.s.rot_interleaved, eps};
-    if (act == XFTHIP_BF16)
-        hipLaunchKernelGGL(latent_prepare_kernel<true>, dim3(v.T), dim3(256), 0, st, p);
-    else
-        hipLaunchKernelGGL(latent_prepare_kernel<false>, dim3(v.T), dim3(256), 0, st, p);
+    const int ch = (L.QR + L.R + 2047) / 2048;
+    XFT_REQUIRE(ch <= 4, "latent_prepare: latents of %d + %d values too wide", L.QR, L.R);
+    if (act == XFTHIP_BF16) {
+        if (ch == 1) hipLaunchKernelGGL((latent_prepare_kernel<true, 1>), dim3(v.T), dim3(256), 0, st, p);
+        else hipLaunchKernelGGL((latent_prepare_kernel<true, 4>), dim3(v.T), dim3(256), 0, st, p);
+    } else {
+        if (ch == 1) hipLaunchKernelGGL((latent_prepare_kernel<false, 1>), dim3(v.T), dim3(256), 0, st, p);
+        else hipLaunchKernelGGL((latent_prepare_kernel<false, 4>), dim3(v.T), dim3(256), 0, st, p);
+    }
     XFT_CHECK_HIP(hipGetLastError());
     return 0;
 }
@@ -604,8 +668,10 @@ int latent_split_count(const PlanLayer &L, int B, int longest, int hint) {
     const long units = (long)B * ((longest * L.s.heads + 31) / 32);
     const int ctx = L.s.window > 0 && L.s.window + longest < hint ? L.s.window + longest : hint;
     const int blocks = (ctx + 31) / 32;
-    const long want = device_cu_count() / units;
-    return (int)(want < 1 ? 1 : (want < blocks ? want : (blocks < 1 ? 1 : blocks)));
+    long want = device_cu_count() / units;
+    want = want < blocks ? want : blocks;
+    want = want < kMaxSplits / 2 ? want : kMaxSplits / 2; // (more parts cost more in the merge than they save)
+    return want < 1 ? 1 : (int)want;
 }
 
 size_t latent_part_floats(const PlanLayer &L) { return mfma_takes(L) ? (size_t)device_cu_count() * 32 * (L.R + 2) : 0; }
@@ -623,11 +689,17 @@ int latent_attention(int act, const PlanLayer &L, const StepView &v, int longest
         const size_t smem = (size_t)2 * 32 * ((L.R + L.RD) * 2 + 16) + 32 * 36 * 4;
         const int ks = (L.R + L.RD) / 32;
         int rc;
-        if (L.R <= 64 && ks <= 6) rc = launch_mfma<1, 6>(p, grid, smem, st);
-        else if (L.R <= 128 && ks <= 8) rc = launch_mfma<2, 8>(p, grid, smem, st);
-        else if (L.R <= 256 && ks <= 12) rc = launch_mfma<4, 12>(p, grid, smem, st);
-        else if (ks <= 18) rc = launch_mfma<8, 18>(p, grid, smem, st);
-        else rc = launch_mfma<8, 20>(p, grid, smem, st);
+        if (L.R == 512 && ks == 18) rc = launch_mfma<8, 18, true>(p, grid, smem, st);
+        else if (L.R == 512 && ks == 17) rc = launch_mfma<8, 17, true>(p, grid, smem, st);
+        else if (L.R == 256 && ks == 10) rc = launch_mfma<4, 10, true>(p, grid, smem, st);
+        else if (L.R == 256 && ks == 9) rc = launch_mfma<4, 9, true>(p, grid, smem, st);
+        else if (L.R == 128 && ks == 6) rc = launch_mfma<2, 6, true>(p, grid, smem, st);
+        else if (L.R == 128 && ks == 5) rc = launch_mfma<2, 5, true>(p, grid, smem, st);
+        else if (L.R == 64 && ks == 3) rc = launch_mfma<1, 3, true>(p, grid, smem, st);
+        else if (L.R <= 64 && ks <= 6) rc = launch_mfma<1, 6, false>(p, grid, smem, st);
+        else if (L.R <= 128 && ks <= 8) rc = launch_mfma<2, 8, false>(p, grid, smem, st);
+        else if (L.R <= 256 && ks <= 12) rc = launch_mfma<4, 12, false>(p, grid, smem, st);
+        else rc = launch_mfma<8, 20, false>(p, grid, smem, st);
         if (rc || p.nsplit == 1) return rc;
         hipLaunchKernelGGL(latent_merge_kernel, dim3(groups, v.B, 32), dim3(128), 0, st, p);
         XFT_CHECK_HIP(hipGetLastError());
@@ -664,9 +736,14 @@ int latent_expanded(const PlanLayer &L, int off, int start, int n, int base, con
     const dim3 grid(L.s.heads, (n + 127) / 128);
     const size_t smem = (size_t)2 * 32 * ((L.D + L.RD) * 2 + 16 + L.V * 2 + 16);
     const int ks = (L.D + L.RD) / 16, vt = L.V / 32;
-    if (ks <= 4 && vt <= 2) return launch_expanded<4, 2>(p, grid, smem, st);
-    if (ks <= 8 && vt <= 4) return launch_expanded<8, 4>(p, grid, smem, st);
-    return launch_expanded<12, 4>(p, grid, smem, st);
+    if (ks == 12 && vt == 4) return launch_expanded<12, 4, true>(p, grid, smem, st);
+    if (ks == 10 && vt == 4) return launch_expanded<10, 4, true>(p, grid, smem, st);
+    if (ks == 8 && vt == 4) return launch_expanded<8, 4, true>(p, grid, smem, st);
+    if (ks == 6 && vt == 2) return launch_expanded<6, 2, true>(p, grid, smem, st);
+    if (ks == 4 && vt == 1) return launch_expanded<4, 1, true>(p, grid, smem, st);
+    if (ks <= 4 && vt <= 2) return launch_expanded<4, 2, false>(p, grid, smem, st);
+    if (ks <= 8 && vt <= 4) return launch_expanded<8, 4, false>(p, grid, smem, st);
+    return launch_expanded<12, 4, false>(p, grid, smem, st);
 }
 
 } // namespace xfthip

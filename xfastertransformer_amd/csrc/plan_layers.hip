@@ -25,25 +25,29 @@ struct NormParams {
     float eps;
 };
 
-__device__ inline float block_sum_256(float v, float *part) {
+template <int NT>
+__device__ inline float block_sum(float v, float *part) {
 #pragma unroll
     for (int off = 32; off > 0; off >>= 1) v += __shfl_xor(v, off, 64);
     if ((threadIdx.x & 63) == 0) part[threadIdx.x >> 6] = v;
     __syncthreads();
-    return (part[0] + part[1]) + (part[2] + part[3]);
+    float s = 0.0f;
+#pragma unroll
+    for (int w = 0; w < NT / 64; ++w) s += part[w];
+    return s;
 }
 
-// one token a workgroup; the row stays in registers (CH float4 a thread), every load is requested before the first use
-template <bool BF16, int CH>
-__global__ __launch_bounds__(256) void plan_norm_kernel(NormParams p) {
-    __shared__ float part[8];
+// one token a workgroup of NT threads; the row stays in registers (CH float4 a thread), every load is requested before the first use
+template <bool BF16, int CH, int NT>
+__global__ __launch_bounds__(NT) void plan_norm_kernel(NormParams p) {
+    __shared__ float part[2 * NT / 64];
     const int t = blockIdx.x;
     const float *xr = p.x + (size_t)(p.rows ? p.rows[t] : t) * p.hidden;
     f32x4 x[CH], y[CH], wpost[CH], wpre[CH];
     const f32x4 zero = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
     for (int c = 0; c < CH; ++c) {
-        const int col = (c * 256 + threadIdx.x) * 4;
+        const int col = (c * NT + threadIdx.x) * 4;
         const bool in = col < p.hidden;
         x[c] = in ? *(const f32x4 *)(xr + col) : zero;
         y[c] = in && p.y ? *(const f32x4 *)(p.y + (size_t)t * p.hidden + col) : zero;
@@ -59,10 +63,10 @@ __global__ __launch_bounds__(256) void plan_norm_kernel(NormParams p) {
         for (int c = 0; c < CH; ++c)
 #pragma unroll
             for (int i = 0; i < 4; ++i) sq = fmaf(y[c][i], y[c][i], sq);
-        const float r = p.y ? 1.0f / sqrtf(block_sum_256(sq, part) / (float)p.width + p.eps) : 0.0f;
+        const float r = p.y ? 1.0f / sqrtf(block_sum<NT>(sq, part) / (float)p.width + p.eps) : 0.0f;
 #pragma unroll
         for (int c = 0; c < CH; ++c) {
-            const int col = (c * 256 + threadIdx.x) * 4;
+            const int col = (c * NT + threadIdx.x) * 4;
             if (col >= p.hidden) continue;
             const uint2 e = *(const uint2 *)(row + col);
             const f32x4 emb = {u2f(e.x << 16), u2f(e.x & 0xFFFF0000u), u2f(e.y << 16), u2f(e.y & 0xFFFF0000u)};
@@ -74,14 +78,14 @@ __global__ __launch_bounds__(256) void plan_norm_kernel(NormParams p) {
         for (int c = 0; c < CH; ++c)
 #pragma unroll
             for (int i = 0; i < 4; ++i) sq = fmaf(y[c][i], y[c][i], sq);
-        const float r = 1.0f / sqrtf(block_sum_256(sq, part) / (float)p.width + p.eps);
+        const float r = 1.0f / sqrtf(block_sum<NT>(sq, part) / (float)p.width + p.eps);
 #pragma unroll
         for (int c = 0; c < CH; ++c) x[c] = x[c] + y[c] * r * wpost[c];
     }
     if (p.y || p.table) {
 #pragma unroll
         for (int c = 0; c < CH; ++c) {
-            const int col = (c * 256 + threadIdx.x) * 4;
+            const int col = (c * NT + threadIdx.x) * 4;
             if (col < p.hidden) *(f32x4 *)(p.x + (size_t)t * p.hidden + col) = x[c];
         }
     }
@@ -91,10 +95,10 @@ __global__ __launch_bounds__(256) void plan_norm_kernel(NormParams p) {
     for (int c = 0; c < CH; ++c)
 #pragma unroll
         for (int i = 0; i < 4; ++i) sq = fmaf(x[c][i], x[c][i], sq);
-    const float r = 1.0f / sqrtf(block_sum_256(sq, part + 4) / (float)p.width + p.eps);
+    const float r = 1.0f / sqrtf(block_sum<NT>(sq, part + NT / 64) / (float)p.width + p.eps);
 #pragma unroll
     for (int c = 0; c < CH; ++c) {
-        const int col = (c * 256 + threadIdx.x) * 4;
+        const int col = (c * NT + threadIdx.x) * 4;
         if (col >= p.hidden) continue;
         const f32x4 v = x[c] * r * wpre[c];
         const size_t at = (size_t)t * p.hidden + col;
@@ -110,11 +114,15 @@ template <bool BF16>
 int launch_norm(const NormParams &p, int T, hipStream_t st) {
     const int ch = (p.hidden + 1023) / 1024;
     XFT_REQUIRE(ch <= 16, "plan_norm: hidden size %d above 16384", p.hidden);
-    if (ch <= 1) hipLaunchKernelGGL((plan_norm_kernel<BF16, 1>), dim3(T), dim3(256), 0, st, p);
-    else if (ch <= 2) hipLaunchKernelGGL((plan_norm_kernel<BF16, 2>), dim3(T), dim3(256), 0, st, p);
-    else if (ch <= 4) hipLaunchKernelGGL((plan_norm_kernel<BF16, 4>), dim3(T), dim3(256), 0, st, p);
-    else if (ch <= 8) hipLaunchKernelGGL((plan_norm_kernel<BF16, 8>), dim3(T), dim3(256), 0, st, p);
-    else hipLaunchKernelGGL((plan_norm_kernel<BF16, 16>), dim3(T), dim3(256), 0, st, p);
+    // few rows: the kernel is one chain of latencies, shorter with the row spread over more threads
+    if (T <= 64 && ch > 1) {
+        if (ch <= 4) hipLaunchKernelGGL((plan_norm_kernel<BF16, 1, 1024>), dim3(T), dim3(1024), 0, st, p);
+        else hipLaunchKernelGGL((plan_norm_kernel<BF16, 4, 1024>), dim3(T), dim3(1024), 0, st, p);
+    } else if (ch <= 1) hipLaunchKernelGGL((plan_norm_kernel<BF16, 1, 256>), dim3(T), dim3(256), 0, st, p);
+    else if (ch <= 2) hipLaunchKernelGGL((plan_norm_kernel<BF16, 2, 256>), dim3(T), dim3(256), 0, st, p);
+    else if (ch <= 4) hipLaunchKernelGGL((plan_norm_kernel<BF16, 4, 256>), dim3(T), dim3(256), 0, st, p);
+    else if (ch <= 8) hipLaunchKernelGGL((plan_norm_kernel<BF16, 8, 256>), dim3(T), dim3(256), 0, st, p);
+    else hipLaunchKernelGGL((plan_norm_kernel<BF16, 16, 256>), dim3(T), dim3(256), 0, st, p);
     XFT_CHECK_HIP(hipGetLastError());
     return 0;
 }
