@@ -11,8 +11,7 @@ import numpy as np
 
 from . import capi  # loads libxft_hip.so (RTLD_GLOBAL) or raises
 
-_HERE = os.path.dirname(os.path.abspath(__file__))
-_LIB_PATH = os.path.join(_HERE, "libxft_layers.so")
+_LIB_PATH = os.path.join(capi.LIB_DIR, "libxft_layers.so")
 if not os.path.exists(_LIB_PATH):
     raise ImportError(f"{_LIB_PATH} is not built; run `python -m xfastertransformer_amd.build`")
 _lib = C.CDLL(_LIB_PATH)

@@ -34,8 +34,12 @@ def _stale(target, sources):
     return any(os.path.getmtime(s) > t for s in sources)
 
 
-def build_hip(force=True):
-    srcs = sorted(glob.glob(os.path.join(CSRC, "*.hip")))
+# what only models with quantised weights need (most of the compile time)
+QUANTISED = {"qgemm_%s_%s.hip" % (k, w) for k in ("skinny", "mfma") for w in ("int8", "int8z", "uint4", "nf4")}
+
+
+def build_hip(force=True, target=LIB_HIP, leave_out=()):
+    srcs = [s for s in sorted(glob.glob(os.path.join(CSRC, "*.hip"))) if os.path.basename(s) not in leave_out]
     deps = srcs + glob.glob(os.path.join(CSRC, "*.h")) + glob.glob(os.path.join(ROOT, "include", "*.h"))
     objdir = os.path.join(CSRC, "build")
     os.makedirs(objdir, exist_ok=True)
@@ -71,19 +75,20 @@ def build_hip(force=True):
         reap(running.pop(0))
     if failed:
         raise RuntimeError("hipcc failed")
-    if force or built or _stale(LIB_HIP, objs):
-        _run([HIPCC, "--offload-arch=gfx950", "-shared", "-fPIC", "-o", LIB_HIP] + objs)
-    return LIB_HIP
+    if force or built or _stale(target, objs):
+        os.makedirs(os.path.dirname(target), exist_ok=True)
+        _run([HIPCC, "--offload-arch=gfx950", "-shared", "-fPIC", "-o", target] + objs)
+    return target
 
 
-def build_host(force=True):
+def build_host(force=True, target=LIB_LAYERS, lib_hip=LIB_HIP):
     """The C++ host layer (xft::invoke* entry points, xft::AutoModel) over the C-ABI; plain g++, no HIP headers."""
     srcs = sorted(glob.glob(os.path.join(CSRC, "host", "*.cpp")))
-    deps = srcs + glob.glob(os.path.join(CSRC, "host", "*.h")) + glob.glob(os.path.join(ROOT, "include", "*.h")) + [LIB_HIP]
-    if force or _stale(LIB_LAYERS, deps):
-        _run([os.environ.get("CXX", "g++"), "-O2", "-std=c++17", "-fPIC", "-shared", "-Wall"] + srcs + ["-o", LIB_LAYERS,
-              "-L" + HERE, "-lxft_hip", "-Wl,-rpath,$ORIGIN"])
-    return LIB_LAYERS
+    deps = srcs + glob.glob(os.path.join(CSRC, "host", "*.h")) + glob.glob(os.path.join(ROOT, "include", "*.h")) + [lib_hip]
+    if force or _stale(target, deps):
+        _run([os.environ.get("CXX", "g++"), "-O2", "-std=c++17", "-fPIC", "-shared", "-Wall"] + srcs + ["-o", target,
+              "-L" + os.path.dirname(lib_hip), "-lxft_hip", "-Wl,-rpath,$ORIGIN"])
+    return target
 
 
 def build_torch(force=True):
@@ -118,11 +123,14 @@ def build_test_drivers(force=True):
 
 
 def use_or_build_plan_libraries():
-    """For programs that may run in a checkout nothing was built in: leaves a built checkout alone."""
-    if os.path.exists(LIB_HIP) and os.path.exists(LIB_LAYERS):
+    """For programs that may run in a checkout nothing was built in: leaves a built checkout alone, else builds what models
+    with BF16 weights need, in a folder of its own, and has the package load that (XFT_LIB_DIR).  Call before importing capi."""
+    if os.environ.get("XFT_LIB_DIR") or (os.path.exists(LIB_HIP) and os.path.exists(LIB_LAYERS)):
         return
-    build_hip(False)
-    build_host(False)
+    folder = os.path.join(CSRC, "build", "bf16")
+    lib_hip = build_hip(False, os.path.join(folder, "libxft_hip.so"), QUANTISED)
+    build_host(False, os.path.join(folder, "libxft_layers.so"), lib_hip)
+    os.environ["XFT_LIB_DIR"] = folder
 
 
 def build_all(force=True):

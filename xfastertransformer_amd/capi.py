@@ -5,7 +5,8 @@ import os
 import numpy as np
 
 _HERE = os.path.dirname(os.path.abspath(__file__))
-LIB_PATH = os.path.join(_HERE, "libxft_hip.so")
+LIB_DIR = os.environ.get("XFT_LIB_DIR") or _HERE
+LIB_PATH = os.path.join(LIB_DIR, "libxft_hip.so")
 
 F32, BF16, FP16, INT8 = 0, 1, 2, 3
 W_INT8, W_UINT4, W_NF4, W_W8A8, W_BF16 = 0, 1, 2, 3, 4

@@ -8,10 +8,11 @@
 
 namespace xfthip {
 
-int qgemm_mfma_int8(const SkinnyParams &p, hipStream_t stream);
-int qgemm_mfma_int8z(const SkinnyParams &p, hipStream_t stream);
-int qgemm_mfma_uint4(const SkinnyParams &p, hipStream_t stream);
-int qgemm_mfma_nf4(const SkinnyParams &p, hipStream_t stream);
+// weak: a library for models with BF16 weights only is built without the quantised kinds (build.py)
+__attribute__((weak)) int qgemm_mfma_int8(const SkinnyParams &p, hipStream_t stream);
+__attribute__((weak)) int qgemm_mfma_int8z(const SkinnyParams &p, hipStream_t stream);
+__attribute__((weak)) int qgemm_mfma_uint4(const SkinnyParams &p, hipStream_t stream);
+__attribute__((weak)) int qgemm_mfma_nf4(const SkinnyParams &p, hipStream_t stream);
 int qgemm_mfma_bf16(const SkinnyParams &p, hipStream_t stream);
 
 namespace {
@@ -173,14 +174,16 @@ int qgemm_mfma(const PackedWeight &pw, const SkinnyParams &p0, hipStream_t strea
         else if (int rc = qgemm_split_reserve(stream, &p.split_part)) return rc;
     }
     if (p.ksplit <= 1) p.ksplit = 0;
-    int rc;
+    int (*kernel)(const SkinnyParams &, hipStream_t) = nullptr;
     switch (pw.kind) {
-        case XFTHIP_W_INT8: rc = p.zero ? qgemm_mfma_int8z(p, stream) : qgemm_mfma_int8(p, stream); break;
-        case XFTHIP_W_UINT4: rc = qgemm_mfma_uint4(p, stream); break;
-        case XFTHIP_W_NF4: rc = qgemm_mfma_nf4(p, stream); break;
-        case XFTHIP_W_BF16: rc = qgemm_mfma_bf16(p, stream); break;
+        case XFTHIP_W_INT8: kernel = p.zero ? qgemm_mfma_int8z : qgemm_mfma_int8; break;
+        case XFTHIP_W_UINT4: kernel = qgemm_mfma_uint4; break;
+        case XFTHIP_W_NF4: kernel = qgemm_mfma_nf4; break;
+        case XFTHIP_W_BF16: kernel = qgemm_mfma_bf16; break;
         default: set_error("qgemm_mfma: weight kind %d not supported", pw.kind); return 2;
     }
+    XFT_REQUIRE(kernel, "qgemm_mfma: this library was built for BF16 weights only");
+    const int rc = kernel(p, stream);
     if (rc || p.ksplit <= 1) return rc;
     const size_t outs = (size_t)p.M * p.N;
     if (p.N % 4 == 0) // the parts are [M][N] fp32 in a 256-byte aligned buffer: 16-byte loads need only N % 4 == 0

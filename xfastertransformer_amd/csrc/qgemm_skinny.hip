@@ -6,9 +6,10 @@
 
 namespace xfthip {
 
-int qgemm_skinny_int8(const SkinnyParams &p, hipStream_t stream);
-int qgemm_skinny_uint4(const SkinnyParams &p, hipStream_t stream);
-int qgemm_skinny_nf4(const SkinnyParams &p, hipStream_t stream);
+// weak: a library for models with BF16 weights only is built without the quantised kinds (build.py)
+__attribute__((weak)) int qgemm_skinny_int8(const SkinnyParams &p, hipStream_t stream);
+__attribute__((weak)) int qgemm_skinny_uint4(const SkinnyParams &p, hipStream_t stream);
+__attribute__((weak)) int qgemm_skinny_nf4(const SkinnyParams &p, hipStream_t stream);
 int qgemm_skinny_bf16(const SkinnyParams &p, hipStream_t stream);
 
 // LDS of the RMSNorm prologue: M rows of K + 8 bf16 values
@@ -45,13 +46,16 @@ int qgemm_skinny(const PackedWeight &pw, const SkinnyParams &p0, hipStream_t str
     p.NTILES = pw.NTILES;
     p.K = pw.K;
     p.N = pw.N;
+    int (*quantised)(const SkinnyParams &, hipStream_t) = nullptr;
     switch (pw.kind) {
-        case XFTHIP_W_INT8: return qgemm_skinny_int8(p, stream);
-        case XFTHIP_W_UINT4: return qgemm_skinny_uint4(p, stream);
-        case XFTHIP_W_NF4: return qgemm_skinny_nf4(p, stream);
+        case XFTHIP_W_INT8: quantised = qgemm_skinny_int8; break;
+        case XFTHIP_W_UINT4: quantised = qgemm_skinny_uint4; break;
+        case XFTHIP_W_NF4: quantised = qgemm_skinny_nf4; break;
         case XFTHIP_W_BF16: return qgemm_skinny_bf16(p, stream);
         default: set_error("qgemm_skinny: weight kind %d not supported", pw.kind); return 2;
     }
+    XFT_REQUIRE(quantised, "qgemm_skinny: this library was built for BF16 weights only");
+    return quantised(p, stream);
 }
 
 } // namespace xfthip
