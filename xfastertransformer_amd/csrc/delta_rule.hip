@@ -282,7 +282,10 @@ __device__ inline float group_sum(float v) {
     v = dpp_add<0x4E>(v); // quad_perm 2 3 0 1
     if constexpr (L >= 8) v = dpp_add<0x141>(v); // row_half_mirror
     if constexpr (L >= 16) v = dpp_add<0x140>(v); // row_mirror
-    if constexpr (L >= 32) v += __shfl_xor(v, 16, 64);
+    if constexpr (L >= 32) { // rows of 16 lanes change places in pairs
+        const auto r = __builtin_amdgcn_permlane16_swap(__builtin_bit_cast(unsigned, v), __builtin_bit_cast(unsigned, v), false, false);
+        v = __builtin_bit_cast(float, r[0]) + __builtin_bit_cast(float, r[1]);
+    }
     return v;
 }
 
@@ -292,27 +295,33 @@ struct ScanParams {
     int H, KH, VD;
 };
 
-// The state's columns (value channels) do not interact: a column is held by L = KD / 8 lanes, 8 key rows each.  With
-// S' = g S the step is a = S'^T k, b = S'^T q, u = beta (v - a), S = S' + k u^T, o = b + (q . k) u: both sums over the key
+// The state's columns (value channels) do not interact.  L lanes hold C neighbouring columns, 4 RV key rows each (KD = 4 L RV).
+// With S' = g S the step is a = S'^T k, b = S'^T q, u = beta (v - a), S = S' + k u^T, o = b + (q . k) u: both sums over the key
 // rows run side by side and the read-out needs none of its own.  q, k, g of CT tokens are staged in LDS, the next CT on
-// their way through registers.  grid (segments, heads, column groups of 256 / L).
-template <int L>
+// their way through registers.  grid (segments, heads, column groups of COLS).
+// One prompt of 32 heads is one wave a SIMD: the time is about 75 vector instructions a token and the latency of the
+// reductions in them.  (KD = 128 as 32 lanes x 4 rows x 2 columns, half the LDS reads: 510 us for 2048 tokens against 440 as
+// 16 x 8 x 1.)
+template <int L, int RV, int C>
 __global__ __launch_bounds__(256) void delta_scan_kernel(ScanParams p) {
-    constexpr int KD = 8 * L, COLS = 256 / L, CT = L == 32 ? 8 : 16; // CT: tokens staged in LDS at a time
+    constexpr int KD = 4 * L * RV, GROUPS = 256 / L, COLS = GROUPS * C, CT = KD > 128 ? 8 : 16;
     constexpr int CHUNK4 = CT * KD / 4; // float4 of one array and chunk
     constexpr int PER = (3 * CHUNK4 + 255) / 256, PERV = (CT * COLS + 255) / 256;
     __shared__ float lds[2][3 * CT * KD];
     __shared__ float vlds[2][CT * COLS];
     __shared__ float sc[2][2 * CT];
-    __shared__ float olds[CT * COLS];
+    __shared__ float olds[2][CT * COLS];
     const int seg = blockIdx.x, head = blockIdx.y, kvh = head / (p.H / p.KH);
     const int n = p.v.seg_len[seg], off = p.v.seg_off[seg];
-    const int li = threadIdx.x % L, lc = threadIdx.x / L;
+    const int li = threadIdx.x % L, lc = threadIdx.x / L * C;
     const int col0 = blockIdx.z * COLS, col = col0 + lc;
-    const bool own = col < p.VD;
-    float *state = p.b.state + (((size_t)p.v.seg_row[seg] * p.H + head) * p.VD + (own ? col : 0)) * KD;
-    f32x4 s0 = {0.f, 0.f, 0.f, 0.f}, s1 = s0;
-    if (p.v.seg_pos[seg] > 0) s0 = *(const f32x4 *)(state + 4 * li), s1 = *(const f32x4 *)(state + 4 * (L + li));
+    const bool own = col < p.VD; // (VD is a multiple of 32: C neighbouring columns are in it or not together)
+    float *state = p.b.state + (((size_t)p.v.seg_row[seg] * p.H + head) * p.VD + (own ? col : 0)) * KD + 4 * li;
+    f32x4 s[C][RV];
+#pragma unroll
+    for (int c = 0; c < C; ++c)
+#pragma unroll
+        for (int r = 0; r < RV; ++r) s[c][r] = p.v.seg_pos[seg] > 0 ? *(const f32x4 *)(state + c * KD + r * 4 * L) : f32x4 {0.f, 0.f, 0.f, 0.f};
 
     f32x4 stage[PER];
     float vstage[PERV], cstage = 0.0f;
@@ -360,28 +369,47 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(ScanParams p) {
         if (c0 + CT < n) fetch(c0 + CT);
         const float *lq = lds[buf] + 4 * li;
         struct Operands {
-            f32x4 q0, q1, k0, k1, g0, g1;
-            float v, beta, qk;
+            f32x4 q[RV], k[RV], g[RV];
+            float v[C], beta, qk;
         };
         auto read = [&](int i) {
             const float *q = lq + i * KD, *k = q + CT * KD, *g = k + CT * KD;
-            return Operands {*(const f32x4 *)q, *(const f32x4 *)(q + 4 * L), *(const f32x4 *)k, *(const f32x4 *)(k + 4 * L), *(const f32x4 *)g,
-                    *(const f32x4 *)(g + 4 * L), vlds[buf][i * COLS + lc], sc[buf][i], sc[buf][CT + i]};
+            Operands x;
+#pragma unroll
+            for (int r = 0; r < RV; ++r) x.q[r] = *(const f32x4 *)(q + r * 4 * L), x.k[r] = *(const f32x4 *)(k + r * 4 * L), x.g[r] = *(const f32x4 *)(g + r * 4 * L);
+#pragma unroll
+            for (int c = 0; c < C; ++c) x.v[c] = vlds[buf][i * COLS + lc + c];
+            x.beta = sc[buf][i], x.qk = sc[buf][CT + i];
+            return x;
         };
         // the operands of the next token are on their way from LDS while this one's sums go round
         auto token = [&](const Operands &x, int i) {
-            float a0 = 0.0f, a1 = 0.0f, b0 = 0.0f, b1 = 0.0f;
+            float a[C], b[C], u[C];
 #pragma unroll
-            for (int r = 0; r < 4; ++r) {
-                s0[r] *= x.g0[r], s1[r] *= x.g1[r];
-                a0 = fmaf(x.k0[r], s0[r], a0), b0 = fmaf(x.q0[r], s0[r], b0);
-                a1 = fmaf(x.k1[r], s1[r], a1), b1 = fmaf(x.q1[r], s1[r], b1);
+            for (int c = 0; c < C; ++c) {
+                a[c] = b[c] = 0.0f;
+#pragma unroll
+                for (int r = 0; r < RV; ++r)
+#pragma unroll
+                    for (int e = 0; e < 4; ++e) {
+                        s[c][r][e] *= x.g[r][e];
+                        a[c] = fmaf(x.k[r][e], s[c][r][e], a[c]), b[c] = fmaf(x.q[r][e], s[c][r][e], b[c]);
+                    }
             }
-            const float a = group_sum<L>(a0 + a1), b = group_sum<L>(b0 + b1);
-            const float u = x.beta * (x.v - a);
 #pragma unroll
-            for (int r = 0; r < 4; ++r) s0[r] = fmaf(x.k0[r], u, s0[r]), s1[r] = fmaf(x.k1[r], u, s1[r]);
-            if (li == 0) olds[i * COLS + lc] = fmaf(x.qk, u, b);
+            for (int c = 0; c < C; ++c) a[c] = group_sum<L>(a[c]), b[c] = group_sum<L>(b[c]);
+#pragma unroll
+            for (int c = 0; c < C; ++c) {
+                u[c] = x.beta * (x.v[c] - a[c]);
+#pragma unroll
+                for (int r = 0; r < RV; ++r)
+#pragma unroll
+                    for (int e = 0; e < 4; ++e) s[c][r][e] = fmaf(x.k[r][e], u[c], s[c][r][e]);
+            }
+            if (li == 0) {
+#pragma unroll
+                for (int c = 0; c < C; ++c) olds[buf][i * COLS + lc + c] = fmaf(x.qk, u[c], b[c]);
+            }
         };
         Operands even = read(0), odd;
         for (int i = 0; i < m; i += 2) {
@@ -391,15 +419,19 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(ScanParams p) {
             even = read(i + 2 < m ? i + 2 : i + 1);
             token(odd, i + 1);
         }
-        if (c0 + CT < n) stash(buf ^ 1); // (the other buffer was last read before the barrier below, one chunk ago)
+        if (c0 + CT < n) stash(buf ^ 1); // (the other buffer, and the other results, were last read before or behind this barrier one chunk ago)
         __syncthreads();
         for (int e = threadIdx.x; e < m * COLS; e += 256) {
             const int c = col0 + e % COLS;
-            if (c < p.VD) p.b.o[((size_t)(off + c0 + e / COLS) * p.H + head) * p.VD + c] = olds[e];
+            if (c < p.VD) p.b.o[((size_t)(off + c0 + e / COLS) * p.H + head) * p.VD + c] = olds[buf][e];
         }
-        __syncthreads();
     }
-    if (own) *(f32x4 *)(state + 4 * li) = s0, *(f32x4 *)(state + 4 * (L + li)) = s1;
+    if (own) {
+#pragma unroll
+        for (int c = 0; c < C; ++c)
+#pragma unroll
+            for (int r = 0; r < RV; ++r) *(f32x4 *)(state + c * KD + r * 4 * L) = s[c][r];
+    }
 }
 
 // The same step for segments of one token: nothing to stage, the kernel is a read and a write of the state.
@@ -523,11 +555,12 @@ int delta_scan(const PlanLayer &L, const StepView &v, const DeltaBuffers &b, hip
         XFT_CHECK_HIP(hipGetLastError());
         return 0;
     }
-    switch (lanes) {
-        case 4: hipLaunchKernelGGL(delta_scan_kernel<4>, grid, dim3(256), 0, st, p); break;
-        case 8: hipLaunchKernelGGL(delta_scan_kernel<8>, grid, dim3(256), 0, st, p); break;
-        case 16: hipLaunchKernelGGL(delta_scan_kernel<16>, grid, dim3(256), 0, st, p); break;
-        case 32: hipLaunchKernelGGL(delta_scan_kernel<32>, grid, dim3(256), 0, st, p); break;
+    auto columns = [&](int per_workgroup) { return dim3(v.B, p.H, (L.VD + per_workgroup - 1) / per_workgroup); };
+    switch (L.KD) {
+        case 32: hipLaunchKernelGGL((delta_scan_kernel<4, 2, 1>), columns(64), dim3(256), 0, st, p); break;
+        case 64: hipLaunchKernelGGL((delta_scan_kernel<8, 2, 1>), columns(32), dim3(256), 0, st, p); break;
+        case 128: hipLaunchKernelGGL((delta_scan_kernel<16, 2, 1>), columns(16), dim3(256), 0, st, p); break;
+        case 256: hipLaunchKernelGGL((delta_scan_kernel<32, 2, 1>), columns(8), dim3(256), 0, st, p); break;
         default: set_error("delta_scan: key dimension %d of a head is above 256", L.s.dim); return 2;
     }
     XFT_CHECK_HIP(hipGetLastError());

@@ -449,7 +449,7 @@ int xfthip_plan_create(const xfthip_plan_config *cfg, const xfthip_plan_layer *l
     XFT_REQUIRE(cfg && layers && out, "xfthip_plan_create: null argument");
     const xfthip_plan_config &c = *cfg;
     XFT_REQUIRE(c.layers > 0 && c.hidden > 0 && c.hidden <= 16384 && c.vocab > 0, "xfthip_plan_create: bad sizes");
-    const bool loop = c.loop_times > 1;
+    const bool loop = c.loop_times > 1 && c.loop_start != c.loop_stop; // (a loop over nothing is none)
     XFT_REQUIRE(!loop || (c.loop_start >= 0 && c.loop_start < c.loop_stop && c.loop_stop <= c.layers), "xfthip_plan_create: loop over layers %d .. %d of %d",
             c.loop_start, c.loop_stop, c.layers);
     xfthip_plan *p = new xfthip_plan();
