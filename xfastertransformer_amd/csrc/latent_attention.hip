@@ -22,6 +22,10 @@ __device__ inline float wave_largest(float v) {
     return v;
 }
 
+typedef __attribute__((ext_vector_type(2))) __bf16 bf16x2;
+// two values -> packed bf16 pair, round to nearest even (v_cvt_pk_bf16_f32)
+__device__ inline uint32_t pack_pair(float lo, float hi) { return __builtin_bit_cast(uint32_t, bf16x2 {(__bf16)lo, (__bf16)hi}); }
+
 template <bool BF16>
 __device__ inline float ldact(const void *p, size_t i) {
     if constexpr (BF16) return bf16_to_f32(((const uint16_t *)p)[i]);
@@ -66,7 +70,7 @@ __device__ inline void store8(void *p, size_t i, const float (&v)[8]) {
     if constexpr (BF16) {
         uint32_t w[4];
 #pragma unroll
-        for (int k = 0; k < 4; ++k) w[k] = f32_bits_to_bf16_sel(f2u(v[2 * k])) | (f32_bits_to_bf16_sel(f2u(v[2 * k + 1])) << 16);
+        for (int k = 0; k < 4; ++k) w[k] = pack_pair(v[2 * k], v[2 * k + 1]);
         *(uint4 *)((uint16_t *)p + i) = make_uint4(w[0], w[1], w[2], w[3]);
     } else {
         *(f32x4 *)((float *)p + i) = f32x4 {v[0], v[1], v[2], v[3]};
@@ -131,21 +135,56 @@ __global__ __launch_bounds__(256) void latent_prepare_kernel(PrepareParams p) {
     }
 }
 
-// one thread a rotated pair
+// One thread eight rotated values: four neighbouring pairs (interleaved), or four pairs of either half.
 template <bool BF16>
 __global__ __launch_bounds__(256) void rotate_q_kernel(StepView v, void *q, int T, int H, int D, int RD, int half, int interleaved, const float *cosT,
         const float *sinT) {
+    const int per = (half + 3) / 4;
     const size_t idx = (size_t)blockIdx.x * 256 + threadIdx.x;
-    if (idx >= (size_t)T * H * half) return;
-    const int i = (int)(idx % half);
-    const size_t th = idx / half;
+    if (idx >= (size_t)T * H * per) return;
+    const int i0 = (int)(idx % per) * 4;
+    const size_t th = idx / per;
     const int pos = v.tok_pos[th / H];
     const size_t at = th * (D + RD) + D;
-    const size_t iu = at + (interleaved ? 2 * i : i), iw = at + (interleaved ? 2 * i + 1 : i + half);
-    const float u = ldact<BF16>(q, iu), w = ldact<BF16>(q, iw);
-    const float cs = cosT[(size_t)pos * half + i], sn = sinT[(size_t)pos * half + i];
-    stact<BF16>(q, iu, fmaf(u, cs, -(w * sn)));
-    stact<BF16>(q, iw, fmaf(w, cs, u * sn));
+    const float *cs = cosT + (size_t)pos * half, *sn = sinT + (size_t)pos * half;
+    if ((half & 3) == 0) {
+        const f32x4 c = *(const f32x4 *)(cs + i0), s = *(const f32x4 *)(sn + i0);
+        if (interleaved) {
+            float x[8], y[8];
+            load8<BF16>(q, at + 2 * i0, x);
+#pragma unroll
+            for (int k = 0; k < 4; ++k) {
+                y[2 * k] = fmaf(x[2 * k], c[k], -(x[2 * k + 1] * s[k]));
+                y[2 * k + 1] = fmaf(x[2 * k + 1], c[k], x[2 * k] * s[k]);
+            }
+            store8<BF16>(q, at + 2 * i0, y);
+        } else {
+            f32x4 a, b;
+            if constexpr (BF16) {
+                const uint2 ua = *(const uint2 *)((const uint16_t *)q + at + i0), ub = *(const uint2 *)((const uint16_t *)q + at + half + i0);
+                a = f32x4 {u2f(ua.x << 16), u2f(ua.x & 0xFFFF0000u), u2f(ua.y << 16), u2f(ua.y & 0xFFFF0000u)};
+                b = f32x4 {u2f(ub.x << 16), u2f(ub.x & 0xFFFF0000u), u2f(ub.y << 16), u2f(ub.y & 0xFFFF0000u)};
+            } else {
+                a = *(const f32x4 *)((const float *)q + at + i0), b = *(const f32x4 *)((const float *)q + at + half + i0);
+            }
+            f32x4 ya, yb;
+#pragma unroll
+            for (int k = 0; k < 4; ++k) ya[k] = fmaf(a[k], c[k], -(b[k] * s[k])), yb[k] = fmaf(b[k], c[k], a[k] * s[k]);
+            if constexpr (BF16) {
+                *(uint2 *)((uint16_t *)q + at + i0) = make_uint2(pack_pair(ya[0], ya[1]), pack_pair(ya[2], ya[3]));
+                *(uint2 *)((uint16_t *)q + at + half + i0) = make_uint2(pack_pair(yb[0], yb[1]), pack_pair(yb[2], yb[3]));
+            } else {
+                *(f32x4 *)((float *)q + at + i0) = ya, *(f32x4 *)((float *)q + at + half + i0) = yb;
+            }
+        }
+        return;
+    }
+    for (int i = i0; i < i0 + 4 && i < half; ++i) {
+        const size_t iu = at + (interleaved ? 2 * i : i), iw = at + (interleaved ? 2 * i + 1 : i + half);
+        const float u = ldact<BF16>(q, iu), w = ldact<BF16>(q, iw);
+        stact<BF16>(q, iu, fmaf(u, cs[i], -(w * sn[i])));
+        stact<BF16>(q, iw, fmaf(w, cs[i], u * sn[i]));
+    }
 }
 
 struct AttendParams {
@@ -215,9 +254,6 @@ typedef __attribute__((ext_vector_type(8))) short s16x8;
 constexpr float kUnseen = -1.0e30f; // score of a masked key, maximum of a column that has seen none
 constexpr float kLog2e = 1.4426950408889634f;
 
-typedef __attribute__((ext_vector_type(2))) __bf16 bf16x2;
-// two values -> packed bf16 pair, round to nearest even (v_cvt_pk_bf16_f32)
-__device__ inline uint32_t pack_pair(float lo, float hi) { return __builtin_bit_cast(uint32_t, bf16x2 {(__bf16)lo, (__bf16)hi}); }
 __device__ inline bf16x8 pack_bf16x8(const float (&v)[8]) {
     u32x4 u;
 #pragma unroll
@@ -324,20 +360,27 @@ __global__ __launch_bounds__(256, 2) void latent_mfma_kernel(MfmaParams p) {
             if (EXACT || ks < ks_n) (ks & 1 ? s1 : s) = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*(const bf16x8 *)(krow + ks * 64), qf[ks], ks & 1 ? s1 : s, 0, 0, 0);
         *(f32x4 *)(sc + (16 * ct_s + i16) * 36 + 16 * tt + 4 * g) = s + s1;
         __syncthreads();
+        // a lane group takes tokens 4 g .. 4 g + 3 and 16 + 4 g .. of the block: the transposed reads below then touch eight
+        // neighbouring rows at a time, which the row pitch spreads over the banks
         bf16x8 pf[2];
         float alpha[2];
+        const bool open = blk * 32 + 31 <= lo && (p.a.window <= 0 || blk * 32 > hi - p.a.window); // every column sees the whole block
 #pragma unroll
         for (int ct = 0; ct < 2; ++ct) {
-            const float *row = sc + (16 * ct + i16) * 36 + 8 * g;
-            const f32x4 x0 = *(const f32x4 *)row, x1 = *(const f32x4 *)(row + 4);
+            const float *row = sc + (16 * ct + i16) * 36 + 4 * g;
+            const f32x4 x0 = *(const f32x4 *)row * scale2, x1 = *(const f32x4 *)(row + 16) * scale2;
             float x[8], bm = kUnseen;
 #pragma unroll
-            for (int j = 0; j < 8; ++j) {
-                const int t = blk * 32 + 8 * g + j;
-                const bool seen = t <= cpos[ct] && (p.a.window <= 0 || t > cpos[ct] - p.a.window);
-                x[j] = seen ? (j < 4 ? x0[j & 3] : x1[j & 3]) * scale2 : kUnseen;
-                bm = fmaxf(bm, x[j]);
+            for (int j = 0; j < 8; ++j) x[j] = j < 4 ? x0[j & 3] : x1[j & 3];
+            if (!open) {
+#pragma unroll
+                for (int j = 0; j < 8; ++j) {
+                    const int t = blk * 32 + 4 * g + (j & 3) + (j < 4 ? 0 : 16);
+                    x[j] = t <= cpos[ct] && (p.a.window <= 0 || t > cpos[ct] - p.a.window) ? x[j] : kUnseen;
+                }
             }
+#pragma unroll
+            for (int j = 0; j < 8; ++j) bm = fmaxf(bm, x[j]);
             bm = fmaxf(bm, __shfl_xor(bm, 16, 64));
             bm = fmaxf(bm, __shfl_xor(bm, 32, 64));
             const float m_new = fmaxf(m[ct], bm);
@@ -346,7 +389,9 @@ __global__ __launch_bounds__(256, 2) void latent_mfma_kernel(MfmaParams p) {
             float sum = 0.0f;
 #pragma unroll
             for (int j = 0; j < 8; ++j) {
-                x[j] = x[j] > 0.5f * kUnseen ? __builtin_amdgcn_exp2f(x[j] - m_new) : 0.0f;
+                // (a column that has seen no key has its reference point at the masked score)
+                const float e = __builtin_amdgcn_exp2f(x[j] - m_new);
+                x[j] = open || x[j] > 0.5f * kUnseen ? e : 0.0f;
                 sum += x[j];
             }
             l[ct] = l[ct] * alpha[ct] + sum;
@@ -356,12 +401,12 @@ __global__ __launch_bounds__(256, 2) void latent_mfma_kernel(MfmaParams p) {
 #pragma unroll
             for (int d = 0; d < DT; ++d) o[d][0] *= alpha[0], o[d][1] *= alpha[1];
         }
-        const unsigned char *vrow = kv + (8 * g + (i16 >> 2)) * pitch + 8 * (i16 & 3);
+        const unsigned char *vrow = kv + (4 * g + (i16 >> 2)) * pitch + 8 * (i16 & 3);
 #pragma unroll
         for (int d = 0; d < DT; ++d) {
             const int tile = wave * DT + d;
             if (EXACT || tile * 16 < R) {
-                const bf16x8 a = transposed_pair(vrow + tile * 32, vrow + tile * 32 + 4 * pitch);
+                const bf16x8 a = transposed_pair(vrow + tile * 32, vrow + tile * 32 + 16 * pitch);
                 o[d][0] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, pf[0], o[d][0], 0, 0, 0);
                 o[d][1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, pf[1], o[d][1], 0, 0, 0);
             }
@@ -653,7 +698,7 @@ int latent_prepare(int act, const PlanLayer &L, const StepView &v, const void *a
 int latent_rotate_q(int act, const PlanLayer &L, const StepView &v, void *q, hipStream_t st) {
     const int half = L.s.rot_dim / 2;
     if (half == 0) return 0;
-    const unsigned blocks = (unsigned)(((size_t)v.T * L.s.heads * half + 255) / 256);
+    const unsigned blocks = (unsigned)(((size_t)v.T * L.s.heads * ((half + 3) / 4) + 255) / 256);
     if (act == XFTHIP_BF16)
         hipLaunchKernelGGL(rotate_q_kernel<true>, dim3(blocks), dim3(256), 0, st, v, q, v.T, L.s.heads, L.D, L.RD, half, L.s.rot_interleaved, L.cosT, L.sinT);
     else
@@ -668,7 +713,7 @@ int latent_split_count(const PlanLayer &L, int B, int longest, int hint) {
     const long units = (long)B * ((longest * L.s.heads + 31) / 32);
     const int ctx = L.s.window > 0 && L.s.window + longest < hint ? L.s.window + longest : hint;
     const int blocks = (ctx + 31) / 32;
-    long want = device_cu_count() / units;
+    long want = device_cu_count() / units; // (two a compute unit: no faster, and twice the merge)
     want = want < blocks ? want : blocks;
     want = want < kMaxSplits / 2 ? want : kMaxSplits / 2; // (more parts cost more in the merge than they save)
     return want < 1 ? 1 : (int)want;
