@@ -282,10 +282,7 @@ __device__ inline float group_sum(float v) {
     v = dpp_add<0x4E>(v); // quad_perm 2 3 0 1
     if constexpr (L >= 8) v = dpp_add<0x141>(v); // row_half_mirror
     if constexpr (L >= 16) v = dpp_add<0x140>(v); // row_mirror
-    if constexpr (L >= 32) { // rows of 16 lanes change places in pairs
-        const auto r = __builtin_amdgcn_permlane16_swap(__builtin_bit_cast(unsigned, v), __builtin_bit_cast(unsigned, v), false, false);
-        v = __builtin_bit_cast(float, r[0]) + __builtin_bit_cast(float, r[1]);
-    }
+    if constexpr (L >= 32) v += __shfl_xor(v, 16, 64);
     return v;
 }
 
