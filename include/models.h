@@ -6,7 +6,7 @@
 //     auto out = model.finalize();
 // for Llama-family model directories (config.ini + .bin files as the reference's convert tools
 // write them, src/models/common_decoder.h:167-262, src/layers/decoder_block.h:205-343) on one
-// MI355X.  Served: greedy search, sampling (top-k / top-p / temperature), repetition penalty, stop
+// MI355X, and for directories with config.json + model.safetensors whose architecture the library knows (layer plans).  Served: greedy search, sampling (top-k / top-p / temperature), repetition penalty, stop
 // words, beam search, the sequence-id (continuous batching) interface in all nine set_input forms,
 // and forward() with the logits of the last or of every position.  Not served: prefix sharing
 // (setPrefix / unsetPrefix print a message and exit(-1), the reference's style for an unsupported

@@ -2,7 +2,8 @@
 src/xfastertransformer/automodel.py (from_pretrained / config / input / forward / generate / is_done /
 finalize with the same argument names and defaults), bound with ctypes to the C entry points of
 libxft_layers.so instead of a Torch custom class.  Token ids go in and come out as torch tensors
-when torch tensors are given, numpy arrays otherwise.  There is no CPU path: without the built
+when torch tensors are given, numpy arrays otherwise.  Directories with config.json + model.safetensors (layer plans) load the
+same way, in bf16 or fp32, and also take steps of unequal parts (set_cache_pool, step).  There is no CPU path: without the built
 libraries the import of this package fails."""
 import ctypes as C
 import os

@@ -28,12 +28,16 @@ __device__ inline float precise_glu(float gate, float up, float limit, float alp
 // A wave: two column tiles (16 weight columns each) x MT row tiles (16 activation rows each).  The weight tile is the MFMA
 // A operand, the activation rows the B operand: a lane ends up with four neighbouring columns of one row.  With fp32
 // activations step j of a 32-row weight tile multiplies rows 8 g + j of the four lane groups g.
-template <bool F32, int MT>
+// KS = 4 (few rows): the four waves of a workgroup take a quarter of K each of the same column tiles, for as many workgroups
+// and as short chains of loads as the weight allows; their sums meet in LDS.
+template <bool F32, int MT, int KS>
 __global__ __launch_bounds__(256) void tile_gemm_kernel(TileGemm p) {
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     const int g = lane >> 4, ml = lane & 15;
-    const int nt0 = (blockIdx.x * 4 + wave) * 2;
-    if (nt0 >= p.NTILES) return;
+    const int nt0 = (KS > 1 ? blockIdx.x : blockIdx.x * 4 + wave) * 2;
+    if (nt0 >= p.NTILES) return; // (KS > 1: the whole workgroup or nobody)
+    const int kper = (p.ktiles + KS - 1) / KS, k0 = KS > 1 ? wave * kper : 0;
+    const int k1 = k0 + kper < p.ktiles ? k0 + kper : p.ktiles;
     const int m0 = blockIdx.y * 16 * MT;
     const uint8_t *w[2];
     int aofs[2];
@@ -56,7 +60,7 @@ __global__ __launch_bounds__(256) void tile_gemm_kernel(TileGemm p) {
 #pragma unroll
         for (int m = 0; m < MT; ++m) acc[t][m] = f32x4 {0.f, 0.f, 0.f, 0.f};
 
-    for (int kt = 0; kt < p.ktiles; ++kt) {
+    for (int kt = k0; kt < k1; ++kt) {
         u32x4 wq[2];
 #pragma unroll
         for (int t = 0; t < 2; ++t) wq[t] = *(const u32x4 *)(w[t] + (size_t)kt * 1024);
@@ -92,6 +96,23 @@ __global__ __launch_bounds__(256) void tile_gemm_kernel(TileGemm p) {
         }
     }
 
+    if constexpr (KS > 1) {
+        __shared__ f32x4 sums[KS - 1][2 * MT][64];
+        if (wave > 0) {
+#pragma unroll
+            for (int t = 0; t < 2; ++t)
+#pragma unroll
+                for (int m = 0; m < MT; ++m) sums[wave - 1][t * MT + m][lane] = acc[t][m];
+        }
+        __syncthreads();
+        if (wave > 0) return;
+#pragma unroll
+        for (int w = 0; w < KS - 1; ++w)
+#pragma unroll
+            for (int t = 0; t < 2; ++t)
+#pragma unroll
+                for (int m = 0; m < MT; ++m) acc[t][m] += sums[w][t * MT + m][lane];
+    }
 #pragma unroll
     for (int m = 0; m < MT; ++m) {
         const int r = m0 + m * 16 + ml;
@@ -136,19 +157,21 @@ int tile_gemm(xfthip_weight_t w, int act_in, int M, const void *A, int lda, int 
     XFT_REQUIRE((long)(blocks - 1) * a_block_stride + pw.K <= lda, "tile_gemm: %d blocks of K=%d reach past the row (%d)", blocks, pw.K, lda);
     XFT_REQUIRE(ldc >= (glu ? pw.N / 2 : pw.N) && (glu != 0) == ((pw.flags & XFTHIP_WF_GATEUP) != 0), "tile_gemm: ldc=%d N=%d glu=%d", ldc, pw.N, glu);
     TileGemm p = {pw.packed, pw.KT, pw.K / 32, pw.NTILES, pw.N, M, A, lda, block_cols / 16, a_block_stride, C, ldc, c_dtype, glu, glu_limit, glu_alpha};
-    const unsigned gx = (unsigned)((pw.NTILES + 7) / 8);
-    const bool few = M <= 16 || (long)gx * ((M + 63) / 64) < 2L * device_cu_count();
-    const unsigned gy = (unsigned)((M + (few ? 16 : 64) - 1) / (few ? 16 : 64));
-    if (act_in == XFTHIP_F32) {
-        if (few)
-            hipLaunchKernelGGL((tile_gemm_kernel<true, 1>), dim3(gx, gy), dim3(256), 0, st, p);
-        else
-            hipLaunchKernelGGL((tile_gemm_kernel<true, 4>), dim3(gx, gy), dim3(256), 0, st, p);
+    const unsigned gx = (unsigned)((pw.NTILES + 7) / 8), gx1 = (unsigned)((pw.NTILES + 1) / 2);
+    const bool f32 = act_in == XFTHIP_F32;
+    auto launch = [&](auto kernel, unsigned x, unsigned y) { hipLaunchKernelGGL(kernel, dim3(x, y), dim3(256), 0, st, p); };
+    if (M <= 16) {
+        if (f32) launch(tile_gemm_kernel<true, 1, 4>, gx1, 1);
+        else launch(tile_gemm_kernel<false, 1, 4>, gx1, 1);
+    } else if (M <= 32) {
+        if (f32) launch(tile_gemm_kernel<true, 2, 4>, gx1, 1);
+        else launch(tile_gemm_kernel<false, 2, 4>, gx1, 1);
+    } else if ((long)gx * ((M + 63) / 64) < 2L * device_cu_count()) {
+        if (f32) launch(tile_gemm_kernel<true, 1, 1>, gx, (unsigned)((M + 15) / 16));
+        else launch(tile_gemm_kernel<false, 1, 1>, gx, (unsigned)((M + 15) / 16));
     } else {
-        if (few)
-            hipLaunchKernelGGL((tile_gemm_kernel<false, 1>), dim3(gx, gy), dim3(256), 0, st, p);
-        else
-            hipLaunchKernelGGL((tile_gemm_kernel<false, 4>), dim3(gx, gy), dim3(256), 0, st, p);
+        if (f32) launch(tile_gemm_kernel<true, 4, 1>, gx, (unsigned)((M + 63) / 64));
+        else launch(tile_gemm_kernel<false, 4, 1>, gx, (unsigned)((M + 63) / 64));
     }
     XFT_CHECK_HIP(hipGetLastError());
     return 0;
