@@ -210,7 +210,7 @@ SHAPES = {  # the absorbed kernel's and the expanded kernel's forms: (R, rotated
     "half": dict(heads=3, dim=128, rot=32, vdim=128, kv_rank=256, q_rank=40),
     "small": dict(heads=5, dim=64, rot=64, vdim=128, kv_rank=128, q_rank=64),
     "odd": dict(heads=3, dim=100, rot=36, vdim=90, kv_rank=300, q_rank=64),
-    "narrow": dict(heads=9, dim=32, rot=32, vdim=32, kv_rank=64, q_rank=96),
+    "narrow": dict(heads=9, dim=32, rot=32, vdim=32, kv_rank=64, q_rank=72),
     "narrow2": dict(heads=16, dim=64, rot=32, vdim=64, kv_rank=64, q_rank=32),
     "very_wide": dict(heads=1, dim=64, rot=32, vdim=64, kv_rank=640, q_rank=32),
 }
@@ -393,6 +393,25 @@ def test_generate(xh, model_dir):
         want = ref.forward(cfg, w, out[b, :-1])[16:]
         for i, row in enumerate(want):
             assert row.max() - row[out[b, 17 + i]] <= 3 * LIMIT["bf16"] * want.std()
+    m.free()
+
+
+def test_steps_larger_than_a_pass(xh, tmp_path):
+    """a step of more tokens than the device model takes at once runs in several passes: the same logits as in portions"""
+    from xfastertransformer_amd.automodel import AutoModel
+    cfg = u.config([u.latent(window=50, heads=1), u.delta(heads=2, kv_heads=1)], width=32)
+    path = str(tmp_path / "model")
+    u.write_model(path, cfg, u.weights(cfg, 30))
+    m = AutoModel.from_pretrained(path, "fp32")
+    m.set_cache_pool(2 * 8320, 2)
+    t = tokens_of(cfg, 8300, 31).tolist()
+    places = [0, 8000, 8191, 8192, 8193, 8299]
+    ids, a = m.step([(None, t, places), (None, t[:100], [0, 99])])
+    m.free_seqs(ids)
+    ids, b0 = m.step([(None, t[:4000], [0, 99])])
+    _, b1 = m.step([(ids[0], t[4000:], [p - 4000 for p in places[1:]])])
+    assert u.rel_rms(a[:6], np.concatenate([b0[:1], b1])).max() < LIMIT["f32"]
+    assert u.rel_rms(a[6:], b0).max() < LIMIT["f32"]
     m.free()
 
 

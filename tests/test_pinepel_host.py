@@ -8,7 +8,7 @@ import numpy as np
 import plan_util as u
 from oracle import pinepel_ref as ref
 
-NARROW = dict(heads=9, dim=32, rot=32, vdim=32, kv_rank=64, q_rank=96)
+NARROW = dict(heads=9, dim=32, rot=32, vdim=32, kv_rank=64, q_rank=72)
 BF16_LIMIT = 0.06  # of the GPU tests
 
 
