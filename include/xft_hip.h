@@ -546,21 +546,28 @@ int xfthip_model_set_moe(xfthip_model_t m, int idx, xfthip_moe_t moe);
 
 /* ---- layer plans: decoder stacks of several kinds of layers --------------------------- */
 /*
- * A plan describes a stack whose layers differ: what mixes the tokens (latent attention or a gated delta-rule recurrence),
- * its sizes, its constants, and the feed-forward behind it, if any.  Keys live in pages of a pool shared by all sequences,
- * recurrent state in one slot a sequence.  The reference has no counterpart; a model built from a plan is a xfthip_model_t and
- * runs behind the same calls as the others.
+ * A plan describes a stack whose layers differ: what mixes the tokens (latent attention, a gated delta-rule recurrence, grouped
+ * attention), its sizes, its constants, and the feed-forward behind it, if any (dense, or routed experts beside an optional shared
+ * one).  Keys live in pages of a pool shared by all sequences, recurrent state in one slot a sequence.  The reference has no
+ * counterpart; a model built from a plan is a xfthip_model_t and runs behind the same calls as the others.
  *
- * Every sublayer has a norm in front and a norm behind it (RMS norms whose stored weights are distances from one), the latter
- * multiplied by a learned scale per channel; layers [loop_start, loop_stop) run loop_times times, every run with its own cache
- * or state, the embedding output joining the residual in front of every pass but the first.
+ * Two arrangements of a layer's sublayers:
+ *   XFTHIP_BLOCK_SANDWICH  one after the other, a norm in front and a norm behind each, the latter multiplied by a learned scale
+ *                          per channel
+ *   XFTHIP_BLOCK_PARALLEL  both read the same residual through a norm of their own, their sum is added to it
+ * and two kinds of norm: RMS norms whose stored weights are distances from one, or tanh(alpha x) * w + b (parallel blocks only).
+ * Layers [loop_start, loop_stop) run loop_times times, every run with its own cache or state, the embedding output joining the
+ * residual in front of every pass but the first.  side_dim > 0: behind its sublayers every layer adds
+ * rms(P (gelu(G x) * e)) * w, e the layer's part of a second embedding of the token.
  */
-enum { XFTHIP_MIXER_LATENT = 1, XFTHIP_MIXER_DELTA = 2 };
+enum { XFTHIP_MIXER_LATENT = 1, XFTHIP_MIXER_DELTA = 2, XFTHIP_MIXER_GROUPED = 3 };
+enum { XFTHIP_BLOCK_SANDWICH = 0, XFTHIP_BLOCK_PARALLEL = 1 };
+enum { XFTHIP_NORM_RMS_ABOUT_ONE = 0, XFTHIP_NORM_DYNAMIC_TANH = 1 };
 typedef struct {
     int mixer;
-    int heads, kv_heads; /* kv_heads: query / key heads of the delta rule */
+    int heads, kv_heads; /* kv_heads: query / key heads of the delta rule, key / value heads of grouped attention */
     int dim, vdim; /* query / key (latent attention: their unrotated part) and value dimensions of a head */
-    /* latent attention */
+    /* latent and grouped attention; rot_dim: width of the rotated part, of a grouped head its first dimensions */
     int rot_dim, kv_rank, q_rank;
     int rot_interleaved; /* 1: pairs (2i, 2i + 1), 0: pairs (i, i + rot_dim / 2) */
     int window; /* tokens a position sees, itself included; 0 = all before it */
@@ -570,24 +577,40 @@ typedef struct {
     /* delta rule */
     int taps; /* of the short convolutions */
     int decay_rank, gate_rank; /* inner widths of the two gates' projections */
-    /* feed-forward (inter 0: none): xfthip_gemm_gateup_clamped */
+    /* feed-forward (inter 0: none; with experts: the shared one): xfthip_gemm_gateup_clamped */
     int inter;
     float glu_limit, glu_alpha;
+    /* grouped attention */
+    int qk_norm; /* RMS norm of every query and key head in front of the rotation */
+    int v_mix; /* values are mixed with those of the first layer that says so: (1 - lambda) v + lambda v_first */
+    /* context extension of the rotation (factor 0: none): frequencies whose pairs turn less than `slow` times within `original`
+     * positions are divided by `factor`, those above `fast` stay, a ramp over the pairs between; cos and sin grow by
+     * 0.1 ln(factor) + 1 */
+    double rot_factor, rot_original, rot_fast, rot_slow;
+    /* routed experts (experts 0: none): softmax over experts + identity outputs, the `top` largest of score + correction, weighted
+     * by their scores; the last `identity` outputs hand the feed-forward's input through */
+    int experts, identity, top, expert_inter;
+    float expert_limit; /* of the experts' gates; the sigmoid's factor is glu_alpha */
 } xfthip_plan_layer;
 typedef struct {
     int layers;
     int hidden, vocab;
     int loop_start, loop_stop, loop_times; /* loop_times <= 1: no loop */
     float eps, logit_scale;
+    int block, norm; /* XFTHIP_BLOCK_*, XFTHIP_NORM_* */
+    int tied_head; /* the head is the embedding table */
+    int side_dim; /* width of a layer's part of the side embedding; 0 = none */
 } xfthip_plan_config;
 typedef struct xfthip_plan *xfthip_plan_t;
 int xfthip_plan_create(const xfthip_plan_config *cfg, const xfthip_plan_layer *layers, xfthip_plan_t *out);
 int xfthip_plan_destroy(xfthip_plan_t p);
 /*
  * Tensors by name, host memory, bf16 bit patterns, row-major [rows, cols] (linear weights [out, in]; vectors cols = 1): layer -1:
- * embed, head, final.norm; a layer: norm1, norm1b, ls1, norm2, norm2b, ls2, mlp.gate / up / down, and in front of its
- * mixer's names "mix.": latent attention dq, dq.norm, uq, dkv, dkv.norm, uk, uv, o, sink; delta rule q, k, v (each with
- * .conv), b, A_log, a1, a2, dt_bias, g1, g2, norm, o.  xfthip_plan_finish checks that all are there, packs and uploads them.
+ * embed, head (unless tied), final.norm, side.embed; a layer: norm1, norm2 (a tanh norm: also .alpha and .b), sandwich blocks also
+ * norm1b, ls1, norm2b, ls2; side.gate / proj / norm; mlp.gate / up / down, with experts mlp.router, mlp.correction,
+ * mlp.e<i>.gate / up / down and mlp.shared.gate / up / down; and in front of its mixer's names "mix.": latent attention dq,
+ * dq.norm, uq, dkv, dkv.norm, uk, uv, o, sink; delta rule q, k, v (each with .conv), b, A_log, a1, a2, dt_bias, g1, g2, norm, o;
+ * grouped attention q, k (each with .norm), v, o, sink, vmix.  xfthip_plan_finish checks that all are there, packs and uploads them.
  */
 int xfthip_plan_set_tensor(xfthip_plan_t p, int layer, const char *name, const uint16_t *data_host, int rows, int cols);
 int xfthip_plan_finish(xfthip_plan_t p);

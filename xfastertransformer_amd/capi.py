@@ -535,15 +535,20 @@ class PlanLayer(C.Structure):
     _fields_ = [("mixer", C.c_int), ("heads", C.c_int), ("kv_heads", C.c_int), ("dim", C.c_int), ("vdim", C.c_int), ("rot_dim", C.c_int),
                 ("kv_rank", C.c_int), ("q_rank", C.c_int), ("rot_interleaved", C.c_int), ("window", C.c_int), ("has_sink", C.c_int),
                 ("scale", C.c_float), ("rot_base", C.c_double), ("taps", C.c_int), ("decay_rank", C.c_int), ("gate_rank", C.c_int),
-                ("inter", C.c_int), ("glu_limit", C.c_float), ("glu_alpha", C.c_float)]
+                ("inter", C.c_int), ("glu_limit", C.c_float), ("glu_alpha", C.c_float), ("qk_norm", C.c_int), ("v_mix", C.c_int),
+                ("rot_factor", C.c_double), ("rot_original", C.c_double), ("rot_fast", C.c_double), ("rot_slow", C.c_double),
+                ("experts", C.c_int), ("identity", C.c_int), ("top", C.c_int), ("expert_inter", C.c_int), ("expert_limit", C.c_float)]
 
 
 class PlanConfig(C.Structure):
     _fields_ = [("layers", C.c_int), ("hidden", C.c_int), ("vocab", C.c_int), ("loop_start", C.c_int), ("loop_stop", C.c_int),
-                ("loop_times", C.c_int), ("eps", C.c_float), ("logit_scale", C.c_float)]
+                ("loop_times", C.c_int), ("eps", C.c_float), ("logit_scale", C.c_float), ("block", C.c_int), ("norm", C.c_int),
+                ("tied_head", C.c_int), ("side_dim", C.c_int)]
 
 
-MIXER_LATENT, MIXER_DELTA = 1, 2
+MIXER_LATENT, MIXER_DELTA, MIXER_GROUPED = 1, 2, 3
+BLOCK_SANDWICH, BLOCK_PARALLEL = 0, 1
+NORM_RMS_ABOUT_ONE, NORM_DYNAMIC_TANH = 0, 1
 lib.xfthip_plan_weight_bytes.restype = C.c_size_t
 lib.xfthip_plan_weight_bytes.argtypes = [C.c_void_p]
 
@@ -551,9 +556,10 @@ lib.xfthip_plan_weight_bytes.argtypes = [C.c_void_p]
 class Plan:
     """A stack of layers of several kinds (xfthip_plan_*).  layers: dicts of PlanLayer fields."""
 
-    def __init__(self, hidden, vocab, layers, loop=(0, 0, 1), eps=1e-6, logit_scale=1.0):
+    def __init__(self, hidden, vocab, layers, loop=(0, 0, 1), eps=1e-6, logit_scale=1.0, block=BLOCK_SANDWICH, norm=NORM_RMS_ABOUT_ONE,
+                 tied_head=0, side_dim=0):
         arr = (PlanLayer * len(layers))(*[PlanLayer(**f) for f in layers])
-        self.cfg = PlanConfig(len(layers), hidden, vocab, loop[0], loop[1], loop[2], eps, logit_scale)
+        self.cfg = PlanConfig(len(layers), hidden, vocab, loop[0], loop[1], loop[2], eps, logit_scale, block, norm, tied_head, side_dim)
         self.layers = layers
         h = C.c_void_p()
         check(lib.xfthip_plan_create(C.byref(self.cfg), arr, C.byref(h)))
@@ -561,7 +567,7 @@ class Plan:
 
     def set(self, layer, name, bits):
         """bits: uint16 bf16 patterns, [rows, cols] or [n]"""
-        bits = np.ascontiguousarray(bits, np.uint16)
+        bits = np.ascontiguousarray(np.atleast_1d(bits), np.uint16)
         rows = bits.shape[0]
         check(lib.xfthip_plan_set_tensor(self.h, layer, name.encode(), _hp(bits), rows, bits.size // rows))
 

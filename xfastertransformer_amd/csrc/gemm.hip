@@ -39,7 +39,8 @@ int gemm_rows_dev(xfthip_weight_t w, int m_max, int m_hint, const int *rows_dev,
 }
 
 int gemm_grouped_rows_dev(const xfthip_weight_t *w, int n_group, const GroupWeight *table_dev, int rows_max, int rows_each_max,
-        const int *rows_dev, int rows_stride, const void *A, int lda, void *C, int ldc, int c_dtype, hipStream_t stream) {
+        const int *rows_dev, int rows_stride, const void *A, int lda, void *C, int ldc, int c_dtype, hipStream_t stream, const int *a_rows,
+        float glu_limit, float glu_alpha) {
     XFT_REQUIRE(w && n_group >= 1 && table_dev && rows_dev && rows_stride >= 3, "gemm_grouped_rows_dev: bad group arguments");
     if (int rc = check_common("gemm_grouped_rows_dev", w[0], rows_max, A, lda, C, ldc)) return rc;
     XFT_REQUIRE(rows_each_max >= 1 && rows_each_max <= rows_max, "gemm_grouped_rows_dev: bad row bounds %d / %d", rows_each_max, rows_max);
@@ -62,13 +63,15 @@ int gemm_grouped_rows_dev(const xfthip_weight_t *w, int n_group, const GroupWeig
     p.ldc = ldc;
     p.c_dtype = c_dtype;
     p.epi = XFTHIP_EPI_NONE;
-    p.gateup = gateup;
+    p.gateup = gateup && glu_alpha > 0.0f ? 2 : gateup;
+    p.glu_limit = glu_limit, p.glu_alpha = glu_alpha;
+    p.a_rows = a_rows;
     p.rows_dev = rows_dev;
     p.group = table_dev;
     p.group_n = n_group;
     p.rows_stride = rows_stride;
     if (rows_each_max <= 32) {
-        XFT_REQUIRE(pw.KT * ktile_of(pw.kind) == pw.K, "gemm_grouped_rows_dev: the few-row form needs K = %d to be a whole number of %d-row weight tiles",
+        XFT_REQUIRE(pw.KT * ktile_of(pw.kind) == pw.K || pw.kind == XFTHIP_W_BF16, "gemm_grouped_rows_dev: the few-row form needs K = %d to be a whole number of %d-row weight tiles",
                 pw.K, ktile_of(pw.kind));
         p.M = rows_each_max; // the few-row kernel: a grid row a weight, each with at most this many rows
         return qgemm_skinny(pw, p, stream);

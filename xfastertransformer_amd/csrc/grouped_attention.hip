@@ -1,0 +1,634 @@
+// Grouped attention of layer plans: every key / value head serves a group of query heads; keys and values live in pages.
+//
+// A page holds, head after head, 64 keys [64][D] and two blocks of 32 tokens of values with the tokens innermost, [V][32]:
+// both are then operands of the matrix units as they lie in memory.
+//
+// Short form (decoded tokens, short portions): 16 columns - neighbouring (token, query head) pairs of one key / value head - a
+// workgroup, straight from memory, the context split over the four waves and over workgroups.  Long form: 128 columns a
+// workgroup, blocks of 32 tokens through LDS.  Scores come out as S^T = K Q^T with the tokens along the registers, in an order
+// chosen (by the row of the key operand a token is put in) so that a lane's probabilities are those of eight neighbouring
+// tokens: the operand of O^T += V^T P^T, whose other side is one 16-byte read.
+#include "plan_dev.h"
+
+namespace xfthip {
+
+namespace {
+
+// first element of a head's part of the page that holds position `pos`
+__device__ inline size_t head_page(const int *table, int pos, int G, int g, int D, int V) {
+    return ((size_t)table[pos / kPageTokens] * G + g) * kPageTokens * (D + V);
+}
+// element of a value behind a head's keys: token `i` of the page, dimension d
+__device__ inline size_t value_at(int D, int V, int i, int d) { return (size_t)kPageTokens * D + ((size_t)(i >> 5) * V + d) * 32 + (i & 31); }
+
+struct PrepareParams {
+    StepView v;
+    GroupedBuffers b;
+    const float *q_norm, *k_norm, *cosT, *sinT; // norms may be null
+    int H, G, D, V, dim, rot, interleaved, lanes; // lanes a head takes (a power of two, 8 values each)
+    int qk_blocks, seg_blocks, keep; // keep: write first_values
+    float share, eps; // share of first_values in the values
+};
+
+// One launch, two kinds of workgroups.  The first qk_blocks: a group of `lanes` threads one query or key head of a token.  The
+// others: one head's values of up to 32 tokens (a block of the cache), turned round through LDS.
+template <bool BF16>
+__global__ __launch_bounds__(256) void grouped_prepare_kernel(PrepareParams p) {
+    const int D = p.D, V = p.V, H = p.H, G = p.G, row_len = H * D + G * (D + V);
+    if ((int)blockIdx.x < p.qk_blocks) {
+        const size_t idx = (size_t)blockIdx.x * 256 + threadIdx.x;
+        const size_t item = idx / p.lanes;
+        const int c = (int)(idx % p.lanes) * 8, heads = H + G;
+        const bool on = item < (size_t)p.v.T * heads && c < D;
+        const int t = on ? (int)(item / heads) : 0, hh = on ? (int)(item % heads) : 0;
+        const size_t at = (size_t)t * row_len + (size_t)hh * D;
+        float x[8], w[8];
+#pragma unroll
+        for (int k = 0; k < 8; ++k) x[k] = 0.0f, w[k] = 1.0f;
+        const float *norm = hh < H ? p.q_norm : p.k_norm;
+        if (on) {
+            load8<BF16>(p.b.a, at + c, x);
+            if (norm) load8<false>(norm, c, w);
+        }
+        float r = 1.0f;
+        if (norm) {
+            float sq = 0.0f;
+#pragma unroll
+            for (int k = 0; k < 8; ++k) sq = fmaf(x[k], x[k], sq);
+            for (int off = p.lanes / 2; off > 0; off >>= 1) sq += __shfl_xor(sq, off, 64);
+            r = 1.0f / sqrtf(sq / (float)p.dim + p.eps);
+        }
+        if (!on) return;
+#pragma unroll
+        for (int k = 0; k < 8; ++k) x[k] = x[k] * r * w[k];
+        const int pos = p.v.tok_pos[t], half = p.rot / 2;
+        const float *cs = p.cosT + (size_t)pos * half, *sn = p.sinT + (size_t)pos * half;
+        if (p.interleaved) {
+#pragma unroll
+            for (int k = 0; k < 4; ++k) {
+                const int i = c / 2 + k;
+                if (i >= half) continue;
+                const float u = x[2 * k], z = x[2 * k + 1], cc = cs[i], ss = sn[i];
+                x[2 * k] = fmaf(u, cc, -(z * ss)), x[2 * k + 1] = fmaf(z, cc, u * ss);
+            }
+        } else {
+#pragma unroll
+            for (int k = 0; k < 8; ++k) {
+                const int d = c + k;
+                if (d >= p.rot) continue;
+                const int i = d < half ? d : d - half, other = d < half ? d + half : i;
+                const float z = ldact<BF16>(p.b.a, at + other) * r * (norm ? norm[other] : 1.0f);
+                x[k] = d < half ? fmaf(x[k], cs[i], -(z * sn[i])) : fmaf(x[k], cs[i], z * sn[i]);
+            }
+        }
+        if (hh < H) {
+            store8<BF16>(p.b.q, ((size_t)t * H + hh) * D + c, x);
+        } else {
+            const int *table = p.v.table + (size_t)p.v.seg_row[p.v.tok_seg[t]] * p.v.table_stride;
+            store8<BF16>(p.b.pool, head_page(table, pos, G, hh - H, D, V) + (size_t)(pos % kPageTokens) * D + c, x);
+        }
+        return;
+    }
+    __shared__ float tile[32][129];
+    int job = (int)blockIdx.x - p.qk_blocks;
+    const int g = job % G;
+    job /= G;
+    const int seg = job / p.seg_blocks, start = p.v.seg_pos[seg], n = p.v.seg_len[seg], off = p.v.seg_off[seg];
+    const int b0 = ((start >> 5) + job % p.seg_blocks) * 32; // positions b0 .. b0 + 31
+    if (b0 >= start + n) return;
+    const int lo = start > b0 ? start : b0, hi = start + n < b0 + 32 ? start + n : b0 + 32;
+    const int *table = p.v.table + (size_t)p.v.seg_row[seg] * p.v.table_stride;
+    const size_t dst = head_page(table, b0, G, g, D, V);
+    for (int d0 = 0; d0 < V; d0 += 128) {
+        const int slice = V - d0 < 128 ? V - d0 : 128;
+        if (d0) __syncthreads();
+        for (int i = threadIdx.x; i < (hi - lo) * (slice / 8); i += 256) {
+            const int tok = lo + i / (slice / 8), c = i % (slice / 8) * 8, t = off + tok - start;
+            const size_t first = ((size_t)t * G + g) * V + d0 + c;
+            float x[8];
+            load8<BF16>(p.b.a, (size_t)t * row_len + (size_t)(H + G) * D + (size_t)g * V + d0 + c, x);
+            if (p.keep) {
+                store8<BF16>(p.b.first_values, first, x);
+            } else if (p.share != 0.0f) {
+                float y[8];
+                load8<BF16>(p.b.first_values, first, y);
+#pragma unroll
+                for (int k = 0; k < 8; ++k) x[k] = (1.0f - p.share) * x[k] + p.share * y[k];
+            }
+#pragma unroll
+            for (int k = 0; k < 8; ++k) tile[tok - b0][c + k] = x[k];
+        }
+        __syncthreads();
+        for (int i = threadIdx.x; i < slice * 4; i += 256) {
+            const int d = i >> 2, t8 = (i & 3) * 8;
+            if (b0 + t8 >= hi || b0 + t8 + 8 <= lo) continue;
+            const size_t at = dst + value_at(D, V, (b0 & 32) + t8, d0 + d);
+            if (b0 + t8 >= lo && b0 + t8 + 8 <= hi) {
+                float x[8];
+#pragma unroll
+                for (int k = 0; k < 8; ++k) x[k] = tile[t8 + k][d];
+                store8<BF16>(p.b.pool, at, x);
+            } else {
+                for (int k = 0; k < 8; ++k)
+                    if (b0 + t8 + k >= lo && b0 + t8 + k < hi) stact<BF16>(p.b.pool, at + k, tile[t8 + k][d]);
+            }
+        }
+    }
+}
+
+struct AttendParams {
+    StepView v;
+    const void *q, *pool;
+    void *out;
+    const float *sink; // or null
+    int H, G, D, V, window;
+    int min_len, max_len; // segments of other lengths are somebody else's
+    float scale;
+    int nsplit, groups; // context splits; column groups of the longest segment
+    float *part; // [segments][G * groups][nsplit][16][V] outputs, behind them as many [2] maxima and sums
+    size_t part_ml;
+};
+
+// Any type, any size: one workgroup a (token, head), 256 keys at a time, a key a thread for the scores and a value
+// dimension a thread for the weighted sum.
+template <bool BF16>
+__global__ __launch_bounds__(256) void grouped_attend_kernel(AttendParams p) {
+    extern __shared__ float smem[];
+    const int D = p.D, V = p.V;
+    float *qs = smem, *ps = qs + D, *o = ps + 256, *part = o + V;
+    const int t = blockIdx.x, h = blockIdx.y, g = h / (p.H / p.G);
+    const int seg = p.v.tok_seg[t], pos = p.v.tok_pos[t];
+    const int *table = p.v.table + (size_t)p.v.seg_row[seg] * p.v.table_stride;
+    for (int c = threadIdx.x; c < D; c += 256) qs[c] = ldact<BF16>(p.q, ((size_t)t * p.H + h) * D + c);
+    for (int c = threadIdx.x; c < V; c += 256) o[c] = 0.0f;
+    const int first = p.window > 0 && pos + 1 > p.window ? pos + 1 - p.window : 0;
+    float m = p.sink ? p.sink[h] : -INFINITY, l = p.sink ? 1.0f : 0.0f; // the sink has no key and no value
+    __syncthreads();
+    for (int k0 = first; k0 <= pos; k0 += 256) {
+        const int j = k0 + threadIdx.x;
+        float s = -INFINITY;
+        if (j <= pos) {
+            const size_t at = head_page(table, j, p.G, g, D, V) + (size_t)(j % kPageTokens) * D;
+            float acc = 0.0f;
+            for (int c = 0; c < D; c += 8) {
+                float k[8];
+                load8<BF16>(p.pool, at + c, k);
+#pragma unroll
+                for (int i = 0; i < 8; ++i) acc = fmaf(qs[c + i], k[i], acc);
+            }
+            s = acc * p.scale;
+        }
+        const float mx = wave_largest(s);
+        if ((threadIdx.x & 63) == 0) part[threadIdx.x >> 6] = mx;
+        __syncthreads();
+        const float m_new = fmaxf(fmaxf(fmaxf(part[0], part[1]), fmaxf(part[2], part[3])), m);
+        const float alpha = expf(m - m_new); // (0 while nothing has been seen)
+        const float e = j <= pos ? expf(s - m_new) : 0.0f;
+        ps[threadIdx.x] = e;
+        const float sum = wave_total(e);
+        if ((threadIdx.x & 63) == 0) part[4 + (threadIdx.x >> 6)] = sum;
+        __syncthreads();
+        l = l * alpha + ((part[4] + part[5]) + (part[6] + part[7]));
+        m = m_new;
+        const int n = pos - k0 + 1 < 256 ? pos - k0 + 1 : 256;
+        for (int c = threadIdx.x; c < V; c += 256) {
+            float acc = o[c] * alpha;
+            for (int i = 0; i < n;) {
+                // the run of tokens up to the end of a value block
+                const int at = k0 + i, run = 32 - (at & 31) < n - i ? 32 - (at & 31) : n - i;
+                const size_t src = head_page(table, at, p.G, g, D, V) + value_at(D, V, at % kPageTokens, c);
+                for (int k = 0; k < run; ++k) acc = fmaf(ps[i + k], ldact<BF16>(p.pool, src + k), acc);
+                i += run;
+            }
+            o[c] = acc;
+        }
+        __syncthreads();
+    }
+    for (int c = threadIdx.x; c < V; c += 256) stact<BF16>(p.out, ((size_t)t * p.H + h) * V + c, o[c] / l);
+}
+
+// BF16, short form.  KS: most 32-dim steps of a key; VT: most 16-dim tiles of a value; EXACT: as many.
+// grid (splits, G * column groups, segments)
+template <int KS, int VT, bool EXACT>
+__global__ __launch_bounds__(256, (KS <= 4 && VT <= 8) ? 3 : 1) void grouped_short_kernel(AttendParams p) {
+    extern __shared__ float merge[]; // [4 waves][16][2] maxima and sums, [4][16][V + 4] outputs
+    const StepView &v = p.v;
+    const int seg = blockIdx.z, n = v.seg_len[seg];
+    const int G = p.G, gs = p.H / G, g = blockIdx.y / p.groups, c0 = (blockIdx.y - g * p.groups) * 16, ncols = n * gs;
+    if (n < p.min_len || n > p.max_len || c0 >= ncols) return;
+    const int D = EXACT ? KS * 32 : p.D, V = EXACT ? VT * 16 : p.V, ks_n = D / 32, vt_n = V / 16;
+    const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lg = lane >> 4, i16 = lane & 15;
+    const int off = v.seg_off[seg], start = v.seg_pos[seg];
+    const int *table = v.table + (size_t)v.seg_row[seg] * v.table_stride;
+    const int last = c0 + 15 < ncols ? c0 + 15 : ncols - 1;
+    const int lo = start + c0 / gs, hi = start + last / gs; // positions of the first and the last column's token
+    const int first_vis = p.window > 0 && lo + 1 > p.window ? lo + 1 - p.window : 0;
+    const int b0 = first_vis >> 5, b1 = (hi >> 5) + 1;
+    const int per = (b1 - b0 + p.nsplit - 1) / p.nsplit;
+    int wb = b0 + (int)blockIdx.x * per, we = wb + per < b1 ? wb + per : b1;
+    const int wper = (we - wb + 3) / 4; // this wave's blocks
+    const int bb = wb + wave * wper, be = bb + wper < we ? bb + wper : we;
+
+    const int c = c0 + i16, cv = c < ncols ? c : ncols - 1;
+    const int cpos = c < ncols ? start + c / gs : -1;
+    bf16x8 qf[KS];
+    {
+        const uint16_t *row = (const uint16_t *)p.q + ((size_t)(off + cv / gs) * p.H + g * gs + cv % gs) * D + 8 * lg;
+#pragma unroll
+        for (int ks = 0; ks < KS; ++ks)
+            if (EXACT || ks < ks_n) qf[ks] = *(const bf16x8 *)(row + ks * 32);
+    }
+    f32x4 o[VT];
+#pragma unroll
+    for (int d = 0; d < VT; ++d) o[d] = f32x4 {0.f, 0.f, 0.f, 0.f};
+    float m = kUnseen, l = 0.0f;
+    const float scale2 = p.scale * kLog2e;
+
+    // row i16 of key tile tt is token 8 (i16 / 4) + 4 tt + i16 % 4 of the block
+    const int krow = (8 * (i16 >> 2) + (i16 & 3)) * D + 8 * lg, vrow = i16 * 32 + 8 * lg;
+    const uint16_t *pool = (const uint16_t *)p.pool;
+    const size_t page_len = (size_t)kPageTokens * (D + V);
+    bf16x8 kf[2][KS], vf[VT];
+    auto load_keys = [&](int blk, int page) {
+        const uint16_t *k = pool + ((size_t)page * G + g) * page_len + (blk & 1) * 32 * D + krow;
+#pragma unroll
+        for (int ks = 0; ks < KS; ++ks)
+            if (EXACT || ks < ks_n) kf[0][ks] = *(const bf16x8 *)(k + ks * 32), kf[1][ks] = *(const bf16x8 *)(k + 4 * D + ks * 32);
+    };
+    auto load_values = [&](int blk, int page) {
+        const uint16_t *w = pool + ((size_t)page * G + g) * page_len + (size_t)kPageTokens * D + (blk & 1) * 32 * V + vrow;
+#pragma unroll
+        for (int d = 0; d < VT; ++d)
+            if (EXACT || d < vt_n) vf[d] = *(const bf16x8 *)(w + d * 512);
+    };
+    int page = bb < be ? table[bb >> 1] : 0;
+    if (bb < be) load_keys(bb, page), load_values(bb, page);
+    for (int blk = bb; blk < be; ++blk) {
+        const bool more = blk + 1 < be;
+        if (more) page = table[(blk + 1) >> 1];
+        f32x4 s0 = {0.f, 0.f, 0.f, 0.f}, s1 = s0;
+#pragma unroll
+        for (int ks = 0; ks < KS; ++ks)
+            if (EXACT || ks < ks_n) {
+                s0 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[0][ks], qf[ks], s0, 0, 0, 0);
+                s1 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[1][ks], qf[ks], s1, 0, 0, 0);
+            }
+        if (more) load_keys(blk + 1, page);
+        s0 *= scale2, s1 *= scale2;
+        float x[8], bm = kUnseen;
+#pragma unroll
+        for (int j = 0; j < 8; ++j) x[j] = j < 4 ? s0[j & 3] : s1[j & 3];
+        const bool open = blk * 32 + 31 <= lo && (p.window <= 0 || blk * 32 > hi - p.window); // every column sees the whole block
+        if (!open) {
+#pragma unroll
+            for (int j = 0; j < 8; ++j) {
+                const int t = blk * 32 + 8 * lg + j;
+                x[j] = t <= cpos && (p.window <= 0 || t > cpos - p.window) ? x[j] : kUnseen;
+            }
+        }
+#pragma unroll
+        for (int j = 0; j < 8; ++j) bm = fmaxf(bm, x[j]);
+        bm = fmaxf(bm, __shfl_xor(bm, 16, 64));
+        bm = fmaxf(bm, __shfl_xor(bm, 32, 64));
+        const float m_new = fmaxf(m, bm);
+        const float alpha = __builtin_amdgcn_exp2f(m - m_new);
+        m = m_new;
+        float sum = 0.0f;
+#pragma unroll
+        for (int j = 0; j < 8; ++j) {
+            // (a column that has seen no key has its reference point at the masked score)
+            const float e = __builtin_amdgcn_exp2f(x[j] - m_new);
+            x[j] = open || x[j] > 0.5f * kUnseen ? e : 0.0f;
+            sum += x[j];
+        }
+        l = l * alpha + sum;
+        const bf16x8 pf = pack_bf16x8(x);
+        if (__builtin_amdgcn_ballot_w64(alpha != 1.0f) != 0) {
+#pragma unroll
+            for (int d = 0; d < VT; ++d) o[d] *= alpha;
+        }
+#pragma unroll
+        for (int d = 0; d < VT; ++d)
+            if (EXACT || d < vt_n) o[d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[d], pf, o[d], 0, 0, 0);
+        if (more) load_values(blk + 1, page);
+    }
+    l += __shfl_xor(l, 16, 64);
+    l += __shfl_xor(l, 32, 64);
+    // the four waves' parts meet in LDS
+    float *ml = merge, *outs = merge + 4 * 16 * 2;
+    const int pitch = V + 4;
+    if (lg == 0) ml[(wave * 16 + i16) * 2] = m, ml[(wave * 16 + i16) * 2 + 1] = l;
+#pragma unroll
+    for (int d = 0; d < VT; ++d)
+        if (EXACT || d < vt_n) *(f32x4 *)(outs + (wave * 16 + i16) * pitch + d * 16 + 4 * lg) = o[d];
+    __syncthreads();
+    const size_t slot0 = (((size_t)seg * gridDim.y + blockIdx.y) * p.nsplit + blockIdx.x) * 16;
+    for (int i = threadIdx.x; i < 16 * (V / 4); i += 256) {
+        const int col = i / (V / 4), d = i % (V / 4) * 4, cc = c0 + col;
+        if (cc >= ncols) continue;
+        float mt = kUnseen, den = 0.0f;
+#pragma unroll
+        for (int w = 0; w < 4; ++w) mt = fmaxf(mt, ml[(w * 16 + col) * 2]);
+        const float s2 = p.sink && p.nsplit == 1 ? p.sink[g * gs + cc % gs] * kLog2e : kUnseen;
+        mt = fmaxf(mt, s2);
+        f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int w = 0; w < 4; ++w) {
+            const float mw = ml[(w * 16 + col) * 2], e = mw > 0.5f * kUnseen ? __builtin_amdgcn_exp2f(mw - mt) : 0.0f;
+            den += ml[(w * 16 + col) * 2 + 1] * e;
+            acc += *(const f32x4 *)(outs + (w * 16 + col) * pitch + d) * e;
+        }
+        if (p.nsplit > 1) {
+            *(f32x4 *)(p.part + (slot0 + col) * V + d) = acc;
+            if (d == 0) *(float2 *)(p.part + p.part_ml + (slot0 + col) * 2) = make_float2(mt, den);
+        } else {
+            if (p.sink) den += __builtin_amdgcn_exp2f(s2 - mt);
+            acc *= 1.0f / den;
+            uint16_t *dst = (uint16_t *)p.out + ((size_t)(off + cc / gs) * p.H + g * gs + cc % gs) * V + d;
+            *(uint2 *)dst = make_uint2(pack_pair(acc[0], acc[1]), pack_pair(acc[2], acc[3]));
+        }
+    }
+}
+
+// sum of a column's splits; grid (G * column groups, segments, 16 columns), 64 threads
+constexpr int kMaxSplits = 64;
+__global__ __launch_bounds__(64) void grouped_merge_kernel(AttendParams p) {
+    __shared__ float w[kMaxSplits];
+    const StepView &v = p.v;
+    const int seg = blockIdx.y, n = v.seg_len[seg], gs = p.H / p.G, V = p.V;
+    const int g = blockIdx.x / p.groups, c = (blockIdx.x - g * p.groups) * 16 + blockIdx.z;
+    if (n < p.min_len || n > p.max_len || c >= n * gs) return;
+    const int head = g * gs + c % gs, lane = threadIdx.x;
+    const size_t slot0 = ((size_t)seg * gridDim.x + blockIdx.x) * p.nsplit * 16 + blockIdx.z;
+    float2 ml = make_float2(kUnseen, 0.0f);
+    if (lane < p.nsplit) ml = *(const float2 *)(p.part + p.part_ml + (slot0 + (size_t)lane * 16) * 2);
+    const float s2 = p.sink ? p.sink[head] * kLog2e : kUnseen;
+    const float mt = fmaxf(wave_largest(ml.x), s2);
+    const float e = ml.x > 0.5f * kUnseen ? __builtin_amdgcn_exp2f(ml.x - mt) : 0.0f;
+    const float den = wave_total(ml.y * e) + (p.sink ? __builtin_amdgcn_exp2f(s2 - mt) : 0.0f);
+    w[lane] = e;
+    __syncthreads();
+    const float inv = 1.0f / den;
+    uint16_t *dst = (uint16_t *)p.out + ((size_t)(v.seg_off[seg] + c / gs) * p.H + head) * V;
+    for (int d = lane * 4; d < V; d += 256) {
+        f32x4 acc[4];
+#pragma unroll
+        for (int i = 0; i < 4; ++i) acc[i] = f32x4 {0.f, 0.f, 0.f, 0.f};
+        for (int s0 = 0; s0 < p.nsplit; s0 += 4) {
+            f32x4 x[4];
+#pragma unroll
+            for (int i = 0; i < 4; ++i) x[i] = *(const f32x4 *)(p.part + (slot0 + (size_t)(s0 + i < p.nsplit ? s0 + i : p.nsplit - 1) * 16) * V + d);
+#pragma unroll
+            for (int i = 0; i < 4; ++i)
+                if (s0 + i < p.nsplit) acc[i] += x[i] * w[s0 + i];
+        }
+        const f32x4 y = ((acc[0] + acc[1]) + (acc[2] + acc[3])) * inv;
+        *(uint2 *)(dst + d) = make_uint2(pack_pair(y[0], y[1]), pack_pair(y[2], y[3]));
+    }
+}
+
+// BF16, long form: 128 columns a workgroup (32 a wave), the visible context in blocks of 32 tokens through LDS, on 32 x 32 tiles.
+// KSM: most 16-dim steps of a key; VTM: most 32-dim tiles of a value; EXACT: as many.  grid (G, column groups, segments)
+template <int KSM, int VTM, bool EXACT>
+__global__ __launch_bounds__(256, (KSM <= 8 && VTM <= 4) ? 2 : 1) void grouped_long_kernel(AttendParams p) {
+    extern __shared__ unsigned char lds[];
+    const StepView &v = p.v;
+    const int seg = blockIdx.z, n = v.seg_len[seg];
+    const int G = p.G, gs = p.H / G, g = blockIdx.x, ncols = n * gs;
+    const int c0 = ((int)gridDim.y - 1 - (int)blockIdx.y) * 128; // the columns with the longest contexts first
+    if (n < p.min_len || n > p.max_len || c0 >= ncols) return;
+    const int D = EXACT ? KSM * 16 : p.D, V = EXACT ? VTM * 32 : p.V, ks_n = D / 16, vt_n = V / 32;
+    const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), h = lane >> 5, cl = lane & 31;
+    const int off = v.seg_off[seg], start = v.seg_pos[seg];
+    const int *table = v.table + (size_t)v.seg_row[seg] * v.table_stride;
+    const int kpitch = D * 2 + 16, vpitch = 80, bufb = 32 * kpitch + V * vpitch;
+    const int c = c0 + wave * 32 + cl, cv = c < ncols ? c : ncols - 1;
+    const int pos = start + cv / gs;
+    const int wc0 = c0 + wave * 32, wc1 = wc0 + 31 < ncols ? wc0 + 31 : ncols - 1;
+    const int wlo = start + wc0 / gs, whi = start + wc1 / gs; // positions of the wave's first and last column
+    const bool wave_on = wc0 < ncols;
+    const int head = g * gs + cv % gs;
+    const size_t orow = (size_t)(off + cv / gs) * p.H + head;
+    bf16x8 qf[KSM];
+    {
+        const uint16_t *row = (const uint16_t *)p.q + orow * D + 8 * h;
+#pragma unroll
+        for (int ks = 0; ks < KSM; ++ks)
+            if (EXACT || ks < ks_n) qf[ks] = *(const bf16x8 *)(row + ks * 16);
+    }
+    f32x16 o[VTM];
+#pragma unroll
+    for (int d = 0; d < VTM; ++d)
+#pragma unroll
+        for (int r = 0; r < 16; ++r) o[d][r] = 0.0f;
+    float m = kUnseen, l = 0.0f;
+    const float scale2 = p.scale * kLog2e;
+    const int lo = start + c0 / gs, last = c0 + 127 < ncols ? c0 + 127 : ncols - 1, hi = start + last / gs;
+    const int first = p.window > 0 && lo + 1 > p.window ? lo + 1 - p.window : 0;
+    const int b0 = first >> 5, b1 = (hi >> 5) + 1;
+    const int wfirst = p.window > 0 && wlo + 1 > p.window ? wlo + 1 - p.window : 0;
+
+    constexpr int PER = KSM / 4 + VTM / 2 + 1; // 16-byte chunks of a block a thread carries (at least D / 64 + V / 64)
+    const int kch = D * 4, chunks = kch + V * 4; // of keys, of both
+    u32x4 stage[PER];
+    int src[PER], step[PER], dst[PER]; // element behind the head's page, way to the second block of the page, byte in LDS
+#pragma unroll
+    for (int i = 0; i < PER; ++i) {
+        int e = i * 256 + threadIdx.x;
+        e = e < chunks ? e : chunks - 1; // (past the block: its last chunk once more)
+        if (e < kch) {
+            src[i] = e * 8, step[i] = 32 * D, dst[i] = (e + e / (D / 8)) * 16; // 16 bytes of padding behind every row before it
+        } else {
+            e -= kch; // four chunks a value row
+            src[i] = kPageTokens * D + e * 8, step[i] = 32 * V, dst[i] = 32 * kpitch + (e >> 2) * vpitch + (e & 3) * 16;
+        }
+    }
+    const uint16_t *pool = (const uint16_t *)p.pool;
+    auto fetch = [&](int blk, int page) {
+        const uint16_t *base = pool + ((size_t)page * G + g) * kPageTokens * (D + V);
+#pragma unroll
+        for (int i = 0; i < PER; ++i)
+            if (i * 256 < chunks) stage[i] = *(const u32x4 *)(base + src[i] + (blk & 1) * step[i]);
+    };
+    // row cl of the key operand is the token with bits 2 and 3 swapped: register 8 t + j of half h is then token 16 t + 8 h + j
+    const int ktok = (cl & 19) | ((cl & 4) << 1) | ((cl & 8) >> 1);
+    fetch(b0, table[b0 >> 1]);
+    int page = b0 + 1 < b1 ? table[(b0 + 1) >> 1] : 0;
+    int buf = 0;
+    for (int blk = b0; blk < b1; ++blk, buf ^= 1) {
+        unsigned char *kb = lds + buf * bufb, *vb = kb + 32 * kpitch;
+#pragma unroll
+        for (int i = 0; i < PER; ++i)
+            if (i * 256 < chunks) *(u32x4 *)(kb + dst[i]) = stage[i];
+        __syncthreads();
+        if (blk + 1 < b1) fetch(blk + 1, page);
+        if (blk + 2 < b1) page = table[(blk + 2) >> 1];
+        const int t0 = blk * 32;
+        if (!wave_on || t0 > whi || t0 + 31 < wfirst) continue; // (the same for the whole wave; the barrier above is all there is)
+        f32x16 s;
+#pragma unroll
+        for (int r = 0; r < 16; ++r) s[r] = 0.0f;
+        const unsigned char *krow = kb + ktok * kpitch + 16 * h;
+#pragma unroll
+        for (int ks = 0; ks < KSM; ++ks)
+            if (EXACT || ks < ks_n) s = __builtin_amdgcn_mfma_f32_32x32x16_bf16(*(const bf16x8 *)(krow + ks * 32), qf[ks], s, 0, 0, 0);
+        const bool masked = t0 + 31 > wlo || (p.window > 0 && t0 + p.window <= whi);
+        float bm = kUnseen;
+#pragma unroll
+        for (int r = 0; r < 16; ++r) s[r] *= scale2;
+        if (masked) {
+#pragma unroll
+            for (int r = 0; r < 16; ++r) {
+                const int t = t0 + 16 * (r >> 3) + 8 * h + (r & 7);
+                s[r] = t <= pos && (p.window <= 0 || t > pos - p.window) ? s[r] : kUnseen;
+            }
+        }
+#pragma unroll
+        for (int r = 0; r < 16; ++r) bm = fmaxf(bm, s[r]);
+        bm = fmaxf(bm, __shfl_xor(bm, 32, 64));
+        const float m_new = bm > m + 8.0f ? bm : m; // (the reference point moves only when it has to)
+        const float alpha = __builtin_amdgcn_exp2f(m - m_new);
+        m = m_new;
+        float sum = 0.0f;
+#pragma unroll
+        for (int r = 0; r < 16; ++r) {
+            const float e = __builtin_amdgcn_exp2f(s[r] - m_new);
+            // (a column that has seen no key yet has its reference point at the masked score)
+            s[r] = !masked || s[r] > 0.5f * kUnseen ? e : 0.0f;
+            sum += s[r];
+        }
+        l = l * alpha + sum;
+        if (__builtin_amdgcn_ballot_w64(alpha != 1.0f) != 0) {
+#pragma unroll
+            for (int d = 0; d < VTM; ++d) o[d] *= alpha;
+        }
+#pragma unroll
+        for (int t = 0; t < 2; ++t) {
+            float pr[8];
+#pragma unroll
+            for (int j = 0; j < 8; ++j) pr[j] = s[8 * t + j];
+            const bf16x8 pf = pack_bf16x8(pr);
+            const unsigned char *vrow = vb + cl * vpitch + t * 32 + h * 16;
+#pragma unroll
+            for (int d = 0; d < VTM; ++d)
+                if (EXACT || d < vt_n) o[d] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(*(const bf16x8 *)(vrow + d * 32 * vpitch), pf, o[d], 0, 0, 0);
+        }
+    }
+    l += __shfl_xor(l, 32, 64);
+    if (c >= ncols) return;
+    float mul = 1.0f;
+    if (p.sink) {
+        const float s2 = p.sink[head] * kLog2e, mt = fmaxf(m, s2);
+        mul = __builtin_amdgcn_exp2f(m - mt);
+        l = l * mul + __builtin_amdgcn_exp2f(s2 - mt);
+    }
+    mul /= l;
+    uint16_t *out = (uint16_t *)p.out + orow * V;
+#pragma unroll
+    for (int d = 0; d < VTM; ++d)
+        if (EXACT || d < vt_n) {
+#pragma unroll
+            for (int q = 0; q < 4; ++q)
+                *(uint2 *)(out + d * 32 + 8 * q + 4 * h) =
+                        make_uint2(pack_pair(o[d][4 * q] * mul, o[d][4 * q + 1] * mul), pack_pair(o[d][4 * q + 2] * mul, o[d][4 * q + 3] * mul));
+        }
+}
+
+template <int KS, int VT, bool EXACT>
+int launch_short(const AttendParams &p, hipStream_t st) {
+    static const hipError_t attr = hipFuncSetAttribute((const void *)grouped_short_kernel<KS, VT, EXACT>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
+    XFT_CHECK_HIP(attr);
+    const size_t smem = (size_t)4 * 16 * (2 + p.V + 4) * 4;
+    hipLaunchKernelGGL((grouped_short_kernel<KS, VT, EXACT>), dim3(p.nsplit, p.G * p.groups, p.v.B), dim3(256), smem, st, p);
+    XFT_CHECK_HIP(hipGetLastError());
+    return 0;
+}
+template <int KSM, int VTM, bool EXACT>
+int launch_long(const AttendParams &p, hipStream_t st) {
+    static const hipError_t attr = hipFuncSetAttribute((const void *)grouped_long_kernel<KSM, VTM, EXACT>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
+    XFT_CHECK_HIP(attr);
+    const size_t smem = (size_t)2 * (32 * (p.D * 2 + 16) + p.V * 80);
+    hipLaunchKernelGGL((grouped_long_kernel<KSM, VTM, EXACT>), dim3(p.G, (p.v.longest * (p.H / p.G) + 127) / 128, p.v.B), dim3(256), smem, st, p);
+    XFT_CHECK_HIP(hipGetLastError());
+    return 0;
+}
+
+bool mfma_takes(const PlanLayer &L) { return L.D <= 256 && L.V <= 256; }
+constexpr int kShortTokens = 16; // longest segment of the short form
+
+} // namespace
+
+int grouped_prepare(int act, const PlanLayer &L, const StepView &v, const GroupedBuffers &b, float eps, hipStream_t st) {
+    const xfthip_plan_layer &s = L.s;
+    PrepareParams p = {v, b, L.q_norm, L.kv_norm, L.cosT, L.sinT, s.heads, s.kv_heads, L.D, L.V, s.dim, s.rot_dim, s.rot_interleaved, 4, 0, 0, L.first_values ? 1 : 0,
+            s.v_mix && !L.first_values ? L.value_share : 0.0f, eps};
+    while (p.lanes * 8 < L.D) p.lanes *= 2;
+    XFT_REQUIRE(p.lanes <= 64, "grouped_prepare: heads of %d values too wide", L.D);
+    p.qk_blocks = (int)(((size_t)v.T * (s.heads + s.kv_heads) * p.lanes + 255) / 256);
+    p.seg_blocks = (v.longest + 62) / 32; // blocks of 32 positions a segment of that length can touch
+    const dim3 grid(p.qk_blocks + v.B * s.kv_heads * p.seg_blocks);
+    if (act == XFTHIP_BF16) hipLaunchKernelGGL(grouped_prepare_kernel<true>, grid, dim3(256), 0, st, p);
+    else hipLaunchKernelGGL(grouped_prepare_kernel<false>, grid, dim3(256), 0, st, p);
+    XFT_CHECK_HIP(hipGetLastError());
+    return 0;
+}
+
+// Parts a context of `hint` tokens is split into: as many as give every compute unit a workgroup, every wave a block permitting.
+int grouped_split_count(const PlanLayer &L, int B, int longest, int hint) {
+    if (!mfma_takes(L)) return 1;
+    longest = longest < kShortTokens ? longest : kShortTokens;
+    const long units = (long)B * L.s.kv_heads * ((longest * (L.s.heads / L.s.kv_heads) + 15) / 16);
+    const int ctx = L.s.window > 0 && L.s.window + longest < hint ? L.s.window + longest : hint;
+    const int most = (ctx + 127) / 128;
+    long want = device_cu_count() / units;
+    want = want < most ? want : most;
+    want = want < kMaxSplits / 2 ? want : kMaxSplits / 2;
+    return want < 1 ? 1 : (int)want;
+}
+
+// (splits times units never exceed the compute units, or nothing is split)
+size_t grouped_part_floats(const PlanLayer &L) {
+    return mfma_takes(L) ? (size_t)device_cu_count() * 16 * (L.V + 2) : 0;
+}
+
+int grouped_attention(int act, const PlanLayer &L, const StepView &v, const void *q, const void *pool, void *out, int hint, float *part, size_t part_floats,
+        hipStream_t st) {
+    const xfthip_plan_layer &s = L.s;
+    AttendParams p = {v, q, pool, out, L.sink, s.heads, s.kv_heads, L.D, L.V, s.window, 0, 1 << 30, s.scale, 1, 1, part, 0};
+    if (act != XFTHIP_BF16 || !mfma_takes(L)) {
+        const size_t smem = (size_t)(L.D + 256 + L.V + 8) * 4;
+        if (act == XFTHIP_BF16) hipLaunchKernelGGL(grouped_attend_kernel<true>, dim3(v.T, s.heads), dim3(256), smem, st, p);
+        else hipLaunchKernelGGL(grouped_attend_kernel<false>, dim3(v.T, s.heads), dim3(256), smem, st, p);
+        XFT_CHECK_HIP(hipGetLastError());
+        return 0;
+    }
+    const int ks = L.D / 32, vt = L.V / 16, gs = s.heads / s.kv_heads;
+    int rc = 0;
+    if (v.longest > kShortTokens) {
+        p.min_len = kShortTokens + 1;
+        if (ks == 4 && vt == 8) rc = launch_long<8, 4, true>(p, st);
+        else if (ks == 6 && vt == 8) rc = launch_long<12, 4, true>(p, st);
+        else if (ks == 2 && vt == 4) rc = launch_long<4, 2, true>(p, st);
+        else if (ks <= 4 && vt <= 8) rc = launch_long<8, 4, false>(p, st);
+        else rc = launch_long<16, 8, false>(p, st);
+        if (rc || v.T == v.longest) return rc; // (a batch of one long segment)
+    }
+    p.min_len = 0, p.max_len = kShortTokens;
+    const int longest = v.longest < kShortTokens ? v.longest : kShortTokens;
+    p.groups = (longest * gs + 15) / 16;
+    p.nsplit = grouped_split_count(L, v.B, longest, hint);
+    const size_t slots = (size_t)v.B * s.kv_heads * p.groups * p.nsplit * 16;
+    p.part_ml = slots * L.V;
+    XFT_REQUIRE(p.nsplit == 1 || slots * (L.V + 2) <= part_floats, "grouped_attention: workspace too small for %zu partial columns", slots);
+    if (ks == 4 && vt == 8) rc = launch_short<4, 8, true>(p, st);
+    else if (ks == 6 && vt == 8) rc = launch_short<6, 8, true>(p, st);
+    else if (ks == 2 && vt == 4) rc = launch_short<2, 4, true>(p, st);
+    else if (ks <= 4 && vt <= 8) rc = launch_short<4, 8, false>(p, st);
+    else rc = launch_short<8, 16, false>(p, st);
+    if (rc || p.nsplit == 1) return rc;
+    hipLaunchKernelGGL(grouped_merge_kernel, dim3(s.kv_heads * p.groups, v.B, 16), dim3(64), 0, st, p);
+    XFT_CHECK_HIP(hipGetLastError());
+    return 0;
+}
+
+} // namespace xfthip

@@ -332,11 +332,58 @@ PlanSpec pinepel(const Json &c, const SafeTensors &w) {
     return s;
 }
 
+// ---- Veterax: grouped attention with normed heads, a sink and values mixed with an earlier layer's, beside routed experts (some of
+// them the identity) and a shared one, both reading the residual through a tanh in the place of a norm; a second embedding of
+// the token joins behind every layer ----
+PlanSpec veterax(const Json &c, const SafeTensors &) {
+    PlanSpec s;
+    s.cfg.hidden = (int)c.integer("width");
+    s.cfg.vocab = (int)c.integer("vocab");
+    s.cfg.eps = (float)c.at("norm").real("eps");
+    s.cfg.logit_scale = 1.0f;
+    s.cfg.loop_times = 1;
+    s.cfg.block = XFTHIP_BLOCK_PARALLEL, s.cfg.norm = XFTHIP_NORM_DYNAMIC_TANH, s.cfg.tied_head = 1;
+    if (c.has("token_side")) s.cfg.side_dim = (int)c.at("token_side").integer("dim");
+    const Json &layers = c.at("layers");
+    for (size_t i = 0; i < layers.items.size(); ++i) {
+        const std::string at = "layer " + std::to_string(i) + ": ";
+        const Json &e = layers.items[i], &m = e.at("mixer");
+        if (e.string("type") != "attention") broken("layer type '" + e.string("type") + "' of config.json is not known");
+        xfthip_plan_layer L {};
+        L.mixer = XFTHIP_MIXER_GROUPED;
+        L.heads = (int)m.integer("heads"), L.kv_heads = (int)m.integer("kv_heads"), L.dim = (int)m.integer("dim"), L.vdim = (int)m.integer("vdim");
+        L.scale = (float)m.real("scale");
+        L.has_sink = 1, L.qk_norm = 1;
+        L.v_mix = m.has("v_mix") && m.at("v_mix").flag ? 1 : 0;
+        const Json &rot = m.at("rot");
+        L.rot_dim = (int)rot.integer("dims"), L.rot_base = rot.real("base"), L.rot_interleaved = 1;
+        if (rot.has("scaling")) {
+            const Json &x = rot.at("scaling");
+            L.rot_factor = x.real("factor"), L.rot_original = x.real("original"), L.rot_fast = x.real("fast"), L.rot_slow = x.real("slow");
+            if (!(L.rot_factor > 0.0)) broken(at + "a rotation scaled by nothing");
+        }
+        if (e.has("mlp")) {
+            const Json &f = e.at("mlp");
+            if (f.string("kind") != "moe") broken("feed-forward '" + f.string("kind") + "' of config.json is not known");
+            const Json &r = f.at("router"), &x = f.at("expert");
+            L.experts = (int)r.integer("experts"), L.top = (int)r.integer("top");
+            L.identity = r.has("identity") ? (int)r.integer("identity") : 0;
+            if (L.experts < 1) broken(at + "a router without experts");
+            L.expert_inter = (int)x.integer("ff"), L.expert_limit = (float)x.real("limit");
+            L.glu_alpha = 1.702f;
+            if (f.has("shared")) L.inter = (int)f.at("shared").integer("ff"), L.glu_limit = (float)f.at("shared").real("limit");
+        }
+        s.layers.push_back(L);
+    }
+    s.cfg.layers = (int)s.layers.size();
+    return s;
+}
+
 struct Architecture {
     const char *name;
     PlanSpec (*describe)(const Json &config, const SafeTensors &weights);
 };
-const Architecture kArchitectures[] = {{"Pinepel", pinepel}};
+const Architecture kArchitectures[] = {{"Pinepel", pinepel}, {"Veterax", veterax}};
 
 const Architecture *find_architecture(const Json &c) {
     if (c.kind != Json::Object || !c.has("architecture") || c.at("architecture").kind != Json::String) return nullptr;

@@ -471,7 +471,9 @@ struct ModelImpl {
             const xfthip_plan_layer &y = planSpec.layers[i];
             const int runs = i >= planSpec.cfg.loop_start && i < planSpec.cfg.loop_stop ? times : 1;
             const double e = planAct == XFTHIP_F32 ? 4 : 2;
-            b += runs * (y.mixer == XFTHIP_MIXER_LATENT ? (double)len * (y.kv_rank + y.rot_dim) * e : (double)y.heads * y.dim * y.vdim * 4);
+            b += runs * (y.mixer == XFTHIP_MIXER_LATENT    ? (double)len * (y.kv_rank + y.rot_dim) * e
+                         : y.mixer == XFTHIP_MIXER_GROUPED ? (double)len * y.kv_heads * (y.dim + y.vdim) * e
+                                                           : (double)y.heads * y.dim * y.vdim * 4);
         }
         return b;
     }

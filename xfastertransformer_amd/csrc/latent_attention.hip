@@ -5,42 +5,11 @@
 // cached rows themselves, and the weighted sum of latents is carried to the value space by W_uv behind the softmax.  All
 // heads of a token then read the same cache rows.  Expanded form: keys and values of every head are made from the latents of
 // the whole context first, which pays when many tokens attend to them.
-#include "plan.h"
+#include "plan_dev.h"
 
 namespace xfthip {
 
 namespace {
-
-__device__ inline float wave_total(float v) {
-#pragma unroll
-    for (int off = 32; off > 0; off >>= 1) v += __shfl_xor(v, off, 64);
-    return v;
-}
-__device__ inline float wave_largest(float v) {
-#pragma unroll
-    for (int off = 32; off > 0; off >>= 1) v = fmaxf(v, __shfl_xor(v, off, 64));
-    return v;
-}
-
-typedef __attribute__((ext_vector_type(2))) __bf16 bf16x2;
-// two values -> packed bf16 pair, round to nearest even (v_cvt_pk_bf16_f32)
-__device__ inline uint32_t pack_pair(float lo, float hi) { return __builtin_bit_cast(uint32_t, bf16x2 {(__bf16)lo, (__bf16)hi}); }
-
-template <bool BF16>
-__device__ inline float ldact(const void *p, size_t i) {
-    if constexpr (BF16) return bf16_to_f32(((const uint16_t *)p)[i]);
-    else return ((const float *)p)[i];
-}
-template <bool BF16>
-__device__ inline void stact(void *p, size_t i, float v) {
-    if constexpr (BF16) ((uint16_t *)p)[i] = f32_to_bf16_ref(v);
-    else ((float *)p)[i] = v;
-}
-
-// cache row of position `pos` of slot `row`
-__device__ inline size_t cache_row(const StepView &v, int row, int pos) {
-    return (size_t)v.table[(size_t)row * v.table_stride + pos / kPageTokens] * kPageTokens + pos % kPageTokens;
-}
 
 struct PrepareParams {
     StepView v;
@@ -51,32 +20,6 @@ struct PrepareParams {
     int QR, RD, q_rank, kv_rank, rot, interleaved;
     float eps;
 };
-
-template <bool BF16>
-__device__ inline void load8(const void *p, size_t i, float (&v)[8]) {
-    if constexpr (BF16) {
-        const uint4 q = *(const uint4 *)((const uint16_t *)p + i);
-        const uint32_t w[4] = {q.x, q.y, q.z, q.w};
-#pragma unroll
-        for (int k = 0; k < 4; ++k) v[2 * k] = u2f(w[k] << 16), v[2 * k + 1] = u2f(w[k] & 0xFFFF0000u);
-    } else {
-        const f32x4 x = *(const f32x4 *)((const float *)p + i), y = *(const f32x4 *)((const float *)p + i + 4);
-#pragma unroll
-        for (int k = 0; k < 4; ++k) v[k] = x[k], v[4 + k] = y[k];
-    }
-}
-template <bool BF16>
-__device__ inline void store8(void *p, size_t i, const float (&v)[8]) {
-    if constexpr (BF16) {
-        uint32_t w[4];
-#pragma unroll
-        for (int k = 0; k < 4; ++k) w[k] = pack_pair(v[2 * k], v[2 * k + 1]);
-        *(uint4 *)((uint16_t *)p + i) = make_uint4(w[0], w[1], w[2], w[3]);
-    } else {
-        *(f32x4 *)((float *)p + i) = f32x4 {v[0], v[1], v[2], v[3]};
-        *(f32x4 *)((float *)p + i + 4) = f32x4 {v[4], v[5], v[6], v[7]};
-    }
-}
 
 // One token a workgroup, 8 neighbouring values a thread and turn; the row and the norm weights are in registers (CH turns)
 // before the sums meet.
@@ -246,20 +189,9 @@ __global__ __launch_bounds__(256) void latent_attend_kernel(AttendParams p) {
     for (int c = threadIdx.x; c < R; c += 256) stact<BF16>(p.out, ((size_t)t * p.H + h) * R + c, o[c] / l);
 }
 
-typedef uint32_t u32x4 __attribute__((ext_vector_type(4)));
 typedef __attribute__((ext_vector_type(4))) short s16x4;
 typedef __attribute__((ext_vector_type(8))) short s16x8;
 #define LDS_PTR(type, p) ((__attribute__((address_space(3))) type *)(p))
-
-constexpr float kUnseen = -1.0e30f; // score of a masked key, maximum of a column that has seen none
-constexpr float kLog2e = 1.4426950408889634f;
-
-__device__ inline bf16x8 pack_bf16x8(const float (&v)[8]) {
-    u32x4 u;
-#pragma unroll
-    for (int i = 0; i < 4; ++i) u[i] = pack_pair(v[2 * i], v[2 * i + 1]);
-    return __builtin_bit_cast(bf16x8, u);
-}
 
 // Two transposing LDS reads: within 16 lanes, lane i names token row i / 4 and dims 4 (i % 4) of a block of 4 tokens x 16 dims
 // and receives the four tokens of dim i.  `second` lies where the lane's other four tokens start.

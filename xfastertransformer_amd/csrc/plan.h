@@ -1,7 +1,7 @@
-// Layer plans: decoder stacks whose layers differ in kind (latent attention, delta-rule recurrence), whose keys live
-// in a page pool shared by all sequences and whose recurrent layers keep a state per sequence slot.  Declarations
-// shared by the plan's driver (plan_model.hip) and its kernels (plan_layers.hip, latent_attention.hip, delta_rule.hip,
-// tile_gemm.hip).
+// Layer plans: decoder stacks whose layers differ in kind (latent attention, grouped attention, delta-rule recurrence), whose
+// keys live in a page pool shared by all sequences and whose recurrent layers keep a state per sequence slot.  Declarations
+// shared by the plan's driver (plan_model.hip) and its kernels (plan_layers.hip, latent_attention.hip, grouped_attention.hip,
+// delta_rule.hip, routed_experts.hip, tile_gemm.hip).
 //
 // Every inner width is padded to whole 32-value groups (the state's key dimension to a power of two) by zero rows and
 // columns of the packed weights, so that the kernels see whole MFMA steps whatever sizes a model has.
@@ -14,7 +14,7 @@
 
 namespace xfthip {
 
-constexpr int kPageTokens = 64; // tokens of a page of the latent cache
+constexpr int kPageTokens = 64; // tokens of a page of the cache
 
 // One step: B segments (one a sequence), T tokens, back to back.  All pointers are device memory.
 struct StepView {
@@ -26,9 +26,16 @@ struct StepView {
     int table_stride;
 };
 
+// what stands in front of a sublayer: an RMS norm with weight w, or, with b set, tanh(alpha x) * w + b
+struct PlanNorm {
+    float *w = nullptr, *b = nullptr;
+    float alpha = 0.0f;
+};
+
 struct PlanLayer {
     xfthip_plan_layer s;
-    // latent attention: padded widths of a head's unrotated / rotated / value part, of the key and the query latent
+    // latent attention: padded widths of a head's unrotated / rotated / value part, of the key and the query latent;
+    // grouped attention: D and V, of the query / key and the value part of a head
     int D = 0, RD = 0, V = 0, R = 0, QR = 0;
     // delta rule: padded key / value width of a head, padded rank of the two gates and columns of one gate
     int KD = 0, VD = 0, rank = 0, gcols = 0;
@@ -36,15 +43,36 @@ struct PlanLayer {
     xfthip_weight_t in = nullptr, o = nullptr, gateup = nullptr, down = nullptr;
     // latent: queries from their latent; W_uk turned round (query -> latent), W_uk and W_uv (latent -> key / value)
     xfthip_weight_t uq = nullptr, absorb = nullptr, uk = nullptr, uv = nullptr;
-    float *q_norm = nullptr, *kv_norm = nullptr, *sink = nullptr;
+    float *q_norm = nullptr, *kv_norm = nullptr, *sink = nullptr; // (grouped attention: weights of the query and the key heads)
+    float value_share = 0.0f; // v_mix: lambda
+    bool first_values = false; // the layer whose values the others mix in
     float *cosT = nullptr, *sinT = nullptr; // [max positions][rot_dim / 2], shared by layers of the same rotation
     // delta rule: both gates' second projections (decay | output gate), filters [channels][taps], exp(A_log), ...
     xfthip_weight_t gates = nullptr;
     float *conv = nullptr, *decay = nullptr, *dt_bias = nullptr, *out_norm = nullptr;
-    // norm weights: 1 + w in front of a sublayer, (1 + w) * layer scale behind it
-    float *pre1 = nullptr, *post1 = nullptr, *pre2 = nullptr, *post2 = nullptr;
+    // routed experts: padded width, weights of one shape by expert and their device table ([experts] gate / up, [experts] down)
+    int eff = 0;
+    std::vector<xfthip_weight_t> egateup, edown;
+    GroupWeight *etable = nullptr;
+    xfthip_weight_t router = nullptr;
+    float *correction = nullptr;
+    // the token's side embedding: into the part's width, back, the norm's weight behind it
+    xfthip_weight_t side_gate = nullptr, side_proj = nullptr;
+    float *side_post = nullptr;
+    // in front of the sublayers (RMS: 1 + w), behind them in sandwich blocks ((1 + w) * layer scale)
+    PlanNorm pre1, pre2;
+    float *post1 = nullptr, *post2 = nullptr;
 
-    int row_in() const { return s.mixer == XFTHIP_MIXER_LATENT ? QR + R + RD : (2 * s.kv_heads * KD + s.heads * VD) + beta_cols() + 2 * rank; }
+    int row_in() const {
+        if (s.mixer == XFTHIP_MIXER_LATENT) return QR + R + RD;
+        if (s.mixer == XFTHIP_MIXER_GROUPED) return s.heads * D + s.kv_heads * (D + V);
+        return (2 * s.kv_heads * KD + s.heads * VD) + beta_cols() + 2 * rank;
+    }
+    bool paged() const { return s.mixer != XFTHIP_MIXER_DELTA; }
+    // elements a token takes in the page pool
+    size_t token_elems() const { return s.mixer == XFTHIP_MIXER_LATENT ? R + RD : (size_t)s.kv_heads * (D + V); }
+    int routes() const { return s.experts + s.identity; }
+    bool feeds_forward() const { return ff > 0 || s.experts > 0; }
     int beta_cols() const { return (s.heads + 31) / 32 * 32; }
     int channels() const { return 2 * s.kv_heads * KD + s.heads * VD; } // of the short convolution: q | k | v
 };
@@ -59,16 +87,79 @@ struct LayerRun {
 
 // x[t] = table[ids[t]] (bf16 table, ids clamped to the vocabulary)
 int plan_embed(const uint16_t *table, const int *ids, float *x, int T, int hidden, int vocab, hipStream_t st);
-// x += rms(y) * post (y may be null), then x += table[ids] (table may be null), then xn = rms(x) * pre (pre may be null).
-// Means over `width` of the `hidden` columns.  rows: xn row i comes from x row rows[i] (only without y and table).
-int plan_norm(int act, float *x, const float *y, const float *post, const uint16_t *table, const int *ids, int vocab, const float *pre, void *xn,
-        const int *rows, int T, int hidden, int width, float eps, hipStream_t st);
+// x += rms(y) * post (y may be null), then x += table[ids] (table may be null), then xn = pre(x) (pre.w may be null) and
+// xn2 = pre2(x) (pre2.w may be null; tanh norms only).  Means over `width` of the `hidden` columns.  rows: xn row i comes from x
+// row rows[i] (only without y and table).
+struct PlanNormArgs {
+    float *x;
+    const float *y, *post;
+    const uint16_t *table;
+    const int *ids;
+    int vocab;
+    PlanNorm pre, pre2;
+    void *xn, *xn2;
+    const int *rows;
+    int hidden, width;
+    float eps;
+};
+int plan_norm(int act, const PlanNormArgs &p, int T, hipStream_t st);
+// out[t][c] = gelu(z[t][c]) * table[ids[t]][first + c] (tanh form of the gelu), c < width; bf16 table [vocab][ld], ids clamped
+int plan_side_gate(int act, const float *z, const uint16_t *table, int ld, int first, const int *ids, int vocab, void *out, int T, int width,
+        hipStream_t st);
 
 // C[t][n] = sum_k A[t][block(n) * a_block_stride + k] W[k][n], block(n) = n / block_cols: a plain product of 32-bit
-// activations (block_cols = 0), or heads side by side.  BF16 weights; act_in / c_dtype XFTHIP_BF16 or XFTHIP_F32; glu: 1
-// the weight holds gate / up pairs (XFTHIP_WF_GATEUP), combined as clamped_glu.
-int tile_gemm(xfthip_weight_t w, int act_in, int M, const void *A, int lda, int block_cols, int a_block_stride, void *C, int ldc, int c_dtype,
-        int glu, float glu_limit, float glu_alpha, hipStream_t st);
+// activations (block_cols = 0), or heads side by side.  BF16 weights; act_in / c_dtype XFTHIP_BF16 or XFTHIP_F32.
+struct TileGemmArgs {
+    int M = 0;
+    const void *A = nullptr;
+    int lda = 0, block_cols = 0, a_block_stride = 0;
+    void *C = nullptr;
+    int ldc = 0, c_dtype = XFTHIP_F32;
+    bool add = false; // C += (fp32)
+    bool glu = false; // the weight holds gate / up pairs (XFTHIP_WF_GATEUP), combined as clamped_glu
+    float glu_limit = 0, glu_alpha = 0;
+    // C = gelu(product) * side[ids[t]][n] (as plan_side_gate)
+    const uint16_t *side = nullptr;
+    int side_ld = 0;
+    const int *side_ids = nullptr;
+    int side_vocab = 0;
+    // weights of one shape behind one launch, M rows at most each: records {rows, first row of A, first row of C} in device memory;
+    // a_rows (or null): row r of A is row a_rows[r]
+    const GroupWeight *group = nullptr;
+    int group_n = 0;
+    const int *group_rows = nullptr, *a_rows = nullptr;
+};
+int tile_gemm(xfthip_weight_t w, int act_in, const TileGemmArgs &a, hipStream_t st);
+
+// ---- routed experts
+struct RouteBuffers {
+    int *sel; // [T][top] router output of a choice
+    float *weight; // [T][top]
+    int *slot_row; // [T][top] row of a choice among the gathered rows; -1: an identity expert
+    int *row_token; // [T * top] token of a gathered row
+    int *group_rows; // [experts][3] records of the expert products
+};
+// softmax over a token's `routes` logits (row pitch ld), the `top` largest of score + correction, lists of tokens by expert
+int route_tokens(const float *logits, int ld, const float *correction, int T, int experts, int routes, int top, const RouteBuffers &b, hipStream_t st);
+// dst[t] = base[t] + sum over choices of weight * (expert output row, or h[t]); base, dst fp32 (base may be null or dst), h of the
+// activation type; narrow (or null): dst once more, of the activation type
+int combine_experts(int act, const float *base, const float *outputs, const void *h, int top, const RouteBuffers &b, float *dst, void *narrow, int T,
+        int hidden, hipStream_t st);
+
+// ---- grouped attention
+struct GroupedBuffers {
+    const void *a; // [T][row_in] of the activation type: q | k | v
+    void *q; // [T][heads][D]
+    void *pool; // pages: by key / value head [64][D] keys, then two blocks of 32 tokens [V][32] values
+    void *first_values; // [T][kv_heads][V]: written by the layer that says so, read by the others that mix
+};
+// norms and rotation of queries and keys, mixing of values, append to the pages
+int grouped_prepare(int act, const PlanLayer &L, const StepView &v, const GroupedBuffers &b, float eps, hipStream_t st);
+// out [T][heads][V]; hint: upper bound of the sequence lengths
+int grouped_attention(int act, const PlanLayer &L, const StepView &v, const void *q, const void *pool, void *out, int hint, float *part, size_t part_floats,
+        hipStream_t st);
+int grouped_split_count(const PlanLayer &L, int B, int longest, int hint);
+size_t grouped_part_floats(const PlanLayer &L);
 
 struct LatentCacheView {
     void *pool; // [pages][kPageTokens][R + RD] of the activation type: normalised latent | rotated shared key part
@@ -116,7 +207,9 @@ struct xfthip_plan {
     std::vector<xfthip::LayerRun> runs;
     int hidden = 0; // width padded to whole 32-value groups
     uint16_t *embedding = nullptr; // [vocab][hidden] bf16
-    float *final_norm = nullptr; // (1 + w) * logit scale
+    xfthip::PlanNorm final_norm; // times the logit scale
+    uint16_t *side_embedding = nullptr; // [vocab][layers * side_pad] bf16
+    int side_pad = 0;
     xfthip_weight_t head = nullptr;
     struct Tensor {
         std::vector<uint16_t> data;
@@ -135,8 +228,8 @@ struct PlanState {
     std::vector<PlanLayer> layers; // the plan's, with this model's rotation tables
     int act = XFTHIP_BF16, esz = 2;
     int slots = 0;
-    // by layer run: page pool of a latent attention, state and convolution inputs of a delta rule
-    std::vector<LatentCacheView> cache;
+    // by layer run: page pool of an attention, state and convolution inputs of a delta rule
+    std::vector<void *> cache;
     std::vector<float *> state;
     std::vector<void *> conv_state;
     // pages: free ones, those of every slot in position order, and the device table [slots][table_stride]
@@ -159,6 +252,10 @@ struct PlanState {
     // scratch (activation type unless float)
     void *xn = nullptr, *a = nullptr, *cq = nullptr, *q = nullptr, *qa = nullptr, *oc = nullptr, *ov = nullptr, *h = nullptr, *on = nullptr;
     float *y = nullptr, *gates = nullptr, *dq = nullptr, *dk = nullptr, *dqk = nullptr, *dg = nullptr, *dv = nullptr, *dbeta = nullptr, *do_ = nullptr;
+    void *xn2 = nullptr, *first_values = nullptr, *side = nullptr, *narrow = nullptr;
+    float *router_logits = nullptr, *expert_out = nullptr, *side_z = nullptr;
+    void *eh = nullptr;
+    RouteBuffers route {};
     void *rows = nullptr, *kx = nullptr, *vx = nullptr; // gathered latents, keys and values of a long segment's context
     float *part = nullptr; // split contexts
     size_t part_floats = 0;

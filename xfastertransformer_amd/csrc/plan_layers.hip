@@ -1,6 +1,6 @@
 // Embedding and norms of layer plans: the norm behind a sublayer, the residual sum, the embedding output that joins in
-// front of a further pass of a loop, and the norm in front of the next sublayer are one kernel.
-#include "plan.h"
+// front of a further pass of a loop, and the norms in front of the next sublayers are one kernel; the gate of the side embedding.
+#include "plan_dev.h"
 
 namespace xfthip {
 
@@ -12,18 +12,6 @@ __global__ void plan_embed_kernel(const uint16_t *__restrict__ table, const int 
     const uint16_t *row = table + (size_t)id * hidden;
     for (int c = threadIdx.x; c < hidden; c += blockDim.x) x[(size_t)blockIdx.x * hidden + c] = bf16_to_f32(row[c]);
 }
-
-struct NormParams {
-    float *x;
-    const float *y, *post;
-    const uint16_t *table;
-    const int *ids, *rows;
-    int vocab;
-    const float *pre;
-    void *xn;
-    int hidden, width;
-    float eps;
-};
 
 template <int NT>
 __device__ inline float block_sum(float v, float *part) {
@@ -39,7 +27,7 @@ __device__ inline float block_sum(float v, float *part) {
 
 // one token a workgroup of NT threads; the row stays in registers (CH float4 a thread), every load is requested before the first use
 template <bool BF16, int CH, int NT>
-__global__ __launch_bounds__(NT) void plan_norm_kernel(NormParams p) {
+__global__ __launch_bounds__(NT) void plan_norm_kernel(PlanNormArgs p) {
     __shared__ float part[2 * NT / 64];
     const int t = blockIdx.x;
     const float *xr = p.x + (size_t)(p.rows ? p.rows[t] : t) * p.hidden;
@@ -52,7 +40,7 @@ __global__ __launch_bounds__(NT) void plan_norm_kernel(NormParams p) {
         x[c] = in ? *(const f32x4 *)(xr + col) : zero;
         y[c] = in && p.y ? *(const f32x4 *)(p.y + (size_t)t * p.hidden + col) : zero;
         wpost[c] = in && p.y ? *(const f32x4 *)(p.post + col) : zero;
-        wpre[c] = in && p.pre ? *(const f32x4 *)(p.pre + col) : zero;
+        wpre[c] = in && p.pre.w && !p.pre.b ? *(const f32x4 *)(p.pre.w + col) : zero;
     }
     if (p.table) {
         int id = p.ids[t];
@@ -89,7 +77,25 @@ __global__ __launch_bounds__(NT) void plan_norm_kernel(NormParams p) {
             if (col < p.hidden) *(f32x4 *)(p.x + (size_t)t * p.hidden + col) = x[c];
         }
     }
-    if (!p.pre) return;
+    if (!p.pre.w) return;
+    if (p.pre.b) { // tanh norms: one value at a time, up to two of them
+#pragma unroll
+        for (int k = 0; k < 2; ++k) {
+            const PlanNorm &n = k ? p.pre2 : p.pre;
+            if (!n.w) break;
+#pragma unroll
+            for (int c = 0; c < CH; ++c) {
+                const int col = (c * NT + threadIdx.x) * 4;
+                if (col >= p.hidden) continue;
+                const f32x4 w = *(const f32x4 *)(n.w + col), b = *(const f32x4 *)(n.b + col);
+                f32x4 v;
+#pragma unroll
+                for (int i = 0; i < 4; ++i) v[i] = fmaf(tanhf(n.alpha * x[c][i]), w[i], b[i]);
+                put4<BF16>(k ? p.xn2 : p.xn, (size_t)t * p.hidden + col, v);
+            }
+        }
+        return;
+    }
     float sq = 0.0f;
 #pragma unroll
     for (int c = 0; c < CH; ++c)
@@ -101,17 +107,36 @@ __global__ __launch_bounds__(NT) void plan_norm_kernel(NormParams p) {
         const int col = (c * NT + threadIdx.x) * 4;
         if (col >= p.hidden) continue;
         const f32x4 v = x[c] * r * wpre[c];
-        const size_t at = (size_t)t * p.hidden + col;
-        if constexpr (BF16)
-            *(uint2 *)((uint16_t *)p.xn + at) = make_uint2(f32_to_bf16_ref(v[0]) | ((uint32_t)f32_to_bf16_ref(v[1]) << 16),
-                    f32_to_bf16_ref(v[2]) | ((uint32_t)f32_to_bf16_ref(v[3]) << 16));
-        else
-            *(f32x4 *)((float *)p.xn + at) = v;
+        put4<BF16>(p.xn, (size_t)t * p.hidden + col, v);
     }
 }
 
+struct SideParams {
+    const float *z;
+    const uint16_t *table;
+    int ld, first;
+    const int *ids;
+    int vocab, T, width;
+    void *out;
+};
 template <bool BF16>
-int launch_norm(const NormParams &p, int T, hipStream_t st) {
+__global__ __launch_bounds__(256) void side_gate_kernel(SideParams p) {
+    const size_t i = ((size_t)blockIdx.x * 256 + threadIdx.x) * 4;
+    if (i >= (size_t)p.T * p.width) return;
+    const int t = (int)(i / p.width), c = (int)(i % p.width);
+    int id = p.ids[t];
+    id = id < 0 ? 0 : (id >= p.vocab ? p.vocab - 1 : id);
+    const f32x4 z = *(const f32x4 *)(p.z + i);
+    const uint2 e = *(const uint2 *)(p.table + (size_t)id * p.ld + p.first + c);
+    const f32x4 emb = {u2f(e.x << 16), u2f(e.x & 0xFFFF0000u), u2f(e.y << 16), u2f(e.y & 0xFFFF0000u)};
+    f32x4 v;
+#pragma unroll
+    for (int k = 0; k < 4; ++k) v[k] = gelu_tanh(z[k]) * emb[k];
+    put4<BF16>(p.out, i, v);
+}
+
+template <bool BF16>
+int launch_norm(const PlanNormArgs &p, int T, hipStream_t st) {
     const int ch = (p.hidden + 1023) / 1024;
     XFT_REQUIRE(ch <= 16, "plan_norm: hidden size %d above 16384", p.hidden);
     // few rows: the kernel is one chain of latencies, shorter with the row spread over more threads
@@ -135,11 +160,20 @@ int plan_embed(const uint16_t *table, const int *ids, float *x, int T, int hidde
     return 0;
 }
 
-int plan_norm(int act, float *x, const float *y, const float *post, const uint16_t *table, const int *ids, int vocab, const float *pre, void *xn,
-        const int *rows, int T, int hidden, int width, float eps, hipStream_t st) {
-    XFT_REQUIRE(T > 0 && x && hidden % 4 == 0 && width <= hidden && (!rows || (!y && !table)), "plan_norm: bad argument");
-    const NormParams p = {x, y, post, table, ids, rows, vocab, pre, xn, hidden, width, eps};
+int plan_norm(int act, const PlanNormArgs &p, int T, hipStream_t st) {
+    XFT_REQUIRE(T > 0 && p.x && p.hidden % 4 == 0 && p.width <= p.hidden && (!p.rows || (!p.y && !p.table)) && (!p.pre2.w || p.pre.b), "plan_norm: bad argument");
     return act == XFTHIP_BF16 ? launch_norm<true>(p, T, st) : launch_norm<false>(p, T, st);
+}
+
+int plan_side_gate(int act, const float *z, const uint16_t *table, int ld, int first, const int *ids, int vocab, void *out, int T, int width,
+        hipStream_t st) {
+    XFT_REQUIRE(T > 0 && width % 4 == 0 && ld % 4 == 0 && first % 4 == 0, "plan_side_gate: bad argument");
+    const SideParams p = {z, table, ld, first, ids, vocab, T, width, out};
+    const dim3 grid((unsigned)(((size_t)T * width / 4 + 255) / 256));
+    if (act == XFTHIP_BF16) hipLaunchKernelGGL(side_gate_kernel<true>, grid, dim3(256), 0, st, p);
+    else hipLaunchKernelGGL(side_gate_kernel<false>, grid, dim3(256), 0, st, p);
+    XFT_CHECK_HIP(hipGetLastError());
+    return 0;
 }
 
 } // namespace xfthip

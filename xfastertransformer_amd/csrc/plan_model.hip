@@ -68,33 +68,71 @@ __global__ void plan_fill_kernel(int *p, int n, int v) {
     if (i < n) p[i] = v;
 }
 
-// rotation tables [positions][dims / 2]: angles in double, as far apart as positions can be
-int rotation_tables(double base, int dims, int positions, float **cosT, float **sinT) {
-    const int half = dims / 2;
-    std::vector<float> c((size_t)positions * half), s((size_t)positions * half);
+// Frequency of pair i of a rotation and the factor on cos and sin.  Context extension: pairs that turn fewer than `slow` times
+// within the original context have their frequency divided by the factor, those above `fast` keep it, a ramp over i between.
+double rotation_frequency(const xfthip_plan_layer &s, int i) {
+    const double f = pow(s.rot_base, -2.0 * i / s.rot_dim);
+    if (s.rot_factor <= 0.0) return f;
+    auto pair_at = [&](double turns) { return s.rot_dim * log(s.rot_original / (2.0 * M_PI * turns)) / (2.0 * log(s.rot_base)); };
+    const double lo = std::max(floor(pair_at(s.rot_fast)), 0.0), hi = std::min(ceil(pair_at(s.rot_slow)), s.rot_dim - 1.0);
+    const double ramp = std::min(std::max((i - lo) / std::max(hi - lo, 0.001), 0.0), 1.0);
+    return f / s.rot_factor * ramp + f * (1.0 - ramp);
+}
+double rotation_magnitude(const xfthip_plan_layer &s) { return s.rot_factor > 0.0 ? 0.1 * log(s.rot_factor) + 1.0 : 1.0; }
+
+// rotation tables [positions][rot_dim / 2]: angles in double, as far apart as positions can be
+int rotation_tables(const xfthip_plan_layer &s, int positions, float **cosT, float **sinT) {
+    const int half = s.rot_dim / 2;
+    const double mul = rotation_magnitude(s);
+    std::vector<float> c((size_t)positions * half), sn((size_t)positions * half);
     for (int i = 0; i < half; ++i) {
-        const double f = pow(base, -2.0 * i / dims);
-        for (int p = 0; p < positions; ++p) c[(size_t)p * half + i] = (float)cos(p * f), s[(size_t)p * half + i] = (float)sin(p * f);
+        const double f = rotation_frequency(s, i);
+        for (int p = 0; p < positions; ++p) c[(size_t)p * half + i] = (float)(cos(p * f) * mul), sn[(size_t)p * half + i] = (float)(sin(p * f) * mul);
     }
     XFT_CHECK_HIP(hipMalloc((void **)cosT, c.size() * 4 + 16));
-    XFT_CHECK_HIP(hipMalloc((void **)sinT, s.size() * 4 + 16));
+    XFT_CHECK_HIP(hipMalloc((void **)sinT, sn.size() * 4 + 16));
     XFT_CHECK_HIP(hipMemcpy(*cosT, c.data(), c.size() * 4, hipMemcpyHostToDevice));
-    XFT_CHECK_HIP(hipMemcpy(*sinT, s.data(), s.size() * 4, hipMemcpyHostToDevice));
+    XFT_CHECK_HIP(hipMemcpy(*sinT, sn.data(), sn.size() * 4, hipMemcpyHostToDevice));
     return 0;
 }
 
 int plan_gemm(xfthip_model *m, xfthip_weight_t w, int M, const void *A, int lda, void *C, int ldc, int c_dtype, hipStream_t st) {
-    if (m->plan->act == XFTHIP_F32) return tile_gemm(w, XFTHIP_F32, M, A, lda, 0, 0, C, ldc, c_dtype, 0, 0, 0, st);
+    if (m->plan->act == XFTHIP_F32) {
+        TileGemmArgs a;
+        a.M = M, a.A = A, a.lda = lda, a.C = C, a.ldc = ldc, a.c_dtype = c_dtype;
+        return tile_gemm(w, XFTHIP_F32, a, st);
+    }
     return xfthip_gemm(w, M, A, lda, C, ldc, c_dtype, XFTHIP_EPI_NONE, nullptr, nullptr, 0, XFTHIP_F32, 1.0f, st);
+}
+
+// a sublayer's last product: into y, or, in parallel blocks, added to the residual
+int plan_gemm_out(xfthip_model *m, xfthip_weight_t w, int M, const void *A, int lda, hipStream_t st) {
+    const PlanState &p = *m->plan;
+    const int hidden = m->cfg.hidden;
+    if (p.plan->cfg.block != XFTHIP_BLOCK_PARALLEL) return plan_gemm(m, w, M, A, lda, p.y, hidden, XFTHIP_F32, st);
+    if (p.act == XFTHIP_F32) {
+        TileGemmArgs a;
+        a.M = M, a.A = A, a.lda = lda, a.C = m->x, a.ldc = hidden, a.add = true;
+        return tile_gemm(w, XFTHIP_F32, a, st);
+    }
+    return xfthip_gemm(w, M, A, lda, m->x, hidden, XFTHIP_F32, XFTHIP_EPI_RESIDENTIAL, nullptr, m->x, hidden, XFTHIP_F32, 1.0f, st);
+}
+
+// heads side by side (block_cols output columns a head, a_block_stride input columns apart)
+int plan_gemm_heads(int act, xfthip_weight_t w, int M, const void *A, int lda, int block_cols, int a_block_stride, void *C, int ldc, int c_dtype, hipStream_t st) {
+    TileGemmArgs a;
+    a.M = M, a.A = A, a.lda = lda, a.block_cols = block_cols, a.a_block_stride = a_block_stride, a.C = C, a.ldc = ldc, a.c_dtype = c_dtype;
+    return tile_gemm(w, act, a, st);
 }
 
 int run_latent(xfthip_model *m, const PlanLayer &L, int run, const StepView &v, hipStream_t st) {
     PlanState &p = *m->plan;
     const int T = v.T, H = L.s.heads, act = p.act, hidden = m->cfg.hidden;
     const int qcols = H * (L.D + L.RD);
+    const LatentCacheView cache = {p.cache[run], L.R, L.RD};
     int rc;
     if ((rc = plan_gemm(m, L.in, T, p.xn, hidden, p.a, L.row_in(), act, st))) return rc;
-    if ((rc = latent_prepare(act, L, v, p.a, p.cq, p.cache[run], m->cfg.rms_eps, st))) return rc;
+    if ((rc = latent_prepare(act, L, v, p.a, p.cq, cache, m->cfg.rms_eps, st))) return rc;
     if ((rc = plan_gemm(m, L.uq, T, p.cq, L.QR, p.q, qcols, act, st))) return rc;
     if ((rc = latent_rotate_q(act, L, v, p.q, st))) return rc;
     // long segments one by one in the expanded form; the others, as far as they are neighbours, together in the absorbed one
@@ -102,12 +140,12 @@ int run_latent(xfthip_model *m, const PlanLayer &L, int run, const StepView &v, 
     const char *q = (const char *)p.q;
     int longest = 0, short_from = -1;
     auto absorb = [&](int from, int to) {
-        return tile_gemm(L.absorb, act, to - from, q + (size_t)from * qcols * p.esz, qcols, L.R, L.D + L.RD, (char *)p.qa + (size_t)from * H * L.R * p.esz, H * L.R,
-                act, 0, 0, 0, st);
+        return plan_gemm_heads(act, L.absorb, to - from, q + (size_t)from * qcols * p.esz, qcols, L.R, L.D + L.RD, (char *)p.qa + (size_t)from * H * L.R * p.esz,
+                H * L.R, act, st);
     };
     auto to_values = [&](int from, int to) {
-        return tile_gemm(L.uv, act, to - from, (char *)p.oc + (size_t)from * H * L.R * p.esz, H * L.R, L.V, L.R, (char *)p.ov + (size_t)from * H * L.V * p.esz,
-                H * L.V, act, 0, 0, 0, st);
+        return plan_gemm_heads(act, L.uv, to - from, (char *)p.oc + (size_t)from * H * L.R * p.esz, H * L.R, L.V, L.R,
+                (char *)p.ov + (size_t)from * H * L.V * p.esz, H * L.V, act, st);
     };
     std::vector<std::pair<int, int>> spans; // token ranges of the absorbed form
     for (size_t i = 0; i < B; ++i) {
@@ -123,7 +161,7 @@ int run_latent(xfthip_model *m, const PlanLayer &L, int run, const StepView &v, 
             short_from = -1;
         }
         if (!expand) continue;
-        if ((rc = latent_gather(v, p.seg_row_host[i], from, rows, p.cache[run], p.rows, st))) return rc;
+        if ((rc = latent_gather(v, p.seg_row_host[i], from, rows, cache, p.rows, st))) return rc;
         if ((rc = xfthip_gemm(L.uk, rows, p.rows, L.R + L.RD, p.kx, H * L.D, XFTHIP_BF16, XFTHIP_EPI_NONE, nullptr, nullptr, 0, XFTHIP_F32, 1.0f, st))) return rc;
         if ((rc = xfthip_gemm(L.uv, rows, p.rows, L.R + L.RD, p.vx, H * L.V, XFTHIP_BF16, XFTHIP_EPI_NONE, nullptr, nullptr, 0, XFTHIP_F32, 1.0f, st))) return rc;
         if ((rc = latent_expanded(L, off, start, n, from, p.q, p.kx, p.vx, p.rows, p.ov, st))) return rc;
@@ -131,11 +169,11 @@ int run_latent(xfthip_model *m, const PlanLayer &L, int run, const StepView &v, 
     if (!spans.empty()) {
         for (auto &s : spans)
             if ((rc = absorb(s.first, s.second))) return rc;
-        if ((rc = latent_attention(act, L, v, longest, p.qa, p.q, p.oc, p.cache[run], m->len_hint, p.part, p.part_floats, st))) return rc;
+        if ((rc = latent_attention(act, L, v, longest, p.qa, p.q, p.oc, cache, m->len_hint, p.part, p.part_floats, st))) return rc;
         for (auto &s : spans)
             if ((rc = to_values(s.first, s.second))) return rc;
     }
-    return plan_gemm(m, L.o, T, p.ov, H * L.V, p.y, hidden, XFTHIP_F32, st);
+    return plan_gemm_out(m, L.o, T, p.ov, H * L.V, st);
 }
 
 int run_delta(xfthip_model *m, const PlanLayer &L, int run, const StepView &v, hipStream_t st) {
@@ -145,48 +183,146 @@ int run_delta(xfthip_model *m, const PlanLayer &L, int run, const StepView &v, h
     const DeltaBuffers b = {p.a, p.gates, p.dq, p.dk, p.dqk, p.dg, p.dv, p.dbeta, p.do_, p.on, p.state[run], p.conv_state[run]};
     if ((rc = plan_gemm(m, L.in, T, p.xn, hidden, p.a, ld, act, st))) return rc;
     const int first = L.channels() + L.beta_cols();
-    if ((rc = tile_gemm(L.gates, act, T, (const char *)p.a + (size_t)first * p.esz, ld, L.gcols, L.rank, p.gates, 2 * L.gcols, XFTHIP_F32, 0, 0, 0, st)))
-        return rc;
+    if ((rc = plan_gemm_heads(act, L.gates, T, (const char *)p.a + (size_t)first * p.esz, ld, L.gcols, L.rank, p.gates, 2 * L.gcols, XFTHIP_F32, st))) return rc;
     if ((rc = delta_prepare(act, L, v, b, st))) return rc;
     if ((rc = delta_scan(L, v, b, st))) return rc;
     if ((rc = delta_output(act, L, v, b, m->cfg.rms_eps, st))) return rc;
-    return plan_gemm(m, L.o, T, p.on, L.s.heads * L.VD, p.y, hidden, XFTHIP_F32, st);
+    return plan_gemm_out(m, L.o, T, p.on, L.s.heads * L.VD, st);
+}
+
+int run_grouped(xfthip_model *m, const PlanLayer &L, int run, const StepView &v, hipStream_t st) {
+    PlanState &p = *m->plan;
+    const int T = v.T, act = p.act;
+    int rc;
+    const GroupedBuffers b = {p.a, p.q, p.cache[run], p.first_values};
+    if ((rc = plan_gemm(m, L.in, T, p.xn, m->cfg.hidden, p.a, L.row_in(), act, st))) return rc;
+    if ((rc = grouped_prepare(act, L, v, b, m->cfg.rms_eps, st))) return rc;
+    if ((rc = grouped_attention(act, L, v, p.q, p.cache[run], p.ov, m->len_hint, p.part, p.part_floats, st))) return rc;
+    return plan_gemm_out(m, L.o, T, p.ov, L.s.heads * L.V, st);
+}
+
+// gate and up projections of a dense or shared feed-forward, combined -> h
+int run_gateup(xfthip_model *m, const PlanLayer &L, int T, const void *in, hipStream_t st) {
+    PlanState &p = *m->plan;
+    const int hidden = m->cfg.hidden;
+    if (p.act != XFTHIP_F32) return xfthip_gemm_gateup_clamped(L.gateup, T, in, hidden, p.h, L.ff, XFTHIP_BF16, L.s.glu_limit, L.s.glu_alpha, st);
+    TileGemmArgs a;
+    a.M = T, a.A = in, a.lda = hidden, a.C = p.h, a.ldc = L.ff, a.c_dtype = XFTHIP_F32, a.glu = true, a.glu_limit = L.s.glu_limit, a.glu_alpha = L.s.glu_alpha;
+    return tile_gemm(L.gateup, XFTHIP_F32, a, st);
+}
+
+// the products of all chosen experts: in -> eh -> expert_out, rows by the lists of the routing
+int run_experts(xfthip_model *m, const PlanLayer &L, int T, const void *in, hipStream_t st) {
+    PlanState &p = *m->plan;
+    const xfthip_plan_layer &s = L.s;
+    const int hidden = m->cfg.hidden, E = s.experts;
+    const int most = s.top < E ? s.top : E; // choices of a token that reach an expert
+    const RouteBuffers &r = p.route;
+    int rc;
+    if (p.act != XFTHIP_F32) {
+        if ((rc = gemm_grouped_rows_dev(L.egateup.data(), E, L.etable, most * T, T, r.group_rows, 3, in, hidden, p.eh, L.eff, XFTHIP_BF16, st, r.row_token,
+                     s.expert_limit, s.glu_alpha)))
+            return rc;
+        return gemm_grouped_rows_dev(L.edown.data(), E, L.etable + E, most * T, T, r.group_rows, 3, p.eh, L.eff, p.expert_out, hidden, XFTHIP_F32, st);
+    }
+    TileGemmArgs a;
+    a.M = T, a.A = in, a.lda = hidden, a.C = p.eh, a.ldc = L.eff, a.c_dtype = XFTHIP_F32, a.glu = true, a.glu_limit = s.expert_limit, a.glu_alpha = s.glu_alpha;
+    a.group = L.etable, a.group_n = E, a.group_rows = r.group_rows, a.a_rows = r.row_token;
+    if ((rc = tile_gemm(L.egateup[0], XFTHIP_F32, a, st))) return rc;
+    TileGemmArgs d;
+    d.M = T, d.A = p.eh, d.lda = L.eff, d.C = p.expert_out, d.ldc = hidden, d.group = L.etable + E, d.group_n = E, d.group_rows = r.group_rows;
+    return tile_gemm(L.edown[0], XFTHIP_F32, d, st);
+}
+
+// The feed-forward: dense, or routed experts beside an optional shared one.  Its result goes where plan_gemm_out puts results; in
+// (activation type) is its input, narrow (or null) receives the residual behind a parallel block, of the activation type.
+int run_feed_forward(xfthip_model *m, const PlanLayer &L, int T, const void *in, void *narrow, hipStream_t st) {
+    PlanState &p = *m->plan;
+    const bool parallel = p.plan->cfg.block == XFTHIP_BLOCK_PARALLEL;
+    const int hidden = m->cfg.hidden;
+    int rc;
+    if (L.ff > 0) {
+        if ((rc = run_gateup(m, L, T, in, st))) return rc;
+        if ((rc = plan_gemm_out(m, L.down, T, p.h, L.ff, st))) return rc;
+    }
+    float *dst = parallel ? m->x : p.y;
+    if (L.s.experts > 0) {
+        const int ld = pad32(L.routes());
+        if ((rc = plan_gemm(m, L.router, T, in, hidden, p.router_logits, ld, XFTHIP_F32, st))) return rc;
+        if ((rc = route_tokens(p.router_logits, ld, L.correction, T, L.s.experts, L.routes(), L.s.top, p.route, st))) return rc;
+        if ((rc = run_experts(m, L, T, in, st))) return rc;
+        return combine_experts(p.act, parallel || L.ff > 0 ? dst : nullptr, p.expert_out, in, L.s.top, p.route, dst, narrow, T, hidden, st);
+    }
+    return narrow ? combine_experts(p.act, dst, nullptr, nullptr, 0, p.route, dst, narrow, T, hidden, st) : 0;
+}
+
+// y = P (gelu(G x) * e) of the token's side embedding; x: the residual in the activation type
+int run_side(xfthip_model *m, const PlanLayer &L, int layer, int T, const void *x, hipStream_t st) {
+    PlanState &p = *m->plan;
+    const xfthip_plan &plan = *p.plan;
+    const int hidden = m->cfg.hidden, pad = plan.side_pad, ld = pad * plan.cfg.layers;
+    int rc;
+    if (p.act == XFTHIP_F32 || T <= 32) { // the gate in the product's epilogue
+        TileGemmArgs a;
+        a.M = T, a.A = x, a.lda = hidden, a.C = p.side, a.ldc = pad, a.c_dtype = p.act;
+        a.side = plan.side_embedding + (size_t)layer * pad, a.side_ld = ld, a.side_ids = p.ids, a.side_vocab = m->cfg.vocab;
+        if ((rc = tile_gemm(L.side_gate, p.act, a, st))) return rc;
+    } else {
+        if ((rc = plan_gemm(m, L.side_gate, T, x, hidden, p.side_z, pad, XFTHIP_F32, st))) return rc;
+        if ((rc = plan_side_gate(p.act, p.side_z, plan.side_embedding, ld, layer * pad, p.ids, m->cfg.vocab, p.side, T, pad, st))) return rc;
+    }
+    return plan_gemm(m, L.side_proj, T, p.side, pad, p.y, hidden, XFTHIP_F32, st);
 }
 
 // all layer runs over the step's tokens, whose embeddings are in m->x
 int plan_layers(xfthip_model *m, const StepView &v, hipStream_t st) {
     PlanState &p = *m->plan;
     const xfthip_plan &plan = *p.plan;
-    const int T = v.T, hidden = m->cfg.hidden, width = plan.cfg.hidden, vocab = m->cfg.vocab;
-    const float eps = m->cfg.rms_eps;
+    const int T = v.T, hidden = m->cfg.hidden;
+    const bool parallel = plan.cfg.block == XFTHIP_BLOCK_PARALLEL;
     const int nruns = (int)plan.runs.size();
     int rc;
-    auto norm = [&](const float *y, const float *post, bool again, const float *pre) {
-        return plan_norm(p.act, m->x, y, post, again ? plan.embedding : nullptr, p.ids, vocab, pre, p.xn, nullptr, T, hidden, width, eps, st);
+    // next: the layer whose first norms follow, or null
+    auto norm = [&](const float *y, const float *post, bool again, const PlanNorm &pre, const PlanNorm &pre2) {
+        const PlanNormArgs a = {m->x, y, post, again ? plan.embedding : nullptr, p.ids, m->cfg.vocab, pre, pre2, p.xn, p.xn2, nullptr, hidden, plan.cfg.hidden,
+                m->cfg.rms_eps};
+        return plan_norm(p.act, a, T, st);
     };
-    if ((rc = norm(nullptr, nullptr, plan.runs[0].add_embedding, p.layers[plan.runs[0].layer].pre1))) return rc;
+    const PlanNorm none;
+    auto enter = [&](const float *y, const float *post, bool again, const PlanLayer *next) {
+        return norm(y, post, again, next ? next->pre1 : none, next && parallel ? next->pre2 : none);
+    };
+    if ((rc = enter(nullptr, nullptr, plan.runs[0].add_embedding, &p.layers[plan.runs[0].layer]))) return rc;
     for (int r = 0; r < nruns; ++r) {
         const PlanLayer &L = p.layers[plan.runs[r].layer];
         const bool last = r + 1 == nruns;
         // (a traced run keeps the embedding of a further pass apart, so that the trace shows the layer's own result)
-        const bool again = !last && plan.runs[r + 1].add_embedding;
-        const float *next = last ? nullptr : p.layers[plan.runs[r + 1].layer].pre1;
-        rc = L.s.mixer == XFTHIP_MIXER_LATENT ? run_latent(m, L, r, v, st) : run_delta(m, L, r, v, st);
+        const bool again = !last && plan.runs[r + 1].add_embedding, join = again && !p.trace;
+        const PlanLayer *next = last ? nullptr : &p.layers[plan.runs[r + 1].layer], *then = p.trace ? nullptr : next;
+        switch (L.s.mixer) {
+            case XFTHIP_MIXER_LATENT: rc = run_latent(m, L, r, v, st); break;
+            case XFTHIP_MIXER_GROUPED: rc = run_grouped(m, L, r, v, st); break;
+            default: rc = run_delta(m, L, r, v, st);
+        }
         if (rc) return rc;
-        const bool ff = L.ff > 0;
-        if ((rc = norm(p.y, L.post1, !ff && again && !p.trace, ff ? L.pre2 : (p.trace ? nullptr : next)))) return rc;
-        if (ff) {
-            if (p.act == XFTHIP_F32)
-                rc = tile_gemm(L.gateup, XFTHIP_F32, T, p.xn, hidden, 0, 0, p.h, L.ff, XFTHIP_F32, 1, L.s.glu_limit, L.s.glu_alpha, st);
-            else
-                rc = xfthip_gemm_gateup_clamped(L.gateup, T, p.xn, hidden, p.h, L.ff, XFTHIP_BF16, L.s.glu_limit, L.s.glu_alpha, st);
-            if (rc) return rc;
-            if ((rc = plan_gemm(m, L.down, T, p.h, L.ff, p.y, hidden, XFTHIP_F32, st))) return rc;
-            if ((rc = norm(p.y, L.post2, again && !p.trace, p.trace ? nullptr : next))) return rc;
+        const bool ff = L.feeds_forward(), side = plan.cfg.side_dim > 0;
+        const void *narrow = p.act == XFTHIP_F32 ? (const void *)m->x : p.narrow; // what the side embedding's gate reads
+        void *narrow_out = side && p.act != XFTHIP_F32 ? p.narrow : nullptr;
+        if (parallel) {
+            if ((ff || narrow_out) && (rc = run_feed_forward(m, L, T, p.xn2, narrow_out, st))) return rc;
+            if (side && (rc = run_side(m, L, plan.runs[r].layer, T, narrow, st))) return rc;
+            if (!last || side)
+                if ((rc = enter(side ? p.y : nullptr, L.side_post, join, then))) return rc;
+        } else {
+            if ((rc = norm(p.y, L.post1, !ff && join, ff ? L.pre2 : then ? then->pre1 : none, none))) return rc;
+            if (ff) {
+                if ((rc = run_feed_forward(m, L, T, p.xn, nullptr, st))) return rc;
+                if ((rc = enter(p.y, L.post2, join, then))) return rc;
+            }
         }
         if (p.trace) {
             XFT_CHECK_HIP(hipMemcpyAsync(p.trace_buf + (size_t)r * T * hidden, m->x, (size_t)T * hidden * 4, hipMemcpyDeviceToDevice, st));
-            if (!last && (rc = norm(nullptr, nullptr, again, next))) return rc;
+            if (!last && (rc = enter(nullptr, nullptr, again, next))) return rc;
         }
     }
     return 0;
@@ -288,8 +424,8 @@ int plan_head(xfthip_model *m, const int *rows_dev, int n, int at, hipStream_t s
     PlanState &p = *m->plan;
     const xfthip_plan &plan = *p.plan;
     const xfthip_model_config &c = m->cfg;
-    if (int rc = plan_norm(p.act, m->x, nullptr, nullptr, nullptr, nullptr, c.vocab, plan.final_norm, p.xn, rows_dev, n, c.hidden, plan.cfg.hidden, c.rms_eps, st))
-        return rc;
+    const PlanNormArgs a = {m->x, nullptr, nullptr, nullptr, nullptr, c.vocab, plan.final_norm, {}, p.xn, nullptr, rows_dev, c.hidden, plan.cfg.hidden, c.rms_eps};
+    if (int rc = plan_norm(p.act, a, n, st)) return rc;
     return plan_gemm(m, plan.head, n, p.xn, c.hidden, m->logits + (size_t)at * c.vocab, c.vocab, XFTHIP_F32, st);
 }
 
@@ -361,6 +497,7 @@ int plan_decode_splits(xfthip_model *m, int B, int hint) {
     int s = 0; // the split counts of the attentions, as far as a recorded step depends on them
     for (auto &L : m->plan->layers)
         if (L.s.mixer == XFTHIP_MIXER_LATENT) s = s * 31 + latent_split_count(L, B, 1, hint);
+        else if (L.s.mixer == XFTHIP_MIXER_GROUPED) s = s * 31 + grouped_split_count(L, B, 1, hint);
     return s;
 }
 
@@ -384,8 +521,8 @@ int plan_reorder(xfthip_model *m, const int *dst, const int *src, int n, hipStre
         const PlanLayer &L = p.layers[p.plan->runs[r].layer];
         size_t need = 0;
         for (int i = 0; i < n; ++i)
-            need += L.s.mixer == XFTHIP_MIXER_LATENT ? from[i].size() * (size_t)kPageTokens * (L.R + L.RD) * p.esz
-                                                     : ((size_t)L.s.heads * L.VD * L.KD * 4 + (size_t)(L.s.taps - 1) * L.channels() * p.esz);
+            need += L.paged() ? from[i].size() * kPageTokens * L.token_elems() * p.esz
+                              : ((size_t)L.s.heads * L.VD * L.KD * 4 + (size_t)(L.s.taps - 1) * L.channels() * p.esz);
         bytes = std::max(bytes, need);
     }
     char *stage = nullptr;
@@ -402,10 +539,10 @@ int plan_reorder(xfthip_model *m, const int *dst, const int *src, int n, hipStre
         for (int write = 0; write < 2; ++write) {
             size_t at = 0;
             for (int i = 0; i < n; ++i) {
-                if (L.s.mixer == XFTHIP_MIXER_LATENT) {
-                    const size_t page = (size_t)kPageTokens * (L.R + L.RD) * p.esz;
+                if (L.paged()) {
+                    const size_t page = kPageTokens * L.token_elems() * p.esz;
                     for (size_t k = 0; k < from[i].size(); ++k, at += page) {
-                        char *pool = (char *)p.cache[r].pool;
+                        char *pool = (char *)p.cache[r];
                         if (write) copy(pool + (size_t)p.held[dst[i]][k] * page, stage + at, page);
                         else copy(stage + at, pool + (size_t)from[i][k] * page, page);
                     }
@@ -450,11 +587,16 @@ int xfthip_plan_create(const xfthip_plan_config *cfg, const xfthip_plan_layer *l
     const xfthip_plan_config &c = *cfg;
     XFT_REQUIRE(c.layers > 0 && c.hidden > 0 && c.hidden <= 16384 && c.vocab > 0, "xfthip_plan_create: bad sizes");
     const bool loop = c.loop_times > 1 && c.loop_start != c.loop_stop; // (a loop over nothing is none)
+    XFT_REQUIRE((c.block == XFTHIP_BLOCK_SANDWICH && c.norm == XFTHIP_NORM_RMS_ABOUT_ONE && c.side_dim == 0)
+                    || (c.block == XFTHIP_BLOCK_PARALLEL && c.norm == XFTHIP_NORM_DYNAMIC_TANH && c.side_dim >= 0),
+            "xfthip_plan_create: block arrangement %d with norm %d and side width %d is not served", c.block, c.norm, c.side_dim);
     XFT_REQUIRE(!loop || (c.loop_start >= 0 && c.loop_start < c.loop_stop && c.loop_stop <= c.layers), "xfthip_plan_create: loop over layers %d .. %d of %d",
             c.loop_start, c.loop_stop, c.layers);
     xfthip_plan *p = new xfthip_plan();
     p->cfg = c;
     p->hidden = pad32(c.hidden);
+    p->side_pad = pad32(c.side_dim);
+    int first_mix = -1; // the first layer with mixed values
     for (int i = 0; i < c.layers; ++i) {
         PlanLayer L;
         L.s = layers[i];
@@ -470,10 +612,24 @@ int xfthip_plan_create(const xfthip_plan_config *cfg, const xfthip_plan_layer *l
             L.VD = pad32(s.vdim);
             L.rank = pad32(std::max(s.decay_rank, s.gate_rank));
             L.gcols = s.heads * std::max(L.KD, L.VD);
+        } else if (s.mixer == XFTHIP_MIXER_GROUPED) {
+            ok = ok && s.kv_heads > 0 && s.heads % s.kv_heads == 0 && s.dim <= 512 && s.vdim <= 512 && s.rot_dim >= 0 && s.rot_dim <= s.dim && s.rot_dim % 2 == 0
+                    && s.window >= 0 && (s.rot_factor <= 0.0 || (s.rot_original > 0.0 && s.rot_fast > 0.0 && s.rot_slow > 0.0));
+            L.D = pad32(s.dim), L.V = pad32(s.vdim);
+            if (ok && s.v_mix) {
+                L.first_values = first_mix < 0;
+                if (first_mix < 0) first_mix = i;
+                const xfthip_plan_layer &f = layers[first_mix];
+                ok = f.kv_heads == s.kv_heads && f.vdim == s.vdim; // values of the same shape
+            }
         } else {
             ok = false;
         }
         L.ff = pad32(s.inter);
+        if (s.experts > 0) {
+            ok = ok && s.identity >= 0 && s.top > 0 && s.top <= L.routes() && s.top <= 64 && L.routes() <= 1024 && s.expert_inter > 0 && s.glu_alpha > 0.0f;
+            L.eff = pad32(s.expert_inter);
+        }
         if (!ok) {
             delete p;
             XFT_REQUIRE(false, "xfthip_plan_create: layer %d has sizes this library does not serve", i);
@@ -495,13 +651,18 @@ int xfthip_plan_create(const xfthip_plan_config *cfg, const xfthip_plan_layer *l
 int xfthip_plan_destroy(xfthip_plan_t p) {
     if (!p) return 0;
     for (PlanLayer &L : p->layers) {
-        for (xfthip_weight_t w : {L.in, L.o, L.gateup, L.down, L.uq, L.absorb, L.uk, L.uv, L.gates}) xfthip_weight_destroy(w);
-        for (float *f : {L.q_norm, L.kv_norm, L.sink, L.conv, L.decay, L.dt_bias, L.out_norm, L.pre1, L.post1, L.pre2, L.post2})
+        for (xfthip_weight_t w : {L.in, L.o, L.gateup, L.down, L.uq, L.absorb, L.uk, L.uv, L.gates, L.router, L.side_gate, L.side_proj}) xfthip_weight_destroy(w);
+        for (auto *list : {&L.egateup, &L.edown})
+            for (xfthip_weight_t w : *list) xfthip_weight_destroy(w);
+        for (float *f : {L.q_norm, L.kv_norm, L.sink, L.conv, L.decay, L.dt_bias, L.out_norm, L.pre1.w, L.pre1.b, L.pre2.w, L.pre2.b, L.post1, L.post2, L.correction,
+                     L.side_post})
             if (f) (void)hipFree(f);
+        if (L.etable) (void)hipFree(L.etable);
     }
     xfthip_weight_destroy(p->head);
     if (p->embedding) (void)hipFree(p->embedding);
-    if (p->final_norm) (void)hipFree(p->final_norm);
+    for (void *b : {(void *)p->final_norm.w, (void *)p->final_norm.b, (void *)p->side_embedding})
+        if (b) (void)hipFree(b);
     delete p;
     return 0;
 }
@@ -556,6 +717,17 @@ int xfthip_plan_finish(xfthip_plan_t p) {
         return v;
     };
     const int W = p->cfg.hidden, Wp = p->hidden, V = p->cfg.vocab;
+    // rows x (parts * width) bf16 -> device, every part padded to `pad` columns
+    auto upload_embedding = [&](const Tensor &t, int parts, int width, int pad, uint16_t **dst) {
+        if (rc) return;
+        std::vector<uint16_t> table((size_t)t.rows * parts * pad, 0);
+        for (int v = 0; v < t.rows; ++v)
+            for (int k = 0; k < parts; ++k) memcpy(&table[((size_t)v * parts + k) * pad], &t.data[((size_t)v * parts + k) * width], (size_t)width * 2);
+        if (hipMalloc((void **)dst, table.size() * 2 + 16) != hipSuccess || hipMemcpy(*dst, table.data(), table.size() * 2, hipMemcpyHostToDevice) != hipSuccess) {
+            set_error("xfthip_plan_finish: upload failed");
+            rc = 1;
+        }
+    };
     auto one_plus = [&](const Tensor &t, const Tensor *scale) {
         std::vector<float> v(Wp, 0.0f);
         for (int i = 0; i < t.rows; ++i) v[i] = (1.0f + bf16_value(t.data[i])) * (scale ? bf16_value(scale->data[i]) : 1.0f);
@@ -564,21 +736,46 @@ int xfthip_plan_finish(xfthip_plan_t p) {
 #define NEED(var, name, r, c)                 \
     const Tensor &var = get(name, r, c);      \
     if (!missing.empty()) break
+    const bool tanh_norm = p->cfg.norm == XFTHIP_NORM_DYNAMIC_TANH, parallel = p->cfg.block == XFTHIP_BLOCK_PARALLEL;
+    // a norm in front of something; mul multiplies its result
+    auto front = [&](const std::string &name, float mul, PlanNorm *dst) {
+        const Tensor &w = get(name.c_str(), W, 1);
+        if (!missing.empty()) return;
+        if (!tanh_norm) {
+            std::vector<float> v = one_plus(w, nullptr);
+            for (float &f : v) f *= mul;
+            upload(v, &dst->w);
+            return;
+        }
+        const Tensor &alpha = get((name + ".alpha").c_str(), 1, 1), &b = get((name + ".b").c_str(), W, 1);
+        if (!missing.empty()) return;
+        std::vector<float> vw = values(w, Wp), vb = values(b, Wp);
+        for (float &f : vw) f *= mul;
+        for (float &f : vb) f *= mul;
+        upload(vw, &dst->w), upload(vb, &dst->b);
+        dst->alpha = bf16_value(alpha.data[0]);
+    };
+    auto gate_up = [&](const Tensor &gate, const Tensor &up, int ff, int pad, xfthip_weight_t *dst) {
+        Matrix gu(Wp, 2 * pad);
+        gu.place(gate, 0, ff, 0, W, 0, 0);
+        gu.place(up, 0, ff, 0, W, 0, pad);
+        pack(gu, XFTHIP_WF_GATEUP, dst);
+    };
+    // [rows, cols] tensor -> weight of `k` inputs and `n` outputs
+    auto plain = [&](const Tensor &t, int k, int n, xfthip_weight_t *dst) {
+        Matrix w(k, n);
+        w.place(t, 0, t.rows, 0, t.cols, 0, 0);
+        pack(w, XFTHIP_WF_NONE, dst);
+    };
     do {
         NEED(embed, "embed", V, W);
-        NEED(head, "head", V, W);
-        NEED(fin, "final.norm", W, 1);
-        std::vector<uint16_t> table((size_t)V * Wp, 0);
-        for (int v = 0; v < V; ++v) memcpy(&table[(size_t)v * Wp], &embed.data[(size_t)v * W], (size_t)W * 2);
-        if (hipMalloc((void **)&p->embedding, table.size() * 2) != hipSuccess
-                || hipMemcpy(p->embedding, table.data(), table.size() * 2, hipMemcpyHostToDevice) != hipSuccess) {
-            set_error("xfthip_plan_finish: upload failed");
-            rc = 1;
-            break;
+        upload_embedding(embed, 1, W, Wp, &p->embedding);
+        front("final.norm", p->cfg.logit_scale, &p->final_norm); // the logits are linear in the normed row
+        if (p->cfg.side_dim > 0) {
+            NEED(side, "side.embed", V, p->cfg.layers * p->cfg.side_dim);
+            upload_embedding(side, p->cfg.layers, p->cfg.side_dim, p->side_pad, &p->side_embedding);
         }
-        std::vector<float> fn = one_plus(fin, nullptr);
-        for (float &f : fn) f *= p->cfg.logit_scale; // the logits are linear in the normed row
-        upload(fn, &p->final_norm);
+        NEED(head, p->cfg.tied_head ? "embed" : "head", V, W);
         Matrix hm(Wp, V);
         hm.place(head, 0, V, 0, W, 0, 0);
         pack(hm, XFTHIP_WF_NONE, &p->head);
@@ -588,26 +785,60 @@ int xfthip_plan_finish(xfthip_plan_t p) {
         const xfthip_plan_layer &s = L.s;
         const int H = s.heads;
         prefix = std::to_string(i) + "/";
-        NEED(n1, "norm1", W, 1);
-        NEED(n1b, "norm1b", W, 1);
-        NEED(ls1, "ls1", W, 1);
-        upload(one_plus(n1, nullptr), &L.pre1);
-        upload(one_plus(n1b, &ls1), &L.post1);
+        front("norm1", 1.0f, &L.pre1);
+        if (L.feeds_forward()) front("norm2", 1.0f, &L.pre2);
+        if (!missing.empty()) break;
+        if (!parallel) {
+            NEED(n1b, "norm1b", W, 1);
+            NEED(ls1, "ls1", W, 1);
+            upload(one_plus(n1b, &ls1), &L.post1);
+            if (L.feeds_forward()) {
+                NEED(n2b, "norm2b", W, 1);
+                NEED(ls2, "ls2", W, 1);
+                upload(one_plus(n2b, &ls2), &L.post2);
+            }
+        }
         if (s.inter > 0) {
-            NEED(n2, "norm2", W, 1);
-            NEED(n2b, "norm2b", W, 1);
-            NEED(ls2, "ls2", W, 1);
-            NEED(gate, "mlp.gate", s.inter, W);
-            NEED(up, "mlp.up", s.inter, W);
-            NEED(down, "mlp.down", W, s.inter);
-            upload(one_plus(n2, nullptr), &L.pre2);
-            upload(one_plus(n2b, &ls2), &L.post2);
-            Matrix gu(Wp, 2 * L.ff), dn(L.ff, Wp);
-            gu.place(gate, 0, s.inter, 0, W, 0, 0);
-            gu.place(up, 0, s.inter, 0, W, 0, L.ff);
-            dn.place(down, 0, W, 0, s.inter, 0, 0);
-            pack(gu, XFTHIP_WF_GATEUP, &L.gateup);
-            pack(dn, XFTHIP_WF_NONE, &L.down);
+            const std::string at = s.experts > 0 ? "mlp.shared." : "mlp.";
+            NEED(gate, (at + "gate").c_str(), s.inter, W);
+            NEED(up, (at + "up").c_str(), s.inter, W);
+            NEED(down, (at + "down").c_str(), W, s.inter);
+            gate_up(gate, up, s.inter, L.ff, &L.gateup);
+            plain(down, L.ff, Wp, &L.down);
+        }
+        if (s.experts > 0) {
+            NEED(router, "mlp.router", L.routes(), W);
+            NEED(correction, "mlp.correction", L.routes(), 1);
+            plain(router, Wp, L.routes(), &L.router);
+            upload(values(correction, L.routes()), &L.correction);
+            L.egateup.assign(s.experts, nullptr), L.edown.assign(s.experts, nullptr);
+            std::vector<GroupWeight> table(2 * (size_t)s.experts);
+            for (int e = 0; e < s.experts && rc == 0; ++e) {
+                const std::string at = "mlp.e" + std::to_string(e) + ".";
+                NEED(gate, (at + "gate").c_str(), s.expert_inter, W);
+                NEED(up, (at + "up").c_str(), s.expert_inter, W);
+                NEED(down, (at + "down").c_str(), W, s.expert_inter);
+                gate_up(gate, up, s.expert_inter, L.eff, &L.egateup[e]);
+                plain(down, L.eff, Wp, &L.edown[e]);
+                if (rc) break;
+                const PackedWeight &g = L.egateup[e]->pw, &d = L.edown[e]->pw;
+                table[e] = {g.packed, g.scale, g.zero}, table[s.experts + e] = {d.packed, d.scale, d.zero};
+            }
+            if (!missing.empty() || rc) break;
+            if (hipMalloc((void **)&L.etable, table.size() * sizeof(GroupWeight)) != hipSuccess
+                    || hipMemcpy(L.etable, table.data(), table.size() * sizeof(GroupWeight), hipMemcpyHostToDevice) != hipSuccess) {
+                set_error("xfthip_plan_finish: upload failed");
+                rc = 1;
+                break;
+            }
+        }
+        if (p->cfg.side_dim > 0) {
+            NEED(gate, "side.gate", p->cfg.side_dim, W);
+            NEED(proj, "side.proj", W, p->cfg.side_dim);
+            NEED(norm, "side.norm", W, 1);
+            plain(gate, Wp, p->side_pad, &L.side_gate);
+            plain(proj, p->side_pad, Wp, &L.side_proj);
+            upload(values(norm, Wp), &L.side_post);
         }
         Matrix in(Wp, L.row_in());
         if (s.mixer == XFTHIP_MIXER_LATENT) {
@@ -642,6 +873,30 @@ int xfthip_plan_finish(xfthip_plan_t p) {
             if (s.has_sink) {
                 NEED(sink, "mix.sink", H, 1);
                 upload(values(sink, H), &L.sink);
+            }
+        } else if (s.mixer == XFTHIP_MIXER_GROUPED) {
+            const int G = s.kv_heads, d = s.dim, dv = s.vdim, k0 = H * L.D, v0 = k0 + G * L.D;
+            NEED(q, "mix.q", H * d, W);
+            NEED(k, "mix.k", G * d, W);
+            NEED(v, "mix.v", G * dv, W);
+            NEED(o, "mix.o", W, H * dv);
+            Matrix mo(H * L.V, Wp);
+            for (int h = 0; h < H; ++h) in.place(q, h * d, d, 0, W, 0, h * L.D), mo.place(o, 0, W, h * dv, dv, h * L.V, 0);
+            for (int h = 0; h < G; ++h) in.place(k, h * d, d, 0, W, 0, k0 + h * L.D), in.place(v, h * dv, dv, 0, W, 0, v0 + h * L.V);
+            pack(mo, XFTHIP_WF_NONE, &L.o);
+            if (s.qk_norm) {
+                NEED(qn, "mix.q.norm", d, 1);
+                NEED(kn, "mix.k.norm", d, 1);
+                upload(values(qn, L.D), &L.q_norm);
+                upload(values(kn, L.D), &L.kv_norm);
+            }
+            if (s.has_sink) {
+                NEED(sink, "mix.sink", H, 1);
+                upload(values(sink, H), &L.sink);
+            }
+            if (s.v_mix && !L.first_values) {
+                NEED(share, "mix.vmix", 1, 1);
+                L.value_share = bf16_value(share.data[0]);
             }
         } else {
             const int KH = s.kv_heads, d = s.dim, dv = s.vdim, n = s.taps;
@@ -710,7 +965,7 @@ int xfthip_model_create_from_plan(xfthip_plan_t plan, int act_dtype, int max_bat
     m->cfg.layers = plan->cfg.layers, m->cfg.hidden = plan->hidden, m->cfg.vocab = plan->cfg.vocab;
     m->cfg.max_batch = max_batch, m->cfg.max_seq = max_seq, m->cfg.max_tokens = max_tokens, m->cfg.max_pos_embed = max_seq;
     m->cfg.rms_eps = plan->cfg.eps;
-    m->final_norm = plan->final_norm;
+    m->final_norm = plan->final_norm.w;
     m->lm_head = plan->head;
     m->row_pos.assign(max_batch, -1);
     PlanState *p = new PlanState();
@@ -736,12 +991,21 @@ int xfthip_model_create_from_plan(xfthip_plan_t plan, int act_dtype, int max_bat
         memcpy(dst, &b, sizeof(b));
     };
     const size_t T = max_tokens, e = p->esz, hidden = plan->hidden;
-    size_t a = 0, cq = 0, q = 0, qa = 0, ov = 0, h = 0, gates = 0, dk = 0, dqk = 0, dg = 0, dv = 0, heads = 0, on = 0;
+    size_t a = 0, cq = 0, q = 0, qa = 0, ov = 0, h = 0, gates = 0, dk = 0, dqk = 0, dg = 0, dv = 0, heads = 0, on = 0, fv = 0;
+    size_t top = 0, experts = 0, routes = 0, eh = 0, eo = 0;
     for (const PlanLayer &L : p->layers) {
         const size_t H = L.s.heads;
         a = std::max(a, (size_t)L.row_in());
         h = std::max(h, (size_t)L.ff);
-        if (L.s.mixer == XFTHIP_MIXER_LATENT) {
+        if (L.s.experts > 0) {
+            const size_t most = std::min(L.s.top, L.s.experts);
+            top = std::max(top, (size_t)L.s.top), experts = std::max(experts, (size_t)L.s.experts), routes = std::max(routes, (size_t)pad32(L.routes()));
+            eh = std::max(eh, most * L.eff), eo = std::max(eo, most * hidden);
+        }
+        if (L.s.mixer == XFTHIP_MIXER_GROUPED) {
+            q = std::max(q, H * L.D), ov = std::max(ov, H * L.V);
+            if (L.s.v_mix) fv = std::max(fv, (size_t)L.s.kv_heads * L.V);
+        } else if (L.s.mixer == XFTHIP_MIXER_LATENT) {
             cq = std::max(cq, (size_t)L.QR), q = std::max(q, H * (L.D + L.RD)), qa = std::max(qa, H * L.R), ov = std::max(ov, H * L.V);
         } else {
             const size_t KH = L.s.kv_heads;
@@ -755,6 +1019,11 @@ int xfthip_model_create_from_plan(xfthip_plan_t plan, int act_dtype, int max_bat
     alloc(&p->ov, T * ov * e), alloc(&p->h, T * h * e), alloc(&p->on, T * on * e);
     alloc(&p->gates, T * gates * 4), alloc(&p->dq, T * dk * 4), alloc(&p->dk, T * dk * 4), alloc(&p->dqk, T * dqk * 4), alloc(&p->dg, T * dg * 4);
     alloc(&p->dv, T * dv * 4), alloc(&p->dbeta, T * heads * 4), alloc(&p->do_, T * dv * 4);
+    if (plan->cfg.block == XFTHIP_BLOCK_PARALLEL) alloc(&p->xn2, T * hidden * e), alloc(&p->narrow, T * hidden * e);
+    alloc(&p->first_values, T * fv * e), alloc(&p->side, T * plan->side_pad * e), alloc(&p->side_z, T * plan->side_pad * 4);
+    alloc(&p->router_logits, T * routes * 4), alloc(&p->eh, T * eh * e), alloc(&p->expert_out, T * eo * 4);
+    alloc(&p->route.sel, T * top * 4), alloc(&p->route.weight, T * top * 4), alloc(&p->route.slot_row, T * top * 4), alloc(&p->route.row_token, T * top * 4);
+    alloc(&p->route.group_rows, experts * 12);
     // the expanded form's context (whole blocks of 32 tokens; cleared: rows behind the end meet zero weights)
     if (act_dtype == XFTHIP_BF16 && max_tokens >= 32) {
         const size_t ctx = pad32(max_seq) + 32;
@@ -764,32 +1033,37 @@ int xfthip_model_create_from_plan(xfthip_plan_t plan, int act_dtype, int max_bat
                 kx = std::max(kx, (size_t)L.s.heads * L.D), vx = std::max(vx, (size_t)L.s.heads * L.V), rl = std::max(rl, (size_t)(L.R + L.RD));
         if (kx) alloc(&p->rows, ctx * rl * e, true), alloc(&p->kx, ctx * kx * e, true), alloc(&p->vx, ctx * vx * e, true);
     }
-    for (const PlanLayer &L : p->layers) p->part_floats = std::max(p->part_floats, L.s.mixer == XFTHIP_MIXER_LATENT ? latent_part_floats(L) : 0);
+    for (const PlanLayer &L : p->layers) {
+        if (L.s.mixer == XFTHIP_MIXER_LATENT) p->part_floats = std::max(p->part_floats, latent_part_floats(L));
+        if (L.s.mixer == XFTHIP_MIXER_GROUPED) p->part_floats = std::max(p->part_floats, grouped_part_floats(L));
+    }
     alloc(&p->part, p->part_floats * 4);
     for (const LayerRun &r : plan->runs) {
         const PlanLayer &L = p->layers[r.layer];
-        LatentCacheView cv = {nullptr, L.R, L.RD};
+        void *pool = nullptr;
         float *state = nullptr;
         void *conv = nullptr;
-        if (L.s.mixer == XFTHIP_MIXER_LATENT) {
+        if (L.paged()) {
             // cleared: keys that lie behind a sequence's end are multiplied by zero weights and must be numbers
-            alloc(&cv.pool, (size_t)p->pages * kPageTokens * (L.R + L.RD) * e, true);
+            alloc(&pool, (size_t)p->pages * kPageTokens * L.token_elems() * e, true);
         } else {
             alloc(&state, (size_t)max_batch * L.s.heads * L.VD * L.KD * 4, true);
             alloc(&conv, (size_t)max_batch * (L.s.taps - 1) * L.channels() * e, true);
         }
-        p->cache.push_back(cv), p->state.push_back(state), p->conv_state.push_back(conv);
+        p->cache.push_back(pool), p->state.push_back(state), p->conv_state.push_back(conv);
     }
     alloc(&p->table, p->table_host.size() * 4, true);
     alloc(&p->desc, (3 * T + 4 * (size_t)max_batch) * 4, true);
     alloc(&p->dec_rows, (size_t)max_batch * 4, true);
     alloc(&p->want, (size_t)p->logit_rows * 4, true);
-    std::map<std::pair<double, int>, std::pair<float *, float *>> rot;
+    std::map<std::vector<double>, std::pair<float *, float *>> rot; // layers of the same rotation share its tables
     for (PlanLayer &L : p->layers) {
-        if (L.s.mixer != XFTHIP_MIXER_LATENT || !ok) continue;
-        auto &t = rot[{L.s.rot_base, L.s.rot_dim}];
+        if (!L.paged() || !ok) continue;
+        const bool extended = L.s.rot_factor > 0.0;
+        auto &t = rot[{L.s.rot_base, (double)L.s.rot_dim, extended ? L.s.rot_factor : 0.0, extended ? L.s.rot_original : 0.0, extended ? L.s.rot_fast : 0.0,
+                extended ? L.s.rot_slow : 0.0}];
         if (!t.first) {
-            ok = rotation_tables(L.s.rot_base, L.s.rot_dim, max_seq, &t.first, &t.second) == 0;
+            ok = rotation_tables(L.s, max_seq, &t.first, &t.second) == 0;
             if (t.first) p->owned.push_back(t.first);
             if (t.second) p->owned.push_back(t.second);
         }

@@ -43,6 +43,7 @@ struct SkinnyParams {
     // rows of C must tile [0, sum of rows) without gaps.
     const GroupWeight *group;
     int group_n, rows_stride;
+    const int *a_rows; // groups only, or null: row r of A (record offset included) is row a_rows[r] of it
 
     // ---- fusions of the decode step (M <= 4, skinny kernel only) ----
     // RMSNorm prologue: when norm_x is set, A is ignored and every workgroup normalises the M rows
@@ -83,9 +84,11 @@ int gemm_rows_dev(xfthip_weight_t w, int m_max, int m_hint, const int *rows_dev,
 // The same for n_group weights of one shape behind one launch: table_dev holds their device pointers, record e
 // of rows_dev (rows_stride ints apart) the rows of weight e; rows_max bounds the sum of the rows, rows_each_max the
 // rows of one weight (up to 32 of those: the few-row kernel, one grid row a weight; more: the tiled kernel, row
-// blocks numbered across the weights); the weights' rows of C tile [0, sum of rows).
+// blocks numbered across the weights); the weights' rows of C tile [0, sum of rows).  a_rows: as in SkinnyParams.
+// glu_alpha > 0: gate / up weights combine as clamped_glu instead of as SwiGLU.
 int gemm_grouped_rows_dev(const xfthip_weight_t *w, int n_group, const GroupWeight *table_dev, int rows_max, int rows_each_max,
-        const int *rows_dev, int rows_stride, const void *A, int lda, void *C, int ldc, int c_dtype, hipStream_t stream);
+        const int *rows_dev, int rows_stride, const void *A, int lda, void *C, int ldc, int c_dtype, hipStream_t stream,
+        const int *a_rows = nullptr, float glu_limit = 0.0f, float glu_alpha = 0.0f);
 
 int gemm_w8a8_from_bf16(xfthip_weight_t w, int M, const void *A, int lda, void *C, int ldc, int c_dtype, int epilogue,
         const float *bias, const void *res, int ldres, int res_dtype, float gamma, hipStream_t stream);

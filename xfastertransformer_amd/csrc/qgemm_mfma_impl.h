@@ -163,7 +163,8 @@ __global__ __launch_bounds__(256 * KG, (DIRECT && KG == 1) ? 2 : 1) void qgemm_m
         mb -= first;
         const int *rec = p.rows_dev + e * p.rows_stride;
         p.M = rec[0];
-        p.A += (size_t)rec[1] * p.lda;
+        if (p.a_rows) p.a_rows += rec[1];
+        else p.A += (size_t)rec[1] * p.lda;
         c_row = part_row = rec[2];
         p.packed = p.group[e].packed;
         p.scale = p.group[e].scale;
@@ -256,6 +257,7 @@ __global__ __launch_bounds__(256 * KG, (DIRECT && KG == 1) ? 2 : 1) void qgemm_m
         } else {
             int row = m0 + a_row0 + i * ROW_STEP;
             row = row < p.M ? row : p.M - 1;
+            if constexpr (DEVROWS) row = p.a_rows ? p.a_rows[row] : row;
             a_off[i] = (uint32_t)row * (uint32_t)p.lda + a_kc * 8;
         }
     }

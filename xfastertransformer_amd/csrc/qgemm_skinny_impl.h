@@ -125,7 +125,7 @@ __global__ __launch_bounds__(512, (STAGE && MT == 1 && NT == 1) ? 4 : 1) void qg
     static_assert(!NORM || (MT == 1 && !KTAIL), "the norm prologue covers M <= 4 without a K tail");
     static_assert(!ROPE || (NT % 2 == 0 && !KTAIL), "the RoPE epilogue works on tile pairs");
     static_assert(!STAGE || (!NORM && !ROPE), "staged activation loads belong to the plain kernels");
-    static_assert(!GROUP || (!NORM && !ROPE && !KTAIL), "grouped launches: plain kernels, whole k tiles");
+    static_assert(!GROUP || (!NORM && !ROPE && (!KTAIL || KIND == XFTHIP_W_BF16)), "grouped launches: plain kernels; K tails for BF16 weights only");
     using T = KindTraits<KIND>;
     constexpr int MPT = T::MPT, KL = T::KL, KTILE = T::KTILE;
     extern __shared__ float smem[];
@@ -146,7 +146,8 @@ __global__ __launch_bounds__(512, (STAGE && MT == 1 && NT == 1) ? 4 : 1) void qg
         }
         if (rec[0] <= 0) return; // uniform: the whole workgroup leaves
         p.M = rec[0] < p.M ? rec[0] : p.M;
-        p.A += (size_t)rec[1] * p.lda;
+        if (GROUP && p.a_rows) p.a_rows += rec[1];
+        else p.A += (size_t)rec[1] * p.lda;
         p.C = (char *)p.C + (size_t)rec[2] * p.ldc * (p.c_dtype == XFTHIP_F32 ? 4 : 2);
     }
 
@@ -230,6 +231,7 @@ __global__ __launch_bounds__(512, (STAGE && MT == 1 && NT == 1) ? 4 : 1) void qg
         for (int m = 0; m < MT; ++m) {
             int row = m * 16 + ml;
             row = row < p.M ? row : p.M - 1;
+            if constexpr (GROUP) row = p.a_rows ? p.a_rows[row] : row;
             abase[m] = p.A + (size_t)row * p.lda + g * KL;
         }
 
@@ -239,6 +241,7 @@ __global__ __launch_bounds__(512, (STAGE && MT == 1 && NT == 1) ? 4 : 1) void qg
         for (int j = 0; j < MT * MPT; ++j) {
             int row = j * RPI + s_row;
             row = row < p.M ? row : p.M - 1;
+            if constexpr (GROUP) row = p.a_rows ? p.a_rows[row] : row;
             s_off[j] = (uint32_t)row * (uint32_t)p.lda;
         }
 
@@ -673,6 +676,12 @@ static int dispatch_tail(const SkinnyParams &p, int kslices, hipStream_t stream)
         if (p.norm_x || p.rope) {
             set_error("qgemm_skinny: the fused prologue / epilogue needs K to be a whole number of weight tiles");
             return 2;
+        }
+        if constexpr (KIND == XFTHIP_W_BF16) {
+            if (p.group) {
+                if (MT == 2 || p.M > 4) return launch<KIND, NT, MT, U, NEED_SUM, true, false, false, true, true>(p, kslices, stream);
+                if constexpr (MT == 1) return launch<KIND, NT, MT, U, NEED_SUM, true, false, false, false, true>(p, kslices, stream);
+            }
         }
         if (MT == 2 || p.M > 4) return launch<KIND, NT, MT, U, NEED_SUM, true, false, false, true>(p, kslices, stream);
         if constexpr (MT == 1) return launch<KIND, NT, MT, U, NEED_SUM, true, false>(p, kslices, stream);

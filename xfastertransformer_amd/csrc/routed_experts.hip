@@ -1,0 +1,187 @@
+// Routing of layer plans' expert feed-forwards: scores, choices and weights of every token, the lists of tokens by expert that
+// the grouped products read, and the weighted sum behind them.  Router outputs past the experts hand the input through.
+#include "plan_dev.h"
+
+namespace xfthip {
+
+namespace {
+
+constexpr int kMaxRoutes = 1024, kMaxTop = 64;
+
+struct RouteParams {
+    const float *logits;
+    const float *correction;
+    int ld, T, experts, routes, top;
+    RouteBuffers b;
+};
+
+// One token a wave: CH router outputs a lane.  The choice scores give way one by one, the lower index first among equals.
+template <int CH>
+__device__ inline void route_one(const RouteParams &p, int t, int lane) {
+    float z[CH], choice[CH], mx = -INFINITY;
+#pragma unroll
+    for (int i = 0; i < CH; ++i) {
+        const int e = i * 64 + lane;
+        z[i] = e < p.routes ? p.logits[(size_t)t * p.ld + e] : -INFINITY;
+        choice[i] = e < p.routes ? p.correction[e] : 0.0f;
+        mx = fmaxf(mx, z[i]);
+    }
+    mx = wave_largest(mx);
+    float sum = 0.0f;
+#pragma unroll
+    for (int i = 0; i < CH; ++i) z[i] = i * 64 + lane < p.routes ? expf(z[i] - mx) : 0.0f, sum += z[i];
+    sum = wave_total(sum);
+#pragma unroll
+    for (int i = 0; i < CH; ++i) {
+        z[i] /= sum;
+        choice[i] = i * 64 + lane < p.routes ? z[i] + choice[i] : -INFINITY;
+    }
+    for (int k = 0; k < p.top; ++k) {
+        float best = -INFINITY, score = 0.0f;
+        int at = 1 << 20;
+#pragma unroll
+        for (int i = 0; i < CH; ++i)
+            if (choice[i] > best) best = choice[i], score = z[i], at = i * 64 + lane;
+#pragma unroll
+        for (int off = 32; off > 0; off >>= 1) {
+            const float ob = __shfl_xor(best, off, 64), os = __shfl_xor(score, off, 64);
+            const int oa = __shfl_xor(at, off, 64);
+            if (ob > best || (ob == best && oa < at)) best = ob, score = os, at = oa;
+        }
+        // (scores that are not numbers choose nothing: the last output, with their weight)
+        const int e = at < p.routes ? at : p.routes - 1;
+        if (lane == 0) p.b.sel[(size_t)t * p.top + k] = e, p.b.weight[(size_t)t * p.top + k] = at < p.routes ? score : sum;
+#pragma unroll
+        for (int i = 0; i < CH; ++i)
+            if (i * 64 + lane == at) choice[i] = -INFINITY;
+    }
+}
+
+// lists of tokens by expert, in one workgroup: count, lay the lists back to back, fill
+__device__ inline void build_lists(const RouteParams &p, int *count, int *first) {
+    const int n = p.T * p.top;
+    for (int e = threadIdx.x; e < p.experts; e += blockDim.x) count[e] = 0;
+    __syncthreads();
+    for (int i = threadIdx.x; i < n; i += blockDim.x) {
+        const int e = p.b.sel[i];
+        p.b.slot_row[i] = e < p.experts ? atomicAdd(&count[e], 1) : -1;
+    }
+    __syncthreads();
+    if (threadIdx.x < 64) {
+        const int per = (p.experts + 63) / 64, e0 = threadIdx.x * per;
+        int own = 0;
+        for (int e = e0; e < e0 + per && e < p.experts; ++e) own += count[e];
+        int upto = own;
+#pragma unroll
+        for (int off = 1; off < 64; off <<= 1) {
+            const int o = __shfl_up(upto, off, 64);
+            if ((int)threadIdx.x >= off) upto += o;
+        }
+        int at = upto - own;
+        for (int e = e0; e < e0 + per && e < p.experts; ++e) {
+            first[e] = at;
+            p.b.group_rows[3 * e] = count[e], p.b.group_rows[3 * e + 1] = at, p.b.group_rows[3 * e + 2] = at;
+            at += count[e];
+        }
+    }
+    __syncthreads();
+    for (int i = threadIdx.x; i < n; i += blockDim.x) {
+        const int e = p.b.sel[i];
+        if (e >= p.experts) continue;
+        const int row = first[e] + p.b.slot_row[i];
+        p.b.slot_row[i] = row;
+        p.b.row_token[row] = i / p.top;
+    }
+}
+
+template <int CH>
+__global__ __launch_bounds__(256) void route_kernel(RouteParams p) {
+    const int t = blockIdx.x * 4 + (threadIdx.x >> 6);
+    if (t < p.T) route_one<CH>(p, t, threadIdx.x & 63);
+}
+__global__ __launch_bounds__(1024) void route_lists_kernel(RouteParams p) {
+    __shared__ int count[kMaxRoutes], first[kMaxRoutes];
+    build_lists(p, count, first);
+}
+// few tokens: both at once
+template <int CH>
+__global__ __launch_bounds__(1024) void route_few_kernel(RouteParams p) {
+    __shared__ int count[kMaxRoutes], first[kMaxRoutes];
+    for (int t = threadIdx.x >> 6; t < p.T; t += 16) route_one<CH>(p, t, threadIdx.x & 63);
+    __syncthreads();
+    build_lists(p, count, first);
+}
+
+struct CombineParams {
+    const float *base, *outputs;
+    const void *h;
+    int top;
+    const float *weight;
+    const int *slot_row;
+    float *dst;
+    void *narrow;
+    int hidden;
+};
+
+// grid (tokens, column chunks of 1024)
+template <bool BF16>
+__global__ __launch_bounds__(256) void combine_experts_kernel(CombineParams p) {
+    const int t = blockIdx.x, c = (blockIdx.y * 256 + threadIdx.x) * 4;
+    if (c >= p.hidden) return;
+    const size_t at = (size_t)t * p.hidden + c;
+    f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+    if (p.base) acc = *(const f32x4 *)(p.base + at);
+    for (int k = 0; k < p.top; ++k) {
+        const int row = p.slot_row[t * p.top + k];
+        const float w = p.weight[t * p.top + k];
+        f32x4 y;
+        if (row >= 0) {
+            y = *(const f32x4 *)(p.outputs + (size_t)row * p.hidden + c);
+        } else if constexpr (BF16) {
+            const uint2 u = *(const uint2 *)((const uint16_t *)p.h + at);
+            y = f32x4 {u2f(u.x << 16), u2f(u.x & 0xFFFF0000u), u2f(u.y << 16), u2f(u.y & 0xFFFF0000u)};
+        } else {
+            y = *(const f32x4 *)((const float *)p.h + at);
+        }
+        acc += y * w;
+    }
+    *(f32x4 *)(p.dst + at) = acc;
+    if (p.narrow) put4<BF16>(p.narrow, at, acc);
+}
+
+template <int CH>
+int launch_route(const RouteParams &p, hipStream_t st) {
+    if (p.T <= 32) {
+        hipLaunchKernelGGL(route_few_kernel<CH>, dim3(1), dim3(1024), 0, st, p);
+    } else {
+        hipLaunchKernelGGL(route_kernel<CH>, dim3((p.T + 3) / 4), dim3(256), 0, st, p);
+        hipLaunchKernelGGL(route_lists_kernel, dim3(1), dim3(1024), 0, st, p);
+    }
+    XFT_CHECK_HIP(hipGetLastError());
+    return 0;
+}
+
+} // namespace
+
+int route_tokens(const float *logits, int ld, const float *correction, int T, int experts, int routes, int top, const RouteBuffers &b, hipStream_t st) {
+    XFT_REQUIRE(T > 0 && experts > 0 && routes >= experts && routes <= kMaxRoutes && top > 0 && top <= routes && top <= kMaxTop && ld >= routes,
+            "route_tokens: %d of %d + %d outputs", top, experts, routes - experts);
+    const RouteParams p = {logits, correction, ld, T, experts, routes, top, b};
+    if (routes <= 64) return launch_route<1>(p, st);
+    if (routes <= 128) return launch_route<2>(p, st);
+    if (routes <= 256) return launch_route<4>(p, st);
+    return launch_route<16>(p, st);
+}
+
+int combine_experts(int act, const float *base, const float *outputs, const void *h, int top, const RouteBuffers &b, float *dst, void *narrow, int T,
+        int hidden, hipStream_t st) {
+    XFT_REQUIRE(T > 0 && dst && hidden % 4 == 0, "combine_experts: bad argument");
+    const CombineParams p = {base, outputs, h, top, b.weight, b.slot_row, dst, narrow, hidden};
+    const dim3 grid(T, (hidden + 1023) / 1024);
+    if (act == XFTHIP_BF16) hipLaunchKernelGGL(combine_experts_kernel<true>, grid, dim3(256), 0, st, p);
+    else hipLaunchKernelGGL(combine_experts_kernel<false>, grid, dim3(256), 0, st, p);
+    XFT_CHECK_HIP(hipGetLastError());
+    return 0;
+}
+
+} // namespace xfthip

@@ -1,8 +1,8 @@
 // Matrix products of layer plans that the weight-only GEMMs do not cover: 32-bit activations (true fp32 products on the
 // fp32 matrix units), and heads side by side (every block of output columns multiplies its own slice of the activation
-// row, the per-head products of latent attention and the two gates of the delta rule).  BF16 weights in the packed layout
-// of common.h.
-#include "plan.h"
+// row, the per-head products of latent attention and the two gates of the delta rule), also for the weights of a group in one
+// launch (experts).  BF16 weights in the packed layout of common.h.
+#include "plan_dev.h"
 
 namespace xfthip {
 
@@ -14,11 +14,14 @@ struct TileGemm {
     const void *A;
     int lda, tiles_per_block, a_block_stride;
     void *C;
-    int ldc, c_dtype, glu;
+    int ldc, c_dtype, glu, add;
     float glu_limit, glu_alpha;
+    const uint16_t *side;
+    int side_ld, side_vocab;
+    const int *side_ids;
+    const GroupWeight *group;
+    const int *group_rows, *a_rows;
 };
-
-typedef uint32_t u32x4 __attribute__((ext_vector_type(4)));
 
 __device__ inline float precise_glu(float gate, float up, float limit, float alpha) {
     const float g = fminf(gate, limit), u = fminf(fmaxf(up, -limit), limit);
@@ -39,6 +42,15 @@ __global__ __launch_bounds__(256) void tile_gemm_kernel(TileGemm p) {
     const int kper = (p.ktiles + KS - 1) / KS, k0 = KS > 1 ? wave * kper : 0;
     const int k1 = k0 + kper < p.ktiles ? k0 + kper : p.ktiles;
     const int m0 = blockIdx.y * 16 * MT;
+    int a_first = 0;
+    if (p.group) { // blockIdx.z: the weight
+        const int *rec = p.group_rows + 3 * blockIdx.z;
+        p.packed = p.group[blockIdx.z].packed;
+        p.M = rec[0] < p.M ? rec[0] : p.M;
+        a_first = rec[1];
+        p.C = (char *)p.C + (size_t)rec[2] * p.ldc * (p.c_dtype == XFTHIP_F32 ? 4 : 2);
+        if (m0 >= p.M) return; // (the whole workgroup)
+    }
     const uint8_t *w[2];
     int aofs[2];
 #pragma unroll
@@ -52,7 +64,8 @@ __global__ __launch_bounds__(256) void tile_gemm_kernel(TileGemm p) {
 #pragma unroll
     for (int m = 0; m < MT; ++m) {
         const int r = m0 + m * 16 + ml;
-        row[m] = (size_t)(r < p.M ? r : p.M - 1) * p.lda + 8 * g;
+        const int ra = a_first + (r < p.M ? r : p.M - 1);
+        row[m] = (size_t)(p.a_rows ? p.a_rows[ra] : ra) * p.lda + 8 * g;
     }
     f32x4 acc[2][MT];
 #pragma unroll
@@ -126,9 +139,23 @@ __global__ __launch_bounds__(256) void tile_gemm_kernel(TileGemm p) {
             }
             continue;
         }
+        const uint16_t *side = nullptr;
+        if (p.side) {
+            int id = p.side_ids[r];
+            id = id < 0 ? 0 : (id >= p.side_vocab ? p.side_vocab - 1 : id);
+            side = p.side + (size_t)id * p.side_ld;
+        }
 #pragma unroll
         for (int t = 0; t < 2; ++t) {
             const int n = (nt0 + t) * 16 + 4 * g;
+            if (side || p.add) {
+#pragma unroll
+                for (int i = 0; i < 4; ++i) {
+                    if (n + i >= p.N) continue;
+                    if (side) acc[t][m][i] = gelu_tanh(acc[t][m][i]) * bf16_to_f32(side[n + i]);
+                    if (p.add) acc[t][m][i] += ((const float *)p.C)[(size_t)r * p.ldc + n + i];
+                }
+            }
             const size_t at = (size_t)r * p.ldc + n;
             if (n + 4 <= p.N && (p.ldc & 3) == 0) {
                 if (p.c_dtype == XFTHIP_F32)
@@ -147,26 +174,30 @@ __global__ __launch_bounds__(256) void tile_gemm_kernel(TileGemm p) {
 
 } // namespace
 
-int tile_gemm(xfthip_weight_t w, int act_in, int M, const void *A, int lda, int block_cols, int a_block_stride, void *C, int ldc, int c_dtype,
-        int glu, float glu_limit, float glu_alpha, hipStream_t st) {
-    XFT_REQUIRE(w && A && C && M > 0, "tile_gemm: null argument");
+int tile_gemm(xfthip_weight_t w, int act_in, const TileGemmArgs &a, hipStream_t st) {
+    XFT_REQUIRE(w && a.A && a.C && a.M > 0, "tile_gemm: null argument");
     const PackedWeight &pw = w->pw;
+    const int M = a.M;
     XFT_REQUIRE(pw.kind == XFTHIP_W_BF16 && pw.K % 32 == 0, "tile_gemm: BF16 weights with K a multiple of 32 (K=%d)", pw.K);
-    XFT_REQUIRE(block_cols % 16 == 0 && lda % 8 == 0 && a_block_stride % 8 == 0 && ((uintptr_t)A & 15) == 0, "tile_gemm: unaligned operands");
-    const int blocks = block_cols ? (pw.N + block_cols - 1) / block_cols : 1;
-    XFT_REQUIRE((long)(blocks - 1) * a_block_stride + pw.K <= lda, "tile_gemm: %d blocks of K=%d reach past the row (%d)", blocks, pw.K, lda);
-    XFT_REQUIRE(ldc >= (glu ? pw.N / 2 : pw.N) && (glu != 0) == ((pw.flags & XFTHIP_WF_GATEUP) != 0), "tile_gemm: ldc=%d N=%d glu=%d", ldc, pw.N, glu);
-    TileGemm p = {pw.packed, pw.KT, pw.K / 32, pw.NTILES, pw.N, M, A, lda, block_cols / 16, a_block_stride, C, ldc, c_dtype, glu, glu_limit, glu_alpha};
+    XFT_REQUIRE(a.block_cols % 16 == 0 && a.lda % 8 == 0 && a.a_block_stride % 8 == 0 && ((uintptr_t)a.A & 15) == 0, "tile_gemm: unaligned operands");
+    const int blocks = a.block_cols ? (pw.N + a.block_cols - 1) / a.block_cols : 1;
+    XFT_REQUIRE((long)(blocks - 1) * a.a_block_stride + pw.K <= a.lda, "tile_gemm: %d blocks of K=%d reach past the row (%d)", blocks, pw.K, a.lda);
+    XFT_REQUIRE(a.ldc >= (a.glu ? pw.N / 2 : pw.N) && a.glu == ((pw.flags & XFTHIP_WF_GATEUP) != 0), "tile_gemm: ldc=%d N=%d glu=%d", a.ldc, pw.N, a.glu);
+    XFT_REQUIRE((!a.add || (a.c_dtype == XFTHIP_F32 && !a.glu)) && (!a.side || (!a.glu && !a.group && a.side_ids)) && (!a.group || a.group_rows),
+            "tile_gemm: options that do not go together");
+    const TileGemm p = {pw.packed, pw.KT, pw.K / 32, pw.NTILES, pw.N, M, a.A, a.lda, a.block_cols / 16, a.a_block_stride, a.C, a.ldc, a.c_dtype, a.glu, a.add,
+            a.glu_limit, a.glu_alpha, a.side, a.side_ld, a.side_vocab, a.side_ids, a.group, a.group_rows, a.a_rows};
+    const unsigned gz = a.group ? (unsigned)a.group_n : 1;
     const unsigned gx = (unsigned)((pw.NTILES + 7) / 8), gx1 = (unsigned)((pw.NTILES + 1) / 2);
     const bool f32 = act_in == XFTHIP_F32;
-    auto launch = [&](auto kernel, unsigned x, unsigned y) { hipLaunchKernelGGL(kernel, dim3(x, y), dim3(256), 0, st, p); };
+    auto launch = [&](auto kernel, unsigned x, unsigned y) { hipLaunchKernelGGL(kernel, dim3(x, y, gz), dim3(256), 0, st, p); };
     if (M <= 16) {
         if (f32) launch(tile_gemm_kernel<true, 1, 4>, gx1, 1);
         else launch(tile_gemm_kernel<false, 1, 4>, gx1, 1);
     } else if (M <= 32) {
         if (f32) launch(tile_gemm_kernel<true, 2, 4>, gx1, 1);
         else launch(tile_gemm_kernel<false, 2, 4>, gx1, 1);
-    } else if ((long)gx * ((M + 63) / 64) < 2L * device_cu_count()) {
+    } else if ((long)gx * ((M + 63) / 64) < 2L * device_cu_count() && !a.group) {
         if (f32) launch(tile_gemm_kernel<true, 1, 1>, gx, (unsigned)((M + 15) / 16));
         else launch(tile_gemm_kernel<false, 1, 1>, gx, (unsigned)((M + 15) / 16));
     } else {
