@@ -55,15 +55,15 @@ def rotate(x, rot, start=0):
     return y
 
 
-def attend(q, k, v, scale, sink):
-    """q [T, H, d], k [T, G, d], v [T, G, e]; every query sees the keys up to its own; sink [H]: one more term of the
-    denominator.  Returns [T, H, e]."""
+def attend(q, k, v, scale, sink, window=0):
+    """q [T, H, d], k [T, G, d], v [T, G, e]; every query sees the keys up to its own (window > 0: the last so many of them);
+    sink [H]: one more term of the denominator.  Returns [T, H, e]."""
     T, H, G = q.shape[0], q.shape[1], k.shape[1]
     i, j = np.arange(T)[:, None], np.arange(T)[None, :]
     out = np.zeros((T, H, v.shape[-1]), q.dtype)
     for h in range(H):
         g = h // (H // G)
-        s = np.where(j <= i, (q[:, h] @ k[:, g].T) * scale, -np.inf)
+        s = np.where((j <= i) & (i - j < (window or T)), (q[:, h] @ k[:, g].T) * scale, -np.inf)
         m = np.maximum(s.max(-1, keepdims=True), sink[h])
         e = np.exp(s - m)
         out[:, h] = (e @ v[:, g]) / (e.sum(-1, keepdims=True) + np.exp(sink[h] - m))
@@ -80,7 +80,7 @@ def attention(h, w, p, m, eps, v_first):
     if v_first is not None:
         lam = w[p + "vmix"]
         v = (1.0 - lam) * own + lam * v_first
-    o = attend(rotate(q, m["rot"]), rotate(k, m["rot"]), v, m["scale"], w[p + "sink"])
+    o = attend(rotate(q, m["rot"]), rotate(k, m["rot"]), v, m["scale"], w[p + "sink"], m.get("_window", 0))
     return o.reshape(T, H * e) @ w[p + "o"].T, own
 
 

@@ -123,6 +123,35 @@ def rel_rms(got, want):
     return np.sqrt(((got - want) ** 2).mean(-1)) / max(want.std(), 1e-9)
 
 
+class Case:
+    """A device model over a plan, held against an oracle: forward(weights, tokens) -> logits."""
+
+    def __init__(self, xh, plan, w, forward, act, limit, slots=4, max_seq=512, max_tokens=None, pool=0):
+        self.w, self.plan, self.limit, self.forward = w, plan, limit, forward
+        self.model = xh.PlanModel(plan, xh.F32 if act == "f32" else xh.BF16, slots, max_seq, max_tokens or max_seq, pool)
+
+    def want(self, tokens):
+        return self.forward(self.w, tokens)
+
+    def check(self, got, want, what, rows=None):
+        err = rel_rms(got, want if rows is None else want[rows])
+        assert err.max() < self.limit, f"{what}: row {int(err.argmax())} of {len(err)} differs by {err.max():.2e} (limit {self.limit})"
+
+    def run(self, slot, tokens, portions, what, want=None):
+        """the sequence in portions of the given sizes (the last size repeats), all logits checked"""
+        want = self.want(tokens) if want is None else want
+        at, i = 0, 0
+        while at < len(tokens):
+            n = min(portions[min(i, len(portions) - 1)], len(tokens) - at)
+            got = self.model.step([(slot, tokens[at:at + n], list(range(n)))])
+            self.check(got, want[at:at + n], f"{what}, portion {i} at {at}")
+            at, i = at + n, i + 1
+
+    def free(self):
+        self.model.free()
+        self.plan.free()
+
+
 # ---- needles: a prompt in which one key decides the answer ------------------------------------------------------------
 def needle_weights(cfg, seed, key_token, strength=6.0):
     """Weights under which the token `key_token` has a key that every query of the latent layers scores far above all

@@ -25,39 +25,9 @@ def xh():
     return capi
 
 
-def act_of(xh, act):
-    return xh.F32 if act == "f32" else xh.BF16
-
-
-class Case:
-    def __init__(self, xh, cfg, seed, act, slots=4, max_seq=512, max_tokens=None, pool=0, bits=None):
-        self.cfg = cfg
-        self.bits = bits or u.weights(cfg, seed)
-        self.w = u.oracle_weights(self.bits)
-        self.plan = u.build_plan(xh, cfg, self.bits)
-        self.model = xh.PlanModel(self.plan, act_of(xh, act), slots, max_seq, max_tokens or max_seq, pool)
-        self.limit = LIMIT[act]
-
-    def want(self, tokens):
-        return ref.forward(self.cfg, self.w, tokens)
-
-    def check(self, got, want, what, rows=None):
-        err = u.rel_rms(got, want if rows is None else want[rows])
-        assert err.max() < self.limit, f"{what}: row {int(err.argmax())} of {len(err)} differs by {err.max():.2e} (limit {self.limit})"
-
-    def run(self, slot, tokens, portions, what, want=None):
-        """the sequence in portions of the given sizes (the last size repeats), all logits checked"""
-        want = self.want(tokens) if want is None else want
-        at, i = 0, 0
-        while at < len(tokens):
-            n = min(portions[min(i, len(portions) - 1)], len(tokens) - at)
-            got = self.model.step([(slot, tokens[at:at + n], list(range(n)))])
-            self.check(got, want[at:at + n], f"{what}, portion {i} at {at}")
-            at, i = at + n, i + 1
-
-    def free(self):
-        self.model.free()
-        self.plan.free()
+def Case(xh, cfg, seed, act, slots=4, max_seq=512, max_tokens=None, pool=0, bits=None):
+    bits = bits or u.weights(cfg, seed)
+    return u.Case(xh, u.build_plan(xh, cfg, bits), u.oracle_weights(bits), lambda w, t: ref.forward(cfg, w, t), act, LIMIT[act], slots, max_seq, max_tokens, pool)
 
 
 def tokens_of(cfg, n, seed):

@@ -1,0 +1,403 @@
+"""Veterax (grouped attention over pages, routed experts, parallel blocks behind tanh norms, side embeddings) on the GPU against the
+plain restatement in oracle/veterax_ref.py: every mechanism alone, whole models, portions, batches, page and slot reuse, page
+borders, long decoding, and generation through AutoModel.  Parity unpinned: the design has no implementation elsewhere."""
+import json
+import os
+import subprocess
+
+import numpy as np
+import pytest
+
+import veterax_util as u
+from oracle import veterax_ref as ref
+
+pytestmark = pytest.mark.gpu
+ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
+
+LIMIT = {"f32": 3e-5, "bf16": 0.06}
+
+
+@pytest.fixture(scope="module")
+def xh():
+    from xfastertransformer_amd import capi
+    capi.init(0)
+    return capi
+
+
+def Case(xh, cfg, seed, act, slots=4, max_seq=512, max_tokens=None, pool=0, bits=None):
+    bits = bits or (u.weights if act == "f32" else u.steady_weights)(cfg, seed)
+    return u.Case(xh, u.build_plan(xh, cfg, bits), u.oracle_weights(bits), lambda w, t: ref.forward(cfg, w, t), act, LIMIT[act], slots, max_seq, max_tokens, pool)
+
+
+def tokens_of(cfg, n, seed):
+    return np.random.default_rng(seed).integers(0, cfg["vocab"], n).astype(int)
+
+
+PLAIN = dict(v_mix=None, scaling=None)
+ALONE = {  # name: (layers, side width)
+    "attention": ([(u.attention(**PLAIN), None)], 0),
+    "one_head": ([(u.attention(heads=1, kv_heads=1, dim=34, vdim=6, scale=1.0, **PLAIN), None)], 0),
+    "equal_heads": ([(u.attention(heads=3, kv_heads=3, dim=32, vdim=32, **PLAIN), None)], 0),
+    "partial_rotation": ([(u.attention(dim=26, rot=10, **PLAIN), None)], 0),
+    "two_rotated": ([(u.attention(dim=8, rot=2, **PLAIN), None)], 0),
+    "context_extension": ([(u.attention(v_mix=False, scaling=(16.0, 32, 4.0, 0.7)), None)], 0),
+    "extension_by_one": ([(u.attention(v_mix=None, scaling=(1.0, 512, 32.0, 1.0)), None)], 0),
+    "wide_heads": ([(u.attention(heads=4, kv_heads=2, dim=200, vdim=136, scale=0.1, **PLAIN), None)], 0),
+    "very_wide_heads": ([(u.attention(heads=2, kv_heads=1, dim=300, vdim=264, scale=0.1, **PLAIN), None)], 0),
+    "many_heads": ([(u.attention(heads=40, kv_heads=2, dim=64, vdim=64, scale=0.2, **PLAIN), None)], 0),
+    "mixed_values": ([(u.attention(v_mix=False), None), (u.attention(), None), (u.attention(heads=4, dim=12), None), (u.attention(), None)], 0),
+    "experts": ([(u.attention(**PLAIN), u.moe(identity=0, shared_ff=0))], 0),
+    "one_expert": ([(u.attention(**PLAIN), u.moe(experts=1, identity=0, top=1, shared_ff=0))], 0),
+    "all_chosen": ([(u.attention(**PLAIN), u.moe(experts=3, identity=2, top=5, shared_ff=0))], 0),
+    "identity_experts": ([(u.attention(**PLAIN), u.moe(experts=2, identity=6, top=4, shared_ff=0))], 0),
+    "shared_expert": ([(u.attention(**PLAIN), u.moe(ff=72, shared_ff=24, limit=0.4, shared_limit=2.0))], 0),
+    "side": ([(u.attention(**PLAIN), None), (u.attention(**PLAIN), None)], 20),
+    "side_and_experts": ([(u.attention(**PLAIN), u.moe()), (u.attention(**PLAIN), None)], 33),
+}
+
+
+@pytest.mark.parametrize("act", ["f32", "bf16"])
+@pytest.mark.parametrize("name", sorted(ALONE))
+def test_mechanism_alone(xh, name, act):
+    """the residual behind every layer and the logits of a prompt, then token by token"""
+    layers, side = ALONE[name]
+    cfg = u.config(layers, side=side)
+    c = Case(xh, cfg, 11, act)
+    t = tokens_of(cfg, 75, 1)
+    streams = []
+    want = ref.forward(cfg, c.w, t, streams)
+    c.model.trace_residual(True)
+    got = c.model.step([(0, t, list(range(len(t))))])
+    tr = c.model.read_residual()
+    assert tr.shape == (len(layers), len(t), cfg["width"])
+    for i, s in enumerate(streams):
+        c.check(tr[i], s, f"{name}: residual behind layer {i}")
+    c.check(got, want, name)
+    c.model.trace_residual(False)
+    c.run(1, t[:20], [1], name + " token by token", want[:20])
+    c.free()
+
+
+@pytest.mark.parametrize("act", ["f32", "bf16"])
+@pytest.mark.parametrize("routes", [(70, 5, 6), (130, 20, 9), (300, 3, 12)], ids=str)
+def test_many_experts(xh, act, routes):
+    """more router outputs than a wave has lanes; few tokens (one product a row or two) and many"""
+    cfg = u.config([(u.attention(heads=2, kv_heads=1, **PLAIN), u.moe(*routes, ff=16, shared_ff=0))], width=40, side=0)
+    bits = u.weights(cfg, 2)
+    if act == "bf16":  # choices by the correction alone: no rounding turns them
+        c = np.random.default_rng(1).permutation(sum(routes[:2])) * 1.0
+        bits["l0.mlp.correction"] = u.bf16_bits(c)
+    c = Case(xh, cfg, 2, act, bits=bits)
+    t = tokens_of(cfg, 140, 3)
+    c.run(0, t, [100, 1, 2, 37], "many experts")
+    c.free()
+
+
+def whole_config(**kw):
+    return u.config([(u.attention(v_mix=False, heads=4, dim=36, rot=20, vdim=12), u.moe()), (u.attention(), u.moe(experts=9, identity=1, top=4, ff=40, shared_ff=0)), (u.attention(heads=8, dim=16, rot=16, base=900.0, scale=0.7), None),
+                     (u.attention(scaling=None), u.moe(experts=3, identity=3, top=2, limit=0.7))], **kw)
+
+
+@pytest.mark.parametrize("act", ["f32", "bf16"])
+@pytest.mark.parametrize("portions", [[300], [1], [2], [3, 2], [64], [63, 1, 65], [31, 33, 2, 1, 120], [17, 16, 15]], ids=str)
+def test_portions(xh, act, portions):
+    cfg = whole_config()
+    c = Case(xh, cfg, 6, act)
+    n = 300 if portions != [1] else 150
+    c.run(0, tokens_of(cfg, n, 3), portions, "portions")
+    c.free()
+
+
+@pytest.mark.parametrize("act", ["f32", "bf16"])
+def test_first_tokens(xh, act):
+    """sequences of 1 .. 6 tokens, in a slot another sequence has used before"""
+    cfg = whole_config()
+    c = Case(xh, cfg, 7, act, slots=1)
+    for n in range(1, 7):
+        c.run(0, tokens_of(cfg, n, 40 + n), [n], f"{n} tokens")
+        c.model.seq_release(0)
+        c.run(0, tokens_of(cfg, n, 50 + n), [1], f"{n} tokens one by one")
+        c.model.seq_release(0)
+    c.free()
+
+
+@pytest.mark.parametrize("act", ["f32", "bf16"])
+def test_unequal_batches_and_reuse(xh, act):
+    """Sequences come, rest, go on and end; portions of some beside single tokens of others; the pool is as small as the
+    live sequences allow, so that pages and slots change hands all the time."""
+    cfg = whole_config()
+    slots, pool = 4, 9 * 64
+    c = Case(xh, cfg, 8, act, slots=slots, max_seq=512, max_tokens=512, pool=pool)
+    rng = np.random.default_rng(9)
+    live, made, steps = {}, 0, 0
+    while made < 14 or live:
+        for s in range(slots):
+            pages = sum(-(-len(q["t"]) // 64) for q in live.values())
+            if s not in live and made < 14 and rng.random() < 0.7:
+                n = int(rng.choice([1, 2, 5, 63, 64, 65, 130, 200]))
+                if pages + -(-n // 64) > 9:
+                    continue
+                t = tokens_of(cfg, n, 100 + made)
+                live[s] = dict(t=t, at=0, want=c.want(t))
+                made += 1
+        entries, expect = [], []
+        for s in rng.permutation(list(live)):
+            q = live[s]
+            if rng.random() < 0.25:
+                continue
+            n = min(int(rng.choice([1, 1, 2, 3, 17, 40, 64, 90])), len(q["t"]) - q["at"])
+            places = list(range(n)) if rng.random() < 0.8 else []
+            entries.append((int(s), q["t"][q["at"]:q["at"] + n], places))
+            if places:
+                expect.append(q["want"][q["at"]:q["at"] + n])
+            q["at"] += n
+        if not entries:
+            continue
+        got = c.model.step(entries)
+        if expect:
+            c.check(got, np.concatenate(expect), f"step {steps}")
+        steps += 1
+        for s in [s for s in live if live[s]["at"] == len(live[s]["t"])]:
+            c.model.seq_release(s)
+            del live[s]
+    assert c.model.pool_pages() == (9, 9)
+    c.free()
+
+
+def test_a_batch_gives_what_each_alone_gives(xh):
+    """single tokens, short and long portions in one step, beyond the few-row products: the same logits as one by one"""
+    cfg = whole_config()
+    for act, limit in (("f32", 1e-5), ("bf16", 0.03)):
+        c = Case(xh, cfg, 16, act, slots=4)
+        seqs = [tokens_of(cfg, n, 20 + n) for n in (130, 70, 41, 9)]
+        cut = [65, 69, 40, 2]
+        alone = [np.concatenate([c.model.step([(s, t[:k], list(range(k)))]), c.model.step([(s, t[k:], list(range(len(t) - k)))])])
+                 for s, (t, k) in enumerate(zip(seqs, cut))]
+        for s in range(4):
+            c.model.seq_release(s)
+        order = [2, 0, 3, 1]
+        got = [c.model.step([(s, seqs[s][:cut[s]], list(range(cut[s]))) for s in order]),
+               c.model.step([(s, seqs[s][cut[s]:], list(range(len(seqs[s]) - cut[s]))) for s in order])]
+        want = [np.concatenate([alone[s][:cut[s]] for s in order]), np.concatenate([alone[s][cut[s]:] for s in order])]
+        for g, w in zip(got, want):
+            assert u.rel_rms(g, w).max() < limit
+        c.free()
+
+
+SHAPES = {  # the attention kernels' forms: (query / key, value) sizes of a head
+    "128_128": dict(heads=4, kv_heads=2, dim=128, vdim=128, rot=64),
+    "192_128": dict(heads=3, kv_heads=1, dim=192, vdim=128, rot=64),
+    "64_64": dict(heads=16, kv_heads=2, dim=64, vdim=64, rot=64),
+    "odd": dict(heads=6, kv_heads=3, dim=90, vdim=70, rot=50),
+    "small": dict(heads=5, kv_heads=5, dim=20, vdim=12, rot=12),
+    "large": dict(heads=2, kv_heads=1, dim=256, vdim=200, rot=128),
+    "larger": dict(heads=1, kv_heads=1, dim=290, vdim=288, rot=32),
+}
+
+
+@pytest.mark.parametrize("act", ["f32", "bf16"])
+@pytest.mark.parametrize("name", sorted(SHAPES))
+@pytest.mark.parametrize("window", [0, 50])
+def test_needle(xh, name, window, act):
+    """One key decides every later answer.  It is planted at a page's border and elsewhere, and read far away, just inside and
+    just outside a window (the kernels' option), in prompts, in portions and by decoded tokens."""
+    m = u.attention(base=5e5, scaling=None, v_mix=None, scale=10.0 / SHAPES[name]["dim"], **SHAPES[name])
+    m["_window"] = window
+    cfg = u.config([(m, None)], width=96, side=0)
+    bits = u.needle_weights(cfg, 3, key_token=7)
+    c = Case(xh, cfg, 0, act, slots=3, max_seq=448, bits=bits)
+    for place in (0, 31, 63, 64, 100, 127):
+        t = np.random.default_rng(place).integers(8, cfg["vocab"], 260)
+        t[place] = 7
+        want = c.want(t)
+        t2 = t.copy()
+        t2[place] = 9
+        seen = u.rel_rms(want, c.want(t2))
+        last = place + (window or 400) - 1  # the last position that sees the needle
+        shows = float(seen[place + 1:min(last, 259) + 1].min())
+        assert shows > 3 * LIMIT["bf16"] and (last + 1 > 259 or seen[last + 1] < 1e-9), f"the needle does not show ({shows:.3f})"
+        c.run(0, t, [260], f"{name} needle at {place}, prompt", want)
+        c.run(1, t, [place + 20, 2, 1, 1, 1, 7], f"{name} needle at {place}, portions", want)
+        if window:
+            c.run(2, t[:last + 4], [last - 2, 1], f"{name} needle at {place}, decoded over the edge", want)
+        for s in range(3):
+            c.model.seq_release(s)
+    c.free()
+
+
+def test_sink_takes_its_weight(xh):
+    """sinks far above every score leave little to the values, one far below nothing to itself"""
+    cfg = u.config([(u.attention(heads=3, kv_heads=1, scale=0.05, **PLAIN), None)], side=0)
+    bits = u.weights(cfg, 4)
+    bits["l0.mix.sink"] = u.bf16_bits(np.array([5.0, -30.0, 2.0]))
+    for act in ("f32", "bf16"):
+        c = Case(xh, cfg, 0, act, bits=bits)
+        t = tokens_of(cfg, 200, 5)
+        want = c.want(t)
+        c.run(0, t, [200], "prompt", want)
+        c.run(1, t, [190, 1], "decoded", want)
+        w2 = dict(c.w, **{"l0.mix.sink": np.full(3, -1e9)})
+        assert u.rel_rms(ref.forward(cfg, w2, t), want).min() > LIMIT["bf16"] * 0.5
+        c.free()
+
+
+def test_split_contexts_and_long_portions(xh):
+    """long contexts over many parts of the chip, decoded, in short and in long portions"""
+    cfg = u.config([(u.attention(heads=8, kv_heads=2, dim=128, vdim=128, rot=64, scale=0.2), None), (u.attention(heads=20, kv_heads=2, dim=64, vdim=128, scale=0.3), None)], width=128)
+    c = Case(xh, cfg, 12, "bf16", slots=3, max_seq=1600, max_tokens=1600)
+    t = tokens_of(cfg, 1500, 6)
+    want = c.want(t)
+    c.run(0, t, [1400, 1, 1, 2, 5, 16, 1, 17, 56], "long", want)
+    for s in (1, 2):
+        c.model.step([(s, t[:700 + s], [])])
+    got = c.model.step([(1, t[701:702], [0]), (2, t[702:705], [0, 1, 2])])
+    c.check(got, want[[701, 702, 703, 704]], "side by side")
+    got = c.model.step([(1, t[702:802], [0, 99]), (2, t[705:706], [0])])
+    c.check(got, want[[702, 801, 705]], "a long portion beside a token")
+    c.free()
+
+
+@pytest.mark.parametrize("act", ["f32", "bf16"])
+def test_long_decoding(xh, act):
+    """greedy decoding by graph replay: every step's chosen ids and the last logits, then the same steps launched one by one"""
+    cfg = whole_config()
+    c = Case(xh, cfg, 13, act, slots=2, max_seq=400, max_tokens=256)
+    prompts = np.stack([tokens_of(cfg, 30, 60), tokens_of(cfg, 30, 61)]).astype(np.int32)
+    runs = []
+    for graph in (True, False):
+        c.model.use_graph(graph)
+        first, logits = c.model.prefill(prompts, want_logits=True)
+        for b in range(2):
+            c.check(logits[b:b + 1], c.want(prompts[b])[-1:], "prompt")
+        ids = [first] + list(c.model.decode(170, 2)) + list(c.model.decode(70, 2))
+        runs.append((np.stack(ids), c.model.logits(2)))
+    np.testing.assert_array_equal(runs[0][0], runs[1][0])
+    np.testing.assert_array_equal(runs[0][1], runs[1][1])
+    ids = runs[0][0]
+    for b in range(2):
+        full = np.concatenate([prompts[b], ids[:-1, b]])
+        want = c.want(full)
+        for i, row in enumerate(want[29:]):
+            assert row.max() - row[ids[i, b]] <= 3 * c.limit * want.std(), f"sequence {b}, step {i}"
+        c.check(runs[0][1][b:b + 1], want[-1:], f"sequence {b}: logits behind 240 decoded tokens")
+    c.free()
+
+
+def test_slots_that_sit_out(xh):
+    cfg = whole_config()
+    c = Case(xh, cfg, 14, "f32", slots=3, max_seq=256)
+    seqs = [list(tokens_of(cfg, n, 70 + n)) for n in (20, 33, 5)]
+    for s, t in enumerate(seqs):
+        c.model.seq_prefill(s, t)
+    for rows in ([2], [0, 2], [1], [2, 1], [0], [0, 1, 2]):
+        for r in rows:
+            i = int(c.want(seqs[r])[-1].argmax())
+            c.model.seq_set_next_id(r, i)
+            seqs[r].append(i)
+        c.model.seq_decode(rows)
+        for r in rows:
+            c.check(c.model.seq_logits(r)[None], c.want(seqs[r])[-1:], f"slot {r} of {rows}")
+    # a copy of a slot goes on by itself
+    c.model.seq_reorder([2, 0], [1, 1], 0, 0)
+    for r in (0, 2):
+        seqs[r] = list(seqs[1])
+    for r, tok in ((0, 3), (1, 4), (2, 5)):
+        c.model.seq_set_next_id(r, tok)
+        seqs[r].append(tok)
+    c.model.seq_decode([0, 1, 2])
+    for r in range(3):
+        c.check(c.model.seq_logits(r)[None], c.want(seqs[r])[-1:], f"copied slot {r}")
+    c.free()
+
+
+def test_broken_plans_are_refused(xh):
+    good = dict(u.plan_layers(u.config([(u.attention(), u.moe())]))[0])
+    for change in (dict(heads=5), dict(rot_dim=21), dict(top=8), dict(top=0), dict(expert_inter=0), dict(dim=600)):
+        with pytest.raises(xh.XftHipError):
+            xh.Plan(72, 90, [dict(good, **change)], block=1, norm=1, tied_head=1)
+    with pytest.raises(xh.XftHipError):  # values that do not fit those they are mixed with
+        xh.Plan(72, 90, [good, dict(good, vdim=30)], block=1, norm=1, tied_head=1)
+    cfg = u.config([(u.attention(), u.moe())])
+    bits = u.weights(cfg, 1)
+    for name in ("l0.mlp.e3.up", "l0.norm2.alpha", "l0.side.proj", "l0.mix.k.norm"):
+        with pytest.raises(xh.XftHipError, match=name.split(".")[-1]):
+            u.build_plan(xh, cfg, {k: v for k, v in bits.items() if k != name})
+
+
+# ---- through the framework's own entry points -----------------------------------------------------------------------------
+@pytest.fixture(scope="module")
+def model_dir(tmp_path_factory):
+    cfg = whole_config()
+    bits = u.steady_weights(cfg, 21)
+    path = str(tmp_path_factory.mktemp("plan") / "model")
+    u.write_model(path, cfg, bits)
+    return path, cfg, u.oracle_weights(bits)
+
+
+def greedy(cfg, w, prompt, n):
+    t = list(prompt)
+    for _ in range(n):
+        t.append(int(ref.forward(cfg, w, t)[-1].argmax()))
+    return t
+
+
+def test_generate(xh, model_dir):
+    from xfastertransformer_amd.automodel import AutoModel
+    path, cfg, w = model_dir
+    m = AutoModel.from_pretrained(path, "fp32")
+    assert m.vocab_size == cfg["vocab"]
+    prompts = [list(tokens_of(cfg, 17, 80)), list(tokens_of(cfg, 17, 81))]
+    expect = [greedy(cfg, w, p, 23) for p in prompts]
+    out = m.generate(np.array(prompts, np.int32), max_length=40)
+    np.testing.assert_array_equal(out, expect)
+    out = m.generate(np.array(prompts[:1], np.int32), max_length=30, num_beams=3)
+    assert out.shape[1] >= 30 and out[0, :17].tolist() == prompts[0]
+    out = m.generate(np.array(prompts, np.int32), max_length=30, do_sample=True, top_k=5)
+    assert out.shape == (2, 30) and out.max() < cfg["vocab"]
+    # sequences by id, of different lengths, stepping and ending independently
+    a, b = m.set_input_cb([prompts[0], prompts[1][:5]], max_length=40)
+    got = {a: [], b: []}
+    for i, x in zip((a, b), m.forward_cb()):
+        got[i].append(x)
+    for ids in ([a, b], [b], [a], [a, b]):
+        m.set_input_cb(seq_ids=ids, max_length=40)
+        for i, x in zip(ids, m.forward_cb()):
+            got[i].append(x)
+    assert prompts[0] + got[a] == expect[0][:17 + 4]
+    assert prompts[1][:5] + got[b] == greedy(cfg, w, prompts[1][:5], 4)
+    m.free_seqs([a, b])
+    m.free()
+    m = AutoModel.from_pretrained(path, "bf16")
+    out = m.generate(np.array(prompts, np.int32), max_length=40)
+    for b in range(2):
+        want = ref.forward(cfg, w, out[b, :-1])[16:]
+        for i, row in enumerate(want):
+            assert row.max() - row[out[b, 17 + i]] <= 3 * LIMIT["bf16"] * want.std()
+    m.free()
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_trace_run(xh, model_dir, tmp_path, dtype):
+    path, cfg, w = model_dir
+    seqs = {"a": tokens_of(cfg, 70, 90), "b": tokens_of(cfg, 9, 91), "c": tokens_of(cfg, 66, 92), "d": tokens_of(cfg, 3, 93), "e": tokens_of(cfg, 80, 94)}
+    plan = [[("a", 60), ("b", 3)], [("b", 1), ("c", 30), ("a", 1)], [("d", 3), ("b", 5), ("a", 2)], [("e", 80), ("c", 36)], [("a", 7)]]
+    at, lines, expect = {k: 0 for k in seqs}, [], {}
+    for n, step in enumerate(plan):
+        entries, rows, end = [], [], []
+        for k, c in step:
+            entries.append(dict(id=k, tokens=seqs[k][at[k]:at[k] + c].tolist(), want=[0, c - 1] if n != 1 else []))
+            rows += [ref.forward(cfg, w, seqs[k])[[at[k], at[k] + c - 1]]] if n != 1 else []
+            at[k] += c
+            if at[k] == len(seqs[k]):
+                end.append(k)
+        lines.append(json.dumps(dict(step=n, entries=entries, end=end)))
+        if rows:
+            expect[n] = np.concatenate(rows)
+    p = subprocess.run([os.path.join(ROOT, "bin", "trace_run"), "--model", path, "--dtype", dtype, "--out", str(tmp_path), "--max-tokens", "384"],
+                       input="\n".join(lines) + "\n", capture_output=True, text=True, timeout=100)
+    assert p.returncode == 0, p.stderr[-2000:]
+    assert [l for l in p.stdout.splitlines() if l.startswith("done")] == ["done %d" % n for n in range(len(plan))]
+    assert not (tmp_path / "1.f32").exists()
+    for n, want in expect.items():
+        got = np.fromfile(tmp_path / ("%d.f32" % n), "<f4").reshape(-1, cfg["vocab"])
+        assert u.rel_rms(got, want).max() < LIMIT["f32" if dtype == "float32" else "bf16"]
