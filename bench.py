@@ -606,6 +606,7 @@ def moe_layer(xh, iters=5):
                      "counts stay on the device)")
 
 
+PLAN_MODELS = ("pinepel", "llama_bf16", "veterax", "mixtral_bf16")
 PLAN_SIZES = {
     # width, ff, heads, query latent (the rest: 128 / 64 query dims, 128 value dims, key latent 512, 128-dim delta heads)
     "2048": dict(width=2048, ff=5632, heads=16, q_rank=768),
@@ -634,6 +635,54 @@ def plan_shapes(sz):
     return kinds * 2, shapes * 2
 
 
+# the stacks with sparse MLPs: key / value heads of 128, experts, chosen, width of an expert and of the shared one, identity outputs
+SPARSE_SIZES = {
+    "2048": dict(kv_heads=4, experts=8, top=2, ff=2816, shared=2816, identity=2),
+    "4096": dict(kv_heads=8, experts=8, top=2, ff=2752, shared=5504, identity=2),
+    "2048x64": dict(kv_heads=4, experts=64, top=6, ff=1408, shared=2816, identity=8),  # (the uniform stack's sparse MLP has 8 experts)
+}
+
+
+def veterax_shapes(sz, sp):
+    """Layer descriptions and tensor shapes of a Veterax stack: grouped attention with mixed values and a sink, routed experts beside a
+    shared one, a side embedding of 256."""
+    W, H, G, S = sz["width"], sz["heads"], sp["kv_heads"], 256
+    layer = dict(mixer=3, heads=H, kv_heads=G, dim=128, vdim=128, rot_dim=128, rot_interleaved=1, rot_base=1e6, rot_factor=4.0, rot_original=8192, rot_fast=32.0,
+                 rot_slow=1.0, scale=128 ** -0.5, has_sink=1, qk_norm=1, v_mix=1, inter=sp["shared"], glu_limit=7.0, glu_alpha=1.702, experts=sp["experts"],
+                 identity=sp["identity"], top=sp["top"], expert_inter=sp["ff"], expert_limit=7.0)
+    n = sp["experts"] + sp["identity"]
+    t = {"mix.q": (H * 128, W), "mix.k": (G * 128, W), "mix.v": (G * 128, W), "mix.q.norm": (128,), "mix.k.norm": (128,), "mix.sink": (H,), "mix.vmix": (1,),
+         "mix.o": (W, H * 128), "mlp.router": (n, W), "mlp.correction": (n,), "side.gate": (S, W), "side.proj": (W, S), "side.norm": (W,)}
+    for n in ("norm1", "norm2"):
+        t[n], t[n + ".b"], t[n + ".alpha"] = (W,), (W,), (1,)
+    for p, ff in [("e%d." % e, sp["ff"]) for e in range(sp["experts"])] + [("shared.", sp["shared"])]:
+        t["mlp." + p + "gate"], t["mlp." + p + "up"], t["mlp." + p + "down"] = (ff, W), (ff, W), (W, ff)
+    return [layer] * 6, [t] * 6, S
+
+
+def build_veterax(xh, sz, sp, vocab=32000):
+    layers, shapes, side = veterax_shapes(sz, sp)
+    W, rng = sz["width"], np.random.default_rng(5)
+    pool = xh.f32_to_bf16_bits(rng.standard_normal(1 << 22, dtype=np.float32) * 0.02)
+    plan = xh.Plan(W, vocab, layers, block=xh.BLOCK_PARALLEL, norm=xh.NORM_DYNAMIC_TANH, tied_head=1, side_dim=side)
+
+    def bits(name, shape):
+        n, leaf = int(np.prod(shape)), name.split(".")[-1]
+        if leaf == "alpha" or leaf.startswith("norm"):
+            return np.full(shape, xh.f32_to_bf16_bits(np.array([0.5 if leaf == "alpha" else 1.0], np.float32))[0], np.uint16)
+        return np.resize(np.roll(pool, int(rng.integers(1 << 20))), n).reshape(shape)
+
+    embed = xh.f32_to_bf16_bits(rng.standard_normal((vocab, W), dtype=np.float32))
+    for n, b in (("embed", embed), ("side.embed", bits("side.embed", (vocab, side * len(layers)))), ("final.norm", bits("norm", (W,))),
+                 ("final.norm.b", bits("b", (W,))), ("final.norm.alpha", bits("alpha", (1,)))):
+        plan.set(-1, n, b)
+    for l, tensors in enumerate(shapes):
+        for n, s in tensors.items():
+            plan.set(l, n, bits(n, s))
+    plan.finish()
+    return plan
+
+
 def build_plan(xh, sz, vocab=32000):
     layers, shapes = plan_shapes(sz)
     pool = xh.f32_to_bf16_bits(np.random.default_rng(5).standard_normal(1 << 22, dtype=np.float32) * 0.02)
@@ -655,42 +704,54 @@ def build_plan(xh, sz, vocab=32000):
     return plan
 
 
-def build_llama_bf16(xh, sz, layers, batch, max_seq, max_tokens, vocab=32000):
-    """The closest uniform stack: same width, feed-forward and layer count, multi-head attention, BF16 weights."""
+def build_llama_bf16(xh, sz, layers, batch, max_seq, max_tokens, vocab=32000, sparse=None):
+    """The closest uniform stack: same width, feed-forward and layer count, multi-head attention, BF16 weights; sparse: grouped
+    key / value heads and the sparse MLP (8 experts, two a token) of these sizes instead."""
     W, F, H = sz["width"], sz["ff"], sz["width"] // 128
+    G = sparse["kv_heads"] if sparse else H
     pool = xh.f32_to_bf16_bits(np.random.default_rng(5).standard_normal(1 << 22, dtype=np.float32) * 0.02)
-    model = xh.Model(layers, W, F, H, H, 128, vocab=vocab, max_batch=batch, max_seq=max_seq, max_tokens=max_tokens, max_pos_embed=max_seq)
+    model = xh.Model(layers, W, sparse["ff"] if sparse else F, H, G, 128, vocab=vocab, max_batch=batch, max_seq=max_seq, max_tokens=max_tokens, max_pos_embed=max_seq)
     ones = np.ones(W, np.float32)
-    ws = []
+    ws, moes = [], []
+
+    def weight(K, N, glu=False):
+        ws.append(xh.Weight(xh.W_BF16, K, N, np.resize(pool, K * N), flags=xh.WF_GATEUP if glu else xh.WF_NONE))
+        return ws[-1]
+
     for l in range(layers):
-        w = [xh.Weight(xh.W_BF16, K, N, np.resize(pool, K * N), flags=xh.WF_GATEUP if i == 2 else xh.WF_NONE)
-             for i, (K, N) in enumerate(((W, 3 * W), (W, W), (W, 2 * F), (F, W)))]
-        model.set_layer(l, *w, ones, ones)
-        ws += w
-    lm = xh.Weight(xh.W_BF16, W, vocab, np.resize(pool, W * vocab))
+        qkv, o = weight(W, (H + 2 * G) * 128), weight(W, W)
+        if sparse:
+            router = np.random.default_rng(l).standard_normal((W, 8), dtype=np.float32) * 0.02
+            moes.append(xh.MoE(W, sparse["ff"], 8, max_tokens, router, ones, beside=moes[0] if moes else None))
+            for e in range(8):
+                moes[-1].set_expert(e, weight(W, 2 * sparse["ff"], True), weight(sparse["ff"], W))
+            model.set_sparse_layer(l, qkv, o, moes[-1], ones)
+        else:
+            model.set_layer(l, qkv, o, weight(W, 2 * F, True), weight(F, W), ones, ones)
+    lm = weight(W, vocab)
     emb = (np.random.default_rng(6).standard_normal((vocab, W), dtype=np.float32) * 0.02).astype(np.float16).view(np.uint16)
     model.set_head(emb, ones, lm)
-    return model, ws + [lm]
+    return model, moes[::-1] + ws
 
 
 def plan_bench(xh, prompt=2048, batches=(1, 8, 32), steps=32, only=None, sizes=None, eager=False):
-    """Prefill (one prompt) and decode (behind prompts of that length) of Pinepel beside the uniform stack, six layers
-    each, in the same run.  Prompts of a decode batch are run one by one."""
+    """Prefill (one prompt) and decode (behind prompts of that length) of Pinepel beside the uniform stack and of Veterax beside the
+    uniform stack with sparse MLPs, six layers each, in the same run.  Prompts of a decode batch are run one by one."""
     out = []
-    for name in sizes or PLAN_SIZES:
-        sz = PLAN_SIZES[name]
-        for which in ("pinepel", "llama_bf16"):
-            if only and which != only:
+    for name in sizes or list(PLAN_SIZES) + [n for n in SPARSE_SIZES if n not in PLAN_SIZES]:
+        sz, sp = PLAN_SIZES[name.split("x")[0]], SPARSE_SIZES[name]
+        for which in PLAN_MODELS:
+            if (only and which != only) or (name not in PLAN_SIZES and which != "veterax"):
                 continue
             B, max_seq = max(batches), prompt + 4 * (steps + 8)
             keep = []
-            if which == "pinepel":
-                plan = build_plan(xh, sz)
+            if which in ("pinepel", "veterax"):
+                plan = build_plan(xh, sz) if which == "pinepel" else build_veterax(xh, sz, sp)
                 model, wbytes = xh.PlanModel(plan, xh.BF16, B, max_seq, prompt), plan.bytes()
                 keep = [plan]
             else:
-                model, keep = build_llama_bf16(xh, sz, 6, B, max_seq, prompt)
-                wbytes = sum(w.bytes() for w in keep)
+                model, keep = build_llama_bf16(xh, sz, 6, B, max_seq, prompt, sparse=sp if which == "mixtral_bf16" else None)
+                wbytes = sum(w.bytes() for w in keep if hasattr(w, "bytes"))
             model.use_graph(not eager)
             ids = np.random.default_rng(7).integers(0, 32000, (1, prompt)).astype(np.int32)
             times = []
@@ -699,11 +760,11 @@ def plan_bench(xh, prompt=2048, batches=(1, 8, 32), steps=32, only=None, sizes=N
                 model.prefill(ids)
                 xh.synchronize()
                 times.append(time.time() - t0)
-            r = dict(model=which, width=sz["width"], layers=6, weight_bytes=wbytes, prompt=prompt, prefill_ms=round(min(times[1:]) * 1e3, 3),
+            r = dict(model=which, size=name, width=sz["width"], layers=6, weight_bytes=wbytes, prompt=prompt, prefill_ms=round(min(times[1:]) * 1e3, 3),
                      prefill_tok_s=round(prompt / min(times[1:]), 1), decode=[])
             for b in batches:
                 for row in range(b):
-                    model.seq_prefill(row, ids[0])
+                    model.seq_prefill(row, np.random.default_rng(7 + row).integers(0, 32000, prompt).astype(np.int32))
                 rows = list(range(b))
                 for _ in range(4):
                     model.seq_decode(rows)
@@ -740,9 +801,9 @@ def main():
     ap.add_argument("--prefill-gemm", action="store_true", help="only the weight-only GEMM sweep: M = 256, 2048 against the MFMA peak, M = 1, 8, 32 against the HBM peak (one JSON line)")
     ap.add_argument("--attention", action="store_true", help="only the GQA attention sweep (one JSON line)")
     ap.add_argument("--moe", action="store_true", help="only the sparse-MLP layer (one JSON line)")
-    ap.add_argument("--plan", action="store_true", help="only the layer-plan stack (Pinepel) beside the uniform BF16 stack of equal size: prefill and decode (one JSON line; progress on stderr)")
-    ap.add_argument("--plan-only", choices=["pinepel", "llama_bf16"], help="with --plan: one of the two")
-    ap.add_argument("--plan-size", choices=sorted(PLAN_SIZES), help="with --plan: one width")
+    ap.add_argument("--plan", action="store_true", help="only the layer-plan stacks (Pinepel, Veterax) beside the uniform BF16 stacks of equal size (dense, sparse MLPs): prefill and decode (one JSON line; progress on stderr)")
+    ap.add_argument("--plan-only", choices=PLAN_MODELS, help="with --plan: one of them")
+    ap.add_argument("--plan-size", choices=sorted(SPARSE_SIZES), help="with --plan: one size")
     ap.add_argument("--no-live-traffic", action="store_true", help="do not run the two rocprofv3 counter passes for roofline.traffic (the recorded figure under profiles/ is reported instead)")
     ap.add_argument("--stream-floor", action="store_true", help="only the read-only streaming floor at the decode GEMVs' byte counts (one JSON line)")
     args = ap.parse_args()

@@ -283,6 +283,22 @@ def test_long_decoding(xh, act):
     c.free()
 
 
+@pytest.mark.parametrize("act", ["f32", "bf16"])
+def test_many_sequences_decode_together(xh, act):
+    """more sequences than the few-row products take, by graph replay"""
+    cfg = whole_config()
+    n = 45
+    c = Case(xh, cfg, 18, act, slots=n, max_seq=64, max_tokens=n * 8)
+    prompts = np.stack([tokens_of(cfg, 7, 200 + i) for i in range(n)]).astype(np.int32)
+    first, _ = c.model.prefill(prompts, want_logits=True)
+    ids = [first] + list(c.model.decode(6, n))
+    logits = c.model.logits(n)
+    for b in range(n):
+        full = np.concatenate([prompts[b], np.stack(ids)[:-1, b]])
+        c.check(logits[b:b + 1], c.want(full)[-1:], f"sequence {b}")
+    c.free()
+
+
 def test_slots_that_sit_out(xh):
     cfg = whole_config()
     c = Case(xh, cfg, 14, "f32", slots=3, max_seq=256)

@@ -350,41 +350,53 @@ __global__ __launch_bounds__(256, (KS <= 4 && VT <= 8) ? 3 : 1) void grouped_sho
     }
 }
 
-// sum of a column's splits; grid (G * column groups, segments, 16 columns), 64 threads
+// sum of a column's splits; grid (G * column groups, segments, 16 columns).  Four neighbouring dimensions a thread, the splits
+// dealt out to as many sets of threads as a workgroup holds.
 constexpr int kMaxSplits = 64;
-__global__ __launch_bounds__(64) void grouped_merge_kernel(AttendParams p) {
-    __shared__ float w[kMaxSplits];
+__global__ __launch_bounds__(256) void grouped_merge_kernel(AttendParams p) {
+    __shared__ float w[kMaxSplits], inv_den;
+    __shared__ f32x4 sums[256];
     const StepView &v = p.v;
     const int seg = blockIdx.y, n = v.seg_len[seg], gs = p.H / p.G, V = p.V;
     const int g = blockIdx.x / p.groups, c = (blockIdx.x - g * p.groups) * 16 + blockIdx.z;
     if (n < p.min_len || n > p.max_len || c >= n * gs) return;
-    const int head = g * gs + c % gs, lane = threadIdx.x;
+    const int head = g * gs + c % gs, per = V / 4, sets = 256 / per;
+    const int set = (int)threadIdx.x / per, d = (int)threadIdx.x % per * 4;
     const size_t slot0 = ((size_t)seg * gridDim.x + blockIdx.x) * p.nsplit * 16 + blockIdx.z;
-    float2 ml = make_float2(kUnseen, 0.0f);
-    if (lane < p.nsplit) ml = *(const float2 *)(p.part + p.part_ml + (slot0 + (size_t)lane * 16) * 2);
-    const float s2 = p.sink ? p.sink[head] * kLog2e : kUnseen;
-    const float mt = fmaxf(wave_largest(ml.x), s2);
-    const float e = ml.x > 0.5f * kUnseen ? __builtin_amdgcn_exp2f(ml.x - mt) : 0.0f;
-    const float den = wave_total(ml.y * e) + (p.sink ? __builtin_amdgcn_exp2f(s2 - mt) : 0.0f);
-    w[lane] = e;
-    __syncthreads();
-    const float inv = 1.0f / den;
-    uint16_t *dst = (uint16_t *)p.out + ((size_t)(v.seg_off[seg] + c / gs) * p.H + head) * V;
-    for (int d = lane * 4; d < V; d += 256) {
-        f32x4 acc[4];
+    // the first outputs are on their way while the weights are worked out
+    const float *src = p.part + slot0 * V + d;
+    const size_t step = (size_t)16 * V;
+    f32x4 x[4];
 #pragma unroll
-        for (int i = 0; i < 4; ++i) acc[i] = f32x4 {0.f, 0.f, 0.f, 0.f};
-        for (int s0 = 0; s0 < p.nsplit; s0 += 4) {
-            f32x4 x[4];
-#pragma unroll
-            for (int i = 0; i < 4; ++i) x[i] = *(const f32x4 *)(p.part + (slot0 + (size_t)(s0 + i < p.nsplit ? s0 + i : p.nsplit - 1) * 16) * V + d);
-#pragma unroll
-            for (int i = 0; i < 4; ++i)
-                if (s0 + i < p.nsplit) acc[i] += x[i] * w[s0 + i];
-        }
-        const f32x4 y = ((acc[0] + acc[1]) + (acc[2] + acc[3])) * inv;
-        *(uint2 *)(dst + d) = make_uint2(pack_pair(y[0], y[1]), pack_pair(y[2], y[3]));
+    for (int i = 0; i < 4; ++i) {
+        const int s = set + i * sets;
+        x[i] = *(const f32x4 *)(src + (s < p.nsplit ? s : 0) * step);
     }
+    if (threadIdx.x < 64) {
+        float2 ml = make_float2(kUnseen, 0.0f);
+        if ((int)threadIdx.x < p.nsplit) ml = *(const float2 *)(p.part + p.part_ml + (slot0 + (size_t)threadIdx.x * 16) * 2);
+        const float s2 = p.sink ? p.sink[head] * kLog2e : kUnseen;
+        const float mt = fmaxf(wave_largest(ml.x), s2);
+        const float e = ml.x > 0.5f * kUnseen ? __builtin_amdgcn_exp2f(ml.x - mt) : 0.0f;
+        const float den = wave_total(ml.y * e) + (p.sink ? __builtin_amdgcn_exp2f(s2 - mt) : 0.0f);
+        w[threadIdx.x] = e;
+        if (threadIdx.x == 0) inv_den = 1.0f / den;
+    }
+    __syncthreads();
+    f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+    if (set < sets) {
+#pragma unroll
+        for (int i = 0; i < 4; ++i)
+            if (set + i * sets < p.nsplit) acc += x[i] * w[set + i * sets];
+        for (int s = set + 4 * sets; s < p.nsplit; s += sets) acc += *(const f32x4 *)(src + s * step) * w[s];
+    }
+    sums[threadIdx.x] = acc;
+    __syncthreads();
+    if (set > 0) return;
+    for (int s = 1; s < sets; ++s) acc += sums[s * per + threadIdx.x];
+    acc *= inv_den;
+    uint16_t *dst = (uint16_t *)p.out + ((size_t)(v.seg_off[seg] + c / gs) * p.H + head) * V + d;
+    *(uint2 *)dst = make_uint2(pack_pair(acc[0], acc[1]), pack_pair(acc[2], acc[3]));
 }
 
 // BF16, long form: 128 columns a workgroup (32 a wave), the visible context in blocks of 32 tokens through LDS, on 32 x 32 tiles.
@@ -626,7 +638,7 @@ int grouped_attention(int act, const PlanLayer &L, const StepView &v, const void
     else if (ks <= 4 && vt <= 8) rc = launch_short<4, 8, false>(p, st);
     else rc = launch_short<8, 16, false>(p, st);
     if (rc || p.nsplit == 1) return rc;
-    hipLaunchKernelGGL(grouped_merge_kernel, dim3(s.kv_heads * p.groups, v.B, 16), dim3(64), 0, st, p);
+    hipLaunchKernelGGL(grouped_merge_kernel, dim3(s.kv_heads * p.groups, v.B, 16), dim3(256), 0, st, p);
     XFT_CHECK_HIP(hipGetLastError());
     return 0;
 }

@@ -97,10 +97,11 @@ int rotation_tables(const xfthip_plan_layer &s, int positions, float **cosT, flo
 }
 
 int plan_gemm(xfthip_model *m, xfthip_weight_t w, int M, const void *A, int lda, void *C, int ldc, int c_dtype, hipStream_t st) {
-    if (m->plan->act == XFTHIP_F32) {
+    // (few rows against few columns: the form with the most waves along K)
+    if (m->plan->act == XFTHIP_F32 || (M <= 32 && w->pw.N <= 256 && w->pw.K >= 1024)) {
         TileGemmArgs a;
         a.M = M, a.A = A, a.lda = lda, a.C = C, a.ldc = ldc, a.c_dtype = c_dtype;
-        return tile_gemm(w, XFTHIP_F32, a, st);
+        return tile_gemm(w, m->plan->act, a, st);
     }
     return xfthip_gemm(w, M, A, lda, C, ldc, c_dtype, XFTHIP_EPI_NONE, nullptr, nullptr, 0, XFTHIP_F32, 1.0f, st);
 }

@@ -37,23 +37,23 @@ __device__ inline void route_one(const RouteParams &p, int t, int lane) {
         choice[i] = i * 64 + lane < p.routes ? z[i] + choice[i] : -INFINITY;
     }
     for (int k = 0; k < p.top; ++k) {
-        float best = -INFINITY, score = 0.0f;
-        int at = 1 << 20;
+        float best = choice[0];
 #pragma unroll
-        for (int i = 0; i < CH; ++i)
-            if (choice[i] > best) best = choice[i], score = z[i], at = i * 64 + lane;
+        for (int i = 1; i < CH; ++i) best = fmaxf(best, choice[i]);
+        best = wave_largest(best);
+        // (scores that are not numbers equal nothing: the last output then, with a weight that is none either)
+        int e = p.routes - 1;
+        float score = sum;
+        bool open = true;
 #pragma unroll
-        for (int off = 32; off > 0; off >>= 1) {
-            const float ob = __shfl_xor(best, off, 64), os = __shfl_xor(score, off, 64);
-            const int oa = __shfl_xor(at, off, 64);
-            if (ob > best || (ob == best && oa < at)) best = ob, score = os, at = oa;
+        for (int i = 0; i < CH; ++i) {
+            const unsigned long long at = open ? __ballot(choice[i] == best) : 0ull;
+            if (at == 0ull) continue;
+            const int who = __ffsll(at) - 1;
+            open = false, e = i * 64 + who, score = __shfl(z[i], who, 64);
+            if (lane == who) choice[i] = -INFINITY;
         }
-        // (scores that are not numbers choose nothing: the last output, with their weight)
-        const int e = at < p.routes ? at : p.routes - 1;
-        if (lane == 0) p.b.sel[(size_t)t * p.top + k] = e, p.b.weight[(size_t)t * p.top + k] = at < p.routes ? score : sum;
-#pragma unroll
-        for (int i = 0; i < CH; ++i)
-            if (i * 64 + lane == at) choice[i] = -INFINITY;
+        if (lane == 0) p.b.sel[(size_t)t * p.top + k] = e < p.routes ? e : p.routes - 1, p.b.weight[(size_t)t * p.top + k] = score;
     }
 }
 

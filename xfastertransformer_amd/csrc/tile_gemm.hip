@@ -28,16 +28,17 @@ __device__ inline float precise_glu(float gate, float up, float limit, float alp
     return g / (1.0f + expf(-alpha * g)) * (u + 1.0f);
 }
 
-// A wave: two column tiles (16 weight columns each) x MT row tiles (16 activation rows each).  The weight tile is the MFMA
+// A wave: TW column tiles (16 weight columns each; two, or one in the 16-wave form) x MT row tiles (16 activation rows each).  The weight tile is the MFMA
 // A operand, the activation rows the B operand: a lane ends up with four neighbouring columns of one row.  With fp32
 // activations step j of a 32-row weight tile multiplies rows 8 g + j of the four lane groups g.
-// KS = 4 (few rows): the four waves of a workgroup take a quarter of K each of the same column tiles, for as many workgroups
-// and as short chains of loads as the weight allows; their sums meet in LDS.
+// KS > 1 (few rows): KS waves of a workgroup take a part of K each of the same column tiles, for as many workgroups and as short
+// chains of loads as the weight allows (16 where there are few columns); their sums meet in LDS.
 template <bool F32, int MT, int KS>
-__global__ __launch_bounds__(256) void tile_gemm_kernel(TileGemm p) {
+__global__ __launch_bounds__(KS > 4 ? 64 * KS : 256) void tile_gemm_kernel(TileGemm p) {
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     const int g = lane >> 4, ml = lane & 15;
-    const int nt0 = (KS > 1 ? blockIdx.x : blockIdx.x * 4 + wave) * 2;
+    constexpr int TW = KS > 4 ? 1 : 2;
+    const int nt0 = (KS > 1 ? blockIdx.x : blockIdx.x * 4 + wave) * TW;
     if (nt0 >= p.NTILES) return; // (KS > 1: the whole workgroup or nobody)
     const int kper = (p.ktiles + KS - 1) / KS, k0 = KS > 1 ? wave * kper : 0;
     const int k1 = k0 + kper < p.ktiles ? k0 + kper : p.ktiles;
@@ -51,15 +52,15 @@ __global__ __launch_bounds__(256) void tile_gemm_kernel(TileGemm p) {
         p.C = (char *)p.C + (size_t)rec[2] * p.ldc * (p.c_dtype == XFTHIP_F32 ? 4 : 2);
         if (m0 >= p.M) return; // (the whole workgroup)
     }
-    const uint8_t *w[2];
-    int aofs[2];
+    const uint8_t *w[TW];
+    int aofs[2] = {0, 0};
 #pragma unroll
-    for (int t = 0; t < 2; ++t) {
+    for (int t = 0; t < TW; ++t) {
         const int nt = nt0 + t < p.NTILES ? nt0 + t : p.NTILES - 1;
         w[t] = p.packed + (size_t)nt * p.KT * 1024 + lane * 16;
         aofs[t] = p.tiles_per_block ? nt / p.tiles_per_block * p.a_block_stride : 0;
     }
-    const bool same = aofs[0] == aofs[1];
+    const bool same = TW == 1 || aofs[0] == aofs[1];
     size_t row[MT];
 #pragma unroll
     for (int m = 0; m < MT; ++m) {
@@ -67,17 +68,27 @@ __global__ __launch_bounds__(256) void tile_gemm_kernel(TileGemm p) {
         const int ra = a_first + (r < p.M ? r : p.M - 1);
         row[m] = (size_t)(p.a_rows ? p.a_rows[ra] : ra) * p.lda + 8 * g;
     }
-    f32x4 acc[2][MT];
+    // the 16-wave form: one result a thread, and what the side embedding says about it is fetched at once
+    float side_value = 1.0f;
+    if constexpr (KS > 4) {
+        const int r = m0 + (int)(threadIdx.x >> 8) * 16 + (int)((threadIdx.x >> 2) & 15), n = nt0 * 16 + 4 * (int)((threadIdx.x >> 6) & 3) + (int)(threadIdx.x & 3);
+        if (p.side && (int)threadIdx.x < MT * 256 && r < p.M && n < p.N) {
+            int id = p.side_ids[r];
+            id = id < 0 ? 0 : (id >= p.side_vocab ? p.side_vocab - 1 : id);
+            side_value = bf16_to_f32(p.side[(size_t)id * p.side_ld + n]);
+        }
+    }
+    f32x4 acc[TW][MT];
 #pragma unroll
-    for (int t = 0; t < 2; ++t)
+    for (int t = 0; t < TW; ++t)
 #pragma unroll
         for (int m = 0; m < MT; ++m) acc[t][m] = f32x4 {0.f, 0.f, 0.f, 0.f};
 
-    for (int kt = k0; kt < k1; ++kt) {
-        u32x4 wq[2];
+    if constexpr (F32) {
+        for (int kt = k0; kt < k1; ++kt) {
+            u32x4 wq[TW];
 #pragma unroll
-        for (int t = 0; t < 2; ++t) wq[t] = *(const u32x4 *)(w[t] + (size_t)kt * 1024);
-        if constexpr (F32) {
+            for (int t = 0; t < TW; ++t) wq[t] = *(const u32x4 *)(w[t] + (size_t)kt * 1024);
             const float *A = (const float *)p.A;
 #pragma unroll
             for (int m = 0; m < MT; ++m) {
@@ -89,7 +100,7 @@ __global__ __launch_bounds__(256) void tile_gemm_kernel(TileGemm p) {
                     a[1][0] = *(const f32x4 *)(A + row[m] + aofs[1] + kt * 32), a[1][1] = *(const f32x4 *)(A + row[m] + aofs[1] + kt * 32 + 4);
                 }
 #pragma unroll
-                for (int t = 0; t < 2; ++t)
+                for (int t = 0; t < TW; ++t)
 #pragma unroll
                     for (int j = 0; j < 8; ++j) {
                         const uint32_t pair = wq[t][j >> 1];
@@ -97,18 +108,56 @@ __global__ __launch_bounds__(256) void tile_gemm_kernel(TileGemm p) {
                         acc[t][m] = __builtin_amdgcn_mfma_f32_16x16x4f32(wv, a[t][j >> 2][j & 3], acc[t][m], 0, 0, 0);
                     }
             }
-        } else {
-            const uint16_t *A = (const uint16_t *)p.A;
+        }
+    } else {
+        // few rows: the loads of UN steps go out together, the chain of round trips is that much shorter
+        constexpr int UN = KS > 1 ? 4 : 1;
+        const uint16_t *A = (const uint16_t *)p.A;
+        for (int kb = k0; kb < k1; kb += UN) {
+            u32x4 wq[UN][TW], a0[UN][MT], a1[UN][MT];
 #pragma unroll
-            for (int m = 0; m < MT; ++m) {
-                u32x4 a0 = *(const u32x4 *)(A + row[m] + aofs[0] + kt * 32), a1 = a0;
-                if (!same) a1 = *(const u32x4 *)(A + row[m] + aofs[1] + kt * 32);
-                acc[0][m] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, wq[0]), __builtin_bit_cast(bf16x8, a0), acc[0][m], 0, 0, 0);
-                acc[1][m] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, wq[1]), __builtin_bit_cast(bf16x8, a1), acc[1][m], 0, 0, 0);
+            for (int u = 0; u < UN; ++u) {
+                const int kt = kb + u < k1 ? kb + u : k1 - 1; // (past the end: the last step's once more, unused)
+#pragma unroll
+                for (int t = 0; t < TW; ++t) wq[u][t] = *(const u32x4 *)(w[t] + (size_t)kt * 1024);
+#pragma unroll
+                for (int m = 0; m < MT; ++m) {
+                    a0[u][m] = *(const u32x4 *)(A + row[m] + aofs[0] + kt * 32);
+                    a1[u][m] = a0[u][m];
+                    if (TW > 1 && !same) a1[u][m] = *(const u32x4 *)(A + row[m] + aofs[1] + kt * 32);
+                }
+            }
+#pragma unroll
+            for (int u = 0; u < UN; ++u) {
+                if (UN > 1 && kb + u >= k1) break;
+#pragma unroll
+                for (int m = 0; m < MT; ++m) {
+                    acc[0][m] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, wq[u][0]), __builtin_bit_cast(bf16x8, a0[u][m]), acc[0][m], 0, 0, 0);
+                    if constexpr (TW > 1)
+                        acc[TW - 1][m] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, wq[u][TW - 1]), __builtin_bit_cast(bf16x8, a1[u][m]), acc[TW - 1][m], 0, 0, 0);
+                }
             }
         }
     }
 
+    if constexpr (KS > 4) {
+        __shared__ f32x4 sums[KS][MT][64];
+#pragma unroll
+        for (int m = 0; m < MT; ++m) sums[wave][m][lane] = acc[0][m];
+        __syncthreads();
+        if ((int)threadIdx.x >= MT * 256) return;
+        const float *part = (const float *)sums + threadIdx.x;
+        float y = 0.0f;
+#pragma unroll
+        for (int w = 0; w < KS; ++w) y += part[w * MT * 256];
+        const int r = m0 + (int)(threadIdx.x >> 8) * 16 + (int)((threadIdx.x >> 2) & 15), n = nt0 * 16 + 4 * (int)((threadIdx.x >> 6) & 3) + (int)(threadIdx.x & 3);
+        if (r >= p.M || n >= p.N) return;
+        const size_t at = (size_t)r * p.ldc + n;
+        if (p.side) y = gelu_tanh(y) * side_value;
+        if (p.add) y += ((const float *)p.C)[at];
+        store_from_f32(p.C, p.c_dtype, at, y);
+        return;
+    } else {
     if constexpr (KS > 1) {
         __shared__ f32x4 sums[KS - 1][2 * MT][64];
         if (wave > 0) {
@@ -170,6 +219,7 @@ __global__ __launch_bounds__(256) void tile_gemm_kernel(TileGemm p) {
             }
         }
     }
+    }
 }
 
 } // namespace
@@ -191,7 +241,11 @@ int tile_gemm(xfthip_weight_t w, int act_in, const TileGemmArgs &a, hipStream_t 
     const unsigned gx = (unsigned)((pw.NTILES + 7) / 8), gx1 = (unsigned)((pw.NTILES + 1) / 2);
     const bool f32 = act_in == XFTHIP_F32;
     auto launch = [&](auto kernel, unsigned x, unsigned y) { hipLaunchKernelGGL(kernel, dim3(x, y, gz), dim3(256), 0, st, p); };
-    if (M <= 16) {
+    auto launch16 = [&](auto kernel, unsigned x, unsigned y) { hipLaunchKernelGGL(kernel, dim3(x, y, gz), dim3(1024), 0, st, p); };
+    const bool deep = pw.NTILES <= 64 && pw.K >= 1024 && !a.block_cols && !a.glu && !a.group; // few columns against a deep K
+    if (!f32 && deep && M <= 32) {
+        launch16(tile_gemm_kernel<false, 1, 16>, (unsigned)pw.NTILES, (unsigned)((M + 15) / 16));
+    } else if (M <= 16) {
         if (f32) launch(tile_gemm_kernel<true, 1, 4>, gx1, 1);
         else launch(tile_gemm_kernel<false, 1, 4>, gx1, 1);
     } else if (M <= 32) {
