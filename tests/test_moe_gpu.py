@@ -117,11 +117,12 @@ def test_mixtral_mlp_four_bit_experts(xh, orc, kind, tokens):
     assert np.abs(got - exp).max() < 2e-2 and _cos(got, exp) >= 0.9999
 
 
-@pytest.mark.parametrize("tokens", [6, 40])
-def test_mixtral_mlp_bf16_experts(xh, orc, tokens):
-    """BF16 expert weights (no codes to widen), per-expert launches and the launch that serves all experts: against a
-    float64 restatement with the same bf16 hand-over points (normalised input, hidden activations)."""
-    hidden, inter, E = 512, 1024, 8
+@pytest.mark.parametrize("hidden,inter", [(512, 1024), (352, 736)], ids=str)
+@pytest.mark.parametrize("tokens", [3, 6, 28, 40])
+def test_mixtral_mlp_bf16_experts(xh, orc, tokens, hidden, inter):
+    """BF16 expert weights (no codes to widen) in the launches that serve all experts, also with depths that are no whole number
+    of load batches: against a float64 restatement with the same bf16 hand-over points (normalised input, hidden activations)."""
+    E = 8
     rng = np.random.default_rng(500 + tokens)
     Wgu = [orc.round_bf16(rng.standard_normal((hidden, 2 * inter)) * 0.05) for _ in range(E)]
     Wdn = [orc.round_bf16(rng.standard_normal((inter, hidden)) * 0.05) for _ in range(E)]

@@ -337,11 +337,11 @@ int xfthip_moe_forward(xfthip_moe_t m, const float *x_in, int in_stride, float *
         uniform = g.kind == g0.kind && g.flags == g0.flags && (g.zero != nullptr) == (g0.zero != nullptr) && d.kind == d0.kind
                 && d.flags == d0.flags && (d.zero != nullptr) == (d0.zero != nullptr);
     }
-    // (the few-row form of the grouped launch has no K-tail variant: a K that is not a whole number of weight
-    // tiles goes expert by expert)
+    // (the few-row form of the grouped launch has a K-tail variant for BF16 weights only: with the other kinds a K that is
+    // not a whole number of weight tiles goes expert by expert)
     if (T <= 32) {
         const PackedWeight &g0 = m->gateup[0]->pw, &d0 = m->down[0]->pw;
-        uniform = uniform && g0.KT * ktile_of(g0.kind) == g0.K && d0.KT * ktile_of(d0.kind) == d0.K;
+        for (const PackedWeight *w : {&g0, &d0}) uniform = uniform && (w->kind == XFTHIP_W_BF16 || w->KT * ktile_of(w->kind) == w->K);
     }
     if (uniform && m->gateup[0]->pw.kind != XFTHIP_W_W8A8 && m->down[0]->pw.kind != XFTHIP_W_W8A8) {
         if (int rc = gemm_grouped_rows_dev(m->gateup.data(), m->E, m->group, 2 * T, T, gemm_rows + 6, 9, m->xg, H, m->h, m->inter, XFTHIP_BF16, st))
