@@ -582,7 +582,7 @@ typedef struct {
     float glu_limit, glu_alpha;
     /* grouped attention */
     int qk_norm; /* RMS norm of every query and key head in front of the rotation */
-    int v_mix; /* values are mixed with those of the first layer that says so: (1 - lambda) v + lambda v_first */
+    int v_mix; /* values move a learned share of the way to those of the first layer that says so */
     /* context extension of the rotation (factor 0: none): frequencies whose pairs turn less than `slow` times within `original`
      * positions are divided by `factor`, those above `fast` stay, a ramp over the pairs between; cos and sin grow by
      * 0.1 ln(factor) + 1 */

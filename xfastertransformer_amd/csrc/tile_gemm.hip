@@ -158,67 +158,67 @@ __global__ __launch_bounds__(KS > 4 ? 64 * KS : 256) void tile_gemm_kernel(TileG
         store_from_f32(p.C, p.c_dtype, at, y);
         return;
     } else {
-    if constexpr (KS > 1) {
-        __shared__ f32x4 sums[KS - 1][2 * MT][64];
-        if (wave > 0) {
+        if constexpr (KS > 1) {
+            __shared__ f32x4 sums[KS - 1][2 * MT][64];
+            if (wave > 0) {
 #pragma unroll
-            for (int t = 0; t < 2; ++t)
+                for (int t = 0; t < 2; ++t)
 #pragma unroll
-                for (int m = 0; m < MT; ++m) sums[wave - 1][t * MT + m][lane] = acc[t][m];
-        }
-        __syncthreads();
-        if (wave > 0) return;
-#pragma unroll
-        for (int w = 0; w < KS - 1; ++w)
-#pragma unroll
-            for (int t = 0; t < 2; ++t)
-#pragma unroll
-                for (int m = 0; m < MT; ++m) acc[t][m] += sums[w][t * MT + m][lane];
-    }
-#pragma unroll
-    for (int m = 0; m < MT; ++m) {
-        const int r = m0 + m * 16 + ml;
-        if (r >= p.M) continue;
-        if (p.glu) { // tile pairs: 16 gate columns, the matching 16 up columns
-#pragma unroll
-            for (int i = 0; i < 4; ++i) {
-                const int n = (nt0 >> 1) * 16 + 4 * g + i;
-                if (n < p.N / 2)
-                    store_from_f32(p.C, p.c_dtype, (size_t)r * p.ldc + n, precise_glu(acc[0][m][i], acc[1][m][i], p.glu_limit, p.glu_alpha));
+                    for (int m = 0; m < MT; ++m) sums[wave - 1][t * MT + m][lane] = acc[t][m];
             }
-            continue;
-        }
-        const uint16_t *side = nullptr;
-        if (p.side) {
-            int id = p.side_ids[r];
-            id = id < 0 ? 0 : (id >= p.side_vocab ? p.side_vocab - 1 : id);
-            side = p.side + (size_t)id * p.side_ld;
+            __syncthreads();
+            if (wave > 0) return;
+#pragma unroll
+            for (int w = 0; w < KS - 1; ++w)
+#pragma unroll
+                for (int t = 0; t < 2; ++t)
+#pragma unroll
+                    for (int m = 0; m < MT; ++m) acc[t][m] += sums[w][t * MT + m][lane];
         }
 #pragma unroll
-        for (int t = 0; t < 2; ++t) {
-            const int n = (nt0 + t) * 16 + 4 * g;
-            if (side || p.add) {
+        for (int m = 0; m < MT; ++m) {
+            const int r = m0 + m * 16 + ml;
+            if (r >= p.M) continue;
+            if (p.glu) { // tile pairs: 16 gate columns, the matching 16 up columns
 #pragma unroll
                 for (int i = 0; i < 4; ++i) {
-                    if (n + i >= p.N) continue;
-                    if (side) acc[t][m][i] = gelu_tanh(acc[t][m][i]) * bf16_to_f32(side[n + i]);
-                    if (p.add) acc[t][m][i] += ((const float *)p.C)[(size_t)r * p.ldc + n + i];
+                    const int n = (nt0 >> 1) * 16 + 4 * g + i;
+                    if (n < p.N / 2)
+                        store_from_f32(p.C, p.c_dtype, (size_t)r * p.ldc + n, precise_glu(acc[0][m][i], acc[1][m][i], p.glu_limit, p.glu_alpha));
+                }
+                continue;
+            }
+            const uint16_t *side = nullptr;
+            if (p.side) {
+                int id = p.side_ids[r];
+                id = id < 0 ? 0 : (id >= p.side_vocab ? p.side_vocab - 1 : id);
+                side = p.side + (size_t)id * p.side_ld;
+            }
+#pragma unroll
+            for (int t = 0; t < 2; ++t) {
+                const int n = (nt0 + t) * 16 + 4 * g;
+                if (side || p.add) {
+#pragma unroll
+                    for (int i = 0; i < 4; ++i) {
+                        if (n + i >= p.N) continue;
+                        if (side) acc[t][m][i] = gelu_tanh(acc[t][m][i]) * bf16_to_f32(side[n + i]);
+                        if (p.add) acc[t][m][i] += ((const float *)p.C)[(size_t)r * p.ldc + n + i];
+                    }
+                }
+                const size_t at = (size_t)r * p.ldc + n;
+                if (n + 4 <= p.N && (p.ldc & 3) == 0) {
+                    if (p.c_dtype == XFTHIP_F32)
+                        *(f32x4 *)((float *)p.C + at) = acc[t][m];
+                    else
+                        *(uint2 *)((uint16_t *)p.C + at) = make_uint2(f32_to_bf16_ref(acc[t][m][0]) | ((uint32_t)f32_to_bf16_ref(acc[t][m][1]) << 16),
+                                f32_to_bf16_ref(acc[t][m][2]) | ((uint32_t)f32_to_bf16_ref(acc[t][m][3]) << 16));
+                } else {
+#pragma unroll
+                    for (int i = 0; i < 4; ++i)
+                        if (n + i < p.N) store_from_f32(p.C, p.c_dtype, at + i, acc[t][m][i]);
                 }
             }
-            const size_t at = (size_t)r * p.ldc + n;
-            if (n + 4 <= p.N && (p.ldc & 3) == 0) {
-                if (p.c_dtype == XFTHIP_F32)
-                    *(f32x4 *)((float *)p.C + at) = acc[t][m];
-                else
-                    *(uint2 *)((uint16_t *)p.C + at) = make_uint2(f32_to_bf16_ref(acc[t][m][0]) | ((uint32_t)f32_to_bf16_ref(acc[t][m][1]) << 16),
-                            f32_to_bf16_ref(acc[t][m][2]) | ((uint32_t)f32_to_bf16_ref(acc[t][m][3]) << 16));
-            } else {
-#pragma unroll
-                for (int i = 0; i < 4; ++i)
-                    if (n + i < p.N) store_from_f32(p.C, p.c_dtype, at + i, acc[t][m][i]);
-            }
         }
-    }
     }
 }
 
