@@ -547,22 +547,30 @@ int xfthip_model_set_moe(xfthip_model_t m, int idx, xfthip_moe_t moe);
 /* ---- layer plans: decoder stacks of several kinds of layers --------------------------- */
 /*
  * A plan describes a stack whose layers differ: what mixes the tokens (latent attention, a gated delta-rule recurrence, grouped
- * attention), its sizes, its constants, and the feed-forward behind it, if any (dense, or routed experts beside an optional shared
- * one).  Keys live in pages of a pool shared by all sequences, recurrent state in one slot a sequence.  The reference has no
+ * attention, a gated linear recurrence, or two of the last three side by side), its sizes, its constants, and the feed-forward
+ * behind it, if any (dense, or routed experts beside an optional shared one).  Keys live in pages of a pool shared by all sequences, recurrent state in one slot a sequence.  The reference has no
  * counterpart; a model built from a plan is a xfthip_model_t and runs behind the same calls as the others.
  *
- * Two arrangements of a layer's sublayers:
+ * Three arrangements of a layer's sublayers:
  *   XFTHIP_BLOCK_SANDWICH  one after the other, a norm in front and a norm behind each, the latter multiplied by a learned scale
  *                          per channel
  *   XFTHIP_BLOCK_PARALLEL  both read the same residual through a norm of their own, their sum is added to it
- * and two kinds of norm: RMS norms whose stored weights are distances from one, or tanh(alpha x) * w + b (parallel blocks only).
+ *   XFTHIP_BLOCK_SERIAL    one after the other, a norm in front of each, their results times residual_mult
+ * and three kinds of norm: RMS norms whose stored weights are distances from one (sandwich), tanh(alpha x) * w + b (parallel), RMS
+ * norms with plain weights (serial).
  * Layers [loop_start, loop_stop) run loop_times times, every run with its own cache or state, the embedding output joining the
  * residual in front of every pass but the first.  side_dim > 0: behind its sublayers every layer adds
  * rms(P (gelu(G x) * e)) * w, e the layer's part of a second embedding of the token.
+ *
+ * The embedding is table[token] * embed_scale; bigram_buckets > 0: plus a row of a second table, that of (previous token * bigram_mul_prev
+ * + token * bigram_mul_cur) mod bigram_buckets, or the row behind the buckets for the first token of a sequence.
  */
-enum { XFTHIP_MIXER_LATENT = 1, XFTHIP_MIXER_DELTA = 2, XFTHIP_MIXER_GROUPED = 3 };
-enum { XFTHIP_BLOCK_SANDWICH = 0, XFTHIP_BLOCK_PARALLEL = 1 };
-enum { XFTHIP_NORM_RMS_ABOUT_ONE = 0, XFTHIP_NORM_DYNAMIC_TANH = 1 };
+enum { XFTHIP_MIXER_LATENT = 1, XFTHIP_MIXER_DELTA = 2, XFTHIP_MIXER_GROUPED = 3, XFTHIP_MIXER_UNIT = 4 };
+enum { XFTHIP_BLOCK_SANDWICH = 0, XFTHIP_BLOCK_PARALLEL = 1, XFTHIP_BLOCK_SERIAL = 2 };
+enum { XFTHIP_NORM_RMS_ABOUT_ONE = 0, XFTHIP_NORM_DYNAMIC_TANH = 1, XFTHIP_NORM_RMS = 2 };
+enum { XFTHIP_QK_NORM_HEAD = 1, XFTHIP_QK_NORM_ALL = 2 };
+enum { XFTHIP_GATE_ELEMENT = 1, XFTHIP_GATE_HEAD = 2 };
+enum { XFTHIP_ROUTE_SOFTMAX = 0, XFTHIP_ROUTE_SIGMOID_GROUPS = 1 };
 typedef struct {
     int mixer;
     int heads, kv_heads; /* kv_heads: query / key heads of the delta rule, key / value heads of grouped attention */
@@ -576,12 +584,14 @@ typedef struct {
     double rot_base;
     /* delta rule */
     int taps; /* of the short convolutions */
-    int decay_rank, gate_rank; /* inner widths of the two gates' projections */
-    /* feed-forward (inter 0: none; with experts: the shared one): xfthip_gemm_gateup_clamped */
+    /* inner widths of the two gates' projections: decays a key channel, a sigmoid on the output; 0: one projection, one decay a head /
+     * a silu on the output */
+    int decay_rank, gate_rank;
+    /* feed-forward (inter 0: none; with experts: the shared one): xfthip_gemm_gateup_clamped; glu_alpha 0: silu(gate) * up, no limits */
     int inter;
     float glu_limit, glu_alpha;
     /* grouped attention */
-    int qk_norm; /* RMS norm of every query and key head in front of the rotation */
+    int qk_norm; /* XFTHIP_QK_NORM_*: RMS norm in front of the rotation, of every query and key head or of all heads at once; 0 = none */
     int v_mix; /* values move a learned share of the way to those of the first layer that says so */
     /* context extension of the rotation (factor 0: none): frequencies whose pairs turn less than `slow` times within `original`
      * positions are divided by `factor`, those above `fast` stay, a ramp over the pairs between; cos and sin grow by
@@ -591,6 +601,24 @@ typedef struct {
      * by their scores; the last `identity` outputs hand the feed-forward's input through */
     int experts, identity, top, expert_inter;
     float expert_limit; /* of the experts' gates; the sigmoid's factor is glu_alpha */
+    /*
+     * beside = 1: not a layer of its own, but a second mixer of the layer before it (mixer fields only): both read the same input, their
+     * results are added.  scaled = 1: the mixer's result is multiplied by mix_scale.
+     */
+    int beside, scaled;
+    float mix_scale;
+    /* grouped attention */
+    int chunk; /* > 0: a position sees those before it in its own chunk of so many tokens (in place of a window) */
+    float softcap; /* > 0: scores pass softcap * tanh(score / softcap) */
+    int distance_bias; /* 1: 2^(-8 (h + 1) / heads) a token of distance is taken off the scores of head h */
+    int qkv_bias; /* q, k, v have biases */
+    int key_values; /* 1: the projected keys, before norm and rotation, are the values; there is no value projection */
+    int out_gate; /* XFTHIP_GATE_*: sigmoid of a projection of the input on every output element or head; 0 = none */
+    int kv_from; /* n > 0: keys and values of record n - 1 (its cache), no projections of its own; n = 0: own ones */
+    /* experts: XFTHIP_ROUTE_*; sigmoid scores: experts form route_groups groups of neighbours, the route_keep with the largest sums of
+     * their two best scores are open; the chosen scores are divided by their sum and multiplied by route_scale; no correction */
+    int router, route_groups, route_keep;
+    float route_scale;
 } xfthip_plan_layer;
 typedef struct {
     int layers;
@@ -600,17 +628,23 @@ typedef struct {
     int block, norm; /* XFTHIP_BLOCK_*, XFTHIP_NORM_* */
     int tied_head; /* the head is the embedding table */
     int side_dim; /* width of a layer's part of the side embedding; 0 = none */
+    float residual_mult; /* serial blocks */
+    float embed_scale; /* 0 = 1 */
+    float logit_softcap; /* > 0: logits pass cap * tanh(logit / cap) */
+    long long bigram_buckets, bigram_mul_prev, bigram_mul_cur;
 } xfthip_plan_config;
 typedef struct xfthip_plan *xfthip_plan_t;
 int xfthip_plan_create(const xfthip_plan_config *cfg, const xfthip_plan_layer *layers, xfthip_plan_t *out);
 int xfthip_plan_destroy(xfthip_plan_t p);
 /*
  * Tensors by name, host memory, bf16 bit patterns, row-major [rows, cols] (linear weights [out, in]; vectors cols = 1): layer -1:
- * embed, head (unless tied), final.norm, side.embed; a layer: norm1, norm2 (a tanh norm: also .alpha and .b), sandwich blocks also
+ * embed, head (unless tied), final.norm, side.embed; a layer (number of its record): norm1, norm2 (a tanh norm: also .alpha and .b), sandwich blocks also
  * norm1b, ls1, norm2b, ls2; side.gate / proj / norm; mlp.gate / up / down, with experts mlp.router, mlp.correction,
  * mlp.e<i>.gate / up / down and mlp.shared.gate / up / down; and in front of its mixer's names "mix.": latent attention dq,
  * dq.norm, uq, dkv, dkv.norm, uk, uv, o, sink; delta rule q, k, v (each with .conv), b, A_log, a1, a2, dt_bias, g1, g2, norm, o;
- * grouped attention q, k (each with .norm), v, o, sink, vmix.  xfthip_plan_finish checks that all are there, packs and uploads them.
+ * grouped attention q, k (each with .norm, .b), v (.b), o, sink, vmix, g; delta rule without ranks a [heads] in place of a1, a2 and g in
+ * place of g1, g2; gated unit (heads = blocks, dim = channels of a block, taps) y, x (each with .b), conv (.b), ra, ri [blocks, dim * dim]
+ * (each with .b), lam, o.  bigram (layer -1).  xfthip_plan_finish checks that all are there, packs and uploads them.
  */
 int xfthip_plan_set_tensor(xfthip_plan_t p, int layer, const char *name, const uint16_t *data_host, int rows, int cols);
 int xfthip_plan_finish(xfthip_plan_t p);

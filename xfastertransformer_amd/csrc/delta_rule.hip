@@ -52,7 +52,7 @@ struct PrepParams {
     StepView v;
     DeltaBuffers b;
     const float *conv, *decay, *dt_bias;
-    int H, KH, KD, VD, taps, ld, channels, beta_col, gcols;
+    int H, KH, KD, VD, taps, ld, channels, beta_col, decay_col, gcols; // decay_col: one decay a head, in the row (or -1)
     float qscale;
 };
 
@@ -113,7 +113,11 @@ __global__ __launch_bounds__(256) void delta_prepare_kernel(PrepParams p) {
     }
     for (int c = lane; c < p.VD; c += 64) p.b.v[((size_t)t * p.H + head) * p.VD + c] = conv(2 * p.KH * p.KD + head * p.VD + c);
     const float a = p.decay[head];
-    for (int c = lane; c < p.KD; c += 64) {
+    if (p.decay_col >= 0) {
+        const float x = load_as_f32(p.b.in, DT, (size_t)t * p.ld + p.decay_col + head) + p.dt_bias[head];
+        if (lane == 0) p.b.g[(size_t)t * p.H + head] = expf(-a * (x > 20.0f ? x : log1pf(expf(x))));
+    }
+    for (int c = lane; c < p.KD && p.decay_col < 0; c += 64) {
         const float x = p.b.gates[(size_t)t * 2 * p.gcols + head * p.KD + c] + p.dt_bias[head * p.KD + c];
         const float sp = x > 20.0f ? x : log1pf(expf(x));
         p.b.g[((size_t)t * p.H + head) * p.KD + c] = expf(-a * sp);
@@ -183,11 +187,11 @@ __global__ __launch_bounds__(256) void delta_prepare_tiled_kernel(PrepParams p) 
         const int c = j * 128 + lane * 2;
         if (qk_head && c < p.KD) open(q[j], head * p.KD + c), open(k[j], (p.KH + head) * p.KD + c);
         if (c < p.VD) open(v[j], vbase + c);
-        dtb[j] = c < p.KD ? *(const float2 *)(p.dt_bias + head * p.KD + c) : make_float2(0.0f, 0.0f);
+        dtb[j] = c < p.KD && p.decay_col < 0 ? *(const float2 *)(p.dt_bias + head * p.KD + c) : make_float2(0.0f, 0.0f);
     }
-    const float decay = p.decay[head];
+    const float decay = p.decay[head], head_dt = p.decay_col >= 0 ? p.dt_bias[head] : 0.0f;
     float2 nq[J], nk[J], nv[J], ng[J]; // the next token's values, requested a token ahead
-    float nb = 0.0f;
+    float nb = 0.0f, nd = 0.0f;
     auto request = [&](int i) {
         const int t = off + i;
         const size_t in_row = (size_t)t * p.ld;
@@ -197,9 +201,10 @@ __global__ __launch_bounds__(256) void delta_prepare_tiled_kernel(PrepParams p) 
             nq[j] = nk[j] = nv[j] = ng[j] = make_float2(0.0f, 0.0f);
             if (qk_head && c < p.KD) nq[j] = load2<BF16>(p.b.in, in_row + head * p.KD + c), nk[j] = load2<BF16>(p.b.in, in_row + (p.KH + head) * p.KD + c);
             if (c < p.VD) nv[j] = load2<BF16>(p.b.in, in_row + vbase + c);
-            if (c < p.KD) ng[j] = *(const float2 *)(p.b.gates + (size_t)t * 2 * p.gcols + head * p.KD + c);
+            if (c < p.KD && p.decay_col < 0) ng[j] = *(const float2 *)(p.b.gates + (size_t)t * 2 * p.gcols + head * p.KD + c);
         }
         nb = ldb<BF16>(p.b.in, in_row + p.beta_col + head);
+        if (p.decay_col >= 0) nd = ldb<BF16>(p.b.in, in_row + p.decay_col + head);
     };
     request(i0);
     for (int i = i0; i < i0 + cnt; ++i) {
@@ -207,7 +212,7 @@ __global__ __launch_bounds__(256) void delta_prepare_tiled_kernel(PrepParams p) 
         float2 xq[J], xk[J], xv[J], xg[J];
 #pragma unroll
         for (int j = 0; j < J; ++j) xq[j] = nq[j], xk[j] = nk[j], xv[j] = nv[j], xg[j] = ng[j];
-        const float bl = nb;
+        const float bl = nb, dl = nd;
         if (i + 1 < i0 + cnt) request(i + 1);
         float sq = 0.0f, sk = 0.0f, dot = 0.0f;
 #pragma unroll
@@ -220,7 +225,7 @@ __global__ __launch_bounds__(256) void delta_prepare_tiled_kernel(PrepParams p) 
                 dot = fmaf(xq[j].x, xk[j].x, fmaf(xq[j].y, xk[j].y, dot));
             }
             if (c < p.VD) *(float2 *)(p.b.v + ((size_t)t * p.H + head) * p.VD + c) = advance(v[j], xv[j]);
-            if (c < p.KD) {
+            if (c < p.KD && p.decay_col < 0) {
                 *(float2 *)(p.b.g + ((size_t)t * p.H + head) * p.KD + c) = make_float2(exp_of<BF16>(-decay * softplus_of<BF16>(xg[j].x + dtb[j].x)),
                         exp_of<BF16>(-decay * softplus_of<BF16>(xg[j].y + dtb[j].y)));
             }
@@ -239,7 +244,10 @@ __global__ __launch_bounds__(256) void delta_prepare_tiled_kernel(PrepParams p) 
             }
             if (lane == 0) p.b.qk[(size_t)t * p.KH + head] = dot;
         }
-        if (lane == 0) p.b.beta[(size_t)t * p.H + head] = sigmoid_of<BF16>(bl);
+        if (lane == 0) {
+            p.b.beta[(size_t)t * p.H + head] = sigmoid_of<BF16>(bl);
+            if (p.decay_col >= 0) p.b.g[(size_t)t * p.H + head] = exp_of<BF16>(-decay * softplus_of<BF16>(dl + head_dt));
+        }
     }
     if (n == 1 && TAPS > 1) { // a single new token: nobody else reads these channels of the slot
         auto keep = [&](const Window &win, int c) {
@@ -255,9 +263,15 @@ __global__ __launch_bounds__(256) void delta_prepare_tiled_kernel(PrepParams p) 
     }
 }
 
+struct TailParams {
+    StepView v;
+    const void *in;
+    int ld, channels, taps;
+    void *conv_state;
+};
 // the last taps - 1 inputs of a segment of several tokens; one thread a channel
 template <bool BF16>
-__global__ __launch_bounds__(256) void conv_tail_kernel(PrepParams p) {
+__global__ __launch_bounds__(256) void conv_tail_kernel(TailParams p) {
     constexpr int DT = BF16 ? XFTHIP_BF16 : XFTHIP_F32;
     const int seg = blockIdx.y, n = p.v.seg_len[seg], ch = blockIdx.x * 256 + threadIdx.x;
     if (n <= 1 || ch >= p.channels) return;
@@ -265,9 +279,9 @@ __global__ __launch_bounds__(256) void conv_tail_kernel(PrepParams p) {
     const int off = p.v.seg_off[seg];
     for (int s = 0; s < p.taps - 1; ++s) { // ascending: slot s is read (as a later source) only by slots below it
         const int from = n - (p.taps - 1) + s;
-        const float x = from >= 0 ? load_as_f32(p.b.in, DT, (size_t)(off + from) * p.ld + ch)
-                                  : load_as_f32(p.b.conv_state, DT, hist + (size_t)(s + n) * p.channels + ch);
-        store_from_f32(p.b.conv_state, DT, hist + (size_t)s * p.channels + ch, x);
+        const float x = from >= 0 ? load_as_f32(p.in, DT, (size_t)(off + from) * p.ld + ch)
+                                  : load_as_f32(p.conv_state, DT, hist + (size_t)(s + n) * p.channels + ch);
+        store_from_f32(p.conv_state, DT, hist + (size_t)s * p.channels + ch, x);
     }
 }
 
@@ -296,17 +310,19 @@ struct ScanParams {
 // With S' = g S the step is a = S'^T k, b = S'^T q, u = beta (v - a), S = S' + k u^T, o = b + (q . k) u: both sums over the key
 // rows run side by side and the read-out needs none of its own.  q, k, g of CT tokens are staged in LDS, the next CT on
 // their way through registers.  grid (segments, heads, column groups of COLS).
+// ONE: one decay a head, a scalar beside beta.
 // One prompt of 32 heads is one wave a SIMD: the time is about 75 vector instructions a token and the latency of the
 // reductions in them.  (KD = 128 as 32 lanes x 4 rows x 2 columns, half the LDS reads: 510 us for 2048 tokens against 440 as
 // 16 x 8 x 1.)
-template <int L, int RV, int C>
+template <int L, int RV, int C, bool ONE>
 __global__ __launch_bounds__(256) void delta_scan_kernel(ScanParams p) {
     constexpr int KD = 4 * L * RV, GROUPS = 256 / L, COLS = GROUPS * C, CT = KD > 128 ? 8 : 16;
     constexpr int CHUNK4 = CT * KD / 4; // float4 of one array and chunk
-    constexpr int PER = (3 * CHUNK4 + 255) / 256, PERV = (CT * COLS + 255) / 256;
-    __shared__ float lds[2][3 * CT * KD];
+    constexpr int ARRAYS = ONE ? 2 : 3, SCALARS = ONE ? 3 : 2; // q, k(, g); beta, q . k(, g)
+    constexpr int PER = (ARRAYS * CHUNK4 + 255) / 256, PERV = (CT * COLS + 255) / 256;
+    __shared__ float lds[2][ARRAYS * CT * KD];
     __shared__ float vlds[2][CT * COLS];
-    __shared__ float sc[2][2 * CT];
+    __shared__ float sc[2][SCALARS * CT];
     __shared__ float olds[2][CT * COLS];
     const int seg = blockIdx.x, head = blockIdx.y, kvh = head / (p.H / p.KH);
     const int n = p.v.seg_len[seg], off = p.v.seg_off[seg];
@@ -328,7 +344,7 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(ScanParams p) {
             const int e = i * 256 + threadIdx.x;
             const int arr = e / CHUNK4, r = e % CHUNK4, tok = r / (KD / 4), d = (r % (KD / 4)) * 4;
             const int t = off + (c0 + tok < n ? c0 + tok : n - 1);
-            if (e < 3 * CHUNK4) {
+            if (e < ARRAYS * CHUNK4) {
                 const float *src = arr == 2 ? p.b.g + ((size_t)t * p.H + head) * KD : (arr ? p.b.k : p.b.q) + ((size_t)t * p.KH + kvh) * KD;
                 stage[i] = *(const f32x4 *)(src + d);
             }
@@ -339,23 +355,23 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(ScanParams p) {
             const int t = off + (c0 + tok < n ? c0 + tok : n - 1);
             if (e < CT * COLS) vstage[i] = p.b.v[((size_t)t * p.H + head) * p.VD + (c < p.VD ? c : p.VD - 1)];
         }
-        if (threadIdx.x < 2 * CT) {
+        if (threadIdx.x < SCALARS * CT) {
             const int tok = threadIdx.x % CT, t = off + (c0 + tok < n ? c0 + tok : n - 1);
-            cstage = threadIdx.x < CT ? p.b.beta[(size_t)t * p.H + head] : p.b.qk[(size_t)t * p.KH + kvh];
+            cstage = threadIdx.x < CT ? p.b.beta[(size_t)t * p.H + head] : threadIdx.x < 2 * CT ? p.b.qk[(size_t)t * p.KH + kvh] : p.b.g[(size_t)t * p.H + head];
         }
     };
     auto stash = [&](int buf) {
 #pragma unroll
         for (int i = 0; i < PER; ++i) {
             const int e = i * 256 + threadIdx.x;
-            if (e < 3 * CHUNK4) *(f32x4 *)(&lds[buf][4 * e]) = stage[i];
+            if (e < ARRAYS * CHUNK4) *(f32x4 *)(&lds[buf][4 * e]) = stage[i];
         }
 #pragma unroll
         for (int i = 0; i < PERV; ++i) {
             const int e = i * 256 + threadIdx.x;
             if (e < CT * COLS) vlds[buf][e] = vstage[i];
         }
-        if (threadIdx.x < 2 * CT) sc[buf][threadIdx.x] = cstage;
+        if (threadIdx.x < SCALARS * CT) sc[buf][threadIdx.x] = cstage;
     };
     fetch(0);
     stash(0);
@@ -366,17 +382,21 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(ScanParams p) {
         if (c0 + CT < n) fetch(c0 + CT);
         const float *lq = lds[buf] + 4 * li;
         struct Operands {
-            f32x4 q[RV], k[RV], g[RV];
-            float v[C], beta, qk;
+            f32x4 q[RV], k[RV], g[ONE ? 1 : RV];
+            float v[C], beta, qk, fade;
         };
         auto read = [&](int i) {
             const float *q = lq + i * KD, *k = q + CT * KD, *g = k + CT * KD;
             Operands x;
 #pragma unroll
-            for (int r = 0; r < RV; ++r) x.q[r] = *(const f32x4 *)(q + r * 4 * L), x.k[r] = *(const f32x4 *)(k + r * 4 * L), x.g[r] = *(const f32x4 *)(g + r * 4 * L);
+            for (int r = 0; r < RV; ++r) {
+                x.q[r] = *(const f32x4 *)(q + r * 4 * L), x.k[r] = *(const f32x4 *)(k + r * 4 * L);
+                if constexpr (!ONE) x.g[r] = *(const f32x4 *)(g + r * 4 * L);
+            }
 #pragma unroll
             for (int c = 0; c < C; ++c) x.v[c] = vlds[buf][i * COLS + lc + c];
             x.beta = sc[buf][i], x.qk = sc[buf][CT + i];
+            if constexpr (ONE) x.fade = sc[buf][2 * CT + i];
             return x;
         };
         // the operands of the next token are on their way from LDS while this one's sums go round
@@ -389,7 +409,8 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(ScanParams p) {
                 for (int r = 0; r < RV; ++r)
 #pragma unroll
                     for (int e = 0; e < 4; ++e) {
-                        s[c][r][e] *= x.g[r][e];
+                        if constexpr (ONE) s[c][r][e] *= x.fade;
+                        else s[c][r][e] *= x.g[r][e];
                         a[c] = fmaf(x.k[r][e], s[c][r][e], a[c]), b[c] = fmaf(x.q[r][e], s[c][r][e], b[c]);
                     }
             }
@@ -432,7 +453,7 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(ScanParams p) {
 }
 
 // The same step for segments of one token: nothing to stage, the kernel is a read and a write of the state.
-template <int L>
+template <int L, bool ONE>
 __global__ __launch_bounds__(256) void delta_step_kernel(ScanParams p) {
     constexpr int KD = 8 * L, COLS = 256 / L;
     const int seg = blockIdx.x, head = blockIdx.y, kvh = head / (p.H / p.KH), t = p.v.seg_off[seg];
@@ -441,9 +462,15 @@ __global__ __launch_bounds__(256) void delta_step_kernel(ScanParams p) {
     float *state = p.b.state + (((size_t)p.v.seg_row[seg] * p.H + head) * p.VD + col) * KD;
     f32x4 s0 = *(const f32x4 *)(state + 4 * li), s1 = *(const f32x4 *)(state + 4 * (L + li));
     const float *q = p.b.q + ((size_t)t * p.KH + kvh) * KD + 4 * li, *k = p.b.k + ((size_t)t * p.KH + kvh) * KD + 4 * li;
-    const float *g = p.b.g + ((size_t)t * p.H + head) * KD + 4 * li;
+    f32x4 g0, g1;
+    if constexpr (ONE) {
+        const float fade = p.b.g[(size_t)t * p.H + head];
+        g0 = g1 = f32x4 {fade, fade, fade, fade};
+    } else {
+        const float *g = p.b.g + ((size_t)t * p.H + head) * KD + 4 * li;
+        g0 = *(const f32x4 *)g, g1 = *(const f32x4 *)(g + 4 * L);
+    }
     const f32x4 q0 = *(const f32x4 *)q, q1 = *(const f32x4 *)(q + 4 * L), k0 = *(const f32x4 *)k, k1 = *(const f32x4 *)(k + 4 * L);
-    const f32x4 g0 = *(const f32x4 *)g, g1 = *(const f32x4 *)(g + 4 * L);
     const float v = p.b.v[((size_t)t * p.H + head) * p.VD + col], beta = p.b.beta[(size_t)t * p.H + head], qk = p.b.qk[(size_t)t * p.KH + kvh];
     if (p.v.seg_pos[seg] == 0) s0 = s1 = f32x4 {0.f, 0.f, 0.f, 0.f};
     float a = 0.0f, b = 0.0f;
@@ -464,12 +491,15 @@ __global__ __launch_bounds__(256) void delta_step_kernel(ScanParams p) {
 
 struct OutParams {
     const float *o, *gates, *norm;
-    void *on;
+    const void *row_gate; // the gate in the rows of the input product (pitch ld), through a silu; or null
+    int ld;
+    void *out; // rows of pitch out_ld
+    int out_ld;
     int H, VD, vdim, gcols, T;
-    float eps;
+    float eps, mul;
 };
 
-// per-head RMS norm times the sigmoid gate; one wave a (token, head)
+// per-head RMS norm times the gate; one wave a (token, head)
 template <bool BF16>
 __global__ __launch_bounds__(256) void delta_output_kernel(OutParams p) {
     const int lane = threadIdx.x & 63;
@@ -484,18 +514,28 @@ __global__ __launch_bounds__(256) void delta_output_kernel(OutParams p) {
         sq = fmaf(x.x, x.x, fmaf(x.y, x.y, sq));
     }
     const float r = 1.0f / sqrtf(wave_total(sq) / (float)p.vdim + p.eps);
+    const float f = r * p.mul;
     for (int c = lane * 2; c < p.VD; c += 128) {
-        const float2 x = *(const float2 *)(o + c), w = *(const float2 *)(p.norm + c), z = *(const float2 *)(gate + c);
-        store2<BF16>(p.on, idx * p.VD + c, make_float2(x.x * r * w.x * sigmoid_of<BF16>(z.x), x.y * r * w.y * sigmoid_of<BF16>(z.y)));
+        const float2 x = *(const float2 *)(o + c), w = *(const float2 *)(p.norm + c);
+        float2 z;
+        if (p.row_gate) {
+            z = load2<BF16>(p.row_gate, (size_t)t * p.ld + head * p.VD + c);
+            z.x = silu_of<BF16>(z.x), z.y = silu_of<BF16>(z.y);
+        } else {
+            z = *(const float2 *)(gate + c);
+            z.x = sigmoid_of<BF16>(z.x), z.y = sigmoid_of<BF16>(z.y);
+        }
+        store2<BF16>(p.out, (size_t)t * p.out_ld + head * p.VD + c, make_float2(x.x * f * w.x * z.x, x.y * f * w.y * z.y));
     }
 }
 
-PrepParams prep_params(const PlanLayer &L, const StepView &v, const DeltaBuffers &b) {
+PrepParams prep_params(int act, const PlanLayer &L, const StepView &v, const DeltaBuffers &b) {
     PrepParams p;
     p.v = v, p.b = b;
+    p.b.in = (char *)b.in + (size_t)L.in_col * (act == XFTHIP_BF16 ? 2 : 4);
     p.conv = L.conv, p.decay = L.decay, p.dt_bias = L.dt_bias;
     p.H = L.s.heads, p.KH = L.s.kv_heads, p.KD = L.KD, p.VD = L.VD, p.taps = L.s.taps;
-    p.ld = L.row_in(), p.channels = L.channels(), p.beta_col = L.channels(), p.gcols = L.gcols;
+    p.ld = L.in_ld, p.channels = L.channels(), p.beta_col = L.channels(), p.decay_col = L.head_decay() ? p.beta_col + L.beta_cols() : -1, p.gcols = L.gcols;
     p.qscale = 1.0f / sqrtf((float)L.s.dim);
     return p;
 }
@@ -503,9 +543,8 @@ PrepParams prep_params(const PlanLayer &L, const StepView &v, const DeltaBuffers
 } // namespace
 
 int delta_prepare(int act, const PlanLayer &L, const StepView &v, const DeltaBuffers &b, hipStream_t st) {
-    const PrepParams p = prep_params(L, v, b);
-    const dim3 grid(v.T, (p.H + 3) / 4), tail((p.channels + 255) / 256, v.B);
-    const bool long_segments = v.longest > 1 && p.taps > 1;
+    const PrepParams p = prep_params(act, L, v, b);
+    const dim3 grid(v.T, (p.H + 3) / 4);
     const int width = p.KD > p.VD ? p.KD : p.VD;
     const bool tiled = p.taps >= 2 && p.taps <= 4 && width <= 256;
     if (tiled) {
@@ -526,13 +565,20 @@ int delta_prepare(int act, const PlanLayer &L, const StepView &v, const DeltaBuf
             default: hipLaunchKernelGGL((delta_prepare_tiled_kernel<false, 4, 2>), tiles, dim3(256), 0, st, p); break;
         }
     }
-    if (act == XFTHIP_BF16) {
-        if (!tiled) hipLaunchKernelGGL(delta_prepare_kernel<true>, grid, dim3(256), 0, st, p);
-        if (long_segments) hipLaunchKernelGGL(conv_tail_kernel<true>, tail, dim3(256), 0, st, p);
-    } else {
-        if (!tiled) hipLaunchKernelGGL(delta_prepare_kernel<false>, grid, dim3(256), 0, st, p);
-        if (long_segments) hipLaunchKernelGGL(conv_tail_kernel<false>, tail, dim3(256), 0, st, p);
+    if (!tiled) {
+        if (act == XFTHIP_BF16) hipLaunchKernelGGL(delta_prepare_kernel<true>, grid, dim3(256), 0, st, p);
+        else hipLaunchKernelGGL(delta_prepare_kernel<false>, grid, dim3(256), 0, st, p);
     }
+    XFT_CHECK_HIP(hipGetLastError());
+    return conv_tail(act, v, p.b.in, p.ld, p.channels, p.taps, b.conv_state, st);
+}
+
+int conv_tail(int act, const StepView &v, const void *in, int ld, int channels, int taps, void *conv_state, hipStream_t st) {
+    if (v.longest <= 1 || taps <= 1) return 0;
+    const TailParams p = {v, in, ld, channels, taps, conv_state};
+    const dim3 grid((channels + 255) / 256, v.B);
+    if (act == XFTHIP_BF16) hipLaunchKernelGGL(conv_tail_kernel<true>, grid, dim3(256), 0, st, p);
+    else hipLaunchKernelGGL(conv_tail_kernel<false>, grid, dim3(256), 0, st, p);
     XFT_CHECK_HIP(hipGetLastError());
     return 0;
 }
@@ -541,23 +587,22 @@ int delta_scan(const PlanLayer &L, const StepView &v, const DeltaBuffers &b, hip
     ScanParams p;
     p.v = v, p.b = b, p.H = L.s.heads, p.KH = L.s.kv_heads, p.VD = L.VD;
     const int lanes = L.KD / 8, cols = 256 / lanes;
+    const bool one = L.head_decay();
     const dim3 grid(v.B, p.H, (L.VD + cols - 1) / cols);
-    if (v.longest == 1 && (lanes == 4 || lanes == 8 || lanes == 16 || lanes == 32)) {
-        switch (lanes) {
-            case 4: hipLaunchKernelGGL(delta_step_kernel<4>, grid, dim3(256), 0, st, p); break;
-            case 8: hipLaunchKernelGGL(delta_step_kernel<8>, grid, dim3(256), 0, st, p); break;
-            case 16: hipLaunchKernelGGL(delta_step_kernel<16>, grid, dim3(256), 0, st, p); break;
-            default: hipLaunchKernelGGL(delta_step_kernel<32>, grid, dim3(256), 0, st, p); break;
-        }
-        XFT_CHECK_HIP(hipGetLastError());
-        return 0;
-    }
-    auto columns = [&](int per_workgroup) { return dim3(v.B, p.H, (L.VD + per_workgroup - 1) / per_workgroup); };
-    switch (L.KD) {
-        case 32: hipLaunchKernelGGL((delta_scan_kernel<4, 2, 1>), columns(64), dim3(256), 0, st, p); break;
-        case 64: hipLaunchKernelGGL((delta_scan_kernel<8, 2, 1>), columns(32), dim3(256), 0, st, p); break;
-        case 128: hipLaunchKernelGGL((delta_scan_kernel<16, 2, 1>), columns(16), dim3(256), 0, st, p); break;
-        case 256: hipLaunchKernelGGL((delta_scan_kernel<32, 2, 1>), columns(8), dim3(256), 0, st, p); break;
+    auto launch = [&](auto several, auto single) {
+        if (one) hipLaunchKernelGGL(single, grid, dim3(256), 0, st, p);
+        else hipLaunchKernelGGL(several, grid, dim3(256), 0, st, p);
+    };
+    const int key = (v.longest == 1 ? 0 : 1000) + L.KD; // (both forms: 256 / lanes columns a workgroup)
+    switch (key) {
+        case 32: launch(delta_step_kernel<4, false>, delta_step_kernel<4, true>); break;
+        case 64: launch(delta_step_kernel<8, false>, delta_step_kernel<8, true>); break;
+        case 128: launch(delta_step_kernel<16, false>, delta_step_kernel<16, true>); break;
+        case 256: launch(delta_step_kernel<32, false>, delta_step_kernel<32, true>); break;
+        case 1032: launch(delta_scan_kernel<4, 2, 1, false>, delta_scan_kernel<4, 2, 1, true>); break;
+        case 1064: launch(delta_scan_kernel<8, 2, 1, false>, delta_scan_kernel<8, 2, 1, true>); break;
+        case 1128: launch(delta_scan_kernel<16, 2, 1, false>, delta_scan_kernel<16, 2, 1, true>); break;
+        case 1256: launch(delta_scan_kernel<32, 2, 1, false>, delta_scan_kernel<32, 2, 1, true>); break;
         default: set_error("delta_scan: key dimension %d of a head is above 256", L.s.dim); return 2;
     }
     XFT_CHECK_HIP(hipGetLastError());
@@ -565,7 +610,10 @@ int delta_scan(const PlanLayer &L, const StepView &v, const DeltaBuffers &b, hip
 }
 
 int delta_output(int act, const PlanLayer &L, const StepView &v, const DeltaBuffers &b, float eps, hipStream_t st) {
-    const OutParams p = {b.o, b.gates, L.out_norm, b.on, L.s.heads, L.VD, L.s.vdim, L.gcols, v.T, eps};
+    const size_t esz = act == XFTHIP_BF16 ? 2 : 4;
+    const size_t gate = (size_t)L.in_col + L.channels() + 2 * L.beta_cols(); // (behind beta and decays)
+    const OutParams p = {b.o, b.gates, L.out_norm, L.silu_gate() ? (const char *)b.in + gate * esz : nullptr, L.in_ld, (char *)b.out + L.out_col * esz, L.out_ld,
+            L.s.heads, L.VD, L.s.vdim, L.gcols, v.T, eps, L.mix_scale};
     const unsigned blocks = (unsigned)(((size_t)v.T * L.s.heads + 3) / 4);
     if (act == XFTHIP_BF16)
         hipLaunchKernelGGL(delta_output_kernel<true>, dim3(blocks), dim3(256), 0, st, p);

@@ -25,68 +25,104 @@ struct PrepareParams {
     StepView v;
     GroupedBuffers b;
     const float *q_norm, *k_norm, *cosT, *sinT; // norms may be null
+    int ld, value_col; // pitch of a's rows, first column of the values
     int H, G, D, V, dim, rot, interleaved, lanes; // lanes a head takes (a power of two, 8 values each)
+    int h0, h1; // heads to move, key heads behind the query heads
+    int all; // norms over all query heads, all key heads: a workgroup a token
     int qk_blocks, seg_blocks, keep; // keep: write first_values
     float share, eps; // share of first_values in the values
 };
 
-// One launch, two kinds of workgroups.  The first qk_blocks: a group of `lanes` threads one query or key head of a token.  The
-// others: one head's values of up to 32 tokens (a block of the cache), turned round through LDS.
+// Eight values of a head from c on, normed (r: factor of the norm, or 1) and rotated, to q or into the page
+template <bool BF16>
+__device__ inline void move_values(const PrepareParams &p, int t, int hh, int c, float (&x)[8], float r) {
+    const int D = p.D, H = p.H, G = p.G;
+    const float *norm = hh < H ? p.q_norm : p.k_norm;
+    if (norm && p.all) norm += (size_t)(hh < H ? hh : hh - H) * D;
+    const size_t at = (size_t)t * p.ld + (size_t)hh * D;
+    float w[8];
+#pragma unroll
+    for (int k = 0; k < 8; ++k) w[k] = 1.0f;
+    if (norm) load8<false>(norm, c, w);
+#pragma unroll
+    for (int k = 0; k < 8; ++k) x[k] = x[k] * r * w[k];
+    const int pos = p.v.tok_pos[t], half = p.rot / 2;
+    const float *cs = p.cosT + (size_t)pos * half, *sn = p.sinT + (size_t)pos * half;
+    if (p.interleaved) {
+#pragma unroll
+        for (int k = 0; k < 4; ++k) {
+            const int i = c / 2 + k;
+            if (i >= half) continue;
+            const float u = x[2 * k], z = x[2 * k + 1], cc = cs[i], ss = sn[i];
+            x[2 * k] = fmaf(u, cc, -(z * ss)), x[2 * k + 1] = fmaf(z, cc, u * ss);
+        }
+    } else {
+#pragma unroll
+        for (int k = 0; k < 8; ++k) {
+            const int d = c + k;
+            if (d >= p.rot) continue;
+            const int i = d < half ? d : d - half, other = d < half ? d + half : i;
+            const float z = ldact<BF16>(p.b.a, at + other) * r * (norm ? norm[other] : 1.0f);
+            x[k] = d < half ? fmaf(x[k], cs[i], -(z * sn[i])) : fmaf(x[k], cs[i], z * sn[i]);
+        }
+    }
+    if (hh < H) {
+        store8<BF16>(p.b.q, ((size_t)t * H + hh) * D + c, x);
+    } else {
+        const int *table = p.v.table + (size_t)p.v.seg_row[p.v.tok_seg[t]] * p.v.table_stride;
+        store8<BF16>(p.b.pool, head_page(table, pos, G, hh - H, D, p.V) + (size_t)(pos % kPageTokens) * D + c, x);
+    }
+}
+
+// One launch, two kinds of workgroups.  The first qk_blocks: a group of `lanes` threads one query or key head of a token (norms over all
+// heads: a workgroup a token).  The others: one head's values of up to 32 tokens (a block of the cache), turned round through LDS.
 template <bool BF16>
 __global__ __launch_bounds__(256) void grouped_prepare_kernel(PrepareParams p) {
-    const int D = p.D, V = p.V, H = p.H, G = p.G, row_len = H * D + G * (D + V);
+    const int D = p.D, V = p.V, H = p.H, G = p.G;
+    if ((int)blockIdx.x < p.qk_blocks && p.all) {
+        __shared__ float part[8];
+        const int t = blockIdx.x, q_end = H * D, end = p.h1 * D; // (h0 is 0)
+        const size_t row = (size_t)t * p.ld;
+        float sq = 0.0f, sk = 0.0f;
+        for (int e = threadIdx.x * 8; e < end; e += 2048) {
+            float x[8], sum = 0.0f;
+            load8<BF16>(p.b.a, row + e, x);
+#pragma unroll
+            for (int k = 0; k < 8; ++k) sum = fmaf(x[k], x[k], sum);
+            if (e < q_end) sq += sum;
+            else sk += sum;
+        }
+        sq = wave_total(sq), sk = wave_total(sk);
+        if ((threadIdx.x & 63) == 0) part[threadIdx.x >> 6] = sq, part[4 + (threadIdx.x >> 6)] = sk;
+        __syncthreads();
+        const float rq = 1.0f / sqrtf(((part[0] + part[1]) + (part[2] + part[3])) / (float)(H * p.dim) + p.eps);
+        const float rk = 1.0f / sqrtf(((part[4] + part[5]) + (part[6] + part[7])) / (float)(G * p.dim) + p.eps);
+        for (int e = threadIdx.x * 8; e < end; e += 2048) {
+            float x[8];
+            load8<BF16>(p.b.a, row + e, x);
+            move_values<BF16>(p, t, e / D, e % D, x, e < q_end ? rq : rk);
+        }
+        return;
+    }
     if ((int)blockIdx.x < p.qk_blocks) {
         const size_t idx = (size_t)blockIdx.x * 256 + threadIdx.x;
         const size_t item = idx / p.lanes;
-        const int c = (int)(idx % p.lanes) * 8, heads = H + G;
+        const int c = (int)(idx % p.lanes) * 8, heads = p.h1 - p.h0;
         const bool on = item < (size_t)p.v.T * heads && c < D;
-        const int t = on ? (int)(item / heads) : 0, hh = on ? (int)(item % heads) : 0;
-        const size_t at = (size_t)t * row_len + (size_t)hh * D;
-        float x[8], w[8];
+        const int t = on ? (int)(item / heads) : 0, hh = on ? (int)(item % heads) + p.h0 : p.h0;
+        float x[8];
 #pragma unroll
-        for (int k = 0; k < 8; ++k) x[k] = 0.0f, w[k] = 1.0f;
-        const float *norm = hh < H ? p.q_norm : p.k_norm;
-        if (on) {
-            load8<BF16>(p.b.a, at + c, x);
-            if (norm) load8<false>(norm, c, w);
-        }
+        for (int k = 0; k < 8; ++k) x[k] = 0.0f;
+        if (on) load8<BF16>(p.b.a, (size_t)t * p.ld + (size_t)hh * D + c, x);
         float r = 1.0f;
-        if (norm) {
+        if (p.q_norm) {
             float sq = 0.0f;
 #pragma unroll
             for (int k = 0; k < 8; ++k) sq = fmaf(x[k], x[k], sq);
             for (int off = p.lanes / 2; off > 0; off >>= 1) sq += __shfl_xor(sq, off, 64);
             r = 1.0f / sqrtf(sq / (float)p.dim + p.eps);
         }
-        if (!on) return;
-#pragma unroll
-        for (int k = 0; k < 8; ++k) x[k] = x[k] * r * w[k];
-        const int pos = p.v.tok_pos[t], half = p.rot / 2;
-        const float *cs = p.cosT + (size_t)pos * half, *sn = p.sinT + (size_t)pos * half;
-        if (p.interleaved) {
-#pragma unroll
-            for (int k = 0; k < 4; ++k) {
-                const int i = c / 2 + k;
-                if (i >= half) continue;
-                const float u = x[2 * k], z = x[2 * k + 1], cc = cs[i], ss = sn[i];
-                x[2 * k] = fmaf(u, cc, -(z * ss)), x[2 * k + 1] = fmaf(z, cc, u * ss);
-            }
-        } else {
-#pragma unroll
-            for (int k = 0; k < 8; ++k) {
-                const int d = c + k;
-                if (d >= p.rot) continue;
-                const int i = d < half ? d : d - half, other = d < half ? d + half : i;
-                const float z = ldact<BF16>(p.b.a, at + other) * r * (norm ? norm[other] : 1.0f);
-                x[k] = d < half ? fmaf(x[k], cs[i], -(z * sn[i])) : fmaf(x[k], cs[i], z * sn[i]);
-            }
-        }
-        if (hh < H) {
-            store8<BF16>(p.b.q, ((size_t)t * H + hh) * D + c, x);
-        } else {
-            const int *table = p.v.table + (size_t)p.v.seg_row[p.v.tok_seg[t]] * p.v.table_stride;
-            store8<BF16>(p.b.pool, head_page(table, pos, G, hh - H, D, V) + (size_t)(pos % kPageTokens) * D + c, x);
-        }
+        if (on) move_values<BF16>(p, t, hh, c, x, r);
         return;
     }
     __shared__ float tile[32][129];
@@ -106,7 +142,7 @@ __global__ __launch_bounds__(256) void grouped_prepare_kernel(PrepareParams p) {
             const int tok = lo + i / (slice / 8), c = i % (slice / 8) * 8, t = off + tok - start;
             const size_t first = ((size_t)t * G + g) * V + d0 + c;
             float x[8];
-            load8<BF16>(p.b.a, (size_t)t * row_len + (size_t)(H + G) * D + (size_t)g * V + d0 + c, x);
+            load8<BF16>(p.b.a, (size_t)t * p.ld + p.value_col + (size_t)g * V + d0 + c, x);
             if (p.keep) {
                 store8<BF16>(p.b.first_values, first, x);
             } else if (p.share != 0.0f) {
@@ -139,15 +175,60 @@ __global__ __launch_bounds__(256) void grouped_prepare_kernel(PrepareParams p) {
 struct AttendParams {
     StepView v;
     const void *q, *pool;
-    void *out;
+    int q_ld; // pitch of a token's queries
+    void *out; // rows of pitch out_ld
+    int out_ld;
     const float *sink; // or null
-    int H, G, D, V, window;
+    // the output: times out_scale, times sigmoid(gate) of every element or head (rows of pitch gate_ld, of the activation type)
+    const void *gate;
+    int gate_kind, gate_ld;
+    float out_scale;
+    float softcap; // or 0
+    int distance_bias;
+    int H, G, D, V, window, chunk;
     int min_len, max_len; // segments of other lengths are somebody else's
     float scale;
     int nsplit, groups; // context splits; column groups of the longest segment
     float *part; // [segments][G * groups][nsplit][16][V] outputs, behind them as many [2] maxima and sums
     size_t part_ml;
 };
+
+// first position that position `pos` sees
+__device__ inline int first_seen(const AttendParams &p, int pos) {
+    if (p.chunk > 0) return pos - pos % p.chunk;
+    return p.window > 0 && pos + 1 > p.window ? pos + 1 - p.window : 0;
+}
+// what a token of distance costs head h
+__device__ inline float head_slope(const AttendParams &p, int h) { return p.distance_bias ? exp2f(-8.0f * (float)(h + 1) / (float)p.H) : 0.0f; }
+
+// factors on four neighbouring outputs of a bf16 row
+__device__ inline f32x4 output_gate(const AttendParams &p, int t, int head, int d) {
+    f32x4 f = {p.out_scale, p.out_scale, p.out_scale, p.out_scale};
+    const uint16_t *row = (const uint16_t *)p.gate + (size_t)t * p.gate_ld;
+    if (p.gate_kind == XFTHIP_GATE_ELEMENT) {
+        const uint2 u = *(const uint2 *)(row + (size_t)head * p.V + d);
+        const f32x4 z = {u2f(u.x << 16), u2f(u.x & 0xFFFF0000u), u2f(u.y << 16), u2f(u.y & 0xFFFF0000u)};
+#pragma unroll
+        for (int k = 0; k < 4; ++k) f[k] *= __builtin_amdgcn_rcpf(1.0f + fast_exp(-z[k]));
+    } else if (p.gate_kind == XFTHIP_GATE_HEAD) {
+        f *= __builtin_amdgcn_rcpf(1.0f + fast_exp(-bf16_to_f32(row[head])));
+    }
+    return f;
+}
+
+// Scores that are more than a scaled product, in units of log2: a cap and a cost of distance
+struct ScoreRule {
+    float twice, cap2, slope2; // 2 log2(e) scale / cap, cap log2(e), slope log2(e)
+    __device__ inline float operator()(float s, float scale2, float distance) const {
+        // cap tanh(x / cap) = cap (1 - 2 / (exp(2 x / cap) + 1))
+        const float x = cap2 > 0.0f ? cap2 * fmaf(-2.0f, __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(s * twice) + 1.0f), 1.0f) : s * scale2;
+        return fmaf(-slope2, distance, x);
+    }
+};
+__device__ inline ScoreRule score_rule(const AttendParams &p, int head) {
+    const bool cap = p.softcap > 0.0f;
+    return ScoreRule {cap ? 2.0f * kLog2e * p.scale / p.softcap : 0.0f, cap ? p.softcap * kLog2e : 0.0f, head_slope(p, head) * kLog2e};
+}
 
 // Any type, any size: one workgroup a (token, head), 256 keys at a time, a key a thread for the scores and a value
 // dimension a thread for the weighted sum.
@@ -159,9 +240,10 @@ __global__ __launch_bounds__(256) void grouped_attend_kernel(AttendParams p) {
     const int t = blockIdx.x, h = blockIdx.y, g = h / (p.H / p.G);
     const int seg = p.v.tok_seg[t], pos = p.v.tok_pos[t];
     const int *table = p.v.table + (size_t)p.v.seg_row[seg] * p.v.table_stride;
-    for (int c = threadIdx.x; c < D; c += 256) qs[c] = ldact<BF16>(p.q, ((size_t)t * p.H + h) * D + c);
+    for (int c = threadIdx.x; c < D; c += 256) qs[c] = ldact<BF16>(p.q, (size_t)t * p.q_ld + (size_t)h * D + c);
     for (int c = threadIdx.x; c < V; c += 256) o[c] = 0.0f;
-    const int first = p.window > 0 && pos + 1 > p.window ? pos + 1 - p.window : 0;
+    const int first = first_seen(p, pos);
+    const float slope = head_slope(p, h);
     float m = p.sink ? p.sink[h] : -INFINITY, l = p.sink ? 1.0f : 0.0f; // the sink has no key and no value
     __syncthreads();
     for (int k0 = first; k0 <= pos; k0 += 256) {
@@ -177,6 +259,8 @@ __global__ __launch_bounds__(256) void grouped_attend_kernel(AttendParams p) {
                 for (int i = 0; i < 8; ++i) acc = fmaf(qs[c + i], k[i], acc);
             }
             s = acc * p.scale;
+            if (p.softcap > 0.0f) s = p.softcap * tanhf(s / p.softcap);
+            s -= slope * (float)(pos - j);
         }
         const float mx = wave_largest(s);
         if ((threadIdx.x & 63) == 0) part[threadIdx.x >> 6] = mx;
@@ -204,12 +288,16 @@ __global__ __launch_bounds__(256) void grouped_attend_kernel(AttendParams p) {
         }
         __syncthreads();
     }
-    for (int c = threadIdx.x; c < V; c += 256) stact<BF16>(p.out, ((size_t)t * p.H + h) * V + c, o[c] / l);
+    for (int c = threadIdx.x; c < V; c += 256) {
+        float y = o[c] / l * p.out_scale;
+        if (p.gate_kind) y /= 1.0f + expf(-ldact<BF16>(p.gate, (size_t)t * p.gate_ld + (p.gate_kind == XFTHIP_GATE_HEAD ? h : h * V + c)));
+        stact<BF16>(p.out, (size_t)t * p.out_ld + (size_t)h * V + c, y);
+    }
 }
 
-// BF16, short form.  KS: most 32-dim steps of a key; VT: most 16-dim tiles of a value; EXACT: as many.
-// grid (splits, G * column groups, segments)
-template <int KS, int VT, bool EXACT>
+// BF16, short form.  KS: most 32-dim steps of a key; VT: most 16-dim tiles of a value; EXACT: as many; RULE: scores are capped or
+// pay for distance.  grid (splits, G * column groups, segments)
+template <int KS, int VT, bool EXACT, bool RULE>
 __global__ __launch_bounds__(256, (KS <= 4 && VT <= 8) ? 3 : 1) void grouped_short_kernel(AttendParams p) {
     extern __shared__ float merge[]; // [4 waves][16][2] maxima and sums, [4][16][V + 4] outputs
     const StepView &v = p.v;
@@ -222,18 +310,20 @@ __global__ __launch_bounds__(256, (KS <= 4 && VT <= 8) ? 3 : 1) void grouped_sho
     const int *table = v.table + (size_t)v.seg_row[seg] * v.table_stride;
     const int last = c0 + 15 < ncols ? c0 + 15 : ncols - 1;
     const int lo = start + c0 / gs, hi = start + last / gs; // positions of the first and the last column's token
-    const int first_vis = p.window > 0 && lo + 1 > p.window ? lo + 1 - p.window : 0;
-    const int b0 = first_vis >> 5, b1 = (hi >> 5) + 1;
+    const int first_lo = first_seen(p, lo), first_hi = first_seen(p, hi);
+    const int b0 = first_lo >> 5, b1 = (hi >> 5) + 1;
     const int per = (b1 - b0 + p.nsplit - 1) / p.nsplit;
     int wb = b0 + (int)blockIdx.x * per, we = wb + per < b1 ? wb + per : b1;
     const int wper = (we - wb + 3) / 4; // this wave's blocks
     const int bb = wb + wave * wper, be = bb + wper < we ? bb + wper : we;
 
     const int c = c0 + i16, cv = c < ncols ? c : ncols - 1;
-    const int cpos = c < ncols ? start + c / gs : -1;
+    const int cpos = c < ncols ? start + c / gs : -1, cfirst = first_seen(p, cpos < 0 ? 0 : cpos);
+    ScoreRule rule;
+    if constexpr (RULE) rule = score_rule(p, g * gs + cv % gs);
     bf16x8 qf[KS];
     {
-        const uint16_t *row = (const uint16_t *)p.q + ((size_t)(off + cv / gs) * p.H + g * gs + cv % gs) * D + 8 * lg;
+        const uint16_t *row = (const uint16_t *)p.q + (size_t)(off + cv / gs) * p.q_ld + (size_t)(g * gs + cv % gs) * D + 8 * lg;
 #pragma unroll
         for (int ks = 0; ks < KS; ++ks)
             if (EXACT || ks < ks_n) qf[ks] = *(const bf16x8 *)(row + ks * 32);
@@ -274,16 +364,19 @@ __global__ __launch_bounds__(256, (KS <= 4 && VT <= 8) ? 3 : 1) void grouped_sho
                 s1 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[1][ks], qf[ks], s1, 0, 0, 0);
             }
         if (more) load_keys(blk + 1, page);
-        s0 *= scale2, s1 *= scale2;
+        if constexpr (!RULE) s0 *= scale2, s1 *= scale2;
         float x[8], bm = kUnseen;
 #pragma unroll
-        for (int j = 0; j < 8; ++j) x[j] = j < 4 ? s0[j & 3] : s1[j & 3];
-        const bool open = blk * 32 + 31 <= lo && (p.window <= 0 || blk * 32 > hi - p.window); // every column sees the whole block
+        for (int j = 0; j < 8; ++j) {
+            x[j] = j < 4 ? s0[j & 3] : s1[j & 3];
+            if constexpr (RULE) x[j] = rule(x[j], scale2, (float)(cpos - (blk * 32 + 8 * lg + j)));
+        }
+        const bool open = blk * 32 + 31 <= lo && blk * 32 >= first_hi; // every column sees the whole block
         if (!open) {
 #pragma unroll
             for (int j = 0; j < 8; ++j) {
                 const int t = blk * 32 + 8 * lg + j;
-                x[j] = t <= cpos && (p.window <= 0 || t > cpos - p.window) ? x[j] : kUnseen;
+                x[j] = t <= cpos && t >= cfirst ? x[j] : kUnseen;
             }
         }
 #pragma unroll
@@ -343,8 +436,9 @@ __global__ __launch_bounds__(256, (KS <= 4 && VT <= 8) ? 3 : 1) void grouped_sho
             if (d == 0) *(float2 *)(p.part + p.part_ml + (slot0 + col) * 2) = make_float2(mt, den);
         } else {
             if (p.sink) den += __builtin_amdgcn_exp2f(s2 - mt);
-            acc *= 1.0f / den;
-            uint16_t *dst = (uint16_t *)p.out + ((size_t)(off + cc / gs) * p.H + g * gs + cc % gs) * V + d;
+            const int t = off + cc / gs, head = g * gs + cc % gs;
+            acc *= output_gate(p, t, head, d) * (1.0f / den);
+            uint16_t *dst = (uint16_t *)p.out + (size_t)t * p.out_ld + (size_t)head * V + d;
             *(uint2 *)dst = make_uint2(pack_pair(acc[0], acc[1]), pack_pair(acc[2], acc[3]));
         }
     }
@@ -394,14 +488,15 @@ __global__ __launch_bounds__(256) void grouped_merge_kernel(AttendParams p) {
     __syncthreads();
     if (set > 0) return;
     for (int s = 1; s < sets; ++s) acc += sums[s * per + threadIdx.x];
-    acc *= inv_den;
-    uint16_t *dst = (uint16_t *)p.out + ((size_t)(v.seg_off[seg] + c / gs) * p.H + head) * V + d;
+    const int t = v.seg_off[seg] + c / gs;
+    acc *= output_gate(p, t, head, d) * inv_den;
+    uint16_t *dst = (uint16_t *)p.out + (size_t)t * p.out_ld + (size_t)head * V + d;
     *(uint2 *)dst = make_uint2(pack_pair(acc[0], acc[1]), pack_pair(acc[2], acc[3]));
 }
 
 // BF16, long form: 128 columns a workgroup (32 a wave), the visible context in blocks of 32 tokens through LDS, on 32 x 32 tiles.
-// KSM: most 16-dim steps of a key; VTM: most 32-dim tiles of a value; EXACT: as many.  grid (G, column groups, segments)
-template <int KSM, int VTM, bool EXACT>
+// KSM: most 16-dim steps of a key; VTM: most 32-dim tiles of a value; EXACT, RULE as above.  grid (G, column groups, segments)
+template <int KSM, int VTM, bool EXACT, bool RULE>
 __global__ __launch_bounds__(256, (KSM <= 8 && VTM <= 4) ? 2 : 1) void grouped_long_kernel(AttendParams p) {
     extern __shared__ unsigned char lds[];
     const StepView &v = p.v;
@@ -420,10 +515,12 @@ __global__ __launch_bounds__(256, (KSM <= 8 && VTM <= 4) ? 2 : 1) void grouped_l
     const int wlo = start + wc0 / gs, whi = start + wc1 / gs; // positions of the wave's first and last column
     const bool wave_on = wc0 < ncols;
     const int head = g * gs + cv % gs;
-    const size_t orow = (size_t)(off + cv / gs) * p.H + head;
+    const int token = off + cv / gs, pos_first = first_seen(p, pos);
+    ScoreRule rule;
+    if constexpr (RULE) rule = score_rule(p, head);
     bf16x8 qf[KSM];
     {
-        const uint16_t *row = (const uint16_t *)p.q + orow * D + 8 * h;
+        const uint16_t *row = (const uint16_t *)p.q + (size_t)token * p.q_ld + (size_t)head * D + 8 * h;
 #pragma unroll
         for (int ks = 0; ks < KSM; ++ks)
             if (EXACT || ks < ks_n) qf[ks] = *(const bf16x8 *)(row + ks * 16);
@@ -436,9 +533,8 @@ __global__ __launch_bounds__(256, (KSM <= 8 && VTM <= 4) ? 2 : 1) void grouped_l
     float m = kUnseen, l = 0.0f;
     const float scale2 = p.scale * kLog2e;
     const int lo = start + c0 / gs, last = c0 + 127 < ncols ? c0 + 127 : ncols - 1, hi = start + last / gs;
-    const int first = p.window > 0 && lo + 1 > p.window ? lo + 1 - p.window : 0;
-    const int b0 = first >> 5, b1 = (hi >> 5) + 1;
-    const int wfirst = p.window > 0 && wlo + 1 > p.window ? wlo + 1 - p.window : 0;
+    const int b0 = first_seen(p, lo) >> 5, b1 = (hi >> 5) + 1;
+    const int wfirst = first_seen(p, wlo), wfirst_hi = first_seen(p, whi);
 
     constexpr int PER = KSM / 4 + VTM / 2 + 1; // 16-byte chunks of a block a thread carries (at least D / 64 + V / 64)
     const int kch = D * 4, chunks = kch + V * 4; // of keys, of both
@@ -484,15 +580,18 @@ __global__ __launch_bounds__(256, (KSM <= 8 && VTM <= 4) ? 2 : 1) void grouped_l
 #pragma unroll
         for (int ks = 0; ks < KSM; ++ks)
             if (EXACT || ks < ks_n) s = __builtin_amdgcn_mfma_f32_32x32x16_bf16(*(const bf16x8 *)(krow + ks * 32), qf[ks], s, 0, 0, 0);
-        const bool masked = t0 + 31 > wlo || (p.window > 0 && t0 + p.window <= whi);
+        const bool masked = t0 + 31 > wlo || t0 < wfirst_hi;
         float bm = kUnseen;
 #pragma unroll
-        for (int r = 0; r < 16; ++r) s[r] *= scale2;
+        for (int r = 0; r < 16; ++r) {
+            if constexpr (RULE) s[r] = rule(s[r], scale2, (float)(pos - (t0 + 16 * (r >> 3) + 8 * h + (r & 7))));
+            else s[r] *= scale2;
+        }
         if (masked) {
 #pragma unroll
             for (int r = 0; r < 16; ++r) {
                 const int t = t0 + 16 * (r >> 3) + 8 * h + (r & 7);
-                s[r] = t <= pos && (p.window <= 0 || t > pos - p.window) ? s[r] : kUnseen;
+                s[r] = t <= pos && t >= pos_first ? s[r] : kUnseen;
             }
         }
 #pragma unroll
@@ -535,34 +634,45 @@ __global__ __launch_bounds__(256, (KSM <= 8 && VTM <= 4) ? 2 : 1) void grouped_l
         l = l * mul + __builtin_amdgcn_exp2f(s2 - mt);
     }
     mul /= l;
-    uint16_t *out = (uint16_t *)p.out + orow * V;
+    uint16_t *out = (uint16_t *)p.out + (size_t)token * p.out_ld + (size_t)head * V;
 #pragma unroll
     for (int d = 0; d < VTM; ++d)
         if (EXACT || d < vt_n) {
 #pragma unroll
-            for (int q = 0; q < 4; ++q)
-                *(uint2 *)(out + d * 32 + 8 * q + 4 * h) =
-                        make_uint2(pack_pair(o[d][4 * q] * mul, o[d][4 * q + 1] * mul), pack_pair(o[d][4 * q + 2] * mul, o[d][4 * q + 3] * mul));
+            for (int q = 0; q < 4; ++q) {
+                const int at = d * 32 + 8 * q + 4 * h;
+                const f32x4 f = output_gate(p, token, head, at) * mul;
+                *(uint2 *)(out + at) = make_uint2(pack_pair(o[d][4 * q] * f[0], o[d][4 * q + 1] * f[1]), pack_pair(o[d][4 * q + 2] * f[2], o[d][4 * q + 3] * f[3]));
+            }
         }
 }
 
-template <int KS, int VT, bool EXACT>
-int launch_short(const AttendParams &p, hipStream_t st) {
-    static const hipError_t attr = hipFuncSetAttribute((const void *)grouped_short_kernel<KS, VT, EXACT>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
+template <int KS, int VT, bool EXACT, bool RULE>
+int launch_short_form(const AttendParams &p, hipStream_t st) {
+    static const hipError_t attr = hipFuncSetAttribute((const void *)grouped_short_kernel<KS, VT, EXACT, RULE>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
     XFT_CHECK_HIP(attr);
     const size_t smem = (size_t)4 * 16 * (2 + p.V + 4) * 4;
-    hipLaunchKernelGGL((grouped_short_kernel<KS, VT, EXACT>), dim3(p.nsplit, p.G * p.groups, p.v.B), dim3(256), smem, st, p);
+    hipLaunchKernelGGL((grouped_short_kernel<KS, VT, EXACT, RULE>), dim3(p.nsplit, p.G * p.groups, p.v.B), dim3(256), smem, st, p);
     XFT_CHECK_HIP(hipGetLastError());
     return 0;
 }
-template <int KSM, int VTM, bool EXACT>
-int launch_long(const AttendParams &p, hipStream_t st) {
-    static const hipError_t attr = hipFuncSetAttribute((const void *)grouped_long_kernel<KSM, VTM, EXACT>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
+template <int KSM, int VTM, bool EXACT, bool RULE>
+int launch_long_form(const AttendParams &p, hipStream_t st) {
+    static const hipError_t attr = hipFuncSetAttribute((const void *)grouped_long_kernel<KSM, VTM, EXACT, RULE>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
     XFT_CHECK_HIP(attr);
     const size_t smem = (size_t)2 * (32 * (p.D * 2 + 16) + p.V * 80);
-    hipLaunchKernelGGL((grouped_long_kernel<KSM, VTM, EXACT>), dim3(p.G, (p.v.longest * (p.H / p.G) + 127) / 128, p.v.B), dim3(256), smem, st, p);
+    hipLaunchKernelGGL((grouped_long_kernel<KSM, VTM, EXACT, RULE>), dim3(p.G, (p.v.longest * (p.H / p.G) + 127) / 128, p.v.B), dim3(256), smem, st, p);
     XFT_CHECK_HIP(hipGetLastError());
     return 0;
+}
+bool has_rule(const AttendParams &p) { return p.softcap > 0.0f || p.distance_bias; }
+template <int KS, int VT, bool EXACT>
+int launch_short(const AttendParams &p, hipStream_t st) {
+    return has_rule(p) ? launch_short_form<KS, VT, EXACT, true>(p, st) : launch_short_form<KS, VT, EXACT, false>(p, st);
+}
+template <int KSM, int VTM, bool EXACT>
+int launch_long(const AttendParams &p, hipStream_t st) {
+    return has_rule(p) ? launch_long_form<KSM, VTM, EXACT, true>(p, st) : launch_long_form<KSM, VTM, EXACT, false>(p, st);
 }
 
 bool mfma_takes(const PlanLayer &L) { return L.D <= 256 && L.V <= 256; }
@@ -570,15 +680,20 @@ constexpr int kShortTokens = 16; // longest segment of the short form
 
 } // namespace
 
-int grouped_prepare(int act, const PlanLayer &L, const StepView &v, const GroupedBuffers &b, float eps, hipStream_t st) {
+int grouped_prepare(int act, const PlanLayer &L, const StepView &v, const GroupedBuffers &b0, float eps, hipStream_t st) {
     const xfthip_plan_layer &s = L.s;
-    PrepareParams p = {v, b, L.q_norm, L.kv_norm, L.cosT, L.sinT, s.heads, s.kv_heads, L.D, L.V, s.dim, s.rot_dim, s.rot_interleaved, 4, 0, 0, L.first_values ? 1 : 0,
+    const bool own = L.kv_from < 0;
+    GroupedBuffers b = b0;
+    b.a = (const char *)b.a + (size_t)L.in_col * (act == XFTHIP_BF16 ? 2 : 4);
+    PrepareParams p = {v, b, L.q_norm, L.kv_norm, L.cosT, L.sinT, L.in_ld, L.value_col(), s.heads, s.kv_heads, L.D, L.V, s.dim, s.rot_dim, s.rot_interleaved, 4,
+            L.moves_queries() ? 0 : s.heads, own ? s.heads + s.kv_heads : s.heads, s.qk_norm == XFTHIP_QK_NORM_ALL ? 1 : 0, 0, 0, L.first_values ? 1 : 0,
             s.v_mix && !L.first_values ? L.value_share : 0.0f, eps};
     while (p.lanes * 8 < L.D) p.lanes *= 2;
     XFT_REQUIRE(p.lanes <= 64, "grouped_prepare: heads of %d values too wide", L.D);
-    p.qk_blocks = (int)(((size_t)v.T * (s.heads + s.kv_heads) * p.lanes + 255) / 256);
-    p.seg_blocks = (v.longest + 62) / 32; // blocks of 32 positions a segment of that length can touch
+    p.qk_blocks = p.h0 >= p.h1 ? 0 : p.all ? v.T : (int)(((size_t)v.T * (p.h1 - p.h0) * p.lanes + 255) / 256);
+    p.seg_blocks = own ? (v.longest + 62) / 32 : 0; // blocks of 32 positions a segment of that length can touch
     const dim3 grid(p.qk_blocks + v.B * s.kv_heads * p.seg_blocks);
+    if (grid.x == 0) return 0;
     if (act == XFTHIP_BF16) hipLaunchKernelGGL(grouped_prepare_kernel<true>, grid, dim3(256), 0, st, p);
     else hipLaunchKernelGGL(grouped_prepare_kernel<false>, grid, dim3(256), 0, st, p);
     XFT_CHECK_HIP(hipGetLastError());
@@ -590,7 +705,8 @@ int grouped_split_count(const PlanLayer &L, int B, int longest, int hint) {
     if (!mfma_takes(L)) return 1;
     longest = longest < kShortTokens ? longest : kShortTokens;
     const long units = (long)B * L.s.kv_heads * ((longest * (L.s.heads / L.s.kv_heads) + 15) / 16);
-    const int ctx = L.s.window > 0 && L.s.window + longest < hint ? L.s.window + longest : hint;
+    const int span = L.s.chunk > 0 ? L.s.chunk : L.s.window;
+    const int ctx = span > 0 && span + longest < hint ? span + longest : hint;
     const int most = (ctx + 127) / 128;
     long want = device_cu_count() / units;
     want = want < most ? want : most;
@@ -603,10 +719,14 @@ size_t grouped_part_floats(const PlanLayer &L) {
     return mfma_takes(L) ? (size_t)device_cu_count() * 16 * (L.V + 2) : 0;
 }
 
-int grouped_attention(int act, const PlanLayer &L, const StepView &v, const void *q, const void *pool, void *out, int hint, float *part, size_t part_floats,
+int grouped_attention(int act, const PlanLayer &L, const StepView &v, const GroupedBuffers &b, void *out, int hint, float *part, size_t part_floats,
         hipStream_t st) {
     const xfthip_plan_layer &s = L.s;
-    AttendParams p = {v, q, pool, out, L.sink, s.heads, s.kv_heads, L.D, L.V, s.window, 0, 1 << 30, s.scale, 1, 1, part, 0};
+    const size_t esz = act == XFTHIP_BF16 ? 2 : 4;
+    const char *rows = (const char *)b.a + L.in_col * esz;
+    AttendParams p = {v, L.moves_queries() ? b.q : rows, b.pool, L.moves_queries() ? s.heads * L.D : L.in_ld, (char *)out + L.out_col * esz, L.out_ld, L.sink,
+            rows + L.gate_col() * esz, s.out_gate, L.in_ld, L.mix_scale, s.softcap, s.distance_bias, s.heads, s.kv_heads, L.D, L.V, s.window, s.chunk, 0, 1 << 30,
+            s.scale, 1, 1, part, 0};
     if (act != XFTHIP_BF16 || !mfma_takes(L)) {
         const size_t smem = (size_t)(L.D + 256 + L.V + 8) * 4;
         if (act == XFTHIP_BF16) hipLaunchKernelGGL(grouped_attend_kernel<true>, dim3(v.T, s.heads), dim3(256), smem, st, p);

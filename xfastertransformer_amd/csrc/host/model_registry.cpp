@@ -379,11 +379,100 @@ PlanSpec veterax(const Json &c, const SafeTensors &) {
     return s;
 }
 
+// ---- Duvadra: pre-norm layers whose mixer is chunked attention with capped scores and a cost of distance (its keys and values
+// perhaps an earlier layer's), or a windowed attention beside a recurrence: with a sink beside a gated delta rule, or with keys that
+// serve as values beside a gated linear recurrence; dense or routed feed-forwards, embeddings of token pairs ----
+PlanSpec duvadra(const Json &c, const SafeTensors &) {
+    PlanSpec s;
+    s.cfg.hidden = (int)c.integer("width");
+    s.cfg.vocab = (int)c.integer("vocab");
+    s.cfg.eps = (float)c.at("norm").real("eps");
+    s.cfg.logit_scale = 1.0f;
+    s.cfg.loop_times = 1;
+    s.cfg.block = XFTHIP_BLOCK_SERIAL, s.cfg.norm = XFTHIP_NORM_RMS;
+    s.cfg.residual_mult = (float)c.real("residual_mult");
+    if (c.has("logit_softcap")) s.cfg.logit_softcap = (float)c.real("logit_softcap");
+    const Json &emb = c.at("embedding");
+    s.cfg.embed_scale = (float)emb.real("scale");
+    if (emb.has("bigram")) {
+        const Json &b = emb.at("bigram");
+        s.cfg.bigram_buckets = b.integer("buckets"), s.cfg.bigram_mul_prev = b.integer("mul_prev"), s.cfg.bigram_mul_cur = b.integer("mul_cur");
+    }
+    auto sizes = [](const Json &m) {
+        xfthip_plan_layer L {};
+        L.heads = (int)m.integer("heads"), L.kv_heads = (int)m.integer("kv_heads"), L.dim = (int)m.integer("dim"), L.vdim = (int)m.integer("vdim");
+        return L;
+    };
+    const Json &layers = c.at("layers");
+    for (size_t i = 0; i < layers.items.size(); ++i) {
+        const std::string at = "layer " + std::to_string(i) + ": ";
+        const Json &e = layers.items[i], &m = e.at("mixer");
+        const std::string &type = e.string("type");
+        const bool one = type == "attention", first = type == "parallel";
+        if (!one && !first && type != "parallel_2") broken("layer type '" + type + "' of config.json is not known");
+        const Json &a = one ? m : m.at("left");
+        xfthip_plan_layer L = sizes(a), R {};
+        L.mixer = XFTHIP_MIXER_GROUPED;
+        L.scale = (float)a.real("scale");
+        const int span = (int)a.at("mask").integer("size");
+        if (span < 1) broken(at + "an empty window or chunk");
+        (one ? L.chunk : L.window) = span;
+        if (one) {
+            L.softcap = (float)a.real("softcap");
+            L.distance_bias = 1, L.out_gate = XFTHIP_GATE_HEAD;
+            if (a.has("kv_from")) {
+                const long j = a.integer("kv_from");
+                if (j < 0 || j >= (long)i) broken(at + "keys and values of a layer that is not before it");
+                L.kv_from = s.record[(size_t)j] + 1;
+            }
+        } else {
+            const Json &r = m.at("right");
+            L.out_gate = XFTHIP_GATE_ELEMENT;
+            L.scaled = 1, L.mix_scale = (float)m.real("left_scale");
+            if (first) {
+                L.qkv_bias = 1, L.has_sink = 1;
+                R = sizes(r);
+                R.mixer = XFTHIP_MIXER_DELTA;
+            } else {
+                L.key_values = 1, L.qk_norm = XFTHIP_QK_NORM_ALL;
+                L.rot_dim = (int)a.at("rot").integer("dims"), L.rot_base = a.at("rot").real("base"), L.rot_interleaved = 1;
+                R.mixer = XFTHIP_MIXER_UNIT;
+                const long width = r.integer("width");
+                R.heads = (int)r.integer("blocks");
+                if (R.heads < 1 || width % R.heads) broken(at + "a recurrence that does not divide into its blocks");
+                R.dim = R.vdim = (int)(width / R.heads);
+            }
+            R.taps = (int)r.integer("conv");
+            R.beside = 1, R.scaled = 1, R.mix_scale = (float)m.real("right_scale");
+        }
+        if (e.has("mlp")) {
+            const Json &f = e.at("mlp");
+            const std::string &kind = f.string("kind");
+            if (kind == "dense") {
+                L.inter = (int)f.integer("ff"), L.glu_limit = (float)f.real("limit"), L.glu_alpha = 1.702f;
+            } else if (kind == "moe") {
+                const Json &r = f.at("router"), &g = r.at("groups");
+                L.experts = (int)r.integer("experts"), L.top = (int)r.integer("top"), L.expert_inter = (int)f.at("expert").integer("ff");
+                if (L.experts < 1) broken(at + "a router without experts");
+                L.router = XFTHIP_ROUTE_SIGMOID_GROUPS;
+                L.route_groups = (int)g.integer("count"), L.route_keep = (int)g.integer("keep"), L.route_scale = (float)r.real("scale");
+            } else {
+                broken("feed-forward '" + kind + "' of config.json is not known");
+            }
+        }
+        s.record.push_back((int)s.layers.size());
+        s.layers.push_back(L);
+        if (!one) s.layers.push_back(R);
+    }
+    s.cfg.layers = (int)s.layers.size();
+    return s;
+}
+
 struct Architecture {
     const char *name;
     PlanSpec (*describe)(const Json &config, const SafeTensors &weights);
 };
-const Architecture kArchitectures[] = {{"Pinepel", pinepel}, {"Veterax", veterax}};
+const Architecture kArchitectures[] = {{"Pinepel", pinepel}, {"Veterax", veterax}, {"Duvadra", duvadra}};
 
 const Architecture *find_architecture(const Json &c) {
     if (c.kind != Json::Object || !c.has("architecture") || c.at("architecture").kind != Json::String) return nullptr;
@@ -427,7 +516,13 @@ xfthip_plan_t load_plan(const std::string &dir, PlanSpec &spec) {
         if (name.size() > 2 && name[0] == 'l' && isdigit((unsigned char)name[1])) {
             char *end = nullptr;
             const long i = strtol(name.c_str() + 1, &end, 10);
-            if (*end == '.' && i < spec.cfg.layers) layer = (int)i, name = std::string(end + 1);
+            const long layers = spec.record.empty() ? spec.cfg.layers : (long)spec.record.size();
+            if (*end == '.' && i < layers) {
+                layer = spec.record.empty() ? (int)i : spec.record[(size_t)i], name = std::string(end + 1);
+                // mixers side by side: 'mix.left.' is the layer's record, 'mix.right.' the one behind it
+                if (name.compare(0, 9, "mix.left.") == 0) name.erase(4, 5);
+                else if (name.compare(0, 10, "mix.right.") == 0) name.erase(4, 6), ++layer;
+            }
         }
         const TensorRef &t = kv.second;
         const long rows = t.shape.empty() ? 1 : t.shape[0], n = t.count();

@@ -57,6 +57,7 @@ private:
 struct PlanSpec {
     xfthip_plan_config cfg {};
     std::vector<xfthip_plan_layer> layers;
+    std::vector<int> record; // of every layer of the model, where some have two mixers (empty: one record a layer)
 };
 
 // is there a config.json whose architecture this build knows; its name

@@ -472,7 +472,8 @@ struct ModelImpl {
             const int runs = i >= planSpec.cfg.loop_start && i < planSpec.cfg.loop_stop ? times : 1;
             const double e = planAct == XFTHIP_F32 ? 4 : 2;
             b += runs * (y.mixer == XFTHIP_MIXER_LATENT    ? (double)len * (y.kv_rank + y.rot_dim) * e
-                         : y.mixer == XFTHIP_MIXER_GROUPED ? (double)len * y.kv_heads * (y.dim + y.vdim) * e
+                         : y.mixer == XFTHIP_MIXER_GROUPED ? (y.kv_from ? 0.0 : (double)len * y.kv_heads * (y.dim + y.vdim) * e)
+                         : y.mixer == XFTHIP_MIXER_UNIT    ? (double)y.heads * y.dim * (4 + (y.taps - 1) * e)
                                                            : (double)y.heads * y.dim * y.vdim * 4);
         }
         return b;
@@ -1693,7 +1694,7 @@ AutoModel::AutoModel(std::string modelPath, xft::DataType dataType, xft::DataTyp
         s.planAct = full ? XFTHIP_F32 : XFTHIP_BF16;
         s.plan = load_plan(modelPath, s.planSpec);
         s.weightBytes = xfthip_plan_weight_bytes(s.plan);
-        s.layers = s.planSpec.cfg.layers, s.hidden = s.planSpec.cfg.hidden, s.vocab = s.planSpec.cfg.vocab;
+        s.layers = s.planSpec.record.empty() ? s.planSpec.cfg.layers : (int)s.planSpec.record.size(), s.hidden = s.planSpec.cfg.hidden, s.vocab = s.planSpec.cfg.vocab;
         s.startId = 0, s.endId = -1; // such a directory names no end token: the caller does
         // nothing in it bounds the positions either; XFT_MAX_POSITIONS does
         s.maxPositions = 8192;

@@ -1,7 +1,7 @@
-// Layer plans: decoder stacks whose layers differ in kind (latent attention, grouped attention, delta-rule recurrence), whose
-// keys live in a page pool shared by all sequences and whose recurrent layers keep a state per sequence slot.  Declarations
-// shared by the plan's driver (plan_model.hip) and its kernels (plan_layers.hip, latent_attention.hip, grouped_attention.hip,
-// delta_rule.hip, routed_experts.hip, tile_gemm.hip).
+// Layer plans: decoder stacks whose layers differ in kind (latent attention, grouped attention, delta-rule recurrence, gated
+// linear recurrence), whose keys live in a page pool shared by all sequences and whose recurrent layers keep a state per sequence
+// slot.  Declarations shared by the plan's driver (plan_model.hip) and its kernels (plan_layers.hip, latent_attention.hip,
+// grouped_attention.hip, delta_rule.hip, gated_unit.hip, routed_experts.hip, tile_gemm.hip).
 //
 // Every inner width is padded to whole 32-value groups (the state's key dimension to a power of two) by zero rows and
 // columns of the packed weights, so that the kernels see whole MFMA steps whatever sizes a model has.
@@ -37,10 +37,17 @@ struct PlanLayer {
     // latent attention: padded widths of a head's unrotated / rotated / value part, of the key and the query latent;
     // grouped attention: D and V, of the query / key and the value part of a head
     int D = 0, RD = 0, V = 0, R = 0, QR = 0;
-    // delta rule: padded key / value width of a head, padded rank of the two gates and columns of one gate
+    // delta rule: padded key / value width of a head, padded rank of the two gates and columns of one gate; gated unit: D, of a block
     int KD = 0, VD = 0, rank = 0, gcols = 0;
+    // Where a mixer finds its projections and puts its result: mixers side by side share the rows of one input product
+    // (row_in() columns from in_col on of in_ld) and of one output product (out_cols() from out_col on of out_ld).
+    int in_col = 0, in_ld = 0, out_col = 0, out_ld = 0;
+    float mix_scale = 1.0f; // of the result
+    int beside = -1; // the record of the mixer next to this one
+    int kv_from = -1; // grouped attention: the record whose cache serves
     int ff = 0; // padded
-    xfthip_weight_t in = nullptr, o = nullptr, gateup = nullptr, down = nullptr;
+    xfthip_weight_t in = nullptr, o = nullptr, gateup = nullptr, down = nullptr; // (in, o: of both mixers, with the first one)
+    float *in_bias = nullptr; // [in_ld] or null
     // latent: queries from their latent; W_uk turned round (query -> latent), W_uk and W_uv (latent -> key / value)
     xfthip_weight_t uq = nullptr, absorb = nullptr, uk = nullptr, uv = nullptr;
     float *q_norm = nullptr, *kv_norm = nullptr, *sink = nullptr; // (grouped attention: weights of the query and the key heads)
@@ -50,6 +57,8 @@ struct PlanLayer {
     // delta rule: both gates' second projections (decay | output gate), filters [channels][taps], exp(A_log), ...
     xfthip_weight_t gates = nullptr;
     float *conv = nullptr, *decay = nullptr, *dt_bias = nullptr, *out_norm = nullptr;
+    // gated unit (conv as above, gates: both square products of every block): filter biases, 8 softplus(lambda), biases [blocks][2][D]
+    float *conv_bias = nullptr, *lambda = nullptr, *gate_bias = nullptr;
     // routed experts: padded width, weights of one shape by expert and their device table ([experts] gate / up, [experts] down)
     int eff = 0;
     std::vector<xfthip_weight_t> egateup, edown;
@@ -63,31 +72,56 @@ struct PlanLayer {
     PlanNorm pre1, pre2;
     float *post1 = nullptr, *post2 = nullptr;
 
+    // columns of the input product: latent: query latent | key latent | shared key part; grouped: q | k | v | gate; delta rule: q | k |
+    // v | beta | decays | gate; gated unit: y | x
     int row_in() const {
         if (s.mixer == XFTHIP_MIXER_LATENT) return QR + R + RD;
-        if (s.mixer == XFTHIP_MIXER_GROUPED) return s.heads * D + s.kv_heads * (D + V);
-        return (2 * s.kv_heads * KD + s.heads * VD) + beta_cols() + 2 * rank;
+        if (s.mixer == XFTHIP_MIXER_GROUPED) return gate_col() + (s.out_gate == XFTHIP_GATE_ELEMENT ? s.heads * V : s.out_gate == XFTHIP_GATE_HEAD ? beta_cols() : 0);
+        if (s.mixer == XFTHIP_MIXER_UNIT) return 2 * s.heads * D;
+        return channels() + beta_cols() + (head_decay() ? beta_cols() : rank) + (silu_gate() ? s.heads * VD : rank);
     }
-    bool paged() const { return s.mixer != XFTHIP_MIXER_DELTA; }
+    int out_cols() const { return s.mixer == XFTHIP_MIXER_UNIT ? s.heads * D : s.heads * (s.mixer == XFTHIP_MIXER_DELTA ? VD : V); }
+    // grouped attention: first columns of values and gate
+    int value_col() const { return s.heads * D + (s.key_values ? 0 : s.kv_heads * D); }
+    int gate_col() const { return s.heads * D + (kv_from >= 0 ? 0 : s.kv_heads * (D + (s.key_values ? 0 : V))); }
+    bool moves_queries() const { return s.rot_dim > 0 || s.qk_norm; } // or they stay in the row
+    bool head_decay() const { return s.decay_rank == 0; }
+    bool silu_gate() const { return s.gate_rank == 0; }
+    bool paged() const { return s.mixer == XFTHIP_MIXER_LATENT || s.mixer == XFTHIP_MIXER_GROUPED; }
     // elements a token takes in the page pool
     size_t token_elems() const { return s.mixer == XFTHIP_MIXER_LATENT ? R + RD : (size_t)s.kv_heads * (D + V); }
+    // floats of a slot's state, channels of the short convolution
+    size_t state_floats() const { return s.mixer == XFTHIP_MIXER_UNIT ? (size_t)s.heads * D : (size_t)s.heads * VD * KD; }
+    int channels() const { return s.mixer == XFTHIP_MIXER_UNIT ? s.heads * D : 2 * s.kv_heads * KD + s.heads * VD; } // (delta rule: q | k | v)
     int routes() const { return s.experts + s.identity; }
     bool feeds_forward() const { return ff > 0 || s.experts > 0; }
     int beta_cols() const { return (s.heads + 31) / 32 * 32; }
-    int channels() const { return 2 * s.kv_heads * KD + s.heads * VD; } // of the short convolution: q | k | v
 };
 
 struct LayerRun {
     int layer;
     bool add_embedding; // the embedding output joins the residual in front of this run
+    int beside = -1; // the record of the layer's second mixer, and its place among caches and states
+    int beside_store = -1;
 };
 
 // ---- kernels -----------------------------------------------------------------------------------------------------
 // (act: XFTHIP_BF16 or XFTHIP_F32, the type of activations between kernels; the residual is fp32)
 
-// x[t] = table[ids[t]] (bf16 table, ids clamped to the vocabulary)
-int plan_embed(const uint16_t *table, const int *ids, float *x, int T, int hidden, int vocab, hipStream_t st);
-// x += rms(y) * post (y may be null), then x += table[ids] (table may be null), then xn = pre(x) (pre.w may be null) and
+// x = table[id] * scale (bf16 tables, ids clamped to the vocabulary), with a pair table: plus its row of (previous token, token) - the
+// row behind the buckets for the first token of a sequence
+struct EmbedTables {
+    const uint16_t *table, *pairs; // pairs: [buckets + 1][hidden] or null
+    int hidden, vocab;
+    float scale;
+    long long buckets, mul_prev, mul_cur;
+};
+// the step's tokens; last_token [slots]: of the tokens a slot has seen
+int plan_embed(const EmbedTables &e, const StepView &v, const int *ids, const int *last_token, float *x, hipStream_t st);
+// logits pass cap * tanh(z / cap)
+int plan_softcap(float *logits, size_t n, float cap, hipStream_t st);
+
+// x += rms(y) * post (y may be null; post null: x += mul * y), then x += table[ids] (table may be null), then xn = pre(x) (pre.w may be null) and
 // xn2 = pre2(x) (pre2.w may be null; tanh norms only).  Means over `width` of the `hidden` columns.  rows: xn row i comes from x
 // row rows[i] (only without y and table).
 struct PlanNormArgs {
@@ -101,6 +135,7 @@ struct PlanNormArgs {
     const int *rows;
     int hidden, width;
     float eps;
+    float mul;
 };
 int plan_norm(int act, const PlanNormArgs &p, int T, hipStream_t st);
 // out[t][c] = gelu(z[t][c]) * table[ids[t]][first + c] (tanh form of the gelu), c < width; bf16 table [vocab][ld], ids clamped
@@ -116,8 +151,9 @@ struct TileGemmArgs {
     void *C = nullptr;
     int ldc = 0, c_dtype = XFTHIP_F32;
     bool add = false; // C += (fp32)
-    bool glu = false; // the weight holds gate / up pairs (XFTHIP_WF_GATEUP), combined as clamped_glu
+    bool glu = false; // the weight holds gate / up pairs (XFTHIP_WF_GATEUP), combined as clamped_glu, or (glu_alpha 0) silu(gate) * up
     float glu_limit = 0, glu_alpha = 0;
+    const float *bias = nullptr; // [N], joins the product (not with glu)
     // C = gelu(product) * side[ids[t]][n] (as plan_side_gate)
     const uint16_t *side = nullptr;
     int side_ld = 0;
@@ -139,8 +175,16 @@ struct RouteBuffers {
     int *row_token; // [T * top] token of a gathered row
     int *group_rows; // [experts][3] records of the expert products
 };
-// softmax over a token's `routes` logits (row pitch ld), the `top` largest of score + correction, lists of tokens by expert
-int route_tokens(const float *logits, int ld, const float *correction, int T, int experts, int routes, int top, const RouteBuffers &b, hipStream_t st);
+// softmax over a token's `routes` logits (row pitch ld), the `top` largest of score + correction; or (groups > 0) sigmoid scores, the `top`
+// largest within the `keep` groups whose two best scores sum highest, divided by their sum and multiplied by `scale`.  Then lists of
+// tokens by expert
+struct RouteRule {
+    int experts, routes, top;
+    const float *correction;
+    int groups, keep;
+    float scale;
+};
+int route_tokens(const float *logits, int ld, const RouteRule &rule, int T, const RouteBuffers &b, hipStream_t st);
 // dst[t] = base[t] + sum over choices of weight * (expert output row, or h[t]); base, dst fp32 (base may be null or dst), h of the
 // activation type; narrow (or null): dst once more, of the activation type
 int combine_experts(int act, const float *base, const float *outputs, const void *h, int top, const RouteBuffers &b, float *dst, void *narrow, int T,
@@ -148,15 +192,15 @@ int combine_experts(int act, const float *base, const float *outputs, const void
 
 // ---- grouped attention
 struct GroupedBuffers {
-    const void *a; // [T][row_in] of the activation type: q | k | v
-    void *q; // [T][heads][D]
+    const void *a; // the step's rows of the input product, of the activation type: q | k | v | gate from in_col on
+    void *q; // [T][heads][D]: normed, rotated queries
     void *pool; // pages: by key / value head [64][D] keys, then two blocks of 32 tokens [V][32] values
     void *first_values; // [T][kv_heads][V]: written by the layer that says so, read by the others that mix
 };
 // norms and rotation of queries and keys, mixing of values, append to the pages
 int grouped_prepare(int act, const PlanLayer &L, const StepView &v, const GroupedBuffers &b, float eps, hipStream_t st);
-// out [T][heads][V]; hint: upper bound of the sequence lengths
-int grouped_attention(int act, const PlanLayer &L, const StepView &v, const void *q, const void *pool, void *out, int hint, float *part, size_t part_floats,
+// out: the step's rows of the output product's input; hint: upper bound of the sequence lengths
+int grouped_attention(int act, const PlanLayer &L, const StepView &v, const GroupedBuffers &b, void *out, int hint, float *part, size_t part_floats,
         hipStream_t st);
 int grouped_split_count(const PlanLayer &L, int B, int longest, int hint);
 size_t grouped_part_floats(const PlanLayer &L);
@@ -186,18 +230,34 @@ int latent_expanded(const PlanLayer &L, int off, int start, int n, int base, con
         hipStream_t st);
 
 struct DeltaBuffers {
-    void *in; // [T][row_in] of the activation type: q | k | v | beta | decay rank | gate rank
+    void *in; // rows of the input product, of the activation type: q | k | v | beta | decay (rank) | gate (rank) from in_col on
     float *gates; // [T][2 * gcols]: decay step (before softplus) | output gate (before the sigmoid)
     float *q, *k, *qk; // [T][kv_heads][KD] twice, [T][kv_heads]
-    float *g, *v, *beta; // [T][heads][KD], [T][heads][VD], [T][heads]
+    float *g, *v, *beta; // [T][heads][KD] (one decay a head: [T][heads]), [T][heads][VD], [T][heads]
     float *o; // [T][heads][VD]
-    void *on; // [T][heads * VD] of the activation type
+    void *out; // rows of the output product's input, of the activation type
     float *state; // [slots][heads][VD][KD]
     void *conv_state; // [slots][taps - 1][channels] of the activation type
 };
+// the last taps - 1 inputs of segments of several tokens: in [T] rows of pitch ld -> conv_state
+int conv_tail(int act, const StepView &v, const void *in, int ld, int channels, int taps, void *conv_state, hipStream_t st);
 int delta_prepare(int act, const PlanLayer &L, const StepView &v, const DeltaBuffers &b, hipStream_t st);
 int delta_scan(const PlanLayer &L, const StepView &v, const DeltaBuffers &b, hipStream_t st);
 int delta_output(int act, const PlanLayer &L, const StepView &v, const DeltaBuffers &b, float eps, hipStream_t st);
+
+// ---- gated linear recurrence: S = a S + sqrt(1 - a^2) i u by channel, a and i gated by the filtered input u itself
+struct UnitBuffers {
+    const void *in; // rows of the input product, of the activation type: y | x from in_col on
+    void *u; // [T][channels] of the activation type
+    float *gates; // [T][blocks][2][D]: r | i before their biases and sigmoids
+    float *carry; // unit_carry_floats()
+    void *out; // rows of the output product's input, of the activation type
+    float *state; // [slots][channels]
+    void *conv_state; // [slots][taps - 1][channels] of the activation type
+};
+int unit_filter(int act, const PlanLayer &L, const StepView &v, const UnitBuffers &b, hipStream_t st);
+int unit_scan(int act, const PlanLayer &L, const StepView &v, const UnitBuffers &b, hipStream_t st);
+size_t unit_carry_floats(const PlanLayer &L, size_t tokens, size_t segments);
 
 } // namespace xfthip
 
@@ -208,6 +268,7 @@ struct xfthip_plan {
     int hidden = 0; // width padded to whole 32-value groups
     uint16_t *embedding = nullptr; // [vocab][hidden] bf16
     xfthip::PlanNorm final_norm; // times the logit scale
+    uint16_t *pair_embedding = nullptr; // [bigram_buckets + 1][hidden] bf16
     uint16_t *side_embedding = nullptr; // [vocab][layers * side_pad] bf16
     int side_pad = 0;
     xfthip_weight_t head = nullptr;
@@ -228,7 +289,9 @@ struct PlanState {
     std::vector<PlanLayer> layers; // the plan's, with this model's rotation tables
     int act = XFTHIP_BF16, esz = 2;
     int slots = 0;
-    // by layer run: page pool of an attention, state and convolution inputs of a delta rule
+    // by layer run, second mixers behind all of them: the record, page pool of an attention, state and convolution inputs of a
+    // recurrence; which page pool an attention reads
+    std::vector<int> store_layer, reads;
     std::vector<void *> cache;
     std::vector<float *> state;
     std::vector<void *> conv_state;
@@ -250,8 +313,9 @@ struct PlanState {
     std::vector<int> logit_of_row; // which row of the logits a slot's last ones are in
     int logit_rows = 0;
     // scratch (activation type unless float)
-    void *xn = nullptr, *a = nullptr, *cq = nullptr, *q = nullptr, *qa = nullptr, *oc = nullptr, *ov = nullptr, *h = nullptr, *on = nullptr;
-    float *y = nullptr, *gates = nullptr, *dq = nullptr, *dk = nullptr, *dqk = nullptr, *dg = nullptr, *dv = nullptr, *dbeta = nullptr, *do_ = nullptr;
+    void *xn = nullptr, *a = nullptr, *cq = nullptr, *q = nullptr, *qa = nullptr, *oc = nullptr, *ov = nullptr, *h = nullptr, *u = nullptr;
+    float *y = nullptr, *gates = nullptr, *dq = nullptr, *dk = nullptr, *dqk = nullptr, *dg = nullptr, *dv = nullptr, *dbeta = nullptr, *do_ = nullptr, *carry = nullptr;
+    int *last_token = nullptr; // [slots]
     void *xn2 = nullptr, *first_values = nullptr, *side = nullptr, *narrow = nullptr;
     float *router_logits = nullptr, *expert_out = nullptr, *side_z = nullptr;
     void *eh = nullptr;

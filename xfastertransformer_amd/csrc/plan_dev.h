@@ -72,6 +72,19 @@ __device__ inline void put4(void *p, size_t i, f32x4 v) {
 // tanh form of the Gaussian error linear unit
 __device__ inline float gelu_tanh(float z) { return 0.5f * z * (1.0f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z))); }
 
+// a row of the residual from a token and the one before it (prev: any value in front of a sequence's first token)
+__device__ inline void embed_token(const EmbedTables &e, int id, bool first, int prev, float *x) {
+    id = id < 0 ? 0 : (id >= e.vocab ? e.vocab - 1 : id);
+    prev = prev < 0 ? 0 : (prev >= e.vocab ? e.vocab - 1 : prev);
+    const uint16_t *row = e.table + (size_t)id * e.hidden;
+    const uint16_t *pair = e.pairs;
+    if (pair) pair += (size_t)(first ? e.buckets : (prev * e.mul_prev + id * e.mul_cur) % e.buckets) * e.hidden;
+    for (int c = threadIdx.x; c < e.hidden; c += blockDim.x) {
+        const float v = bf16_to_f32(row[c]) * e.scale;
+        x[c] = pair ? v + bf16_to_f32(pair[c]) : v;
+    }
+}
+
 typedef uint32_t u32x4 __attribute__((ext_vector_type(4)));
 constexpr float kUnseen = -1.0e30f; // score of a masked key, maximum of a column that has seen none
 constexpr float kLog2e = 1.4426950408889634f;

@@ -6,11 +6,15 @@ namespace xfthip {
 
 namespace {
 
-__global__ void plan_embed_kernel(const uint16_t *__restrict__ table, const int *__restrict__ ids, float *__restrict__ x, int hidden, int vocab) {
-    int id = ids[blockIdx.x];
-    id = id < 0 ? 0 : (id >= vocab ? vocab - 1 : id);
-    const uint16_t *row = table + (size_t)id * hidden;
-    for (int c = threadIdx.x; c < hidden; c += blockDim.x) x[(size_t)blockIdx.x * hidden + c] = bf16_to_f32(row[c]);
+__global__ void plan_embed_kernel(EmbedTables e, StepView v, const int *__restrict__ ids, const int *__restrict__ last_token, float *__restrict__ x) {
+    const int t = blockIdx.x, seg = v.tok_seg[t];
+    const int prev = v.tok_pos[t] == 0 ? -1 : t > v.seg_off[seg] ? ids[t - 1] : last_token[v.seg_row[seg]];
+    embed_token(e, ids[t], v.tok_pos[t] == 0, prev, x + (size_t)t * e.hidden);
+}
+
+__global__ __launch_bounds__(256) void plan_softcap_kernel(float *z, size_t n, float cap) {
+    const size_t i = (size_t)blockIdx.x * 256 + threadIdx.x;
+    if (i < n) z[i] = cap * tanhf(z[i] / cap);
 }
 
 template <int NT>
@@ -39,7 +43,7 @@ __global__ __launch_bounds__(NT) void plan_norm_kernel(PlanNormArgs p) {
         const bool in = col < p.hidden;
         x[c] = in ? *(const f32x4 *)(xr + col) : zero;
         y[c] = in && p.y ? *(const f32x4 *)(p.y + (size_t)t * p.hidden + col) : zero;
-        wpost[c] = in && p.y ? *(const f32x4 *)(p.post + col) : zero;
+        wpost[c] = in && p.post ? *(const f32x4 *)(p.post + col) : zero;
         wpre[c] = in && p.pre.w && !p.pre.b ? *(const f32x4 *)(p.pre.w + col) : zero;
     }
     if (p.table) {
@@ -60,6 +64,9 @@ __global__ __launch_bounds__(NT) void plan_norm_kernel(PlanNormArgs p) {
             const f32x4 emb = {u2f(e.x << 16), u2f(e.x & 0xFFFF0000u), u2f(e.y << 16), u2f(e.y & 0xFFFF0000u)};
             x[c] = (x[c] + y[c] * r * wpost[c]) + emb;
         }
+    } else if (p.y && !p.post) {
+#pragma unroll
+        for (int c = 0; c < CH; ++c) x[c] = x[c] + y[c] * p.mul;
     } else if (p.y) {
         float sq = 0.0f;
 #pragma unroll
@@ -154,14 +161,23 @@ int launch_norm(const PlanNormArgs &p, int T, hipStream_t st) {
 
 } // namespace
 
-int plan_embed(const uint16_t *table, const int *ids, float *x, int T, int hidden, int vocab, hipStream_t st) {
-    hipLaunchKernelGGL(plan_embed_kernel, dim3(T), dim3(256), 0, st, table, ids, x, hidden, vocab);
+int plan_embed(const EmbedTables &e, const StepView &v, const int *ids, const int *last_token, float *x, hipStream_t st) {
+    hipLaunchKernelGGL(plan_embed_kernel, dim3(v.T), dim3(256), 0, st, e, v, ids, last_token, x);
+    XFT_CHECK_HIP(hipGetLastError());
+    return 0;
+}
+
+int plan_softcap(float *logits, size_t n, float cap, hipStream_t st) {
+    XFT_REQUIRE(n > 0 && cap > 0.0f, "plan_softcap: bad argument");
+    hipLaunchKernelGGL(plan_softcap_kernel, dim3((unsigned)((n + 255) / 256)), dim3(256), 0, st, logits, n, cap);
     XFT_CHECK_HIP(hipGetLastError());
     return 0;
 }
 
 int plan_norm(int act, const PlanNormArgs &p, int T, hipStream_t st) {
-    XFT_REQUIRE(T > 0 && p.x && p.hidden % 4 == 0 && p.width <= p.hidden && (!p.rows || (!p.y && !p.table)) && (!p.pre2.w || p.pre.b), "plan_norm: bad argument");
+    XFT_REQUIRE(T > 0 && p.x && p.hidden % 4 == 0 && p.width <= p.hidden && (!p.rows || (!p.y && !p.table)) && (!p.pre2.w || p.pre.b)
+                    && (!p.table || !p.y || p.post),
+            "plan_norm: bad argument");
     return act == XFTHIP_BF16 ? launch_norm<true>(p, T, st) : launch_norm<false>(p, T, st);
 }
 

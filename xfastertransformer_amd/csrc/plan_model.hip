@@ -9,7 +9,7 @@
 #include <map>
 
 #include "model_impl.h"
-#include "plan.h"
+#include "plan_dev.h"
 
 namespace xfthip {
 
@@ -43,24 +43,27 @@ struct Matrix { // [K][N] bf16, zero where nothing is placed
     }
 };
 
-__global__ void plan_decode_begin_kernel(const uint16_t *table, const int *dec_rows, const int *pos, const int *ids, float *x, int hidden, int vocab,
-        int *tok_seg, int *tok_pos, int *tok_ids, int *seg, int seg_cap, int *log, const int *step, int max_seq) {
-    const int b = blockIdx.x, row = dec_rows[b];
-    int id = ids[row], at = pos[row];
+__global__ void plan_decode_begin_kernel(EmbedTables e, const int *dec_rows, const int *pos, const int *ids, float *x, int *last_token, int *tok_seg,
+        int *tok_pos, int *tok_ids, int *seg, int seg_cap, int *log, const int *step, int max_seq) {
+    const int b = blockIdx.x, row = dec_rows[b], id = ids[row], prev = last_token[row];
+    int at = pos[row];
     at = at < 0 ? 0 : (at >= max_seq ? max_seq - 1 : at);
+    __syncthreads(); // (all have read the token before)
     if (threadIdx.x == 0) {
         log[(size_t)step[0] * gridDim.x + b] = id;
         tok_seg[b] = b, tok_pos[b] = at, tok_ids[b] = id;
         seg[b] = row, seg[seg_cap + b] = b, seg[2 * seg_cap + b] = 1, seg[3 * seg_cap + b] = at;
+        last_token[row] = id;
     }
-    id = id < 0 ? 0 : (id >= vocab ? vocab - 1 : id);
-    const uint16_t *src = table + (size_t)id * hidden;
-    for (int c = threadIdx.x; c < hidden; c += blockDim.x) x[(size_t)b * hidden + c] = bf16_to_f32(src[c]);
+    embed_token(e, id, at == 0, prev, x + (size_t)b * e.hidden);
 }
 
-__global__ void plan_set_pos_kernel(const int *seg, int seg_cap, int n, int *pos) {
+// behind a step: where its sequences stand, and the last token of each
+__global__ void plan_advance_kernel(const int *seg, int seg_cap, int n, const int *ids, int *pos, int *last_token) {
     const int b = blockIdx.x * blockDim.x + threadIdx.x;
-    if (b < n) pos[seg[b]] = seg[3 * seg_cap + b] + seg[2 * seg_cap + b];
+    if (b >= n) return;
+    pos[seg[b]] = seg[3 * seg_cap + b] + seg[2 * seg_cap + b];
+    last_token[seg[b]] = ids[seg[seg_cap + b] + seg[2 * seg_cap + b] - 1];
 }
 
 __global__ void plan_fill_kernel(int *p, int n, int v) {
@@ -96,14 +99,20 @@ int rotation_tables(const xfthip_plan_layer &s, int positions, float **cosT, flo
     return 0;
 }
 
-int plan_gemm(xfthip_model *m, xfthip_weight_t w, int M, const void *A, int lda, void *C, int ldc, int c_dtype, hipStream_t st) {
+int plan_gemm(xfthip_model *m, xfthip_weight_t w, int M, const void *A, int lda, void *C, int ldc, int c_dtype, hipStream_t st, const float *bias = nullptr) {
     // (few rows against few columns: the form with the most waves along K)
     if (m->plan->act == XFTHIP_F32 || (M <= 32 && w->pw.N <= 256 && w->pw.K >= 1024)) {
         TileGemmArgs a;
-        a.M = M, a.A = A, a.lda = lda, a.C = C, a.ldc = ldc, a.c_dtype = c_dtype;
+        a.M = M, a.A = A, a.lda = lda, a.C = C, a.ldc = ldc, a.c_dtype = c_dtype, a.bias = bias;
         return tile_gemm(w, m->plan->act, a, st);
     }
-    return xfthip_gemm(w, M, A, lda, C, ldc, c_dtype, XFTHIP_EPI_NONE, nullptr, nullptr, 0, XFTHIP_F32, 1.0f, st);
+    return xfthip_gemm(w, M, A, lda, C, ldc, c_dtype, bias ? XFTHIP_EPI_BIAS : XFTHIP_EPI_NONE, bias, nullptr, 0, XFTHIP_F32, 1.0f, st);
+}
+
+// the product in front of a layer's mixers -> a
+int plan_gemm_in(xfthip_model *m, const PlanLayer &L, int T, hipStream_t st) {
+    const PlanState &p = *m->plan;
+    return plan_gemm(m, L.in, T, p.xn, m->cfg.hidden, p.a, L.in_ld, p.act, st, L.in_bias);
 }
 
 // a sublayer's last product: into y, or, in parallel blocks, added to the residual
@@ -128,11 +137,11 @@ int plan_gemm_heads(int act, xfthip_weight_t w, int M, const void *A, int lda, i
 
 int run_latent(xfthip_model *m, const PlanLayer &L, int run, const StepView &v, hipStream_t st) {
     PlanState &p = *m->plan;
-    const int T = v.T, H = L.s.heads, act = p.act, hidden = m->cfg.hidden;
+    const int T = v.T, H = L.s.heads, act = p.act;
     const int qcols = H * (L.D + L.RD);
     const LatentCacheView cache = {p.cache[run], L.R, L.RD};
     int rc;
-    if ((rc = plan_gemm(m, L.in, T, p.xn, hidden, p.a, L.row_in(), act, st))) return rc;
+    if ((rc = plan_gemm_in(m, L, T, st))) return rc;
     if ((rc = latent_prepare(act, L, v, p.a, p.cq, cache, m->cfg.rms_eps, st))) return rc;
     if ((rc = plan_gemm(m, L.uq, T, p.cq, L.QR, p.q, qcols, act, st))) return rc;
     if ((rc = latent_rotate_q(act, L, v, p.q, st))) return rc;
@@ -177,35 +186,64 @@ int run_latent(xfthip_model *m, const PlanLayer &L, int run, const StepView &v, 
     return plan_gemm_out(m, L.o, T, p.ov, H * L.V, st);
 }
 
-int run_delta(xfthip_model *m, const PlanLayer &L, int run, const StepView &v, hipStream_t st) {
+int mix_delta(xfthip_model *m, const PlanLayer &L, int store, const StepView &v, hipStream_t st) {
     PlanState &p = *m->plan;
-    const int T = v.T, act = p.act, hidden = m->cfg.hidden, ld = L.row_in();
+    const int act = p.act;
     int rc;
-    const DeltaBuffers b = {p.a, p.gates, p.dq, p.dk, p.dqk, p.dg, p.dv, p.dbeta, p.do_, p.on, p.state[run], p.conv_state[run]};
-    if ((rc = plan_gemm(m, L.in, T, p.xn, hidden, p.a, ld, act, st))) return rc;
-    const int first = L.channels() + L.beta_cols();
-    if ((rc = plan_gemm_heads(act, L.gates, T, (const char *)p.a + (size_t)first * p.esz, ld, L.gcols, L.rank, p.gates, 2 * L.gcols, XFTHIP_F32, st))) return rc;
+    const DeltaBuffers b = {p.a, p.gates, p.dq, p.dk, p.dqk, p.dg, p.dv, p.dbeta, p.do_, p.ov, p.state[store], p.conv_state[store]};
+    if (L.gates) {
+        const int first = L.in_col + L.channels() + L.beta_cols();
+        if ((rc = plan_gemm_heads(act, L.gates, v.T, (const char *)p.a + (size_t)first * p.esz, L.in_ld, L.gcols, L.rank, p.gates, 2 * L.gcols, XFTHIP_F32, st)))
+            return rc;
+    }
     if ((rc = delta_prepare(act, L, v, b, st))) return rc;
     if ((rc = delta_scan(L, v, b, st))) return rc;
-    if ((rc = delta_output(act, L, v, b, m->cfg.rms_eps, st))) return rc;
-    return plan_gemm_out(m, L.o, T, p.on, L.s.heads * L.VD, st);
+    return delta_output(act, L, v, b, m->cfg.rms_eps, st);
 }
 
-int run_grouped(xfthip_model *m, const PlanLayer &L, int run, const StepView &v, hipStream_t st) {
+int mix_grouped(xfthip_model *m, const PlanLayer &L, int store, const StepView &v, hipStream_t st) {
     PlanState &p = *m->plan;
-    const int T = v.T, act = p.act;
     int rc;
-    const GroupedBuffers b = {p.a, p.q, p.cache[run], p.first_values};
-    if ((rc = plan_gemm(m, L.in, T, p.xn, m->cfg.hidden, p.a, L.row_in(), act, st))) return rc;
-    if ((rc = grouped_prepare(act, L, v, b, m->cfg.rms_eps, st))) return rc;
-    if ((rc = grouped_attention(act, L, v, p.q, p.cache[run], p.ov, m->len_hint, p.part, p.part_floats, st))) return rc;
-    return plan_gemm_out(m, L.o, T, p.ov, L.s.heads * L.V, st);
+    const GroupedBuffers b = {p.a, p.q, p.cache[p.reads[store]], p.first_values};
+    if ((rc = grouped_prepare(p.act, L, v, b, m->cfg.rms_eps, st))) return rc;
+    return grouped_attention(p.act, L, v, b, p.ov, m->len_hint, p.part, p.part_floats, st);
+}
+
+int mix_unit(xfthip_model *m, const PlanLayer &L, int store, const StepView &v, hipStream_t st) {
+    PlanState &p = *m->plan;
+    int rc;
+    const UnitBuffers b = {p.a, p.u, p.gates, p.carry, p.ov, p.state[store], p.conv_state[store]};
+    if ((rc = unit_filter(p.act, L, v, b, st))) return rc;
+    if ((rc = plan_gemm_heads(p.act, L.gates, v.T, p.u, L.channels(), 2 * L.D, L.D, p.gates, 2 * L.channels(), XFTHIP_F32, st))) return rc;
+    return unit_scan(p.act, L, v, b, st);
+}
+
+// between the input and the output product of a mixer
+int mix(xfthip_model *m, const PlanLayer &L, int store, const StepView &v, hipStream_t st) {
+    switch (L.s.mixer) {
+        case XFTHIP_MIXER_GROUPED: return mix_grouped(m, L, store, v, st);
+        case XFTHIP_MIXER_UNIT: return mix_unit(m, L, store, v, st);
+        default: return mix_delta(m, L, store, v, st);
+    }
+}
+
+int run_mixers(xfthip_model *m, int run, const StepView &v, hipStream_t st) {
+    PlanState &p = *m->plan;
+    const LayerRun &r = p.plan->runs[run];
+    const PlanLayer &L = p.layers[r.layer];
+    if (L.s.mixer == XFTHIP_MIXER_LATENT) return run_latent(m, L, run, v, st);
+    int rc;
+    if ((rc = plan_gemm_in(m, L, v.T, st))) return rc;
+    if ((rc = mix(m, L, run, v, st))) return rc;
+    if (r.beside >= 0 && (rc = mix(m, p.layers[r.beside], r.beside_store, v, st))) return rc;
+    return plan_gemm_out(m, L.o, v.T, p.ov, L.out_ld, st);
 }
 
 // gate and up projections of a dense or shared feed-forward, combined -> h
 int run_gateup(xfthip_model *m, const PlanLayer &L, int T, const void *in, hipStream_t st) {
     PlanState &p = *m->plan;
     const int hidden = m->cfg.hidden;
+    if (p.act != XFTHIP_F32 && L.s.glu_alpha == 0.0f) return xfthip_gemm_gateup_silu(L.gateup, T, in, hidden, p.h, L.ff, XFTHIP_BF16, st);
     if (p.act != XFTHIP_F32) return xfthip_gemm_gateup_clamped(L.gateup, T, in, hidden, p.h, L.ff, XFTHIP_BF16, L.s.glu_limit, L.s.glu_alpha, st);
     TileGemmArgs a;
     a.M = T, a.A = in, a.lda = hidden, a.C = p.h, a.ldc = L.ff, a.c_dtype = XFTHIP_F32, a.glu = true, a.glu_limit = L.s.glu_limit, a.glu_alpha = L.s.glu_alpha;
@@ -249,8 +287,10 @@ int run_feed_forward(xfthip_model *m, const PlanLayer &L, int T, const void *in,
     float *dst = parallel ? m->x : p.y;
     if (L.s.experts > 0) {
         const int ld = pad32(L.routes());
+        const RouteRule rule = {L.s.experts, L.routes(), L.s.top, L.correction, L.s.router == XFTHIP_ROUTE_SIGMOID_GROUPS ? L.s.route_groups : 0, L.s.route_keep,
+                L.s.route_scale};
         if ((rc = plan_gemm(m, L.router, T, in, hidden, p.router_logits, ld, XFTHIP_F32, st))) return rc;
-        if ((rc = route_tokens(p.router_logits, ld, L.correction, T, L.s.experts, L.routes(), L.s.top, p.route, st))) return rc;
+        if ((rc = route_tokens(p.router_logits, ld, rule, T, p.route, st))) return rc;
         if ((rc = run_experts(m, L, T, in, st))) return rc;
         return combine_experts(p.act, parallel || L.ff > 0 ? dst : nullptr, p.expert_out, in, L.s.top, p.route, dst, narrow, T, hidden, st);
     }
@@ -286,7 +326,7 @@ int plan_layers(xfthip_model *m, const StepView &v, hipStream_t st) {
     // next: the layer whose first norms follow, or null
     auto norm = [&](const float *y, const float *post, bool again, const PlanNorm &pre, const PlanNorm &pre2) {
         const PlanNormArgs a = {m->x, y, post, again ? plan.embedding : nullptr, p.ids, m->cfg.vocab, pre, pre2, p.xn, p.xn2, nullptr, hidden, plan.cfg.hidden,
-                m->cfg.rms_eps};
+                m->cfg.rms_eps, plan.cfg.residual_mult};
         return plan_norm(p.act, a, T, st);
     };
     const PlanNorm none;
@@ -300,12 +340,7 @@ int plan_layers(xfthip_model *m, const StepView &v, hipStream_t st) {
         // (a traced run keeps the embedding of a further pass apart, so that the trace shows the layer's own result)
         const bool again = !last && plan.runs[r + 1].add_embedding, join = again && !p.trace;
         const PlanLayer *next = last ? nullptr : &p.layers[plan.runs[r + 1].layer], *then = p.trace ? nullptr : next;
-        switch (L.s.mixer) {
-            case XFTHIP_MIXER_LATENT: rc = run_latent(m, L, r, v, st); break;
-            case XFTHIP_MIXER_GROUPED: rc = run_grouped(m, L, r, v, st); break;
-            default: rc = run_delta(m, L, r, v, st);
-        }
-        if (rc) return rc;
+        if ((rc = run_mixers(m, r, v, st))) return rc;
         const bool ff = L.feeds_forward(), side = plan.cfg.side_dim > 0;
         const void *narrow = p.act == XFTHIP_F32 ? (const void *)m->x : p.narrow; // what the side embedding's gate reads
         void *narrow_out = side && p.act != XFTHIP_F32 ? p.narrow : nullptr;
@@ -341,6 +376,12 @@ StepView view_of(const xfthip_model *m, int B, int T, int longest) {
     const PlanState &p = *m->plan;
     const int cap = p.slots;
     return StepView {B, T, longest, p.tok_seg, p.tok_pos, p.seg, p.seg + cap, p.seg + 2 * cap, p.seg + 3 * cap, p.table, p.table_stride};
+}
+
+EmbedTables embed_tables(const xfthip_model *m) {
+    const xfthip_plan &plan = *m->plan->plan;
+    const xfthip_plan_config &c = plan.cfg;
+    return EmbedTables {plan.embedding, plan.pair_embedding, m->cfg.hidden, m->cfg.vocab, c.embed_scale, c.bigram_buckets, c.bigram_mul_prev, c.bigram_mul_cur};
 }
 
 } // namespace
@@ -401,7 +442,8 @@ int plan_run(xfthip_model *m, int n, const int *rows, const int *lens, const int
     XFT_CHECK_HIP(hipMemcpyAsync(p.tok_pos, hp, (size_t)T * 4, hipMemcpyHostToDevice, st));
     XFT_CHECK_HIP(hipMemcpyAsync(p.ids, hi, (size_t)T * 4, hipMemcpyHostToDevice, st));
     XFT_CHECK_HIP(hipMemcpyAsync(p.seg, hg, (size_t)4 * cap * 4, hipMemcpyHostToDevice, st));
-    if (int rc = plan_embed(p.plan->embedding, p.ids, m->x, (int)T, c.hidden, c.vocab, st)) return rc;
+    const StepView view = view_of(m, n, (int)T, longest);
+    if (int rc = plan_embed(embed_tables(m), view, p.ids, p.last_token, m->x, st)) return rc;
     m->len_hint = deepest;
     if (p.trace) {
         const size_t need = p.plan->runs.size() * (size_t)T * c.hidden;
@@ -414,8 +456,8 @@ int plan_run(xfthip_model *m, int n, const int *rows, const int *lens, const int
         }
         p.trace_tokens = (int)T;
     }
-    if (int rc = plan_layers(m, view_of(m, n, (int)T, longest), st)) return rc;
-    hipLaunchKernelGGL(plan_set_pos_kernel, dim3((n + 63) / 64), dim3(64), 0, st, p.seg, cap, n, m->pos);
+    if (int rc = plan_layers(m, view, st)) return rc;
+    hipLaunchKernelGGL(plan_advance_kernel, dim3((n + 63) / 64), dim3(64), 0, st, p.seg, cap, n, p.ids, m->pos, p.last_token);
     XFT_CHECK_HIP(hipGetLastError());
     for (int i = 0; i < n; ++i) m->row_pos[rows[i]] = std::max(m->row_pos[rows[i]], 0) + lens[i];
     return 0;
@@ -425,9 +467,11 @@ int plan_head(xfthip_model *m, const int *rows_dev, int n, int at, hipStream_t s
     PlanState &p = *m->plan;
     const xfthip_plan &plan = *p.plan;
     const xfthip_model_config &c = m->cfg;
-    const PlanNormArgs a = {m->x, nullptr, nullptr, nullptr, nullptr, c.vocab, plan.final_norm, {}, p.xn, nullptr, rows_dev, c.hidden, plan.cfg.hidden, c.rms_eps};
+    const PlanNormArgs a = {m->x, nullptr, nullptr, nullptr, nullptr, c.vocab, plan.final_norm, {}, p.xn, nullptr, rows_dev, c.hidden, plan.cfg.hidden, c.rms_eps, 0.0f};
     if (int rc = plan_norm(p.act, a, n, st)) return rc;
-    return plan_gemm(m, plan.head, n, p.xn, c.hidden, m->logits + (size_t)at * c.vocab, c.vocab, XFTHIP_F32, st);
+    float *logits = m->logits + (size_t)at * c.vocab;
+    if (int rc = plan_gemm(m, plan.head, n, p.xn, c.hidden, logits, c.vocab, XFTHIP_F32, st)) return rc;
+    return plan.cfg.logit_softcap > 0.0f ? plan_softcap(logits, (size_t)n * c.vocab, plan.cfg.logit_softcap, st) : 0;
 }
 
 int plan_logits(xfthip_model *m, const int *list, int n, float *logits_host, hipStream_t st) {
@@ -479,7 +523,7 @@ int plan_decode_begin(xfthip_model *m, int steps, hipStream_t st) {
 int plan_decode_step(xfthip_model *m, int B, hipStream_t st) {
     PlanState &p = *m->plan;
     const xfthip_model_config &c = m->cfg;
-    hipLaunchKernelGGL(plan_decode_begin_kernel, dim3(B), dim3(256), 0, st, p.plan->embedding, p.dec_rows, m->pos, m->ids, m->x, c.hidden, c.vocab, p.tok_seg,
+    hipLaunchKernelGGL(plan_decode_begin_kernel, dim3(B), dim3(256), 0, st, embed_tables(m), p.dec_rows, m->pos, m->ids, m->x, p.last_token, p.tok_seg,
             p.tok_pos, p.ids, p.seg, p.slots, m->idlog, m->step, c.max_seq);
     XFT_CHECK_HIP(hipGetLastError());
     const bool trace = p.trace;
@@ -518,14 +562,15 @@ int plan_reorder(xfthip_model *m, const int *dst, const int *src, int n, hipStre
     }
     // (a slot whose pages another one reads keeps them: it is a destination itself only if it is listed, with as many or more pages)
     size_t bytes = 0;
-    for (size_t r = 0; r < p.plan->runs.size(); ++r) {
-        const PlanLayer &L = p.layers[p.plan->runs[r].layer];
+    const size_t stores = p.store_layer.size();
+    for (size_t r = 0; r < stores; ++r) {
+        const PlanLayer &L = p.layers[p.store_layer[r]];
         size_t need = 0;
         for (int i = 0; i < n; ++i)
-            need += L.paged() ? from[i].size() * kPageTokens * L.token_elems() * p.esz
-                              : ((size_t)L.s.heads * L.VD * L.KD * 4 + (size_t)(L.s.taps - 1) * L.channels() * p.esz);
+            need += L.paged() ? from[i].size() * kPageTokens * L.token_elems() * p.esz : L.state_floats() * 4 + (size_t)(L.s.taps - 1) * L.channels() * p.esz;
         bytes = std::max(bytes, need);
     }
+    bytes = std::max(bytes, (size_t)n * 4);
     char *stage = nullptr;
     XFT_CHECK_HIP(hipMalloc((void **)&stage, bytes + 16));
     int rc = 0;
@@ -535,8 +580,14 @@ int plan_reorder(xfthip_model *m, const int *dst, const int *src, int n, hipStre
     auto copy = [&](void *d, const void *s, size_t b) {
         if (e == hipSuccess && b) e = hipMemcpyAsync(d, s, b, hipMemcpyDeviceToDevice, st);
     };
-    for (size_t r = 0; r < p.plan->runs.size() && rc == 0; ++r) {
-        const PlanLayer &L = p.layers[p.plan->runs[r].layer];
+    for (int write = 0; write < 2 && rc == 0; ++write)
+        for (int i = 0; i < n; ++i) {
+            if (write) copy(p.last_token + dst[i], stage + 4 * (size_t)i, 4);
+            else copy(stage + 4 * (size_t)i, p.last_token + src[i], 4);
+        }
+    for (size_t r = 0; r < stores && rc == 0; ++r) {
+        const PlanLayer &L = p.layers[p.store_layer[r]];
+        if (L.kv_from >= 0) continue; // (what it reads is another record's)
         for (int write = 0; write < 2; ++write) {
             size_t at = 0;
             for (int i = 0; i < n; ++i) {
@@ -548,7 +599,7 @@ int plan_reorder(xfthip_model *m, const int *dst, const int *src, int n, hipStre
                         else copy(stage + at, pool + (size_t)from[i][k] * page, page);
                     }
                 } else {
-                    const size_t sb = (size_t)L.s.heads * L.VD * L.KD * 4, cb = (size_t)(L.s.taps - 1) * L.channels() * p.esz;
+                    const size_t sb = L.state_floats() * 4, cb = (size_t)(L.s.taps - 1) * L.channels() * p.esz;
                     char *state = (char *)p.state[r], *conv = (char *)p.conv_state[r];
                     if (write) {
                         copy(state + dst[i] * sb, stage + at, sb);
@@ -589,12 +640,16 @@ int xfthip_plan_create(const xfthip_plan_config *cfg, const xfthip_plan_layer *l
     XFT_REQUIRE(c.layers > 0 && c.hidden > 0 && c.hidden <= 16384 && c.vocab > 0, "xfthip_plan_create: bad sizes");
     const bool loop = c.loop_times > 1 && c.loop_start != c.loop_stop; // (a loop over nothing is none)
     XFT_REQUIRE((c.block == XFTHIP_BLOCK_SANDWICH && c.norm == XFTHIP_NORM_RMS_ABOUT_ONE && c.side_dim == 0)
-                    || (c.block == XFTHIP_BLOCK_PARALLEL && c.norm == XFTHIP_NORM_DYNAMIC_TANH && c.side_dim >= 0),
+                    || (c.block == XFTHIP_BLOCK_PARALLEL && c.norm == XFTHIP_NORM_DYNAMIC_TANH && c.side_dim >= 0)
+                    || (c.block == XFTHIP_BLOCK_SERIAL && c.norm == XFTHIP_NORM_RMS && c.side_dim == 0 && !loop),
             "xfthip_plan_create: block arrangement %d with norm %d and side width %d is not served", c.block, c.norm, c.side_dim);
     XFT_REQUIRE(!loop || (c.loop_start >= 0 && c.loop_start < c.loop_stop && c.loop_stop <= c.layers), "xfthip_plan_create: loop over layers %d .. %d of %d",
             c.loop_start, c.loop_stop, c.layers);
+    XFT_REQUIRE(c.bigram_buckets >= 0 && c.bigram_buckets < (1ll << 31) - 1 && (c.embed_scale == 0.0f || c.embed_scale == 1.0f || !loop) && c.logit_softcap >= 0.0f,
+            "xfthip_plan_create: bad embedding or logit constants");
     xfthip_plan *p = new xfthip_plan();
     p->cfg = c;
+    if (c.embed_scale == 0.0f) p->cfg.embed_scale = 1.0f;
     p->hidden = pad32(c.hidden);
     p->side_pad = pad32(c.side_dim);
     int first_mix = -1; // the first layer with mixed values
@@ -607,15 +662,17 @@ int xfthip_plan_create(const xfthip_plan_config *cfg, const xfthip_plan_layer *l
             ok = ok && s.rot_dim > 0 && s.rot_dim % 2 == 0 && s.kv_rank > 0 && s.kv_rank <= 1024 && s.q_rank > 0 && s.window >= 0;
             L.D = pad32(s.dim), L.RD = pad32(s.rot_dim), L.V = pad32(s.vdim), L.R = pad32(s.kv_rank), L.QR = pad32(s.q_rank);
         } else if (s.mixer == XFTHIP_MIXER_DELTA) {
-            ok = ok && s.kv_heads > 0 && s.heads % s.kv_heads == 0 && s.dim <= 256 && s.taps >= 1 && s.decay_rank > 0 && s.gate_rank > 0;
+            ok = ok && s.kv_heads > 0 && s.heads % s.kv_heads == 0 && s.dim <= 256 && s.taps >= 1 && s.decay_rank >= 0 && s.gate_rank >= 0
+                    && (s.decay_rank > 0) == (s.gate_rank > 0);
             L.KD = 32;
             while (L.KD < s.dim) L.KD *= 2;
             L.VD = pad32(s.vdim);
             L.rank = pad32(std::max(s.decay_rank, s.gate_rank));
-            L.gcols = s.heads * std::max(L.KD, L.VD);
+            if (L.rank > 0) L.gcols = s.heads * std::max(L.KD, L.VD);
         } else if (s.mixer == XFTHIP_MIXER_GROUPED) {
             ok = ok && s.kv_heads > 0 && s.heads % s.kv_heads == 0 && s.dim <= 512 && s.vdim <= 512 && s.rot_dim >= 0 && s.rot_dim <= s.dim && s.rot_dim % 2 == 0
-                    && s.window >= 0 && (s.rot_factor <= 0.0 || (s.rot_original > 0.0 && s.rot_fast > 0.0 && s.rot_slow > 0.0));
+                    && s.window >= 0 && s.chunk >= 0 && !(s.window > 0 && s.chunk > 0) && s.softcap >= 0.0f && s.qk_norm >= 0 && s.qk_norm <= XFTHIP_QK_NORM_ALL
+                    && s.out_gate >= 0 && s.out_gate <= XFTHIP_GATE_HEAD && (!s.key_values || (s.dim == s.vdim && !s.v_mix)) && (s.rot_factor <= 0.0 || (s.rot_original > 0.0 && s.rot_fast > 0.0 && s.rot_slow > 0.0));
             L.D = pad32(s.dim), L.V = pad32(s.vdim);
             if (ok && s.v_mix) {
                 L.first_values = first_mix < 0;
@@ -623,13 +680,38 @@ int xfthip_plan_create(const xfthip_plan_config *cfg, const xfthip_plan_layer *l
                 const xfthip_plan_layer &f = layers[first_mix];
                 ok = f.kv_heads == s.kv_heads && f.vdim == s.vdim; // values of the same shape
             }
+            if (ok && s.kv_from != 0) { // a record before this one with keys and values of its own and of the same shape
+                ok = s.kv_from > 0 && s.kv_from <= i && !loop && !s.v_mix;
+                const xfthip_plan_layer &f = layers[ok ? s.kv_from - 1 : 0];
+                ok = ok && f.mixer == XFTHIP_MIXER_GROUPED && f.kv_from == 0 && f.kv_heads == s.kv_heads && f.dim == s.dim && f.vdim == s.vdim;
+                if (ok) L.kv_from = s.kv_from - 1;
+            }
+        } else if (s.mixer == XFTHIP_MIXER_UNIT) {
+            ok = ok && s.taps >= 1;
+            L.D = pad32(s.dim);
         } else {
             ok = false;
         }
         L.ff = pad32(s.inter);
         if (s.experts > 0) {
-            ok = ok && s.identity >= 0 && s.top > 0 && s.top <= L.routes() && s.top <= 64 && L.routes() <= 1024 && s.expert_inter > 0 && s.glu_alpha > 0.0f;
+            ok = ok && s.identity >= 0 && s.top > 0 && s.top <= L.routes() && s.top <= 64 && L.routes() <= 1024 && s.expert_inter > 0 && s.glu_alpha >= 0.0f;
+            if (ok && s.router == XFTHIP_ROUTE_SIGMOID_GROUPS)
+                ok = s.identity == 0 && s.route_groups > 0 && s.experts % s.route_groups == 0 && s.route_keep > 0 && s.route_keep <= s.route_groups
+                        && s.top <= s.route_keep * (s.experts / s.route_groups);
+            else ok = ok && s.router == XFTHIP_ROUTE_SOFTMAX;
             L.eff = pad32(s.expert_inter);
+        }
+        if (s.scaled) L.mix_scale = s.mix_scale;
+        L.in_ld = L.row_in(), L.out_ld = L.out_cols();
+        if (s.beside) { // joins the layer before it, whose projections it continues
+            ok = ok && i > 0 && !loop && !layers[i - 1].beside && layers[i - 1].mixer != XFTHIP_MIXER_LATENT && s.mixer != XFTHIP_MIXER_LATENT && s.inter == 0
+                    && s.experts == 0;
+            if (ok) {
+                PlanLayer &f = p->layers[i - 1];
+                f.beside = i;
+                L.in_col = f.in_ld, L.out_col = f.out_ld;
+                f.in_ld = L.in_ld += f.in_ld, f.out_ld = L.out_ld += f.out_ld;
+            }
         }
         if (!ok) {
             delete p;
@@ -638,13 +720,17 @@ int xfthip_plan_create(const xfthip_plan_config *cfg, const xfthip_plan_layer *l
         p->layers.push_back(L);
     }
     auto add = [&](int from, int to, bool again) {
-        for (int i = from; i < to; ++i) p->runs.push_back({i, again && i == from});
+        for (int i = from; i < to; ++i)
+            if (!p->layers[i].s.beside) p->runs.push_back({i, again && i == from, p->layers[i].beside});
     };
     add(0, loop ? c.loop_start : c.layers, false);
     if (loop) {
         for (int t = 0; t < c.loop_times; ++t) add(c.loop_start, c.loop_stop, t > 0);
         add(c.loop_stop, c.layers, false);
     }
+    int stores = (int)p->runs.size();
+    for (LayerRun &r : p->runs)
+        if (r.beside >= 0) r.beside_store = stores++;
     *out = p;
     return 0;
 }
@@ -656,13 +742,13 @@ int xfthip_plan_destroy(xfthip_plan_t p) {
         for (auto *list : {&L.egateup, &L.edown})
             for (xfthip_weight_t w : *list) xfthip_weight_destroy(w);
         for (float *f : {L.q_norm, L.kv_norm, L.sink, L.conv, L.decay, L.dt_bias, L.out_norm, L.pre1.w, L.pre1.b, L.pre2.w, L.pre2.b, L.post1, L.post2, L.correction,
-                     L.side_post})
+                     L.side_post, L.in_bias, L.conv_bias, L.lambda, L.gate_bias})
             if (f) (void)hipFree(f);
         if (L.etable) (void)hipFree(L.etable);
     }
     xfthip_weight_destroy(p->head);
     if (p->embedding) (void)hipFree(p->embedding);
-    for (void *b : {(void *)p->final_norm.w, (void *)p->final_norm.b, (void *)p->side_embedding})
+    for (void *b : {(void *)p->final_norm.w, (void *)p->final_norm.b, (void *)p->side_embedding, (void *)p->pair_embedding})
         if (b) (void)hipFree(b);
     delete p;
     return 0;
@@ -737,13 +823,13 @@ int xfthip_plan_finish(xfthip_plan_t p) {
 #define NEED(var, name, r, c)                 \
     const Tensor &var = get(name, r, c);      \
     if (!missing.empty()) break
-    const bool tanh_norm = p->cfg.norm == XFTHIP_NORM_DYNAMIC_TANH, parallel = p->cfg.block == XFTHIP_BLOCK_PARALLEL;
+    const bool tanh_norm = p->cfg.norm == XFTHIP_NORM_DYNAMIC_TANH, sandwich = p->cfg.block == XFTHIP_BLOCK_SANDWICH;
     // a norm in front of something; mul multiplies its result
     auto front = [&](const std::string &name, float mul, PlanNorm *dst) {
         const Tensor &w = get(name.c_str(), W, 1);
         if (!missing.empty()) return;
         if (!tanh_norm) {
-            std::vector<float> v = one_plus(w, nullptr);
+            std::vector<float> v = p->cfg.norm == XFTHIP_NORM_RMS ? values(w, Wp) : one_plus(w, nullptr);
             for (float &f : v) f *= mul;
             upload(v, &dst->w);
             return;
@@ -768,10 +854,196 @@ int xfthip_plan_finish(xfthip_plan_t p) {
         w.place(t, 0, t.rows, 0, t.cols, 0, 0);
         pack(w, XFTHIP_WF_NONE, dst);
     };
+    // a mixer's part of the layer's two products, and its own tensors
+    auto mixer = [&](PlanLayer &L, Matrix &in, Matrix &mo, std::vector<float> &bias, bool &biased) {
+        const xfthip_plan_layer &s = L.s;
+        const int H = s.heads, c0 = L.in_col, r0 = L.out_col;
+        do {
+            if (s.mixer == XFTHIP_MIXER_LATENT) {
+                const int d = s.dim, r = s.rot_dim, dv = s.vdim, R = s.kv_rank;
+                NEED(dq, "mix.dq", s.q_rank, W);
+                NEED(dqn, "mix.dq.norm", s.q_rank, 1);
+                NEED(uq, "mix.uq", H * (d + r), s.q_rank);
+                NEED(dkv, "mix.dkv", R + r, W);
+                NEED(dkvn, "mix.dkv.norm", R, 1);
+                NEED(uk, "mix.uk", H * d, R);
+                NEED(uv, "mix.uv", H * dv, R);
+                NEED(o, "mix.o", W, H * dv);
+                in.place(dq, 0, s.q_rank, 0, W, 0, c0);
+                in.place(dkv, 0, R, 0, W, 0, c0 + L.QR);
+                in.place(dkv, R, r, 0, W, 0, c0 + L.QR + L.R);
+                Matrix mq(L.QR, H * (L.D + L.RD)), ma(L.D, H * L.R), mk(L.R, H * L.D), mv(L.R, H * L.V);
+                for (int h = 0; h < H; ++h) {
+                    mq.place(uq, h * (d + r), d, 0, s.q_rank, 0, h * (L.D + L.RD));
+                    mq.place(uq, h * (d + r) + d, r, 0, s.q_rank, 0, h * (L.D + L.RD) + L.D);
+                    ma.place_turned(uk, h * d, d, 0, R, 0, h * L.R);
+                    mk.place(uk, h * d, d, 0, R, 0, h * L.D);
+                    mv.place(uv, h * dv, dv, 0, R, 0, h * L.V);
+                    mo.place(o, 0, W, h * dv, dv, r0 + h * L.V, 0);
+                }
+                pack(mq, XFTHIP_WF_NONE, &L.uq);
+                pack(ma, XFTHIP_WF_NONE, &L.absorb);
+                pack(mk, XFTHIP_WF_NONE, &L.uk);
+                pack(mv, XFTHIP_WF_NONE, &L.uv);
+                upload(values(dqn, L.QR), &L.q_norm);
+                upload(values(dkvn, L.R), &L.kv_norm);
+                if (s.has_sink) {
+                    NEED(sink, "mix.sink", H, 1);
+                    upload(values(sink, H), &L.sink);
+                }
+            } else if (s.mixer == XFTHIP_MIXER_GROUPED) {
+                const int G = s.kv_heads, d = s.dim, dv = s.vdim, k0 = c0 + H * L.D, v0 = c0 + L.value_col(), g0 = c0 + L.gate_col();
+                const bool own = L.kv_from < 0;
+                // a projection of n heads of width w, each padded to `pad` columns from c on
+                auto project = [&](const char *name, int n, int w, int pad, int c, bool with_bias) {
+                    const Tensor &t = get(name, n * w, W);
+                    if (!missing.empty()) return;
+                    for (int h = 0; h < n; ++h) in.place(t, h * w, w, 0, W, 0, c + h * pad);
+                    if (!with_bias) return;
+                    const Tensor &b = get((std::string(name) + ".b").c_str(), n * w, 1);
+                    if (!missing.empty()) return;
+                    for (int x = 0; x < n * w; ++x) bias[c + x / w * pad + x % w] = bf16_value(b.data[x]);
+                    biased = true;
+                };
+                project("mix.q", H, d, L.D, c0, s.qkv_bias);
+                if (own) project("mix.k", G, d, L.D, k0, s.qkv_bias);
+                if (own && !s.key_values) project("mix.v", G, dv, L.V, v0, s.qkv_bias);
+                if (s.out_gate == XFTHIP_GATE_ELEMENT) project("mix.g", H, dv, L.V, g0, false);
+                if (s.out_gate == XFTHIP_GATE_HEAD) project("mix.g", H, 1, 1, g0, false);
+                NEED(o, "mix.o", W, H * dv);
+                for (int h = 0; h < H; ++h) mo.place(o, 0, W, h * dv, dv, r0 + h * L.V, 0);
+                if (s.qk_norm == XFTHIP_QK_NORM_HEAD) {
+                    NEED(qn, "mix.q.norm", d, 1);
+                    NEED(kn, "mix.k.norm", d, 1);
+                    upload(values(qn, L.D), &L.q_norm);
+                    upload(values(kn, L.D), &L.kv_norm);
+                } else if (s.qk_norm == XFTHIP_QK_NORM_ALL) {
+                    auto spread = [&](const Tensor &t, int n) {
+                        std::vector<float> v((size_t)n * L.D, 0.0f);
+                        for (int x = 0; x < n * d; ++x) v[(size_t)(x / d) * L.D + x % d] = bf16_value(t.data[x]);
+                        return v;
+                    };
+                    NEED(qn, "mix.q.norm", H * d, 1);
+                    upload(spread(qn, H), &L.q_norm);
+                    if (own) {
+                        NEED(kn, "mix.k.norm", G * d, 1);
+                        upload(spread(kn, G), &L.kv_norm);
+                    }
+                }
+                if (s.has_sink) {
+                    NEED(sink, "mix.sink", H, 1);
+                    upload(values(sink, H), &L.sink);
+                }
+                if (s.v_mix && !L.first_values) {
+                    NEED(share, "mix.vmix", 1, 1);
+                    L.value_share = bf16_value(share.data[0]);
+                }
+            } else if (s.mixer == XFTHIP_MIXER_UNIT) {
+                const int B = s.heads, d = s.dim, n = s.taps, C = B * d, P = B * L.D;
+                NEED(y, "mix.y", C, W);
+                NEED(yb, "mix.y.b", C, 1);
+                NEED(x, "mix.x", C, W);
+                NEED(xb, "mix.x.b", C, 1);
+                NEED(cv, "mix.conv", C, n);
+                NEED(cb, "mix.conv.b", C, 1);
+                NEED(ra, "mix.ra", B, d * d);
+                NEED(rab, "mix.ra.b", B, d);
+                NEED(ri, "mix.ri", B, d * d);
+                NEED(rib, "mix.ri.b", B, d);
+                NEED(lam, "mix.lam", C, 1);
+                NEED(o, "mix.o", W, C);
+                std::vector<float> conv((size_t)P * n, 0.0f), conv_bias(P, 0.0f), lambda(P, 0.0f), gate_bias((size_t)2 * P, 0.0f);
+                Matrix gt(L.D, 2 * P);
+                for (int b = 0; b < B; ++b) {
+                    in.place(y, b * d, d, 0, W, 0, c0 + b * L.D);
+                    in.place(x, b * d, d, 0, W, 0, c0 + P + b * L.D);
+                    mo.place(o, 0, W, b * d, d, r0 + b * L.D, 0);
+                    for (int e = 0; e < d; ++e) {
+                        const int from = b * d + e, to = b * L.D + e;
+                        bias[c0 + to] = bf16_value(yb.data[from]), bias[c0 + P + to] = bf16_value(xb.data[from]);
+                        for (int k = 0; k < n; ++k) conv[(size_t)to * n + k] = bf16_value(cv.data[(size_t)from * n + k]);
+                        conv_bias[to] = bf16_value(cb.data[from]);
+                        const double z = bf16_value(lam.data[from]);
+                        lambda[to] = (float)(8.0 * (z > 0.0 ? z + log1p(exp(-z)) : log1p(exp(z))));
+                        gate_bias[(size_t)2 * b * L.D + e] = bf16_value(rab.data[from]), gate_bias[(size_t)(2 * b + 1) * L.D + e] = bf16_value(rib.data[from]);
+                        for (int k = 0; k < d; ++k) { // (square matrices [out, in])
+                            gt.w[(size_t)k * gt.N + 2 * b * L.D + e] = ra.data[((size_t)b * d + e) * d + k];
+                            gt.w[(size_t)k * gt.N + (2 * b + 1) * L.D + e] = ri.data[((size_t)b * d + e) * d + k];
+                        }
+                    }
+                }
+                biased = true;
+                pack(gt, XFTHIP_WF_NONE, &L.gates);
+                upload(conv, &L.conv), upload(conv_bias, &L.conv_bias), upload(lambda, &L.lambda), upload(gate_bias, &L.gate_bias);
+            } else {
+                const int KH = s.kv_heads, d = s.dim, dv = s.vdim, n = s.taps;
+                NEED(q, "mix.q", KH * d, W);
+                NEED(k, "mix.k", KH * d, W);
+                NEED(v, "mix.v", H * dv, W);
+                NEED(qc, "mix.q.conv", KH * d, n);
+                NEED(kc, "mix.k.conv", KH * d, n);
+                NEED(vc, "mix.v.conv", H * dv, n);
+                NEED(b, "mix.b", H, W);
+                NEED(al, "mix.A_log", H, 1);
+                NEED(nm, "mix.norm", dv, 1);
+                NEED(o, "mix.o", W, H * dv);
+                std::vector<float> conv((size_t)L.channels() * n, 0.0f), dec(H);
+                const int k0 = KH * L.KD, v0 = 2 * KH * L.KD, b0 = c0 + L.channels(), a0 = b0 + L.beta_cols(), g0 = a0 + (L.head_decay() ? L.beta_cols() : L.rank);
+                auto filters = [&](const Tensor &t, int from, int count, int to) {
+                    for (int i2 = 0; i2 < count * n; ++i2) conv[(size_t)to * n + i2] = bf16_value(t.data[(size_t)from * n + i2]);
+                };
+                for (int h = 0; h < KH; ++h) {
+                    in.place(q, h * d, d, 0, W, 0, c0 + h * L.KD);
+                    in.place(k, h * d, d, 0, W, 0, c0 + k0 + h * L.KD);
+                    filters(qc, h * d, d, h * L.KD);
+                    filters(kc, h * d, d, k0 + h * L.KD);
+                }
+                for (int h = 0; h < H; ++h) {
+                    in.place(v, h * dv, dv, 0, W, 0, c0 + v0 + h * L.VD);
+                    filters(vc, h * dv, dv, v0 + h * L.VD);
+                    mo.place(o, 0, W, h * dv, dv, r0 + h * L.VD, 0);
+                    dec[h] = expf(bf16_value(al.data[h]));
+                }
+                in.place(b, 0, H, 0, W, 0, b0);
+                if (L.head_decay()) {
+                    NEED(ad, "mix.a", H, W);
+                    NEED(dt, "mix.dt_bias", H, 1);
+                    NEED(g, "mix.g", H * dv, W);
+                    in.place(ad, 0, H, 0, W, 0, a0);
+                    for (int h = 0; h < H; ++h) in.place(g, h * dv, dv, 0, W, 0, g0 + h * L.VD);
+                    upload(values(dt, H), &L.dt_bias);
+                } else {
+                    NEED(a1, "mix.a1", s.decay_rank, W);
+                    NEED(a2, "mix.a2", H * d, s.decay_rank);
+                    NEED(dt, "mix.dt_bias", H * d, 1);
+                    NEED(g1, "mix.g1", s.gate_rank, W);
+                    NEED(g2, "mix.g2", H * dv, s.gate_rank);
+                    std::vector<float> dtb((size_t)H * L.KD, 0.0f);
+                    Matrix gt(L.rank, 2 * L.gcols);
+                    for (int h = 0; h < H; ++h) {
+                        gt.place(a2, h * d, d, 0, s.decay_rank, 0, h * L.KD);
+                        gt.place(g2, h * dv, dv, 0, s.gate_rank, 0, L.gcols + h * L.VD);
+                        for (int e = 0; e < d; ++e) dtb[(size_t)h * L.KD + e] = bf16_value(dt.data[(size_t)h * d + e]);
+                    }
+                    in.place(a1, 0, s.decay_rank, 0, W, 0, a0);
+                    in.place(g1, 0, s.gate_rank, 0, W, 0, g0);
+                    pack(gt, XFTHIP_WF_NONE, &L.gates);
+                    upload(dtb, &L.dt_bias);
+                }
+                upload(conv, &L.conv);
+                upload(dec, &L.decay);
+                upload(values(nm, L.VD), &L.out_norm);
+            }
+        } while (false);
+    };
     do {
         NEED(embed, "embed", V, W);
         upload_embedding(embed, 1, W, Wp, &p->embedding);
         front("final.norm", p->cfg.logit_scale, &p->final_norm); // the logits are linear in the normed row
+        if (p->cfg.bigram_buckets > 0) {
+            NEED(pairs, "bigram", (int)p->cfg.bigram_buckets + 1, W);
+            upload_embedding(pairs, 1, W, Wp, &p->pair_embedding);
+        }
         if (p->cfg.side_dim > 0) {
             NEED(side, "side.embed", V, p->cfg.layers * p->cfg.side_dim);
             upload_embedding(side, p->cfg.layers, p->cfg.side_dim, p->side_pad, &p->side_embedding);
@@ -784,12 +1056,12 @@ int xfthip_plan_finish(xfthip_plan_t p) {
     for (int i = 0; i < p->cfg.layers && missing.empty() && rc == 0; ++i) do {
         PlanLayer &L = p->layers[i];
         const xfthip_plan_layer &s = L.s;
-        const int H = s.heads;
+        if (s.beside) break; // (with the layer before it)
         prefix = std::to_string(i) + "/";
         front("norm1", 1.0f, &L.pre1);
         if (L.feeds_forward()) front("norm2", 1.0f, &L.pre2);
         if (!missing.empty()) break;
-        if (!parallel) {
+        if (sandwich) {
             NEED(n1b, "norm1b", W, 1);
             NEED(ls1, "ls1", W, 1);
             upload(one_plus(n1b, &ls1), &L.post1);
@@ -809,9 +1081,11 @@ int xfthip_plan_finish(xfthip_plan_t p) {
         }
         if (s.experts > 0) {
             NEED(router, "mlp.router", L.routes(), W);
-            NEED(correction, "mlp.correction", L.routes(), 1);
             plain(router, Wp, L.routes(), &L.router);
-            upload(values(correction, L.routes()), &L.correction);
+            if (s.router == XFTHIP_ROUTE_SOFTMAX) {
+                NEED(correction, "mlp.correction", L.routes(), 1);
+                upload(values(correction, L.routes()), &L.correction);
+            }
             L.egateup.assign(s.experts, nullptr), L.edown.assign(s.experts, nullptr);
             std::vector<GroupWeight> table(2 * (size_t)s.experts);
             for (int e = 0; e < s.experts && rc == 0; ++e) {
@@ -841,113 +1115,18 @@ int xfthip_plan_finish(xfthip_plan_t p) {
             plain(proj, p->side_pad, Wp, &L.side_proj);
             upload(values(norm, Wp), &L.side_post);
         }
-        Matrix in(Wp, L.row_in());
-        if (s.mixer == XFTHIP_MIXER_LATENT) {
-            const int d = s.dim, r = s.rot_dim, dv = s.vdim, R = s.kv_rank;
-            NEED(dq, "mix.dq", s.q_rank, W);
-            NEED(dqn, "mix.dq.norm", s.q_rank, 1);
-            NEED(uq, "mix.uq", H * (d + r), s.q_rank);
-            NEED(dkv, "mix.dkv", R + r, W);
-            NEED(dkvn, "mix.dkv.norm", R, 1);
-            NEED(uk, "mix.uk", H * d, R);
-            NEED(uv, "mix.uv", H * dv, R);
-            NEED(o, "mix.o", W, H * dv);
-            in.place(dq, 0, s.q_rank, 0, W, 0, 0);
-            in.place(dkv, 0, R, 0, W, 0, L.QR);
-            in.place(dkv, R, r, 0, W, 0, L.QR + L.R);
-            Matrix mq(L.QR, H * (L.D + L.RD)), ma(L.D, H * L.R), mk(L.R, H * L.D), mv(L.R, H * L.V), mo(H * L.V, Wp);
-            for (int h = 0; h < H; ++h) {
-                mq.place(uq, h * (d + r), d, 0, s.q_rank, 0, h * (L.D + L.RD));
-                mq.place(uq, h * (d + r) + d, r, 0, s.q_rank, 0, h * (L.D + L.RD) + L.D);
-                ma.place_turned(uk, h * d, d, 0, R, 0, h * L.R);
-                mk.place(uk, h * d, d, 0, R, 0, h * L.D);
-                mv.place(uv, h * dv, dv, 0, R, 0, h * L.V);
-                mo.place(o, 0, W, h * dv, dv, h * L.V, 0);
-            }
-            pack(mq, XFTHIP_WF_NONE, &L.uq);
-            pack(ma, XFTHIP_WF_NONE, &L.absorb);
-            pack(mk, XFTHIP_WF_NONE, &L.uk);
-            pack(mv, XFTHIP_WF_NONE, &L.uv);
-            pack(mo, XFTHIP_WF_NONE, &L.o);
-            upload(values(dqn, L.QR), &L.q_norm);
-            upload(values(dkvn, L.R), &L.kv_norm);
-            if (s.has_sink) {
-                NEED(sink, "mix.sink", H, 1);
-                upload(values(sink, H), &L.sink);
-            }
-        } else if (s.mixer == XFTHIP_MIXER_GROUPED) {
-            const int G = s.kv_heads, d = s.dim, dv = s.vdim, k0 = H * L.D, v0 = k0 + G * L.D;
-            NEED(q, "mix.q", H * d, W);
-            NEED(k, "mix.k", G * d, W);
-            NEED(v, "mix.v", G * dv, W);
-            NEED(o, "mix.o", W, H * dv);
-            Matrix mo(H * L.V, Wp);
-            for (int h = 0; h < H; ++h) in.place(q, h * d, d, 0, W, 0, h * L.D), mo.place(o, 0, W, h * dv, dv, h * L.V, 0);
-            for (int h = 0; h < G; ++h) in.place(k, h * d, d, 0, W, 0, k0 + h * L.D), in.place(v, h * dv, dv, 0, W, 0, v0 + h * L.V);
-            pack(mo, XFTHIP_WF_NONE, &L.o);
-            if (s.qk_norm) {
-                NEED(qn, "mix.q.norm", d, 1);
-                NEED(kn, "mix.k.norm", d, 1);
-                upload(values(qn, L.D), &L.q_norm);
-                upload(values(kn, L.D), &L.kv_norm);
-            }
-            if (s.has_sink) {
-                NEED(sink, "mix.sink", H, 1);
-                upload(values(sink, H), &L.sink);
-            }
-            if (s.v_mix && !L.first_values) {
-                NEED(share, "mix.vmix", 1, 1);
-                L.value_share = bf16_value(share.data[0]);
-            }
-        } else {
-            const int KH = s.kv_heads, d = s.dim, dv = s.vdim, n = s.taps;
-            NEED(q, "mix.q", KH * d, W);
-            NEED(k, "mix.k", KH * d, W);
-            NEED(v, "mix.v", H * dv, W);
-            NEED(qc, "mix.q.conv", KH * d, n);
-            NEED(kc, "mix.k.conv", KH * d, n);
-            NEED(vc, "mix.v.conv", H * dv, n);
-            NEED(b, "mix.b", H, W);
-            NEED(al, "mix.A_log", H, 1);
-            NEED(nm, "mix.norm", dv, 1);
-            NEED(a1, "mix.a1", s.decay_rank, W);
-            NEED(a2, "mix.a2", H * d, s.decay_rank);
-            NEED(dt, "mix.dt_bias", H * d, 1);
-            NEED(g1, "mix.g1", s.gate_rank, W);
-            NEED(g2, "mix.g2", H * dv, s.gate_rank);
-            NEED(o, "mix.o", W, H * dv);
-            std::vector<float> conv((size_t)L.channels() * n, 0.0f), dtb((size_t)H * L.KD, 0.0f), dec(H);
-            const int k0 = KH * L.KD, v0 = 2 * KH * L.KD, b0 = L.channels(), a0 = b0 + L.beta_cols(), g0 = a0 + L.rank;
-            auto filters = [&](const Tensor &t, int from, int count, int to) {
-                for (int i2 = 0; i2 < count * n; ++i2) conv[(size_t)to * n + i2] = bf16_value(t.data[(size_t)from * n + i2]);
-            };
-            for (int h = 0; h < KH; ++h) {
-                in.place(q, h * d, d, 0, W, 0, h * L.KD);
-                in.place(k, h * d, d, 0, W, 0, k0 + h * L.KD);
-                filters(qc, h * d, d, h * L.KD);
-                filters(kc, h * d, d, k0 + h * L.KD);
-            }
-            Matrix gt(L.rank, 2 * L.gcols), mo(H * L.VD, Wp);
-            for (int h = 0; h < H; ++h) {
-                in.place(v, h * dv, dv, 0, W, 0, v0 + h * L.VD);
-                filters(vc, h * dv, dv, v0 + h * L.VD);
-                gt.place(a2, h * d, d, 0, s.decay_rank, 0, h * L.KD);
-                gt.place(g2, h * dv, dv, 0, s.gate_rank, 0, L.gcols + h * L.VD);
-                mo.place(o, 0, W, h * dv, dv, h * L.VD, 0);
-                for (int e = 0; e < d; ++e) dtb[(size_t)h * L.KD + e] = bf16_value(dt.data[(size_t)h * d + e]);
-                dec[h] = expf(bf16_value(al.data[h]));
-            }
-            in.place(b, 0, H, 0, W, 0, b0);
-            in.place(a1, 0, s.decay_rank, 0, W, 0, a0);
-            in.place(g1, 0, s.gate_rank, 0, W, 0, g0);
-            pack(gt, XFTHIP_WF_NONE, &L.gates);
-            pack(mo, XFTHIP_WF_NONE, &L.o);
-            upload(conv, &L.conv);
-            upload(dtb, &L.dt_bias);
-            upload(dec, &L.decay);
-            upload(values(nm, L.VD), &L.out_norm);
+        // the mixer, or both: one input product, one output product
+        Matrix in(Wp, L.in_ld), mo(L.out_ld, Wp);
+        std::vector<float> bias(L.in_ld, 0.0f);
+        bool biased = false;
+        for (int k = i; k >= 0 && missing.empty() && rc == 0; k = k == i ? L.beside : -1) {
+            if (k != i) prefix = std::to_string(k) + "/";
+            mixer(p->layers[k], in, mo, bias, biased);
         }
+        if (!missing.empty() || rc) break;
         pack(in, XFTHIP_WF_NONE, &L.in);
+        pack(mo, XFTHIP_WF_NONE, &L.o);
+        if (biased) upload(bias, &L.in_bias);
     } while (false);
 #undef NEED
     XFT_REQUIRE(missing.empty(), "xfthip_plan_finish: tensor %s", missing.c_str());
@@ -992,11 +1171,11 @@ int xfthip_model_create_from_plan(xfthip_plan_t plan, int act_dtype, int max_bat
         memcpy(dst, &b, sizeof(b));
     };
     const size_t T = max_tokens, e = p->esz, hidden = plan->hidden;
-    size_t a = 0, cq = 0, q = 0, qa = 0, ov = 0, h = 0, gates = 0, dk = 0, dqk = 0, dg = 0, dv = 0, heads = 0, on = 0, fv = 0;
+    size_t a = 0, cq = 0, q = 0, qa = 0, ov = 0, h = 0, gates = 0, dk = 0, dqk = 0, dg = 0, dv = 0, heads = 0, fv = 0, u = 0, carry = 0;
     size_t top = 0, experts = 0, routes = 0, eh = 0, eo = 0;
     for (const PlanLayer &L : p->layers) {
         const size_t H = L.s.heads;
-        a = std::max(a, (size_t)L.row_in());
+        a = std::max(a, (size_t)L.in_ld), ov = std::max(ov, (size_t)L.out_ld);
         h = std::max(h, (size_t)L.ff);
         if (L.s.experts > 0) {
             const size_t most = std::min(L.s.top, L.s.experts);
@@ -1004,20 +1183,24 @@ int xfthip_model_create_from_plan(xfthip_plan_t plan, int act_dtype, int max_bat
             eh = std::max(eh, most * L.eff), eo = std::max(eo, most * hidden);
         }
         if (L.s.mixer == XFTHIP_MIXER_GROUPED) {
-            q = std::max(q, H * L.D), ov = std::max(ov, H * L.V);
+            q = std::max(q, H * L.D);
             if (L.s.v_mix) fv = std::max(fv, (size_t)L.s.kv_heads * L.V);
+        } else if (L.s.mixer == XFTHIP_MIXER_UNIT) {
+            gates = std::max(gates, (size_t)2 * L.channels()), u = std::max(u, (size_t)L.channels());
+            carry = std::max(carry, unit_carry_floats(L, max_tokens, max_batch));
         } else if (L.s.mixer == XFTHIP_MIXER_LATENT) {
-            cq = std::max(cq, (size_t)L.QR), q = std::max(q, H * (L.D + L.RD)), qa = std::max(qa, H * L.R), ov = std::max(ov, H * L.V);
+            cq = std::max(cq, (size_t)L.QR), q = std::max(q, H * (L.D + L.RD)), qa = std::max(qa, H * L.R);
         } else {
             const size_t KH = L.s.kv_heads;
-            gates = std::max(gates, (size_t)2 * L.gcols), dk = std::max(dk, KH * L.KD), dqk = std::max(dqk, KH), dg = std::max(dg, H * L.KD);
-            dv = std::max(dv, H * L.VD), heads = std::max(heads, H), on = std::max(on, H * L.VD);
+            gates = std::max(gates, (size_t)2 * L.gcols), dk = std::max(dk, KH * L.KD), dqk = std::max(dqk, KH), dg = std::max(dg, L.head_decay() ? H : H * L.KD);
+            dv = std::max(dv, H * L.VD), heads = std::max(heads, H);
         }
     }
     alloc(&p->xn, std::max(T, (size_t)p->logit_rows) * hidden * e);
     alloc(&p->y, T * hidden * 4);
     alloc(&p->a, T * a * e), alloc(&p->cq, T * cq * e), alloc(&p->q, T * q * e), alloc(&p->qa, T * qa * e), alloc(&p->oc, T * qa * e);
-    alloc(&p->ov, T * ov * e), alloc(&p->h, T * h * e), alloc(&p->on, T * on * e);
+    alloc(&p->ov, T * ov * e), alloc(&p->h, T * h * e), alloc(&p->u, T * u * e);
+    alloc(&p->carry, carry * 4), alloc(&p->last_token, (size_t)max_batch * 4, true);
     alloc(&p->gates, T * gates * 4), alloc(&p->dq, T * dk * 4), alloc(&p->dk, T * dk * 4), alloc(&p->dqk, T * dqk * 4), alloc(&p->dg, T * dg * 4);
     alloc(&p->dv, T * dv * 4), alloc(&p->dbeta, T * heads * 4), alloc(&p->do_, T * dv * 4);
     if (plan->cfg.block == XFTHIP_BLOCK_PARALLEL) alloc(&p->xn2, T * hidden * e), alloc(&p->narrow, T * hidden * e);
@@ -1039,19 +1222,25 @@ int xfthip_model_create_from_plan(xfthip_plan_t plan, int act_dtype, int max_bat
         if (L.s.mixer == XFTHIP_MIXER_GROUPED) p->part_floats = std::max(p->part_floats, grouped_part_floats(L));
     }
     alloc(&p->part, p->part_floats * 4);
-    for (const LayerRun &r : plan->runs) {
-        const PlanLayer &L = p->layers[r.layer];
+    for (const LayerRun &r : plan->runs) p->store_layer.push_back(r.layer);
+    for (const LayerRun &r : plan->runs)
+        if (r.beside >= 0) p->store_layer.push_back(r.beside);
+    for (size_t k = 0; k < p->store_layer.size(); ++k) {
+        const PlanLayer &L = p->layers[p->store_layer[k]];
         void *pool = nullptr;
         float *state = nullptr;
         void *conv = nullptr;
-        if (L.paged()) {
+        int from = (int)k;
+        if (L.kv_from >= 0) {
+            for (from = 0; p->store_layer[from] != L.kv_from;) ++from;
+        } else if (L.paged()) {
             // cleared: keys that lie behind a sequence's end are multiplied by zero weights and must be numbers
             alloc(&pool, (size_t)p->pages * kPageTokens * L.token_elems() * e, true);
         } else {
-            alloc(&state, (size_t)max_batch * L.s.heads * L.VD * L.KD * 4, true);
+            alloc(&state, (size_t)max_batch * L.state_floats() * 4, true);
             alloc(&conv, (size_t)max_batch * (L.s.taps - 1) * L.channels() * e, true);
         }
-        p->cache.push_back(pool), p->state.push_back(state), p->conv_state.push_back(conv);
+        p->reads.push_back(from), p->cache.push_back(pool), p->state.push_back(state), p->conv_state.push_back(conv);
     }
     alloc(&p->table, p->table_host.size() * 4, true);
     alloc(&p->desc, (3 * T + 4 * (size_t)max_batch) * 4, true);
@@ -1059,7 +1248,7 @@ int xfthip_model_create_from_plan(xfthip_plan_t plan, int act_dtype, int max_bat
     alloc(&p->want, (size_t)p->logit_rows * 4, true);
     std::map<std::vector<double>, std::pair<float *, float *>> rot; // layers of the same rotation share its tables
     for (PlanLayer &L : p->layers) {
-        if (!L.paged() || !ok) continue;
+        if (!L.paged() || L.s.rot_dim == 0 || !ok) continue;
         const bool extended = L.s.rot_factor > 0.0;
         auto &t = rot[{L.s.rot_base, (double)L.s.rot_dim, extended ? L.s.rot_factor : 0.0, extended ? L.s.rot_original : 0.0, extended ? L.s.rot_fast : 0.0,
                 extended ? L.s.rot_slow : 0.0}];

@@ -12,12 +12,87 @@ struct RouteParams {
     const float *logits;
     const float *correction;
     int ld, T, experts, routes, top;
+    int groups, keep; // groups 0: softmax and correction
+    float scale;
     RouteBuffers b;
 };
+
+__device__ inline float sigmoid(float z) { return 1.0f / (1.0f + expf(-z)); }
+
+// Sigmoid scores, the choice within the best groups of neighbouring experts; one token a wave, a group a lane (in turns of 64) for
+// the groups' scores.  Equal groups: the lower one first.
+template <int CH>
+__device__ inline void route_groups(const RouteParams &p, int t, int lane) {
+    const float *logits = p.logits + (size_t)t * p.ld;
+    const int n = p.routes / p.groups;
+    float z[CH], choice[CH], group[CH];
+#pragma unroll
+    for (int i = 0; i < CH; ++i) {
+        const int e = i * 64 + lane;
+        z[i] = e < p.routes ? sigmoid(logits[e]) : 0.0f;
+        choice[i] = -INFINITY;
+        group[i] = -INFINITY;
+        if (e < p.groups) { // (at most as many groups as outputs)
+            const float *g = logits + (size_t)e * n;
+            float a = g[0], b = -INFINITY;
+#pragma unroll 4
+            for (int k = 1; k < n; ++k) {
+                const float x = g[k];
+                b = fmaxf(b, fminf(a, x)), a = fmaxf(a, x);
+            }
+            group[i] = sigmoid(a) + (n > 1 ? sigmoid(b) : 0.0f);
+        }
+    }
+    for (int k = 0; k < p.keep; ++k) {
+        float best = group[0];
+#pragma unroll
+        for (int i = 1; i < CH; ++i) best = fmaxf(best, group[i]);
+        best = wave_largest(best);
+        int chosen = p.groups - 1;
+        bool open = true;
+#pragma unroll
+        for (int i = 0; i < CH; ++i) {
+            const unsigned long long at = open ? __ballot(group[i] == best) : 0ull;
+            if (at == 0ull) continue;
+            const int who = __ffsll(at) - 1;
+            open = false, chosen = i * 64 + who;
+            if (lane == who) group[i] = -INFINITY;
+        }
+#pragma unroll
+        for (int i = 0; i < CH; ++i) {
+            const int e = i * 64 + lane;
+            if (e < p.routes && e / n == chosen) choice[i] = z[i];
+        }
+    }
+    float sum = 0.0f;
+    for (int k = 0; k < p.top; ++k) {
+        float best = choice[0];
+#pragma unroll
+        for (int i = 1; i < CH; ++i) best = fmaxf(best, choice[i]);
+        best = wave_largest(best);
+        int e = p.routes - 1; // (scores that are not numbers equal nothing)
+        bool open = true;
+#pragma unroll
+        for (int i = 0; i < CH; ++i) {
+            const unsigned long long at = open ? __ballot(choice[i] == best) : 0ull;
+            if (at == 0ull) continue;
+            const int who = __ffsll(at) - 1;
+            open = false, e = i * 64 + who;
+            if (lane == who) choice[i] = -INFINITY;
+        }
+        sum += best;
+        if (lane == 0) p.b.sel[(size_t)t * p.top + k] = e < p.routes ? e : p.routes - 1;
+        if (lane == 0) p.b.weight[(size_t)t * p.top + k] = best;
+    }
+    const float f = p.scale / (sum + 1e-20f);
+    if (lane == 0)
+        for (int k = 0; k < p.top; ++k) p.b.weight[(size_t)t * p.top + k] *= f;
+}
 
 // One token a wave: CH router outputs a lane.  The choice scores give way one by one, the lower index first among equals.
 template <int CH>
 __device__ inline void route_one(const RouteParams &p, int t, int lane) {
+    if (p.groups > 0) return route_groups<CH>(p, t, lane);
     float z[CH], choice[CH], mx = -INFINITY;
 #pragma unroll
     for (int i = 0; i < CH; ++i) {
@@ -163,10 +238,12 @@ int launch_route(const RouteParams &p, hipStream_t st) {
 
 } // namespace
 
-int route_tokens(const float *logits, int ld, const float *correction, int T, int experts, int routes, int top, const RouteBuffers &b, hipStream_t st) {
-    XFT_REQUIRE(T > 0 && experts > 0 && routes >= experts && routes <= kMaxRoutes && top > 0 && top <= routes && top <= kMaxTop && ld >= routes,
-            "route_tokens: %d of %d + %d outputs", top, experts, routes - experts);
-    const RouteParams p = {logits, correction, ld, T, experts, routes, top, b};
+int route_tokens(const float *logits, int ld, const RouteRule &r, int T, const RouteBuffers &b, hipStream_t st) {
+    const int routes = r.routes;
+    XFT_REQUIRE(T > 0 && r.experts > 0 && routes >= r.experts && routes <= kMaxRoutes && r.top > 0 && r.top <= routes && r.top <= kMaxTop && ld >= routes
+                    && (r.groups > 0 ? routes == r.experts && routes % r.groups == 0 && r.keep > 0 && r.keep <= r.groups : r.correction != nullptr),
+            "route_tokens: %d of %d + %d outputs", r.top, r.experts, routes - r.experts);
+    const RouteParams p = {logits, r.correction, ld, T, r.experts, routes, r.top, r.groups, r.keep, r.scale, b};
     if (routes <= 64) return launch_route<1>(p, st);
     if (routes <= 128) return launch_route<2>(p, st);
     if (routes <= 256) return launch_route<4>(p, st);

@@ -16,6 +16,7 @@ struct TileGemm {
     void *C;
     int ldc, c_dtype, glu, add;
     float glu_limit, glu_alpha;
+    const float *bias;
     const uint16_t *side;
     int side_ld, side_vocab;
     const int *side_ids;
@@ -24,6 +25,7 @@ struct TileGemm {
 };
 
 __device__ inline float precise_glu(float gate, float up, float limit, float alpha) {
+    if (alpha == 0.0f) return gate / (1.0f + expf(-gate)) * up; // no limits
     const float g = fminf(gate, limit), u = fminf(fmaxf(up, -limit), limit);
     return g / (1.0f + expf(-alpha * g)) * (u + 1.0f);
 }
@@ -153,6 +155,7 @@ __global__ __launch_bounds__(KS > 4 ? 64 * KS : 256) void tile_gemm_kernel(TileG
         const int r = m0 + (int)(threadIdx.x >> 8) * 16 + (int)((threadIdx.x >> 2) & 15), n = nt0 * 16 + 4 * (int)((threadIdx.x >> 6) & 3) + (int)(threadIdx.x & 3);
         if (r >= p.M || n >= p.N) return;
         const size_t at = (size_t)r * p.ldc + n;
+        if (p.bias) y += p.bias[n];
         if (p.side) y = gelu_tanh(y) * side_value;
         if (p.add) y += ((const float *)p.C)[at];
         store_from_f32(p.C, p.c_dtype, at, y);
@@ -197,10 +200,11 @@ __global__ __launch_bounds__(KS > 4 ? 64 * KS : 256) void tile_gemm_kernel(TileG
 #pragma unroll
             for (int t = 0; t < 2; ++t) {
                 const int n = (nt0 + t) * 16 + 4 * g;
-                if (side || p.add) {
+                if (side || p.add || p.bias) {
 #pragma unroll
                     for (int i = 0; i < 4; ++i) {
                         if (n + i >= p.N) continue;
+                        if (p.bias) acc[t][m][i] += p.bias[n + i];
                         if (side) acc[t][m][i] = gelu_tanh(acc[t][m][i]) * bf16_to_f32(side[n + i]);
                         if (p.add) acc[t][m][i] += ((const float *)p.C)[(size_t)r * p.ldc + n + i];
                     }
@@ -233,10 +237,11 @@ int tile_gemm(xfthip_weight_t w, int act_in, const TileGemmArgs &a, hipStream_t 
     const int blocks = a.block_cols ? (pw.N + a.block_cols - 1) / a.block_cols : 1;
     XFT_REQUIRE((long)(blocks - 1) * a.a_block_stride + pw.K <= a.lda, "tile_gemm: %d blocks of K=%d reach past the row (%d)", blocks, pw.K, a.lda);
     XFT_REQUIRE(a.ldc >= (a.glu ? pw.N / 2 : pw.N) && a.glu == ((pw.flags & XFTHIP_WF_GATEUP) != 0), "tile_gemm: ldc=%d N=%d glu=%d", a.ldc, pw.N, a.glu);
+    XFT_REQUIRE(!a.bias || (!a.glu && !a.group), "tile_gemm: a bias joins plain products only");
     XFT_REQUIRE((!a.add || (a.c_dtype == XFTHIP_F32 && !a.glu)) && (!a.side || (!a.glu && !a.group && a.side_ids)) && (!a.group || a.group_rows),
             "tile_gemm: options that do not go together");
     const TileGemm p = {pw.packed, pw.KT, pw.K / 32, pw.NTILES, pw.N, M, a.A, a.lda, a.block_cols / 16, a.a_block_stride, a.C, a.ldc, a.c_dtype, a.glu, a.add,
-            a.glu_limit, a.glu_alpha, a.side, a.side_ld, a.side_vocab, a.side_ids, a.group, a.group_rows, a.a_rows};
+            a.glu_limit, a.glu_alpha, a.bias, a.side, a.side_ld, a.side_vocab, a.side_ids, a.group, a.group_rows, a.a_rows};
     const unsigned gz = a.group ? (unsigned)a.group_n : 1;
     const unsigned gx = (unsigned)((pw.NTILES + 7) / 8), gx1 = (unsigned)((pw.NTILES + 1) / 2);
     const bool f32 = act_in == XFTHIP_F32;
