@@ -606,7 +606,7 @@ def moe_layer(xh, iters=5):
                      "counts stay on the device)")
 
 
-PLAN_MODELS = ("pinepel", "llama_bf16", "veterax", "mixtral_bf16")
+PLAN_MODELS = ("pinepel", "llama_bf16", "veterax", "duvadra", "mixtral_bf16")
 PLAN_SIZES = {
     # width, ff, heads, query latent (the rest: 128 / 64 query dims, 128 value dims, key latent 512, 128-dim delta heads)
     "2048": dict(width=2048, ff=5632, heads=16, q_rank=768),
@@ -635,11 +635,12 @@ def plan_shapes(sz):
     return kinds * 2, shapes * 2
 
 
-# the stacks with sparse MLPs: key / value heads of 128, experts, chosen, width of an expert and of the shared one, identity outputs
+# the stacks with sparse MLPs: key / value heads of 128, experts (and their groups), chosen, width of an expert; Veterax: width of the
+# shared one, identity outputs
 SPARSE_SIZES = {
-    "2048": dict(kv_heads=4, experts=8, top=2, ff=2816, shared=2816, identity=2),
-    "4096": dict(kv_heads=8, experts=8, top=2, ff=2752, shared=5504, identity=2),
-    "2048x64": dict(kv_heads=4, experts=64, top=6, ff=1408, shared=2816, identity=8),  # (the uniform stack's sparse MLP has 8 experts)
+    "2048": dict(kv_heads=4, experts=8, groups=4, top=2, ff=2816, shared=2816, identity=2),
+    "4096": dict(kv_heads=8, experts=8, groups=4, top=2, ff=2752, shared=5504, identity=2),
+    "2048x64": dict(kv_heads=4, experts=64, groups=8, top=6, ff=1408, shared=2816, identity=8),  # (the uniform stack's sparse MLP has 8 experts)
 }
 
 
@@ -675,6 +676,60 @@ def build_veterax(xh, sz, sp, vocab=32000):
     embed = xh.f32_to_bf16_bits(rng.standard_normal((vocab, W), dtype=np.float32))
     for n, b in (("embed", embed), ("side.embed", bits("side.embed", (vocab, side * len(layers)))), ("final.norm", bits("norm", (W,))),
                  ("final.norm.b", bits("b", (W,))), ("final.norm.alpha", bits("alpha", (1,)))):
+        plan.set(-1, n, b)
+    for l, tensors in enumerate(shapes):
+        for n, s in tensors.items():
+            plan.set(l, n, bits(n, s))
+    plan.finish()
+    return plan
+
+
+def duvadra_layers(sz, sp):
+    """Records (mixers side by side are two) and tensor shapes of a Duvadra stack: a windowed attention with a sink beside a gated delta
+    rule, chunked attention, a keyed attention beside a gated linear recurrence, chunked attention on the second layer's keys, and the
+    first and the third once more; routed experts behind every layer."""
+    W, H, G, E = sz["width"], sz["heads"], sp["kv_heads"], sp["experts"]
+    scale, near = 128 ** -0.5, 1024
+    ff = dict(experts=E, top=sp["top"], expert_inter=sp["ff"], router=1, route_groups=sp["groups"], route_keep=sp["groups"] // 2, route_scale=2.5)
+    own = dict(mixer=3, heads=H, kv_heads=G, dim=128, vdim=128, scale=scale, **ff)
+    chunked = dict(own, chunk=near, softcap=30.0, distance_bias=1, out_gate=2)
+    windowed = dict(own, window=near, has_sink=1, qkv_bias=1, out_gate=1, scaled=1, mix_scale=0.6)
+    keyed = dict(own, window=near, key_values=1, qk_norm=2, rot_dim=64, rot_base=1e6, rot_interleaved=1, out_gate=1, scaled=1, mix_scale=0.6)
+    delta = dict(mixer=2, heads=H, kv_heads=H // 2, dim=128, vdim=128, taps=4, beside=1, scaled=1, mix_scale=0.8)
+    unit = dict(mixer=4, heads=W // 256, dim=256, vdim=256, taps=4, beside=1, scaled=1, mix_scale=0.8)
+    norms = {"norm1": (W,), "norm2": (W,), "mlp.router": (E, W)}
+    for e in range(E):
+        norms.update({"mlp.e%d.gate" % e: (sp["ff"], W), "mlp.e%d.up" % e: (sp["ff"], W), "mlp.e%d.down" % e: (W, sp["ff"])})
+    q, k, v, o = ({"mix." + n: s} for n, s in (("q", (H * 128, W)), ("k", (G * 128, W)), ("v", (G * 128, W)), ("o", (W, H * 128))))
+    biases = {"mix.q.b": (H * 128,), "mix.k.b": (G * 128,), "mix.v.b": (G * 128,), "mix.sink": (H,), "mix.g": (H * 128, W)}
+    w_shapes = dict(norms, **q, **k, **v, **o, **biases)
+    k_shapes = dict(norms, **q, **k, **o, **{"mix.q.norm": (H * 128,), "mix.k.norm": (G * 128,), "mix.g": (H * 128, W)})
+    d_shapes = {"mix.b": (H, W), "mix.a": (H, W), "mix.A_log": (H,), "mix.dt_bias": (H,), "mix.norm": (128,), "mix.g": (H * 128, W), "mix.o": (W, H * 128)}
+    for n, rows in (("q", H * 64), ("k", H * 64), ("v", H * 128)):
+        d_shapes["mix." + n], d_shapes["mix." + n + ".conv"] = (rows, W), (rows, 4)
+    u_shapes = {"mix.y": (W, W), "mix.y.b": (W,), "mix.x": (W, W), "mix.x.b": (W,), "mix.conv": (W, 4), "mix.conv.b": (W,), "mix.lam": (W,), "mix.o": (W, W)}
+    for n in ("ra", "ri"):
+        u_shapes["mix." + n], u_shapes["mix." + n + ".b"] = (W // 256, 256 * 256), (W // 256, 256)
+    first, third = [(windowed, w_shapes), (delta, d_shapes)], [(keyed, k_shapes), (unit, u_shapes)]
+    gate = {"mix.g": (H, W)}
+    records = first + [(chunked, dict(norms, **q, **k, **v, **o, **gate))] + third + [(dict(chunked, kv_from=3), dict(norms, **q, **o, **gate))] + first + third
+    return [r for r, _ in records], [t for _, t in records]
+
+
+def build_duvadra(xh, sz, sp, vocab=32000):
+    layers, shapes = duvadra_layers(sz, sp)
+    W, rng, pairs = sz["width"], np.random.default_rng(5), 65521
+    pool = xh.f32_to_bf16_bits(rng.standard_normal(1 << 22, dtype=np.float32) * 0.02)
+    plan = xh.Plan(W, vocab, layers, block=xh.BLOCK_SERIAL, norm=xh.NORM_RMS, residual_mult=0.5, embed_scale=1.0, logit_softcap=30.0, bigram=(pairs, 31, 7))
+    one = xh.f32_to_bf16_bits(np.ones(1, np.float32))[0]
+
+    def bits(name, shape):
+        if "norm" in name.split(".")[-1]:
+            return np.full(shape, one, np.uint16)
+        return np.resize(np.roll(pool, int(rng.integers(1 << 20))), int(np.prod(shape))).reshape(shape)
+
+    embed = xh.f32_to_bf16_bits(rng.standard_normal((vocab, W), dtype=np.float32))
+    for n, b in (("embed", embed), ("bigram", bits("bigram", (pairs + 1, W))), ("head", bits("head", (vocab, W))), ("final.norm", bits("final.norm", (W,)))):
         plan.set(-1, n, b)
     for l, tensors in enumerate(shapes):
         for n, s in tensors.items():
@@ -735,18 +790,18 @@ def build_llama_bf16(xh, sz, layers, batch, max_seq, max_tokens, vocab=32000, sp
 
 
 def plan_bench(xh, prompt=2048, batches=(1, 8, 32), steps=32, only=None, sizes=None, eager=False):
-    """Prefill (one prompt) and decode (behind prompts of that length) of Pinepel beside the uniform stack and of Veterax beside the
-    uniform stack with sparse MLPs, six layers each, in the same run.  Prompts of a decode batch are run one by one."""
+    """Prefill (one prompt) and decode (behind prompts of that length) of Pinepel beside the uniform stack and of Veterax and Duvadra
+    beside the uniform stack with sparse MLPs, six layers each, in the same run.  Prompts of a decode batch are run one by one."""
     out = []
     for name in sizes or list(PLAN_SIZES) + [n for n in SPARSE_SIZES if n not in PLAN_SIZES]:
         sz, sp = PLAN_SIZES[name.split("x")[0]], SPARSE_SIZES[name]
         for which in PLAN_MODELS:
-            if (only and which != only) or (name not in PLAN_SIZES and which != "veterax"):
+            if (only and which != only) or (name not in PLAN_SIZES and which not in ("veterax", "duvadra")):
                 continue
             B, max_seq = max(batches), prompt + 4 * (steps + 8)
             keep = []
-            if which in ("pinepel", "veterax"):
-                plan = build_plan(xh, sz) if which == "pinepel" else build_veterax(xh, sz, sp)
+            if which in ("pinepel", "veterax", "duvadra"):
+                plan = build_plan(xh, sz) if which == "pinepel" else (build_veterax if which == "veterax" else build_duvadra)(xh, sz, sp)
                 model, wbytes = xh.PlanModel(plan, xh.BF16, B, max_seq, prompt), plan.bytes()
                 keep = [plan]
             else:
@@ -801,7 +856,7 @@ def main():
     ap.add_argument("--prefill-gemm", action="store_true", help="only the weight-only GEMM sweep: M = 256, 2048 against the MFMA peak, M = 1, 8, 32 against the HBM peak (one JSON line)")
     ap.add_argument("--attention", action="store_true", help="only the GQA attention sweep (one JSON line)")
     ap.add_argument("--moe", action="store_true", help="only the sparse-MLP layer (one JSON line)")
-    ap.add_argument("--plan", action="store_true", help="only the layer-plan stacks (Pinepel, Veterax) beside the uniform BF16 stacks of equal size (dense, sparse MLPs): prefill and decode (one JSON line; progress on stderr)")
+    ap.add_argument("--plan", action="store_true", help="only the layer-plan stacks (Pinepel, Veterax, Duvadra) beside the uniform BF16 stacks of equal size (dense, sparse MLPs): prefill and decode (one JSON line; progress on stderr)")
     ap.add_argument("--plan-only", choices=PLAN_MODELS, help="with --plan: one of them")
     ap.add_argument("--plan-size", choices=sorted(SPARSE_SIZES), help="with --plan: one size")
     ap.add_argument("--no-live-traffic", action="store_true", help="do not run the two rocprofv3 counter passes for roofline.traffic (the recorded figure under profiles/ is reported instead)")
