@@ -692,7 +692,7 @@ def duvadra_layers(sz, sp):
     scale, near = 128 ** -0.5, 1024
     ff = dict(experts=E, top=sp["top"], expert_inter=sp["ff"], router=1, route_groups=sp["groups"], route_keep=sp["groups"] // 2, route_scale=2.5)
     own = dict(mixer=3, heads=H, kv_heads=G, dim=128, vdim=128, scale=scale, **ff)
-    chunked = dict(own, chunk=near, softcap=30.0, distance_bias=1, out_gate=2)
+    chunked = dict(own, chunk=4096, softcap=30.0, distance_bias=1, out_gate=2)
     windowed = dict(own, window=near, has_sink=1, qkv_bias=1, out_gate=1, scaled=1, mix_scale=0.6)
     keyed = dict(own, window=near, key_values=1, qk_norm=2, rot_dim=64, rot_base=1e6, rot_interleaved=1, out_gate=1, scaled=1, mix_scale=0.6)
     delta = dict(mixer=2, heads=H, kv_heads=H // 2, dim=128, vdim=128, taps=4, beside=1, scaled=1, mix_scale=0.8)

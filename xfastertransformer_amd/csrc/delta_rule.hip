@@ -1,17 +1,11 @@
 // The gated delta-rule recurrence of layer plans: short convolutions, unit norms, decays and step sizes (delta_prepare), the
 // walk over the tokens with the state in registers (delta_scan), the gated per-head norm behind it (delta_output).
 // Everything between the projections' outputs and the output projection's input is fp32.
-#include "plan.h"
+#include "plan_dev.h"
 
 namespace xfthip {
 
 namespace {
-
-__device__ inline float wave_total(float v) {
-#pragma unroll
-    for (int off = 32; off > 0; off >>= 1) v += __shfl_xor(v, off, 64);
-    return v;
-}
 
 template <bool BF16>
 __device__ inline float ldb(const void *p, size_t i) {
@@ -129,21 +123,6 @@ __global__ __launch_bounds__(256) void delta_prepare_kernel(PrepParams p) {
 // head, two neighbouring channels a lane, the convolutions' last inputs in registers - every input is read once and every
 // result leaves as a pair.  grid (token tiles of a segment, ceil(heads / 4), segments)
 constexpr int kPrepTokens = 8;
-
-template <bool BF16>
-__device__ inline float2 load2(const void *p, size_t i) {
-    if constexpr (BF16) {
-        const uint32_t u = *(const uint32_t *)((const uint16_t *)p + i);
-        return make_float2(u2f(u << 16), u2f(u & 0xFFFF0000u));
-    } else {
-        return *(const float2 *)((const float *)p + i);
-    }
-}
-template <bool BF16>
-__device__ inline void store2(void *p, size_t i, float2 v) {
-    if constexpr (BF16) *(uint32_t *)((uint16_t *)p + i) = f32_bits_to_bf16_sel(f2u(v.x)) | (f32_bits_to_bf16_sel(f2u(v.y)) << 16);
-    else *(float2 *)((float *)p + i) = v;
-}
 
 template <bool BF16, int TAPS, int J> // J: turns of 128 channels that cover a head's width
 __global__ __launch_bounds__(256) void delta_prepare_tiled_kernel(PrepParams p) {

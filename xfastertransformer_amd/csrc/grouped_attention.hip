@@ -224,6 +224,19 @@ struct ScoreRule {
         const float x = cap2 > 0.0f ? cap2 * fmaf(-2.0f, __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(s * twice) + 1.0f), 1.0f) : s * scale2;
         return fmaf(-slope2, distance, x);
     }
+    // N scores of a column; value r stands ahead(r) tokens closer than `distance`
+    template <int N, class S, class F>
+    __device__ inline void all(S &s, float scale2, float distance, F ahead) const {
+        const float far = -slope2 * distance;
+        if (cap2 > 0.0f) {
+#pragma unroll
+            for (int r = 0; r < N; ++r)
+                s[r] = fmaf(-2.0f * cap2, __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(s[r] * twice) + 1.0f), fmaf(slope2, ahead(r), cap2 + far));
+        } else {
+#pragma unroll
+            for (int r = 0; r < N; ++r) s[r] = fmaf(s[r], scale2, fmaf(slope2, ahead(r), far));
+        }
+    }
 };
 __device__ inline ScoreRule score_rule(const AttendParams &p, int head) {
     const bool cap = p.softcap > 0.0f;
@@ -582,10 +595,11 @@ __global__ __launch_bounds__(256, (KSM <= 8 && VTM <= 4) ? 2 : 1) void grouped_l
             if (EXACT || ks < ks_n) s = __builtin_amdgcn_mfma_f32_32x32x16_bf16(*(const bf16x8 *)(krow + ks * 32), qf[ks], s, 0, 0, 0);
         const bool masked = t0 + 31 > wlo || t0 < wfirst_hi;
         float bm = kUnseen;
+        if constexpr (RULE) {
+            rule.all<16>(s, scale2, (float)(pos - (t0 + 8 * h)), [](int r) { return (float)(16 * (r >> 3) + (r & 7)); });
+        } else {
 #pragma unroll
-        for (int r = 0; r < 16; ++r) {
-            if constexpr (RULE) s[r] = rule(s[r], scale2, (float)(pos - (t0 + 16 * (r >> 3) + 8 * h + (r & 7))));
-            else s[r] *= scale2;
+            for (int r = 0; r < 16; ++r) s[r] *= scale2;
         }
         if (masked) {
 #pragma unroll

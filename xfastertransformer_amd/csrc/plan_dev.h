@@ -32,6 +32,22 @@ __device__ inline void stact(void *p, size_t i, float v) {
     else ((float *)p)[i] = v;
 }
 
+// neighbouring pairs
+template <bool BF16>
+__device__ inline float2 load2(const void *p, size_t i) {
+    if constexpr (BF16) {
+        const uint32_t u = *(const uint32_t *)((const uint16_t *)p + i);
+        return make_float2(u2f(u << 16), u2f(u & 0xFFFF0000u));
+    } else {
+        return *(const float2 *)((const float *)p + i);
+    }
+}
+template <bool BF16>
+__device__ inline void store2(void *p, size_t i, float2 v) {
+    if constexpr (BF16) *(uint32_t *)((uint16_t *)p + i) = f32_bits_to_bf16_sel(f2u(v.x)) | (f32_bits_to_bf16_sel(f2u(v.y)) << 16);
+    else *(float2 *)((float *)p + i) = v;
+}
+
 // cache row of position `pos` of slot `row`
 __device__ inline size_t cache_row(const StepView &v, int row, int pos) {
     return (size_t)v.table[(size_t)row * v.table_stride + pos / kPageTokens] * kPageTokens + pos % kPageTokens;
@@ -79,9 +95,11 @@ __device__ inline void embed_token(const EmbedTables &e, int id, bool first, int
     const uint16_t *row = e.table + (size_t)id * e.hidden;
     const uint16_t *pair = e.pairs;
     if (pair) pair += (size_t)(first ? e.buckets : (prev * e.mul_prev + id * e.mul_cur) % e.buckets) * e.hidden;
-    for (int c = threadIdx.x; c < e.hidden; c += blockDim.x) {
-        const float v = bf16_to_f32(row[c]) * e.scale;
-        x[c] = pair ? v + bf16_to_f32(pair[c]) : v;
+    for (int c = threadIdx.x * 4; c < e.hidden; c += blockDim.x * 4) { // (rows are whole 32-value groups)
+        const uint2 a = *(const uint2 *)(row + c), b = pair ? *(const uint2 *)(pair + c) : make_uint2(0, 0);
+        const f32x4 v = {u2f(a.x << 16), u2f(a.x & 0xFFFF0000u), u2f(a.y << 16), u2f(a.y & 0xFFFF0000u)};
+        const f32x4 w = {u2f(b.x << 16), u2f(b.x & 0xFFFF0000u), u2f(b.y << 16), u2f(b.y & 0xFFFF0000u)};
+        *(f32x4 *)(x + c) = v * e.scale + w;
     }
 }
 
