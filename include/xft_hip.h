@@ -148,6 +148,9 @@ int xfthip_gemm(xfthip_weight_t w, int M, const void *A, int lda, void *C, int l
  */
 int xfthip_gemm_gateup_silu(xfthip_weight_t w, int M, const void *A, int lda, void *out, int ldo, int out_dtype,
         xfthip_stream_t stream);
+/* The same with a bias on both products (fp32 [2 I] in device memory: I of the gate, I of the other; no counterpart in the reference). */
+int xfthip_gemm_gateup_silu_bias(xfthip_weight_t w, int M, const void *A, int lda, void *out, int ldo, int out_dtype, const float *bias,
+        xfthip_stream_t stream);
 /* out[M,I] = g * sigmoid(alpha * g) * (u + 1) with g = min(A*Wgate, limit), u = A*Wup held to [-limit, limit], for a weight
  * created with XFTHIP_WF_GATEUP (no counterpart in the reference). */
 int xfthip_gemm_gateup_clamped(xfthip_weight_t w, int M, const void *A, int lda, void *out, int ldo, int out_dtype, float limit, float alpha,
@@ -547,17 +550,17 @@ int xfthip_model_set_moe(xfthip_model_t m, int idx, xfthip_moe_t moe);
 /* ---- layer plans: decoder stacks of several kinds of layers --------------------------- */
 /*
  * A plan describes a stack whose layers differ: what mixes the tokens (latent attention, a gated delta-rule recurrence, grouped
- * attention, a gated linear recurrence, or two of the last three side by side), its sizes, its constants, and the feed-forward
- * behind it, if any (dense, or routed experts beside an optional shared one).  Keys live in pages of a pool shared by all sequences, recurrent state in one slot a sequence.  The reference has no
+ * attention, a gated linear recurrence, gated linear attention, or two of the last four side by side), its sizes, its constants, and the
+ * feed-forward behind it, if any (dense, or routed experts beside an optional shared one).  Keys live in pages of a pool shared by all sequences, recurrent state in one slot a sequence.  The reference has no
  * counterpart; a model built from a plan is a xfthip_model_t and runs behind the same calls as the others.
  *
  * Three arrangements of a layer's sublayers:
- *   XFTHIP_BLOCK_SANDWICH  one after the other, a norm in front and a norm behind each, the latter multiplied by a learned scale
- *                          per channel
+ *   XFTHIP_BLOCK_SANDWICH  one after the other, a norm in front and a norm behind each, the latter (norms about one only) multiplied
+ *                          by a learned scale per channel
  *   XFTHIP_BLOCK_PARALLEL  both read the same residual through a norm of their own, their sum is added to it
  *   XFTHIP_BLOCK_SERIAL    one after the other, a norm in front of each, their results times residual_mult
  * and three kinds of norm: RMS norms whose stored weights are distances from one (sandwich), tanh(alpha x) * w + b (parallel), RMS
- * norms with plain weights (serial).
+ * norms with plain weights (serial, sandwich), the latter perhaps in norm_groups equal parts of the row, each divided by its own root mean square.
  * Layers [loop_start, loop_stop) run loop_times times, every run with its own cache or state, the embedding output joining the
  * residual in front of every pass but the first.  side_dim > 0: behind its sublayers every layer adds
  * rms(P (gelu(G x) * e)) * w, e the layer's part of a second embedding of the token.
@@ -565,10 +568,10 @@ int xfthip_model_set_moe(xfthip_model_t m, int idx, xfthip_moe_t moe);
  * The embedding is table[token] * embed_scale; bigram_buckets > 0: plus a row of a second table, that of (previous token * bigram_mul_prev
  * + token * bigram_mul_cur) mod bigram_buckets, or the row behind the buckets for the first token of a sequence.
  */
-enum { XFTHIP_MIXER_LATENT = 1, XFTHIP_MIXER_DELTA = 2, XFTHIP_MIXER_GROUPED = 3, XFTHIP_MIXER_UNIT = 4 };
+enum { XFTHIP_MIXER_LATENT = 1, XFTHIP_MIXER_DELTA = 2, XFTHIP_MIXER_GROUPED = 3, XFTHIP_MIXER_UNIT = 4, XFTHIP_MIXER_LINEAR = 5 };
 enum { XFTHIP_BLOCK_SANDWICH = 0, XFTHIP_BLOCK_PARALLEL = 1, XFTHIP_BLOCK_SERIAL = 2 };
 enum { XFTHIP_NORM_RMS_ABOUT_ONE = 0, XFTHIP_NORM_DYNAMIC_TANH = 1, XFTHIP_NORM_RMS = 2 };
-enum { XFTHIP_QK_NORM_HEAD = 1, XFTHIP_QK_NORM_ALL = 2 };
+enum { XFTHIP_QK_NORM_HEAD = 1, XFTHIP_QK_NORM_ALL = 2, XFTHIP_QK_NORM_UNIT = 3 };
 enum { XFTHIP_GATE_ELEMENT = 1, XFTHIP_GATE_HEAD = 2 };
 enum { XFTHIP_ROUTE_SOFTMAX = 0, XFTHIP_ROUTE_SIGMOID_GROUPS = 1 };
 typedef struct {
@@ -582,16 +585,17 @@ typedef struct {
     int has_sink; /* a learned logit a head in the softmax denominator */
     float scale;
     double rot_base;
-    /* delta rule */
+    /* delta rule; grouped attention (0: none): filters on the projected queries, keys and values, in front of norm and rotation */
     int taps; /* of the short convolutions */
     /* inner widths of the two gates' projections: decays a key channel, a sigmoid on the output; 0: one projection, one decay a head /
-     * a silu on the output */
+     * a silu on the output.  Linear attention: decay_rank > 0, a silu on the output */
     int decay_rank, gate_rank;
     /* feed-forward (inter 0: none; with experts: the shared one): xfthip_gemm_gateup_clamped; glu_alpha 0: silu(gate) * up, no limits */
     int inter;
     float glu_limit, glu_alpha;
     /* grouped attention */
-    int qk_norm; /* XFTHIP_QK_NORM_*: RMS norm in front of the rotation, of every query and key head or of all heads at once; 0 = none */
+    int qk_norm; /* XFTHIP_QK_NORM_*: RMS norm in front of the rotation, of every query and key head (with weights, or UNIT: without) or of
+                    all heads at once; 0 = none */
     int v_mix; /* values move a learned share of the way to those of the first layer that says so */
     /* context extension of the rotation (factor 0: none): frequencies whose pairs turn less than `slow` times within `original`
      * positions are divided by `factor`, those above `fast` stay, a ramp over the pairs between; cos and sin grow by
@@ -603,7 +607,8 @@ typedef struct {
     float expert_limit; /* of the experts' gates; the sigmoid's factor is glu_alpha */
     /*
      * beside = 1: not a layer of its own, but a second mixer of the layer before it (mixer fields only): both read the same input, their
-     * results are added.  scaled = 1: the mixer's result is multiplied by mix_scale.
+     * results are added.  scaled = 1: the mixer's result is multiplied by mix_scale.  result_norm = 1 (both of a pair or neither; below):
+     * each result is RMS-normed over the width, with a weight, before that.
      */
     int beside, scaled;
     float mix_scale;
@@ -619,6 +624,13 @@ typedef struct {
      * their two best scores are open; the chosen scores are divided by their sum and multiplied by route_scale; no correction */
     int router, route_groups, route_keep;
     float route_scale;
+    int result_norm; /* mixers side by side, see above */
+    /* grouped attention */
+    int keep_first; /* with a window: the first keep_first tokens of a sequence stay visible */
+    int pool; /* with a window, > 0: blocks of so many tokens that lie wholly before it are seen as the means of their keys and values */
+    int v_rot; /* 1: values are rotated by their position over all vdim dimensions (rot_base, pairs as the keys'), outputs back by theirs */
+    int o_bias, mlp_bias; /* the output projection, all three projections of a dense feed-forward have biases */
+    float tau; /* linear attention: decays are sigmoid(z)^(1 / tau) */
 } xfthip_plan_layer;
 typedef struct {
     int layers;
@@ -632,6 +644,7 @@ typedef struct {
     float embed_scale; /* 0 = 1 */
     float logit_softcap; /* > 0: logits pass cap * tanh(logit / cap) */
     long long bigram_buckets, bigram_mul_prev, bigram_mul_cur;
+    int norm_groups; /* XFTHIP_NORM_RMS: parts of a row in the norms around the sublayers and in front of the head; 0 = 1 */
 } xfthip_plan_config;
 typedef struct xfthip_plan *xfthip_plan_t;
 int xfthip_plan_create(const xfthip_plan_config *cfg, const xfthip_plan_layer *layers, xfthip_plan_t *out);
@@ -639,11 +652,11 @@ int xfthip_plan_destroy(xfthip_plan_t p);
 /*
  * Tensors by name, host memory, bf16 bit patterns, row-major [rows, cols] (linear weights [out, in]; vectors cols = 1): layer -1:
  * embed, head (unless tied), final.norm, side.embed; a layer (number of its record): norm1, norm2 (a tanh norm: also .alpha and .b), sandwich blocks also
- * norm1b, ls1, norm2b, ls2; side.gate / proj / norm; mlp.gate / up / down, with experts mlp.router, mlp.correction,
+ * norm1b, norm2b (norms about one: and ls1, ls2); side.gate / proj / norm; mlp.gate / up / down (.b), with experts mlp.router, mlp.correction,
  * mlp.e<i>.gate / up / down and mlp.shared.gate / up / down; and in front of its mixer's names "mix.": latent attention dq,
  * dq.norm, uq, dkv, dkv.norm, uk, uv, o, sink; delta rule q, k, v (each with .conv), b, A_log, a1, a2, dt_bias, g1, g2, norm, o;
- * grouped attention q, k (each with .norm, .b), v (.b), o, sink, vmix, g; delta rule without ranks a [heads] in place of a1, a2 and g in
- * place of g1, g2; gated unit (heads = blocks, dim = channels of a block, taps) y, x (each with .b), conv (.b), ra, ri [blocks, dim * dim]
+ * grouped attention q, k (each with .norm, .b, .conv), v (.b, .conv), o (.b), sink, vmix, g; delta rule without ranks a [heads] in place of a1,
+ * a2 and g in place of g1, g2; linear attention q, k, v, g, a1, a2 (.b), norm, o; with result_norm also out; gated unit (heads = blocks, dim = channels of a block, taps) y, x (each with .b), conv (.b), ra, ri [blocks, dim * dim]
  * (each with .b), lam, o.  bigram (layer -1).  xfthip_plan_finish checks that all are there, packs and uploads them.
  */
 int xfthip_plan_set_tensor(xfthip_plan_t p, int layer, const char *name, const uint16_t *data_host, int rows, int cols);

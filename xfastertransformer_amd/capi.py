@@ -245,6 +245,10 @@ def gemm_gateup_silu(w, A_dev, M, lda, out_dev, ldo, out_dtype=BF16, stream=None
     check(lib.xfthip_gemm_gateup_silu(w.h, M, A_dev, lda, out_dev, ldo, out_dtype, stream))
 
 
+def gemm_gateup_silu_bias(w, A_dev, M, lda, out_dev, ldo, bias_dev, out_dtype=BF16, stream=None):
+    check(lib.xfthip_gemm_gateup_silu_bias(w.h, M, A_dev, lda, out_dev, ldo, out_dtype, bias_dev, stream))
+
+
 class Timer:
     """HIP-event timer on a given stream (None = default stream)."""
 
@@ -540,20 +544,21 @@ class PlanLayer(C.Structure):
                 ("experts", C.c_int), ("identity", C.c_int), ("top", C.c_int), ("expert_inter", C.c_int), ("expert_limit", C.c_float),
                 ("beside", C.c_int), ("scaled", C.c_int), ("mix_scale", C.c_float), ("chunk", C.c_int), ("softcap", C.c_float), ("distance_bias", C.c_int),
                 ("qkv_bias", C.c_int), ("key_values", C.c_int), ("out_gate", C.c_int), ("kv_from", C.c_int), ("router", C.c_int), ("route_groups", C.c_int),
-                ("route_keep", C.c_int), ("route_scale", C.c_float)]
+                ("route_keep", C.c_int), ("route_scale", C.c_float), ("result_norm", C.c_int), ("keep_first", C.c_int), ("pool", C.c_int), ("v_rot", C.c_int),
+                ("o_bias", C.c_int), ("mlp_bias", C.c_int), ("tau", C.c_float)]
 
 
 class PlanConfig(C.Structure):
     _fields_ = [("layers", C.c_int), ("hidden", C.c_int), ("vocab", C.c_int), ("loop_start", C.c_int), ("loop_stop", C.c_int),
                 ("loop_times", C.c_int), ("eps", C.c_float), ("logit_scale", C.c_float), ("block", C.c_int), ("norm", C.c_int),
                 ("tied_head", C.c_int), ("side_dim", C.c_int), ("residual_mult", C.c_float), ("embed_scale", C.c_float), ("logit_softcap", C.c_float),
-                ("bigram_buckets", C.c_longlong), ("bigram_mul_prev", C.c_longlong), ("bigram_mul_cur", C.c_longlong)]
+                ("bigram_buckets", C.c_longlong), ("bigram_mul_prev", C.c_longlong), ("bigram_mul_cur", C.c_longlong), ("norm_groups", C.c_int)]
 
 
-MIXER_LATENT, MIXER_DELTA, MIXER_GROUPED, MIXER_UNIT = 1, 2, 3, 4
+MIXER_LATENT, MIXER_DELTA, MIXER_GROUPED, MIXER_UNIT, MIXER_LINEAR = 1, 2, 3, 4, 5
 BLOCK_SANDWICH, BLOCK_PARALLEL, BLOCK_SERIAL = 0, 1, 2
 NORM_RMS_ABOUT_ONE, NORM_DYNAMIC_TANH, NORM_RMS = 0, 1, 2
-QK_NORM_HEAD, QK_NORM_ALL = 1, 2
+QK_NORM_HEAD, QK_NORM_ALL, QK_NORM_UNIT = 1, 2, 3
 GATE_ELEMENT, GATE_HEAD = 1, 2
 ROUTE_SOFTMAX, ROUTE_SIGMOID_GROUPS = 0, 1
 lib.xfthip_plan_weight_bytes.restype = C.c_size_t
@@ -564,10 +569,10 @@ class Plan:
     """A stack of layers of several kinds (xfthip_plan_*).  layers: dicts of PlanLayer fields."""
 
     def __init__(self, hidden, vocab, layers, loop=(0, 0, 1), eps=1e-6, logit_scale=1.0, block=BLOCK_SANDWICH, norm=NORM_RMS_ABOUT_ONE,
-                 tied_head=0, side_dim=0, residual_mult=1.0, embed_scale=1.0, logit_softcap=0.0, bigram=(0, 0, 0)):
+                 tied_head=0, side_dim=0, residual_mult=1.0, embed_scale=1.0, logit_softcap=0.0, bigram=(0, 0, 0), norm_groups=0):
         arr = (PlanLayer * len(layers))(*[PlanLayer(**f) for f in layers])
         self.cfg = PlanConfig(len(layers), hidden, vocab, loop[0], loop[1], loop[2], eps, logit_scale, block, norm, tied_head, side_dim, residual_mult,
-                              embed_scale, logit_softcap, *bigram)
+                              embed_scale, logit_softcap, *bigram, norm_groups)
         self.layers = layers
         h = C.c_void_p()
         check(lib.xfthip_plan_create(C.byref(self.cfg), arr, C.byref(h)))

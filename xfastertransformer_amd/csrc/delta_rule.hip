@@ -13,35 +13,6 @@ __device__ inline float ldb(const void *p, size_t i) {
     else return ((const float *)p)[i];
 }
 
-// exp, x / (1 + exp(-x)), 1 / (1 + exp(-x)) and log(1 + exp(x)): the library functions with 32-bit activations; with bf16
-// ones the hardware's exp2 / log2 / reciprocal, each good to a few units in the last place (log(1 + y) through
-// y log(u) / (u - 1), u = 1 + y rounded, which keeps small y exact)
-template <bool FAST>
-__device__ inline float exp_of(float x) {
-    if constexpr (FAST) return fast_exp(x);
-    else return expf(x);
-}
-template <bool FAST>
-__device__ inline float sigmoid_of(float x) {
-    if constexpr (FAST) return __builtin_amdgcn_rcpf(1.0f + fast_exp(-x));
-    else return 1.0f / (1.0f + expf(-x));
-}
-template <bool FAST>
-__device__ inline float silu_of(float x) {
-    if constexpr (FAST) return x * __builtin_amdgcn_rcpf(1.0f + fast_exp(-x));
-    else return x / (1.0f + expf(-x));
-}
-template <bool FAST>
-__device__ inline float softplus_of(float x) {
-    if (x > 20.0f) return x;
-    if constexpr (FAST) {
-        const float y = fast_exp(x), u = 1.0f + y, d = u - 1.0f;
-        return d > 0.0f ? y * (__logf(u) * __builtin_amdgcn_rcpf(d)) : y;
-    } else {
-        return log1pf(expf(x));
-    }
-}
-
 struct PrepParams {
     StepView v;
     DeltaBuffers b;
@@ -262,21 +233,6 @@ __global__ __launch_bounds__(256) void conv_tail_kernel(TailParams p) {
                                   : load_as_f32(p.conv_state, DT, hist + (size_t)(s + n) * p.channels + ch);
         store_from_f32(p.conv_state, DT, hist + (size_t)s * p.channels + ch, x);
     }
-}
-
-template <int CTRL>
-__device__ inline float dpp_add(float v) {
-    return v + __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), CTRL, 0xF, 0xF, true));
-}
-// sum over aligned groups of L lanes, the same in all of them
-template <int L>
-__device__ inline float group_sum(float v) {
-    v = dpp_add<0xB1>(v); // quad_perm 1 0 3 2
-    v = dpp_add<0x4E>(v); // quad_perm 2 3 0 1
-    if constexpr (L >= 8) v = dpp_add<0x141>(v); // row_half_mirror
-    if constexpr (L >= 16) v = dpp_add<0x140>(v); // row_mirror
-    if constexpr (L >= 32) v += __shfl_xor(v, 16, 64);
-    return v;
 }
 
 struct ScanParams {
@@ -519,6 +475,16 @@ PrepParams prep_params(int act, const PlanLayer &L, const StepView &v, const Del
     return p;
 }
 
+int launch_output(int act, const PlanLayer &L, int T, OutParams p, float eps, hipStream_t st) {
+    p.out = (char *)p.out + (size_t)L.out_col * (act == XFTHIP_BF16 ? 2 : 4), p.out_ld = L.out_ld;
+    p.H = L.s.heads, p.VD = L.VD, p.vdim = L.s.vdim, p.gcols = L.gcols, p.T = T, p.eps = eps, p.mul = L.mix_scale;
+    const unsigned blocks = (unsigned)(((size_t)T * p.H + 3) / 4);
+    if (act == XFTHIP_BF16) hipLaunchKernelGGL(delta_output_kernel<true>, dim3(blocks), dim3(256), 0, st, p);
+    else hipLaunchKernelGGL(delta_output_kernel<false>, dim3(blocks), dim3(256), 0, st, p);
+    XFT_CHECK_HIP(hipGetLastError());
+    return 0;
+}
+
 } // namespace
 
 int delta_prepare(int act, const PlanLayer &L, const StepView &v, const DeltaBuffers &b, hipStream_t st) {
@@ -589,17 +555,12 @@ int delta_scan(const PlanLayer &L, const StepView &v, const DeltaBuffers &b, hip
 }
 
 int delta_output(int act, const PlanLayer &L, const StepView &v, const DeltaBuffers &b, float eps, hipStream_t st) {
-    const size_t esz = act == XFTHIP_BF16 ? 2 : 4;
-    const size_t gate = (size_t)L.in_col + L.channels() + 2 * L.beta_cols(); // (behind beta and decays)
-    const OutParams p = {b.o, b.gates, L.out_norm, L.silu_gate() ? (const char *)b.in + gate * esz : nullptr, L.in_ld, (char *)b.out + L.out_col * esz, L.out_ld,
-            L.s.heads, L.VD, L.s.vdim, L.gcols, v.T, eps, L.mix_scale};
-    const unsigned blocks = (unsigned)(((size_t)v.T * L.s.heads + 3) / 4);
-    if (act == XFTHIP_BF16)
-        hipLaunchKernelGGL(delta_output_kernel<true>, dim3(blocks), dim3(256), 0, st, p);
-    else
-        hipLaunchKernelGGL(delta_output_kernel<false>, dim3(blocks), dim3(256), 0, st, p);
-    XFT_CHECK_HIP(hipGetLastError());
-    return 0;
+    if (L.silu_gate()) return gated_head_norm(act, L, v.T, b.o, b.in, b.out, eps, st);
+    return launch_output(act, L, v.T, {b.o, b.gates, L.out_norm, nullptr, L.in_ld, b.out}, eps, st);
+}
+
+int gated_head_norm(int act, const PlanLayer &L, int T, const float *o, const void *in, void *out, float eps, hipStream_t st) {
+    return launch_output(act, L, T, {o, nullptr, L.out_norm, (const char *)in + (size_t)L.out_gate_col() * (act == XFTHIP_BF16 ? 2 : 4), L.in_ld, out}, eps, st);
 }
 
 } // namespace xfthip

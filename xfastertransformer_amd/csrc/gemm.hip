@@ -118,6 +118,11 @@ int xfthip_gemm(xfthip_weight_t w, int M, const void *A, int lda, void *C, int l
 
 int xfthip_gemm_gateup_silu(xfthip_weight_t w, int M, const void *A, int lda, void *out, int ldo, int out_dtype,
         xfthip_stream_t stream) {
+    return xfthip_gemm_gateup_silu_bias(w, M, A, lda, out, ldo, out_dtype, nullptr, stream);
+}
+
+int xfthip_gemm_gateup_silu_bias(xfthip_weight_t w, int M, const void *A, int lda, void *out, int ldo, int out_dtype, const float *bias,
+        xfthip_stream_t stream) {
     if (int rc = check_common("xfthip_gemm_gateup_silu", w, M, A, lda, out, ldo)) return rc;
     const PackedWeight &pw = w->pw;
     XFT_REQUIRE(pw.flags & XFTHIP_WF_GATEUP, "xfthip_gemm_gateup_silu: weight was not created with XFTHIP_WF_GATEUP");
@@ -132,6 +137,7 @@ int xfthip_gemm_gateup_silu(xfthip_weight_t w, int M, const void *A, int lda, vo
     p.ldc = ldo;
     p.c_dtype = out_dtype;
     p.gateup = 1;
+    p.bias = bias;
     if (M <= 32) return qgemm_skinny(pw, p, (hipStream_t)stream);
     return qgemm_mfma(pw, p, (hipStream_t)stream);
 }

@@ -8,6 +8,10 @@
 // workgroup, blocks of 32 tokens through LDS.  Scores come out as S^T = K Q^T with the tokens along the registers, in an order
 // chosen (by the row of the key operand a token is put in) so that a lane's probabilities are those of eight neighbouring
 // tokens: the operand of O^T += V^T P^T, whose other side is one 16-byte read.
+//
+// What a window leaves out but a position sees all the same - the first tokens of the sequence, or the means of whole blocks of tokens,
+// which have pages of their own - is a number of blocks in front of the window's: both forms walk them like the others.
+// The two values of a rotated pair are neighbours (PlanLayer::head_place).
 #include "plan_dev.h"
 
 namespace xfthip {
@@ -25,13 +29,66 @@ struct PrepareParams {
     StepView v;
     GroupedBuffers b;
     const float *q_norm, *k_norm, *cosT, *sinT; // norms may be null
+    const float *cosV, *sinV; // rotation of the values, or null
+    const uint16_t *filter; // [taps][channels] bf16, or null
+    int taps, channels;
+    int normed; // heads are divided by their root mean square (with or without weights)
+    int pool; // tokens of a block whose mean is kept, or 0
     int ld, value_col; // pitch of a's rows, first column of the values
-    int H, G, D, V, dim, rot, interleaved, lanes; // lanes a head takes (a power of two, 8 values each)
+    int H, G, D, V, dim, vdim, rot, lanes; // lanes a head takes (a power of two, 8 values each)
     int h0, h1; // heads to move, key heads behind the query heads
     int all; // norms over all query heads, all key heads: a workgroup a token
     int qk_blocks, seg_blocks, keep; // keep: write first_values
     float share, eps; // share of first_values in the values
 };
+
+// Eight neighbouring channels of token t's row from c on, behind their filter if there is one.  The only new token of a sequence shifts the
+// filter's inputs in place: a channel belongs to one thread.  (longer segments: conv_tail)
+template <bool BF16>
+__device__ inline void filtered8(const PrepareParams &p, int t, int c, float (&x)[8]) {
+    load8<BF16>(p.b.a, (size_t)t * p.ld + c, x);
+    if (!p.filter) return;
+    const int seg = p.v.tok_seg[t], pos = p.v.tok_pos[t], local = t - p.v.seg_off[seg], keep = p.taps - 1;
+    const size_t hist = (size_t)p.v.seg_row[seg] * keep * p.channels + c;
+    float y[8], w[8], in[8];
+    load8<true>(p.filter, (size_t)keep * p.channels + c, w);
+#pragma unroll
+    for (int k = 0; k < 8; ++k) y[k] = w[k] * x[k];
+    for (int back = 1; back <= keep && back <= pos; ++back) {
+        if (local >= back) load8<BF16>(p.b.a, (size_t)(t - back) * p.ld + c, in);
+        else load8<BF16>(p.b.conv_state, hist + (size_t)(keep + local - back) * p.channels, in);
+        load8<true>(p.filter, (size_t)(keep - back) * p.channels + c, w);
+#pragma unroll
+        for (int k = 0; k < 8; ++k) y[k] = fmaf(w[k], in[k], y[k]);
+    }
+    if (p.v.seg_len[seg] == 1 && keep > 0) {
+        for (int s = 0; s + 1 < keep; ++s) {
+            load8<BF16>(p.b.conv_state, hist + (size_t)(s + 1) * p.channels, in);
+            store8<BF16>(p.b.conv_state, hist + (size_t)s * p.channels, in);
+        }
+        store8<BF16>(p.b.conv_state, hist + (size_t)(keep - 1) * p.channels, x);
+    }
+#pragma unroll
+    for (int k = 0; k < 8; ++k) x[k] = y[k];
+}
+
+// neighbouring pairs from dimension c on, turned by the angles of their tables' row (or back)
+template <int N, bool BACK, class X>
+__device__ inline void turn_pairs(X &x, const float *cs, const float *sn, int c, int half) {
+#pragma unroll
+    for (int k = 0; k < N / 2; ++k) {
+        const int i = c / 2 + k;
+        if (i >= half) continue;
+        const float u = x[2 * k], z = x[2 * k + 1], cc = cs[i], ss = BACK ? -sn[i] : sn[i];
+        x[2 * k] = fmaf(u, cc, -(z * ss)), x[2 * k + 1] = fmaf(z, cc, u * ss);
+    }
+}
+
+template <bool BF16>
+__device__ inline float stored(float x) { // as memory holds it
+    if constexpr (BF16) return bf16_to_f32(f32_to_bf16_ref(x));
+    else return x;
+}
 
 // Eight values of a head from c on, normed (r: factor of the norm, or 1) and rotated, to q or into the page
 template <bool BF16>
@@ -39,7 +96,6 @@ __device__ inline void move_values(const PrepareParams &p, int t, int hh, int c,
     const int D = p.D, H = p.H, G = p.G;
     const float *norm = hh < H ? p.q_norm : p.k_norm;
     if (norm && p.all) norm += (size_t)(hh < H ? hh : hh - H) * D;
-    const size_t at = (size_t)t * p.ld + (size_t)hh * D;
     float w[8];
 #pragma unroll
     for (int k = 0; k < 8; ++k) w[k] = 1.0f;
@@ -47,31 +103,27 @@ __device__ inline void move_values(const PrepareParams &p, int t, int hh, int c,
 #pragma unroll
     for (int k = 0; k < 8; ++k) x[k] = x[k] * r * w[k];
     const int pos = p.v.tok_pos[t], half = p.rot / 2;
-    const float *cs = p.cosT + (size_t)pos * half, *sn = p.sinT + (size_t)pos * half;
-    if (p.interleaved) {
-#pragma unroll
-        for (int k = 0; k < 4; ++k) {
-            const int i = c / 2 + k;
-            if (i >= half) continue;
-            const float u = x[2 * k], z = x[2 * k + 1], cc = cs[i], ss = sn[i];
-            x[2 * k] = fmaf(u, cc, -(z * ss)), x[2 * k + 1] = fmaf(z, cc, u * ss);
-        }
-    } else {
-#pragma unroll
-        for (int k = 0; k < 8; ++k) {
-            const int d = c + k;
-            if (d >= p.rot) continue;
-            const int i = d < half ? d : d - half, other = d < half ? d + half : i;
-            const float z = ldact<BF16>(p.b.a, at + other) * r * (norm ? norm[other] : 1.0f);
-            x[k] = d < half ? fmaf(x[k], cs[i], -(z * sn[i])) : fmaf(x[k], cs[i], z * sn[i]);
-        }
-    }
+    turn_pairs<8, false>(x, p.cosT + (size_t)pos * half, p.sinT + (size_t)pos * half, c, half);
     if (hh < H) {
         store8<BF16>(p.b.q, ((size_t)t * H + hh) * D + c, x);
-    } else {
-        const int *table = p.v.table + (size_t)p.v.seg_row[p.v.tok_seg[t]] * p.v.table_stride;
-        store8<BF16>(p.b.pool, head_page(table, pos, G, hh - H, D, p.V) + (size_t)(pos % kPageTokens) * D + c, x);
+        return;
     }
+    const int seg = p.v.tok_seg[t], slot = p.v.seg_row[seg];
+    const int *table = p.v.table + (size_t)slot * p.v.table_stride;
+    store8<BF16>(p.b.pool, head_page(table, pos, G, hh - H, D, p.V) + (size_t)(pos % kPageTokens) * D + c, x);
+    if (p.pool == 0 || p.v.seg_len[seg] != 1 || (pos + 1) % p.pool != 0) return;
+    // the only new token of a sequence, and its block is full: the others of the block are there already
+#pragma unroll
+    for (int k = 0; k < 8; ++k) x[k] = stored<BF16>(x[k]);
+    for (int j = pos - p.pool + 1; j < pos; ++j) {
+        load8<BF16>(p.b.pool, head_page(table, j, G, hh - H, D, p.V) + (size_t)(j % kPageTokens) * D + c, w);
+#pragma unroll
+        for (int k = 0; k < 8; ++k) x[k] += w[k];
+    }
+#pragma unroll
+    for (int k = 0; k < 8; ++k) x[k] /= (float)p.pool;
+    const int block = pos / p.pool;
+    store8<BF16>(p.b.means, head_page(p.b.means_table + (size_t)slot * p.b.means_stride, block, G, hh - H, D, p.V) + (size_t)(block % kPageTokens) * D + c, x);
 }
 
 // One launch, two kinds of workgroups.  The first qk_blocks: a group of `lanes` threads one query or key head of a token (norms over all
@@ -113,9 +165,9 @@ __global__ __launch_bounds__(256) void grouped_prepare_kernel(PrepareParams p) {
         float x[8];
 #pragma unroll
         for (int k = 0; k < 8; ++k) x[k] = 0.0f;
-        if (on) load8<BF16>(p.b.a, (size_t)t * p.ld + (size_t)hh * D + c, x);
+        if (on) filtered8<BF16>(p, t, hh * D + c, x);
         float r = 1.0f;
-        if (p.q_norm) {
+        if (p.normed) {
             float sq = 0.0f;
 #pragma unroll
             for (int k = 0; k < 8; ++k) sq = fmaf(x[k], x[k], sq);
@@ -142,7 +194,11 @@ __global__ __launch_bounds__(256) void grouped_prepare_kernel(PrepareParams p) {
             const int tok = lo + i / (slice / 8), c = i % (slice / 8) * 8, t = off + tok - start;
             const size_t first = ((size_t)t * G + g) * V + d0 + c;
             float x[8];
-            load8<BF16>(p.b.a, (size_t)t * p.ld + p.value_col + (size_t)g * V + d0 + c, x);
+            filtered8<BF16>(p, t, p.value_col + g * V + d0 + c, x);
+            if (p.cosV) {
+                const size_t row = (size_t)tok * (p.vdim / 2);
+                turn_pairs<8, false>(x, p.cosV + row, p.sinV + row, d0 + c, p.vdim / 2);
+            }
             if (p.keep) {
                 store8<BF16>(p.b.first_values, first, x);
             } else if (p.share != 0.0f) {
@@ -169,6 +225,56 @@ __global__ __launch_bounds__(256) void grouped_prepare_kernel(PrepareParams p) {
                     if (b0 + t8 + k >= lo && b0 + t8 + k < hi) stact<BF16>(p.b.pool, at + k, tile[t8 + k][d]);
             }
         }
+        if (p.pool == 0 || n != 1 || (start + 1) % p.pool != 0) continue; // (as for keys)
+        for (int d = threadIdx.x; d < slice; d += 256) {
+            float sum = stored<BF16>(tile[start - b0][d]);
+            for (int j = start - p.pool + 1; j < start; ++j)
+                sum += ldact<BF16>(p.b.pool, head_page(table, j, G, g, D, V) + value_at(D, V, j % kPageTokens, d0 + d));
+            const int block = start / p.pool;
+            stact<BF16>(p.b.means, head_page(p.b.means_table + (size_t)p.v.seg_row[seg] * p.b.means_stride, block, G, g, D, V)
+                    + value_at(D, V, block % kPageTokens, d0 + d), sum / (float)p.pool);
+        }
+    }
+}
+
+// Means of the blocks that segments of several tokens fill: a workgroup one block of one head.  grid (heads * blocks, segments)
+template <bool BF16>
+__global__ __launch_bounds__(256) void grouped_means_kernel(PrepareParams p) {
+    const int D = p.D, V = p.V, G = p.G, seg = blockIdx.y, n = p.v.seg_len[seg], start = p.v.seg_pos[seg], g = blockIdx.x % G;
+    const int block = start / p.pool + (int)(blockIdx.x / G);
+    if (n == 1 || (block + 1) * p.pool > start + n) return;
+    const int *table = p.v.table + (size_t)p.v.seg_row[seg] * p.v.table_stride;
+    const size_t dst = head_page(p.b.means_table + (size_t)p.v.seg_row[seg] * p.b.means_stride, block, G, g, D, V);
+    const int first = block * p.pool, end = first + p.pool;
+    const float inv = 1.0f / (float)p.pool;
+    for (int i = threadIdx.x; i < D / 8 + V; i += 256) {
+        if (i < D / 8) {
+            float x[8] = {0.0f, 0.0f, 0.0f, 0.0f, 0.0f, 0.0f, 0.0f, 0.0f}, w[8];
+            for (int j = first; j < end; ++j) {
+                load8<BF16>(p.b.pool, head_page(table, j, G, g, D, V) + (size_t)(j % kPageTokens) * D + i * 8, w);
+#pragma unroll
+                for (int k = 0; k < 8; ++k) x[k] += w[k];
+            }
+#pragma unroll
+            for (int k = 0; k < 8; ++k) x[k] *= inv;
+            store8<BF16>(p.b.means, dst + (size_t)(block % kPageTokens) * D + i * 8, x);
+        } else {
+            const int d = i - D / 8;
+            float sum = 0.0f;
+            for (int j = first; j < end;) { // (runs of tokens of a value block, eight at a time where they are whole)
+                const size_t at = head_page(table, j, G, g, D, V) + value_at(D, V, j % kPageTokens, d);
+                if (j % 8 == 0 && j + 8 <= end) {
+                    float w[8];
+                    load8<BF16>(p.b.pool, at, w);
+                    sum += ((w[0] + w[1]) + (w[2] + w[3])) + ((w[4] + w[5]) + (w[6] + w[7]));
+                    j += 8;
+                } else {
+                    sum += ldact<BF16>(p.b.pool, at);
+                    ++j;
+                }
+            }
+            stact<BF16>(p.b.means, dst + value_at(D, V, block % kPageTokens, d), sum * inv);
+        }
     }
 }
 
@@ -186,6 +292,13 @@ struct AttendParams {
     float softcap; // or 0
     int distance_bias;
     int H, G, D, V, window, chunk;
+    // in front of the window: first tokens that stay visible, or means of blocks of `block` tokens
+    int keep_first, block;
+    const void *means;
+    const int *means_table;
+    int means_stride;
+    const float *cosV, *sinV; // outputs are turned back by their position, or null
+    int vhalf;
     int min_len, max_len; // segments of other lengths are somebody else's
     float scale;
     int nsplit, groups; // context splits; column groups of the longest segment
@@ -197,6 +310,16 @@ struct AttendParams {
 __device__ inline int first_seen(const AttendParams &p, int pos) {
     if (p.chunk > 0) return pos - pos % p.chunk;
     return p.window > 0 && pos + 1 > p.window ? pos + 1 - p.window : 0;
+}
+// entries in front of the window that position `pos` sees (kept first tokens: those that the window does not reach)
+__device__ inline int front_seen(const AttendParams &p, int pos) {
+    if (p.block == 0) return p.keep_first;
+    return pos + 1 - p.window >= p.block ? (pos + 1 - p.window) / p.block : 0;
+}
+// a position's outputs from dimension d on, turned back
+template <int N, class X>
+__device__ inline void turn_back(const AttendParams &p, int pos, int d, X &x) {
+    if (p.cosV) turn_pairs<N, true>(x, p.cosV + (size_t)pos * p.vhalf, p.sinV + (size_t)pos * p.vhalf, d, p.vhalf);
 }
 // what a token of distance costs head h
 __device__ inline float head_slope(const AttendParams &p, int h) { return p.distance_bias ? exp2f(-8.0f * (float)(h + 1) / (float)p.H) : 0.0f; }
@@ -259,59 +382,92 @@ __global__ __launch_bounds__(256) void grouped_attend_kernel(AttendParams p) {
     const float slope = head_slope(p, h);
     float m = p.sink ? p.sink[h] : -INFINITY, l = p.sink ? 1.0f : 0.0f; // the sink has no key and no value
     __syncthreads();
-    for (int k0 = first; k0 <= pos; k0 += 256) {
-        const int j = k0 + threadIdx.x;
-        float s = -INFINITY;
-        if (j <= pos) {
-            const size_t at = head_page(table, j, p.G, g, D, V) + (size_t)(j % kPageTokens) * D;
-            float acc = 0.0f;
-            for (int c = 0; c < D; c += 8) {
-                float k[8];
-                load8<BF16>(p.pool, at + c, k);
-#pragma unroll
-                for (int i = 0; i < 8; ++i) acc = fmaf(qs[c + i], k[i], acc);
+    // the entries in front of the window, then the window's
+    const int front = front_seen(p, pos), ahead = p.block == 0 && front > first ? first : front;
+    for (int stretch = 0; stretch < 2; ++stretch) {
+        const bool mean = stretch == 0 && p.block > 0;
+        const int begin = stretch ? first : 0, end = stretch ? pos : ahead - 1;
+        const void *pool = mean ? p.means : p.pool;
+        const int *pages = mean ? p.means_table + (size_t)p.v.seg_row[seg] * p.means_stride : table;
+        for (int k0 = begin; k0 <= end; k0 += 256) {
+            const int j = k0 + threadIdx.x;
+            float s = -INFINITY;
+            if (j <= end) {
+                const size_t at = head_page(pages, j, p.G, g, D, V) + (size_t)(j % kPageTokens) * D;
+                float acc = 0.0f;
+                for (int c = 0; c < D; c += 8) {
+                    float k[8];
+                    load8<BF16>(pool, at + c, k);
+    #pragma unroll
+                    for (int i = 0; i < 8; ++i) acc = fmaf(qs[c + i], k[i], acc);
+                }
+                s = acc * p.scale;
+                if (p.softcap > 0.0f) s = p.softcap * tanhf(s / p.softcap);
+                s -= slope * (float)(pos - j);
             }
-            s = acc * p.scale;
-            if (p.softcap > 0.0f) s = p.softcap * tanhf(s / p.softcap);
-            s -= slope * (float)(pos - j);
-        }
-        const float mx = wave_largest(s);
-        if ((threadIdx.x & 63) == 0) part[threadIdx.x >> 6] = mx;
-        __syncthreads();
-        const float m_new = fmaxf(fmaxf(fmaxf(part[0], part[1]), fmaxf(part[2], part[3])), m);
-        const float alpha = expf(m - m_new); // (0 while nothing has been seen)
-        const float e = j <= pos ? expf(s - m_new) : 0.0f;
-        ps[threadIdx.x] = e;
-        const float sum = wave_total(e);
-        if ((threadIdx.x & 63) == 0) part[4 + (threadIdx.x >> 6)] = sum;
-        __syncthreads();
-        l = l * alpha + ((part[4] + part[5]) + (part[6] + part[7]));
-        m = m_new;
-        const int n = pos - k0 + 1 < 256 ? pos - k0 + 1 : 256;
-        for (int c = threadIdx.x; c < V; c += 256) {
-            float acc = o[c] * alpha;
-            for (int i = 0; i < n;) {
-                // the run of tokens up to the end of a value block
-                const int at = k0 + i, run = 32 - (at & 31) < n - i ? 32 - (at & 31) : n - i;
-                const size_t src = head_page(table, at, p.G, g, D, V) + value_at(D, V, at % kPageTokens, c);
-                for (int k = 0; k < run; ++k) acc = fmaf(ps[i + k], ldact<BF16>(p.pool, src + k), acc);
-                i += run;
+            const float mx = wave_largest(s);
+            if ((threadIdx.x & 63) == 0) part[threadIdx.x >> 6] = mx;
+            __syncthreads();
+            const float m_new = fmaxf(fmaxf(fmaxf(part[0], part[1]), fmaxf(part[2], part[3])), m);
+            const float alpha = expf(m - m_new); // (0 while nothing has been seen)
+            const float e = j <= end ? expf(s - m_new) : 0.0f;
+            ps[threadIdx.x] = e;
+            const float sum = wave_total(e);
+            if ((threadIdx.x & 63) == 0) part[4 + (threadIdx.x >> 6)] = sum;
+            __syncthreads();
+            l = l * alpha + ((part[4] + part[5]) + (part[6] + part[7]));
+            m = m_new;
+            const int n = end - k0 + 1 < 256 ? end - k0 + 1 : 256;
+            for (int c = threadIdx.x; c < V; c += 256) {
+                float acc = o[c] * alpha;
+                for (int i = 0; i < n;) {
+                    // the run of tokens up to the end of a value block
+                    const int at = k0 + i, run = 32 - (at & 31) < n - i ? 32 - (at & 31) : n - i;
+                    const size_t src = head_page(pages, at, p.G, g, D, V) + value_at(D, V, at % kPageTokens, c);
+                    for (int k = 0; k < run; ++k) acc = fmaf(ps[i + k], ldact<BF16>(pool, src + k), acc);
+                    i += run;
+                }
+                o[c] = acc;
             }
-            o[c] = acc;
+            __syncthreads();
         }
-        __syncthreads();
     }
     for (int c = threadIdx.x; c < V; c += 256) {
-        float y = o[c] / l * p.out_scale;
-        if (p.gate_kind) y /= 1.0f + expf(-ldact<BF16>(p.gate, (size_t)t * p.gate_ld + (p.gate_kind == XFTHIP_GATE_HEAD ? h : h * V + c)));
-        stact<BF16>(p.out, (size_t)t * p.out_ld + (size_t)h * V + c, y);
+        float y[2] = {o[c & ~1], o[c | 1]}; // (V is even)
+        turn_back<2>(p, pos, c & ~1, y);
+        y[0] = (c & 1 ? y[1] : y[0]) / l * p.out_scale;
+        if (p.gate_kind) y[0] /= 1.0f + expf(-ldact<BF16>(p.gate, (size_t)t * p.gate_ld + (p.gate_kind == XFTHIP_GATE_HEAD ? h : h * V + c)));
+        stact<BF16>(p.out, (size_t)t * p.out_ld + (size_t)h * V + c, y[0]);
     }
 }
 
-// BF16, short form.  KS: most 32-dim steps of a key; VT: most 16-dim tiles of a value; EXACT: as many; RULE: scores are capped or
-// pay for distance.  grid (splits, G * column groups, segments)
-template <int KS, int VT, bool EXACT, bool RULE>
+// What the kernels know beforehand: plain scores; scores that are capped or pay for distance; entries in front of a window, with either
+// kind of score, and outputs that are turned back
+enum { kPlain, kRule, kFront };
+
+// The blocks of 32 entries that columns of positions lo .. hi see: those in front of the window, then the window's.  For `kFront`
+struct FrontBlocks {
+    int n, seen_lo, keep; // blocks; entries that the first column sees; kept first tokens (0: means)
+    const uint16_t *means;
+    const int *table;
+};
+__device__ inline FrontBlocks front_blocks(const AttendParams &p, int slot, int lo, int hi) {
+    FrontBlocks f;
+    if (p.block > 0) {
+        f.n = (front_seen(p, hi) + 31) >> 5, f.seen_lo = front_seen(p, lo), f.keep = 0;
+    } else {
+        const int b0 = first_seen(p, lo) >> 5, n = (p.keep_first + 31) >> 5;
+        f.n = n < b0 ? n : b0, f.seen_lo = f.keep = p.keep_first;
+    }
+    f.means = (const uint16_t *)p.means, f.table = p.means_table + (size_t)slot * p.means_stride;
+    return f;
+}
+
+// BF16, short form.  KS: most 32-dim steps of a key; VT: most 16-dim tiles of a value; EXACT: as many; FORM: see above.
+// grid (splits, G * column groups, segments)
+template <int KS, int VT, bool EXACT, int FORM>
 __global__ __launch_bounds__(256, (KS <= 4 && VT <= 8) ? 3 : 1) void grouped_short_kernel(AttendParams p) {
+    constexpr bool FRONT = FORM == kFront;
     extern __shared__ float merge[]; // [4 waves][16][2] maxima and sums, [4][16][V + 4] outputs
     const StepView &v = p.v;
     const int seg = blockIdx.z, n = v.seg_len[seg];
@@ -324,7 +480,10 @@ __global__ __launch_bounds__(256, (KS <= 4 && VT <= 8) ? 3 : 1) void grouped_sho
     const int last = c0 + 15 < ncols ? c0 + 15 : ncols - 1;
     const int lo = start + c0 / gs, hi = start + last / gs; // positions of the first and the last column's token
     const int first_lo = first_seen(p, lo), first_hi = first_seen(p, hi);
-    const int b0 = first_lo >> 5, b1 = (hi >> 5) + 1;
+    const int b1 = (hi >> 5) + 1;
+    FrontBlocks front {};
+    if constexpr (FRONT) front = front_blocks(p, v.seg_row[seg], lo, hi);
+    const int b0 = (first_lo >> 5) - front.n; // (blocks in front have numbers from b0 on, as if they were neighbours of the window's)
     const int per = (b1 - b0 + p.nsplit - 1) / p.nsplit;
     int wb = b0 + (int)blockIdx.x * per, we = wb + per < b1 ? wb + per : b1;
     const int wper = (we - wb + 3) / 4; // this wave's blocks
@@ -332,8 +491,10 @@ __global__ __launch_bounds__(256, (KS <= 4 && VT <= 8) ? 3 : 1) void grouped_sho
 
     const int c = c0 + i16, cv = c < ncols ? c : ncols - 1;
     const int cpos = c < ncols ? start + c / gs : -1, cfirst = first_seen(p, cpos < 0 ? 0 : cpos);
+    const int cfront = FRONT && p.block > 0 ? front_seen(p, cpos) : p.keep_first;
+    const bool ruled = FORM == kRule || (FRONT && (p.softcap > 0.0f || p.distance_bias));
     ScoreRule rule;
-    if constexpr (RULE) rule = score_rule(p, g * gs + cv % gs);
+    if constexpr (FORM != kPlain) rule = score_rule(p, g * gs + cv % gs);
     bf16x8 qf[KS];
     {
         const uint16_t *row = (const uint16_t *)p.q + (size_t)(off + cv / gs) * p.q_ld + (size_t)(g * gs + cv % gs) * D + 8 * lg;
@@ -352,23 +513,32 @@ __global__ __launch_bounds__(256, (KS <= 4 && VT <= 8) ? 3 : 1) void grouped_sho
     const uint16_t *pool = (const uint16_t *)p.pool;
     const size_t page_len = (size_t)kPageTokens * (D + V);
     bf16x8 kf[2][KS], vf[VT];
-    auto load_keys = [&](int blk, int page) {
-        const uint16_t *k = pool + ((size_t)page * G + g) * page_len + (blk & 1) * 32 * D + krow;
+    // block `at` of the walk: its number among those in front of the window or of all, where its page begins
+    auto in_front = [&](int at) { return FRONT && at < b0 + front.n; };
+    auto number = [&](int at) { return in_front(at) ? at - b0 : at; };
+    auto page_of = [&](int at) {
+        const int n = number(at) >> 1;
+        if (FRONT && front.keep == 0 && in_front(at)) return front.means + ((size_t)front.table[n] * G + g) * page_len;
+        return pool + ((size_t)table[n] * G + g) * page_len;
+    };
+    auto load_keys = [&](int at, const uint16_t *page) {
+        const uint16_t *k = page + (number(at) & 1) * 32 * D + krow;
 #pragma unroll
         for (int ks = 0; ks < KS; ++ks)
             if (EXACT || ks < ks_n) kf[0][ks] = *(const bf16x8 *)(k + ks * 32), kf[1][ks] = *(const bf16x8 *)(k + 4 * D + ks * 32);
     };
-    auto load_values = [&](int blk, int page) {
-        const uint16_t *w = pool + ((size_t)page * G + g) * page_len + (size_t)kPageTokens * D + (blk & 1) * 32 * V + vrow;
+    auto load_values = [&](int at, const uint16_t *page) {
+        const uint16_t *w = page + (size_t)kPageTokens * D + (number(at) & 1) * 32 * V + vrow;
 #pragma unroll
         for (int d = 0; d < VT; ++d)
             if (EXACT || d < vt_n) vf[d] = *(const bf16x8 *)(w + d * 512);
     };
-    int page = bb < be ? table[bb >> 1] : 0;
+    const uint16_t *page = bb < be ? page_of(bb) : pool;
     if (bb < be) load_keys(bb, page), load_values(bb, page);
-    for (int blk = bb; blk < be; ++blk) {
-        const bool more = blk + 1 < be;
-        if (more) page = table[(blk + 1) >> 1];
+    for (int at = bb; at < be; ++at) {
+        const bool more = at + 1 < be;
+        if (more) page = page_of(at + 1);
+        const int t0 = number(at) * 32;
         f32x4 s0 = {0.f, 0.f, 0.f, 0.f}, s1 = s0;
 #pragma unroll
         for (int ks = 0; ks < KS; ++ks)
@@ -376,20 +546,21 @@ __global__ __launch_bounds__(256, (KS <= 4 && VT <= 8) ? 3 : 1) void grouped_sho
                 s0 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[0][ks], qf[ks], s0, 0, 0, 0);
                 s1 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[1][ks], qf[ks], s1, 0, 0, 0);
             }
-        if (more) load_keys(blk + 1, page);
-        if constexpr (!RULE) s0 *= scale2, s1 *= scale2;
+        if (more) load_keys(at + 1, page);
+        if (!ruled) s0 *= scale2, s1 *= scale2;
         float x[8], bm = kUnseen;
 #pragma unroll
         for (int j = 0; j < 8; ++j) {
             x[j] = j < 4 ? s0[j & 3] : s1[j & 3];
-            if constexpr (RULE) x[j] = rule(x[j], scale2, (float)(cpos - (blk * 32 + 8 * lg + j)));
+            if (ruled) x[j] = rule(x[j], scale2, (float)(cpos - (t0 + 8 * lg + j)));
         }
-        const bool open = blk * 32 + 31 <= lo && blk * 32 >= first_hi; // every column sees the whole block
+        const bool open = in_front(at) ? t0 + 31 < front.seen_lo : t0 + 31 <= lo && t0 >= first_hi; // every column sees the whole block
         if (!open) {
 #pragma unroll
             for (int j = 0; j < 8; ++j) {
-                const int t = blk * 32 + 8 * lg + j;
-                x[j] = t <= cpos && t >= cfirst ? x[j] : kUnseen;
+                const int t = t0 + 8 * lg + j;
+                const bool seen = in_front(at) ? t < cfront : t <= cpos && (t >= cfirst || (FRONT && t < front.keep));
+                x[j] = seen ? x[j] : kUnseen;
             }
         }
 #pragma unroll
@@ -416,7 +587,7 @@ __global__ __launch_bounds__(256, (KS <= 4 && VT <= 8) ? 3 : 1) void grouped_sho
 #pragma unroll
         for (int d = 0; d < VT; ++d)
             if (EXACT || d < vt_n) o[d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[d], pf, o[d], 0, 0, 0);
-        if (more) load_values(blk + 1, page);
+        if (more) load_values(at + 1, page);
     }
     l += __shfl_xor(l, 16, 64);
     l += __shfl_xor(l, 32, 64);
@@ -450,6 +621,7 @@ __global__ __launch_bounds__(256, (KS <= 4 && VT <= 8) ? 3 : 1) void grouped_sho
         } else {
             if (p.sink) den += __builtin_amdgcn_exp2f(s2 - mt);
             const int t = off + cc / gs, head = g * gs + cc % gs;
+            if constexpr (FRONT) turn_back<4>(p, start + cc / gs, d, acc);
             acc *= output_gate(p, t, head, d) * (1.0f / den);
             uint16_t *dst = (uint16_t *)p.out + (size_t)t * p.out_ld + (size_t)head * V + d;
             *(uint2 *)dst = make_uint2(pack_pair(acc[0], acc[1]), pack_pair(acc[2], acc[3]));
@@ -502,15 +674,17 @@ __global__ __launch_bounds__(256) void grouped_merge_kernel(AttendParams p) {
     if (set > 0) return;
     for (int s = 1; s < sets; ++s) acc += sums[s * per + threadIdx.x];
     const int t = v.seg_off[seg] + c / gs;
+    turn_back<4>(p, v.seg_pos[seg] + c / gs, d, acc);
     acc *= output_gate(p, t, head, d) * inv_den;
     uint16_t *dst = (uint16_t *)p.out + (size_t)t * p.out_ld + (size_t)head * V + d;
     *(uint2 *)dst = make_uint2(pack_pair(acc[0], acc[1]), pack_pair(acc[2], acc[3]));
 }
 
 // BF16, long form: 128 columns a workgroup (32 a wave), the visible context in blocks of 32 tokens through LDS, on 32 x 32 tiles.
-// KSM: most 16-dim steps of a key; VTM: most 32-dim tiles of a value; EXACT, RULE as above.  grid (G, column groups, segments)
-template <int KSM, int VTM, bool EXACT, bool RULE>
+// KSM: most 16-dim steps of a key; VTM: most 32-dim tiles of a value; EXACT, FORM as above.  grid (G, column groups, segments)
+template <int KSM, int VTM, bool EXACT, int FORM>
 __global__ __launch_bounds__(256, (KSM <= 8 && VTM <= 4) ? 2 : 1) void grouped_long_kernel(AttendParams p) {
+    constexpr bool FRONT = FORM == kFront;
     extern __shared__ unsigned char lds[];
     const StepView &v = p.v;
     const int seg = blockIdx.z, n = v.seg_len[seg];
@@ -529,8 +703,9 @@ __global__ __launch_bounds__(256, (KSM <= 8 && VTM <= 4) ? 2 : 1) void grouped_l
     const bool wave_on = wc0 < ncols;
     const int head = g * gs + cv % gs;
     const int token = off + cv / gs, pos_first = first_seen(p, pos);
+    const bool ruled = FORM == kRule || (FRONT && (p.softcap > 0.0f || p.distance_bias));
     ScoreRule rule;
-    if constexpr (RULE) rule = score_rule(p, head);
+    if constexpr (FORM != kPlain) rule = score_rule(p, head);
     bf16x8 qf[KSM];
     {
         const uint16_t *row = (const uint16_t *)p.q + (size_t)token * p.q_ld + (size_t)head * D + 8 * h;
@@ -546,7 +721,11 @@ __global__ __launch_bounds__(256, (KSM <= 8 && VTM <= 4) ? 2 : 1) void grouped_l
     float m = kUnseen, l = 0.0f;
     const float scale2 = p.scale * kLog2e;
     const int lo = start + c0 / gs, last = c0 + 127 < ncols ? c0 + 127 : ncols - 1, hi = start + last / gs;
-    const int b0 = first_seen(p, lo) >> 5, b1 = (hi >> 5) + 1;
+    FrontBlocks front {};
+    if constexpr (FRONT) front = front_blocks(p, v.seg_row[seg], lo, hi);
+    const int b0 = (first_seen(p, lo) >> 5) - front.n, b1 = (hi >> 5) + 1; // (numbers as in the short form)
+    int pos_front = 0, wfront_lo = 0, wfront_hi = 0; // entries in front that the column, the wave's first and its last column see
+    if constexpr (FRONT) pos_front = front_seen(p, pos), wfront_lo = front_seen(p, wlo), wfront_hi = front_seen(p, whi);
     const int wfirst = first_seen(p, wlo), wfirst_hi = first_seen(p, whi);
 
     constexpr int PER = KSM / 4 + VTM / 2 + 1; // 16-byte chunks of a block a thread carries (at least D / 64 + V / 64)
@@ -565,27 +744,31 @@ __global__ __launch_bounds__(256, (KSM <= 8 && VTM <= 4) ? 2 : 1) void grouped_l
         }
     }
     const uint16_t *pool = (const uint16_t *)p.pool;
-    auto fetch = [&](int blk, int page) {
-        const uint16_t *base = pool + ((size_t)page * G + g) * kPageTokens * (D + V);
+    auto in_front = [&](int at) { return FRONT && at < b0 + front.n; };
+    auto number = [&](int at) { return in_front(at) ? at - b0 : at; };
+    auto page_of = [&](int at) { return FRONT && front.keep == 0 && in_front(at) ? front.table[number(at) >> 1] : table[number(at) >> 1]; };
+    auto fetch = [&](int at, int page) {
+        const uint16_t *base = (FRONT && front.keep == 0 && in_front(at) ? front.means : pool) + ((size_t)page * G + g) * kPageTokens * (D + V);
 #pragma unroll
         for (int i = 0; i < PER; ++i)
-            if (i * 256 < chunks) stage[i] = *(const u32x4 *)(base + src[i] + (blk & 1) * step[i]);
+            if (i * 256 < chunks) stage[i] = *(const u32x4 *)(base + src[i] + (number(at) & 1) * step[i]);
     };
     // row cl of the key operand is the token with bits 2 and 3 swapped: register 8 t + j of half h is then token 16 t + 8 h + j
     const int ktok = (cl & 19) | ((cl & 4) << 1) | ((cl & 8) >> 1);
-    fetch(b0, table[b0 >> 1]);
-    int page = b0 + 1 < b1 ? table[(b0 + 1) >> 1] : 0;
+    fetch(b0, page_of(b0));
+    int page = b0 + 1 < b1 ? page_of(b0 + 1) : 0;
     int buf = 0;
-    for (int blk = b0; blk < b1; ++blk, buf ^= 1) {
+    for (int at = b0; at < b1; ++at, buf ^= 1) {
         unsigned char *kb = lds + buf * bufb, *vb = kb + 32 * kpitch;
 #pragma unroll
         for (int i = 0; i < PER; ++i)
             if (i * 256 < chunks) *(u32x4 *)(kb + dst[i]) = stage[i];
         __syncthreads();
-        if (blk + 1 < b1) fetch(blk + 1, page);
-        if (blk + 2 < b1) page = table[(blk + 2) >> 1];
-        const int t0 = blk * 32;
-        if (!wave_on || t0 > whi || t0 + 31 < wfirst) continue; // (the same for the whole wave; the barrier above is all there is)
+        if (at + 1 < b1) fetch(at + 1, page);
+        if (at + 2 < b1) page = page_of(at + 2);
+        const int t0 = number(at) * 32;
+        const bool none = in_front(at) ? t0 >= wfront_hi : t0 > whi || (t0 + 31 < wfirst && !(FRONT && t0 < front.keep));
+        if (!wave_on || none) continue; // (the same for the whole wave; the barrier above is all there is)
         f32x16 s;
 #pragma unroll
         for (int r = 0; r < 16; ++r) s[r] = 0.0f;
@@ -593,9 +776,9 @@ __global__ __launch_bounds__(256, (KSM <= 8 && VTM <= 4) ? 2 : 1) void grouped_l
 #pragma unroll
         for (int ks = 0; ks < KSM; ++ks)
             if (EXACT || ks < ks_n) s = __builtin_amdgcn_mfma_f32_32x32x16_bf16(*(const bf16x8 *)(krow + ks * 32), qf[ks], s, 0, 0, 0);
-        const bool masked = t0 + 31 > wlo || t0 < wfirst_hi;
+        const bool masked = in_front(at) ? t0 + 31 >= wfront_lo : t0 + 31 > wlo || t0 < wfirst_hi;
         float bm = kUnseen;
-        if constexpr (RULE) {
+        if (ruled) {
             rule.all<16>(s, scale2, (float)(pos - (t0 + 8 * h)), [](int r) { return (float)(16 * (r >> 3) + (r & 7)); });
         } else {
 #pragma unroll
@@ -605,7 +788,8 @@ __global__ __launch_bounds__(256, (KSM <= 8 && VTM <= 4) ? 2 : 1) void grouped_l
 #pragma unroll
             for (int r = 0; r < 16; ++r) {
                 const int t = t0 + 16 * (r >> 3) + 8 * h + (r & 7);
-                s[r] = t <= pos && t >= pos_first ? s[r] : kUnseen;
+                const bool seen = in_front(at) ? t < pos_front : t <= pos && (t >= pos_first || (FRONT && t < front.keep));
+                s[r] = seen ? s[r] : kUnseen;
             }
         }
 #pragma unroll
@@ -656,37 +840,48 @@ __global__ __launch_bounds__(256, (KSM <= 8 && VTM <= 4) ? 2 : 1) void grouped_l
             for (int q = 0; q < 4; ++q) {
                 const int at = d * 32 + 8 * q + 4 * h;
                 const f32x4 f = output_gate(p, token, head, at) * mul;
-                *(uint2 *)(out + at) = make_uint2(pack_pair(o[d][4 * q] * f[0], o[d][4 * q + 1] * f[1]), pack_pair(o[d][4 * q + 2] * f[2], o[d][4 * q + 3] * f[3]));
+                f32x4 y = {o[d][4 * q], o[d][4 * q + 1], o[d][4 * q + 2], o[d][4 * q + 3]};
+                if constexpr (FRONT) turn_back<4>(p, pos, at, y);
+                y *= f;
+                *(uint2 *)(out + at) = make_uint2(pack_pair(y[0], y[1]), pack_pair(y[2], y[3]));
             }
         }
 }
 
-template <int KS, int VT, bool EXACT, bool RULE>
+template <int KS, int VT, bool EXACT, int FORM>
 int launch_short_form(const AttendParams &p, hipStream_t st) {
-    static const hipError_t attr = hipFuncSetAttribute((const void *)grouped_short_kernel<KS, VT, EXACT, RULE>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
+    static const hipError_t attr = hipFuncSetAttribute((const void *)grouped_short_kernel<KS, VT, EXACT, FORM>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
     XFT_CHECK_HIP(attr);
     const size_t smem = (size_t)4 * 16 * (2 + p.V + 4) * 4;
-    hipLaunchKernelGGL((grouped_short_kernel<KS, VT, EXACT, RULE>), dim3(p.nsplit, p.G * p.groups, p.v.B), dim3(256), smem, st, p);
+    hipLaunchKernelGGL((grouped_short_kernel<KS, VT, EXACT, FORM>), dim3(p.nsplit, p.G * p.groups, p.v.B), dim3(256), smem, st, p);
     XFT_CHECK_HIP(hipGetLastError());
     return 0;
 }
-template <int KSM, int VTM, bool EXACT, bool RULE>
+template <int KSM, int VTM, bool EXACT, int FORM>
 int launch_long_form(const AttendParams &p, hipStream_t st) {
-    static const hipError_t attr = hipFuncSetAttribute((const void *)grouped_long_kernel<KSM, VTM, EXACT, RULE>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
+    static const hipError_t attr = hipFuncSetAttribute((const void *)grouped_long_kernel<KSM, VTM, EXACT, FORM>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
     XFT_CHECK_HIP(attr);
     const size_t smem = (size_t)2 * (32 * (p.D * 2 + 16) + p.V * 80);
-    hipLaunchKernelGGL((grouped_long_kernel<KSM, VTM, EXACT, RULE>), dim3(p.G, (p.v.longest * (p.H / p.G) + 127) / 128, p.v.B), dim3(256), smem, st, p);
+    hipLaunchKernelGGL((grouped_long_kernel<KSM, VTM, EXACT, FORM>), dim3(p.G, (p.v.longest * (p.H / p.G) + 127) / 128, p.v.B), dim3(256), smem, st, p);
     XFT_CHECK_HIP(hipGetLastError());
     return 0;
 }
-bool has_rule(const AttendParams &p) { return p.softcap > 0.0f || p.distance_bias; }
+int form_of(const AttendParams &p) { return p.keep_first > 0 || p.block > 0 || p.cosV ? kFront : p.softcap > 0.0f || p.distance_bias ? kRule : kPlain; }
 template <int KS, int VT, bool EXACT>
 int launch_short(const AttendParams &p, hipStream_t st) {
-    return has_rule(p) ? launch_short_form<KS, VT, EXACT, true>(p, st) : launch_short_form<KS, VT, EXACT, false>(p, st);
+    switch (form_of(p)) {
+        case kFront: return launch_short_form<KS, VT, EXACT, kFront>(p, st);
+        case kRule: return launch_short_form<KS, VT, EXACT, kRule>(p, st);
+        default: return launch_short_form<KS, VT, EXACT, kPlain>(p, st);
+    }
 }
 template <int KSM, int VTM, bool EXACT>
 int launch_long(const AttendParams &p, hipStream_t st) {
-    return has_rule(p) ? launch_long_form<KSM, VTM, EXACT, true>(p, st) : launch_long_form<KSM, VTM, EXACT, false>(p, st);
+    switch (form_of(p)) {
+        case kFront: return launch_long_form<KSM, VTM, EXACT, kFront>(p, st);
+        case kRule: return launch_long_form<KSM, VTM, EXACT, kRule>(p, st);
+        default: return launch_long_form<KSM, VTM, EXACT, kPlain>(p, st);
+    }
 }
 
 bool mfma_takes(const PlanLayer &L) { return L.D <= 256 && L.V <= 256; }
@@ -699,8 +894,8 @@ int grouped_prepare(int act, const PlanLayer &L, const StepView &v, const Groupe
     const bool own = L.kv_from < 0;
     GroupedBuffers b = b0;
     b.a = (const char *)b.a + (size_t)L.in_col * (act == XFTHIP_BF16 ? 2 : 4);
-    PrepareParams p = {v, b, L.q_norm, L.kv_norm, L.cosT, L.sinT, L.in_ld, L.value_col(), s.heads, s.kv_heads, L.D, L.V, s.dim, s.rot_dim, s.rot_interleaved, 4,
-            L.moves_queries() ? 0 : s.heads, own ? s.heads + s.kv_heads : s.heads, s.qk_norm == XFTHIP_QK_NORM_ALL ? 1 : 0, 0, 0, L.first_values ? 1 : 0,
+    PrepareParams p = {v, b, L.q_norm, L.kv_norm, L.cosT, L.sinT, L.cosV, L.sinV, L.filter, s.taps, L.channels(), s.qk_norm != 0, s.pool, L.in_ld, L.value_col(),
+            s.heads, s.kv_heads, L.D, L.V, s.dim, s.vdim, s.rot_dim, 4, L.moves_queries() ? 0 : s.heads, own ? s.heads + s.kv_heads : s.heads, s.qk_norm == XFTHIP_QK_NORM_ALL ? 1 : 0, 0, 0, L.first_values ? 1 : 0,
             s.v_mix && !L.first_values ? L.value_share : 0.0f, eps};
     while (p.lanes * 8 < L.D) p.lanes *= 2;
     XFT_REQUIRE(p.lanes <= 64, "grouped_prepare: heads of %d values too wide", L.D);
@@ -711,6 +906,14 @@ int grouped_prepare(int act, const PlanLayer &L, const StepView &v, const Groupe
     if (act == XFTHIP_BF16) hipLaunchKernelGGL(grouped_prepare_kernel<true>, grid, dim3(256), 0, st, p);
     else hipLaunchKernelGGL(grouped_prepare_kernel<false>, grid, dim3(256), 0, st, p);
     XFT_CHECK_HIP(hipGetLastError());
+    if (L.filters())
+        if (int rc = conv_tail(act, v, b.a, L.in_ld, L.channels(), s.taps, b.conv_state, st)) return rc;
+    if (s.pool > 0 && v.longest > 1) {
+        const dim3 blocks(s.kv_heads * (v.longest / s.pool + 1), v.B);
+        if (act == XFTHIP_BF16) hipLaunchKernelGGL(grouped_means_kernel<true>, blocks, dim3(256), 0, st, p);
+        else hipLaunchKernelGGL(grouped_means_kernel<false>, blocks, dim3(256), 0, st, p);
+        XFT_CHECK_HIP(hipGetLastError());
+    }
     return 0;
 }
 
@@ -720,7 +923,8 @@ int grouped_split_count(const PlanLayer &L, int B, int longest, int hint) {
     longest = longest < kShortTokens ? longest : kShortTokens;
     const long units = (long)B * L.s.kv_heads * ((longest * (L.s.heads / L.s.kv_heads) + 15) / 16);
     const int span = L.s.chunk > 0 ? L.s.chunk : L.s.window;
-    const int ctx = span > 0 && span + longest < hint ? span + longest : hint;
+    const int ahead = L.s.pool > 0 ? hint / L.s.pool : L.s.keep_first; // entries in front of a window
+    const int ctx = span > 0 && span + ahead + longest < hint ? span + ahead + longest : hint;
     const int most = (ctx + 127) / 128;
     long want = device_cu_count() / units;
     want = want < most ? want : most;
@@ -739,8 +943,8 @@ int grouped_attention(int act, const PlanLayer &L, const StepView &v, const Grou
     const size_t esz = act == XFTHIP_BF16 ? 2 : 4;
     const char *rows = (const char *)b.a + L.in_col * esz;
     AttendParams p = {v, L.moves_queries() ? b.q : rows, b.pool, L.moves_queries() ? s.heads * L.D : L.in_ld, (char *)out + L.out_col * esz, L.out_ld, L.sink,
-            rows + L.gate_col() * esz, s.out_gate, L.in_ld, L.mix_scale, s.softcap, s.distance_bias, s.heads, s.kv_heads, L.D, L.V, s.window, s.chunk, 0, 1 << 30,
-            s.scale, 1, 1, part, 0};
+            rows + L.gate_col() * esz, s.out_gate, L.in_ld, L.mix_scale, s.softcap, s.distance_bias, s.heads, s.kv_heads, L.D, L.V, s.window, s.chunk, s.keep_first, s.pool,
+            b.means, b.means_table, b.means_stride, L.cosV, L.sinV, s.vdim / 2, 0, 1 << 30, s.scale, 1, 1, part, 0};
     if (act != XFTHIP_BF16 || !mfma_takes(L)) {
         const size_t smem = (size_t)(L.D + 256 + L.V + 8) * 4;
         if (act == XFTHIP_BF16) hipLaunchKernelGGL(grouped_attend_kernel<true>, dim3(v.T, s.heads), dim3(256), smem, st, p);

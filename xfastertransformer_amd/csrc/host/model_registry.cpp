@@ -468,11 +468,70 @@ PlanSpec duvadra(const Json &c, const SafeTensors &) {
     return s;
 }
 
+// ---- Balenex: norms in groups on both sides of every sublayer; a windowed attention with unit heads that sees older tokens as means of blocks, or
+// an attention with filters, turned values and a window beside the first tokens next to gated linear attention, their normed results
+// added; dense feed-forwards, biases nearly everywhere ----
+PlanSpec balenex(const Json &c, const SafeTensors &w) {
+    PlanSpec s;
+    s.cfg.hidden = (int)c.integer("width");
+    s.cfg.vocab = (int)c.integer("vocab");
+    s.cfg.eps = (float)c.at("norm").real("eps");
+    s.cfg.norm_groups = (int)c.at("norm").integer("groups");
+    if (s.cfg.norm_groups < 1) broken("norms without groups");
+    s.cfg.logit_scale = 1.0f;
+    s.cfg.loop_times = 1;
+    s.cfg.block = XFTHIP_BLOCK_SANDWICH, s.cfg.norm = XFTHIP_NORM_RMS;
+    const Json &layers = c.at("layers");
+    for (size_t i = 0; i < layers.items.size(); ++i) {
+        const std::string at = "layer " + std::to_string(i) + ": ";
+        const Json &e = layers.items[i], &m = e.at("mixer");
+        const std::string &type = e.string("type");
+        const bool one = type == "attention";
+        if (!one && type != "parallel") broken("layer type '" + type + "' of config.json is not known");
+        const Json &a = one ? m : m.at("left");
+        xfthip_plan_layer L {}, R {};
+        L.mixer = XFTHIP_MIXER_GROUPED;
+        L.heads = (int)a.integer("heads"), L.kv_heads = (int)a.integer("kv_heads"), L.dim = (int)a.integer("dim"), L.vdim = (int)a.integer("vdim");
+        L.scale = (float)a.real("scale");
+        L.qkv_bias = 1;
+        L.window = (int)a.at("mask").integer("size");
+        if (L.window < 1) broken(at + "an empty window");
+        if (one) {
+            L.o_bias = 1, L.qk_norm = XFTHIP_QK_NORM_UNIT;
+            L.pool = (int)a.at("mask").integer("pool");
+            if (L.pool < 1) broken(at + "empty blocks");
+        } else {
+            L.qk_norm = XFTHIP_QK_NORM_HEAD;
+            L.keep_first = (int)a.at("mask").integer("keep_first");
+            L.taps = (int)a.integer("conv");
+            L.rot_dim = (int)a.at("rot").integer("dims"), L.rot_base = a.at("rot").real("base");
+            L.v_rot = 1;
+            const Json &r = m.at("right");
+            R.mixer = XFTHIP_MIXER_LINEAR;
+            R.heads = (int)r.integer("heads"), R.dim = (int)r.integer("dim"), R.vdim = (int)r.integer("vdim");
+            R.tau = (float)r.real("tau");
+            R.decay_rank = (int)first_dim(w, "l" + std::to_string(i) + ".mix.right.a1");
+            R.beside = 1;
+            L.result_norm = R.result_norm = 1, L.scaled = R.scaled = 1, L.mix_scale = R.mix_scale = 0.5f;
+        }
+        if (e.has("mlp")) {
+            const Json &f = e.at("mlp");
+            if (f.string("kind") != "dense") broken("feed-forward '" + f.string("kind") + "' of config.json is not known");
+            L.inter = (int)f.integer("ff"), L.mlp_bias = 1;
+        }
+        s.record.push_back((int)s.layers.size());
+        s.layers.push_back(L);
+        if (!one) s.layers.push_back(R);
+    }
+    s.cfg.layers = (int)s.layers.size();
+    return s;
+}
+
 struct Architecture {
     const char *name;
     PlanSpec (*describe)(const Json &config, const SafeTensors &weights);
 };
-const Architecture kArchitectures[] = {{"Pinepel", pinepel}, {"Veterax", veterax}, {"Duvadra", duvadra}};
+const Architecture kArchitectures[] = {{"Pinepel", pinepel}, {"Veterax", veterax}, {"Duvadra", duvadra}, {"Balenex", balenex}};
 
 const Architecture *find_architecture(const Json &c) {
     if (c.kind != Json::Object || !c.has("architecture") || c.at("architecture").kind != Json::String) return nullptr;

@@ -472,7 +472,7 @@ struct ModelImpl {
             const int runs = i >= planSpec.cfg.loop_start && i < planSpec.cfg.loop_stop ? times : 1;
             const double e = planAct == XFTHIP_F32 ? 4 : 2;
             b += runs * (y.mixer == XFTHIP_MIXER_LATENT    ? (double)len * (y.kv_rank + y.rot_dim) * e
-                         : y.mixer == XFTHIP_MIXER_GROUPED ? (y.kv_from ? 0.0 : (double)len * y.kv_heads * (y.dim + y.vdim) * e)
+                         : y.mixer == XFTHIP_MIXER_GROUPED ? (y.kv_from ? 0.0 : (double)len * y.kv_heads * (y.dim + y.vdim) * e * (y.pool > 0 ? 1.0 + 1.0 / y.pool : 1.0))
                          : y.mixer == XFTHIP_MIXER_UNIT    ? (double)y.heads * y.dim * (4 + (y.taps - 1) * e)
                                                            : (double)y.heads * y.dim * y.vdim * 4);
         }

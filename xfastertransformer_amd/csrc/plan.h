@@ -1,7 +1,7 @@
 // Layer plans: decoder stacks whose layers differ in kind (latent attention, grouped attention, delta-rule recurrence, gated
-// linear recurrence), whose keys live in a page pool shared by all sequences and whose recurrent layers keep a state per sequence
+// linear recurrence, gated linear attention), whose keys live in a page pool shared by all sequences and whose recurrent layers keep a state per sequence
 // slot.  Declarations shared by the plan's driver (plan_model.hip) and its kernels (plan_layers.hip, latent_attention.hip,
-// grouped_attention.hip, delta_rule.hip, gated_unit.hip, routed_experts.hip, tile_gemm.hip).
+// grouped_attention.hip, delta_rule.hip, gated_unit.hip, linear_attention.hip, routed_experts.hip, tile_gemm.hip).
 //
 // Every inner width is padded to whole 32-value groups (the state's key dimension to a power of two) by zero rows and
 // columns of the packed weights, so that the kernels see whole MFMA steps whatever sizes a model has.
@@ -37,23 +37,29 @@ struct PlanLayer {
     // latent attention: padded widths of a head's unrotated / rotated / value part, of the key and the query latent;
     // grouped attention: D and V, of the query / key and the value part of a head
     int D = 0, RD = 0, V = 0, R = 0, QR = 0;
-    // delta rule: padded key / value width of a head, padded rank of the two gates and columns of one gate; gated unit: D, of a block
+    // delta rule, linear attention: padded key / value width of a head, padded rank of the gates and columns of one gate; gated unit: D, of
+    // a block
     int KD = 0, VD = 0, rank = 0, gcols = 0;
     // Where a mixer finds its projections and puts its result: mixers side by side share the rows of one input product
     // (row_in() columns from in_col on of in_ld) and of one output product (out_cols() from out_col on of out_ld).
     int in_col = 0, in_ld = 0, out_col = 0, out_ld = 0;
     float mix_scale = 1.0f; // of the result
+    float *result_norm = nullptr; // weights of the norm of the result (times its scale), or null; then each of a pair has an output product
     int beside = -1; // the record of the mixer next to this one
     int kv_from = -1; // grouped attention: the record whose cache serves
     int ff = 0; // padded
     xfthip_weight_t in = nullptr, o = nullptr, gateup = nullptr, down = nullptr; // (in, o: of both mixers, with the first one)
     float *in_bias = nullptr; // [in_ld] or null
+    float *o_bias = nullptr, *gateup_bias = nullptr, *down_bias = nullptr; // [hidden], [2 ff], [hidden] or null
     // latent: queries from their latent; W_uk turned round (query -> latent), W_uk and W_uv (latent -> key / value)
     xfthip_weight_t uq = nullptr, absorb = nullptr, uk = nullptr, uv = nullptr;
     float *q_norm = nullptr, *kv_norm = nullptr, *sink = nullptr; // (grouped attention: weights of the query and the key heads)
     float value_share = 0.0f; // v_mix: lambda
     bool first_values = false; // the layer whose values the others mix in
     float *cosT = nullptr, *sinT = nullptr; // [max positions][rot_dim / 2], shared by layers of the same rotation
+    float *cosV = nullptr, *sinV = nullptr; // [max positions][vdim / 2]: of rotated values
+    uint16_t *filter = nullptr; // grouped attention: filters [taps][channels], bf16
+    int means_table = 0; // grouped attention: the page table of block means, or 0
     // delta rule: both gates' second projections (decay | output gate), filters [channels][taps], exp(A_log), ...
     xfthip_weight_t gates = nullptr;
     float *conv = nullptr, *decay = nullptr, *dt_bias = nullptr, *out_norm = nullptr;
@@ -73,26 +79,40 @@ struct PlanLayer {
     float *post1 = nullptr, *post2 = nullptr;
 
     // columns of the input product: latent: query latent | key latent | shared key part; grouped: q | k | v | gate; delta rule: q | k |
-    // v | beta | decays | gate; gated unit: y | x
+    // v | beta | decays | gate; linear attention: q | k | v | decays | gate; gated unit: y | x
     int row_in() const {
         if (s.mixer == XFTHIP_MIXER_LATENT) return QR + R + RD;
         if (s.mixer == XFTHIP_MIXER_GROUPED) return gate_col() + (s.out_gate == XFTHIP_GATE_ELEMENT ? s.heads * V : s.out_gate == XFTHIP_GATE_HEAD ? beta_cols() : 0);
         if (s.mixer == XFTHIP_MIXER_UNIT) return 2 * s.heads * D;
+        if (s.mixer == XFTHIP_MIXER_LINEAR) return channels() + rank + s.heads * VD;
         return channels() + beta_cols() + (head_decay() ? beta_cols() : rank) + (silu_gate() ? s.heads * VD : rank);
     }
-    int out_cols() const { return s.mixer == XFTHIP_MIXER_UNIT ? s.heads * D : s.heads * (s.mixer == XFTHIP_MIXER_DELTA ? VD : V); }
+    int out_cols() const { return s.mixer == XFTHIP_MIXER_UNIT ? s.heads * D : s.heads * (s.mixer == XFTHIP_MIXER_DELTA || s.mixer == XFTHIP_MIXER_LINEAR ? VD : V); }
+    // delta rule, linear attention: first column of a gate in the rows
+    int out_gate_col() const { return in_col + channels() + (s.mixer == XFTHIP_MIXER_LINEAR ? rank : 2 * beta_cols()); }
     // grouped attention: first columns of values and gate
     int value_col() const { return s.heads * D + (s.key_values ? 0 : s.kv_heads * D); }
     int gate_col() const { return s.heads * D + (kv_from >= 0 ? 0 : s.kv_heads * (D + (s.key_values ? 0 : V))); }
-    bool moves_queries() const { return s.rot_dim > 0 || s.qk_norm; } // or they stay in the row
+    bool filters() const { return s.mixer == XFTHIP_MIXER_GROUPED && s.taps > 0; }
+    bool moves_queries() const { return s.rot_dim > 0 || s.qk_norm || filters(); } // or they stay in the row
+    // Grouped attention keeps the two values of a rotated pair side by side, whatever the model's order (the packed weights see to it):
+    // where dimension d of a query / key head or of a value head of the model is kept
+    int head_place(int d) const { return !s.rot_interleaved && d < s.rot_dim ? beside_partner(d, s.rot_dim / 2) : d; }
+    int value_place(int d) const { return s.key_values ? head_place(d) : s.v_rot && !s.rot_interleaved ? beside_partner(d, s.vdim / 2) : d; }
+    static int beside_partner(int d, int half) { return d < half ? 2 * d : 2 * (d - half) + 1; }
     bool head_decay() const { return s.decay_rank == 0; }
     bool silu_gate() const { return s.gate_rank == 0; }
     bool paged() const { return s.mixer == XFTHIP_MIXER_LATENT || s.mixer == XFTHIP_MIXER_GROUPED; }
     // elements a token takes in the page pool
     size_t token_elems() const { return s.mixer == XFTHIP_MIXER_LATENT ? R + RD : (size_t)s.kv_heads * (D + V); }
-    // floats of a slot's state, channels of the short convolution
-    size_t state_floats() const { return s.mixer == XFTHIP_MIXER_UNIT ? (size_t)s.heads * D : (size_t)s.heads * VD * KD; }
-    int channels() const { return s.mixer == XFTHIP_MIXER_UNIT ? s.heads * D : 2 * s.kv_heads * KD + s.heads * VD; } // (delta rule: q | k | v)
+    // floats of a slot's state, channels of the short convolution, elements of a slot's inputs of it
+    size_t state_floats() const { return paged() ? 0 : s.mixer == XFTHIP_MIXER_UNIT ? (size_t)s.heads * D : (size_t)s.heads * VD * KD; }
+    int channels() const { // (q | k | v; gated unit: x)
+        if (s.mixer == XFTHIP_MIXER_UNIT) return s.heads * D;
+        if (s.mixer == XFTHIP_MIXER_GROUPED) return s.heads * D + s.kv_heads * (D + V);
+        return 2 * (s.mixer == XFTHIP_MIXER_LINEAR ? s.heads : s.kv_heads) * KD + s.heads * VD;
+    }
+    size_t history() const { return s.mixer != XFTHIP_MIXER_LATENT && s.taps > 1 ? (size_t)(s.taps - 1) * channels() : 0; }
     int routes() const { return s.experts + s.identity; }
     bool feeds_forward() const { return ff > 0 || s.experts > 0; }
     int beta_cols() const { return (s.heads + 31) / 32 * 32; }
@@ -121,8 +141,10 @@ int plan_embed(const EmbedTables &e, const StepView &v, const int *ids, const in
 // logits pass cap * tanh(z / cap)
 int plan_softcap(float *logits, size_t n, float cap, hipStream_t st);
 
+// With y2: y = rms(y) * mix1 + rms(y2) * mix2 first, means over the width.  Then
 // x += rms(y) * post (y may be null; post null: x += mul * y), then x += table[ids] (table may be null), then xn = pre(x) (pre.w may be null) and
-// xn2 = pre2(x) (pre2.w may be null; tanh norms only).  Means over `width` of the `hidden` columns.  rows: xn row i comes from x
+// xn2 = pre2(x) (pre2.w may be null; tanh norms only).  Means over `width` of the `hidden` columns, with groups > 1 over each of so many
+// equal parts of them.  rows: xn row i comes from x
 // row rows[i] (only without y and table).
 struct PlanNormArgs {
     float *x;
@@ -136,6 +158,8 @@ struct PlanNormArgs {
     int hidden, width;
     float eps;
     float mul;
+    int groups = 1;
+    const float *y2 = nullptr, *mix1 = nullptr, *mix2 = nullptr;
 };
 int plan_norm(int act, const PlanNormArgs &p, int T, hipStream_t st);
 // out[t][c] = gelu(z[t][c]) * table[ids[t]][first + c] (tanh form of the gelu), c < width; bf16 table [vocab][ld], ids clamped
@@ -153,7 +177,8 @@ struct TileGemmArgs {
     bool add = false; // C += (fp32)
     bool glu = false; // the weight holds gate / up pairs (XFTHIP_WF_GATEUP), combined as clamped_glu, or (glu_alpha 0) silu(gate) * up
     float glu_limit = 0, glu_alpha = 0;
-    const float *bias = nullptr; // [N], joins the product (not with glu)
+    const float *bias = nullptr; // [N], joins the product (glu: of the gates, behind them of the others)
+    float decay_tau = 0; // > 0: C = sigmoid(product)^(1 / decay_tau)
     // C = gelu(product) * side[ids[t]][n] (as plan_side_gate)
     const uint16_t *side = nullptr;
     int side_ld = 0;
@@ -196,8 +221,12 @@ struct GroupedBuffers {
     void *q; // [T][heads][D]: normed, rotated queries
     void *pool; // pages: by key / value head [64][D] keys, then two blocks of 32 tokens [V][32] values
     void *first_values; // [T][kv_heads][V]: written by the layer that says so, read by the others that mix
+    void *conv_state; // filters: [slots][taps - 1][channels] of the activation type
+    void *means; // pages as the pool's: means of blocks of tokens, a block an entry; their table [slots][means_stride]
+    const int *means_table;
+    int means_stride;
 };
-// norms and rotation of queries and keys, mixing of values, append to the pages
+// filters, norms and rotation of queries and keys, mixing or rotation of values, append to the pages, means of the blocks that are full
 int grouped_prepare(int act, const PlanLayer &L, const StepView &v, const GroupedBuffers &b, float eps, hipStream_t st);
 // out: the step's rows of the output product's input; hint: upper bound of the sequence lengths
 int grouped_attention(int act, const PlanLayer &L, const StepView &v, const GroupedBuffers &b, void *out, int hint, float *part, size_t part_floats,
@@ -245,6 +274,19 @@ int delta_prepare(int act, const PlanLayer &L, const StepView &v, const DeltaBuf
 int delta_scan(const PlanLayer &L, const StepView &v, const DeltaBuffers &b, hipStream_t st);
 int delta_output(int act, const PlanLayer &L, const StepView &v, const DeltaBuffers &b, float eps, hipStream_t st);
 
+// ---- gated linear attention: S = diag(alpha) S + k v^T, o = S^T q
+struct LinearBuffers {
+    const void *in; // rows of the input product, of the activation type: q | k | v | decays (rank) | gate from in_col on
+    const float *alpha; // [T][heads][KD]
+    float *o; // [T][heads][VD]
+    void *out; // rows of the output product's input, of the activation type
+    float *state; // [slots][heads][VD][KD]
+};
+// the recurrence, the norm of every head and the gate
+int linear_attention(int act, const PlanLayer &L, const StepView &v, const LinearBuffers &b, float eps, hipStream_t st);
+// norm of every head of o [T][heads][VD] and silu gate (delta_output behind other recurrences)
+int gated_head_norm(int act, const PlanLayer &L, int T, const float *o, const void *in, void *out, float eps, hipStream_t st);
+
 // ---- gated linear recurrence: S = a S + sqrt(1 - a^2) i u by channel, a and i gated by the filtered input u itself
 struct UnitBuffers {
     const void *in; // rows of the input product, of the activation type: y | x from in_col on
@@ -283,6 +325,16 @@ struct xfthip_plan {
 
 namespace xfthip {
 
+// Pages of 64 entries, `unit` tokens an entry (1: keys and values of tokens; more: means of blocks of tokens): free ones, those of every slot
+// in position order, and the table [slots][stride], of which `at` is the place in the tables' common buffers.
+struct PageTable {
+    int unit = 1, pages = 0, stride = 0;
+    size_t at = 0;
+    std::vector<int> free_pages;
+    std::vector<std::vector<int>> held;
+    int pages_for(int tokens) const { return (tokens / unit + kPageTokens - 1) / kPageTokens; }
+};
+
 // What a model from a plan adds to xfthip_model: the page pool and the state slots, scratch, the step's description.
 struct PlanState {
     xfthip_plan *plan = nullptr;
@@ -294,12 +346,9 @@ struct PlanState {
     std::vector<int> store_layer, reads;
     std::vector<void *> cache;
     std::vector<float *> state;
-    std::vector<void *> conv_state;
-    // pages: free ones, those of every slot in position order, and the device table [slots][table_stride]
-    int pages = 0, table_stride = 0;
-    std::vector<int> free_pages;
-    std::vector<std::vector<int>> held;
-    std::vector<int> table_host;
+    std::vector<void *> conv_state, means;
+    std::vector<PageTable> tables; // the first: of tokens
+    std::vector<int> table_host; // all tables, and on the device
     int *table = nullptr;
     bool table_dirty = true;
     // step description on the device, its host image (pinned) and the views into it
@@ -314,7 +363,7 @@ struct PlanState {
     int logit_rows = 0;
     // scratch (activation type unless float)
     void *xn = nullptr, *a = nullptr, *cq = nullptr, *q = nullptr, *qa = nullptr, *oc = nullptr, *ov = nullptr, *h = nullptr, *u = nullptr;
-    float *y = nullptr, *gates = nullptr, *dq = nullptr, *dk = nullptr, *dqk = nullptr, *dg = nullptr, *dv = nullptr, *dbeta = nullptr, *do_ = nullptr, *carry = nullptr;
+    float *y = nullptr, *y2 = nullptr, *gates = nullptr, *dq = nullptr, *dk = nullptr, *dqk = nullptr, *dg = nullptr, *dv = nullptr, *dbeta = nullptr, *do_ = nullptr, *carry = nullptr;
     int *last_token = nullptr; // [slots]
     void *xn2 = nullptr, *first_values = nullptr, *side = nullptr, *narrow = nullptr;
     float *router_logits = nullptr, *expert_out = nullptr, *side_z = nullptr;
@@ -323,7 +372,6 @@ struct PlanState {
     void *rows = nullptr, *kx = nullptr, *vx = nullptr; // gathered latents, keys and values of a long segment's context
     float *part = nullptr; // split contexts
     size_t part_floats = 0;
-    std::vector<float *> tables; // rotation tables
     std::vector<void *> owned; // every device buffer above
     bool trace = false;
     float *trace_buf = nullptr;

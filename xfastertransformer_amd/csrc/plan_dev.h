@@ -85,6 +85,50 @@ __device__ inline void put4(void *p, size_t i, f32x4 v) {
     else *(f32x4 *)((float *)p + i) = v;
 }
 
+// exp, x / (1 + exp(-x)), 1 / (1 + exp(-x)) and log(1 + exp(x)): the library functions with 32-bit activations; with bf16
+// ones the hardware's exp2 / log2 / reciprocal, each good to a few units in the last place (log(1 + y) through
+// y log(u) / (u - 1), u = 1 + y rounded, which keeps small y exact)
+template <bool FAST>
+__device__ inline float exp_of(float x) {
+    if constexpr (FAST) return fast_exp(x);
+    else return expf(x);
+}
+template <bool FAST>
+__device__ inline float sigmoid_of(float x) {
+    if constexpr (FAST) return __builtin_amdgcn_rcpf(1.0f + fast_exp(-x));
+    else return 1.0f / (1.0f + expf(-x));
+}
+template <bool FAST>
+__device__ inline float silu_of(float x) {
+    if constexpr (FAST) return x * __builtin_amdgcn_rcpf(1.0f + fast_exp(-x));
+    else return x / (1.0f + expf(-x));
+}
+template <bool FAST>
+__device__ inline float softplus_of(float x) {
+    if (x > 20.0f) return x;
+    if constexpr (FAST) {
+        const float y = fast_exp(x), u = 1.0f + y, d = u - 1.0f;
+        return d > 0.0f ? y * (__logf(u) * __builtin_amdgcn_rcpf(d)) : y;
+    } else {
+        return log1pf(expf(x));
+    }
+}
+
+template <int CTRL>
+__device__ inline float dpp_add(float v) {
+    return v + __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), CTRL, 0xF, 0xF, true));
+}
+// sum over aligned groups of L lanes, the same in all of them
+template <int L>
+__device__ inline float group_sum(float v) {
+    v = dpp_add<0xB1>(v); // quad_perm 1 0 3 2
+    v = dpp_add<0x4E>(v); // quad_perm 2 3 0 1
+    if constexpr (L >= 8) v = dpp_add<0x141>(v); // row_half_mirror
+    if constexpr (L >= 16) v = dpp_add<0x140>(v); // row_mirror
+    if constexpr (L >= 32) v += __shfl_xor(v, 16, 64);
+    return v;
+}
+
 // tanh form of the Gaussian error linear unit
 __device__ inline float gelu_tanh(float z) { return 0.5f * z * (1.0f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z))); }
 

@@ -118,6 +118,113 @@ __global__ __launch_bounds__(NT) void plan_norm_kernel(PlanNormArgs p) {
     }
 }
 
+// Factors 1 / sqrt(mean + eps) of the groups a thread's values belong to.  `unit` lanes (a power of two) add the squares of their
+// neighbouring values up before the sums meet in LDS; unit 0: groups that are no whole number of float4, by value.
+template <int CH, int NT>
+__device__ inline void group_factors(const f32x4 (&v)[CH], const PlanNormArgs &p, int unit, float *sums, f32x4 (&r)[CH]) {
+    const int size = p.width / p.groups;
+    __syncthreads(); // (the sums of an earlier norm have been read)
+#pragma unroll
+    for (int c = 0; c < CH; ++c) {
+        const int at = c * NT + threadIdx.x; // float4 of the row
+        const f32x4 q = v[c] * v[c];
+        if (unit == 0) {
+            if (at * 4 < p.hidden) *(f32x4 *)(sums + at * 4) = q;
+            continue;
+        }
+        float s = (q[0] + q[1]) + (q[2] + q[3]);
+        for (int off = 1; off < unit; off <<= 1) s += __shfl_xor(s, off, 64);
+        if (at % unit == 0 && at * 4 < p.hidden) sums[at / unit] = s;
+    }
+    __syncthreads();
+#pragma unroll
+    for (int c = 0; c < CH; ++c) {
+        const int col = (c * NT + threadIdx.x) * 4;
+        r[c] = f32x4 {0.f, 0.f, 0.f, 0.f};
+        if (unit > 0) {
+            if (col >= p.width) continue;
+            const int n = size / (4 * unit);
+            const float *part = sums + (size_t)(col / size) * n;
+            float s = 0.0f;
+            for (int k = 0; k < n; ++k) s += part[k];
+            const float f = 1.0f / sqrtf(s / (float)size + p.eps);
+            r[c] = f32x4 {f, f, f, f};
+        } else {
+            for (int i = 0; i < 4; ++i) {
+                if (col + i >= p.width) break;
+                const float *part = sums + (size_t)((col + i) / size) * size;
+                float s = 0.0f;
+                for (int k = 0; k < size; ++k) s += part[k];
+                r[c][i] = 1.0f / sqrtf(s / (float)size + p.eps);
+            }
+        }
+    }
+}
+
+// The same steps with norms in groups and with the results of two mixers that meet here: y = rms(y) mix1 + rms(y2) mix2, x += norm(y) post,
+// xn = norm(x) pre
+template <bool BF16, int CH, int NT>
+__global__ __launch_bounds__(NT) void plan_group_norm_kernel(PlanNormArgs p, int unit) {
+    extern __shared__ float sums[];
+    __shared__ float part[2][NT / 64];
+    const int t = blockIdx.x;
+    const float *xr = p.x + (size_t)(p.rows ? p.rows[t] : t) * p.hidden;
+    f32x4 x[CH], y[CH], z[CH], wpost[CH], wpre[CH], r[CH];
+    const f32x4 zero = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int c = 0; c < CH; ++c) {
+        const int col = (c * NT + threadIdx.x) * 4;
+        const bool in = col < p.hidden;
+        x[c] = in ? *(const f32x4 *)(xr + col) : zero;
+        y[c] = in && p.y ? *(const f32x4 *)(p.y + (size_t)t * p.hidden + col) : zero;
+        z[c] = in && p.y2 ? *(const f32x4 *)(p.y2 + (size_t)t * p.hidden + col) : zero;
+        wpost[c] = in && p.post ? *(const f32x4 *)(p.post + col) : zero;
+        wpre[c] = in && p.pre.w ? *(const f32x4 *)(p.pre.w + col) : zero;
+    }
+    if (p.y2) {
+        float s1 = 0.0f, s2 = 0.0f;
+#pragma unroll
+        for (int c = 0; c < CH; ++c)
+#pragma unroll
+            for (int i = 0; i < 4; ++i) s1 = fmaf(y[c][i], y[c][i], s1), s2 = fmaf(z[c][i], z[c][i], s2);
+        s1 = wave_total(s1), s2 = wave_total(s2);
+        if ((threadIdx.x & 63) == 0) part[0][threadIdx.x >> 6] = s1, part[1][threadIdx.x >> 6] = s2;
+        __syncthreads();
+        s1 = s2 = 0.0f;
+#pragma unroll
+        for (int w = 0; w < NT / 64; ++w) s1 += part[0][w], s2 += part[1][w];
+        const float r1 = 1.0f / sqrtf(s1 / (float)p.width + p.eps), r2 = 1.0f / sqrtf(s2 / (float)p.width + p.eps);
+#pragma unroll
+        for (int c = 0; c < CH; ++c) {
+            const int col = (c * NT + threadIdx.x) * 4;
+            if (col >= p.hidden) continue;
+            y[c] = y[c] * r1 * *(const f32x4 *)(p.mix1 + col) + z[c] * r2 * *(const f32x4 *)(p.mix2 + col);
+        }
+    }
+    if (p.y) {
+        if (p.post) {
+            group_factors<CH, NT>(y, p, unit, sums, r);
+#pragma unroll
+            for (int c = 0; c < CH; ++c) x[c] = x[c] + y[c] * r[c] * wpost[c];
+        } else {
+#pragma unroll
+            for (int c = 0; c < CH; ++c) x[c] = x[c] + y[c] * p.mul;
+        }
+#pragma unroll
+        for (int c = 0; c < CH; ++c) {
+            const int col = (c * NT + threadIdx.x) * 4;
+            if (col < p.hidden) *(f32x4 *)(p.x + (size_t)t * p.hidden + col) = x[c];
+        }
+    }
+    if (!p.pre.w) return;
+    group_factors<CH, NT>(x, p, unit, sums, r);
+#pragma unroll
+    for (int c = 0; c < CH; ++c) {
+        const int col = (c * NT + threadIdx.x) * 4;
+        if (col < p.hidden) put4<BF16>(p.xn, (size_t)t * p.hidden + col, x[c] * r[c] * wpre[c]);
+    }
+}
+
 struct SideParams {
     const float *z;
     const uint16_t *table;
@@ -140,6 +247,27 @@ __global__ __launch_bounds__(256) void side_gate_kernel(SideParams p) {
 #pragma unroll
     for (int k = 0; k < 4; ++k) v[k] = gelu_tanh(z[k]) * emb[k];
     put4<BF16>(p.out, i, v);
+}
+
+template <bool BF16>
+int launch_group_norm(const PlanNormArgs &p, int T, hipStream_t st) {
+    const int ch = (p.hidden + 1023) / 1024, size = p.width / p.groups;
+    XFT_REQUIRE(ch <= 16, "plan_norm: hidden size %d above 16384", p.hidden);
+    int unit = 0;
+    if (size % 4 == 0)
+        for (unit = 1; unit < 64 && size % (8 * unit) == 0;) unit *= 2;
+    const size_t smem = unit ? (size_t)p.hidden / (4 * unit) * 4 + 16 : (size_t)p.hidden * 4;
+    auto launch = [&](void (*kernel)(PlanNormArgs, int), int threads) { hipLaunchKernelGGL(kernel, dim3(T), dim3(threads), smem, st, p, unit); };
+    if (T <= 64 && ch > 1) {
+        if (ch <= 4) launch(plan_group_norm_kernel<BF16, 1, 1024>, 1024);
+        else launch(plan_group_norm_kernel<BF16, 4, 1024>, 1024);
+    } else if (ch <= 1) launch(plan_group_norm_kernel<BF16, 1, 256>, 256);
+    else if (ch <= 2) launch(plan_group_norm_kernel<BF16, 2, 256>, 256);
+    else if (ch <= 4) launch(plan_group_norm_kernel<BF16, 4, 256>, 256);
+    else if (ch <= 8) launch(plan_group_norm_kernel<BF16, 4, 512>, 512);
+    else launch(plan_group_norm_kernel<BF16, 4, 1024>, 1024);
+    XFT_CHECK_HIP(hipGetLastError());
+    return 0;
 }
 
 template <bool BF16>
@@ -178,6 +306,10 @@ int plan_norm(int act, const PlanNormArgs &p, int T, hipStream_t st) {
     XFT_REQUIRE(T > 0 && p.x && p.hidden % 4 == 0 && p.width <= p.hidden && (!p.rows || (!p.y && !p.table)) && (!p.pre2.w || p.pre.b)
                     && (!p.table || !p.y || p.post),
             "plan_norm: bad argument");
+    if (p.groups > 1 || p.y2) {
+        XFT_REQUIRE(p.width % p.groups == 0 && !p.table && !p.pre.b && !p.pre2.w && (!p.y2 || (p.y && p.mix1 && p.mix2)), "plan_norm: options that do not go together");
+        return act == XFTHIP_BF16 ? launch_group_norm<true>(p, T, st) : launch_group_norm<false>(p, T, st);
+    }
     return act == XFTHIP_BF16 ? launch_norm<true>(p, T, st) : launch_norm<false>(p, T, st);
 }
 

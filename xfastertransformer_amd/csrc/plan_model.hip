@@ -116,16 +116,16 @@ int plan_gemm_in(xfthip_model *m, const PlanLayer &L, int T, hipStream_t st) {
 }
 
 // a sublayer's last product: into y, or, in parallel blocks, added to the residual
-int plan_gemm_out(xfthip_model *m, xfthip_weight_t w, int M, const void *A, int lda, hipStream_t st) {
+int plan_gemm_out(xfthip_model *m, xfthip_weight_t w, int M, const void *A, int lda, const float *bias, hipStream_t st) {
     const PlanState &p = *m->plan;
     const int hidden = m->cfg.hidden;
-    if (p.plan->cfg.block != XFTHIP_BLOCK_PARALLEL) return plan_gemm(m, w, M, A, lda, p.y, hidden, XFTHIP_F32, st);
+    if (p.plan->cfg.block != XFTHIP_BLOCK_PARALLEL) return plan_gemm(m, w, M, A, lda, p.y, hidden, XFTHIP_F32, st, bias);
     if (p.act == XFTHIP_F32) {
         TileGemmArgs a;
-        a.M = M, a.A = A, a.lda = lda, a.C = m->x, a.ldc = hidden, a.add = true;
+        a.M = M, a.A = A, a.lda = lda, a.C = m->x, a.ldc = hidden, a.add = true, a.bias = bias;
         return tile_gemm(w, XFTHIP_F32, a, st);
     }
-    return xfthip_gemm(w, M, A, lda, m->x, hidden, XFTHIP_F32, XFTHIP_EPI_RESIDENTIAL, nullptr, m->x, hidden, XFTHIP_F32, 1.0f, st);
+    return xfthip_gemm(w, M, A, lda, m->x, hidden, XFTHIP_F32, XFTHIP_EPI_RESIDENTIAL, bias, m->x, hidden, XFTHIP_F32, 1.0f, st);
 }
 
 // heads side by side (block_cols output columns a head, a_block_stride input columns apart)
@@ -183,7 +183,7 @@ int run_latent(xfthip_model *m, const PlanLayer &L, int run, const StepView &v, 
         for (auto &s : spans)
             if ((rc = to_values(s.first, s.second))) return rc;
     }
-    return plan_gemm_out(m, L.o, T, p.ov, H * L.V, st);
+    return plan_gemm_out(m, L.o, T, p.ov, H * L.V, nullptr, st);
 }
 
 int mix_delta(xfthip_model *m, const PlanLayer &L, int store, const StepView &v, hipStream_t st) {
@@ -204,7 +204,8 @@ int mix_delta(xfthip_model *m, const PlanLayer &L, int store, const StepView &v,
 int mix_grouped(xfthip_model *m, const PlanLayer &L, int store, const StepView &v, hipStream_t st) {
     PlanState &p = *m->plan;
     int rc;
-    const GroupedBuffers b = {p.a, p.q, p.cache[p.reads[store]], p.first_values};
+    const PageTable &t = p.tables[L.means_table];
+    const GroupedBuffers b = {p.a, p.q, p.cache[p.reads[store]], p.first_values, p.conv_state[store], p.means[store], p.table + t.at, t.stride};
     if ((rc = grouped_prepare(p.act, L, v, b, m->cfg.rms_eps, st))) return rc;
     return grouped_attention(p.act, L, v, b, p.ov, m->len_hint, p.part, p.part_floats, st);
 }
@@ -218,11 +219,21 @@ int mix_unit(xfthip_model *m, const PlanLayer &L, int store, const StepView &v, 
     return unit_scan(p.act, L, v, b, st);
 }
 
+int mix_linear(xfthip_model *m, const PlanLayer &L, int store, const StepView &v, hipStream_t st) {
+    PlanState &p = *m->plan;
+    TileGemmArgs a; // the decays
+    a.M = v.T, a.A = (const char *)p.a + (size_t)(L.in_col + L.channels()) * p.esz, a.lda = L.in_ld, a.block_cols = L.s.heads * L.KD, a.C = p.gates;
+    a.ldc = L.s.heads * L.KD, a.bias = L.dt_bias, a.decay_tau = L.s.tau;
+    if (int rc = tile_gemm(L.gates, p.act, a, st)) return rc;
+    return linear_attention(p.act, L, v, {p.a, p.gates, p.do_, p.ov, p.state[store]}, m->cfg.rms_eps, st);
+}
+
 // between the input and the output product of a mixer
 int mix(xfthip_model *m, const PlanLayer &L, int store, const StepView &v, hipStream_t st) {
     switch (L.s.mixer) {
         case XFTHIP_MIXER_GROUPED: return mix_grouped(m, L, store, v, st);
         case XFTHIP_MIXER_UNIT: return mix_unit(m, L, store, v, st);
+        case XFTHIP_MIXER_LINEAR: return mix_linear(m, L, store, v, st);
         default: return mix_delta(m, L, store, v, st);
     }
 }
@@ -236,17 +247,22 @@ int run_mixers(xfthip_model *m, int run, const StepView &v, hipStream_t st) {
     if ((rc = plan_gemm_in(m, L, v.T, st))) return rc;
     if ((rc = mix(m, L, run, v, st))) return rc;
     if (r.beside >= 0 && (rc = mix(m, p.layers[r.beside], r.beside_store, v, st))) return rc;
-    return plan_gemm_out(m, L.o, v.T, p.ov, L.out_ld, st);
+    if (L.result_norm) { // the results meet behind norms of their own
+        const PlanLayer &S = p.layers[r.beside];
+        if ((rc = plan_gemm(m, S.o, v.T, (const char *)p.ov + (size_t)S.out_col * p.esz, S.out_ld, p.y2, m->cfg.hidden, XFTHIP_F32, st, S.o_bias))) return rc;
+    }
+    return plan_gemm_out(m, L.o, v.T, p.ov, L.out_ld, L.o_bias, st);
 }
 
 // gate and up projections of a dense or shared feed-forward, combined -> h
 int run_gateup(xfthip_model *m, const PlanLayer &L, int T, const void *in, hipStream_t st) {
     PlanState &p = *m->plan;
     const int hidden = m->cfg.hidden;
-    if (p.act != XFTHIP_F32 && L.s.glu_alpha == 0.0f) return xfthip_gemm_gateup_silu(L.gateup, T, in, hidden, p.h, L.ff, XFTHIP_BF16, st);
+    if (p.act != XFTHIP_F32 && L.s.glu_alpha == 0.0f) return xfthip_gemm_gateup_silu_bias(L.gateup, T, in, hidden, p.h, L.ff, XFTHIP_BF16, L.gateup_bias, st);
     if (p.act != XFTHIP_F32) return xfthip_gemm_gateup_clamped(L.gateup, T, in, hidden, p.h, L.ff, XFTHIP_BF16, L.s.glu_limit, L.s.glu_alpha, st);
     TileGemmArgs a;
     a.M = T, a.A = in, a.lda = hidden, a.C = p.h, a.ldc = L.ff, a.c_dtype = XFTHIP_F32, a.glu = true, a.glu_limit = L.s.glu_limit, a.glu_alpha = L.s.glu_alpha;
+    a.bias = L.gateup_bias;
     return tile_gemm(L.gateup, XFTHIP_F32, a, st);
 }
 
@@ -282,7 +298,7 @@ int run_feed_forward(xfthip_model *m, const PlanLayer &L, int T, const void *in,
     int rc;
     if (L.ff > 0) {
         if ((rc = run_gateup(m, L, T, in, st))) return rc;
-        if ((rc = plan_gemm_out(m, L.down, T, p.h, L.ff, st))) return rc;
+        if ((rc = plan_gemm_out(m, L.down, T, p.h, L.ff, L.down_bias, st))) return rc;
     }
     float *dst = parallel ? m->x : p.y;
     if (L.s.experts > 0) {
@@ -324,14 +340,16 @@ int plan_layers(xfthip_model *m, const StepView &v, hipStream_t st) {
     const int nruns = (int)plan.runs.size();
     int rc;
     // next: the layer whose first norms follow, or null
-    auto norm = [&](const float *y, const float *post, bool again, const PlanNorm &pre, const PlanNorm &pre2) {
-        const PlanNormArgs a = {m->x, y, post, again ? plan.embedding : nullptr, p.ids, m->cfg.vocab, pre, pre2, p.xn, p.xn2, nullptr, hidden, plan.cfg.hidden,
-                m->cfg.rms_eps, plan.cfg.residual_mult};
+    // pair: the layer whose mixers' results meet here, or null
+    auto norm = [&](const float *y, const float *post, bool again, const PlanNorm &pre, const PlanNorm &pre2, const PlanLayer *pair) {
+        PlanNormArgs a = {m->x, y, post, again ? plan.embedding : nullptr, p.ids, m->cfg.vocab, pre, pre2, p.xn, p.xn2, nullptr, hidden, plan.cfg.hidden,
+                m->cfg.rms_eps, plan.cfg.residual_mult, plan.cfg.norm_groups};
+        if (pair && pair->result_norm) a.y2 = p.y2, a.mix1 = pair->result_norm, a.mix2 = p.layers[pair->beside].result_norm;
         return plan_norm(p.act, a, T, st);
     };
     const PlanNorm none;
     auto enter = [&](const float *y, const float *post, bool again, const PlanLayer *next) {
-        return norm(y, post, again, next ? next->pre1 : none, next && parallel ? next->pre2 : none);
+        return norm(y, post, again, next ? next->pre1 : none, next && parallel ? next->pre2 : none, nullptr);
     };
     if ((rc = enter(nullptr, nullptr, plan.runs[0].add_embedding, &p.layers[plan.runs[0].layer]))) return rc;
     for (int r = 0; r < nruns; ++r) {
@@ -350,7 +368,7 @@ int plan_layers(xfthip_model *m, const StepView &v, hipStream_t st) {
             if (!last || side)
                 if ((rc = enter(side ? p.y : nullptr, L.side_post, join, then))) return rc;
         } else {
-            if ((rc = norm(p.y, L.post1, !ff && join, ff ? L.pre2 : then ? then->pre1 : none, none))) return rc;
+            if ((rc = norm(p.y, L.post1, !ff && join, ff ? L.pre2 : then ? then->pre1 : none, none, &L))) return rc;
             if (ff) {
                 if ((rc = run_feed_forward(m, L, T, p.xn, nullptr, st))) return rc;
                 if ((rc = enter(p.y, L.post2, join, then))) return rc;
@@ -375,7 +393,7 @@ int upload_table(PlanState &p, hipStream_t st) {
 StepView view_of(const xfthip_model *m, int B, int T, int longest) {
     const PlanState &p = *m->plan;
     const int cap = p.slots;
-    return StepView {B, T, longest, p.tok_seg, p.tok_pos, p.seg, p.seg + cap, p.seg + 2 * cap, p.seg + 3 * cap, p.table, p.table_stride};
+    return StepView {B, T, longest, p.tok_seg, p.tok_pos, p.seg, p.seg + cap, p.seg + 2 * cap, p.seg + 3 * cap, p.table, p.tables[0].stride};
 }
 
 EmbedTables embed_tables(const xfthip_model *m) {
@@ -388,23 +406,26 @@ EmbedTables embed_tables(const xfthip_model *m) {
 
 int plan_reserve(xfthip_model *m, int row, int tokens) {
     PlanState &p = *m->plan;
-    const int need = (tokens + kPageTokens - 1) / kPageTokens;
-    XFT_REQUIRE(need <= p.table_stride, "the sequence of slot %d is longer than the model's %d positions", row, m->cfg.max_seq);
-    while ((int)p.held[row].size() < need) {
-        XFT_REQUIRE(!p.free_pages.empty(), "the page pool (%d pages of %d tokens) is exhausted", p.pages, kPageTokens);
-        const int page = p.free_pages.back();
-        p.free_pages.pop_back();
-        p.table_host[(size_t)row * p.table_stride + p.held[row].size()] = page;
-        p.held[row].push_back(page);
-        p.table_dirty = true;
+    for (PageTable &t : p.tables) {
+        const int need = t.pages_for(tokens);
+        XFT_REQUIRE(need <= t.stride, "the sequence of slot %d is longer than the model's %d positions", row, m->cfg.max_seq);
+        while ((int)t.held[row].size() < need) {
+            XFT_REQUIRE(!t.free_pages.empty(), "the page pool (%d pages of %d entries, %d tokens each) is exhausted", t.pages, kPageTokens, t.unit);
+            const int page = t.free_pages.back();
+            t.free_pages.pop_back();
+            p.table_host[t.at + (size_t)row * t.stride + t.held[row].size()] = page;
+            t.held[row].push_back(page);
+            p.table_dirty = true;
+        }
     }
     return 0;
 }
 
 void plan_release(xfthip_model *m, int row) {
-    PlanState &p = *m->plan;
-    for (size_t i = p.held[row].size(); i-- > 0;) p.free_pages.push_back(p.held[row][i]);
-    p.held[row].clear();
+    for (PageTable &t : m->plan->tables) {
+        for (size_t i = t.held[row].size(); i-- > 0;) t.free_pages.push_back(t.held[row][i]);
+        t.held[row].clear();
+    }
 }
 
 int plan_run(xfthip_model *m, int n, const int *rows, const int *lens, const int *ids, hipStream_t st) {
@@ -467,7 +488,8 @@ int plan_head(xfthip_model *m, const int *rows_dev, int n, int at, hipStream_t s
     PlanState &p = *m->plan;
     const xfthip_plan &plan = *p.plan;
     const xfthip_model_config &c = m->cfg;
-    const PlanNormArgs a = {m->x, nullptr, nullptr, nullptr, nullptr, c.vocab, plan.final_norm, {}, p.xn, nullptr, rows_dev, c.hidden, plan.cfg.hidden, c.rms_eps, 0.0f};
+    const PlanNormArgs a = {m->x, nullptr, nullptr, nullptr, nullptr, c.vocab, plan.final_norm, {}, p.xn, nullptr, rows_dev, c.hidden, plan.cfg.hidden, c.rms_eps, 0.0f,
+            plan.cfg.norm_groups};
     if (int rc = plan_norm(p.act, a, n, st)) return rc;
     float *logits = m->logits + (size_t)at * c.vocab;
     if (int rc = plan_gemm(m, plan.head, n, p.xn, c.hidden, logits, c.vocab, XFTHIP_F32, st)) return rc;
@@ -551,30 +573,46 @@ int plan_decode_splits(xfthip_model *m, int B, int hint) {
 int plan_reorder(xfthip_model *m, const int *dst, const int *src, int n, hipStream_t st) {
     PlanState &p = *m->plan;
     XFT_CHECK_HIP(hipStreamSynchronize(st));
-    std::vector<std::vector<int>> from(n);
-    for (int i = 0; i < n; ++i) from[i] = p.held[src[i]];
-    for (int i = 0; i < n; ++i) {
-        const int have = (int)p.held[dst[i]].size(), want = (int)from[i].size();
-        for (int k = have; k > want; --k) {
-            p.free_pages.push_back(p.held[dst[i]].back());
-            p.held[dst[i]].pop_back();
-        }
+    std::vector<std::vector<std::vector<int>>> from(p.tables.size()); // pages of the sources, by table
+    for (size_t t = 0; t < p.tables.size(); ++t) {
+        PageTable &pt = p.tables[t];
+        for (int i = 0; i < n; ++i) from[t].push_back(pt.held[src[i]]);
+        for (int i = 0; i < n; ++i)
+            while (pt.held[dst[i]].size() > from[t][i].size()) {
+                pt.free_pages.push_back(pt.held[dst[i]].back());
+                pt.held[dst[i]].pop_back();
+            }
     }
     // (a slot whose pages another one reads keeps them: it is a destination itself only if it is listed, with as many or more pages)
-    size_t bytes = 0;
-    const size_t stores = p.store_layer.size();
-    for (size_t r = 0; r < stores; ++r) {
+    // what a record keeps: pages of some table, and so many bytes a slot
+    struct Kept {
+        char *base;
+        int table; // or -1: by slot
+        size_t bytes; // of a page or a slot
+    };
+    auto kept = [&](size_t r) {
         const PlanLayer &L = p.layers[p.store_layer[r]];
-        size_t need = 0;
-        for (int i = 0; i < n; ++i)
-            need += L.paged() ? from[i].size() * kPageTokens * L.token_elems() * p.esz : L.state_floats() * 4 + (size_t)(L.s.taps - 1) * L.channels() * p.esz;
-        bytes = std::max(bytes, need);
-    }
-    bytes = std::max(bytes, (size_t)n * 4);
+        std::vector<Kept> k;
+        if (L.kv_from >= 0) return k; // (what it reads is another record's)
+        const size_t page = kPageTokens * L.token_elems() * p.esz;
+        if (L.paged()) k.push_back({(char *)p.cache[r], 0, page});
+        if (L.means_table) k.push_back({(char *)p.means[r], L.means_table, page});
+        if (L.state_floats()) k.push_back({(char *)p.state[r], -1, L.state_floats() * 4});
+        if (L.history()) k.push_back({(char *)p.conv_state[r], -1, L.history() * p.esz});
+        return k;
+    };
+    size_t bytes = (size_t)n * 4;
+    const size_t stores = p.store_layer.size();
+    for (size_t r = 0; r < stores; ++r)
+        for (const Kept &k : kept(r)) {
+            size_t need = 0;
+            for (int i = 0; i < n; ++i) need += k.bytes * (k.table < 0 ? 1 : from[k.table][i].size());
+            bytes = std::max(bytes, need);
+        }
     char *stage = nullptr;
     XFT_CHECK_HIP(hipMalloc((void **)&stage, bytes + 16));
     int rc = 0;
-    for (int i = 0; i < n && rc == 0; ++i) rc = plan_reserve(m, dst[i], (int)from[i].size() * kPageTokens);
+    for (int i = 0; i < n && rc == 0; ++i) rc = plan_reserve(m, dst[i], (int)from[0][i].size() * kPageTokens);
     if (rc == 0) rc = upload_table(p, st);
     hipError_t e = hipSuccess;
     auto copy = [&](void *d, const void *s, size_t b) {
@@ -585,34 +623,20 @@ int plan_reorder(xfthip_model *m, const int *dst, const int *src, int n, hipStre
             if (write) copy(p.last_token + dst[i], stage + 4 * (size_t)i, 4);
             else copy(stage + 4 * (size_t)i, p.last_token + src[i], 4);
         }
-    for (size_t r = 0; r < stores && rc == 0; ++r) {
-        const PlanLayer &L = p.layers[p.store_layer[r]];
-        if (L.kv_from >= 0) continue; // (what it reads is another record's)
-        for (int write = 0; write < 2; ++write) {
-            size_t at = 0;
-            for (int i = 0; i < n; ++i) {
-                if (L.paged()) {
-                    const size_t page = kPageTokens * L.token_elems() * p.esz;
-                    for (size_t k = 0; k < from[i].size(); ++k, at += page) {
-                        char *pool = (char *)p.cache[r];
-                        if (write) copy(pool + (size_t)p.held[dst[i]][k] * page, stage + at, page);
-                        else copy(stage + at, pool + (size_t)from[i][k] * page, page);
+    for (size_t r = 0; r < stores && rc == 0; ++r)
+        for (const Kept &k : kept(r))
+            for (int write = 0; write < 2; ++write) {
+                size_t at = 0;
+                for (int i = 0; i < n; ++i) {
+                    const size_t count = k.table < 0 ? 1 : from[k.table][i].size();
+                    for (size_t j = 0; j < count; ++j, at += k.bytes) {
+                        const int place = k.table < 0 ? (write ? dst[i] : src[i]) : write ? p.tables[k.table].held[dst[i]][j] : from[k.table][i][j];
+                        char *there = k.base + (size_t)place * k.bytes;
+                        if (write) copy(there, stage + at, k.bytes);
+                        else copy(stage + at, there, k.bytes);
                     }
-                } else {
-                    const size_t sb = L.state_floats() * 4, cb = (size_t)(L.s.taps - 1) * L.channels() * p.esz;
-                    char *state = (char *)p.state[r], *conv = (char *)p.conv_state[r];
-                    if (write) {
-                        copy(state + dst[i] * sb, stage + at, sb);
-                        copy(conv + dst[i] * cb, stage + at + sb, cb);
-                    } else {
-                        copy(stage + at, state + src[i] * sb, sb);
-                        copy(stage + at + sb, conv + src[i] * cb, cb);
-                    }
-                    at += sb + cb;
                 }
             }
-        }
-    }
     if (e == hipSuccess) e = hipStreamSynchronize(st);
     (void)hipFree(stage);
     if (rc) return rc;
@@ -639,7 +663,7 @@ int xfthip_plan_create(const xfthip_plan_config *cfg, const xfthip_plan_layer *l
     const xfthip_plan_config &c = *cfg;
     XFT_REQUIRE(c.layers > 0 && c.hidden > 0 && c.hidden <= 16384 && c.vocab > 0, "xfthip_plan_create: bad sizes");
     const bool loop = c.loop_times > 1 && c.loop_start != c.loop_stop; // (a loop over nothing is none)
-    XFT_REQUIRE((c.block == XFTHIP_BLOCK_SANDWICH && c.norm == XFTHIP_NORM_RMS_ABOUT_ONE && c.side_dim == 0)
+    XFT_REQUIRE((c.block == XFTHIP_BLOCK_SANDWICH && (c.norm == XFTHIP_NORM_RMS_ABOUT_ONE || c.norm == XFTHIP_NORM_RMS) && c.side_dim == 0)
                     || (c.block == XFTHIP_BLOCK_PARALLEL && c.norm == XFTHIP_NORM_DYNAMIC_TANH && c.side_dim >= 0)
                     || (c.block == XFTHIP_BLOCK_SERIAL && c.norm == XFTHIP_NORM_RMS && c.side_dim == 0 && !loop),
             "xfthip_plan_create: block arrangement %d with norm %d and side width %d is not served", c.block, c.norm, c.side_dim);
@@ -647,9 +671,12 @@ int xfthip_plan_create(const xfthip_plan_config *cfg, const xfthip_plan_layer *l
             c.loop_start, c.loop_stop, c.layers);
     XFT_REQUIRE(c.bigram_buckets >= 0 && c.bigram_buckets < (1ll << 31) - 1 && (c.embed_scale == 0.0f || c.embed_scale == 1.0f || !loop) && c.logit_softcap >= 0.0f,
             "xfthip_plan_create: bad embedding or logit constants");
+    XFT_REQUIRE(c.norm_groups >= 0 && (c.norm_groups <= 1 || (c.norm == XFTHIP_NORM_RMS && c.hidden % c.norm_groups == 0 && !loop)),
+            "xfthip_plan_create: %d groups of a norm over %d values", c.norm_groups, c.hidden);
     xfthip_plan *p = new xfthip_plan();
     p->cfg = c;
     if (c.embed_scale == 0.0f) p->cfg.embed_scale = 1.0f;
+    if (c.norm_groups == 0) p->cfg.norm_groups = 1;
     p->hidden = pad32(c.hidden);
     p->side_pad = pad32(c.side_dim);
     int first_mix = -1; // the first layer with mixed values
@@ -671,8 +698,11 @@ int xfthip_plan_create(const xfthip_plan_config *cfg, const xfthip_plan_layer *l
             if (L.rank > 0) L.gcols = s.heads * std::max(L.KD, L.VD);
         } else if (s.mixer == XFTHIP_MIXER_GROUPED) {
             ok = ok && s.kv_heads > 0 && s.heads % s.kv_heads == 0 && s.dim <= 512 && s.vdim <= 512 && s.rot_dim >= 0 && s.rot_dim <= s.dim && s.rot_dim % 2 == 0
-                    && s.window >= 0 && s.chunk >= 0 && !(s.window > 0 && s.chunk > 0) && s.softcap >= 0.0f && s.qk_norm >= 0 && s.qk_norm <= XFTHIP_QK_NORM_ALL
+                    && s.window >= 0 && s.chunk >= 0 && !(s.window > 0 && s.chunk > 0) && s.softcap >= 0.0f && s.qk_norm >= 0 && s.qk_norm <= XFTHIP_QK_NORM_UNIT
                     && s.out_gate >= 0 && s.out_gate <= XFTHIP_GATE_HEAD && (!s.key_values || (s.dim == s.vdim && !s.v_mix)) && (s.rot_factor <= 0.0 || (s.rot_original > 0.0 && s.rot_fast > 0.0 && s.rot_slow > 0.0));
+            ok = ok && s.taps >= 0 && (s.taps == 0 || (s.qk_norm != XFTHIP_QK_NORM_ALL && !s.v_mix && !s.key_values && s.kv_from == 0))
+                    && s.keep_first >= 0 && s.pool >= 0 && ((s.keep_first == 0 && s.pool == 0) || s.window > 0) && !(s.keep_first > 0 && s.pool > 0) && !(s.pool > 0 && s.distance_bias)
+                    && !(s.pool > 0 && s.kv_from != 0) && (!s.v_rot || (s.vdim % 2 == 0 && s.rot_base > 0.0 && !s.key_values && !s.v_mix && s.kv_from == 0));
             L.D = pad32(s.dim), L.V = pad32(s.vdim);
             if (ok && s.v_mix) {
                 L.first_values = first_mix < 0;
@@ -683,15 +713,24 @@ int xfthip_plan_create(const xfthip_plan_config *cfg, const xfthip_plan_layer *l
             if (ok && s.kv_from != 0) { // a record before this one with keys and values of its own and of the same shape
                 ok = s.kv_from > 0 && s.kv_from <= i && !loop && !s.v_mix;
                 const xfthip_plan_layer &f = layers[ok ? s.kv_from - 1 : 0];
-                ok = ok && f.mixer == XFTHIP_MIXER_GROUPED && f.kv_from == 0 && f.kv_heads == s.kv_heads && f.dim == s.dim && f.vdim == s.vdim;
+                ok = ok && f.mixer == XFTHIP_MIXER_GROUPED && f.kv_from == 0 && f.kv_heads == s.kv_heads && f.dim == s.dim && f.vdim == s.vdim && !f.v_rot;
+                const bool moved = s.rot_dim > 0 && !s.rot_interleaved, f_moved = f.rot_dim > 0 && !f.rot_interleaved; // (and the same order of dimensions)
+                ok = ok && moved == f_moved && (!moved || s.rot_dim == f.rot_dim);
                 if (ok) L.kv_from = s.kv_from - 1;
             }
         } else if (s.mixer == XFTHIP_MIXER_UNIT) {
             ok = ok && s.taps >= 1;
             L.D = pad32(s.dim);
+        } else if (s.mixer == XFTHIP_MIXER_LINEAR) {
+            ok = ok && s.dim <= 256 && s.taps <= 1 && s.decay_rank > 0 && s.gate_rank == 0 && s.tau > 0.0f;
+            L.KD = 32;
+            while (L.KD < s.dim) L.KD *= 2;
+            L.VD = pad32(s.vdim), L.rank = pad32(s.decay_rank);
         } else {
             ok = false;
         }
+        ok = ok && (!s.o_bias || (s.mixer == XFTHIP_MIXER_GROUPED && (!s.beside || s.result_norm))) && (!s.mlp_bias || (s.inter > 0 && s.experts == 0 && s.glu_alpha == 0.0f))
+                && (!s.result_norm || c.block != XFTHIP_BLOCK_PARALLEL);
         L.ff = pad32(s.inter);
         if (s.experts > 0) {
             ok = ok && s.identity >= 0 && s.top > 0 && s.top <= L.routes() && s.top <= 64 && L.routes() <= 1024 && s.expert_inter > 0 && s.glu_alpha >= 0.0f;
@@ -701,11 +740,11 @@ int xfthip_plan_create(const xfthip_plan_config *cfg, const xfthip_plan_layer *l
             else ok = ok && s.router == XFTHIP_ROUTE_SOFTMAX;
             L.eff = pad32(s.expert_inter);
         }
-        if (s.scaled) L.mix_scale = s.mix_scale;
+        if (s.scaled && !s.result_norm) L.mix_scale = s.mix_scale;
         L.in_ld = L.row_in(), L.out_ld = L.out_cols();
         if (s.beside) { // joins the layer before it, whose projections it continues
             ok = ok && i > 0 && !loop && !layers[i - 1].beside && layers[i - 1].mixer != XFTHIP_MIXER_LATENT && s.mixer != XFTHIP_MIXER_LATENT && s.inter == 0
-                    && s.experts == 0;
+                    && s.experts == 0 && !s.result_norm == !layers[i - 1].result_norm && (s.result_norm || !layers[i - 1].o_bias);
             if (ok) {
                 PlanLayer &f = p->layers[i - 1];
                 f.beside = i;
@@ -713,6 +752,7 @@ int xfthip_plan_create(const xfthip_plan_config *cfg, const xfthip_plan_layer *l
                 f.in_ld = L.in_ld += f.in_ld, f.out_ld = L.out_ld += f.out_ld;
             }
         }
+        if (s.result_norm && !s.beside) ok = ok && i + 1 < c.layers && layers[i + 1].beside;
         if (!ok) {
             delete p;
             XFT_REQUIRE(false, "xfthip_plan_create: layer %d has sizes this library does not serve", i);
@@ -742,8 +782,9 @@ int xfthip_plan_destroy(xfthip_plan_t p) {
         for (auto *list : {&L.egateup, &L.edown})
             for (xfthip_weight_t w : *list) xfthip_weight_destroy(w);
         for (float *f : {L.q_norm, L.kv_norm, L.sink, L.conv, L.decay, L.dt_bias, L.out_norm, L.pre1.w, L.pre1.b, L.pre2.w, L.pre2.b, L.post1, L.post2, L.correction,
-                     L.side_post, L.in_bias, L.conv_bias, L.lambda, L.gate_bias})
+                     L.side_post, L.in_bias, L.conv_bias, L.lambda, L.gate_bias, L.o_bias, L.gateup_bias, L.down_bias, L.result_norm})
             if (f) (void)hipFree(f);
+        if (L.filter) (void)hipFree(L.filter);
         if (L.etable) (void)hipFree(L.etable);
     }
     xfthip_weight_destroy(p->head);
@@ -811,6 +852,13 @@ int xfthip_plan_finish(xfthip_plan_t p) {
         for (int v = 0; v < t.rows; ++v)
             for (int k = 0; k < parts; ++k) memcpy(&table[((size_t)v * parts + k) * pad], &t.data[((size_t)v * parts + k) * width], (size_t)width * 2);
         if (hipMalloc((void **)dst, table.size() * 2 + 16) != hipSuccess || hipMemcpy(*dst, table.data(), table.size() * 2, hipMemcpyHostToDevice) != hipSuccess) {
+            set_error("xfthip_plan_finish: upload failed");
+            rc = 1;
+        }
+    };
+    auto upload_bits = [&](const std::vector<uint16_t> &v, uint16_t **dst) {
+        if (rc) return;
+        if (hipMalloc((void **)dst, v.size() * 2 + 16) != hipSuccess || hipMemcpy(*dst, v.data(), v.size() * 2, hipMemcpyHostToDevice) != hipSuccess) {
             set_error("xfthip_plan_finish: upload failed");
             rc = 1;
         }
@@ -894,35 +942,56 @@ int xfthip_plan_finish(xfthip_plan_t p) {
             } else if (s.mixer == XFTHIP_MIXER_GROUPED) {
                 const int G = s.kv_heads, d = s.dim, dv = s.vdim, k0 = c0 + H * L.D, v0 = c0 + L.value_col(), g0 = c0 + L.gate_col();
                 const bool own = L.kv_from < 0;
-                // a projection of n heads of width w, each padded to `pad` columns from c on
-                auto project = [&](const char *name, int n, int w, int pad, int c, bool with_bias) {
+                // where the dimensions of a head are kept
+                std::vector<int> same, head, value;
+                for (int x = 0; x < std::max(d, dv); ++x) same.push_back(x), head.push_back(L.head_place(x)), value.push_back(L.value_place(x));
+                std::vector<uint16_t> filter(L.filters() ? (size_t)s.taps * L.channels() : 0, 0);
+                // a projection of n heads of width w, each padded to `pad` columns from c on, with its bias and filters
+                auto project = [&](const char *name, int n, int w, int pad, int c, const std::vector<int> &place, bool with_bias, bool with_filter) {
                     const Tensor &t = get(name, n * w, W);
                     if (!missing.empty()) return;
-                    for (int h = 0; h < n; ++h) in.place(t, h * w, w, 0, W, 0, c + h * pad);
-                    if (!with_bias) return;
-                    const Tensor &b = get((std::string(name) + ".b").c_str(), n * w, 1);
-                    if (!missing.empty()) return;
-                    for (int x = 0; x < n * w; ++x) bias[c + x / w * pad + x % w] = bf16_value(b.data[x]);
-                    biased = true;
+                    const bool in_order = std::equal(place.begin(), place.begin() + w, same.begin());
+                    for (int h = 0; h < n && in_order; ++h) in.place(t, h * w, w, 0, W, 0, c + h * pad);
+                    for (int x = 0; x < n * w && !in_order; ++x) in.place(t, x, 1, 0, W, 0, c + x / w * pad + place[x % w]);
+                    if (with_bias) {
+                        const Tensor &b = get((std::string(name) + ".b").c_str(), n * w, 1);
+                        if (!missing.empty()) return;
+                        for (int x = 0; x < n * w; ++x) bias[c + x / w * pad + place[x % w]] = bf16_value(b.data[x]);
+                        biased = true;
+                    }
+                    if (with_filter) {
+                        const Tensor &f = get((std::string(name) + ".conv").c_str(), n * w, s.taps);
+                        if (!missing.empty()) return;
+                        for (int x = 0; x < n * w; ++x)
+                            for (int j = 0; j < s.taps; ++j) filter[(size_t)j * L.channels() + c - c0 + x / w * pad + place[x % w]] = f.data[(size_t)x * s.taps + j];
+                    }
                 };
-                project("mix.q", H, d, L.D, c0, s.qkv_bias);
-                if (own) project("mix.k", G, d, L.D, k0, s.qkv_bias);
-                if (own && !s.key_values) project("mix.v", G, dv, L.V, v0, s.qkv_bias);
-                if (s.out_gate == XFTHIP_GATE_ELEMENT) project("mix.g", H, dv, L.V, g0, false);
-                if (s.out_gate == XFTHIP_GATE_HEAD) project("mix.g", H, 1, 1, g0, false);
+                project("mix.q", H, d, L.D, c0, head, s.qkv_bias, L.filters());
+                if (own) project("mix.k", G, d, L.D, k0, head, s.qkv_bias, L.filters());
+                if (own && !s.key_values) project("mix.v", G, dv, L.V, v0, value, s.qkv_bias, L.filters());
+                if (s.out_gate == XFTHIP_GATE_ELEMENT) project("mix.g", H, dv, L.V, g0, value, false, false);
+                if (s.out_gate == XFTHIP_GATE_HEAD) project("mix.g", H, 1, 1, g0, same, false, false);
                 NEED(o, "mix.o", W, H * dv);
-                for (int h = 0; h < H; ++h) mo.place(o, 0, W, h * dv, dv, r0 + h * L.V, 0);
+                for (int h = 0; h < H; ++h)
+                    for (int x = 0; x < dv; ++x) mo.place(o, 0, W, h * dv + x, 1, r0 + h * L.V + value[x], 0);
+                auto spread = [&](const Tensor &t, int n) {
+                    std::vector<float> v((size_t)n * L.D, 0.0f);
+                    for (int x = 0; x < n * d; ++x) v[(size_t)(x / d) * L.D + head[x % d]] = bf16_value(t.data[x]);
+                    return v;
+                };
+                if (L.filters()) upload_bits(filter, &L.filter);
+                if (s.o_bias) {
+                    NEED(ob, "mix.o.b", W, 1);
+                    std::vector<float> v = values(ob, Wp);
+                    for (float &f : v) f *= L.mix_scale;
+                    upload(v, &L.o_bias);
+                }
                 if (s.qk_norm == XFTHIP_QK_NORM_HEAD) {
                     NEED(qn, "mix.q.norm", d, 1);
                     NEED(kn, "mix.k.norm", d, 1);
-                    upload(values(qn, L.D), &L.q_norm);
-                    upload(values(kn, L.D), &L.kv_norm);
+                    upload(spread(qn, 1), &L.q_norm);
+                    upload(spread(kn, 1), &L.kv_norm);
                 } else if (s.qk_norm == XFTHIP_QK_NORM_ALL) {
-                    auto spread = [&](const Tensor &t, int n) {
-                        std::vector<float> v((size_t)n * L.D, 0.0f);
-                        for (int x = 0; x < n * d; ++x) v[(size_t)(x / d) * L.D + x % d] = bf16_value(t.data[x]);
-                        return v;
-                    };
                     NEED(qn, "mix.q.norm", H * d, 1);
                     upload(spread(qn, H), &L.q_norm);
                     if (own) {
@@ -975,6 +1044,32 @@ int xfthip_plan_finish(xfthip_plan_t p) {
                 biased = true;
                 pack(gt, XFTHIP_WF_NONE, &L.gates);
                 upload(conv, &L.conv), upload(conv_bias, &L.conv_bias), upload(lambda, &L.lambda), upload(gate_bias, &L.gate_bias);
+            } else if (s.mixer == XFTHIP_MIXER_LINEAR) {
+                const int d = s.dim, dv = s.vdim, k0 = H * L.KD, v0 = 2 * H * L.KD, a0 = c0 + L.channels(), g0 = a0 + L.rank;
+                NEED(q, "mix.q", H * d, W);
+                NEED(k, "mix.k", H * d, W);
+                NEED(v, "mix.v", H * dv, W);
+                NEED(g, "mix.g", H * dv, W);
+                NEED(a1, "mix.a1", s.decay_rank, W);
+                NEED(a2, "mix.a2", H * d, s.decay_rank);
+                NEED(ab, "mix.a2.b", H * d, 1);
+                NEED(nm, "mix.norm", dv, 1);
+                NEED(o, "mix.o", W, H * dv);
+                std::vector<float> ab_values((size_t)H * L.KD, 0.0f);
+                Matrix gt(L.rank, H * L.KD);
+                for (int h = 0; h < H; ++h) {
+                    in.place(q, h * d, d, 0, W, 0, c0 + h * L.KD);
+                    in.place(k, h * d, d, 0, W, 0, c0 + k0 + h * L.KD);
+                    in.place(v, h * dv, dv, 0, W, 0, c0 + v0 + h * L.VD);
+                    in.place(g, h * dv, dv, 0, W, 0, g0 + h * L.VD);
+                    mo.place(o, 0, W, h * dv, dv, r0 + h * L.VD, 0);
+                    gt.place(a2, h * d, d, 0, s.decay_rank, 0, h * L.KD);
+                    for (int e = 0; e < d; ++e) ab_values[(size_t)h * L.KD + e] = bf16_value(ab.data[(size_t)h * d + e]);
+                }
+                in.place(a1, 0, s.decay_rank, 0, W, 0, a0);
+                pack(gt, XFTHIP_WF_NONE, &L.gates);
+                upload(ab_values, &L.dt_bias);
+                upload(values(nm, L.VD), &L.out_norm);
             } else {
                 const int KH = s.kv_heads, d = s.dim, dv = s.vdim, n = s.taps;
                 NEED(q, "mix.q", KH * d, W);
@@ -1034,6 +1129,12 @@ int xfthip_plan_finish(xfthip_plan_t p) {
                 upload(dec, &L.decay);
                 upload(values(nm, L.VD), &L.out_norm);
             }
+            if (s.result_norm) {
+                NEED(rn, "mix.out", W, 1);
+                std::vector<float> v = values(rn, Wp);
+                for (float &f : v) f *= s.scaled ? s.mix_scale : 1.0f;
+                upload(v, &L.result_norm);
+            }
         } while (false);
     };
     do {
@@ -1061,7 +1162,14 @@ int xfthip_plan_finish(xfthip_plan_t p) {
         front("norm1", 1.0f, &L.pre1);
         if (L.feeds_forward()) front("norm2", 1.0f, &L.pre2);
         if (!missing.empty()) break;
-        if (sandwich) {
+        if (sandwich && p->cfg.norm == XFTHIP_NORM_RMS) { // no further scale
+            NEED(n1b, "norm1b", W, 1);
+            upload(values(n1b, Wp), &L.post1);
+            if (L.feeds_forward()) {
+                NEED(n2b, "norm2b", W, 1);
+                upload(values(n2b, Wp), &L.post2);
+            }
+        } else if (sandwich) {
             NEED(n1b, "norm1b", W, 1);
             NEED(ls1, "ls1", W, 1);
             upload(one_plus(n1b, &ls1), &L.post1);
@@ -1078,6 +1186,14 @@ int xfthip_plan_finish(xfthip_plan_t p) {
             NEED(down, (at + "down").c_str(), W, s.inter);
             gate_up(gate, up, s.inter, L.ff, &L.gateup);
             plain(down, L.ff, Wp, &L.down);
+            if (s.mlp_bias) {
+                NEED(gb, (at + "gate.b").c_str(), s.inter, 1);
+                NEED(ub, (at + "up.b").c_str(), s.inter, 1);
+                NEED(db, (at + "down.b").c_str(), W, 1);
+                std::vector<float> v = values(gb, L.ff), u = values(ub, L.ff);
+                v.insert(v.end(), u.begin(), u.end());
+                upload(v, &L.gateup_bias), upload(values(db, Wp), &L.down_bias);
+            }
         }
         if (s.experts > 0) {
             NEED(router, "mlp.router", L.routes(), W);
@@ -1125,7 +1241,16 @@ int xfthip_plan_finish(xfthip_plan_t p) {
         }
         if (!missing.empty() || rc) break;
         pack(in, XFTHIP_WF_NONE, &L.in);
-        pack(mo, XFTHIP_WF_NONE, &L.o);
+        if (s.result_norm) { // an output product each: rows of the common one
+            for (int k : {i, L.beside}) {
+                PlanLayer &own = p->layers[k];
+                Matrix part(own.out_cols(), Wp);
+                memcpy(part.w.data(), &mo.w[(size_t)own.out_col * Wp], part.w.size() * 2);
+                pack(part, XFTHIP_WF_NONE, &own.o);
+            }
+        } else {
+            pack(mo, XFTHIP_WF_NONE, &L.o);
+        }
         if (biased) upload(bias, &L.in_bias);
     } while (false);
 #undef NEED
@@ -1151,11 +1276,24 @@ int xfthip_model_create_from_plan(xfthip_plan_t plan, int act_dtype, int max_bat
     PlanState *p = new PlanState();
     m->plan = p;
     p->plan = plan, p->layers = plan->layers, p->act = act_dtype, p->esz = act_dtype == XFTHIP_F32 ? 4 : 2, p->slots = max_batch;
-    p->table_stride = (max_seq + kPageTokens - 1) / kPageTokens;
-    p->pages = pool_tokens > 0 ? (pool_tokens + kPageTokens - 1) / kPageTokens : max_batch * p->table_stride;
-    for (int i = p->pages; i-- > 0;) p->free_pages.push_back(i);
-    p->held.resize(max_batch);
-    p->table_host.assign((size_t)max_batch * p->table_stride, 0);
+    // a table of tokens, and one for every size of block whose means some layer keeps
+    auto add_table = [&](int unit) {
+        for (size_t t = 1; t < p->tables.size(); ++t)
+            if (p->tables[t].unit == unit) return (int)t;
+        PageTable t;
+        t.unit = unit, t.at = p->table_host.size();
+        t.stride = std::max(t.pages_for(max_seq), 1);
+        if (p->tables.empty()) t.pages = pool_tokens > 0 ? (pool_tokens + kPageTokens - 1) / kPageTokens : max_batch * t.stride;
+        else t.pages = std::min(p->tables[0].pages / unit + max_batch, max_batch * t.stride); // (every slot may end in a part of a page)
+        for (int i = t.pages; i-- > 0;) t.free_pages.push_back(i);
+        t.held.resize(max_batch);
+        p->table_host.resize(t.at + (size_t)max_batch * t.stride, 0);
+        p->tables.push_back(t);
+        return (int)p->tables.size() - 1;
+    };
+    add_table(1);
+    for (PlanLayer &L : p->layers)
+        if (L.s.mixer == XFTHIP_MIXER_GROUPED && L.s.pool > 0) L.means_table = add_table(L.s.pool);
     p->logit_of_row.resize(max_batch);
     for (int r = 0; r < max_batch; ++r) p->logit_of_row[r] = r;
     p->logit_rows = std::max(max_batch, 64);
@@ -1171,12 +1309,14 @@ int xfthip_model_create_from_plan(xfthip_plan_t plan, int act_dtype, int max_bat
         memcpy(dst, &b, sizeof(b));
     };
     const size_t T = max_tokens, e = p->esz, hidden = plan->hidden;
+    bool normed_results = false;
     size_t a = 0, cq = 0, q = 0, qa = 0, ov = 0, h = 0, gates = 0, dk = 0, dqk = 0, dg = 0, dv = 0, heads = 0, fv = 0, u = 0, carry = 0;
     size_t top = 0, experts = 0, routes = 0, eh = 0, eo = 0;
     for (const PlanLayer &L : p->layers) {
         const size_t H = L.s.heads;
         a = std::max(a, (size_t)L.in_ld), ov = std::max(ov, (size_t)L.out_ld);
         h = std::max(h, (size_t)L.ff);
+        normed_results = normed_results || L.s.result_norm;
         if (L.s.experts > 0) {
             const size_t most = std::min(L.s.top, L.s.experts);
             top = std::max(top, (size_t)L.s.top), experts = std::max(experts, (size_t)L.s.experts), routes = std::max(routes, (size_t)pad32(L.routes()));
@@ -1188,6 +1328,8 @@ int xfthip_model_create_from_plan(xfthip_plan_t plan, int act_dtype, int max_bat
         } else if (L.s.mixer == XFTHIP_MIXER_UNIT) {
             gates = std::max(gates, (size_t)2 * L.channels()), u = std::max(u, (size_t)L.channels());
             carry = std::max(carry, unit_carry_floats(L, max_tokens, max_batch));
+        } else if (L.s.mixer == XFTHIP_MIXER_LINEAR) {
+            gates = std::max(gates, H * L.KD), dv = std::max(dv, H * L.VD);
         } else if (L.s.mixer == XFTHIP_MIXER_LATENT) {
             cq = std::max(cq, (size_t)L.QR), q = std::max(q, H * (L.D + L.RD)), qa = std::max(qa, H * L.R);
         } else {
@@ -1198,6 +1340,7 @@ int xfthip_model_create_from_plan(xfthip_plan_t plan, int act_dtype, int max_bat
     }
     alloc(&p->xn, std::max(T, (size_t)p->logit_rows) * hidden * e);
     alloc(&p->y, T * hidden * 4);
+    if (normed_results) alloc(&p->y2, T * hidden * 4);
     alloc(&p->a, T * a * e), alloc(&p->cq, T * cq * e), alloc(&p->q, T * q * e), alloc(&p->qa, T * qa * e), alloc(&p->oc, T * qa * e);
     alloc(&p->ov, T * ov * e), alloc(&p->h, T * h * e), alloc(&p->u, T * u * e);
     alloc(&p->carry, carry * 4), alloc(&p->last_token, (size_t)max_batch * 4, true);
@@ -1227,37 +1370,47 @@ int xfthip_model_create_from_plan(xfthip_plan_t plan, int act_dtype, int max_bat
         if (r.beside >= 0) p->store_layer.push_back(r.beside);
     for (size_t k = 0; k < p->store_layer.size(); ++k) {
         const PlanLayer &L = p->layers[p->store_layer[k]];
-        void *pool = nullptr;
+        void *pool = nullptr, *means = nullptr;
         float *state = nullptr;
         void *conv = nullptr;
         int from = (int)k;
         if (L.kv_from >= 0) {
             for (from = 0; p->store_layer[from] != L.kv_from;) ++from;
-        } else if (L.paged()) {
-            // cleared: keys that lie behind a sequence's end are multiplied by zero weights and must be numbers
-            alloc(&pool, (size_t)p->pages * kPageTokens * L.token_elems() * e, true);
         } else {
-            alloc(&state, (size_t)max_batch * L.state_floats() * 4, true);
-            alloc(&conv, (size_t)max_batch * (L.s.taps - 1) * L.channels() * e, true);
+            // cleared: keys that lie behind a sequence's end are multiplied by zero weights and must be numbers
+            const size_t page = kPageTokens * L.token_elems() * e;
+            if (L.paged()) alloc(&pool, p->tables[0].pages * page, true);
+            if (L.means_table) alloc(&means, p->tables[L.means_table].pages * page, true);
+            if (L.state_floats()) alloc(&state, (size_t)max_batch * L.state_floats() * 4, true);
+            if (L.history()) alloc(&conv, max_batch * L.history() * e, true);
         }
-        p->reads.push_back(from), p->cache.push_back(pool), p->state.push_back(state), p->conv_state.push_back(conv);
+        p->reads.push_back(from), p->cache.push_back(pool), p->state.push_back(state), p->conv_state.push_back(conv), p->means.push_back(means);
     }
     alloc(&p->table, p->table_host.size() * 4, true);
     alloc(&p->desc, (3 * T + 4 * (size_t)max_batch) * 4, true);
     alloc(&p->dec_rows, (size_t)max_batch * 4, true);
     alloc(&p->want, (size_t)p->logit_rows * 4, true);
     std::map<std::vector<double>, std::pair<float *, float *>> rot; // layers of the same rotation share its tables
-    for (PlanLayer &L : p->layers) {
-        if (!L.paged() || L.s.rot_dim == 0 || !ok) continue;
-        const bool extended = L.s.rot_factor > 0.0;
-        auto &t = rot[{L.s.rot_base, (double)L.s.rot_dim, extended ? L.s.rot_factor : 0.0, extended ? L.s.rot_original : 0.0, extended ? L.s.rot_fast : 0.0,
-                extended ? L.s.rot_slow : 0.0}];
+    auto tables_of = [&](const xfthip_plan_layer &s, float **cosT, float **sinT) {
+        const bool extended = s.rot_factor > 0.0;
+        auto &t = rot[{s.rot_base, (double)s.rot_dim, extended ? s.rot_factor : 0.0, extended ? s.rot_original : 0.0, extended ? s.rot_fast : 0.0,
+                extended ? s.rot_slow : 0.0}];
         if (!t.first) {
-            ok = rotation_tables(L.s, max_seq, &t.first, &t.second) == 0;
+            ok = rotation_tables(s, max_seq, &t.first, &t.second) == 0;
             if (t.first) p->owned.push_back(t.first);
             if (t.second) p->owned.push_back(t.second);
         }
-        L.cosT = t.first, L.sinT = t.second;
+        *cosT = t.first, *sinT = t.second;
+    };
+    for (PlanLayer &L : p->layers) {
+        if (!L.paged() || L.s.rot_dim == 0 || !ok) continue;
+        tables_of(L.s, &L.cosT, &L.sinT);
+    }
+    for (PlanLayer &L : p->layers) {
+        if (L.s.mixer != XFTHIP_MIXER_GROUPED || !L.s.v_rot || !ok) continue;
+        xfthip_plan_layer values = L.s;
+        values.rot_dim = L.s.vdim, values.rot_factor = 0.0;
+        tables_of(values, &L.cosV, &L.sinV);
     }
     ok = ok && hipHostMalloc((void **)&p->desc_host, (3 * T + 5 * (size_t)max_batch + p->logit_rows + p->table_host.size()) * 4) == hipSuccess
             && hipHostMalloc((void **)&p->logits_pinned, (size_t)p->logit_rows * plan->cfg.vocab * 4) == hipSuccess;
@@ -1304,8 +1457,8 @@ int xfthip_model_read_residual(xfthip_model_t m, float *out_host, int *runs, int
 
 int xfthip_model_pool_pages(xfthip_model_t m, int *free_pages, int *total_pages) {
     XFT_REQUIRE(m && m->plan, "xfthip_model_pool_pages: only for models from a plan");
-    if (free_pages) *free_pages = (int)m->plan->free_pages.size();
-    if (total_pages) *total_pages = m->plan->pages;
+    if (free_pages) *free_pages = (int)m->plan->tables[0].free_pages.size();
+    if (total_pages) *total_pages = m->plan->tables[0].pages;
     return 0;
 }
 

@@ -21,7 +21,7 @@ struct SkinnyParams {
     void *C;
     int ldc, c_dtype;
     int epi;
-    const float *bias;
+    const float *bias; // [N]; gateup: of the gate columns, behind them of the others
     const void *res;
     int ldres, res_dtype;
     float gamma;

@@ -749,11 +749,12 @@ __global__ __launch_bounds__(256 * KG, (DIRECT && KG == 1) ? 2 : 1) void qgemm_m
     };
     if (p.gateup) {
         // packed columns alternate 16 gate / 16 up: lanes nl < 16 hold gate, nl >= 16 the matching up
-        float s[WN], z[WN];
+        float s[WN], z[WN], bv[WN];
 #pragma unroll
         for (int t = 0; t < WN; ++t) {
-            const int np = (n32_0 + t) * 32 + nl;
+            const int np = (n32_0 + t) * 32 + nl, col = (n32_0 + t) * 16 + (nl & 15);
             s[t] = 1.0f, z[t] = 0.0f;
+            bv[t] = p.bias && col < p.N / 2 ? p.bias[(nl < 16 ? 0 : p.N / 2) + col] : 0.0f;
             if constexpr (KIND != XFTHIP_W_BF16) s[t] = p.scale[np < p.NTILES * 16 ? np : 0];
             if constexpr (KIND == XFTHIP_W_UINT4 || (KIND == XFTHIP_W_INT8 && NEED_SUM)) z[t] = p.zero ? p.zero[np < p.NTILES * 16 ? np : 0] : 0.0f;
         }
@@ -775,6 +776,7 @@ __global__ __launch_bounds__(256 * KG, (DIRECT && KG == 1) ? 2 : 1) void qgemm_m
                     } else if constexpr (KIND == XFTHIP_W_NF4) {
                         x = s[t] * x;
                     }
+                    x += bv[t];
                     const float other = __shfl_xor(x, 16, 64); // gate <-> up partner
                     put_at(put_base, 16 * t, j, p.gateup == 2 ? clamped_glu(x, other, p.glu_limit, p.glu_alpha) : other * silu_big(x));
                 }

@@ -604,8 +604,9 @@ __global__ __launch_bounds__(512, (STAGE && MT == 1 && NT == 1) ? 4 : 1) void qg
                 const int out_col = (blk * PAIRS + pr) * 16 + c;
                 if (m >= p.M || out_col >= p.N / 2) continue;
                 const float sumA = need_sum ? total_sum(m) : 0.0f;
-                const float gate = column_value(m, pr * 32 + c, sumA);
-                const float up = column_value(m, pr * 32 + 16 + c, sumA);
+                float gate = column_value(m, pr * 32 + c, sumA);
+                float up = column_value(m, pr * 32 + 16 + c, sumA);
+                if (p.bias) gate += p.bias[out_col], up += p.bias[p.N / 2 + out_col];
                 const float y = p.gateup == 2 ? clamped_glu(gate, up, p.glu_limit, p.glu_alpha) : up * silu_f(gate);
                 store_from_f32(p.C, p.c_dtype, (size_t)m * p.ldc + out_col, y);
             }

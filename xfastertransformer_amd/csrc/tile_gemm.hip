@@ -17,6 +17,7 @@ struct TileGemm {
     int ldc, c_dtype, glu, add;
     float glu_limit, glu_alpha;
     const float *bias;
+    float decay; // 1 / decay_tau, or 0
     const uint16_t *side;
     int side_ld, side_vocab;
     const int *side_ids;
@@ -29,6 +30,10 @@ __device__ inline float precise_glu(float gate, float up, float limit, float alp
     const float g = fminf(gate, limit), u = fminf(fmaxf(up, -limit), limit);
     return g / (1.0f + expf(-alpha * g)) * (u + 1.0f);
 }
+
+// sigmoid(z)^power
+template <bool FAST>
+__device__ inline float decay_of(float z, float power) { return exp_of<FAST>(-power * softplus_of<FAST>(-z)); }
 
 // A wave: TW column tiles (16 weight columns each; two, or one in the 16-wave form) x MT row tiles (16 activation rows each).  The weight tile is the MFMA
 // A operand, the activation rows the B operand: a lane ends up with four neighbouring columns of one row.  With fp32
@@ -156,6 +161,7 @@ __global__ __launch_bounds__(KS > 4 ? 64 * KS : 256) void tile_gemm_kernel(TileG
         if (r >= p.M || n >= p.N) return;
         const size_t at = (size_t)r * p.ldc + n;
         if (p.bias) y += p.bias[n];
+        if (p.decay > 0.0f) y = decay_of<!F32>(y, p.decay);
         if (p.side) y = gelu_tanh(y) * side_value;
         if (p.add) y += ((const float *)p.C)[at];
         store_from_f32(p.C, p.c_dtype, at, y);
@@ -186,8 +192,9 @@ __global__ __launch_bounds__(KS > 4 ? 64 * KS : 256) void tile_gemm_kernel(TileG
 #pragma unroll
                 for (int i = 0; i < 4; ++i) {
                     const int n = (nt0 >> 1) * 16 + 4 * g + i;
-                    if (n < p.N / 2)
-                        store_from_f32(p.C, p.c_dtype, (size_t)r * p.ldc + n, precise_glu(acc[0][m][i], acc[1][m][i], p.glu_limit, p.glu_alpha));
+                    if (n >= p.N / 2) continue;
+                    const float gate = acc[0][m][i] + (p.bias ? p.bias[n] : 0.0f), up = acc[1][m][i] + (p.bias ? p.bias[p.N / 2 + n] : 0.0f);
+                    store_from_f32(p.C, p.c_dtype, (size_t)r * p.ldc + n, precise_glu(gate, up, p.glu_limit, p.glu_alpha));
                 }
                 continue;
             }
@@ -200,11 +207,12 @@ __global__ __launch_bounds__(KS > 4 ? 64 * KS : 256) void tile_gemm_kernel(TileG
 #pragma unroll
             for (int t = 0; t < 2; ++t) {
                 const int n = (nt0 + t) * 16 + 4 * g;
-                if (side || p.add || p.bias) {
+                if (side || p.add || p.bias || p.decay > 0.0f) {
 #pragma unroll
                     for (int i = 0; i < 4; ++i) {
                         if (n + i >= p.N) continue;
                         if (p.bias) acc[t][m][i] += p.bias[n + i];
+                        if (p.decay > 0.0f) acc[t][m][i] = decay_of<!F32>(acc[t][m][i], p.decay);
                         if (side) acc[t][m][i] = gelu_tanh(acc[t][m][i]) * bf16_to_f32(side[n + i]);
                         if (p.add) acc[t][m][i] += ((const float *)p.C)[(size_t)r * p.ldc + n + i];
                     }
@@ -237,11 +245,12 @@ int tile_gemm(xfthip_weight_t w, int act_in, const TileGemmArgs &a, hipStream_t 
     const int blocks = a.block_cols ? (pw.N + a.block_cols - 1) / a.block_cols : 1;
     XFT_REQUIRE((long)(blocks - 1) * a.a_block_stride + pw.K <= a.lda, "tile_gemm: %d blocks of K=%d reach past the row (%d)", blocks, pw.K, a.lda);
     XFT_REQUIRE(a.ldc >= (a.glu ? pw.N / 2 : pw.N) && a.glu == ((pw.flags & XFTHIP_WF_GATEUP) != 0), "tile_gemm: ldc=%d N=%d glu=%d", a.ldc, pw.N, a.glu);
-    XFT_REQUIRE(!a.bias || (!a.glu && !a.group), "tile_gemm: a bias joins plain products only");
+    XFT_REQUIRE(!a.bias || !a.group, "tile_gemm: no bias in groups");
+    XFT_REQUIRE(a.decay_tau >= 0.0f && (a.decay_tau == 0.0f || (!a.glu && !a.add && !a.side && !a.group)), "tile_gemm: decays of plain products only");
     XFT_REQUIRE((!a.add || (a.c_dtype == XFTHIP_F32 && !a.glu)) && (!a.side || (!a.glu && !a.group && a.side_ids)) && (!a.group || a.group_rows),
             "tile_gemm: options that do not go together");
     const TileGemm p = {pw.packed, pw.KT, pw.K / 32, pw.NTILES, pw.N, M, a.A, a.lda, a.block_cols / 16, a.a_block_stride, a.C, a.ldc, a.c_dtype, a.glu, a.add,
-            a.glu_limit, a.glu_alpha, a.bias, a.side, a.side_ld, a.side_vocab, a.side_ids, a.group, a.group_rows, a.a_rows};
+            a.glu_limit, a.glu_alpha, a.bias, a.decay_tau > 0.0f ? 1.0f / a.decay_tau : 0.0f, a.side, a.side_ld, a.side_vocab, a.side_ids, a.group, a.group_rows, a.a_rows};
     const unsigned gz = a.group ? (unsigned)a.group_n : 1;
     const unsigned gx = (unsigned)((pw.NTILES + 7) / 8), gx1 = (unsigned)((pw.NTILES + 1) / 2);
     const bool f32 = act_in == XFTHIP_F32;
