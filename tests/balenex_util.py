@@ -6,7 +6,7 @@ from plan_util import Case, bf16_bits, bf16_values, oracle_weights, rel_rms  # n
 import plan_util
 
 
-def pooled(heads=6, kv_heads=2, dim=20, vdim=28, window=29, pool=5, scale=0.9):
+def pooled(heads=6, kv_heads=2, dim=20, vdim=28, window=9, pool=3, scale=0.2):
     return dict(type="attention", mixer=dict(heads=heads, kv_heads=kv_heads, dim=dim, vdim=vdim, mask=dict(size=window, pool=pool), scale=scale))
 
 
@@ -39,8 +39,11 @@ def weights(cfg, seed):
         elif leaf == "conv":
             x *= 0.6
         elif leaf != "embed":
-            x *= (2.0 if leaf in ("k", "q") else 1.0) / np.sqrt(shape[-1])
+            x *= (2.0 if leaf in ("q", "k", "v") else 1.0) / np.sqrt(shape[-1])
         out[name] = bf16_bits(x)
+    for name in out:  # (a read-out near zero would have its sign, and the normed result, decided by rounding)
+        if name.endswith("right.k"):
+            out[name] = bf16_bits(0.6 * bf16_values(out[name]) + 0.8 * bf16_values(out[name[:-1] + "q"]))
     return out
 
 

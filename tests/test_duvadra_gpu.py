@@ -396,8 +396,8 @@ def test_broken_plans_are_refused(xh):
                 [left, dict(right, inter=8)], [left, dict(right, decay_rank=4)]):
         with pytest.raises(xh.XftHipError):
             xh.Plan(72, 90, bad, **stack)
-    with pytest.raises(xh.XftHipError):  # plain norms belong to serial blocks
-        xh.Plan(72, 90, [attention], block=0, norm=2)
+    with pytest.raises(xh.XftHipError):  # plain norms do not belong to parallel blocks
+        xh.Plan(72, 90, [attention], block=1, norm=2)
     cfg = u.config([(u.windowed_delta(), u.moe()), (u.keyed_unit(), None)])
     bits = u.weights(cfg, 1)
     for name in ("bigram", "l0.mlp.e3.up", "l0.norm2", "l0.mix.left.k.b", "l0.mix.right.dt_bias", "l1.mix.left.k.norm", "l1.mix.right.ri.b"):

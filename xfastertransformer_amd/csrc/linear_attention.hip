@@ -26,8 +26,8 @@ struct LinearParams {
 
 // sums of two values over aligned groups of 32 lanes: of `a` in the first 16 of them, of `b` in the others
 __device__ inline float two_sums(float a, float b) {
-    const auto x = __builtin_amdgcn_permlane16_swap(__builtin_bit_cast(unsigned, a), __builtin_bit_cast(unsigned, b), false, false);
-    return group_sum<16>(__builtin_bit_cast(float, x[0]) + __builtin_bit_cast(float, x[1]));
+    const auto x = __builtin_amdgcn_permlane16_swap(f2u(a), f2u(b), false, false);
+    return group_sum<16>(u2f(x[0]) + u2f(x[1]));
 }
 
 // A walk over a segment's tokens with the state in registers.  The state's columns (value channels) do not interact: L lanes hold C neighbouring
