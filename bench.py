@@ -606,7 +606,7 @@ def moe_layer(xh, iters=5):
                      "counts stay on the device)")
 
 
-PLAN_MODELS = ("pinepel", "llama_bf16", "veterax", "duvadra", "mixtral_bf16")
+PLAN_MODELS = ("pinepel", "balenex", "llama_bf16", "veterax", "duvadra", "mixtral_bf16")
 PLAN_SIZES = {
     # width, ff, heads, query latent (the rest: 128 / 64 query dims, 128 value dims, key latent 512, 128-dim delta heads)
     "2048": dict(width=2048, ff=5632, heads=16, q_rank=768),
@@ -738,6 +738,50 @@ def build_duvadra(xh, sz, sp, vocab=32000):
     return plan
 
 
+def balenex_layers(sz, sp):
+    """Records (mixers side by side are two) and tensor shapes of a Balenex stack: a filtered attention with 64 kept tokens beside gated linear
+    attention, then two windowed attentions that see older tokens as means of 16, twice over; windows of 1024, dense feed-forwards."""
+    W, F, H, G = sz["width"], sz["ff"], sz["heads"], sp["kv_heads"]
+    own = dict(mixer=3, heads=H, kv_heads=G, dim=128, vdim=128, scale=128 ** -0.5, window=1024, qkv_bias=1, inter=F, mlp_bias=1)
+    result = dict(result_norm=1, scaled=1, mix_scale=0.5)
+    pooled = dict(own, qk_norm=3, pool=16, o_bias=1)
+    left = dict(own, qk_norm=1, keep_first=64, taps=4, rot_dim=64, rot_base=1e6, v_rot=1, **result)
+    right = dict(mixer=5, heads=H, dim=128, vdim=128, tau=16.0, decay_rank=64, beside=1, **result)
+    common = {"norm1": (W,), "norm1b": (W,), "norm2": (W,), "norm2b": (W,), "mlp.gate": (F, W), "mlp.gate.b": (F,), "mlp.up": (F, W), "mlp.up.b": (F,),
+              "mlp.down": (W, F), "mlp.down.b": (W,), "mix.o": (W, H * 128)}
+    for n, rows in (("q", H * 128), ("k", G * 128), ("v", G * 128)):
+        common["mix." + n], common["mix." + n + ".b"] = (rows, W), (rows,)
+    l_shapes = dict(common, **{"mix.q.norm": (128,), "mix.k.norm": (128,), "mix.out": (W,), "mix.q.conv": (H * 128, 4), "mix.k.conv": (G * 128, 4), "mix.v.conv": (G * 128, 4)})
+    r_shapes = {"mix.a1": (64, W), "mix.a2": (H * 128, 64), "mix.a2.b": (H * 128,), "mix.norm": (128,), "mix.out": (W,), "mix.o": (W, H * 128)}
+    for n in "qkvg":
+        r_shapes["mix." + n] = (H * 128, W)
+    p_shapes = dict(common, **{"mix.o.b": (W,)})
+    records = [(left, l_shapes), (right, r_shapes), (pooled, p_shapes), (pooled, p_shapes)] * 2
+    return [r for r, _ in records], [t for _, t in records]
+
+
+def build_balenex(xh, sz, sp, vocab=32000):
+    layers, shapes = balenex_layers(sz, sp)
+    W, rng = sz["width"], np.random.default_rng(5)
+    pool = xh.f32_to_bf16_bits(rng.standard_normal(1 << 22, dtype=np.float32) * 0.02)
+    plan = xh.Plan(W, vocab, layers, block=xh.BLOCK_SANDWICH, norm=xh.NORM_RMS, norm_groups=8)
+    one = xh.f32_to_bf16_bits(np.ones(1, np.float32))[0]
+
+    def bits(name, shape):
+        if "norm" in name.split(".")[-1] or name.endswith(".out"):
+            return np.full(shape, one, np.uint16)
+        return np.resize(np.roll(pool, int(rng.integers(1 << 20))), int(np.prod(shape))).reshape(shape)
+
+    embed = xh.f32_to_bf16_bits(rng.standard_normal((vocab, W), dtype=np.float32))
+    for n, b in (("embed", embed), ("head", bits("head", (vocab, W))), ("final.norm", bits("final.norm", (W,)))):
+        plan.set(-1, n, b)
+    for l, tensors in enumerate(shapes):
+        for n, s in tensors.items():
+            plan.set(l, n, bits(n, s))
+    plan.finish()
+    return plan
+
+
 def build_plan(xh, sz, vocab=32000):
     layers, shapes = plan_shapes(sz)
     pool = xh.f32_to_bf16_bits(np.random.default_rng(5).standard_normal(1 << 22, dtype=np.float32) * 0.02)
@@ -790,7 +834,7 @@ def build_llama_bf16(xh, sz, layers, batch, max_seq, max_tokens, vocab=32000, sp
 
 
 def plan_bench(xh, prompt=2048, batches=(1, 8, 32), steps=32, only=None, sizes=None, eager=False):
-    """Prefill (one prompt) and decode (behind prompts of that length) of Pinepel beside the uniform stack and of Veterax and Duvadra
+    """Prefill (one prompt) and decode (behind prompts of that length) of Pinepel and Balenex beside the uniform stack and of Veterax and Duvadra
     beside the uniform stack with sparse MLPs, six layers each, in the same run.  Prompts of a decode batch are run one by one."""
     out = []
     for name in sizes or list(PLAN_SIZES) + [n for n in SPARSE_SIZES if n not in PLAN_SIZES]:
@@ -800,8 +844,9 @@ def plan_bench(xh, prompt=2048, batches=(1, 8, 32), steps=32, only=None, sizes=N
                 continue
             B, max_seq = max(batches), prompt + 4 * (steps + 8)
             keep = []
-            if which in ("pinepel", "veterax", "duvadra"):
-                plan = build_plan(xh, sz) if which == "pinepel" else (build_veterax if which == "veterax" else build_duvadra)(xh, sz, sp)
+            if which in ("pinepel", "balenex", "veterax", "duvadra"):
+                build = dict(balenex=build_balenex, veterax=build_veterax, duvadra=build_duvadra)
+                plan = build_plan(xh, sz) if which == "pinepel" else build[which](xh, sz, sp)
                 model, wbytes = xh.PlanModel(plan, xh.BF16, B, max_seq, prompt), plan.bytes()
                 keep = [plan]
             else:
@@ -856,7 +901,7 @@ def main():
     ap.add_argument("--prefill-gemm", action="store_true", help="only the weight-only GEMM sweep: M = 256, 2048 against the MFMA peak, M = 1, 8, 32 against the HBM peak (one JSON line)")
     ap.add_argument("--attention", action="store_true", help="only the GQA attention sweep (one JSON line)")
     ap.add_argument("--moe", action="store_true", help="only the sparse-MLP layer (one JSON line)")
-    ap.add_argument("--plan", action="store_true", help="only the layer-plan stacks (Pinepel, Veterax, Duvadra) beside the uniform BF16 stacks of equal size (dense, sparse MLPs): prefill and decode (one JSON line; progress on stderr)")
+    ap.add_argument("--plan", action="store_true", help="only the layer-plan stacks (Pinepel, Balenex, Veterax, Duvadra) beside the uniform BF16 stacks of equal size (dense, sparse MLPs): prefill and decode (one JSON line; progress on stderr)")
     ap.add_argument("--plan-only", choices=PLAN_MODELS, help="with --plan: one of them")
     ap.add_argument("--plan-size", choices=sorted(SPARSE_SIZES), help="with --plan: one size")
     ap.add_argument("--no-live-traffic", action="store_true", help="do not run the two rocprofv3 counter passes for roofline.traffic (the recorded figure under profiles/ is reported instead)")
