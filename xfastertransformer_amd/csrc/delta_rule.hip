@@ -273,27 +273,25 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(ScanParams p) {
 
     f32x4 stage[PER];
     float vstage[PERV], cstage = 0.0f;
+    // (threads without a part fetch the last one: a load under a condition would be waited for before the next one goes out)
     auto fetch = [&](int c0) {
 #pragma unroll
         for (int i = 0; i < PER; ++i) {
-            const int e = i * 256 + threadIdx.x;
+            const int part = i * 256 + (int)threadIdx.x, e = part < ARRAYS * CHUNK4 ? part : ARRAYS * CHUNK4 - 1;
             const int arr = e / CHUNK4, r = e % CHUNK4, tok = r / (KD / 4), d = (r % (KD / 4)) * 4;
             const int t = off + (c0 + tok < n ? c0 + tok : n - 1);
-            if (e < ARRAYS * CHUNK4) {
-                const float *src = arr == 2 ? p.b.g + ((size_t)t * p.H + head) * KD : (arr ? p.b.k : p.b.q) + ((size_t)t * p.KH + kvh) * KD;
-                stage[i] = *(const f32x4 *)(src + d);
-            }
+            const float *src = arr == 2 ? p.b.g + ((size_t)t * p.H + head) * KD : (arr ? p.b.k : p.b.q) + ((size_t)t * p.KH + kvh) * KD;
+            stage[i] = *(const f32x4 *)(src + d);
         }
 #pragma unroll
         for (int i = 0; i < PERV; ++i) {
-            const int e = i * 256 + threadIdx.x, tok = e / COLS, c = col0 + e % COLS;
+            const int part = i * 256 + (int)threadIdx.x, e = part < CT * COLS ? part : CT * COLS - 1, tok = e / COLS, c = col0 + e % COLS;
             const int t = off + (c0 + tok < n ? c0 + tok : n - 1);
-            if (e < CT * COLS) vstage[i] = p.b.v[((size_t)t * p.H + head) * p.VD + (c < p.VD ? c : p.VD - 1)];
+            vstage[i] = p.b.v[((size_t)t * p.H + head) * p.VD + (c < p.VD ? c : p.VD - 1)];
         }
-        if (threadIdx.x < SCALARS * CT) {
-            const int tok = threadIdx.x % CT, t = off + (c0 + tok < n ? c0 + tok : n - 1);
-            cstage = threadIdx.x < CT ? p.b.beta[(size_t)t * p.H + head] : threadIdx.x < 2 * CT ? p.b.qk[(size_t)t * p.KH + kvh] : p.b.g[(size_t)t * p.H + head];
-        }
+        const int tok = threadIdx.x % CT, t = off + (c0 + tok < n ? c0 + tok : n - 1);
+        const float *scalar = threadIdx.x < CT ? p.b.beta + (size_t)t * p.H + head : threadIdx.x < 2 * CT || !ONE ? p.b.qk + (size_t)t * p.KH + kvh : p.b.g + (size_t)t * p.H + head;
+        cstage = *scalar;
     };
     auto stash = [&](int buf) {
 #pragma unroll
@@ -308,6 +306,10 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(ScanParams p) {
         }
         if (threadIdx.x < SCALARS * CT) sc[buf][threadIdx.x] = cstage;
     };
+#pragma unroll
+    for (int c = 0; c < C; ++c)
+#pragma unroll
+        for (int r = 0; r < RV; ++r) arrived(s[c][r]);
     fetch(0);
     stash(0);
     __syncthreads();

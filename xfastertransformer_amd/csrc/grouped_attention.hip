@@ -247,35 +247,43 @@ __global__ __launch_bounds__(256) void grouped_means_kernel(PrepareParams p) {
     const size_t dst = head_page(p.b.means_table + (size_t)p.v.seg_row[seg] * p.b.means_stride, block, G, g, D, V);
     const int first = block * p.pool, end = first + p.pool;
     const float inv = 1.0f / (float)p.pool;
-    for (int i = threadIdx.x; i < D / 8 + V; i += 256) {
-        if (i < D / 8) {
-            float x[8] = {0.0f, 0.0f, 0.0f, 0.0f, 0.0f, 0.0f, 0.0f, 0.0f}, w[8];
-            for (int j = first; j < end; ++j) {
-                load8<BF16>(p.b.pool, head_page(table, j, G, g, D, V) + (size_t)(j % kPageTokens) * D + i * 8, w);
+    // keys: p.lanes threads a token, the sets of threads take turns; values: a thread a dimension
+    __shared__ float sums[256 * 8];
+    const int sets = 256 / p.lanes, set = (int)threadIdx.x / p.lanes, c = (int)threadIdx.x % p.lanes * 8;
+    float x[8] = {0.0f, 0.0f, 0.0f, 0.0f, 0.0f, 0.0f, 0.0f, 0.0f};
+    for (int j = first + set; j < end && c < D; j += sets) {
+        float w[8];
+        load8<BF16>(p.b.pool, head_page(table, j, G, g, D, V) + (size_t)(j % kPageTokens) * D + c, w);
 #pragma unroll
-                for (int k = 0; k < 8; ++k) x[k] += w[k];
-            }
-#pragma unroll
-            for (int k = 0; k < 8; ++k) x[k] *= inv;
-            store8<BF16>(p.b.means, dst + (size_t)(block % kPageTokens) * D + i * 8, x);
-        } else {
-            const int d = i - D / 8;
-            float sum = 0.0f;
-            for (int j = first; j < end;) { // (runs of tokens of a value block, eight at a time where they are whole)
-                const size_t at = head_page(table, j, G, g, D, V) + value_at(D, V, j % kPageTokens, d);
-                if (j % 8 == 0 && j + 8 <= end) {
-                    float w[8];
-                    load8<BF16>(p.b.pool, at, w);
-                    sum += ((w[0] + w[1]) + (w[2] + w[3])) + ((w[4] + w[5]) + (w[6] + w[7]));
-                    j += 8;
-                } else {
-                    sum += ldact<BF16>(p.b.pool, at);
-                    ++j;
-                }
-            }
-            stact<BF16>(p.b.means, dst + value_at(D, V, block % kPageTokens, d), sum * inv);
-        }
+        for (int k = 0; k < 8; ++k) x[k] += w[k];
     }
+#pragma unroll
+    for (int k = 0; k < 8; ++k) sums[k * 256 + threadIdx.x] = x[k];
+    for (int d = threadIdx.x; d < V; d += 256) {
+        float sum = 0.0f;
+        for (int j = first; j < end;) { // (runs of tokens of a value block, eight at a time where they are whole)
+            const size_t at = head_page(table, j, G, g, D, V) + value_at(D, V, j % kPageTokens, d);
+            if (j % 8 == 0 && j + 8 <= end) {
+                float w[8];
+                load8<BF16>(p.b.pool, at, w);
+                sum += ((w[0] + w[1]) + (w[2] + w[3])) + ((w[4] + w[5]) + (w[6] + w[7]));
+                j += 8;
+            } else {
+                sum += ldact<BF16>(p.b.pool, at);
+                ++j;
+            }
+        }
+        stact<BF16>(p.b.means, dst + value_at(D, V, block % kPageTokens, d), sum * inv);
+    }
+    __syncthreads();
+    if (set > 0 || c >= D) return;
+#pragma unroll
+    for (int k = 0; k < 8; ++k) {
+        x[k] = 0.0f;
+        for (int t = 0; t < sets && t < p.pool; ++t) x[k] += sums[k * 256 + t * p.lanes + threadIdx.x];
+        x[k] *= inv;
+    }
+    store8<BF16>(p.b.means, dst + (size_t)(block % kPageTokens) * D + c, x);
 }
 
 struct AttendParams {

@@ -1,6 +1,8 @@
 // Gated linear attention of layer plans: per head S = diag(alpha) S + k v^T and o = S^T q, alpha a decay of every key channel, then the norm of
 // every head and a silu gate.  Queries, keys and values are read from the rows of the input product, the decays come out of their product's
 // epilogue; between those and the output projection's input everything is fp32.
+#include <type_traits>
+
 #include "plan_dev.h"
 
 namespace xfthip {
@@ -30,38 +32,46 @@ __device__ inline float two_sums(float a, float b) {
     return group_sum<16>(u2f(x[0]) + u2f(x[1]));
 }
 
-// A walk over a segment's tokens with the state in registers.  The state's columns (value channels) do not interact: L lanes hold C neighbouring
-// columns, 4 RV key rows each (KD = 4 L RV).  A token is S = g S + k v and a sum over the key rows that nothing waits for.  q, k, g of
-// CT tokens are staged in LDS, the next CT on their way through registers.  grid (segments, heads, column groups of COLS)
-template <bool BF16, int L, int RV, int C>
+// A walk over a segment's tokens with the state in registers.  The state's columns (value channels) do not interact: L lanes hold two
+// neighbouring columns, E key rows each (KD = E L).  A token is S = g S + k v and a sum over the key rows that nothing waits for.  q, k, g, v
+// of CT tokens are staged in LDS, the next CT on their way through registers.  grid (segments, heads, column groups of COLS)
+// (2048 tokens, 32 heads of 128: bound by one wave a SIMD and 33 vector instructions a token)
+template <int L, int E>
+struct ScanShape {
+    static constexpr int KD = E * L, COLS = 256 / L * 2, CT = KD > 128 ? 16 : 32;
+    static constexpr size_t lds_floats = 2 * (3 * CT * KD + 2 * CT * COLS);
+};
+template <bool BF16, int L, int E>
 __global__ __launch_bounds__(256) void linear_scan_kernel(LinearParams p) {
-    constexpr int KD = 4 * L * RV, COLS = 256 / L * C, CT = KD > 128 ? 8 : 16;
+    typedef float Rows __attribute__((ext_vector_type(E)));
+    typedef typename std::conditional<BF16, uint16_t, float>::type Act;
+    constexpr int KD = ScanShape<L, E>::KD, COLS = ScanShape<L, E>::COLS, CT = ScanShape<L, E>::CT;
     constexpr int QK8 = 2 * CT * KD / 8, G4 = CT * KD / 4; // groups of eight of q and k, float4 of the decays of a chunk
     constexpr int PERQ = (QK8 + 255) / 256, PERG = (G4 + 255) / 256, PERV = (CT * COLS + 255) / 256;
-    __shared__ float lds[2][3 * CT * KD];
-    __shared__ float vlds[2][CT * COLS];
-    __shared__ float olds[2][CT * COLS];
+    extern __shared__ __align__(16) float scan_lds[]; // twice: q, k, g [CT][KD], v, o [CT][COLS]
+    constexpr int HALF = 3 * CT * KD + 2 * CT * COLS, V0 = 3 * CT * KD, O0 = V0 + CT * COLS;
     const int seg = blockIdx.x, head = blockIdx.y, n = p.v.seg_len[seg], off = p.v.seg_off[seg];
-    const int li = threadIdx.x % L, lc = threadIdx.x / L * C, col0 = blockIdx.z * COLS, col = col0 + lc;
-    const bool own = col < p.VD; // (VD is a multiple of 32: C neighbouring columns are in it or not together)
-    float *state = p.state + (((size_t)p.v.seg_row[seg] * p.H + head) * p.VD + (own ? col : 0)) * KD + 4 * li;
+    const int li = threadIdx.x % L, lc = threadIdx.x / L * 2, col0 = blockIdx.z * COLS, col = col0 + lc;
+    const bool own = col < p.VD; // (VD is a multiple of 32: neighbouring columns are in it or not together)
+    float *state = p.state + (((size_t)p.v.seg_row[seg] * p.H + head) * p.VD + (own ? col : 0)) * KD + E * li;
     const int vcol = 2 * p.H * KD + head * p.VD;
-    f32x4 s[C][RV];
+    Rows s[2];
 #pragma unroll
-    for (int c = 0; c < C; ++c)
-#pragma unroll
-        for (int r = 0; r < RV; ++r) s[c][r] = p.v.seg_pos[seg] > 0 ? *(const f32x4 *)(state + c * KD + r * 4 * L) : f32x4 {0.f, 0.f, 0.f, 0.f};
+    for (int c = 0; c < 2; ++c) {
+        s[c] = p.v.seg_pos[seg] > 0 ? *(const Rows *)(state + c * KD) : (Rows)0.0f;
+        arrived(s[c]);
+    }
 
     constexpr int WORDS = BF16 ? 1 : 2; // of 16 bytes that hold eight activations
     u32x4 qk[PERQ][WORDS];
     f32x4 g[PERG];
-    float vs[PERV];
+    Act vs[PERV];
     auto token_at = [&](int i) { return off + (i < n ? i : n - 1); };
+    // (threads without a part take the last one too: a load under a condition would be waited for before the next one goes out)
     auto fetch = [&](int c0) {
 #pragma unroll
         for (int i = 0; i < PERQ; ++i) {
-            const int e = i * 256 + threadIdx.x, k = e / (QK8 / 2), r = e % (QK8 / 2);
-            if (e >= QK8) continue;
+            const int part = i * 256 + (int)threadIdx.x, e = part < QK8 ? part : QK8 - 1, k = e / (QK8 / 2), r = e % (QK8 / 2);
             const size_t at = (size_t)token_at(c0 + r / (KD / 8)) * p.ld + (size_t)(k * p.H + head) * KD + r % (KD / 8) * 8;
             const u32x4 *src = (const u32x4 *)((const char *)p.in + at * (BF16 ? 2 : 4));
 #pragma unroll
@@ -69,22 +79,20 @@ __global__ __launch_bounds__(256) void linear_scan_kernel(LinearParams p) {
         }
 #pragma unroll
         for (int i = 0; i < PERG; ++i) {
-            const int e = i * 256 + threadIdx.x;
-            if (e < G4) g[i] = *(const f32x4 *)(p.alpha + ((size_t)token_at(c0 + e / (KD / 4)) * p.H + head) * KD + e % (KD / 4) * 4);
+            const int part = i * 256 + (int)threadIdx.x, e = part < G4 ? part : G4 - 1;
+            g[i] = *(const f32x4 *)(p.alpha + ((size_t)token_at(c0 + e / (KD / 4)) * p.H + head) * KD + e % (KD / 4) * 4);
         }
 #pragma unroll
         for (int i = 0; i < PERV; ++i) {
-            const int e = i * 256 + threadIdx.x, c = col0 + e % COLS;
-            if (e < CT * COLS) vs[i] = ldact<BF16>(p.in, (size_t)token_at(c0 + e / COLS) * p.ld + vcol + (c < p.VD ? c : p.VD - 1));
+            const int part = i * 256 + (int)threadIdx.x, e = part < CT * COLS ? part : CT * COLS - 1, c = col0 + e % COLS;
+            vs[i] = ((const Act *)p.in)[(size_t)token_at(c0 + e / COLS) * p.ld + vcol + (c < p.VD ? c : p.VD - 1)];
         }
     };
-    auto stash = [&](int buf) {
+    auto stash = [&](int c0, float *lds) { // (a token past the end: decays of one, a key of zero)
 #pragma unroll
         for (int i = 0; i < PERQ; ++i) {
-            const int e = i * 256 + threadIdx.x;
-            if (e >= QK8) continue;
-            const float mul = e < QK8 / 2 ? p.qscale : 1.0f;
-            float *dst = &lds[buf][8 * e];
+            const int part = i * 256 + (int)threadIdx.x, e = part < QK8 ? part : QK8 - 1;
+            const float mul = e < QK8 / 2 ? p.qscale : c0 + e % (QK8 / 2) / (KD / 8) < n ? 1.0f : 0.0f;
             f32x4 lo, hi;
             if constexpr (BF16) {
 #pragma unroll
@@ -95,86 +103,99 @@ __global__ __launch_bounds__(256) void linear_scan_kernel(LinearParams p) {
             } else {
                 lo = __builtin_bit_cast(f32x4, qk[i][0]), hi = __builtin_bit_cast(f32x4, qk[i][WORDS - 1]);
             }
-            *(f32x4 *)dst = lo * mul, *(f32x4 *)(dst + 4) = hi * mul;
+            *(f32x4 *)(lds + 8 * e) = lo * mul, *(f32x4 *)(lds + 8 * e + 4) = hi * mul;
         }
 #pragma unroll
         for (int i = 0; i < PERG; ++i) {
-            const int e = i * 256 + threadIdx.x;
-            if (e < G4) *(f32x4 *)(&lds[buf][2 * CT * KD + 4 * e]) = g[i];
+            const int part = i * 256 + (int)threadIdx.x, e = part < G4 ? part : G4 - 1;
+            *(f32x4 *)(lds + 2 * CT * KD + 4 * e) = c0 + e / (KD / 4) < n ? g[i] : f32x4 {1.f, 1.f, 1.f, 1.f};
         }
 #pragma unroll
         for (int i = 0; i < PERV; ++i) {
-            const int e = i * 256 + threadIdx.x;
-            if (e < CT * COLS) vlds[buf][e] = vs[i];
+            const int part = i * 256 + (int)threadIdx.x, e = part < CT * COLS ? part : CT * COLS - 1;
+            if constexpr (BF16) lds[V0 + e] = bf16_to_f32(vs[i]);
+            else lds[V0 + e] = vs[i];
         }
     };
     fetch(0);
-    stash(0);
+    stash(0, scan_lds);
     __syncthreads();
     int buf = 0;
     for (int c0 = 0; c0 < n; c0 += CT, buf ^= 1) {
+        float *lds = scan_lds + buf * HALF;
         const int m = n - c0 < CT ? n - c0 : CT;
-        if (c0 + CT < n) fetch(c0 + CT);
+        fetch(c0 + CT);
         struct Operands {
-            f32x4 q[RV], k[RV], g[RV];
-            float v[C];
+            Rows q, k, g;
+            float2 v;
         };
-        auto read = [&](int i) {
-            const float *q = lds[buf] + i * KD + 4 * li, *k = q + CT * KD, *a = k + CT * KD;
-            Operands x;
+        auto read = [&](Operands (&x)[2], int i) {
 #pragma unroll
-            for (int r = 0; r < RV; ++r)
-                x.q[r] = *(const f32x4 *)(q + r * 4 * L), x.k[r] = *(const f32x4 *)(k + r * 4 * L), x.g[r] = *(const f32x4 *)(a + r * 4 * L);
-#pragma unroll
-            for (int c = 0; c < C; ++c) x.v[c] = vlds[buf][i * COLS + lc + c];
-            return x;
-        };
-        auto token = [&](const Operands &x, int i) {
-            float o[C];
-#pragma unroll
-            for (int c = 0; c < C; ++c) {
-                o[c] = 0.0f;
-#pragma unroll
-                for (int r = 0; r < RV; ++r)
-#pragma unroll
-                    for (int e = 0; e < 4; ++e) {
-                        s[c][r][e] = fmaf(x.g[r][e], s[c][r][e], x.k[r][e] * x.v[c]);
-                        o[c] = fmaf(x.q[r][e], s[c][r][e], o[c]);
-                    }
+            for (int b = 0; b < 2; ++b) {
+                const float *q = lds + (i + b) * KD + E * li, *k = q + CT * KD, *a = k + CT * KD;
+                x[b] = Operands {*(const Rows *)q, *(const Rows *)k, *(const Rows *)a, *(const float2 *)(lds + V0 + (i + b) * COLS + lc)};
             }
-            if constexpr (L == 32 && C == 2) {
-                const float sum = two_sums(o[0], o[1]);
-                if (li % 16 == 0) olds[buf][i * COLS + lc + li / 16] = sum;
+        };
+        float o[4][2];
+        auto tokens = [&](const Operands (&x)[2], int first) {
+#pragma unroll
+            for (int b = 0; b < 2; ++b)
+#pragma unroll
+                for (int c = 0; c < 2; ++c) {
+                    const float v = c ? x[b].v.y : x[b].v.x;
+                    float sum = 0.0f;
+#pragma unroll
+                    for (int e = 0; e < E; ++e) {
+                        s[c][e] = fmaf(x[b].g[e], s[c][e], x[b].k[e] * v);
+                        sum = fmaf(x[b].q[e], s[c][e], sum);
+                    }
+                    o[first + b][c] = sum;
+                }
+        };
+        // Four tokens at a time, whose sums go round side by side; a pair's operands are asked for a pair ahead (more reads in flight than
+        // the hardware counts would be waited for).  Tokens past the segment's end change nothing: stash.
+        Operands even[2], odd[2];
+        read(even, 0), read(odd, 2);
+        for (int i = 0; i < m; i += 4) {
+            const int next = i + 4 < CT ? i + 4 : 0;
+            tokens(even, 0);
+            read(even, next);
+            __builtin_amdgcn_sched_barrier(0);
+            tokens(odd, 2);
+            read(odd, next + 2);
+            __builtin_amdgcn_sched_barrier(0);
+            float *dst = lds + O0 + i * COLS + lc;
+            if constexpr (L == 32) {
+                float sum[4];
+#pragma unroll
+                for (int b = 0; b < 4; ++b) sum[b] = two_sums(o[b][0], o[b][1]);
+                if (li % 16 == 0) {
+#pragma unroll
+                    for (int b = 0; b < 4; ++b) dst[b * COLS + li / 16] = sum[b];
+                }
             } else {
 #pragma unroll
-                for (int c = 0; c < C; ++c) o[c] = group_sum<L>(o[c]);
+                for (int b = 0; b < 4; ++b) o[b][0] = group_sum<L>(o[b][0]), o[b][1] = group_sum<L>(o[b][1]);
                 if (li == 0) {
 #pragma unroll
-                    for (int c = 0; c < C; ++c) olds[buf][i * COLS + lc + c] = o[c];
+                    for (int b = 0; b < 4; ++b) *(float2 *)(dst + b * COLS) = make_float2(o[b][0], o[b][1]);
                 }
             }
-        };
-        // the operands of the next token are on their way from LDS while this one's sum goes round
-        Operands even = read(0), odd;
-        for (int i = 0; i < m; i += 2) {
-            odd = read(i + 1 < m ? i + 1 : i);
-            token(even, i);
-            if (i + 1 >= m) break;
-            even = read(i + 2 < m ? i + 2 : i + 1);
-            token(odd, i + 1);
         }
-        if (c0 + CT < n) stash(buf ^ 1); // (the other buffer, and the other results, were last read before or behind this barrier one chunk ago)
+        stash(c0 + CT, scan_lds + (buf ^ 1) * HALF); // (the other buffer, and the other results, were last read before or behind this barrier one chunk ago)
         __syncthreads();
-        for (int e = threadIdx.x; e < m * COLS; e += 256) {
-            const int c = col0 + e % COLS;
-            if (c < p.VD) p.o[((size_t)(off + c0 + e / COLS) * p.H + head) * p.VD + c] = olds[buf][e];
+        float y[PERV];
+#pragma unroll
+        for (int i = 0; i < PERV; ++i) y[i] = lds[O0 + (i * 256 + (int)threadIdx.x) % (CT * COLS)];
+#pragma unroll
+        for (int i = 0; i < PERV; ++i) {
+            const int e = i * 256 + (int)threadIdx.x, c = col0 + e % COLS;
+            if (e < m * COLS && c < p.VD) p.o[((size_t)(off + c0 + e / COLS) * p.H + head) * p.VD + c] = y[i];
         }
     }
     if (own) {
 #pragma unroll
-        for (int c = 0; c < C; ++c)
-#pragma unroll
-            for (int r = 0; r < RV; ++r) *(f32x4 *)(state + c * KD + r * 4 * L) = s[c][r];
+        for (int c = 0; c < 2; ++c) *(Rows *)(state + c * KD) = s[c];
     }
 }
 
@@ -224,19 +245,23 @@ __global__ __launch_bounds__(kStepThreads) void linear_step_kernel(LinearParams 
         stact<BF16>(p.out, (size_t)t * p.out_ld + head * p.VD + c, os[c] * f * p.norm[c] * silu_of<BF16>(ldact<BF16>(p.gate, row + head * p.VD + c)));
 }
 
-template <bool BF16>
-int launch_scan(int KD, const LinearParams &p, hipStream_t st) {
-    auto launch = [&](void (*kernel)(LinearParams), int cols) {
-        hipLaunchKernelGGL(kernel, dim3(p.v.B, p.H, (p.VD + cols - 1) / cols), dim3(256), 0, st, p);
-    };
-    switch (KD) {
-        case 32: launch(linear_scan_kernel<BF16, 8, 1, 2>, 64); break;
-        case 64: launch(linear_scan_kernel<BF16, 16, 1, 2>, 32); break;
-        case 128: launch(linear_scan_kernel<BF16, 32, 1, 2>, 16); break;
-        default: launch(linear_scan_kernel<BF16, 32, 2, 2>, 16); break;
-    }
+template <bool BF16, int L, int E>
+int launch_scan_shape(const LinearParams &p, hipStream_t st) {
+    using S = ScanShape<L, E>;
+    static const hipError_t attr = hipFuncSetAttribute((const void *)linear_scan_kernel<BF16, L, E>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
+    XFT_CHECK_HIP(attr);
+    hipLaunchKernelGGL((linear_scan_kernel<BF16, L, E>), dim3(p.v.B, p.H, (p.VD + S::COLS - 1) / S::COLS), dim3(256), S::lds_floats * 4, st, p);
     XFT_CHECK_HIP(hipGetLastError());
     return 0;
+}
+template <bool BF16>
+int launch_scan(int KD, const LinearParams &p, hipStream_t st) {
+    switch (KD) {
+        case 32: return launch_scan_shape<BF16, 8, 4>(p, st);
+        case 64: return launch_scan_shape<BF16, 16, 4>(p, st);
+        case 128: return launch_scan_shape<BF16, 32, 4>(p, st);
+        default: return launch_scan_shape<BF16, 32, 8>(p, st);
+    }
 }
 
 template <bool BF16>

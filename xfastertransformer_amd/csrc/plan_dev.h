@@ -129,6 +129,13 @@ __device__ inline float group_sum(float v) {
     return v;
 }
 
+// The value is in its register from here on.  What is loaded in front of a loop and changed in it would otherwise be waited for inside, and
+// with it the loads that the loop has just sent ahead.
+template <class V>
+__device__ inline void arrived(V &v) {
+    asm volatile("" : "+v"(v));
+}
+
 // tanh form of the Gaussian error linear unit
 __device__ inline float gelu_tanh(float z) { return 0.5f * z * (1.0f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z))); }
 

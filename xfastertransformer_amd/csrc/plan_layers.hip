@@ -263,7 +263,7 @@ int launch_group_norm(const PlanNormArgs &p, int T, hipStream_t st) {
         else launch(plan_group_norm_kernel<BF16, 4, 1024>, 1024);
     } else if (ch <= 1) launch(plan_group_norm_kernel<BF16, 1, 256>, 256);
     else if (ch <= 2) launch(plan_group_norm_kernel<BF16, 2, 256>, 256);
-    else if (ch <= 4) launch(plan_group_norm_kernel<BF16, 4, 256>, 256);
+    else if (ch <= 4) launch(plan_group_norm_kernel<BF16, 2, 512>, 512);
     else if (ch <= 8) launch(plan_group_norm_kernel<BF16, 4, 512>, 512);
     else launch(plan_group_norm_kernel<BF16, 4, 1024>, 1024);
     XFT_CHECK_HIP(hipGetLastError());

@@ -31,9 +31,16 @@ __device__ inline float precise_glu(float gate, float up, float limit, float alp
     return g / (1.0f + expf(-alpha * g)) * (u + 1.0f);
 }
 
-// sigmoid(z)^power
+// sigmoid(z)^power.  (FAST: log(1 + exp(-z)) may be off by a rounding of 1, which is a rounding of the result)
 template <bool FAST>
-__device__ inline float decay_of(float z, float power) { return exp_of<FAST>(-power * softplus_of<FAST>(-z)); }
+__device__ inline float decay_of(float z, float power) {
+    if constexpr (FAST) {
+        const float x = -kLog2e * z;
+        return __builtin_amdgcn_exp2f(-power * (x > 80.0f ? x : __builtin_amdgcn_logf(1.0f + __builtin_amdgcn_exp2f(x))));
+    } else {
+        return expf(-power * softplus_of<false>(-z));
+    }
+}
 
 // A wave: TW column tiles (16 weight columns each; two, or one in the 16-wave form) x MT row tiles (16 activation rows each).  The weight tile is the MFMA
 // A operand, the activation rows the B operand: a lane ends up with four neighbouring columns of one row.  With fp32
@@ -262,6 +269,9 @@ int tile_gemm(xfthip_weight_t w, int act_in, const TileGemmArgs &a, hipStream_t 
     } else if (M <= 16) {
         if (f32) launch(tile_gemm_kernel<true, 1, 4>, gx1, 1);
         else launch(tile_gemm_kernel<false, 1, 4>, gx1, 1);
+    } else if (!f32 && a.decay_tau > 0.0f) { // (a shallow K and a long epilogue: smaller tiles.  2048 rows x 4096 columns, K = 64: 24 us against 30)
+        if (M <= 32) launch(tile_gemm_kernel<false, 1, 4>, gx1, 2);
+        else launch(tile_gemm_kernel<false, 2, 1>, gx, (unsigned)((M + 31) / 32));
     } else if (M <= 32) {
         if (f32) launch(tile_gemm_kernel<true, 2, 4>, gx1, 1);
         else launch(tile_gemm_kernel<false, 2, 4>, gx1, 1);
