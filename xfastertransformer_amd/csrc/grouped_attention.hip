@@ -38,49 +38,87 @@ struct PrepareParams {
     int H, G, D, V, dim, vdim, rot, lanes; // lanes a head takes (a power of two, 8 values each)
     int h0, h1; // heads to move, key heads behind the query heads
     int all; // norms over all query heads, all key heads: a workgroup a token
-    int qk_blocks, seg_blocks, keep; // keep: write first_values
+    int v_blocks, seg_blocks, keep; // keep: write first_values
     float share, eps; // share of first_values in the values
 };
 
-// Eight neighbouring channels of token t's row from c on, behind their filter if there is one.  The only new token of a sequence shifts the
-// filter's inputs in place: a channel belongs to one thread.  (longer segments: conv_tail)
-template <bool BF16>
+// Eight neighbouring channels of token t's row from c on, behind their filter.  TAPS: of the filter (0: none, -1: any number).  The only new
+// token of a sequence shifts the filter's inputs in place: a channel belongs to one thread.  (longer segments: conv_tail)
+template <bool BF16, int TAPS>
 __device__ inline void filtered8(const PrepareParams &p, int t, int c, float (&x)[8]) {
     load8<BF16>(p.b.a, (size_t)t * p.ld + c, x);
-    if (!p.filter) return;
-    const int seg = p.v.tok_seg[t], pos = p.v.tok_pos[t], local = t - p.v.seg_off[seg], keep = p.taps - 1;
+    if constexpr (TAPS == 0) return;
+    const int seg = p.v.tok_seg[t], pos = p.v.tok_pos[t], local = t - p.v.seg_off[seg], keep = TAPS > 0 ? TAPS - 1 : p.taps - 1;
     const size_t hist = (size_t)p.v.seg_row[seg] * keep * p.channels + c;
-    float y[8], w[8], in[8];
-    load8<true>(p.filter, (size_t)keep * p.channels + c, w);
+    const bool alone = p.v.seg_len[seg] == 1;
+    // the input `back` tokens before this one: of the step, or kept from earlier ones (nothing in front of the sequence, but something to read)
+    auto input = [&](int back, float (&in)[8]) {
+        const bool here = local >= back;
+        load8<BF16>(here ? p.b.a : p.b.conv_state, here ? (size_t)(t - back) * p.ld + c : hist + (size_t)(keep + local - back) * p.channels, in);
+    };
+    float y[8];
+    if constexpr (TAPS > 0) {
+        float in[TAPS][8], w[TAPS][8];
 #pragma unroll
-    for (int k = 0; k < 8; ++k) y[k] = w[k] * x[k];
-    for (int back = 1; back <= keep && back <= pos; ++back) {
-        if (local >= back) load8<BF16>(p.b.a, (size_t)(t - back) * p.ld + c, in);
-        else load8<BF16>(p.b.conv_state, hist + (size_t)(keep + local - back) * p.channels, in);
-        load8<true>(p.filter, (size_t)(keep - back) * p.channels + c, w);
-#pragma unroll
-        for (int k = 0; k < 8; ++k) y[k] = fmaf(w[k], in[k], y[k]);
-    }
-    if (p.v.seg_len[seg] == 1 && keep > 0) {
-        for (int s = 0; s + 1 < keep; ++s) {
-            load8<BF16>(p.b.conv_state, hist + (size_t)(s + 1) * p.channels, in);
-            store8<BF16>(p.b.conv_state, hist + (size_t)s * p.channels, in);
+        for (int back = 0; back < TAPS; ++back) {
+            if (back > 0) input(back, in[back]);
+            load8<true>(p.filter, (size_t)(keep - back) * p.channels + c, w[back]);
         }
-        store8<BF16>(p.b.conv_state, hist + (size_t)(keep - 1) * p.channels, x);
+#pragma unroll
+        for (int k = 0; k < 8; ++k) in[0][k] = x[k], y[k] = w[0][k] * x[k];
+#pragma unroll
+        for (int back = 1; back < TAPS; ++back)
+#pragma unroll
+            for (int k = 0; k < 8; ++k) y[k] = fmaf(w[back][k], back <= pos ? in[back][k] : 0.0f, y[k]);
+        if (alone) {
+#pragma unroll
+            for (int s = 0; s < TAPS - 1; ++s) store8<BF16>(p.b.conv_state, hist + (size_t)s * p.channels, in[TAPS - 2 - s]);
+        }
+    } else {
+        float in[8], w[8];
+        load8<true>(p.filter, (size_t)keep * p.channels + c, w);
+#pragma unroll
+        for (int k = 0; k < 8; ++k) y[k] = w[k] * x[k];
+        for (int back = 1; back <= keep && back <= pos; ++back) {
+            input(back, in);
+            load8<true>(p.filter, (size_t)(keep - back) * p.channels + c, w);
+#pragma unroll
+            for (int k = 0; k < 8; ++k) y[k] = fmaf(w[k], in[k], y[k]);
+        }
+        if (alone && keep > 0) {
+            for (int s = 0; s + 1 < keep; ++s) {
+                load8<BF16>(p.b.conv_state, hist + (size_t)(s + 1) * p.channels, in);
+                store8<BF16>(p.b.conv_state, hist + (size_t)s * p.channels, in);
+            }
+            store8<BF16>(p.b.conv_state, hist + (size_t)(keep - 1) * p.channels, x);
+        }
     }
 #pragma unroll
     for (int k = 0; k < 8; ++k) x[k] = y[k];
 }
 
-// neighbouring pairs from dimension c on, turned by the angles of their tables' row (or back)
+// N / 2 neighbouring pairs from dimension c (a multiple of N) on, turned by the angles of their tables' row (or back)
 template <int N, bool BACK, class X>
 __device__ inline void turn_pairs(X &x, const float *cs, const float *sn, int c, int half) {
+    const int first = c / 2;
+    if (first >= half) return;
+    float cc[N / 2], ss[N / 2];
+    if (N == 8 && half % 4 == 0) {
+        const f32x4 a = *(const f32x4 *)(cs + first), b = *(const f32x4 *)(sn + first);
+#pragma unroll
+        for (int k = 0; k < N / 2; ++k) cc[k] = a[k], ss[k] = b[k];
+    } else {
+#pragma unroll
+        for (int k = 0; k < N / 2; ++k) { // (past the rotated part: its last pair's, unused)
+            const int i = first + k < half ? first + k : half - 1;
+            cc[k] = cs[i], ss[k] = sn[i];
+        }
+    }
 #pragma unroll
     for (int k = 0; k < N / 2; ++k) {
-        const int i = c / 2 + k;
-        if (i >= half) continue;
-        const float u = x[2 * k], z = x[2 * k + 1], cc = cs[i], ss = BACK ? -sn[i] : sn[i];
-        x[2 * k] = fmaf(u, cc, -(z * ss)), x[2 * k + 1] = fmaf(z, cc, u * ss);
+        const float u = x[2 * k], z = x[2 * k + 1], turn = BACK ? -ss[k] : ss[k];
+        const bool on = first + k < half;
+        x[2 * k] = on ? fmaf(u, cc[k], -(z * turn)) : u, x[2 * k + 1] = on ? fmaf(z, cc[k], u * turn) : z;
     }
 }
 
@@ -126,14 +164,15 @@ __device__ inline void move_values(const PrepareParams &p, int t, int hh, int c,
     store8<BF16>(p.b.means, head_page(p.b.means_table + (size_t)slot * p.b.means_stride, block, G, hh - H, D, p.V) + (size_t)(block % kPageTokens) * D + c, x);
 }
 
-// One launch, two kinds of workgroups.  The first qk_blocks: a group of `lanes` threads one query or key head of a token (norms over all
-// heads: a workgroup a token).  The others: one head's values of up to 32 tokens (a block of the cache), turned round through LDS.
-template <bool BF16>
+// One launch, two kinds of workgroups.  The first v_blocks: one head's values of up to 32 tokens (a block of the cache), turned round through
+// LDS (the longer way, so they go first).  The others: a group of `lanes` threads one query or key head of a token (norms over all heads: a
+// workgroup a token).
+template <bool BF16, int TAPS>
 __global__ __launch_bounds__(256) void grouped_prepare_kernel(PrepareParams p) {
     const int D = p.D, V = p.V, H = p.H, G = p.G;
-    if ((int)blockIdx.x < p.qk_blocks && p.all) {
+    if ((int)blockIdx.x >= p.v_blocks && p.all) {
         __shared__ float part[8];
-        const int t = blockIdx.x, q_end = H * D, end = p.h1 * D; // (h0 is 0)
+        const int t = (int)blockIdx.x - p.v_blocks, q_end = H * D, end = p.h1 * D; // (h0 is 0)
         const size_t row = (size_t)t * p.ld;
         float sq = 0.0f, sk = 0.0f;
         for (int e = threadIdx.x * 8; e < end; e += 2048) {
@@ -156,8 +195,8 @@ __global__ __launch_bounds__(256) void grouped_prepare_kernel(PrepareParams p) {
         }
         return;
     }
-    if ((int)blockIdx.x < p.qk_blocks) {
-        const size_t idx = (size_t)blockIdx.x * 256 + threadIdx.x;
+    if ((int)blockIdx.x >= p.v_blocks) {
+        const size_t idx = (size_t)((int)blockIdx.x - p.v_blocks) * 256 + threadIdx.x;
         const size_t item = idx / p.lanes;
         const int c = (int)(idx % p.lanes) * 8, heads = p.h1 - p.h0;
         const bool on = item < (size_t)p.v.T * heads && c < D;
@@ -165,7 +204,7 @@ __global__ __launch_bounds__(256) void grouped_prepare_kernel(PrepareParams p) {
         float x[8];
 #pragma unroll
         for (int k = 0; k < 8; ++k) x[k] = 0.0f;
-        if (on) filtered8<BF16>(p, t, hh * D + c, x);
+        if (on) filtered8<BF16, TAPS>(p, t, hh * D + c, x);
         float r = 1.0f;
         if (p.normed) {
             float sq = 0.0f;
@@ -178,7 +217,7 @@ __global__ __launch_bounds__(256) void grouped_prepare_kernel(PrepareParams p) {
         return;
     }
     __shared__ float tile[32][129];
-    int job = (int)blockIdx.x - p.qk_blocks;
+    int job = blockIdx.x;
     const int g = job % G;
     job /= G;
     const int seg = job / p.seg_blocks, start = p.v.seg_pos[seg], n = p.v.seg_len[seg], off = p.v.seg_off[seg];
@@ -194,7 +233,7 @@ __global__ __launch_bounds__(256) void grouped_prepare_kernel(PrepareParams p) {
             const int tok = lo + i / (slice / 8), c = i % (slice / 8) * 8, t = off + tok - start;
             const size_t first = ((size_t)t * G + g) * V + d0 + c;
             float x[8];
-            filtered8<BF16>(p, t, p.value_col + g * V + d0 + c, x);
+            filtered8<BF16, TAPS>(p, t, p.value_col + g * V + d0 + c, x);
             if (p.cosV) {
                 const size_t row = (size_t)tok * (p.vdim / 2);
                 turn_pairs<8, false>(x, p.cosV + row, p.sinV + row, d0 + c, p.vdim / 2);
@@ -907,12 +946,22 @@ int grouped_prepare(int act, const PlanLayer &L, const StepView &v, const Groupe
             s.v_mix && !L.first_values ? L.value_share : 0.0f, eps};
     while (p.lanes * 8 < L.D) p.lanes *= 2;
     XFT_REQUIRE(p.lanes <= 64, "grouped_prepare: heads of %d values too wide", L.D);
-    p.qk_blocks = p.h0 >= p.h1 ? 0 : p.all ? v.T : (int)(((size_t)v.T * (p.h1 - p.h0) * p.lanes + 255) / 256);
+    const int qk_blocks = p.h0 >= p.h1 ? 0 : p.all ? v.T : (int)(((size_t)v.T * (p.h1 - p.h0) * p.lanes + 255) / 256);
     p.seg_blocks = own ? (v.longest + 62) / 32 : 0; // blocks of 32 positions a segment of that length can touch
-    const dim3 grid(p.qk_blocks + v.B * s.kv_heads * p.seg_blocks);
+    p.v_blocks = v.B * s.kv_heads * p.seg_blocks;
+    const dim3 grid(p.v_blocks + qk_blocks);
     if (grid.x == 0) return 0;
-    if (act == XFTHIP_BF16) hipLaunchKernelGGL(grouped_prepare_kernel<true>, grid, dim3(256), 0, st, p);
-    else hipLaunchKernelGGL(grouped_prepare_kernel<false>, grid, dim3(256), 0, st, p);
+    auto launch = [&](void (*bf16)(PrepareParams), void (*f32)(PrepareParams)) {
+        if (act == XFTHIP_BF16) hipLaunchKernelGGL(bf16, grid, dim3(256), 0, st, p);
+        else hipLaunchKernelGGL(f32, grid, dim3(256), 0, st, p);
+    };
+    switch (L.filters() ? s.taps : 0) {
+        case 0: launch(grouped_prepare_kernel<true, 0>, grouped_prepare_kernel<false, 0>); break;
+        case 2: launch(grouped_prepare_kernel<true, 2>, grouped_prepare_kernel<false, 2>); break;
+        case 3: launch(grouped_prepare_kernel<true, 3>, grouped_prepare_kernel<false, 3>); break;
+        case 4: launch(grouped_prepare_kernel<true, 4>, grouped_prepare_kernel<false, 4>); break;
+        default: launch(grouped_prepare_kernel<true, -1>, grouped_prepare_kernel<false, -1>);
+    }
     XFT_CHECK_HIP(hipGetLastError());
     if (L.filters())
         if (int rc = conv_tail(act, v, b.a, L.in_ld, L.channels(), s.taps, b.conv_state, st)) return rc;
